@@ -6,7 +6,7 @@
 //   0 nothing   1 lane 0 of wave 0: fence(acquire, agent)   2 lane 0: fence(release, agent) then fence(acquire, agent)
 //   3 as 1 but the stores are NOT drained first
 // The host then reads the buffer back and counts pieces that do not hold their value.
-// Build + run on the GPU box:  hipcc -O3 --offload-arch=gfx950 tools/buffer_inv_probe.hip -o /tmp/bip && /tmp/bip
+// Build + run on the GPU box:  hipcc -O3 -Xclang -target-feature -Xclang -packed-fp32-ops --offload-arch=gfx950 tools/buffer_inv_probe.hip -o /tmp/bip && /tmp/bip
 #include <hip/hip_runtime.h>
 #include <stdio.h>
 #include <stdlib.h>

@@ -27,6 +27,7 @@ def main():
         with tempfile.TemporaryDirectory() as d:
             out = os.path.join(d, "k.s")
             subprocess.run(["/opt/rocm/bin/hipcc", "-O3", "-std=c++17", "-ffp-contract=off", "--offload-arch=gfx950",
+                            "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
                             "-I" + os.path.join(ROOT, "include"), "--cuda-device-only", "-S", "-o", out, SRC],
                            check=True, capture_output=True)
             text = open(out).read()

@@ -1,5 +1,5 @@
 // r05 probe: v_mfma_scale_f32_16x16x128_f8f6f4 / _32x32x64_ with OCP e4m3 operands on gfx950 — operand lane map, scale
-// semantics, issue rate.  hipcc --offload-arch=gfx950 -O3 tools/mfma_f8f6f4_probe.hip -o /tmp/mfma_f8_probe && /tmp/mfma_f8_probe
+// semantics, issue rate.  hipcc --offload-arch=gfx950 -O3 -Xclang -target-feature -Xclang -packed-fp32-ops tools/mfma_f8f6f4_probe.hip -o /tmp/mfma_f8_probe && /tmp/mfma_f8_probe
 //   (1) exact-integer check of the assumed map: lane l holds, for row (A) / column (B) l & 15, the 32 consecutive k
 //       32 (l >> 4) .. + 31 in its 8 operand registers (byte j of the 32-byte fragment = k 32 (l >> 4) + j); D as every
 //       16x16 MFMA (col = l & 15, row = 4 (l >> 4) + reg).  Asymmetric A and B.

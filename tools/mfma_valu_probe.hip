@@ -2,7 +2,7 @@
 // on gfx950 (r04; design input for csrc/prefill_attn64.hip).  Each variant runs a loop whose body holds 16 independent
 // v_mfma_f32_16x16x32_bf16 (16 accumulators) with a fixed filler after every MFMA; one workgroup of 256 threads per CU
 // (LDS request blocks a second one), time from s_memtime of wave 0 and from the wall clock.
-// Build + run on the GPU box:  hipcc -O3 --offload-arch=gfx950 tools/mfma_valu_probe.hip -o /tmp/mvp && /tmp/mvp
+// Build + run on the GPU box:  hipcc -O3 -Xclang -target-feature -Xclang -packed-fp32-ops --offload-arch=gfx950 tools/mfma_valu_probe.hip -o /tmp/mvp && /tmp/mvp
 #include <hip/hip_runtime.h>
 #include <stdio.h>
 #include <stdlib.h>

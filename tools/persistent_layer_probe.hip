@@ -7,7 +7,7 @@
 //       streaming (a 4 KiB-per-lane read loop) between two barriers;
 //   (b) the host/graph cost of launching that grid cooperatively (hipLaunchCooperativeKernel) against a plain launch, eager
 //       and replayed from a captured graph.
-// Build + run on the GPU box:  hipcc -O3 --offload-arch=gfx950 tools/persistent_layer_probe.hip -o /tmp/plp && /tmp/plp
+// Build + run on the GPU box:  hipcc -O3 -Xclang -target-feature -Xclang -packed-fp32-ops --offload-arch=gfx950 tools/persistent_layer_probe.hip -o /tmp/plp && /tmp/plp
 #include <hip/hip_runtime.h>
 #include <stdio.h>
 #include <stdlib.h>

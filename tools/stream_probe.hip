@@ -2,7 +2,7 @@
 //   mode 0: contiguous — a wave instruction reads 1 KiB contiguous (fragment-major / packed layout)
 //   mode 1: row fragments — a wave instruction reads 16 rows x 64 B, rows `row_bytes` apart (gemm_smallm today)
 // Each wave keeps 8 x 16 B loads in flight (unrolled), 4 waves per workgroup, WGs stream `bytes_per_wg`.
-// build: hipcc --offload-arch=gfx950 -O3 -o stream_probe tools/stream_probe.hip
+// build: hipcc --offload-arch=gfx950 -O3 -Xclang -target-feature -Xclang -packed-fp32-ops -o stream_probe tools/stream_probe.hip
 #include <hip/hip_runtime.h>
 #include <stdio.h>
 #include <stdlib.h>
