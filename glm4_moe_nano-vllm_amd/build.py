@@ -20,7 +20,8 @@ LIBDIR = os.path.join(HERE, "lib")
 LIB = os.path.join(LIBDIR, "libglm4moe_hip.so")
 ARCH = "gfx950"
 SOURCES = ["api", "elementwise", "moe_misc", "paged_attn", "prefill_attn", "gemm_smallm", "gemm_tinym", "gemm_largem",
-           "decode_engine", "oneshot_allreduce"]
+           "decode_engine", "oneshot_allreduce", "seq_norm", "gemm_f32", "latent_attn",
+           "window_attn"]
 # kernels that were measured against the shipped ones and lost: only in the study library (`--study`), with their tests
 STUDY_SOURCES = ["prefill_attn64", "prefill_attn_persist"]
 STUDY_TAG = "_study"

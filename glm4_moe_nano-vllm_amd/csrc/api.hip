@@ -13,7 +13,7 @@ void glm_set_error(const char* fmt, ...) {
     va_end(ap);
 }
 
-extern "C" int glm_abi_version(void) { return 10; }
+extern "C" int glm_abi_version(void) { return 11; }
 extern "C" const char* glm_last_error(void) { return g_err; }
 
 // ---- launch-path options: name, environment variable read once, default ------------------------------------------------
@@ -138,6 +138,31 @@ extern "C" int glm_gemm_bf16(const void* x, int64_t ldx, const void* w, int64_t 
         if (rc != GLM_ERR_UNSUPPORTED) return rc;
     }
     return dispatch(GEMM_PLAIN, p, glm_s(stream));
+}
+
+extern "C" int glm_gemm_bf16_act(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* bias, void* y, int64_t ldy,
+                                 int64_t M, int N, int K, int out_f32, int act, float act_a, float act_b, glm_stream_t stream) {
+    GLM_CHECK_ARG(x && w && y, GLM_ERR_INVALID, "glm_gemm_bf16_act: null pointer");
+    GLM_CHECK_ARG(M >= 0 && N > 0 && K > 0 && ldx >= K && ldy >= N && ldw >= K, GLM_ERR_INVALID,
+                  "glm_gemm_bf16_act: bad shape M=%ld N=%d K=%d ldx=%ld ldy=%ld", (long)M, N, K, (long)ldx, (long)ldy);
+    GLM_CHECK_ARG(act >= GLM_ACT_NONE && act <= GLM_ACT_SOFTCAP, GLM_ERR_INVALID, "glm_gemm_bf16_act: unknown activation %d", act);
+    GLM_CHECK_ARG(!out_f32 || (glm_aligned16(y) && ldy % 4 == 0), GLM_ERR_UNSUPPORTED, "glm_gemm_bf16_act: fp32 rows need 16-byte alignment");
+    GemmParams p;
+    memset(&p, 0, sizeof(p));
+    p.x = (const bf16_t*)x; p.ldx = ldx;
+    p.w = (const bf16_t*)w; p.ldw = ldw;
+    p.bias = (const bf16_t*)bias;
+    p.y = (bf16_t*)y; p.ldy = ldy;  // (fp32 output: only the alignment checks look at y)
+    if (out_f32) p.yf = (float*)y;
+    p.R = M; p.N = N; p.K = K; p.G = 1;
+    p.act = GlmAct{act, act_a, act_b};
+    if (M <= 0) return GLM_OK;
+    if (M == 1 && tinym_enabled()) {
+        const int rc = glm_launch_gemm_tinym(GEMM_PLAIN, p, 1, glm_s(stream));
+        if (rc != GLM_ERR_UNSUPPORTED) return rc;
+    }
+    if (M >= LARGEM_MIN_AVG_ROWS) return glm_launch_gemm_largem(GEMM_ACT, p, glm_s(stream));
+    return glm_launch_gemm_smallm(GEMM_PLAIN, p, glm_s(stream));
 }
 
 extern "C" int glm_gemm_qkv_rope_store(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* bias, int64_t T,

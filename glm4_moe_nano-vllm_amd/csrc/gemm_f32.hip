@@ -1,0 +1,86 @@
+// gemm_f32.hip — y = act(x · W^T + bias) in true fp32 (vector FMAs, no reduced-precision matrix mode), optionally batched.
+// gfx950 only.  For models that are served in 32-bit: exactness first; a 64 x 64 tile per workgroup, 4 x 4 outputs per
+// thread, 16-wide K slabs through LDS.  Every output is one fixed-order sum over K, whatever the number of rows.
+#include "gemm_internal.h"
+
+namespace {
+
+constexpr int GF_B = 64, GF_K = 16, GF_PAD = 4;
+
+struct GemmF32Args {
+    const float *x, *w, *bias;
+    float* y;
+    int64_t ldx, xb, ldw, wb, ldy, yb, M;
+    int N, K;
+    GlmAct act;
+};
+
+__global__ __launch_bounds__(256) void gemm_f32_kernel(const GemmF32Args a) {
+    __shared__ __attribute__((aligned(16))) float sx[GF_K][GF_B + GF_PAD], sw[GF_K][GF_B + GF_PAD];
+    const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4;
+    const int64_t m0 = (int64_t)blockIdx.y * GF_B;
+    const int n0 = blockIdx.x * GF_B;
+    const float* x = a.x + blockIdx.z * a.xb;
+    const float* w = a.w + blockIdx.z * a.wb;
+    float acc[4][4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] = 0.f;
+    const int lr = tid >> 2, lk = (tid & 3) * 4;  // row and K offset this thread stages
+    for (int k0 = 0; k0 < a.K; k0 += GF_K) {
+        f32x4_t vx = {0.f, 0.f, 0.f, 0.f}, vw = {0.f, 0.f, 0.f, 0.f};
+        if (k0 + lk < a.K) {  // K is a multiple of 4
+            if (m0 + lr < a.M) vx = *reinterpret_cast<const f32x4_t*>(x + (m0 + lr) * a.ldx + k0 + lk);
+            if (n0 + lr < a.N) vw = *reinterpret_cast<const f32x4_t*>(w + (int64_t)(n0 + lr) * a.ldw + k0 + lk);
+        }
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            sx[lk + i][lr] = vx[i];
+            sw[lk + i][lr] = vw[i];
+        }
+        __syncthreads();
+#pragma unroll
+        for (int k = 0; k < GF_K; ++k) {
+            const f32x4_t xv = *reinterpret_cast<const f32x4_t*>(&sx[k][ty * 4]);
+            const f32x4_t wv = *reinterpret_cast<const f32x4_t*>(&sw[k][tx * 4]);
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) acc[i][j] = fmaf(xv[i], wv[j], acc[i][j]);
+        }
+    }
+    float* y = a.y + blockIdx.z * a.yb;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int64_t m = m0 + ty * 4 + i;
+        if (m >= a.M) continue;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int n = n0 + tx * 4 + j;
+            if (n >= a.N) continue;
+            float v = acc[i][j];
+            if (a.bias) v += a.bias[n];
+            y[m * a.ldy + n] = glm_act_precise(a.act, v);
+        }
+    }
+}
+
+}  // namespace
+
+extern "C" int glm_gemm_f32(const float* x, int64_t ldx, int64_t xb, const float* w, int64_t ldw, int64_t wb, const float* bias, float* y,
+                            int64_t ldy, int64_t yb, int64_t M, int N, int K, int batch, int act, float act_a, float act_b, glm_stream_t stream) {
+    GLM_CHECK_ARG(x && w && y && M >= 0 && N > 0 && K > 0 && batch > 0 && ldx >= K && ldw >= K && ldy >= N, GLM_ERR_INVALID,
+                  "glm_gemm_f32: bad shape M=%ld N=%d K=%d", (long)M, N, K);
+    GLM_CHECK_ARG(K % 4 == 0 && ldx % 4 == 0 && ldw % 4 == 0 && xb % 4 == 0 && wb % 4 == 0 && glm_aligned16(x) && glm_aligned16(w), GLM_ERR_UNSUPPORTED,
+                  "glm_gemm_f32: needs K, ldx, ldw, batch strides %% 4 == 0 and 16-byte aligned operands (K=%d)", K);
+    GLM_CHECK_ARG(act >= GLM_ACT_NONE && act <= GLM_ACT_SOFTCAP, GLM_ERR_INVALID, "glm_gemm_f32: unknown activation %d", act);
+    const int64_t gy = (M + GF_B - 1) / GF_B;
+    GLM_CHECK_ARG(gy <= 65535 && batch <= 65535, GLM_ERR_UNSUPPORTED, "glm_gemm_f32: too many rows (%ld)", (long)M);
+    if (M == 0) return GLM_OK;
+    GemmF32Args a = {x, w, bias, y, ldx, xb, ldw, wb, ldy, yb, M, N, K, {act, act_a, act_b}};
+    hipLaunchKernelGGL(gemm_f32_kernel, dim3((unsigned)((N + GF_B - 1) / GF_B), (unsigned)gy, (unsigned)batch), dim3(256), 0, glm_s(stream), a);
+    GLM_CHECK_LAUNCH("glm_gemm_f32");
+    return GLM_OK;
+}

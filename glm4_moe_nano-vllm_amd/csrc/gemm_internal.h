@@ -6,7 +6,34 @@ enum GemmMode : int {
     GEMM_PLAIN = 0,   // y[r,n] = bf16(acc + bias[n])                              (a5, a10)
     GEMM_GATEUP = 1,  // act[r,i] = bf16(bf16(silu(bf16(g))) * bf16(u)), W rows gate|up  (a13)
     GEMM_DOWN = 2,    // y[r,n] = bf16(bf16(acc) * scale[r]) for groups < n_scaled    (a12/a13)
+    GEMM_ACT = 3,     // gemm_largem only: GEMM_PLAIN followed by p.act and / or an fp32 output row (p.yf) — its own instantiation,
+                      // so that the plain kernel's epilogue stays as it is; the decode bodies take p.act / p.yf in GEMM_PLAIN
 };
+
+// activation on the fp32 accumulator of a projection (after the bias)
+enum : int { GLM_ACT_NONE = GLM_EPI_NONE, GLM_ACT_XIELU = GLM_EPI_XIELU, GLM_ACT_SOFTCAP = GLM_EPI_SOFTCAP };
+struct GlmAct {
+    int kind;
+    float a, b;
+};
+// z > 0: a z^2 + z / 2;  z <= 0: b (exp(z) - 1 - z) + z / 2.   The fp32 form, for fp32 outputs.
+__device__ __forceinline__ float glm_act_precise(const GlmAct& t, float z) {
+    if (t.kind == GLM_ACT_XIELU) return z > 0.f ? t.a * z * z + 0.5f * z : t.b * (expm1f(z) - z) + 0.5f * z;
+    if (t.kind == GLM_ACT_SOFTCAP) return t.a * tanhf(z / t.a);
+    return z;
+}
+// ... for outputs that are rounded to bf16 right away: exp on the hardware exp2 unit, its absolute error (1e-7) far below the
+// rounding of the result; a series where exp(z) - 1 - z cancels
+__device__ __forceinline__ float glm_act_fast(const GlmAct& t, float z) {
+    if (t.kind == GLM_ACT_XIELU) {
+        const float zn = fminf(z, 0.f);
+        const float far = __builtin_amdgcn_exp2f(1.4426950408889634f * zn) - 1.0f - zn;
+        const float near = zn * zn * (0.5f + zn * (1.0f / 6.0f + zn * (1.0f / 24.0f)));
+        const float e = zn > -0.0625f ? near : far;
+        return z > 0.f ? t.a * z * z + 0.5f * z : t.b * e + 0.5f * z;
+    }
+    return glm_act_precise(t, z);
+}
 
 struct GemmParams {
     const bf16_t* x;      // activations, row r_src at x + r_src*ldx, K contiguous
@@ -53,6 +80,9 @@ struct GemmParams {
     const float* qkv_cs;         // cos_sin_cache [max_pos, 64] = cos(32) | sin(32)
     int64_t qkv_nslots;
     int qkv_nh, qkv_nkv;
+    // dense projections: activation in the epilogue; yf != nullptr: fp32 output rows at yf + r*ldy instead of y
+    GlmAct act;
+    float* yf;
 };
 
 // weight-streaming kernels for few rows per group (decode); returns GLM_* code

@@ -138,6 +138,19 @@ __device__ __forceinline__ void smallm_epilogue(const GemmParams& p, f32x4_t (&a
                     if (scaled) a = rbf(a) * sc;
                     o[r] = a;
                 }
+                if (MODE == GEMM_PLAIN) {
+                    if (p.yf != nullptr) {
+                        f32x4_t v;
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) v[r] = glm_act_precise(p.act, o[r]);
+                        *reinterpret_cast<f32x4_t*>(p.yf + (int64_t)(m0 + row) * p.ldy + n) = v;
+                        continue;
+                    }
+                    if (p.act.kind != GLM_ACT_NONE) {
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) o[r] = glm_act_fast(p.act, o[r]);
+                    }
+                }
                 u32x2_t v = {pack2bf(o[0], o[1]), pack2bf(o[2], o[3])};
                 *reinterpret_cast<u32x2_t*>(yrow + n) = v;
             }

@@ -492,6 +492,17 @@ __global__ __launch_bounds__(TM_NT) void gemm_tinym_kernel(const TinyParams tp) 
                     if (scaled) a = rbf(a) * sc;
                     v[r] = a;
                 }
+                if (MODE == GEMM_PLAIN && !TAIL) {
+                    if (p.yf != nullptr) {
+#pragma unroll
+                        for (int r = 0; r < RPW; ++r) p.yf[row * p.ldy + t.ncol + r] = glm_act_precise(p.act, v[r]);
+                        continue;
+                    }
+                    if (p.act.kind != GLM_ACT_NONE) {
+#pragma unroll
+                        for (int r = 0; r < RPW; ++r) v[r] = glm_act_fast(p.act, v[r]);
+                    }
+                }
                 if constexpr (RPW == 4) {
                     const u32x2_t o2 = u32x2_t{pack2bf(v[0], v[1]), pack2bf(v[2], v[3])};
                     if (TAIL)  // read by another workgroup of this launch: write-through (Guideline 16 R1)

@@ -1,0 +1,673 @@
+// latent_attn.hip — attention over a paged cache of latent rows (one row c of `rank` values per token, shared by all heads),
+// with a sliding window and a learned sink per head, in the ABSORBED form: with k = W_uk c and v = W_uv c,
+//
+//     q . k = (W_uk^T q) . c          sum_j p_j v_j = W_uv (sum_j p_j c_j)
+//
+// so a query row attends directly over the cached latents, every row of which is read once for all heads.  The form for few
+// query rows per sequence (decode, short portions); long portions expand k and v (window_attn.hip).  gfx950 only.
+//
+//   latent_prepare   one launch: latent norm + cache store of the step's tokens, and q' = W_uk^T q of the absorbed rows
+//   latent_attn      split-KV flash loop over the pages; rows are (token, head) pairs; fp32 scores and softmax
+//   latent_up        merge of the KV splits (with the sink's mass) and out = W_uv ctx
+//
+// Roofline of latent_attn at decode: HBM — window * rank * 2 bytes per sequence, read once.  4 waves share every 32-key tile
+// through a ring of LDS-DMA stages (two tiles in flight): S^T = C . Q^T with the K dimension split over wave pairs and the keys
+// over the pairs' members, partial scores exchanged through LDS, the softmax evaluated redundantly by every wave, and
+// O^T += C^T . P^T with the latent dimension split over the waves.  One LDS image serves both products: chunk ^ swz(key) with
+// swz(key) = (key & 3) << 1 | (key >> 2) & 1 is conflict-free for the ds_read_b128 row reads and for the transposed
+// ds_read_b64_tr_b16 reads.  Keys outside the sequence's range and padding columns are fetched from a page of zeros, never
+// from unused cache memory (whatever lies there would turn a zero weight into a NaN).
+#include "common.h"
+#include "attn_lds.h"
+
+namespace {
+
+constexpr float LOG2E = 1.4426950408889634f;
+constexpr int LA_BT = 2048;  // block-table entries a workgroup caches in LDS
+
+__device__ const u32x4_t la_zero_page[4] = {};
+
+// ---------------------------------------------------------------------------------------------------------------------------
+struct PrepArgs {
+    const void* qc;        // [T, ldq] projection rows: q heads at h*dimp, raw latent at c_off
+    int64_t ldq;
+    int c_off;
+    int64_t T, Ta;         // rows; rows [0, Ta) are absorbed
+    int H, dimp, rank, rp; // rp = rank rounded up to 8
+    const float* norm_w;   // [rp]
+    float eps;
+    const int32_t* slots;  // [T] cache row of the token, < 0: none
+    void* cache;           // [n_slots, rp]
+    int64_t n_slots;
+    const int32_t* crow;   // [T] row of c_out, < 0: none (nullptr: no c_out)
+    void* c_out;           // [n_crows, rp]
+    int64_t n_crows;
+    const bf16_t* wukt;    // [H, rp, dimp]
+    bf16_t* qa;            // [Ta, H, rp]
+};
+
+template <typename E>
+__device__ __forceinline__ float la_ld(const void* p, int64_t i) {
+    if constexpr (sizeof(E) == 2) return bf2f(reinterpret_cast<const bf16_t*>(p)[i]);
+    else return reinterpret_cast<const float*>(p)[i];
+}
+template <typename E>
+__device__ __forceinline__ void la_st(void* p, int64_t i, float v) {
+    if constexpr (sizeof(E) == 2) reinterpret_cast<bf16_t*>(p)[i] = f2bf(v);
+    else reinterpret_cast<float*>(p)[i] = v;
+}
+
+// latent norm of one token by one wave
+template <typename E>
+__device__ void latent_norm_row(const PrepArgs& a, int64_t t, int lane) {
+    const int64_t base = t * a.ldq + a.c_off;
+    float s = 0.f;
+    for (int i = lane; i < a.rank; i += 64) {
+        const float v = la_ld<E>(a.qc, base + i);
+        s += v * v;
+    }
+    const float r = 1.0f / sqrtf(wave_sum(s) / (float)a.rank + a.eps);
+    const int64_t slot = a.slots[t];
+    const bool st = slot >= 0 && slot < a.n_slots;
+    int64_t row = a.crow ? a.crow[t] : -1;
+    if (row >= a.n_crows) row = -1;
+    for (int i = lane; i < a.rp; i += 64) {
+        const float v = i < a.rank ? la_ld<E>(a.qc, base + i) * r * a.norm_w[i] : 0.f;
+        if (st) la_st<E>(a.cache, slot * a.rp + i, v);
+        if (row >= 0) la_st<E>(a.c_out, row * a.rp + i, v);
+    }
+}
+
+constexpr int PREP_TT = 4;  // 16-token tiles per absorb workgroup
+
+__global__ __launch_bounds__(256) void latent_prepare_kernel(const PrepArgs a, int n_absorb) {
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+    if ((int)blockIdx.x >= n_absorb) {
+        const int64_t t = (int64_t)((int)blockIdx.x - n_absorb) * 4 + wid;
+        if (t < a.T) latent_norm_row<bf16_t>(a, t, lane);
+        return;
+    }
+    // q'[t, h, r] = sum_d W_uk[h, d, r] q[t, h, d]: 64 latent rows x 64 tokens per workgroup, 16 x 64 per wave
+    const int nr = (a.rp + 63) / 64;
+    int b = blockIdx.x;
+    const int rb = b % nr;
+    b /= nr;
+    const int h = b % a.H;
+    const int64_t t0 = (int64_t)(b / a.H) * (16 * PREP_TT);
+    const int c = lane & 15, g = lane >> 4;
+    const int r0 = rb * 64 + wid * 16;
+    const int ar = r0 + c;  // A row of this lane
+    const bf16_t* q = reinterpret_cast<const bf16_t*>(a.qc);
+    f32x4_t acc[PREP_TT];
+#pragma unroll
+    for (int i = 0; i < PREP_TT; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    for (int k = 8 * g; k < ((a.dimp + 31) & ~31); k += 32) {
+        u32x4_t av = {0, 0, 0, 0};
+        if (k < a.dimp && ar < a.rp) av = *reinterpret_cast<const u32x4_t*>(a.wukt + ((int64_t)h * a.rp + ar) * a.dimp + k);
+#pragma unroll
+        for (int i = 0; i < PREP_TT; ++i) {
+            const int64_t t = t0 + 16 * i + c;
+            u32x4_t bv = {0, 0, 0, 0};
+            if (k < a.dimp && t < a.Ta) bv = *reinterpret_cast<const u32x4_t*>(q + t * a.ldq + (int64_t)h * a.dimp + k);
+            acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, av), __builtin_bit_cast(bf16x8_t, bv), acc[i], 0, 0, 0);
+        }
+    }
+    const int r = r0 + 4 * g;
+    if (r < a.rp) {
+#pragma unroll
+        for (int i = 0; i < PREP_TT; ++i) {
+            const int64_t t = t0 + 16 * i + c;
+            if (t < a.Ta)
+                *reinterpret_cast<u32x2_t*>(a.qa + (t * a.H + h) * a.rp + r) = u32x2_t{pack2bf(acc[i][0], acc[i][1]), pack2bf(acc[i][2], acc[i][3])};
+        }
+    }
+}
+
+__global__ __launch_bounds__(256) void latent_norm_f32_kernel(const PrepArgs a) {
+    const int64_t t = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (t < a.T) latent_norm_row<float>(a, t, threadIdx.x & 63);
+}
+
+// cache rows -> contiguous rows (the history in front of a long portion): one wave per row, 16-byte chunks
+__global__ __launch_bounds__(256) void latent_gather_kernel(const uint8_t* cache, int64_t n_slots, const int32_t* slots, const int32_t* rows, int64_t n,
+                                                            uint8_t* out, int64_t n_rows, int row_bytes) {
+    const int64_t i = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (i >= n) return;
+    const int64_t s = slots[i], r = rows[i];
+    if (s < 0 || s >= n_slots || r < 0 || r >= n_rows) return;
+    for (int o = (threadIdx.x & 63) * 16; o < row_bytes; o += 1024)
+        *reinterpret_cast<u32x4_t*>(out + r * row_bytes + o) = *reinterpret_cast<const u32x4_t*>(cache + s * row_bytes + o);
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------
+struct AttnArgs {
+    const void* qa;           // [Ta, H, rp]
+    const void* cache;        // [n_blocks, block_size, rp]
+    const int32_t *tile_tok, *tile_n;  // [n_tiles] first row and row count of a tile (one sequence)
+    const int32_t *pos, *seq_of;       // [T]
+    const int32_t* bt;        // [S, bt_stride]
+    int64_t bt_stride;
+    int64_t n_blocks;
+    int bs_shift;             // log2(block size)
+    int64_t Ta;
+    int H, rank, rp, window;
+    float scale;
+    const float* sink;        // [H]
+    int n_tiles, hb, n_hg, tq, nsplit;  // heads per workgroup, head groups, tokens per tile (at most)
+    bf16_t* ctx;              // nsplit == 1: [Ta, H, rp] normalised context
+    float* part_o;            // nsplit > 1: [Ta * H, nsplit, rp] unnormalised
+    float* part_ml;           // [Ta * H, nsplit, 2] running maximum (log2 units), mass
+};
+
+template <int NCT, int MT>
+__global__ __launch_bounds__(256, 1) void latent_attn_kernel(const AttnArgs a) {
+    constexpr int RPAD = NCT * 64, ROWB = RPAD * 2, TILEB = 32 * ROWB, CPR = RPAD / 8;
+    constexpr int NST = 3 * TILEB <= 112 * 1024 ? 3 : 2;
+    constexpr int SLAB = 2 * MT * 2 * 1024;
+    constexpr int FG = NCT < 8 ? NCT : 8;  // fragments per request group
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int c = lane & 15, g = lane >> 4;
+    const int kt = w & 1, kh = w >> 1;  // key half and K half of this wave's scores
+    int id = blockIdx.x;
+    const int split = id % a.nsplit;
+    id /= a.nsplit;
+    const int hg = id % a.n_hg, tile = id / a.n_hg;
+    const int h0 = hg * a.hb, hb = min(a.hb, a.H - h0);
+    const int tok0 = a.tile_tok[tile];
+    const int ntok = min(a.tile_n[tile], a.tq);
+    if (tok0 < 0 || tok0 >= a.Ta || ntok <= 0) return;
+    const int p0 = a.pos[tok0], p1 = p0 + ntok - 1, seq = a.seq_of[tok0];
+    const int nrows = ntok * hb;
+    const int lo = max(0, p0 - a.window + 1);
+    const int ntile = p0 < 0 ? 0 : (p1 - lo + 32) >> 5;  // 32-key tiles of the whole range
+    const int per = (ntile + a.nsplit - 1) / a.nsplit;
+    const int t0 = split * per, t1 = min(t0 + per, ntile), n = t1 - t0;
+    if (n <= 0) {  // an empty split (or an unused row): no mass
+        for (int r = tid; r < nrows; r += 256) {
+            const int64_t grow = (int64_t)(tok0 + r / hb) * a.H + h0 + r % hb;
+            if (a.nsplit > 1) {
+                a.part_ml[(grow * a.nsplit + split) * 2] = -INFINITY;
+                a.part_ml[(grow * a.nsplit + split) * 2 + 1] = 0.f;
+            } else {
+                for (int d = 0; d < a.rp; ++d) a.ctx[grow * a.rp + d] = 0;
+            }
+        }
+        return;
+    }
+    const int bs = 1 << a.bs_shift, bmask = bs - 1;
+    const int klo = lo + t0 * 32;                 // first key of this split
+    const int khi = min(p1, lo + t1 * 32 - 1);    // last key of this split
+    const int blk0 = klo >> a.bs_shift, nblk = (khi >> a.bs_shift) - blk0 + 1;
+    int* bt_lds = reinterpret_cast<int*>(smem + NST * TILEB + SLAB);
+    for (int i = tid; i < min(nblk, LA_BT); i += 256) {
+        const int64_t b = a.bt[(int64_t)seq * a.bt_stride + blk0 + i];
+        bt_lds[i] = (int)min(max(b, (int64_t)0), a.n_blocks - 1);
+    }
+    // query rows of this lane (one per row tile) and their fragments: K step 2 i + kh of wave pair kh
+    int rpos[MT];
+    int64_t grow[MT];
+    u32x4_t qf[MT][NCT];
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+        const int r = 16 * m + c;
+        const bool ok = r < nrows;
+        const int to = ok ? r / hb : 0, hd = ok ? r % hb : 0;
+        rpos[m] = ok ? p0 + to : -1;
+        grow[m] = (int64_t)(tok0 + to) * a.H + h0 + hd;
+        const bf16_t* q = reinterpret_cast<const bf16_t*>(a.qa) + grow[m] * a.rp;
+#pragma unroll
+        for (int i = 0; i < NCT; ++i) {
+            const int k = 32 * (2 * i + kh) + 8 * g;
+            qf[m][i] = u32x4_t{0, 0, 0, 0};
+            if (ok && k < a.rp) qf[m][i] = *reinterpret_cast<const u32x4_t*>(q + k);
+        }
+    }
+    __syncthreads();
+    const unsigned base = lds_addr(smem), slab = base + NST * TILEB, bt_addr = slab + SLAB;
+    const bf16_t* cache = reinterpret_cast<const bf16_t*>(a.cache);
+    auto issue = [&](int it) {
+        const int k0 = klo + it * 32;
+        int b0, b1;
+        {
+            const int i0 = (k0 >> a.bs_shift) - blk0, i1 = min(i0 + 1, nblk - 1);
+            asm volatile("ds_read_b32 %0, %2\n\tds_read_b32 %1, %3\n\ts_waitcnt lgkmcnt(0)"
+                         : "=&v"(b0), "=&v"(b1) : "v"(bt_addr + i0 * 4), "v"(bt_addr + i1 * 4) : "memory");
+            b0 = __builtin_amdgcn_readfirstlane(b0);
+            b1 = __builtin_amdgcn_readfirstlane(b1);
+        }
+        const int first = k0 >> a.bs_shift;
+        char* st = smem + (it % NST) * TILEB;
+#pragma unroll
+        for (int i = 0; i < NCT; ++i) {
+            const int q = (w * NCT + i) * 64 + lane;
+            const int row = q / CPR, ch = (q % CPR) ^ attn_swz(row);
+            const int key = k0 + row;
+            const int blk = (key >> a.bs_shift) == first ? b0 : b1;
+            const bf16_t* src = cache + (((int64_t)blk << a.bs_shift) + (key & bmask)) * a.rp + ch * 8;
+            const void* s = (key <= khi && ch * 8 < a.rp) ? (const void*)src : (const void*)la_zero_page;
+            lds_dma16(s, st + (w * NCT + i) * 1024);
+        }
+    };
+    f32x4_t acc[MT][NCT];
+    float m_run[MT], l_run[MT];
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+        m_run[m] = -INFINITY;
+        l_run[m] = 0.f;
+#pragma unroll
+        for (int d = 0; d < NCT; ++d) acc[m][d] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    }
+    // loop-invariant LDS offsets of this lane's fragment reads
+    const unsigned k_rel = (16 * kt + c) * ROWB + (((4 * kh + g) ^ attn_swz(c)) << 4);
+    const int qq = (lane >> 2) & 3, pp = lane & 3, vrow = 4 * g + qq;
+    const unsigned v_rel = vrow * ROWB + (((2 * w + (pp >> 1)) ^ attn_swz(vrow)) << 4) + ((pp & 1) << 3);
+    const float sc = a.scale * LOG2E;
+#pragma unroll
+    for (int m = 0; m < MT; ++m)
+#pragma unroll
+        for (int i = 0; i < NCT; ++i) asm volatile("" : "+v"(qf[m][i]));  // landed before the ring starts counting vmcnt
+#pragma unroll
+    for (int i = 0; i < NST - 1; ++i)
+        if (i < n) issue(i);
+    for (int it = 0; it < n; ++it) {
+        if (NST == 3 && it + 1 < n) wait_vm<NCT>();
+        else wait_vm<0>();
+        __builtin_amdgcn_s_barrier();
+        if (it + NST - 1 < n) issue(it + NST - 1);
+        const unsigned st = base + (it % NST) * TILEB;
+        // ---- partial scores: keys 16 kt .. of the tile, K steps of parity kh ----
+        f32x4_t s[MT];
+#pragma unroll
+        for (int m = 0; m < MT; ++m) s[m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        static_for<(NCT + FG - 1) / FG>([&](auto G) {
+            constexpr int i0 = decltype(G)::value * FG, ni = NCT - i0 < FG ? NCT - i0 : FG;
+            u32x4_t kf[FG];
+            static_for<ni>([&](auto I) { constexpr int i = decltype(I)::value; lds_read_b128<(i0 + i) * 128>(kf[i], st + k_rel); });
+            wait_lds();
+#pragma unroll
+            for (int i = 0; i < ni; ++i) asm volatile("" : "+v"(kf[i]));
+#pragma unroll
+            for (int i = 0; i < ni; ++i)
+#pragma unroll
+                for (int m = 0; m < MT; ++m)
+                    s[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, kf[i]), __builtin_bit_cast(bf16x8_t, qf[m][i0 + i]), s[m], 0, 0, 0);
+        });
+#pragma unroll
+        for (int m = 0; m < MT; ++m) {
+            f32x4_t v;  // (an ordinary vector instruction between the matrix pipe's result and the store below)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) v[r] = s[m][r] * sc;
+            asm volatile("ds_write_b128 %0, %1" ::"v"(slab + ((kh * MT + m) * 2 + kt) * 1024 + lane * 16), "v"(v) : "memory");
+        }
+        wait_lds();
+        __builtin_amdgcn_s_barrier();
+        // ---- online softmax of row c of every row tile: this lane holds keys 16 t + 4 g + r ----
+        const int kbase = klo + it * 32 + 4 * g;
+        bf16x8_t pf[MT];
+#pragma unroll
+        for (int m = 0; m < MT; ++m) {
+            f32x4_t sv[2][2];
+#pragma unroll
+            for (int t = 0; t < 2; ++t)
+#pragma unroll
+                for (int k2 = 0; k2 < 2; ++k2)
+                    asm volatile("ds_read_b128 %0, %1" : "=v"(sv[t][k2]) : "v"(slab + ((k2 * MT + m) * 2 + t) * 1024 + lane * 16));
+            wait_lds();
+            asm volatile("" : "+v"(sv[0][0]), "+v"(sv[0][1]), "+v"(sv[1][0]), "+v"(sv[1][1]));
+            float mx = -INFINITY, x[2][4];
+#pragma unroll
+            for (int t = 0; t < 2; ++t)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const int d = rpos[m] - (kbase + 16 * t + r);
+                    const bool vis = d >= 0 && d < a.window && kbase + 16 * t + r <= khi;
+                    x[t][r] = vis ? sv[t][0][r] + sv[t][1][r] : -INFINITY;
+                    mx = fmaxf(mx, x[t][r]);
+                }
+            mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+            mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+            const float m_new = fmaxf(m_run[m], mx);
+            const float m_use = m_new == -INFINITY ? 0.f : m_new;
+            if (__any(m_new > m_run[m])) {
+                const float alpha = __builtin_amdgcn_exp2f(m_run[m] - m_use);
+                l_run[m] *= alpha;
+#pragma unroll
+                for (int d = 0; d < NCT; ++d) acc[m][d] *= alpha;
+            }
+            m_run[m] = m_new;
+#pragma unroll
+            for (int t = 0; t < 2; ++t)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const float p = __builtin_amdgcn_exp2f(x[t][r] - m_use);
+                    l_run[m] += p;
+                    pf[m][4 * t + r] = (__bf16)p;
+                }
+        }
+        // ---- O^T += C^T . P^T on this wave's latent columns ----
+        static_for<(NCT + FG - 1) / FG>([&](auto G) {
+            constexpr int d0 = decltype(G)::value * FG, nd = NCT - d0 < FG ? NCT - d0 : FG;
+            u32x2_t vf[FG][2];
+            static_for<nd>([&](auto I) {
+                constexpr int d = decltype(I)::value;
+                lds_read_tr16_b64<(d0 + d) * 128>(vf[d][0], st + v_rel);
+                lds_read_tr16_b64<(d0 + d) * 128>(vf[d][1], st + v_rel + 16 * ROWB);
+            });
+            wait_lds();
+#pragma unroll
+            for (int d = 0; d < nd; ++d) asm volatile("" : "+v"(vf[d][0]), "+v"(vf[d][1]));
+#pragma unroll
+            for (int d = 0; d < nd; ++d) {
+                const u32x4_t vv = {vf[d][0][0], vf[d][0][1], vf[d][1][0], vf[d][1][1]};
+#pragma unroll
+                for (int m = 0; m < MT; ++m)
+                    acc[m][d0 + d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, vv), pf[m], acc[m][d0 + d], 0, 0, 0);
+            }
+        });
+    }
+    // ---- rows out: lane holds dims 64 d + 16 w + 4 g .. of row c ----
+#pragma unroll
+    for (int m = 0; m < MT; ++m) {
+        float l = l_run[m];
+        l += __shfl_xor(l, 16, 64);
+        l += __shfl_xor(l, 32, 64);
+        const bool ok = 16 * m + c < nrows;
+        if (!ok) continue;
+        if (a.nsplit == 1) {
+            const float sk = a.sink[grow[m] % a.H] * LOG2E;
+            const float M = fmaxf(m_run[m], sk);
+            const float f = __builtin_amdgcn_exp2f(m_run[m] - M);
+            const float inv = f / (l * f + __builtin_amdgcn_exp2f(sk - M));
+#pragma unroll
+            for (int d = 0; d < NCT; ++d) {
+                const int dim = 64 * d + 16 * w + 4 * g;
+                if (dim < a.rp)
+                    *reinterpret_cast<u32x2_t*>(a.ctx + grow[m] * a.rp + dim) =
+                        u32x2_t{pack2bf(acc[m][d][0] * inv, acc[m][d][1] * inv), pack2bf(acc[m][d][2] * inv, acc[m][d][3] * inv)};
+            }
+        } else {
+            const int64_t pr = grow[m] * a.nsplit + split;
+#pragma unroll
+            for (int d = 0; d < NCT; ++d) {
+                const int dim = 64 * d + 16 * w + 4 * g;
+                if (dim < a.rp) *reinterpret_cast<f32x4_t*>(a.part_o + pr * a.rp + dim) = acc[m][d];
+            }
+            if (w == 0 && g == 0) {
+                a.part_ml[pr * 2] = m_run[m];
+                a.part_ml[pr * 2 + 1] = l;
+            }
+        }
+    }
+}
+
+template <int NCT, int MT>
+int launch_latent_attn(const AttnArgs& a, hipStream_t st) {
+    constexpr int TILEB = 32 * NCT * 128;
+    constexpr int NST = 3 * TILEB <= 112 * 1024 ? 3 : 2;
+    constexpr int LDS = NST * TILEB + 2 * MT * 2 * 1024 + LA_BT * 4;
+    static_assert(LDS <= 160 * 1024, "LDS of a CU");
+    auto kern = latent_attn_kernel<NCT, MT>;
+    GLM_SET_MAX_LDS(kern, LDS, "glm_latent_attn");
+    const int64_t grid = (int64_t)a.n_tiles * a.n_hg * a.nsplit;
+    GLM_CHECK_ARG(grid < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_latent_attn: grid too large");
+    hipLaunchKernelGGL(kern, dim3((unsigned)grid), dim3(256), LDS, st, a);
+    GLM_CHECK_LAUNCH("glm_latent_attn");
+    return GLM_OK;
+}
+
+template <int NCT>
+int launch_latent_attn_mt(const AttnArgs& a, int mt, hipStream_t st) {
+    if (mt == 1) return launch_latent_attn<NCT, 1>(a, st);
+    if constexpr (NCT > 6) return launch_latent_attn<NCT, 2>(a, st);  // (four row tiles would not fit the registers)
+    else return mt == 2 ? launch_latent_attn<NCT, 2>(a, st) : launch_latent_attn<NCT, 4>(a, st);
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------
+// fp32: one wave per (token, head), 64 keys per step (one per lane), then the latent dimensions over the lanes
+constexpr int LF_MAXR = 2048;
+
+template <int NV>  // latent values per lane
+__global__ __launch_bounds__(256) void latent_attn_f32_kernel(const AttnArgs a, float* ctx) {
+    extern __shared__ __attribute__((aligned(16))) float sq[];  // [4][rp]
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
+    const int64_t grow = (int64_t)blockIdx.x * 4 + wid;
+    const bool live = grow < a.Ta * a.H;
+    const int64_t t = live ? grow / a.H : 0;
+    const int h = live ? (int)(grow % a.H) : 0;
+    const int p = a.pos[t];
+    float* q = sq + wid * a.rp;
+    const float* qa = reinterpret_cast<const float*>(a.qa) + (t * a.H + h) * a.rp;
+    for (int i = lane; i < a.rp; i += 64) q[i] = qa[i];
+    __syncthreads();
+    if (!live) return;
+    float acc[NV];
+#pragma unroll
+    for (int i = 0; i < NV; ++i) acc[i] = 0.f;
+    float m = a.sink[h], l = 1.0f;  // the sink's mass is in from the start
+    const int lo = max(0, p - a.window + 1);
+    const int32_t* bt = a.bt + (int64_t)a.seq_of[t] * a.bt_stride;
+    const float* cache = reinterpret_cast<const float*>(a.cache);
+    const int bs = 1 << a.bs_shift;
+    for (int k0 = lo; k0 <= p; k0 += 64) {
+        const int key = k0 + lane;
+        int64_t row = 0;
+        float s = -INFINITY;
+        if (key <= p) {
+            const int64_t b = min(max((int64_t)bt[key >> a.bs_shift], (int64_t)0), a.n_blocks - 1);
+            row = (b << a.bs_shift) + (key & (bs - 1));
+            const float* cr = cache + row * a.rp;
+            float d = 0.f;
+            for (int i = 0; i < a.rp; i += 4) {
+                const f32x4_t cv = *reinterpret_cast<const f32x4_t*>(cr + i), qv = *reinterpret_cast<const f32x4_t*>(q + i);
+                d = fmaf(cv[0], qv[0], d);
+                d = fmaf(cv[1], qv[1], d);
+                d = fmaf(cv[2], qv[2], d);
+                d = fmaf(cv[3], qv[3], d);
+            }
+            s = d * a.scale;
+        }
+        const float m_new = fmaxf(m, wave_max(s));
+        const float alpha = expf(m - m_new);
+        const float pv = key <= p ? expf(s - m_new) : 0.f;
+        l = l * alpha + wave_sum(pv);
+#pragma unroll
+        for (int i = 0; i < NV; ++i) acc[i] *= alpha;
+        m = m_new;
+        const int nk = min(64, p - k0 + 1);
+        for (int k = 0; k < nk; ++k) {
+            const float pk = __shfl(pv, k, 64);
+            const int64_t rk = __shfl((long long)row, k, 64);
+#pragma unroll
+            for (int i = 0; i < NV; ++i)
+                if (lane + 64 * i < a.rp) acc[i] = fmaf(pk, cache[rk * a.rp + lane + 64 * i], acc[i]);
+        }
+    }
+    const float inv = 1.0f / l;
+#pragma unroll
+    for (int i = 0; i < NV; ++i)
+        if (lane + 64 * i < a.rp) ctx[grow * a.rp + lane + 64 * i] = p < 0 ? 0.f : acc[i] * inv;
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------
+struct UpArgs {
+    const bf16_t* ctx;
+    const float *part_o, *part_ml, *sink;
+    int nsplit;
+    const bf16_t* wuv;   // [H, vdimp, rp]
+    bf16_t* out;         // [T, ldo], head h at h*vdimp
+    int64_t ldo, Ta;
+    int H, vdimp, rp;
+};
+
+// out[t, h, :] = W_uv[h] . ctx[t, h, :]: 16 tokens and up to 64 value rows of one head per workgroup (16 rows per wave)
+__global__ __launch_bounds__(256) void latent_up_kernel(const UpArgs a) {
+    extern __shared__ __attribute__((aligned(16))) char smem_up[];
+    bf16_t* sx = reinterpret_cast<bf16_t*>(smem_up);  // [16][pitch]
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+    const int c = lane & 15, g = lane >> 4;
+    const int kp = (a.rp + 31) & ~31, pitch = kp + 8;
+    const int h = blockIdx.x % a.H, vc = blockIdx.x / a.H;
+    const int64_t t0 = (int64_t)blockIdx.y * 16;
+    const int nk4 = kp / 4;
+    __shared__ float s_f[16][64];  // per token and split: weight of the split's sums
+    if (a.nsplit > 1) {
+        if (tid < 16) {
+            const int64_t t = t0 + tid;
+            if (t < a.Ta) {
+                const float* ml = a.part_ml + (t * a.H + h) * a.nsplit * 2;
+                const float sk = a.sink[h] * LOG2E;
+                float M = sk, L = 0.f;
+                for (int s = 0; s < a.nsplit; ++s) M = fmaxf(M, ml[2 * s]);
+                for (int s = 0; s < a.nsplit; ++s) L += ml[2 * s + 1] > 0.f ? ml[2 * s + 1] * __builtin_amdgcn_exp2f(ml[2 * s] - M) : 0.f;
+                L += __builtin_amdgcn_exp2f(sk - M);
+                for (int s = 0; s < a.nsplit; ++s) s_f[tid][s] = ml[2 * s + 1] > 0.f ? __builtin_amdgcn_exp2f(ml[2 * s] - M) / L : 0.f;
+            }
+        }
+        __syncthreads();
+    }
+    for (int i = tid; i < 16 * nk4; i += 256) {
+        const int r = i / nk4, k = (i % nk4) * 4;
+        const int64_t t = t0 + r;
+        u32x2_t v = {0, 0};
+        if (t < a.Ta && k < a.rp) {
+            const int64_t grow = t * a.H + h;
+            if (a.nsplit == 1) {
+                v = *reinterpret_cast<const u32x2_t*>(a.ctx + grow * a.rp + k);
+            } else {
+                f32x4_t o = {0.f, 0.f, 0.f, 0.f};
+                for (int s = 0; s < a.nsplit; ++s) {
+                    const float f = s_f[r][s];
+                    if (f != 0.f) {  // an empty split's sums were never written
+                        const f32x4_t x = *reinterpret_cast<const f32x4_t*>(a.part_o + (grow * a.nsplit + s) * a.rp + k);
+#pragma unroll
+                        for (int j = 0; j < 4; ++j) o[j] += f * x[j];
+                    }
+                }
+                v = u32x2_t{pack2bf(o[0], o[1]), pack2bf(o[2], o[3])};
+            }
+        }
+        *reinterpret_cast<u32x2_t*>(sx + r * pitch + k) = v;
+    }
+    __syncthreads();
+    const int v0 = vc * 64 + wid * 16;
+    if (v0 >= a.vdimp) return;
+    const int ar = min(v0 + c, a.vdimp - 1);
+    f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+    const bf16_t* wr = a.wuv + ((int64_t)h * a.vdimp + ar) * a.rp;
+    for (int k = 8 * g; k < kp; k += 32) {
+        u32x4_t av = {0, 0, 0, 0};
+        if (k < a.rp) av = *reinterpret_cast<const u32x4_t*>(wr + k);
+        const u32x4_t bv = *reinterpret_cast<const u32x4_t*>(sx + c * pitch + k);
+        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, av), __builtin_bit_cast(bf16x8_t, bv), acc, 0, 0, 0);
+    }
+    const int v = v0 + 4 * g;
+    if (t0 + c < a.Ta && v < a.vdimp)
+        *reinterpret_cast<u32x2_t*>(a.out + (t0 + c) * a.ldo + (int64_t)h * a.vdimp + v) = u32x2_t{pack2bf(acc[0], acc[1]), pack2bf(acc[2], acc[3])};
+}
+
+int pick_nct(int rp) {
+    for (int n : {1, 2, 3, 4, 6, 8, 9, 16})
+        if (rp <= 64 * n) return n;
+    return -1;
+}
+
+}  // namespace
+
+extern "C" int glm_latent_prepare(const void* qc, int64_t ldq, int c_off, int64_t T, int64_t Ta, int H, int dimp, int rank, int rp, const float* norm_w,
+                                  float eps, const int32_t* slots, void* cache, int64_t n_slots, const int32_t* crow, void* c_out, int64_t n_crows,
+                                  const void* wukt, void* qa, int act_f32, glm_stream_t stream) {
+    GLM_CHECK_ARG(qc && norm_w && slots && cache && T >= 0 && Ta >= 0 && Ta <= T && H > 0 && rank > 0 && rp >= rank && rp % 8 == 0 && c_off % 8 == 0 &&
+                      ldq % 8 == 0 && ldq >= (int64_t)c_off + rank && dimp % 8 == 0 && c_off >= H * dimp && n_slots > 0 && (!crow || (c_out && n_crows > 0)),
+                  GLM_ERR_INVALID, "glm_latent_prepare: bad shape T=%ld Ta=%ld H=%d dimp=%d rank=%d", (long)T, (long)Ta, H, dimp, rank);
+    GLM_CHECK_ARG(act_f32 || Ta == 0 || (wukt && qa && glm_aligned16(wukt) && glm_aligned16(qc)), GLM_ERR_INVALID, "glm_latent_prepare: absorbed rows need W_uk^T and q'");
+    if (T == 0) return GLM_OK;
+    PrepArgs a = {qc, ldq, c_off, T, Ta, H, dimp, rank, rp, norm_w, eps, slots, cache, n_slots, crow, c_out, n_crows, (const bf16_t*)wukt, (bf16_t*)qa};
+    const int64_t nnorm = (T + 3) / 4;
+    if (act_f32) {
+        hipLaunchKernelGGL(latent_norm_f32_kernel, dim3((unsigned)nnorm), dim3(256), 0, glm_s(stream), a);
+    } else {
+        const int64_t nabs = Ta > 0 ? (int64_t)((rp + 63) / 64) * H * ((Ta + 16 * PREP_TT - 1) / (16 * PREP_TT)) : 0;
+        GLM_CHECK_ARG(nabs + nnorm < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_latent_prepare: grid too large");
+        hipLaunchKernelGGL(latent_prepare_kernel, dim3((unsigned)(nabs + nnorm)), dim3(256), 0, glm_s(stream), a, (int)nabs);
+    }
+    GLM_CHECK_LAUNCH("glm_latent_prepare");
+    return GLM_OK;
+}
+
+extern "C" int glm_latent_gather(const void* cache, int64_t n_slots, const int32_t* slots, const int32_t* rows, int64_t n, void* out, int64_t n_rows,
+                                 int row_bytes, glm_stream_t stream) {
+    GLM_CHECK_ARG(cache && slots && rows && out && n >= 0 && row_bytes > 0 && row_bytes % 16 == 0 && glm_aligned16(cache) && glm_aligned16(out), GLM_ERR_INVALID,
+                  "glm_latent_gather: bad arguments (n=%ld row_bytes=%d)", (long)n, row_bytes);
+    if (n == 0) return GLM_OK;
+    hipLaunchKernelGGL(latent_gather_kernel, dim3((unsigned)((n + 3) / 4)), dim3(256), 0, glm_s(stream), (const uint8_t*)cache, n_slots, slots, rows, n,
+                       (uint8_t*)out, n_rows, row_bytes);
+    GLM_CHECK_LAUNCH("glm_latent_gather");
+    return GLM_OK;
+}
+
+// rows per tile the absorbed kernel takes (16, 32 or 64) for a latent of rp columns
+extern "C" int glm_latent_attn_max_rows(int rp) {
+    const int n = pick_nct(rp);
+    return n < 0 ? 0 : (n > 6 ? 32 : 64);
+}
+
+extern "C" int glm_latent_attn(const void* qa, const void* cache, int64_t n_blocks, int block_size, const int32_t* tile_tok, const int32_t* tile_n,
+                               int n_tiles, int tokens_per_tile, const int32_t* pos, const int32_t* seq_of, const int32_t* block_tables, int64_t bt_stride,
+                               int64_t Ta, int H, int rank, int rp, int window, float scale, const float* sink, int nsplit, void* ctx, float* part_o,
+                               float* part_ml, int act_f32, glm_stream_t stream) {
+    GLM_CHECK_ARG(qa && cache && pos && seq_of && block_tables && sink && n_blocks > 0 && Ta >= 0 && H > 0 && rank > 0 && rp >= rank && rp % 8 == 0 && window > 0 &&
+                      bt_stride > 0, GLM_ERR_INVALID, "glm_latent_attn: bad shape Ta=%ld H=%d rp=%d window=%d", (long)Ta, H, rp, window);
+    int sh = 0;
+    while ((1 << sh) < block_size) ++sh;
+    GLM_CHECK_ARG((1 << sh) == block_size && block_size >= 32, GLM_ERR_UNSUPPORTED, "glm_latent_attn: block size %d is not a power of two >= 32", block_size);
+    if (Ta == 0) return GLM_OK;
+    AttnArgs a = {qa, cache, tile_tok, tile_n, pos, seq_of, block_tables, bt_stride, n_blocks, sh, Ta, H, rank, rp, window, scale, sink,
+                  n_tiles, 0, 0, tokens_per_tile, nsplit, (bf16_t*)ctx, part_o, part_ml};
+    hipStream_t st = glm_s(stream);
+    if (act_f32) {
+        GLM_CHECK_ARG(ctx && rp <= LF_MAXR, GLM_ERR_UNSUPPORTED, "glm_latent_attn(fp32): latent of %d columns", rp);
+        const int64_t nb = (Ta * H + 3) / 4;
+        const size_t lds = (size_t)4 * rp * 4;
+        if (rp <= 128) hipLaunchKernelGGL(latent_attn_f32_kernel<2>, dim3((unsigned)nb), dim3(256), lds, st, a, (float*)ctx);
+        else if (rp <= 512) hipLaunchKernelGGL(latent_attn_f32_kernel<8>, dim3((unsigned)nb), dim3(256), lds, st, a, (float*)ctx);
+        else hipLaunchKernelGGL(latent_attn_f32_kernel<32>, dim3((unsigned)nb), dim3(256), lds, st, a, (float*)ctx);
+        GLM_CHECK_LAUNCH("glm_latent_attn(fp32)");
+        return GLM_OK;
+    }
+    GLM_CHECK_ARG(tile_tok && tile_n && n_tiles > 0 && tokens_per_tile > 0 && nsplit >= 1 && nsplit <= 64, GLM_ERR_INVALID, "glm_latent_attn: bad tiles");
+    GLM_CHECK_ARG(nsplit > 1 ? (part_o && part_ml) : ctx != nullptr, GLM_ERR_INVALID, "glm_latent_attn: no output for %d splits", nsplit);
+    const int nct = pick_nct(rp), maxrows = glm_latent_attn_max_rows(rp);
+    GLM_CHECK_ARG(nct > 0, GLM_ERR_UNSUPPORTED, "glm_latent_attn: latent of %d columns", rp);
+    a.n_hg = (H + maxrows - 1) / maxrows;
+    a.hb = (H + a.n_hg - 1) / a.n_hg;
+    GLM_CHECK_ARG(tokens_per_tile * a.hb <= maxrows, GLM_ERR_INVALID, "glm_latent_attn: %d tokens x %d heads exceed %d rows", tokens_per_tile, a.hb, maxrows);
+    const int64_t range = ((int64_t)bt_stride * block_size < (int64_t)window + tokens_per_tile ? (int64_t)bt_stride * block_size : (int64_t)window + tokens_per_tile);
+    GLM_CHECK_ARG((range / nsplit + 64) / block_size + 2 <= LA_BT, GLM_ERR_UNSUPPORTED, "glm_latent_attn: %ld keys per split exceed the block-table slice", (long)(range / nsplit));
+    const int rows = tokens_per_tile * a.hb, mt = rows <= 16 ? 1 : rows <= 32 ? 2 : 4;
+    switch (nct) {
+        case 1: return launch_latent_attn_mt<1>(a, mt, st);
+        case 2: return launch_latent_attn_mt<2>(a, mt, st);
+        case 3: return launch_latent_attn_mt<3>(a, mt, st);
+        case 4: return launch_latent_attn_mt<4>(a, mt, st);
+        case 6: return launch_latent_attn_mt<6>(a, mt, st);
+        case 8: return launch_latent_attn_mt<8>(a, mt, st);
+        case 9: return launch_latent_attn_mt<9>(a, mt, st);
+        default: return launch_latent_attn_mt<16>(a, mt, st);
+    }
+}
+
+extern "C" int glm_latent_up(const void* ctx, const float* part_o, const float* part_ml, const float* sink, int nsplit, const void* wuv, void* out,
+                             int64_t ldo, int64_t Ta, int H, int vdimp, int rp, glm_stream_t stream) {
+    GLM_CHECK_ARG(sink && wuv && out && Ta >= 0 && H > 0 && vdimp > 0 && vdimp % 8 == 0 && rp % 8 == 0 && ldo >= (int64_t)H * vdimp && ldo % 4 == 0 && nsplit >= 1 &&
+                      nsplit <= 64 && (nsplit > 1 ? (part_o && part_ml) : ctx != nullptr), GLM_ERR_INVALID, "glm_latent_up: bad shape Ta=%ld H=%d vdimp=%d", (long)Ta, H, vdimp);
+    GLM_CHECK_ARG((Ta + 15) / 16 <= 65535, GLM_ERR_UNSUPPORTED, "glm_latent_up: too many rows");
+    if (Ta == 0) return GLM_OK;
+    UpArgs a = {(const bf16_t*)ctx, part_o, part_ml, sink, nsplit, (const bf16_t*)wuv, (bf16_t*)out, ldo, Ta, H, vdimp, rp};
+    const size_t lds = (size_t)16 * (((rp + 31) & ~31) + 8) * 2;
+    GLM_CHECK_ARG(lds <= 56 * 1024, GLM_ERR_UNSUPPORTED, "glm_latent_up: latent of %d columns", rp);
+    hipLaunchKernelGGL(latent_up_kernel, dim3((unsigned)(H * ((vdimp + 63) / 64)), (unsigned)((Ta + 15) / 16)), dim3(256), lds, glm_s(stream), a);
+    GLM_CHECK_LAUNCH("glm_latent_up");
+    return GLM_OK;
+}

@@ -1,0 +1,286 @@
+// seq_norm.hip — what happens between two sublayers of a decoder with a 32-bit residual stream, norms in front of and behind
+// every sublayer and a short causal convolution over time on what a sublayer reads:
+//
+//     x_out = x_in + rms(y) * g_post          (y: the finished sublayer's output, optional)
+//     h     = rms(x_out) * g_pre              (optional)
+//     h     = h + conv(h)                     (optional; depthwise, causal, TAPS taps)
+//
+// in ONE launch.  gfx950 only.  Roofline: HBM — x_in and y are read once from HBM (the second pass over a row hits the L2),
+// x_out and h written once.
+//
+// The convolution needs the h of the TAPS-1 tokens before.  Inside a step's rows they are RECOMPUTED from x_in and y (a halo
+// of TAPS-1 rows per workgroup: no hand-off between workgroups, x_out goes to another buffer than x_in); for tokens of
+// earlier steps they come from the sequence's state rows.  The state is double-buffered per sequence (a step reads row set
+// state_in and writes row set state_out), because the workgroup that writes a portion's last inputs is not the one that reads
+// the previous portion's.  Everything is fp32 up to the store of h, and a token's h is the same arithmetic whether it was
+// computed in this step or kept from an earlier one: cutting a sequence differently gives the same bits here.
+#include "common.h"
+
+namespace {
+
+struct SeqNormArgs {
+    const float* x_in;        // [T, ldx], row r or row_index[r]
+    const int32_t* row_index; // optional gather of x_in / y rows (no convolution then)
+    int64_t ldx;
+    float* x_out;             // [T, ldx] or nullptr
+    void* x_cast;             // [T, ldc] x_out in the activation dtype, or nullptr
+    int64_t ldc;
+    const void* y;            // [T, ldy] or nullptr
+    int64_t ldy;
+    int y_f32, n_slabs;       // fp32 y: sum of n_slabs slabs (K-slice partial sums)
+    int64_t slab_stride;
+    const float* g_post;      // [wp]
+    const float* g_pre;       // [wp] or nullptr
+    const float* conv_w;      // [TAPS][wp] or nullptr
+    float* state;             // [state rows][TAPS-1][wp]
+    const int32_t* pos;       // [T] position of the row in its sequence (< 0: unused row)
+    const int32_t* seq_of;    // [T]
+    const int32_t* q_start;   // [S+1] first row of every sequence's portion
+    const int32_t* state_in;  // [S]
+    const int32_t* state_out; // [S] (< 0: keep nothing)
+    int64_t n_state;          // state rows
+    void* h;                  // [T, ldh]
+    int64_t ldh;
+    int act_f32;              // activation dtype: 0 bf16, 1 fp32
+    int64_t T;
+    int width, wp;            // true width (the mean's divisor), padded width (multiple of 8, zero padding)
+    float eps;
+};
+
+constexpr int SN_NT = 256;
+
+__device__ __forceinline__ f32x4_t sn_load_y(const SeqNormArgs& a, int64_t row, int col) {
+    if (!a.y_f32) {
+        const u32x2_t u = *reinterpret_cast<const u32x2_t*>(reinterpret_cast<const bf16_t*>(a.y) + row * a.ldy + col);
+        return f32x4_t{bflo(u[0]), bfhi(u[0]), bflo(u[1]), bfhi(u[1])};
+    }
+    const float* p = reinterpret_cast<const float*>(a.y) + row * a.ldy + col;
+    f32x4_t v = *reinterpret_cast<const f32x4_t*>(p);
+    for (int s = 1; s < a.n_slabs; ++s) v += *reinterpret_cast<const f32x4_t*>(p + s * a.slab_stride);
+    return v;
+}
+
+__device__ __forceinline__ float sn_sumsq(const f32x4_t& v) { return v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3]; }
+
+// x_out of one row at four columns
+__device__ __forceinline__ f32x4_t sn_x(const SeqNormArgs& a, int64_t row, int col, float ry) {
+    f32x4_t x = *reinterpret_cast<const f32x4_t*>(a.x_in + row * a.ldx + col);
+    if (a.y) {
+        const f32x4_t y = sn_load_y(a, row, col), g = *reinterpret_cast<const f32x4_t*>(a.g_post + col);
+#pragma unroll
+        for (int i = 0; i < 4; ++i) x[i] = x[i] + y[i] * ry * g[i];
+    }
+    return x;
+}
+
+__device__ __forceinline__ void sn_store(void* base, int64_t off, int f32, const f32x4_t& v) {
+    if (f32) *reinterpret_cast<f32x4_t*>(reinterpret_cast<float*>(base) + off) = v;
+    else *reinterpret_cast<u32x2_t*>(reinterpret_cast<bf16_t*>(base) + off) = u32x2_t{pack2bf(v[0], v[1]), pack2bf(v[2], v[3])};
+}
+
+// TR rows per workgroup; TAPS = 1: no convolution
+template <int TAPS, int TR>
+__global__ __launch_bounds__(SN_NT) void seq_norm_kernel(const SeqNormArgs a) {
+    constexpr int HALO = TAPS - 1, NR = TR + HALO;
+    __shared__ float s_ry[NR], s_rx[NR], s_red[2][SN_NT / 64];
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+    const int64_t r0 = (int64_t)blockIdx.x * TR;
+    const int64_t r1 = min(r0 + TR, a.T);  // rows [r0, r1) belong to this workgroup
+    const float inv_w = 1.0f / (float)a.width;
+    int64_t lo = r0;  // first halo row that is needed: rows of the same sequence only
+    if constexpr (TAPS > 1) lo = max(r0 - HALO, (int64_t)a.q_start[a.seq_of[r0]]);
+    auto src = [&](int64_t r) -> int64_t { return a.row_index ? a.row_index[r] : r; };
+
+    // ---- pass 1: the two reciprocal root mean squares of every row ----
+    if constexpr (TR == 1) {  // the whole workgroup on one row at a time
+        for (int64_t r = lo; r < r1; ++r) {
+            const int64_t row = src(r);
+            float ry = 0.f, s = 0.f;
+            if (a.y) {
+                for (int c = tid * 4; c < a.wp; c += SN_NT * 4) s += sn_sumsq(sn_load_y(a, row, c));
+                s = wave_sum(s);
+                if (lane == 0) s_red[0][wid] = s;
+                __syncthreads();
+                s = 0.f;
+#pragma unroll
+                for (int w = 0; w < SN_NT / 64; ++w) s += s_red[0][w];
+                ry = 1.0f / sqrtf(s * inv_w + a.eps);
+            }
+            if (a.g_pre) {
+                s = 0.f;
+                for (int c = tid * 4; c < a.wp; c += SN_NT * 4) s += sn_sumsq(sn_x(a, row, c, ry));
+                s = wave_sum(s);
+                if (lane == 0) s_red[1][wid] = s;
+                __syncthreads();
+                s = 0.f;
+#pragma unroll
+                for (int w = 0; w < SN_NT / 64; ++w) s += s_red[1][w];
+            }
+            if (tid == 0) {
+                s_ry[r - r0 + HALO] = ry;
+                s_rx[r - r0 + HALO] = 1.0f / sqrtf(s * inv_w + a.eps);
+            }
+            __syncthreads();
+        }
+    } else {
+        for (int64_t r = lo + wid; r < r1; r += SN_NT / 64) {
+            const int64_t row = src(r);
+            float ry = 0.f, s = 0.f;
+            if (a.y) {
+                for (int c = lane * 4; c < a.wp; c += 256) s += sn_sumsq(sn_load_y(a, row, c));
+                ry = 1.0f / sqrtf(wave_sum(s) * inv_w + a.eps);
+            }
+            if (a.g_pre) {
+                s = 0.f;
+                for (int c = lane * 4; c < a.wp; c += 256) s += sn_sumsq(sn_x(a, row, c, ry));
+                s = wave_sum(s);
+            }
+            if (lane == 0) {
+                s_ry[r - r0 + HALO] = ry;
+                s_rx[r - r0 + HALO] = 1.0f / sqrtf(s * inv_w + a.eps);
+            }
+        }
+        __syncthreads();
+    }
+
+    // ---- pass 2: four columns per thread, down the rows; the last HALO inputs of the convolution ride in registers ----
+    for (int c = tid * 4; c < a.wp; c += SN_NT * 4) {
+        f32x4_t gp = {0.f, 0.f, 0.f, 0.f};
+        if (a.g_pre) gp = *reinterpret_cast<const f32x4_t*>(a.g_pre + c);
+        f32x4_t w[TAPS], hist[TAPS];  // hist[k-1]: h of k tokens ago
+        if constexpr (TAPS > 1) {
+#pragma unroll
+            for (int j = 0; j < TAPS; ++j) w[j] = *reinterpret_cast<const f32x4_t*>(a.conv_w + (int64_t)j * a.wp + c);
+        }
+        auto pre = [&](int64_t r, const f32x4_t& x) {
+            const float rx = s_rx[r - r0 + HALO];
+            f32x4_t h;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) h[i] = x[i] * rx * gp[i];
+            return h;
+        };
+        int cur = -1;  // sequence whose history `hist` holds
+        for (int64_t r = r0; r < r1; ++r) {
+            const f32x4_t x = sn_x(a, src(r), c, s_ry[r - r0 + HALO]);
+            if (a.x_out) *reinterpret_cast<f32x4_t*>(a.x_out + r * a.ldx + c) = x;
+            if (a.x_cast) sn_store(a.x_cast, r * a.ldc + c, a.act_f32, x);
+            if (!a.g_pre) continue;
+            const f32x4_t h = pre(r, x);
+            f32x4_t o = h;
+            if constexpr (TAPS > 1) {
+                const int s = a.seq_of[r], p = a.pos[r], qs = a.q_start[s];
+                if (s != cur) {
+                    cur = s;
+                    const int64_t sin = min(max((int64_t)a.state_in[s], (int64_t)0), a.n_state - 1);
+#pragma unroll
+                    for (int k = 1; k < TAPS; ++k) {
+                        f32x4_t v = {0.f, 0.f, 0.f, 0.f};
+                        if (p - k >= 0) {
+                            if (r - k >= qs) v = pre(r - k, sn_x(a, r - k, c, s_ry[r - k - r0 + HALO]));
+                            else v = *reinterpret_cast<const f32x4_t*>(a.state + (sin * HALO + (HALO - (qs - (r - k)))) * a.wp + c);
+                        }
+                        hist[k - 1] = v;
+                    }
+                }
+                f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int k = HALO; k >= 1; --k)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) acc[i] = acc[i] + w[TAPS - 1 - k][i] * hist[k - 1][i];
+#pragma unroll
+                for (int i = 0; i < 4; ++i) o[i] = h[i] + (acc[i] + w[TAPS - 1][i] * h[i]);
+#pragma unroll
+                for (int k = HALO; k >= 2; --k) hist[k - 1] = hist[k - 2];
+                hist[0] = h;
+                const int qe = a.q_start[s + 1];
+                const int64_t so = a.state_out[s];
+                if (so >= 0 && so < a.n_state && p >= 0) {
+                    const int e = qe - 1 - (int)r;  // tokens of the portion behind this one
+                    if (e < HALO) *reinterpret_cast<f32x4_t*>(a.state + (so * HALO + (HALO - 1 - e)) * a.wp + c) = h;
+                    if (e == 0 && qe - qs < HALO) {  // a portion shorter than the history: the older inputs move up
+                        const int64_t sin = min(max((int64_t)a.state_in[s], (int64_t)0), a.n_state - 1);
+                        for (int i = 0; i < HALO - (qe - qs); ++i)
+                            *reinterpret_cast<f32x4_t*>(a.state + (so * HALO + i) * a.wp + c) =
+                                *reinterpret_cast<const f32x4_t*>(a.state + (sin * HALO + i + (qe - qs)) * a.wp + c);
+                    }
+                }
+            }
+            sn_store(a.h, r * a.ldh + c, a.act_f32, o);
+        }
+    }
+}
+
+template <int TAPS>
+int launch_seq_norm(const SeqNormArgs& a, hipStream_t st) {
+    // few rows (decode): one row per workgroup; many: 16 rows share a halo
+    if (a.T <= 512) hipLaunchKernelGGL((seq_norm_kernel<TAPS, 1>), dim3((unsigned)a.T), dim3(SN_NT), 0, st, a);
+    else hipLaunchKernelGGL((seq_norm_kernel<TAPS, 16>), dim3((unsigned)((a.T + 15) / 16)), dim3(SN_NT), 0, st, a);
+    GLM_CHECK_LAUNCH("glm_seq_norm");
+    return GLM_OK;
+}
+
+// one workgroup per token row: fp32 residual row and (optionally) the row in the activation dtype
+__global__ __launch_bounds__(SN_NT) void embed_rows_kernel(const int64_t* ids, const void* table, int64_t ldw, int64_t vocab, float* x,
+                                                           int64_t ldx, void* cast, int64_t ldc, int act_f32, int width, int wp) {
+    const int64_t t = blockIdx.x;
+    const int64_t id = ids[t];
+    const bool ok = id >= 0 && id < vocab;
+    for (int c = threadIdx.x; c < wp; c += SN_NT) {
+        float v = 0.f;
+        if (ok && c < width) v = act_f32 ? reinterpret_cast<const float*>(table)[id * ldw + c] : bf2f(reinterpret_cast<const bf16_t*>(table)[id * ldw + c]);
+        x[t * ldx + c] = v;
+        if (cast) {
+            if (act_f32) reinterpret_cast<float*>(cast)[t * ldc + c] = v;
+            else reinterpret_cast<bf16_t*>(cast)[t * ldc + c] = f2bf(v);
+        }
+    }
+}
+
+}  // namespace
+
+extern "C" int glm_seq_norm_taps(int taps) {
+    for (int t : {1, 2, 3, 4, 6, 8, 16, 32})
+        if (taps >= 1 && taps <= t) return t;
+    return -1;
+}
+
+extern "C" int glm_seq_norm(const float* x_in, const int32_t* row_index, int64_t ldx, float* x_out, void* x_cast, int64_t ldc,
+                            const void* y, int64_t ldy, int y_f32, int n_slabs, int64_t slab_stride, const float* g_post,
+                            const float* g_pre, const float* conv_w, int taps, float* state, int64_t n_state, const int32_t* pos,
+                            const int32_t* seq_of, const int32_t* q_start, const int32_t* state_in, const int32_t* state_out,
+                            void* h, int64_t ldh, int act_f32, int64_t T, int width, int wp, float eps, glm_stream_t stream) {
+    GLM_CHECK_ARG(x_in && T >= 0 && width > 0 && wp >= width && wp % 8 == 0 && ldx >= wp && ldx % 4 == 0, GLM_ERR_INVALID,
+                  "glm_seq_norm: bad shape T=%ld width=%d wp=%d ldx=%ld", (long)T, width, wp, (long)ldx);
+    GLM_CHECK_ARG(!y || (g_post && ldy >= wp && ldy % 4 == 0 && n_slabs >= 1 && (y_f32 || n_slabs == 1)), GLM_ERR_INVALID,
+                  "glm_seq_norm: bad sublayer output (ldy=%ld slabs=%d)", (long)ldy, n_slabs);
+    GLM_CHECK_ARG((!g_pre) == (!h) && (!h || (ldh >= wp && ldh % 4 == 0)) && (!x_cast || (ldc >= wp && ldc % 4 == 0)), GLM_ERR_INVALID,
+                  "glm_seq_norm: bad output (ldh=%ld ldc=%ld)", (long)ldh, (long)ldc);
+    GLM_CHECK_ARG(taps == 1 || (conv_w && g_pre && state && n_state > 0 && pos && seq_of && q_start && state_in && state_out && !row_index && x_out != x_in),
+                  GLM_ERR_INVALID, "glm_seq_norm: the convolution needs weights, state, positions and x_out apart from x_in");
+    GLM_CHECK_ARG(taps >= 1 && glm_seq_norm_taps(taps) == taps, GLM_ERR_UNSUPPORTED, "glm_seq_norm: %d taps (see glm_seq_norm_taps)", taps);
+    GLM_CHECK_ARG(T < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_seq_norm: too many rows");
+    if (T == 0) return GLM_OK;
+    SeqNormArgs a = {x_in, row_index, ldx, x_out, x_cast, ldc, y, ldy, y_f32, n_slabs, slab_stride, g_post, g_pre, conv_w, state,
+                     pos, seq_of, q_start, state_in, state_out, n_state, h, ldh, act_f32, T, width, wp, eps};
+    hipStream_t st = glm_s(stream);
+    switch (taps) {
+        case 1: return launch_seq_norm<1>(a, st);
+        case 2: return launch_seq_norm<2>(a, st);
+        case 3: return launch_seq_norm<3>(a, st);
+        case 4: return launch_seq_norm<4>(a, st);
+        case 6: return launch_seq_norm<6>(a, st);
+        case 8: return launch_seq_norm<8>(a, st);
+        case 16: return launch_seq_norm<16>(a, st);
+        default: return launch_seq_norm<32>(a, st);
+    }
+}
+
+extern "C" int glm_embed_rows(const int64_t* ids, const void* table, int64_t ldw, int64_t vocab, float* x, int64_t ldx, void* cast,
+                              int64_t ldc, int act_f32, int64_t T, int width, int wp, glm_stream_t stream) {
+    GLM_CHECK_ARG(ids && table && x && T >= 0 && width > 0 && wp >= width && ldw >= width && ldx >= wp && (!cast || ldc >= wp), GLM_ERR_INVALID,
+                  "glm_embed_rows: bad shape T=%ld width=%d wp=%d", (long)T, width, wp);
+    if (T == 0) return GLM_OK;
+    hipLaunchKernelGGL(embed_rows_kernel, dim3((unsigned)T), dim3(SN_NT), 0, glm_s(stream), ids, table, ldw, vocab, x, ldx, cast, ldc, act_f32, width, wp);
+    GLM_CHECK_LAUNCH("glm_embed_rows");
+    return GLM_OK;
+}

@@ -10,6 +10,8 @@ from dataclasses import dataclass
 
 import torch
 
+from nanovllm.models.registry import find_model
+
 
 def normalise_hf_config(cfg) -> types.SimpleNamespace:
     d = cfg if isinstance(cfg, dict) else (cfg.to_dict() if hasattr(cfg, "to_dict") else dict(vars(cfg)))
@@ -48,16 +50,25 @@ class Config:
     enforce_eager: bool = False
     hf_config: object | None = None
     eos: int = -1
-    kvcache_block_size: int = 256
+    kvcache_block_size: int = 0   # 0: the model's default (GLM-4-MoE: 256)
     num_kvcache_blocks: int = -1
+    dtype: str | None = None      # activation dtype of models that run in several ("bfloat16", "float32"); None: bfloat16
 
     def __post_init__(self):
         assert os.path.isdir(self.model)
-        assert self.kvcache_block_size % 256 == 0
         assert 1 <= self.tensor_parallel_size <= 8
         if self.hf_config is None:
             with open(os.path.join(self.model, "config.json")) as f:
                 self.hf_config = json.load(f)
-        self.hf_config = normalise_hf_config(self.hf_config)
+        self.entry = find_model(self.hf_config)
+        self.hf_config = self.entry.read_config(self.hf_config)
+        if self.dtype is not None:
+            if self.dtype not in self.entry.dtypes:
+                raise ValueError(f"{self.entry.name} runs in {' / '.join(self.entry.dtypes)}, not {self.dtype}")
+            if self.entry.step_batches:
+                self.hf_config.torch_dtype = getattr(torch, self.dtype)
+        self.kvcache_block_size = self.kvcache_block_size or self.entry.default_block_size
+        assert self.kvcache_block_size % self.entry.block_multiple == 0
         self.max_model_len = min(self.max_model_len, self.hf_config.max_position_embeddings)
-        assert self.max_num_batched_tokens >= self.max_model_len
+        # (step batches cut prompts into portions: a prompt may be longer than a step)
+        assert self.entry.step_batches or self.max_num_batched_tokens >= self.max_model_len

@@ -12,7 +12,7 @@ import torch.multiprocessing as mp
 
 from nanovllm.config import Config
 from nanovllm.engine.model_runner import ModelRunner
-from nanovllm.engine.scheduler import Scheduler
+from nanovllm.engine.scheduler import Scheduler, StepScheduler
 from nanovllm.engine.sequence import Sequence
 from nanovllm.sampling_params import SamplingParams
 
@@ -45,7 +45,7 @@ class LLMEngine:
         self.tokenizer = self._load_tokenizer(config.model)
         if self.tokenizer is not None and self.tokenizer.eos_token_id is not None:
             config.eos = self.tokenizer.eos_token_id
-        self.scheduler = Scheduler(config)
+        self.scheduler = StepScheduler(config) if config.entry.step_batches else Scheduler(config)
         self._closed = False
         atexit.register(self.exit)
 
@@ -74,6 +74,13 @@ class LLMEngine:
         self.scheduler.add(Sequence(prompt, sampling_params))
 
     def step(self):
+        if self.config.entry.step_batches:
+            batch = self.scheduler.schedule()
+            token_ids = self.model_runner.call("run_chunks", [c for _, c in batch])
+            self.scheduler.postprocess(batch, token_ids)
+            outputs = [(s.seq_id, s.completion_token_ids) for s, _ in batch if s.is_finished]
+            rows = sum(len(c.tokens) for _, c in batch)
+            return outputs, rows if rows > len(batch) else -rows
         seqs, is_prefill = self.scheduler.schedule()
         token_ids = self.model_runner.call("run", seqs, is_prefill)
         self.scheduler.postprocess(seqs, token_ids)

@@ -14,8 +14,8 @@ import torch.distributed as dist
 
 from nanovllm.config import Config
 from nanovllm.engine.sequence import Sequence
+from nanovllm.engine.step_batch import Chunk, build_step
 from nanovllm.layers.sampler import Sampler
-from nanovllm.models.glm4_moe.model import Glm4MoeForCausalLM
 from nanovllm.utils.context import get_context, reset_context, set_context
 
 
@@ -64,17 +64,19 @@ class ModelRunner:
         torch.set_default_dtype(hf.torch_dtype)
         try:
             with torch.device(self.device):
-                model_type = getattr(hf, "model_type", "glm4_moe")
-                if model_type != "glm4_moe":
-                    raise NotImplementedError(f"model_type {model_type!r}: only glm4_moe is built here")
-                self.model = Glm4MoeForCausalLM(hf)
+                self.model = config.entry.load_class()(hf)
                 self.model.load_weights(config.model)
                 self.sampler = Sampler()
-                self.warmup_model()
-                self.reserve_workspaces()
-                self.allocate_kv_cache()
-                if not self.enforce_eager:
-                    self.capture_graphs()
+                if config.entry.step_batches:
+                    self.allocate_step_cache()
+                    if not self.enforce_eager:
+                        self.capture_step_graphs()
+                else:
+                    self.warmup_model()
+                    self.reserve_workspaces()
+                    self.allocate_kv_cache()
+                    if not self.enforce_eager:
+                        self.capture_graphs()
         finally:
             torch.set_default_dtype(old_dtype)
 
@@ -82,6 +84,7 @@ class ModelRunner:
     def exit(self):
         if not self.enforce_eager:
             self.graphs = {}
+            self.step_graphs = {}
         torch.cuda.synchronize()
         if self.world_size > 1:
             dist.barrier()
@@ -265,3 +268,82 @@ class ModelRunner:
             from nanovllm.distributed.expert_parallel import EPExperts
             EPExperts.clear_overflow()
         self.graph_vars = gv
+
+    # ------------------------------------------------------------------ step batches (engine/step_batch.py)
+    def allocate_step_cache(self):
+        """Cache blocks and state slots.  Without a given number of blocks: what the memory holds beside the working set of
+        the largest step, measured by running one over a small cache."""
+        cfg, m = self.config, self.model
+        slots, bs = cfg.max_num_seqs, self.block_size
+        if cfg.num_kvcache_blocks <= 0:
+            n = cfg.max_num_batched_tokens
+            m.allocate(-(-n // bs) + 1, bs, 1, self.device)
+            torch.cuda.reset_peak_memory_stats()
+            self.step_logits([Chunk([0] * n, 0, list(range(-(-n // bs))), 0, 1, [n - 1])])
+            torch.cuda.synchronize()
+            free, total = torch.cuda.mem_get_info()
+            st = torch.cuda.memory_stats()
+            working = st["allocated_bytes.all.peak"] - st["allocated_bytes.all.current"]
+            m.allocate(1, bs, 1, self.device)
+            torch.cuda.empty_cache()
+            free, total = torch.cuda.mem_get_info()
+            budget = int(total * cfg.gpu_memory_utilization) - (total - free) - working - slots * m.state_bytes_per_slot()
+            cfg.num_kvcache_blocks = budget // (m.cache_bytes_per_token() * bs)
+            if self.world_size > 1:   # the ranks must agree on the pool
+                t = torch.tensor([cfg.num_kvcache_blocks], dtype=torch.int64, device="cpu")
+                dist.all_reduce(t, op=dist.ReduceOp.MIN, group=self.ctrl_group)
+                cfg.num_kvcache_blocks = int(t)
+        assert cfg.num_kvcache_blocks > 0, "no memory left for the KV cache"
+        m.allocate(cfg.num_kvcache_blocks, bs, slots, self.device)
+
+    def _to_device(self, host) -> torch.Tensor:
+        return torch.from_numpy(host).pin_memory().to(self.device, non_blocking=True)
+
+    @torch.inference_mode()
+    def step_logits(self, chunks: list[Chunk]) -> torch.Tensor:
+        """Run one step batch: fp32 logits of the wanted rows, in chunk order."""
+        B = len(chunks)
+        if (getattr(self, "step_graphs", None) and B <= self.step_graph_bs[-1]
+                and all(len(c.tokens) == 1 and len(c.block_table) <= self.step_graph_width for c in chunks)):
+            bucket = next(b for b in self.step_graph_bs if b >= B)
+            g = self.step_graphs[bucket]
+            host, _, rows = build_step(chunks, self.model, self.block_size, pad_rows=bucket, table_width=self.step_graph_width)
+            g["buf"].copy_(self._to_device(host))
+            g["graph"].replay()
+            want = [r for c, r in zip(chunks, rows) if c.want]
+            return g["logits"][: B].clone() if want == list(range(B)) else g["logits"][want]
+        host, on_device, _ = build_step(chunks, self.model, self.block_size)
+        return self.model(on_device(self._to_device(host)))
+
+    def run_chunks(self, chunks: list[Chunk]):
+        """One step of generation: tokens sampled for the portions that ask for logits (their last place)."""
+        logits = self.step_logits(chunks)
+        if self.rank != 0:
+            return None
+        temps = [c.temperature for c in chunks if c.want]
+        if not temps:
+            torch.cuda.synchronize()
+            return []
+        return self.sampler(logits, self._dev(temps, torch.float32)).tolist()
+
+    @torch.inference_mode()
+    def capture_step_graphs(self):
+        """The whole decode step (embedding to logits) in one HIP graph per batch-size bucket, over a fixed input buffer."""
+        cfg = self.config
+        max_bs = min(cfg.max_num_seqs, 512)
+        width = self.step_graph_width = -(-cfg.max_model_len // self.block_size)
+        self.step_graph_bs = sorted({b for b in (1, 2, 4, 8) if b <= max_bs} | set(range(16, max_bs + 1, 16)) | {max_bs})
+        graphs, pool = {}, None
+        for bs in reversed(self.step_graph_bs):
+            host, on_device, _ = build_step([], self.model, self.block_size, pad_rows=bs, table_width=width)
+            buf = self._to_device(host)
+            meta = on_device(buf)
+            self.model(meta)  # warm-up
+            torch.cuda.synchronize()
+            g = torch.cuda.CUDAGraph()
+            with torch.cuda.graph(g, pool):
+                logits = self.model(meta)
+            pool = pool or g.pool()
+            graphs[bs] = dict(graph=g, buf=buf, logits=logits)
+            torch.cuda.synchronize()
+        self.step_graphs = graphs

@@ -137,6 +137,28 @@ _SIGNATURES = {
                                             c_void_p, c_void_p, c_void_p, c_float, c_void_p]),
     "glm_add_rmsnorm_partial": (c_int, [c_void_p, c_int, c_int64, c_void_p, c_void_p, c_void_p, c_void_p,
                                         c_int64, c_int, c_float, c_void_p]),
+    "glm_gemm_bf16_act": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int,
+        c_int, c_int, c_int, c_float, c_float, c_void_p]),
+    "glm_gemm_f32": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_int64,
+        c_int64, c_int64, c_int, c_int, c_int, c_int, c_float, c_float, c_void_p]),
+    "glm_seq_norm_taps": (c_int, [c_int]),
+    "glm_seq_norm": (c_int, [c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_int, c_int,
+        c_int64, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p,
+        c_void_p, c_void_p, c_int64, c_int, c_int64, c_int, c_int, c_float, c_void_p]),
+    "glm_embed_rows": (c_int, [c_void_p, c_void_p, c_int64, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_int,
+        c_int64, c_int, c_int, c_void_p]),
+    "glm_latent_prepare": (c_int, [c_void_p, c_int64, c_int, c_int64, c_int64, c_int, c_int, c_int, c_int, c_void_p,
+        c_float, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int, c_void_p]),
+    "glm_latent_gather": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_int, c_void_p]),
+    "glm_latent_attn_max_rows": (c_int, [c_int]),
+    "glm_latent_attn": (c_int, [c_void_p, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p,
+        c_void_p, c_void_p, c_int64, c_int64, c_int, c_int, c_int, c_int, c_float, c_void_p, c_int, c_void_p, c_void_p,
+        c_void_p, c_int, c_void_p]),
+    "glm_latent_up": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int64, c_int64,
+        c_int, c_int, c_int, c_void_p]),
+    "glm_window_attn_prefill": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_void_p,
+        c_void_p, c_void_p, c_void_p, c_int, c_int, c_int64, c_int64, c_int, c_int, c_int, c_int, c_float, c_void_p,
+        c_void_p]),
 }
 
 EXPORTED_SYMBOLS = tuple(_SIGNATURES)
@@ -1182,3 +1204,210 @@ def gemm_bf16(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None
     _check(load_library().glm_gemm_bf16(_p(x2), x2.stride(0), _p(w), w.stride(0), _p(bias), _p(y), N,
                                         M, N, K, _stream()), "glm_gemm_bf16")
     return y.view(*x.shape[:-1], N)
+
+
+# ------------------------------------------------------------------------------------------
+# decoders with a 32-bit residual stream, latent attention and short convolutions over time (no counterpart in the
+# reference).  Activations are bf16 or fp32 (`act dtype`): every op below takes either and picks the kernel by dtype.
+ACT_NONE, ACT_XIELU, ACT_SOFTCAP = 0, 1, 2
+NO_ACT = (ACT_NONE, 0.0, 0.0)
+
+
+def round8(n: int) -> int:
+    return (n + 7) // 8 * 8
+
+
+def _is_f32(dtype) -> int:
+    if dtype == torch.float32:
+        return 1
+    if dtype == torch.bfloat16:
+        return 0
+    raise TypeError(f"activations are bfloat16 or float32, not {dtype}")
+
+
+def linear_act(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, act=NO_ACT, out_f32: bool = False) -> torch.Tensor:
+    """act(x @ w.T + bias), x [M, K], w [N, K] (row pitches free), in x's dtype or — out_f32 — unrounded fp32."""
+    M, K = x.shape
+    N = w.shape[0]
+    assert w.shape[1] == K and w.dtype == x.dtype and x.stride(1) == 1 and w.stride(1) == 1
+    f32 = _is_f32(x.dtype)
+    assert bias is None or (bias.dtype == x.dtype and bias.numel() == N and bias.is_contiguous())
+    y = torch.empty((M, N), dtype=torch.float32 if (f32 or out_f32) else x.dtype, device=x.device)
+    if f32:
+        _check(load_library().glm_gemm_f32(_p(x), x.stride(0), 0, _p(w), w.stride(0), 0, _p(bias), _p(y), N, 0, M, N, K, 1, *act,
+                                           _stream()), "glm_gemm_f32")
+    elif act[0] == ACT_NONE and not out_f32:
+        _check(load_library().glm_gemm_bf16(_p(x), x.stride(0), _p(w), w.stride(0), _p(bias), _p(y), N, M, N, K, _stream()),
+               "glm_gemm_bf16")
+    else:
+        _check(load_library().glm_gemm_bf16_act(_p(x), x.stride(0), _p(w), w.stride(0), _p(bias), _p(y), N, M, N, K,
+                                                int(out_f32), *act, _stream()), "glm_gemm_bf16_act")
+    return y
+
+
+def batched_gemm_f32(x: torch.Tensor, w: torch.Tensor, y: torch.Tensor) -> None:
+    """y[b] = x[b] @ w[b].T for strided fp32 views x [B, M, K], w [B, N, K], y [B, M, N]."""
+    B, M, K = x.shape
+    N = w.shape[1]
+    assert w.shape == (B, N, K) and y.shape == (B, M, N) and x.stride(2) == w.stride(2) == y.stride(2) == 1
+    assert x.dtype == w.dtype == y.dtype == torch.float32
+    _check(load_library().glm_gemm_f32(_p(x), x.stride(1), x.stride(0), _p(w), w.stride(1), w.stride(0), None, _p(y), y.stride(1),
+                                       y.stride(0), M, N, K, B, *NO_ACT, _stream()), "glm_gemm_f32")
+
+
+def embed_rows(ids: torch.Tensor, table: torch.Tensor, wp: int, cast: torch.Tensor | None = None) -> torch.Tensor:
+    """fp32 residual rows [T, wp] of the token ids; `cast` ([T, >= wp], the table's dtype) receives a copy."""
+    T = ids.numel()
+    assert ids.dtype == torch.int64 and table.stride(1) == 1
+    x = torch.empty((T, wp), dtype=torch.float32, device=table.device)
+    assert cast is None or (cast.shape[0] == T and cast.stride(1) == 1 and cast.dtype == table.dtype)
+    _check(load_library().glm_embed_rows(_p(ids), _p(table), table.stride(0), table.shape[0], _p(x), wp, _p(cast),
+                                         cast.stride(0) if cast is not None else wp, _is_f32(table.dtype), T, table.shape[1], wp,
+                                         _stream()), "glm_embed_rows")
+    return x
+
+
+def seq_norm_taps(taps: int) -> int:
+    t = load_library().glm_seq_norm_taps(taps)
+    if t < 0:
+        raise NotImplementedError(f"a convolution over {taps} tokens is not built")
+    return t
+
+
+def seq_norm(x: torch.Tensor, width: int, eps: float, y=None, g_post: torch.Tensor | None = None,
+             g_pre: torch.Tensor | None = None, conv=None, meta=None, rows: torch.Tensor | None = None, act_dtype=torch.bfloat16,
+             x_cast: torch.Tensor | None = None, keep_x: bool = True):
+    """Between two sublayers (glm_seq_norm): returns (x_out, h).  y: the finished sublayer's output [T, wp] (bf16, fp32 or a
+    PartialSum), g_post its norm's gain; g_pre the gain of the norm in front of the next sublayer (None: no h); conv =
+    (weights [taps, wp], state [n, taps-1, wp]) with the step's `meta` (pos, seq_of, q_start, state_in, state_out); rows:
+    gather of rows (no convolution); x_cast receives x_out in the activation dtype."""
+    wp = x.shape[1]
+    assert x.dtype == torch.float32 and x.is_contiguous() and wp % 8 == 0 and width <= wp
+    T = rows.numel() if rows is not None else x.shape[0]
+    yp, ldy, y_f32, ns, sstride = None, wp, 0, 1, 0
+    if y is not None:
+        t = y.part if isinstance(y, PartialSum) else y
+        assert t.is_contiguous() and t.shape[-2:] == x.shape and g_post is not None and g_post.numel() == wp
+        yp, ldy, y_f32 = _p(t), t.shape[-1], _is_f32(t.dtype)
+        if t.dim() == 3:
+            ns, sstride = t.shape[0], t.shape[1] * t.shape[2]
+    x_out = torch.empty((T, wp), dtype=torch.float32, device=x.device) if (y is not None and keep_x) else None
+    h = torch.empty((T, wp), dtype=act_dtype, device=x.device) if g_pre is not None else None
+    w = st = pos = seq_of = q_start = s_in = s_out = None
+    taps, n_state = 1, 0
+    if conv is not None:
+        w, st = conv
+        taps, n_state = w.shape[0], st.shape[0]
+        assert w.dtype == st.dtype == torch.float32 and w.is_contiguous() and st.is_contiguous() and w.shape[1] == wp
+        assert taps == 1 or (st.shape[1:] == (taps - 1, wp) and meta is not None and rows is None)
+    if taps > 1:
+        pos, seq_of, q_start, s_in, s_out = meta.pos, meta.seq_of, meta.q_start, meta.state_in, meta.state_out
+        assert pos.numel() == seq_of.numel() == T and q_start.numel() == s_in.numel() + 1 == s_out.numel() + 1
+        if y is None:
+            assert x_out is None
+    for g in (g_post, g_pre):
+        assert g is None or (g.dtype == torch.float32 and g.is_contiguous() and g.numel() == wp)
+    assert x_cast is None or (x_cast.dtype == act_dtype and x_cast.stride(1) == 1 and x_cast.shape[0] == T)
+    _check(load_library().glm_seq_norm(
+        _p(x), _p(rows), wp, _p(x_out), _p(x_cast), x_cast.stride(0) if x_cast is not None else wp, yp, ldy, y_f32, ns, sstride,
+        _p(g_post) if y is not None else None, _p(g_pre), _p(w) if taps > 1 else None, taps, _p(st) if taps > 1 else None, n_state,
+        _p(pos), _p(seq_of), _p(q_start), _p(s_in), _p(s_out), _p(h), wp, _is_f32(act_dtype), T, width, wp, eps, _stream()),
+        "glm_seq_norm")
+    return (x if x_out is None else x_out), h
+
+
+def latent_prepare(qc: torch.Tensor, c_off: int, heads: int, dimp: int, rank: int, norm_w: torch.Tensor, eps: float,
+                   slots: torch.Tensor, cache: torch.Tensor, Ta: int, wukt: torch.Tensor, crow: torch.Tensor | None = None,
+                   n_crows: int = 0):
+    """Latent norm + cache store of every row of qc, q' = W_uk^T q of the first Ta rows.  Returns (q' [Ta, H, rp], c_out
+    [n_crows, rp] or None)."""
+    T, rp, f32 = qc.shape[0], cache.shape[-1], _is_f32(qc.dtype)
+    assert qc.stride(1) == 1 and cache.is_contiguous() and cache.dtype == qc.dtype and slots.numel() == T
+    assert slots.dtype == torch.int32 and norm_w.dtype == torch.float32 and norm_w.numel() == rp and wukt.shape == (heads, rp, dimp)
+    assert wukt.is_contiguous() and (crow is None or (crow.dtype == torch.int32 and crow.numel() == T))
+    qa = torch.empty((Ta, heads, rp), dtype=qc.dtype, device=qc.device)
+    c_out = torch.empty((n_crows, rp), dtype=qc.dtype, device=qc.device) if crow is not None else None
+    _check(load_library().glm_latent_prepare(
+        _p(qc), qc.stride(0), c_off, T, Ta, heads, dimp, rank, rp, _p(norm_w), eps, _p(slots), _p(cache), cache.numel() // rp,
+        _p(crow), _p(c_out), n_crows, _p(wukt), _p(qa) if Ta else None, f32, _stream()), "glm_latent_prepare")
+    if f32 and Ta:
+        q = qc[:Ta, : heads * dimp].view(Ta, heads, dimp)
+        batched_gemm_f32(q.transpose(0, 1), wukt, qa.transpose(0, 1))
+    return qa, c_out
+
+
+def latent_gather(cache: torch.Tensor, slots: torch.Tensor, rows: torch.Tensor, out: torch.Tensor) -> None:
+    """out[rows[i]] = cache row slots[i]."""
+    rp = cache.shape[-1]
+    assert out.shape[1] == rp and out.dtype == cache.dtype and out.is_contiguous() and cache.is_contiguous()
+    assert slots.dtype == rows.dtype == torch.int32 and slots.numel() == rows.numel()
+    _check(load_library().glm_latent_gather(_p(cache), cache.numel() // rp, _p(slots), _p(rows), slots.numel(), _p(out), out.shape[0],
+                                            rp * cache.element_size(), _stream()), "glm_latent_gather")
+
+
+def latent_attn_max_rows(rp: int) -> int:
+    n = load_library().glm_latent_attn_max_rows(rp)
+    if n <= 0:
+        raise NotImplementedError(f"a latent of {rp} columns is not built")
+    return n
+
+
+def latent_tokens_per_tile(rp: int, heads: int) -> int:
+    """Query tokens of one sequence that share a workgroup's pass over the cache."""
+    rows = latent_attn_max_rows(rp)
+    groups = -(-heads // rows)
+    return max(1, rows // -(-heads // groups))
+
+
+def latent_attn(qa: torch.Tensor, cache: torch.Tensor, tile_tok: torch.Tensor, tile_n: torch.Tensor, tokens_per_tile: int,
+                pos: torch.Tensor, seq_of: torch.Tensor, block_tables: torch.Tensor, rank: int, window: int, scale: float,
+                sink: torch.Tensor, wuv: torch.Tensor, out: torch.Tensor, num_splits: int = 0) -> None:
+    """Absorbed attention of the rows qa [Ta, H, rp] over the paged latents, then W_uv: writes out[:Ta] ([T, H * vdimp])."""
+    Ta, H, rp = qa.shape
+    n_blocks, bs, _ = cache.shape
+    vdimp = wuv.shape[1]
+    if Ta == 0:
+        return
+    assert qa.is_contiguous() and cache.is_contiguous() and cache.dtype == qa.dtype and wuv.is_contiguous()
+    assert wuv.shape == (H, vdimp, rp) and sink.dtype == torch.float32 and sink.numel() == H and block_tables.stride(1) == 1
+    for t in (tile_tok, tile_n, pos, seq_of, block_tables):
+        assert t.dtype == torch.int32
+    assert pos.numel() >= Ta and seq_of.numel() >= Ta and out.stride(1) == 1 and out.shape[0] >= Ta and out.shape[1] == H * vdimp
+    lib, f32 = load_library(), _is_f32(qa.dtype)
+    ctx = part_o = part_ml = None
+    ns = 1
+    if not f32:
+        # enough (tile, head group, KV split) workgroups to cover the chip, at least four 32-key tiles per split
+        rows = latent_attn_max_rows(rp)
+        wgs = tile_tok.numel() * -(-H // rows)
+        keys = min(window + tokens_per_tile, block_tables.shape[1] * bs)
+        ns = num_splits or max(1, min(64, 512 // max(1, wgs), -(-keys // 128)))
+    if ns == 1:
+        ctx = torch.empty((Ta, H, rp), dtype=qa.dtype, device=qa.device)
+    else:
+        part_o = torch.empty((Ta * H, ns, rp), dtype=torch.float32, device=qa.device)
+        part_ml = torch.empty((Ta * H, ns, 2), dtype=torch.float32, device=qa.device)
+    _check(lib.glm_latent_attn(_p(qa), _p(cache), n_blocks, bs, _p(tile_tok), _p(tile_n), tile_tok.numel(), tokens_per_tile, _p(pos),
+                               _p(seq_of), _p(block_tables), block_tables.stride(0), Ta, H, rank, rp, window, scale, _p(sink), ns,
+                               _p(ctx), _p(part_o), _p(part_ml), f32, _stream()), "glm_latent_attn")
+    if f32:
+        batched_gemm_f32(ctx.transpose(0, 1), wuv, out[:Ta].view(Ta, H, vdimp).transpose(0, 1))
+        return
+    _check(lib.glm_latent_up(_p(ctx), _p(part_o), _p(part_ml), _p(sink), ns, _p(wuv), _p(out), out.stride(0), Ta, H, vdimp, rp,
+                             _stream()), "glm_latent_up")
+
+
+def window_attn_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, out: torch.Tensor, q_start: torch.Tensor,
+                        k_start: torch.Tensor, tile_seq: torch.Tensor, tile_off: torch.Tensor, heads: int, dk: int, dv: int,
+                        window: int, scale: float, sink: torch.Tensor) -> None:
+    """q, out: rows of the step's long portions (views with free row pitch); k, v: expanded rows, see the header."""
+    _bf16(q, "q"); _bf16(k, "k"); _bf16(v, "v"); _bf16(out, "out")
+    assert q.shape[1] == k.shape[1] == heads * dk and v.shape[1] == out.shape[1] == heads * dv and k.stride(0) == v.stride(0)
+    assert k.shape[0] == v.shape[0] and out.shape[0] == q.shape[0] and sink.dtype == torch.float32 and sink.numel() == heads
+    for t in (q_start, k_start, tile_seq, tile_off):
+        assert t.dtype == torch.int32
+    S = q_start.numel() - 1
+    assert k_start.numel() == S + 1 and tile_seq.numel() == tile_off.numel()
+    _check(load_library().glm_window_attn_prefill(
+        _p(q), q.stride(0), _p(k), _p(v), k.stride(0), _p(out), out.stride(0), _p(q_start), _p(k_start), _p(tile_seq), _p(tile_off),
+        tile_seq.numel(), S, q.shape[0], k.shape[0], heads, dk, dv, window, scale, _p(sink), _stream()), "glm_window_attn_prefill")

@@ -155,3 +155,39 @@ class RowParallelLinear(LinearBase):
         if self.tp_size > 1:
             get_tp_group().all_reduce(y)
         return y
+
+
+class PaddedLinear(nn.Module):
+    """Projection whose output is a row of blocks (heads, latents ...), each padded to a multiple of 8 columns, and whose input
+    may be such a row too: any size runs on the kernels, padding is zero weights.  bf16 or fp32, activation in the epilogue.
+
+    in_size: input columns, or a list of block sizes (the input's own padded layout); out_blocks: PADDED sizes of the output
+    blocks.  load() takes one [rows, columns] tensor per output block, columns unpadded."""
+
+    def __init__(self, in_size, out_blocks: list[int], dtype):
+        super().__init__()
+        self.in_blocks = list(in_size) if isinstance(in_size, (list, tuple)) else [in_size]
+        self.out_blocks = list(out_blocks)
+        assert all(b % 8 == 0 for b in self.out_blocks)
+        self.K = sum(hip_ops.round8(b) for b in self.in_blocks)
+        self.N = sum(self.out_blocks)
+        self.dtype = dtype
+        self.weight = None
+
+    def load(self, blocks: list[torch.Tensor], device) -> None:
+        assert len(blocks) == len(self.out_blocks)
+        full = torch.zeros(self.N, self.K, dtype=self.dtype, device=device)
+        r = 0
+        for size, w in zip(self.out_blocks, blocks):
+            w = w.to(device=device, dtype=self.dtype)
+            assert w.shape[0] <= size and w.shape[1] == sum(self.in_blocks), (w.shape, size, self.in_blocks)
+            c = k = 0
+            for b in self.in_blocks:
+                full[r: r + w.shape[0], k: k + b] = w[:, c: c + b]
+                c, k = c + b, k + hip_ops.round8(b)
+            r += size
+        self.weight = hip_ops.padded_weight(self.N, self.K, dtype=self.dtype, device=device)
+        self.weight.copy_(full)
+
+    def forward(self, x: torch.Tensor, bias: torch.Tensor | None = None, act=hip_ops.NO_ACT, out_f32: bool = False) -> torch.Tensor:
+        return hip_ops.linear_act(x, self.weight, bias, act, out_f32)

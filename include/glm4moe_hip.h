@@ -487,6 +487,66 @@ int glm_comm_ipc_close(void* ptr);
 int glm_allreduce_oneshot(const void* in, void* out, void* const* peer_bufs, void* const* peer_flags, int rank, int world,
                           int64_t n, int64_t n_max, void* state, glm_stream_t stream);
 
+/* ---- decoders with a 32-bit residual stream, latent attention and short convolutions over time (Dafolorn) ---------------------
+ * No counterpart in the reference.  act_f32: activation dtype, 0 = bf16, 1 = fp32.  Sizes are padded to multiples of 8 with
+ * zero weights by the caller; kernels never read uninitialised memory into a product.                                       */
+
+/* activations of a projection's fp32 result: xIELU (z > 0: a z^2 + z/2; z <= 0: b (exp(z) - 1 - z) + z/2), soft cap a tanh(z/a) */
+#define GLM_EPI_NONE    0
+#define GLM_EPI_XIELU   1
+#define GLM_EPI_SOFTCAP 2
+/* y = act(x . W^T + bias): glm_gemm_bf16 with an activation in the epilogue and, with out_f32, fp32 output rows (unrounded).  */
+int glm_gemm_bf16_act(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* bias, void* y, int64_t ldy, int64_t M,
+                      int N, int K, int out_f32, int act, float act_a, float act_b, glm_stream_t stream);
+/* the same in true fp32, `batch` products at strides xb / wb / yb (elements).  K % 4 == 0.                                     */
+int glm_gemm_f32(const float* x, int64_t ldx, int64_t xb, const float* w, int64_t ldw, int64_t wb, const float* bias, float* y,
+                 int64_t ldy, int64_t yb, int64_t M, int N, int K, int batch, int act, float act_a, float act_b,
+                 glm_stream_t stream);
+
+/* Between two sublayers: x_out = x_in + rms(y) g_post (y bf16, or the sum of n_slabs fp32 slabs); h = rms(x_out) g_pre, then
+ * h += depthwise causal convolution over time.  Gains and conv_w [taps][wp] fp32; x fp32.  Rows of a step: row t belongs to
+ * sequence seq_of[t] at position pos[t] (< 0: unused), sequence s has rows [q_start[s], q_start[s+1]).  state
+ * [n_state][taps-1][wp] fp32 keeps the last taps-1 inputs of the convolution, oldest first: set state_in[s] is read, set
+ * state_out[s] (another one; < 0: none) written.  taps: a value glm_seq_norm_taps returns (1 = no convolution; then row_index
+ * may gather the x_in / y rows); x_out, x_cast (x_out in the activation dtype), y, g_pre + h are optional.                    */
+int glm_seq_norm_taps(int taps); /* smallest supported count >= taps (pad with zero weights in front), -1: none */
+int glm_seq_norm(const float* x_in, const int32_t* row_index, int64_t ldx, float* x_out, void* x_cast, int64_t ldc, const void* y,
+                 int64_t ldy, int y_f32, int n_slabs, int64_t slab_stride, const float* g_post, const float* g_pre,
+                 const float* conv_w, int taps, float* state, int64_t n_state, const int32_t* pos, const int32_t* seq_of,
+                 const int32_t* q_start, const int32_t* state_in, const int32_t* state_out, void* h, int64_t ldh, int act_f32,
+                 int64_t T, int width, int wp, float eps, glm_stream_t stream);
+/* embedding rows as the fp32 residual and, optionally, in the activation dtype; columns [width, wp) are zeros                 */
+int glm_embed_rows(const int64_t* ids, const void* table, int64_t ldw, int64_t vocab, float* x, int64_t ldx, void* cast,
+                   int64_t ldc, int act_f32, int64_t T, int width, int wp, glm_stream_t stream);
+
+/* Latent attention over a paged cache [n_blocks, block_size, rp] of latent rows (rp = rank rounded up to 8).
+ * prepare: row t of qc holds the query heads at h*dimp and the raw latent at c_off; c = rms(raw) norm_w goes to cache row
+ * slots[t] (< 0: none) and to row crow[t] of c_out; for rows [0, Ta): qa[t, h, :] = W_uk[h]^T q[t, h, :] (wukt [H, rp, dimp]; bf16 only). */
+int glm_latent_prepare(const void* qc, int64_t ldq, int c_off, int64_t T, int64_t Ta, int H, int dimp, int rank, int rp,
+                       const float* norm_w, float eps, const int32_t* slots, void* cache, int64_t n_slots, const int32_t* crow,
+                       void* c_out, int64_t n_crows, const void* wukt, void* qa, int act_f32, glm_stream_t stream);
+int glm_latent_gather(const void* cache, int64_t n_slots, const int32_t* slots, const int32_t* rows, int64_t n, void* out,
+                      int64_t n_rows, int row_bytes, glm_stream_t stream);
+/* attn: query row (t, h) sees the latents of positions (pos[t] - window, pos[t]] of its sequence; softmax with the extra mass
+ * exp(sink[h]).  Tiles: tile i covers tile_n[i] <= tokens_per_tile consecutive rows of one sequence from tile_tok[i]; tokens x
+ * heads of a tile <= glm_latent_attn_max_rows(rp).  nsplit == 1: ctx [Ta, H, rp] normalised (bf16 / fp32); else part_o
+ * [Ta*H, nsplit, rp], part_ml [Ta*H, nsplit, 2] for glm_latent_up.  fp32: tiles unused, nsplit 1.
+ * up: out[t, h*vdimp ..] = W_uv[h] ctx[t, h, :] (wuv [H, vdimp, rp]).                                                         */
+int glm_latent_attn_max_rows(int rp);
+int glm_latent_attn(const void* qa, const void* cache, int64_t n_blocks, int block_size, const int32_t* tile_tok,
+                    const int32_t* tile_n, int n_tiles, int tokens_per_tile, const int32_t* pos, const int32_t* seq_of,
+                    const int32_t* block_tables, int64_t bt_stride, int64_t Ta, int H, int rank, int rp, int window, float scale,
+                    const float* sink, int nsplit, void* ctx, float* part_o, float* part_ml, int act_f32, glm_stream_t stream);
+int glm_latent_up(const void* ctx, const float* part_o, const float* part_ml, const float* sink, int nsplit, const void* wuv,
+                  void* out, int64_t ldo, int64_t Ta, int H, int vdimp, int rp, glm_stream_t stream);
+/* Prompts and long portions, bf16: q rows [q_start[s], q_start[s+1]) against expanded k / v rows [k_start[s], k_start[s+1]) — the
+ * portion's own tokens last, in front of them the history the window still reaches.  Head h at h*dk (q, k) / h*dv (v, out).
+ * Tiles of 128 query rows: (sequence, first row inside the portion).  dk, dv <= 256, multiples of 8.                          */
+int glm_window_attn_prefill(const void* q, int64_t ldq, const void* k, const void* v, int64_t ldkv, void* out, int64_t ldo,
+                            const int32_t* q_start, const int32_t* k_start, const int32_t* tile_seq, const int32_t* tile_off,
+                            int n_tiles, int S, int64_t Tq, int64_t Tk, int H, int dk, int dv, int window, float scale,
+                            const float* sink, glm_stream_t stream);
+
 #ifdef __cplusplus
 }
 #endif
