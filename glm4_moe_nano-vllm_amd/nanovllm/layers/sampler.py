@@ -14,7 +14,9 @@ class Sampler(nn.Module):
     def forward(self, logits: torch.Tensor, temperatures: torch.Tensor):
         if torch.all(temperatures == 0):
             return torch.argmax(logits, dim=-1)
-        logits = logits.float().div_(temperatures.unsqueeze(dim=1))
-        probs = torch.softmax(logits, dim=-1)
+        # out of place: the caller may hand over fp32 logits it still owns.  A temperature of 0 beside others: that row is greedy.
+        greedy = temperatures == 0
+        scaled = logits.float() / torch.where(greedy, 1.0, temperatures).unsqueeze(dim=1)
+        probs = torch.softmax(scaled, dim=-1)
         noise = torch.empty_like(probs).exponential_(1).clamp_min_(1e-10)
-        return probs.div_(noise).argmax(dim=-1)
+        return torch.where(greedy, torch.argmax(logits, dim=-1), (probs / noise).argmax(dim=-1))
