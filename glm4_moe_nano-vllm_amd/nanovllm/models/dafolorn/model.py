@@ -14,7 +14,7 @@ from nanovllm.layers.dense_mlp import DenseMLP
 from nanovllm.layers.latent_attention import LatentAttention
 from nanovllm.layers.linear import PaddedLinear
 from nanovllm.layers.seq_norm import SublayerEntry, norm_gain
-from nanovllm.utils.loader import load_one, load_prefixed
+from nanovllm.utils.loader import load_prefixed
 from .config import layer_runs
 
 
@@ -32,10 +32,10 @@ class DafolornLayer(nn.Module):
             self.mlp = DenseMLP(cfg.hidden_size, spec.ff, dt)
         self.g_post1 = self.g_post2 = None
 
-    def load_weights(self, path: str, prefix: str, device) -> None:
-        t = {k[len(prefix) + 1:]: v for k, v in load_prefixed(path, prefix).items()}
+    def load_from(self, fetch, prefix: str, device) -> None:
+        t = {k[len(prefix) + 1:]: v for k, v in fetch(prefix).items()}
         if not t:
-            raise ValueError(f"no tensors under '{prefix}' in '{path}'")
+            raise ValueError(f"no tensors under '{prefix}'")
         wp = self.entry1.wp
         sub = lambda p: {k[len(p):]: v for k, v in t.items() if k.startswith(p)}  # noqa: E731
         self.entry1.load(t["norm1"], t["canon1"], device)
@@ -69,13 +69,17 @@ class DafolornForCausalLM(nn.Module):
 
     # ------------------------------------------------------------------ weights
     def load_weights(self, path: str) -> None:
+        self.load_from(lambda prefix: load_prefixed(path, prefix))
+
+    def load_from(self, fetch) -> None:
+        """fetch(prefix) -> the tensors `prefix` and `prefix.*` of a checkpoint, by full name."""
         cfg, dev = self.config, torch.empty(0).device  # the engine builds models under torch.device(...)
         V, w, wp = cfg.vocab_size, cfg.hidden_size, cfg.padded_width
 
         def need(name):
-            t = load_one(path, name)
+            t = fetch(name).get(name)
             if t is None:
-                raise ValueError(f"'{name}' not found in '{path}'")
+                raise ValueError(f"'{name}' not found in the checkpoint")
             return t
 
         table = hip_ops.padded_weight(hip_ops.round8(V), wp, dtype=self.dtype, device=dev)
@@ -89,7 +93,7 @@ class DafolornForCausalLM(nn.Module):
             step[:, :w] = need("loop.step").to(device=dev, dtype=self.dtype)
             self.loop_step = step
         for i, layer in enumerate(self.layers):
-            layer.load_weights(path, f"l{i}", dev)
+            layer.load_from(fetch, f"l{i}", dev)
 
     # ------------------------------------------------------------------ cache and state
     @property
