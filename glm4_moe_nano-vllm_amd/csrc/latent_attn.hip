@@ -23,7 +23,7 @@
 namespace {
 
 constexpr float LOG2E = 1.4426950408889634f;
-constexpr int LA_BT = 2048;  // block-table entries a workgroup caches in LDS
+constexpr int LA_BT = 1024;  // block-table entries a workgroup caches in LDS
 
 __device__ const u32x4_t la_zero_page[4] = {};
 
@@ -46,35 +46,53 @@ struct PrepArgs {
     bf16_t* qa;            // [Ta, H, rp]
 };
 
+// latent norm of one token by one wave, eight columns per lane and step (the padding columns of the projection are zeros)
 template <typename E>
-__device__ __forceinline__ float la_ld(const void* p, int64_t i) {
-    if constexpr (sizeof(E) == 2) return bf2f(reinterpret_cast<const bf16_t*>(p)[i]);
-    else return reinterpret_cast<const float*>(p)[i];
+__device__ __forceinline__ void la_ld8(const void* p, int64_t i, float (&v)[8]) {
+    if constexpr (sizeof(E) == 2) {
+        const u32x4_t u = *reinterpret_cast<const u32x4_t*>(reinterpret_cast<const bf16_t*>(p) + i);
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            v[2 * j] = bflo(u[j]);
+            v[2 * j + 1] = bfhi(u[j]);
+        }
+    } else {
+        const float* f = reinterpret_cast<const float*>(p) + i;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v[j] = f[j];
+    }
 }
 template <typename E>
-__device__ __forceinline__ void la_st(void* p, int64_t i, float v) {
-    if constexpr (sizeof(E) == 2) reinterpret_cast<bf16_t*>(p)[i] = f2bf(v);
-    else reinterpret_cast<float*>(p)[i] = v;
+__device__ __forceinline__ void la_st8(void* p, int64_t i, const float (&v)[8]) {
+    if constexpr (sizeof(E) == 2) {
+        *reinterpret_cast<u32x4_t*>(reinterpret_cast<bf16_t*>(p) + i) =
+            u32x4_t{pack2bf(v[0], v[1]), pack2bf(v[2], v[3]), pack2bf(v[4], v[5]), pack2bf(v[6], v[7])};
+    } else {
+        float* f = reinterpret_cast<float*>(p) + i;
+#pragma unroll
+        for (int j = 0; j < 8; ++j) f[j] = v[j];
+    }
 }
-
-// latent norm of one token by one wave
 template <typename E>
 __device__ void latent_norm_row(const PrepArgs& a, int64_t t, int lane) {
     const int64_t base = t * a.ldq + a.c_off;
-    float s = 0.f;
-    for (int i = lane; i < a.rank; i += 64) {
-        const float v = la_ld<E>(a.qc, base + i);
-        s += v * v;
-    }
-    const float r = 1.0f / sqrtf(wave_sum(s) / (float)a.rank + a.eps);
     const int64_t slot = a.slots[t];
     const bool st = slot >= 0 && slot < a.n_slots;
     int64_t row = a.crow ? a.crow[t] : -1;
     if (row >= a.n_crows) row = -1;
-    for (int i = lane; i < a.rp; i += 64) {
-        const float v = i < a.rank ? la_ld<E>(a.qc, base + i) * r * a.norm_w[i] : 0.f;
-        if (st) la_st<E>(a.cache, slot * a.rp + i, v);
-        if (row >= 0) la_st<E>(a.c_out, row * a.rp + i, v);
+    float v[8], s = 0.f;
+    for (int i = lane * 8; i < a.rp; i += 512) {
+        la_ld8<E>(a.qc, base + i, v);
+#pragma unroll
+        for (int j = 0; j < 8; ++j) s += v[j] * v[j];
+    }
+    const float r = 1.0f / sqrtf(wave_sum(s) / (float)a.rank + a.eps);
+    for (int i = lane * 8; i < a.rp; i += 512) {
+        if (a.rp > 512) la_ld8<E>(a.qc, base + i, v);  // (one step: the values are still in registers)
+#pragma unroll
+        for (int j = 0; j < 8; ++j) v[j] = v[j] * r * a.norm_w[i + j];
+        if (st) la_st8<E>(a.cache, slot * a.rp + i, v);
+        if (row >= 0) la_st8<E>(a.c_out, row * a.rp + i, v);
     }
 }
 
@@ -159,11 +177,20 @@ struct AttnArgs {
     float* part_ml;           // [Ta * H, nsplit, 2] running maximum (log2 units), mass
 };
 
+// Two workgroups per CU where registers and LDS allow (one computes while the other waits), else one with a deeper ring.
 template <int NCT, int MT>
-__global__ __launch_bounds__(256, 1) void latent_attn_kernel(const AttnArgs a) {
+struct LaCfg {
+    static constexpr int TILEB = 32 * NCT * 128, SLAB = 2 * MT * 2 * 1024;
+    static constexpr bool TWO = NCT <= 8 && MT * NCT <= 16;
+    static constexpr int NST = TWO ? (3 * TILEB + SLAB + LA_BT * 4 <= 80 * 1024 ? 3 : 2) : (3 * TILEB <= 112 * 1024 ? 3 : 2);
+    static constexpr int LDS = NST * TILEB + SLAB + LA_BT * 4;
+    static_assert(LDS <= (TWO ? 80 : 160) * 1024, "LDS of a CU");
+};
+
+template <int NCT, int MT>
+__global__ __launch_bounds__(256, (LaCfg<NCT, MT>::TWO ? 2 : 1)) void latent_attn_kernel(const AttnArgs a) {
     constexpr int RPAD = NCT * 64, ROWB = RPAD * 2, TILEB = 32 * ROWB, CPR = RPAD / 8;
-    constexpr int NST = 3 * TILEB <= 112 * 1024 ? 3 : 2;
-    constexpr int SLAB = 2 * MT * 2 * 1024;
+    constexpr int NST = LaCfg<NCT, MT>::NST, SLAB = LaCfg<NCT, MT>::SLAB;
     constexpr int FG = NCT < 8 ? NCT : 8;  // fragments per request group
     extern __shared__ __attribute__((aligned(16))) char smem[];
     const int tid = threadIdx.x, lane = tid & 63;
@@ -180,7 +207,9 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(const AttnArgs a) {
     if (tok0 < 0 || tok0 >= a.Ta || ntok <= 0) return;
     const int p0 = a.pos[tok0], p1 = p0 + ntok - 1, seq = a.seq_of[tok0];
     const int nrows = ntok * hb;
-    const int lo = max(0, p0 - a.window + 1);
+    // tiles start at multiples of 32, so that a tile lies in one cache block; the keys in front of the window's first are old
+    // latents of the same sequence (masked), keys behind the last row's are fetched from the zero page
+    const int lo = max(0, p0 - a.window + 1) & ~31;
     const int ntile = p0 < 0 ? 0 : (p1 - lo + 32) >> 5;  // 32-key tiles of the whole range
     const int per = (ntile + a.nsplit - 1) / a.nsplit;
     const int t0 = split * per, t1 = min(t0 + per, ntile), n = t1 - t0;
@@ -227,27 +256,30 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(const AttnArgs a) {
     __syncthreads();
     const unsigned base = lds_addr(smem), slab = base + NST * TILEB, bt_addr = slab + SLAB;
     const bf16_t* cache = reinterpret_cast<const bf16_t*>(a.cache);
+    // per-lane source offsets (elements) of the DMA pieces inside a tile: constant over the tiles
+    unsigned off[NCT];
+    int orow[NCT];
+    const bool padded = RPAD != a.rp;
+#pragma unroll
+    for (int i = 0; i < NCT; ++i) {
+        const int q = (w * NCT + i) * 64 + lane, row = q / CPR, ch = (q % CPR) ^ attn_swz(row);
+        orow[i] = (padded && ch * 8 >= a.rp) ? 1 << 30 : row;
+        off[i] = (unsigned)(row * a.rp + ch * 8);
+    }
     auto issue = [&](int it) {
         const int k0 = klo + it * 32;
-        int b0, b1;
-        {
-            const int i0 = (k0 >> a.bs_shift) - blk0, i1 = min(i0 + 1, nblk - 1);
-            asm volatile("ds_read_b32 %0, %2\n\tds_read_b32 %1, %3\n\ts_waitcnt lgkmcnt(0)"
-                         : "=&v"(b0), "=&v"(b1) : "v"(bt_addr + i0 * 4), "v"(bt_addr + i1 * 4) : "memory");
-            b0 = __builtin_amdgcn_readfirstlane(b0);
-            b1 = __builtin_amdgcn_readfirstlane(b1);
-        }
-        const int first = k0 >> a.bs_shift;
-        char* st = smem + (it % NST) * TILEB;
+        int blk;
+        asm volatile("ds_read_b32 %0, %1\n\ts_waitcnt lgkmcnt(0)" : "=v"(blk) : "v"(bt_addr + ((k0 >> a.bs_shift) - blk0) * 4) : "memory");
+        blk = __builtin_amdgcn_readfirstlane(blk);
+        const bf16_t* src = cache + (((int64_t)blk << a.bs_shift) + (k0 & bmask)) * a.rp;
+        char* st = smem + (it % NST) * TILEB + w * NCT * 1024;
+        const int left = khi - k0;
+        if (left >= 31 && !padded) {
 #pragma unroll
-        for (int i = 0; i < NCT; ++i) {
-            const int q = (w * NCT + i) * 64 + lane;
-            const int row = q / CPR, ch = (q % CPR) ^ attn_swz(row);
-            const int key = k0 + row;
-            const int blk = (key >> a.bs_shift) == first ? b0 : b1;
-            const bf16_t* src = cache + (((int64_t)blk << a.bs_shift) + (key & bmask)) * a.rp + ch * 8;
-            const void* s = (key <= khi && ch * 8 < a.rp) ? (const void*)src : (const void*)la_zero_page;
-            lds_dma16(s, st + (w * NCT + i) * 1024);
+            for (int i = 0; i < NCT; ++i) lds_dma16(src + off[i], st + i * 1024);
+        } else {
+#pragma unroll
+            for (int i = 0; i < NCT; ++i) lds_dma16(orow[i] <= left ? (const void*)(src + off[i]) : (const void*)la_zero_page, st + i * 1024);
         }
     };
     f32x4_t acc[MT][NCT];
@@ -305,6 +337,7 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(const AttnArgs a) {
         __builtin_amdgcn_s_barrier();
         // ---- online softmax of row c of every row tile: this lane holds keys 16 t + 4 g + r ----
         const int kbase = klo + it * 32 + 4 * g;
+        const bool inner = klo + it * 32 > p1 - a.window && klo + it * 32 + 31 <= p0;  // every row sees every key
         bf16x8_t pf[MT];
 #pragma unroll
         for (int m = 0; m < MT; ++m) {
@@ -317,26 +350,38 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(const AttnArgs a) {
             wait_lds();
             asm volatile("" : "+v"(sv[0][0]), "+v"(sv[0][1]), "+v"(sv[1][0]), "+v"(sv[1][1]));
             float mx = -INFINITY, x[2][4];
+            if (inner) {
 #pragma unroll
-            for (int t = 0; t < 2; ++t)
+                for (int t = 0; t < 2; ++t)
 #pragma unroll
-                for (int r = 0; r < 4; ++r) {
-                    const int d = rpos[m] - (kbase + 16 * t + r);
-                    const bool vis = d >= 0 && d < a.window && kbase + 16 * t + r <= khi;
-                    x[t][r] = vis ? sv[t][0][r] + sv[t][1][r] : -INFINITY;
-                    mx = fmaxf(mx, x[t][r]);
-                }
-            mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-            mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-            const float m_new = fmaxf(m_run[m], mx);
-            const float m_use = m_new == -INFINITY ? 0.f : m_new;
-            if (__any(m_new > m_run[m])) {
-                const float alpha = __builtin_amdgcn_exp2f(m_run[m] - m_use);
+                    for (int r = 0; r < 4; ++r) {
+                        x[t][r] = sv[t][0][r] + sv[t][1][r];
+                        mx = fmaxf(mx, x[t][r]);
+                    }
+            } else {
+                const int d0 = rpos[m] - kbase;
+#pragma unroll
+                for (int t = 0; t < 2; ++t)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) {
+                        const int d = d0 - 16 * t - r;
+                        x[t][r] = (rpos[m] >= 0 && d >= 0 && d < a.window) ? sv[t][0][r] + sv[t][1][r] : -INFINITY;
+                        mx = fmaxf(mx, x[t][r]);
+                    }
+            }
+            // the reference point is raised only when a score exceeds it by more than 2^8 (it cancels in the end); it is the
+            // same in the four lanes that share a row
+            if (__any(mx > m_run[m] + 8.0f || (m_run[m] == -INFINITY && mx > -INFINITY))) {
+                mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+                mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+                const float m_new = fmaxf(m_run[m], mx);
+                const float alpha = m_new == -INFINITY ? 1.0f : __builtin_amdgcn_exp2f(m_run[m] - m_new);
                 l_run[m] *= alpha;
 #pragma unroll
                 for (int d = 0; d < NCT; ++d) acc[m][d] *= alpha;
+                m_run[m] = m_new;
             }
-            m_run[m] = m_new;
+            const float m_use = m_run[m] == -INFINITY ? 0.f : m_run[m];
 #pragma unroll
             for (int t = 0; t < 2; ++t)
 #pragma unroll
@@ -404,10 +449,7 @@ __global__ __launch_bounds__(256, 1) void latent_attn_kernel(const AttnArgs a) {
 
 template <int NCT, int MT>
 int launch_latent_attn(const AttnArgs& a, hipStream_t st) {
-    constexpr int TILEB = 32 * NCT * 128;
-    constexpr int NST = 3 * TILEB <= 112 * 1024 ? 3 : 2;
-    constexpr int LDS = NST * TILEB + 2 * MT * 2 * 1024 + LA_BT * 4;
-    static_assert(LDS <= 160 * 1024, "LDS of a CU");
+    constexpr int LDS = LaCfg<NCT, MT>::LDS;
     auto kern = latent_attn_kernel<NCT, MT>;
     GLM_SET_MAX_LDS(kern, LDS, "glm_latent_attn");
     const int64_t grid = (int64_t)a.n_tiles * a.n_hg * a.nsplit;
@@ -491,80 +533,79 @@ __global__ __launch_bounds__(256) void latent_attn_f32_kernel(const AttnArgs a, 
 }
 
 // ---------------------------------------------------------------------------------------------------------------------------
+// ctx = (sum over the KV splits, each brought to the common maximum) / (mass of the splits + the sink's): one wave per (token, head)
+__global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, const float* __restrict__ sink,
+                                                           int nsplit, bf16_t* __restrict__ ctx, int64_t rows, int H, int rp) {
+    const int lane = threadIdx.x & 63;
+    const int64_t grow = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (grow >= rows) return;
+    float m = -INFINITY, l = 0.f;
+    if (lane < nsplit) {
+        m = part_ml[(grow * nsplit + lane) * 2];
+        l = part_ml[(grow * nsplit + lane) * 2 + 1];
+    }
+    const float sk = sink[grow % H] * LOG2E;
+    const float M = fmaxf(wave_max(m), sk);
+    const float e = l > 0.f ? __builtin_amdgcn_exp2f(m - M) : 0.f;
+    const float f = e / (wave_sum(l * e) + __builtin_amdgcn_exp2f(sk - M));  // 0: an empty split, its sums were never written
+    for (int k = lane * 4; k < rp; k += 256) {
+        const float* p = part_o + grow * nsplit * rp + k;
+        f32x4_t o = {0.f, 0.f, 0.f, 0.f};
+        for (int s0 = 0; s0 < nsplit; s0 += 8) {
+            f32x4_t x[8];
+#pragma unroll
+            for (int j = 0; j < 8; ++j) x[j] = *reinterpret_cast<const f32x4_t*>(p + (int64_t)min(s0 + j, nsplit - 1) * rp);
+#pragma unroll
+            for (int j = 0; j < 8; ++j) {
+                const float fs = s0 + j < nsplit ? __shfl(f, s0 + j, 64) : 0.f;
+                if (fs != 0.f) {
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) o[i] += fs * x[j][i];
+                }
+            }
+        }
+        *reinterpret_cast<u32x2_t*>(ctx + grow * rp + k) = u32x2_t{pack2bf(o[0], o[1]), pack2bf(o[2], o[3])};
+    }
+}
+
 struct UpArgs {
-    const bf16_t* ctx;
-    const float *part_o, *part_ml, *sink;
-    int nsplit;
+    const bf16_t* ctx;   // [Ta, H, rp]
     const bf16_t* wuv;   // [H, vdimp, rp]
     bf16_t* out;         // [T, ldo], head h at h*vdimp
     int64_t ldo, Ta;
     int H, vdimp, rp;
 };
 
-// out[t, h, :] = W_uv[h] . ctx[t, h, :]: 16 tokens and up to 64 value rows of one head per workgroup (16 rows per wave)
+// out[t, h, :] = W_uv[h] . ctx[t, h, :]: per wave 16 tokens and 16 value rows of one head, operands straight from memory, eight
+// K steps of both in flight
 __global__ __launch_bounds__(256) void latent_up_kernel(const UpArgs a) {
-    extern __shared__ __attribute__((aligned(16))) char smem_up[];
-    bf16_t* sx = reinterpret_cast<bf16_t*>(smem_up);  // [16][pitch]
-    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+    const int lane = threadIdx.x & 63, wid = threadIdx.x >> 6;
     const int c = lane & 15, g = lane >> 4;
-    const int kp = (a.rp + 31) & ~31, pitch = kp + 8;
-    const int h = blockIdx.x % a.H, vc = blockIdx.x / a.H;
-    const int64_t t0 = (int64_t)blockIdx.y * 16;
-    const int nk4 = kp / 4;
-    __shared__ float s_f[16][64];  // per token and split: weight of the split's sums
-    if (a.nsplit > 1) {
-        if (tid < 16) {
-            const int64_t t = t0 + tid;
-            if (t < a.Ta) {
-                const float* ml = a.part_ml + (t * a.H + h) * a.nsplit * 2;
-                const float sk = a.sink[h] * LOG2E;
-                float M = sk, L = 0.f;
-                for (int s = 0; s < a.nsplit; ++s) M = fmaxf(M, ml[2 * s]);
-                for (int s = 0; s < a.nsplit; ++s) L += ml[2 * s + 1] > 0.f ? ml[2 * s + 1] * __builtin_amdgcn_exp2f(ml[2 * s] - M) : 0.f;
-                L += __builtin_amdgcn_exp2f(sk - M);
-                for (int s = 0; s < a.nsplit; ++s) s_f[tid][s] = ml[2 * s + 1] > 0.f ? __builtin_amdgcn_exp2f(ml[2 * s] - M) / L : 0.f;
-            }
-        }
-        __syncthreads();
-    }
-    for (int i = tid; i < 16 * nk4; i += 256) {
-        const int r = i / nk4, k = (i % nk4) * 4;
-        const int64_t t = t0 + r;
-        u32x2_t v = {0, 0};
-        if (t < a.Ta && k < a.rp) {
-            const int64_t grow = t * a.H + h;
-            if (a.nsplit == 1) {
-                v = *reinterpret_cast<const u32x2_t*>(a.ctx + grow * a.rp + k);
-            } else {
-                f32x4_t o = {0.f, 0.f, 0.f, 0.f};
-                for (int s = 0; s < a.nsplit; ++s) {
-                    const float f = s_f[r][s];
-                    if (f != 0.f) {  // an empty split's sums were never written
-                        const f32x4_t x = *reinterpret_cast<const f32x4_t*>(a.part_o + (grow * a.nsplit + s) * a.rp + k);
-#pragma unroll
-                        for (int j = 0; j < 4; ++j) o[j] += f * x[j];
-                    }
-                }
-                v = u32x2_t{pack2bf(o[0], o[1]), pack2bf(o[2], o[3])};
-            }
-        }
-        *reinterpret_cast<u32x2_t*>(sx + r * pitch + k) = v;
-    }
-    __syncthreads();
-    const int v0 = vc * 64 + wid * 16;
-    if (v0 >= a.vdimp) return;
-    const int ar = min(v0 + c, a.vdimp - 1);
+    const int nv = (a.vdimp + 15) / 16;
+    const int item = blockIdx.x * 4 + wid;
+    if (item >= a.H * nv) return;
+    const int h = item / nv, v0 = (item % nv) * 16;
+    const int64_t t = (int64_t)blockIdx.y * 16 + c;
+    const bf16_t* wr = a.wuv + ((int64_t)h * a.vdimp + min(v0 + c, a.vdimp - 1)) * a.rp;
+    const bf16_t* xr = a.ctx + (min(t, a.Ta - 1) * a.H + h) * a.rp;
     f32x4_t acc = {0.f, 0.f, 0.f, 0.f};
-    const bf16_t* wr = a.wuv + ((int64_t)h * a.vdimp + ar) * a.rp;
-    for (int k = 8 * g; k < kp; k += 32) {
-        u32x4_t av = {0, 0, 0, 0};
-        if (k < a.rp) av = *reinterpret_cast<const u32x4_t*>(wr + k);
-        const u32x4_t bv = *reinterpret_cast<const u32x4_t*>(sx + c * pitch + k);
-        acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, av), __builtin_bit_cast(bf16x8_t, bv), acc, 0, 0, 0);
+    for (int k0 = 0; k0 < a.rp; k0 += 256) {
+        u32x4_t av[8], bv[8];
+#pragma unroll
+        for (int i = 0; i < 8; ++i) {
+            const int k = k0 + 32 * i + 8 * g;
+            const bool ok = k < a.rp;
+            av[i] = *reinterpret_cast<const u32x4_t*>(wr + (ok ? k : 0));
+            bv[i] = *reinterpret_cast<const u32x4_t*>(xr + (ok ? k : 0));
+            if (!ok) av[i] = bv[i] = u32x4_t{0, 0, 0, 0};
+        }
+#pragma unroll
+        for (int i = 0; i < 8; ++i)
+            acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, av[i]), __builtin_bit_cast(bf16x8_t, bv[i]), acc, 0, 0, 0);
     }
     const int v = v0 + 4 * g;
-    if (t0 + c < a.Ta && v < a.vdimp)
-        *reinterpret_cast<u32x2_t*>(a.out + (t0 + c) * a.ldo + (int64_t)h * a.vdimp + v) = u32x2_t{pack2bf(acc[0], acc[1]), pack2bf(acc[2], acc[3])};
+    if (t < a.Ta && v < a.vdimp)
+        *reinterpret_cast<u32x2_t*>(a.out + t * a.ldo + (int64_t)h * a.vdimp + v) = u32x2_t{pack2bf(acc[0], acc[1]), pack2bf(acc[2], acc[3])};
 }
 
 int pick_nct(int rp) {
@@ -658,16 +699,25 @@ extern "C" int glm_latent_attn(const void* qa, const void* cache, int64_t n_bloc
     }
 }
 
-extern "C" int glm_latent_up(const void* ctx, const float* part_o, const float* part_ml, const float* sink, int nsplit, const void* wuv, void* out,
-                             int64_t ldo, int64_t Ta, int H, int vdimp, int rp, glm_stream_t stream) {
-    GLM_CHECK_ARG(sink && wuv && out && Ta >= 0 && H > 0 && vdimp > 0 && vdimp % 8 == 0 && rp % 8 == 0 && ldo >= (int64_t)H * vdimp && ldo % 4 == 0 && nsplit >= 1 &&
-                      nsplit <= 64 && (nsplit > 1 ? (part_o && part_ml) : ctx != nullptr), GLM_ERR_INVALID, "glm_latent_up: bad shape Ta=%ld H=%d vdimp=%d", (long)Ta, H, vdimp);
+extern "C" int glm_latent_merge(const float* part_o, const float* part_ml, const float* sink, int nsplit, void* ctx, int64_t Ta, int H, int rp,
+                                glm_stream_t stream) {
+    GLM_CHECK_ARG(part_o && part_ml && sink && ctx && nsplit >= 1 && nsplit <= 64 && Ta >= 0 && H > 0 && rp > 0 && rp % 8 == 0, GLM_ERR_INVALID,
+                  "glm_latent_merge: bad shape Ta=%ld H=%d rp=%d splits=%d", (long)Ta, H, rp, nsplit);
+    GLM_CHECK_ARG(Ta * H < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_latent_merge: too many rows");
+    if (Ta == 0) return GLM_OK;
+    hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)((Ta * H + 3) / 4)), dim3(256), 0, glm_s(stream), part_o, part_ml, sink, nsplit, (bf16_t*)ctx, Ta * H, H, rp);
+    GLM_CHECK_LAUNCH("glm_latent_merge");
+    return GLM_OK;
+}
+
+extern "C" int glm_latent_up(const void* ctx, const void* wuv, void* out, int64_t ldo, int64_t Ta, int H, int vdimp, int rp, glm_stream_t stream) {
+    GLM_CHECK_ARG(ctx && wuv && out && Ta >= 0 && H > 0 && vdimp > 0 && vdimp % 8 == 0 && rp > 0 && rp % 8 == 0 && ldo >= (int64_t)H * vdimp && ldo % 4 == 0 &&
+                      glm_aligned16(ctx) && glm_aligned16(wuv), GLM_ERR_INVALID, "glm_latent_up: bad shape Ta=%ld H=%d vdimp=%d", (long)Ta, H, vdimp);
     GLM_CHECK_ARG((Ta + 15) / 16 <= 65535, GLM_ERR_UNSUPPORTED, "glm_latent_up: too many rows");
     if (Ta == 0) return GLM_OK;
-    UpArgs a = {(const bf16_t*)ctx, part_o, part_ml, sink, nsplit, (const bf16_t*)wuv, (bf16_t*)out, ldo, Ta, H, vdimp, rp};
-    const size_t lds = (size_t)16 * (((rp + 31) & ~31) + 8) * 2;
-    GLM_CHECK_ARG(lds <= 56 * 1024, GLM_ERR_UNSUPPORTED, "glm_latent_up: latent of %d columns", rp);
-    hipLaunchKernelGGL(latent_up_kernel, dim3((unsigned)(H * ((vdimp + 63) / 64)), (unsigned)((Ta + 15) / 16)), dim3(256), lds, glm_s(stream), a);
+    UpArgs a = {(const bf16_t*)ctx, (const bf16_t*)wuv, (bf16_t*)out, ldo, Ta, H, vdimp, rp};
+    const int items = H * ((vdimp + 15) / 16);
+    hipLaunchKernelGGL(latent_up_kernel, dim3((unsigned)((items + 3) / 4), (unsigned)((Ta + 15) / 16)), dim3(256), 0, glm_s(stream), a);
     GLM_CHECK_LAUNCH("glm_latent_up");
     return GLM_OK;
 }

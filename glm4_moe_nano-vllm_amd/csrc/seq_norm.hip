@@ -5,8 +5,8 @@
 //     h     = rms(x_out) * g_pre              (optional)
 //     h     = h + conv(h)                     (optional; depthwise, causal, TAPS taps)
 //
-// in ONE launch.  gfx950 only.  Roofline: HBM — x_in and y are read once from HBM (the second pass over a row hits the L2),
-// x_out and h written once.
+// in ONE launch.  gfx950 only.  Roofline: HBM — x_in and y are read once, x_out and h written once (seq_norm_stream_kernel; the
+// two-pass seq_norm_kernel, which reads a row again, is for very wide rows and very long convolutions).
 //
 // The convolution needs the h of the TAPS-1 tokens before.  Inside a step's rows they are RECOMPUTED from x_in and y (a halo
 // of TAPS-1 rows per workgroup: no hand-off between workgroups, x_out goes to another buffer than x_in); for tokens of
@@ -210,8 +210,200 @@ __global__ __launch_bounds__(SN_NT) void seq_norm_kernel(const SeqNormArgs a) {
     }
 }
 
+// ---- one pass: every thread owns eight columns and keeps its gains, taps and the convolution's history in registers; the rows of
+// the workgroup's run go by one after the other, the next row's loads in flight.  The reduction over a row's x_out^2 and the one
+// over the next row's y^2 share a barrier. ----
+template <int CTRL, int ROWS>
+__device__ __forceinline__ float sn_dpp_add(float v) {
+    return v + __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, ROWS, 0xf, false));
+}
+__device__ __forceinline__ float sn_wave_sum(float v) {  // the sum over the wave, in lane 63
+    v = sn_dpp_add<0x111, 0xf>(v);  // row_shr:1
+    v = sn_dpp_add<0x112, 0xf>(v);
+    v = sn_dpp_add<0x114, 0xf>(v);
+    v = sn_dpp_add<0x118, 0xf>(v);
+    v = sn_dpp_add<0x142, 0xa>(v);  // row_bcast:15
+    v = sn_dpp_add<0x143, 0xc>(v);  // row_bcast:31
+    return v;
+}
+
+struct Row8 {
+    f32x4_t a, b;
+};
+__device__ __forceinline__ Row8 sn_ld8f(const float* p) { return {*reinterpret_cast<const f32x4_t*>(p), *reinterpret_cast<const f32x4_t*>(p + 4)}; }
+__device__ __forceinline__ void sn_st8f(float* p, const Row8& v) {
+    *reinterpret_cast<f32x4_t*>(p) = v.a;
+    *reinterpret_cast<f32x4_t*>(p + 4) = v.b;
+}
+__device__ __forceinline__ void sn_st8(void* base, int64_t off, int f32, const Row8& v) {
+    if (f32) sn_st8f(reinterpret_cast<float*>(base) + off, v);
+    else
+        *reinterpret_cast<u32x4_t*>(reinterpret_cast<bf16_t*>(base) + off) =
+            u32x4_t{pack2bf(v.a[0], v.a[1]), pack2bf(v.a[2], v.a[3]), pack2bf(v.b[0], v.b[1]), pack2bf(v.b[2], v.b[3])};
+}
+__device__ __forceinline__ float sn_sumsq8(const Row8& v) { return sn_sumsq(v.a) + sn_sumsq(v.b); }
+
+template <int TAPS, int NT>
+__global__ __launch_bounds__(NT) void seq_norm_stream_kernel(const SeqNormArgs a, int tr) {
+    constexpr int HALO = TAPS - 1, NW = NT / 64;
+    __shared__ float s_red[2][2][NW];
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+    const int c = tid * 8;
+    const bool on = c < a.wp;
+    const int64_t r0 = (int64_t)blockIdx.x * tr, r1 = min(r0 + tr, a.T);
+    const float inv_w = 1.0f / (float)a.width;
+    int s = 0, qs = 0, qe = 0;
+    int64_t lo = r0;
+    if constexpr (TAPS > 1) {
+        s = a.seq_of[r0];
+        qs = a.q_start[s];
+        qe = a.q_start[s + 1];
+        lo = max(r0 - HALO, (int64_t)qs);
+    }
+    const Row8 zero = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+    Row8 gq = zero, gp = zero, w[TAPS], hist[TAPS];
+    if (on) {
+        if (a.y) gq = sn_ld8f(a.g_post + c);
+        if (a.g_pre) gp = sn_ld8f(a.g_pre + c);
+        if constexpr (TAPS > 1) {
+#pragma unroll
+            for (int j = 0; j < TAPS; ++j) w[j] = sn_ld8f(a.conv_w + (int64_t)j * a.wp + c);
+        }
+    }
+    if (TAPS > 1 && !on) {
+#pragma unroll
+        for (int j = 0; j < TAPS; ++j) w[j] = zero;
+    }
+#pragma unroll
+    for (int j = 0; j < TAPS; ++j) hist[j] = zero;
+    auto load_x = [&](int64_t r) { return on ? sn_ld8f(a.x_in + (a.row_index ? a.row_index[r] : r) * a.ldx + c) : zero; };
+    auto load_y = [&](int64_t r) -> Row8 {
+        if (!a.y || !on) return zero;
+        const int64_t row = a.row_index ? a.row_index[r] : r;
+        if (!a.y_f32) {
+            const u32x4_t u = *reinterpret_cast<const u32x4_t*>(reinterpret_cast<const bf16_t*>(a.y) + row * a.ldy + c);
+            return {{bflo(u[0]), bfhi(u[0]), bflo(u[1]), bfhi(u[1])}, {bflo(u[2]), bfhi(u[2]), bflo(u[3]), bfhi(u[3])}};
+        }
+        return {sn_load_y(a, row, c), sn_load_y(a, row, c + 4)};
+    };
+    // sums over the workgroup of two values per thread
+    auto reduce2 = [&](float u, float v, int par, float& su, float& sv) {
+        u = sn_wave_sum(u);
+        v = sn_wave_sum(v);
+        if (lane == 63) {
+            s_red[par][0][wid] = u;
+            s_red[par][1][wid] = v;
+        }
+        __syncthreads();
+        su = sv = 0.f;
+#pragma unroll
+        for (int i = 0; i < NW; ++i) {
+            su += s_red[par][0][i];
+            sv += s_red[par][1][i];
+        }
+    };
+    Row8 x = load_x(lo), y = load_y(lo), xn = zero, yn = zero;
+    float ry = 0.f, su, sv;
+    int par = 0;
+    if (a.y) {
+        reduce2(sn_sumsq8(y), 0.f, par, su, sv);
+        ry = 1.0f / sqrtf(su * inv_w + a.eps);
+        par ^= 1;
+    }
+    for (int64_t r = lo; r < r1; ++r) {
+        const bool more = r + 1 < r1;
+        if (more) {
+            xn = load_x(r + 1);
+            yn = load_y(r + 1);
+        }
+        if (a.y) {
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                x.a[i] = x.a[i] + y.a[i] * ry * gq.a[i];
+                x.b[i] = x.b[i] + y.b[i] * ry * gq.b[i];
+            }
+        }
+        if (r >= r0 && on) {
+            if (a.x_out) sn_st8f(a.x_out + r * a.ldx + c, x);
+            if (a.x_cast) sn_st8(a.x_cast, r * a.ldc + c, a.act_f32, x);
+        }
+        reduce2(sn_sumsq8(x), more ? sn_sumsq8(yn) : 0.f, par, su, sv);
+        par ^= 1;
+        if (a.g_pre) {
+            const float rx = 1.0f / sqrtf(su * inv_w + a.eps);
+            Row8 h, o;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                h.a[i] = x.a[i] * rx * gp.a[i];
+                h.b[i] = x.b[i] * rx * gp.b[i];
+            }
+            o = h;
+            if constexpr (TAPS > 1) {
+                if (r == qe) {  // the next sequence's portion begins
+                    s = a.seq_of[r];
+                    qs = a.q_start[s];
+                    qe = a.q_start[s + 1];
+                }
+                const int64_t sin = min(max((int64_t)a.state_in[s], (int64_t)0), a.n_state - 1);
+                if (r == qs) {
+                    const int p = a.pos[r];
+#pragma unroll
+                    for (int k = 1; k < TAPS; ++k)
+                        hist[k - 1] = (on && p - k >= 0) ? sn_ld8f(a.state + (sin * HALO + (HALO - k)) * a.wp + c) : zero;
+                }
+                Row8 acc = zero;
+#pragma unroll
+                for (int k = HALO; k >= 1; --k)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) {
+                        acc.a[i] = acc.a[i] + w[TAPS - 1 - k].a[i] * hist[k - 1].a[i];
+                        acc.b[i] = acc.b[i] + w[TAPS - 1 - k].b[i] * hist[k - 1].b[i];
+                    }
+#pragma unroll
+                for (int i = 0; i < 4; ++i) {
+                    o.a[i] = h.a[i] + (acc.a[i] + w[TAPS - 1].a[i] * h.a[i]);
+                    o.b[i] = h.b[i] + (acc.b[i] + w[TAPS - 1].b[i] * h.b[i]);
+                }
+                const int64_t so = a.state_out[s];
+                const int e = qe - 1 - (int)r;  // tokens of the portion behind this one
+                if (r >= r0 && e < HALO && on && so >= 0 && so < a.n_state && a.pos[r] >= 0) {
+                    sn_st8f(a.state + (so * HALO + (HALO - 1 - e)) * a.wp + c, h);
+                    if (e == 0)  // a portion shorter than the history: the older inputs move up
+                        for (int i = 0; i < HALO - (qe - qs); ++i)
+                            sn_st8f(a.state + (so * HALO + i) * a.wp + c, sn_ld8f(a.state + (sin * HALO + i + (qe - qs)) * a.wp + c));
+                }
+#pragma unroll
+                for (int k = HALO; k >= 2; --k) hist[k - 1] = hist[k - 2];
+                hist[0] = h;
+            }
+            if (r >= r0 && on) sn_st8(a.h, r * a.ldh + c, a.act_f32, o);
+        }
+        if (a.y) ry = 1.0f / sqrtf(sv * inv_w + a.eps);
+        x = xn;
+        y = yn;
+    }
+}
+
+template <int TAPS, int NT>
+int launch_seq_norm_stream(const SeqNormArgs& a, hipStream_t st) {
+    // decode: one row per workgroup; else runs of rows long enough to spread the halo and the register setup, short enough
+    // to fill the chip
+    int tr = a.T <= 512 ? 1 : (int)((a.T + 1023) / 1024);
+    if (tr > 1) tr = tr < 8 ? 8 : tr > 32 ? 32 : tr;
+    hipLaunchKernelGGL((seq_norm_stream_kernel<TAPS, NT>), dim3((unsigned)((a.T + tr - 1) / tr)), dim3(NT), 0, st, a, tr);
+    GLM_CHECK_LAUNCH("glm_seq_norm");
+    return GLM_OK;
+}
+
 template <int TAPS>
 int launch_seq_norm(const SeqNormArgs& a, hipStream_t st) {
+    if constexpr (TAPS <= 8) {
+        if (a.wp <= 512) return launch_seq_norm_stream<TAPS, 64>(a, st);
+        if (a.wp <= 1024) return launch_seq_norm_stream<TAPS, 128>(a, st);
+        if (a.wp <= 2048) return launch_seq_norm_stream<TAPS, 256>(a, st);
+        if (a.wp <= 4096) return launch_seq_norm_stream<TAPS, 512>(a, st);
+        if (TAPS <= 4 && a.wp <= 8192) return launch_seq_norm_stream<TAPS, (TAPS <= 4 ? 1024 : 512)>(a, st);
+    }
     // few rows (decode): one row per workgroup; many: 16 rows share a halo
     if (a.T <= 512) hipLaunchKernelGGL((seq_norm_kernel<TAPS, 1>), dim3((unsigned)a.T), dim3(SN_NT), 0, st, a);
     else hipLaunchKernelGGL((seq_norm_kernel<TAPS, 16>), dim3((unsigned)((a.T + 15) / 16)), dim3(SN_NT), 0, st, a);

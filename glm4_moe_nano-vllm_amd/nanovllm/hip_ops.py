@@ -154,8 +154,8 @@ _SIGNATURES = {
     "glm_latent_attn": (c_int, [c_void_p, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p,
         c_void_p, c_void_p, c_int64, c_int64, c_int, c_int, c_int, c_int, c_float, c_void_p, c_int, c_void_p, c_void_p,
         c_void_p, c_int, c_void_p]),
-    "glm_latent_up": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_void_p, c_int64, c_int64,
-        c_int, c_int, c_int, c_void_p]),
+    "glm_latent_merge": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int64, c_int, c_int, c_void_p]),
+    "glm_latent_up": (c_int, [c_void_p, c_void_p, c_void_p, c_int64, c_int64, c_int, c_int, c_int, c_void_p]),
     "glm_window_attn_prefill": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_void_p,
         c_void_p, c_void_p, c_void_p, c_int, c_int, c_int64, c_int64, c_int, c_int, c_int, c_int, c_float, c_void_p,
         c_void_p]),
@@ -1374,7 +1374,7 @@ def latent_attn(qa: torch.Tensor, cache: torch.Tensor, tile_tok: torch.Tensor, t
         assert t.dtype == torch.int32
     assert pos.numel() >= Ta and seq_of.numel() >= Ta and out.stride(1) == 1 and out.shape[0] >= Ta and out.shape[1] == H * vdimp
     lib, f32 = load_library(), _is_f32(qa.dtype)
-    ctx = part_o = part_ml = None
+    part_o = part_ml = None
     ns = 1
     if not f32:
         # enough (tile, head group, KV split) workgroups to cover the chip, at least four 32-key tiles per split
@@ -1382,9 +1382,8 @@ def latent_attn(qa: torch.Tensor, cache: torch.Tensor, tile_tok: torch.Tensor, t
         wgs = tile_tok.numel() * -(-H // rows)
         keys = min(window + tokens_per_tile, block_tables.shape[1] * bs)
         ns = num_splits or max(1, min(64, 512 // max(1, wgs), -(-keys // 128)))
-    if ns == 1:
-        ctx = torch.empty((Ta, H, rp), dtype=qa.dtype, device=qa.device)
-    else:
+    ctx = torch.empty((Ta, H, rp), dtype=qa.dtype, device=qa.device)
+    if ns > 1:
         part_o = torch.empty((Ta * H, ns, rp), dtype=torch.float32, device=qa.device)
         part_ml = torch.empty((Ta * H, ns, 2), dtype=torch.float32, device=qa.device)
     _check(lib.glm_latent_attn(_p(qa), _p(cache), n_blocks, bs, _p(tile_tok), _p(tile_n), tile_tok.numel(), tokens_per_tile, _p(pos),
@@ -1393,8 +1392,9 @@ def latent_attn(qa: torch.Tensor, cache: torch.Tensor, tile_tok: torch.Tensor, t
     if f32:
         batched_gemm_f32(ctx.transpose(0, 1), wuv, out[:Ta].view(Ta, H, vdimp).transpose(0, 1))
         return
-    _check(lib.glm_latent_up(_p(ctx), _p(part_o), _p(part_ml), _p(sink), ns, _p(wuv), _p(out), out.stride(0), Ta, H, vdimp, rp,
-                             _stream()), "glm_latent_up")
+    if ns > 1:
+        _check(lib.glm_latent_merge(_p(part_o), _p(part_ml), _p(sink), ns, _p(ctx), Ta, H, rp, _stream()), "glm_latent_merge")
+    _check(lib.glm_latent_up(_p(ctx), _p(wuv), _p(out), out.stride(0), Ta, H, vdimp, rp, _stream()), "glm_latent_up")
 
 
 def window_attn_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, out: torch.Tensor, q_start: torch.Tensor,

@@ -530,15 +530,17 @@ int glm_latent_gather(const void* cache, int64_t n_slots, const int32_t* slots, 
 /* attn: query row (t, h) sees the latents of positions (pos[t] - window, pos[t]] of its sequence; softmax with the extra mass
  * exp(sink[h]).  Tiles: tile i covers tile_n[i] <= tokens_per_tile consecutive rows of one sequence from tile_tok[i]; tokens x
  * heads of a tile <= glm_latent_attn_max_rows(rp).  nsplit == 1: ctx [Ta, H, rp] normalised (bf16 / fp32); else part_o
- * [Ta*H, nsplit, rp], part_ml [Ta*H, nsplit, 2] for glm_latent_up.  fp32: tiles unused, nsplit 1.
+ * [Ta*H, nsplit, rp], part_ml [Ta*H, nsplit, 2] for glm_latent_merge, which forms ctx.  fp32: tiles unused, nsplit 1.
  * up: out[t, h*vdimp ..] = W_uv[h] ctx[t, h, :] (wuv [H, vdimp, rp]).                                                         */
 int glm_latent_attn_max_rows(int rp);
 int glm_latent_attn(const void* qa, const void* cache, int64_t n_blocks, int block_size, const int32_t* tile_tok,
                     const int32_t* tile_n, int n_tiles, int tokens_per_tile, const int32_t* pos, const int32_t* seq_of,
                     const int32_t* block_tables, int64_t bt_stride, int64_t Ta, int H, int rank, int rp, int window, float scale,
                     const float* sink, int nsplit, void* ctx, float* part_o, float* part_ml, int act_f32, glm_stream_t stream);
-int glm_latent_up(const void* ctx, const float* part_o, const float* part_ml, const float* sink, int nsplit, const void* wuv,
-                  void* out, int64_t ldo, int64_t Ta, int H, int vdimp, int rp, glm_stream_t stream);
+int glm_latent_merge(const float* part_o, const float* part_ml, const float* sink, int nsplit, void* ctx, int64_t Ta, int H, int rp,
+                     glm_stream_t stream);
+int glm_latent_up(const void* ctx, const void* wuv, void* out, int64_t ldo, int64_t Ta, int H, int vdimp, int rp,
+                  glm_stream_t stream);
 /* Prompts and long portions, bf16: q rows [q_start[s], q_start[s+1]) against expanded k / v rows [k_start[s], k_start[s+1]) — the
  * portion's own tokens last, in front of them the history the window still reaches.  Head h at h*dk (q, k) / h*dv (v, out).
  * Tiles of 128 query rows: (sequence, first row inside the portion).  dk, dv <= 256, multiples of 8.                          */
