@@ -6,8 +6,11 @@ enum GemmMode : int {
     GEMM_PLAIN = 0,   // y[r,n] = bf16(acc + bias[n])                              (a5, a10)
     GEMM_GATEUP = 1,  // act[r,i] = bf16(bf16(silu(bf16(g))) * bf16(u)), W rows gate|up  (a13)
     GEMM_DOWN = 2,    // y[r,n] = bf16(bf16(acc) * scale[r]) for groups < n_scaled    (a12/a13)
-    GEMM_ACT = 3,     // gemm_largem only: GEMM_PLAIN followed by p.act and / or an fp32 output row (p.yf) — its own instantiation,
-                      // so that the plain kernel's epilogue stays as it is; the decode bodies take p.act / p.yf in GEMM_PLAIN
+    // gemm_largem only.  GEMM_PLAIN followed by p.act and / or fp32 output rows (p.yf), and its common case without anything left
+    // to decide in the epilogue: their own instantiations, so that the plain kernel's epilogue stays as it is.  (The decode
+    // bodies take p.act / p.yf in GEMM_PLAIN.)
+    GEMM_ACT = 3,
+    GEMM_XIELU = 4,  // xIELU, bf16 rows
 };
 
 // activation on the fp32 accumulator of a projection (after the bias)
@@ -22,17 +25,14 @@ __device__ __forceinline__ float glm_act_precise(const GlmAct& t, float z) {
     if (t.kind == GLM_ACT_SOFTCAP) return t.a * tanhf(z / t.a);
     return z;
 }
-// ... for outputs that are rounded to bf16 right away: exp on the hardware exp2 unit, its absolute error (1e-7) far below the
-// rounding of the result; a series where exp(z) - 1 - z cancels
+// ... for outputs that are rounded to bf16 right away: exp on the hardware exp2 unit.  Near zero exp(z) - 1 - z cancels to an
+// absolute error of 1e-7 beside the z / 2 that is added to it.
+__device__ __forceinline__ float glm_xielu_fast(float a, float b, float z) {
+    const float neg = b * (__builtin_amdgcn_exp2f(1.4426950408889634f * fminf(z, 0.f)) - 1.0f - z);
+    return (z > 0.f ? a * z * z : neg) + 0.5f * z;
+}
 __device__ __forceinline__ float glm_act_fast(const GlmAct& t, float z) {
-    if (t.kind == GLM_ACT_XIELU) {
-        const float zn = fminf(z, 0.f);
-        const float far = __builtin_amdgcn_exp2f(1.4426950408889634f * zn) - 1.0f - zn;
-        const float near = zn * zn * (0.5f + zn * (1.0f / 6.0f + zn * (1.0f / 24.0f)));
-        const float e = zn > -0.0625f ? near : far;
-        return z > 0.f ? t.a * z * z + 0.5f * z : t.b * e + 0.5f * z;
-    }
-    return glm_act_precise(t, z);
+    return t.kind == GLM_ACT_XIELU ? glm_xielu_fast(t.a, t.b, z) : glm_act_precise(t, z);
 }
 
 struct GemmParams {

@@ -306,7 +306,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
     constexpr bool PARK = C::PH8 && (VAR & LM_PARK) != 0 && (VAR & LM_WIDEST) != 0 && (VAR & LM_NOSTORE) == 0;
     constexpr int PARK_N = 4;
     constexpr bool CONT = (VAR & LM_CONT) != 0 && C::PH8 && (VAR & LM_QW) != 0 && (VAR & LM_RFIRST) != 0 && (VAR & LM_P3X) == 0 &&
-                          !PARK && !C::A8 && !C::W8 && !WSCALE && MODE != GEMM_PLAIN && MODE != GEMM_ACT && (VAR & LM_EPIORD) != 0;
+                          !PARK && !C::A8 && !C::W8 && !WSCALE && (MODE == GEMM_GATEUP || MODE == GEMM_DOWN) && (VAR & LM_EPIORD) != 0;
     int* sh = reinterpret_cast<int*>(smem + C::NSTAGE * C::STAGE - ((C::ALIAS_SH || PARK) ? 16 : 0));
     const int tid = threadIdx.x, lane = tid & 63;
     const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -1554,8 +1554,9 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
                     } else {
                         float a = acc[t][mt][r];
                         if constexpr (WSCALE) a *= wsv[t][r];
-                        if ((MODE == GEMM_PLAIN || MODE == GEMM_ACT) && p.bias) a += bf2f(p.bias[min(ncol_w + 16 * t + 4 * g4 + r, p.N - 1)]);
+                        if ((MODE == GEMM_PLAIN || MODE == GEMM_ACT || MODE == GEMM_XIELU) && p.bias) a += bf2f(p.bias[min(ncol_w + 16 * t + 4 * g4 + r, p.N - 1)]);
                         if (scaled) a = rbf(a) * sc;
+                        if (MODE == GEMM_XIELU) a = glm_xielu_fast(p.act.a, p.act.b, a);
                         if (MODE == GEMM_ACT) a = p.yf != nullptr ? glm_act_precise(p.act, a) : glm_act_fast(p.act, a);
                         o[r] = a;
                     }
@@ -1702,7 +1703,7 @@ int launch_largem(const GemmParams& p, hipStream_t st) {
     const int64_t avg_rows = (p.R_hint > 0 ? p.R_hint : p.R) / (p.G > 0 ? p.G : 1);
     // ... and a projection onto <= 128 columns (the router logits at prefill: N = E = 64) is one column tile however the rows
     // are cut, so its parallelism is its row-block count: 128-row blocks (75.8 -> 55.1 us at T = 16384)
-    const bool use_b = ch == 2 || (ch == 0 && avg_rows >= 192 && !((MODE == GEMM_PLAIN || MODE == GEMM_ACT) && p.offs == nullptr && p.N <= 128));
+    const bool use_b = ch == 2 || (ch == 0 && avg_rows >= 192 && !((MODE == GEMM_PLAIN || MODE == GEMM_ACT || MODE == GEMM_XIELU) && p.offs == nullptr && p.N <= 128));
     // the lean load phase addresses x and the group's weights through 32-bit buffer offsets and has no K tail path
     // default (tools/largem_ab.py, one process, T = 16384): the quadrant-phase loop with 4 x 2-tile quadrants and the
     // fragment reads of a load interval issued before its DMA, no priority flips (86531: +1 % over 86019), epilogue
@@ -1721,7 +1722,7 @@ int launch_largem(const GemmParams& p, hipStream_t st) {
             glm_set_error("gemm_largem(fp8 weights): shape not covered (K=%d N=%d ldw=%ld)", p.K, p.N, (long)p.ldw);
             return GLM_ERR_UNSUPPORTED;
         }
-        if constexpr (MODE == GEMM_PLAIN || MODE == GEMM_ACT) {
+        if constexpr (MODE == GEMM_PLAIN || MODE == GEMM_ACT || MODE == GEMM_XIELU) {
             glm_set_error("gemm_largem(fp8 weights): only the grouped expert projections are quantised");
             return GLM_ERR_UNSUPPORTED;
         } else {
@@ -1837,6 +1838,7 @@ int glm_launch_gemm_largem(int mode, const GemmParams& p, hipStream_t st) {
                   p.K, p.N);
     if (mode == GEMM_GATEUP) return launch_largem<GEMM_GATEUP>(p, st);
     if (mode == GEMM_DOWN) return launch_largem<GEMM_DOWN>(p, st);
+    if (mode == GEMM_ACT && p.yf == nullptr && p.act.kind == GLM_ACT_XIELU) return launch_largem<GEMM_XIELU>(p, st);
     if (mode == GEMM_ACT) return launch_largem<GEMM_ACT>(p, st);
     return launch_largem<GEMM_PLAIN>(p, st);
 }

@@ -31,7 +31,7 @@ struct SeqNormArgs {
     int64_t slab_stride;
     const float* g_post;      // [wp]
     const float* g_pre;       // [wp] or nullptr
-    const float* conv_w;      // [TAPS][wp] or nullptr
+    const bf16_t* conv_w;     // [TAPS][wp] or nullptr (bf16 in either activation dtype: the checkpoint's values)
     float* state;             // [state rows][TAPS-1][wp]
     const int32_t* pos;       // [T] position of the row in its sequence (< 0: unused row)
     const int32_t* seq_of;    // [T]
@@ -150,7 +150,10 @@ __global__ __launch_bounds__(SN_NT) void seq_norm_kernel(const SeqNormArgs a) {
         f32x4_t w[TAPS], hist[TAPS];  // hist[k-1]: h of k tokens ago
         if constexpr (TAPS > 1) {
 #pragma unroll
-            for (int j = 0; j < TAPS; ++j) w[j] = *reinterpret_cast<const f32x4_t*>(a.conv_w + (int64_t)j * a.wp + c);
+            for (int j = 0; j < TAPS; ++j) {
+                const u32x2_t u = *reinterpret_cast<const u32x2_t*>(a.conv_w + (int64_t)j * a.wp + c);
+                w[j] = f32x4_t{bflo(u[0]), bfhi(u[0]), bflo(u[1]), bfhi(u[1])};
+            }
         }
         auto pre = [&](int64_t r, const f32x4_t& x) {
             const float rx = s_rx[r - r0 + HALO];
@@ -244,7 +247,7 @@ __device__ __forceinline__ void sn_st8(void* base, int64_t off, int f32, const R
 __device__ __forceinline__ float sn_sumsq8(const Row8& v) { return sn_sumsq(v.a) + sn_sumsq(v.b); }
 
 template <int TAPS, int NT>
-__global__ __launch_bounds__(NT) void seq_norm_stream_kernel(const SeqNormArgs a, int tr) {
+__global__ __launch_bounds__(NT, (TAPS <= 4 && NT <= 512 ? 4 : 1)) void seq_norm_stream_kernel(const SeqNormArgs a, int tr) {
     constexpr int HALO = TAPS - 1, NW = NT / 64;
     __shared__ float s_red[2][2][NW];
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
@@ -261,30 +264,36 @@ __global__ __launch_bounds__(NT) void seq_norm_stream_kernel(const SeqNormArgs a
         lo = max(r0 - HALO, (int64_t)qs);
     }
     const Row8 zero = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
-    Row8 gq = zero, gp = zero, w[TAPS], hist[TAPS];
+    Row8 gq = zero, gp = zero, hist[TAPS];
+    u32x4_t w[TAPS];  // eight taps packed
     if (on) {
         if (a.y) gq = sn_ld8f(a.g_post + c);
         if (a.g_pre) gp = sn_ld8f(a.g_pre + c);
         if constexpr (TAPS > 1) {
 #pragma unroll
-            for (int j = 0; j < TAPS; ++j) w[j] = sn_ld8f(a.conv_w + (int64_t)j * a.wp + c);
+            for (int j = 0; j < TAPS; ++j) w[j] = *reinterpret_cast<const u32x4_t*>(a.conv_w + (int64_t)j * a.wp + c);
         }
     }
     if (TAPS > 1 && !on) {
 #pragma unroll
-        for (int j = 0; j < TAPS; ++j) w[j] = zero;
+        for (int j = 0; j < TAPS; ++j) w[j] = u32x4_t{0, 0, 0, 0};
     }
 #pragma unroll
     for (int j = 0; j < TAPS; ++j) hist[j] = zero;
-    auto load_x = [&](int64_t r) { return on ? sn_ld8f(a.x_in + (a.row_index ? a.row_index[r] : r) * a.ldx + c) : zero; };
-    auto load_y = [&](int64_t r) -> Row8 {
-        if (!a.y || !on) return zero;
+    auto tap = [](const u32x4_t& p, int i) { return (i & 1) ? bfhi(p[i >> 1]) : bflo(p[i >> 1]); };
+    auto load_row = [&](int64_t r, Row8& x, Row8& y) {
+        if (!on) return;
         const int64_t row = a.row_index ? a.row_index[r] : r;
+        x = sn_ld8f(a.x_in + row * a.ldx + c);
+        if (!a.y) return;
         if (!a.y_f32) {
             const u32x4_t u = *reinterpret_cast<const u32x4_t*>(reinterpret_cast<const bf16_t*>(a.y) + row * a.ldy + c);
-            return {{bflo(u[0]), bfhi(u[0]), bflo(u[1]), bfhi(u[1])}, {bflo(u[2]), bfhi(u[2]), bflo(u[3]), bfhi(u[3])}};
+            y.a = f32x4_t{bflo(u[0]), bfhi(u[0]), bflo(u[1]), bfhi(u[1])};
+            y.b = f32x4_t{bflo(u[2]), bfhi(u[2]), bflo(u[3]), bfhi(u[3])};
+        } else {
+            y.a = sn_load_y(a, row, c);
+            y.b = sn_load_y(a, row, c + 4);
         }
-        return {sn_load_y(a, row, c), sn_load_y(a, row, c + 4)};
     };
     // sums over the workgroup of two values per thread
     auto reduce2 = [&](float u, float v, int par, float& su, float& sv) {
@@ -302,7 +311,8 @@ __global__ __launch_bounds__(NT) void seq_norm_stream_kernel(const SeqNormArgs a
             sv += s_red[par][1][i];
         }
     };
-    Row8 x = load_x(lo), y = load_y(lo), xn = zero, yn = zero;
+    Row8 x = zero, y = zero, xn = zero, yn = zero;
+    load_row(lo, x, y);
     float ry = 0.f, su, sv;
     int par = 0;
     if (a.y) {
@@ -312,10 +322,11 @@ __global__ __launch_bounds__(NT) void seq_norm_stream_kernel(const SeqNormArgs a
     }
     for (int64_t r = lo; r < r1; ++r) {
         const bool more = r + 1 < r1;
-        if (more) {
-            xn = load_x(r + 1);
-            yn = load_y(r + 1);
+        if constexpr (TAPS > 1) {  // opaque: unpacked outside the loop the taps would take twice the registers
+#pragma unroll
+            for (int j = 0; j < TAPS; ++j) asm volatile("" : "+v"(w[j]));
         }
+        if (more) load_row(r + 1, xn, yn);
         if (a.y) {
 #pragma unroll
             for (int i = 0; i < 4; ++i) {
@@ -348,21 +359,23 @@ __global__ __launch_bounds__(NT) void seq_norm_stream_kernel(const SeqNormArgs a
                 if (r == qs) {
                     const int p = a.pos[r];
 #pragma unroll
-                    for (int k = 1; k < TAPS; ++k)
-                        hist[k - 1] = (on && p - k >= 0) ? sn_ld8f(a.state + (sin * HALO + (HALO - k)) * a.wp + c) : zero;
+                    for (int k = 1; k < TAPS; ++k) {
+                        hist[k - 1] = zero;
+                        if (on && p - k >= 0) hist[k - 1] = sn_ld8f(a.state + (sin * HALO + (HALO - k)) * a.wp + c);
+                    }
                 }
                 Row8 acc = zero;
 #pragma unroll
                 for (int k = HALO; k >= 1; --k)
 #pragma unroll
                     for (int i = 0; i < 4; ++i) {
-                        acc.a[i] = acc.a[i] + w[TAPS - 1 - k].a[i] * hist[k - 1].a[i];
-                        acc.b[i] = acc.b[i] + w[TAPS - 1 - k].b[i] * hist[k - 1].b[i];
+                        acc.a[i] = acc.a[i] + tap(w[TAPS - 1 - k], i) * hist[k - 1].a[i];
+                        acc.b[i] = acc.b[i] + tap(w[TAPS - 1 - k], 4 + i) * hist[k - 1].b[i];
                     }
 #pragma unroll
                 for (int i = 0; i < 4; ++i) {
-                    o.a[i] = h.a[i] + (acc.a[i] + w[TAPS - 1].a[i] * h.a[i]);
-                    o.b[i] = h.b[i] + (acc.b[i] + w[TAPS - 1].b[i] * h.b[i]);
+                    o.a[i] = h.a[i] + (acc.a[i] + tap(w[TAPS - 1], i) * h.a[i]);
+                    o.b[i] = h.b[i] + (acc.b[i] + tap(w[TAPS - 1], 4 + i) * h.b[i]);
                 }
                 const int64_t so = a.state_out[s];
                 const int e = qe - 1 - (int)r;  // tokens of the portion behind this one
@@ -388,7 +401,7 @@ template <int TAPS, int NT>
 int launch_seq_norm_stream(const SeqNormArgs& a, hipStream_t st) {
     // decode: one row per workgroup; else runs of rows long enough to spread the halo and the register setup, short enough
     // to fill the chip
-    int tr = a.T <= 512 ? 1 : (int)((a.T + 1023) / 1024);
+    int tr = a.T <= 512 ? 1 : (int)((a.T + 511) / 512);
     if (tr > 1) tr = tr < 8 ? 8 : tr > 32 ? 32 : tr;
     hipLaunchKernelGGL((seq_norm_stream_kernel<TAPS, NT>), dim3((unsigned)((a.T + tr - 1) / tr)), dim3(NT), 0, st, a, tr);
     GLM_CHECK_LAUNCH("glm_seq_norm");
@@ -438,7 +451,7 @@ extern "C" int glm_seq_norm_taps(int taps) {
 
 extern "C" int glm_seq_norm(const float* x_in, const int32_t* row_index, int64_t ldx, float* x_out, void* x_cast, int64_t ldc,
                             const void* y, int64_t ldy, int y_f32, int n_slabs, int64_t slab_stride, const float* g_post,
-                            const float* g_pre, const float* conv_w, int taps, float* state, int64_t n_state, const int32_t* pos,
+                            const float* g_pre, const void* conv_w, int taps, float* state, int64_t n_state, const int32_t* pos,
                             const int32_t* seq_of, const int32_t* q_start, const int32_t* state_in, const int32_t* state_out,
                             void* h, int64_t ldh, int act_f32, int64_t T, int width, int wp, float eps, glm_stream_t stream) {
     GLM_CHECK_ARG(x_in && T >= 0 && width > 0 && wp >= width && wp % 8 == 0 && ldx >= wp && ldx % 4 == 0, GLM_ERR_INVALID,
@@ -452,7 +465,7 @@ extern "C" int glm_seq_norm(const float* x_in, const int32_t* row_index, int64_t
     GLM_CHECK_ARG(taps >= 1 && glm_seq_norm_taps(taps) == taps, GLM_ERR_UNSUPPORTED, "glm_seq_norm: %d taps (see glm_seq_norm_taps)", taps);
     GLM_CHECK_ARG(T < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_seq_norm: too many rows");
     if (T == 0) return GLM_OK;
-    SeqNormArgs a = {x_in, row_index, ldx, x_out, x_cast, ldc, y, ldy, y_f32, n_slabs, slab_stride, g_post, g_pre, conv_w, state,
+    SeqNormArgs a = {x_in, row_index, ldx, x_out, x_cast, ldc, y, ldy, y_f32, n_slabs, slab_stride, g_post, g_pre, (const bf16_t*)conv_w, state,
                      pos, seq_of, q_start, state_in, state_out, n_state, h, ldh, act_f32, T, width, wp, eps};
     hipStream_t st = glm_s(stream);
     switch (taps) {

@@ -1279,7 +1279,7 @@ def seq_norm(x: torch.Tensor, width: int, eps: float, y=None, g_post: torch.Tens
              x_cast: torch.Tensor | None = None, keep_x: bool = True):
     """Between two sublayers (glm_seq_norm): returns (x_out, h).  y: the finished sublayer's output [T, wp] (bf16, fp32 or a
     PartialSum), g_post its norm's gain; g_pre the gain of the norm in front of the next sublayer (None: no h); conv =
-    (weights [taps, wp], state [n, taps-1, wp]) with the step's `meta` (pos, seq_of, q_start, state_in, state_out); rows:
+    (bf16 weights [taps, wp], fp32 state [n, taps-1, wp]) with the step's `meta` (pos, seq_of, q_start, state_in, state_out); rows:
     gather of rows (no convolution); x_cast receives x_out in the activation dtype."""
     wp = x.shape[1]
     assert x.dtype == torch.float32 and x.is_contiguous() and wp % 8 == 0 and width <= wp
@@ -1298,7 +1298,7 @@ def seq_norm(x: torch.Tensor, width: int, eps: float, y=None, g_post: torch.Tens
     if conv is not None:
         w, st = conv
         taps, n_state = w.shape[0], st.shape[0]
-        assert w.dtype == st.dtype == torch.float32 and w.is_contiguous() and st.is_contiguous() and w.shape[1] == wp
+        assert w.dtype == torch.bfloat16 and st.dtype == torch.float32 and w.is_contiguous() and st.is_contiguous() and w.shape[1] == wp
         assert taps == 1 or (st.shape[1:] == (taps - 1, wp) and meta is not None and rows is None)
     if taps > 1:
         pos, seq_of, q_start, s_in, s_out = meta.pos, meta.seq_of, meta.q_start, meta.state_in, meta.state_out

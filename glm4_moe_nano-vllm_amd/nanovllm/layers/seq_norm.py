@@ -32,8 +32,8 @@ class SublayerEntry(nn.Module):
     def load(self, norm_w: torch.Tensor, conv_w: torch.Tensor, device) -> None:
         self.g_pre = norm_gain(norm_w, self.wp, device)
         assert conv_w.shape[0] == self.width and conv_w.shape[1] <= self.taps
-        w = torch.zeros(self.taps, self.wp, dtype=torch.float32, device=device)
-        w[self.taps - conv_w.shape[1]:, : self.width] = conv_w.to(device=device, dtype=torch.float32).t()
+        w = torch.zeros(self.taps, self.wp, dtype=torch.bfloat16, device=device)
+        w[self.taps - conv_w.shape[1]:, : self.width] = conv_w.to(device=device, dtype=torch.bfloat16).t()
         self.conv_w = w
 
     def state_bytes(self) -> int:

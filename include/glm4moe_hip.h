@@ -504,7 +504,7 @@ int glm_gemm_f32(const float* x, int64_t ldx, int64_t xb, const float* w, int64_
                  glm_stream_t stream);
 
 /* Between two sublayers: x_out = x_in + rms(y) g_post (y bf16, or the sum of n_slabs fp32 slabs); h = rms(x_out) g_pre, then
- * h += depthwise causal convolution over time.  Gains and conv_w [taps][wp] fp32; x fp32.  Rows of a step: row t belongs to
+ * h += depthwise causal convolution over time.  Gains fp32, conv_w [taps][wp] bf16, x fp32.  Rows of a step: row t belongs to
  * sequence seq_of[t] at position pos[t] (< 0: unused), sequence s has rows [q_start[s], q_start[s+1]).  state
  * [n_state][taps-1][wp] fp32 keeps the last taps-1 inputs of the convolution, oldest first: set state_in[s] is read, set
  * state_out[s] (another one; < 0: none) written.  taps: a value glm_seq_norm_taps returns (1 = no convolution; then row_index
@@ -512,7 +512,7 @@ int glm_gemm_f32(const float* x, int64_t ldx, int64_t xb, const float* w, int64_
 int glm_seq_norm_taps(int taps); /* smallest supported count >= taps (pad with zero weights in front), -1: none */
 int glm_seq_norm(const float* x_in, const int32_t* row_index, int64_t ldx, float* x_out, void* x_cast, int64_t ldc, const void* y,
                  int64_t ldy, int y_f32, int n_slabs, int64_t slab_stride, const float* g_post, const float* g_pre,
-                 const float* conv_w, int taps, float* state, int64_t n_state, const int32_t* pos, const int32_t* seq_of,
+                 const void* conv_w, int taps, float* state, int64_t n_state, const int32_t* pos, const int32_t* seq_of,
                  const int32_t* q_start, const int32_t* state_in, const int32_t* state_out, void* h, int64_t ldh, int act_f32,
                  int64_t T, int width, int wp, float eps, glm_stream_t stream);
 /* embedding rows as the fp32 residual and, optionally, in the activation dtype; columns [width, wp) are zeros                 */

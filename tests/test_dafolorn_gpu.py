@@ -69,7 +69,7 @@ def test_seq_norm(width, taps, y_kind):
     x = {s: torch.randn(n, width, generator=g(s)) for s, n in L.items()}
     y = {s: torch.randn(n, width, generator=g(10 + s)).to(torch.bfloat16).float() for s, n in L.items()}
     gp, gq = 1 + 0.2 * torch.randn(width, generator=g(20)), 1 + 0.2 * torch.randn(width, generator=g(21))
-    cw = torch.randn(width, taps, generator=g(22))
+    cw = torch.randn(width, taps, generator=g(22)).to(torch.bfloat16).float()
     conv = torch.zeros(tp, wp)
     conv[tp - taps:, :width] = cw.T
     ref_x = {s: (x[s].double() + O.unit_rms(y[s].double(), eps) * gp.double()) if y_kind != "none" else x[s].double() for s in L}
@@ -86,7 +86,7 @@ def test_seq_norm(width, taps, y_kind):
             xs, ys = dev(cut(x)), cut(y)
             yk = {"none": None, "bf16": dev(ys, torch.bfloat16), "f32": dev(ys),
                   "slabs": hip_ops.PartialSum(dev(torch.stack([ys * 0.25, ys * 0.75])))}[y_kind]
-            xo, h = hip_ops.seq_norm(xs, width, eps, y=yk, g_post=dev(pad(gp)), g_pre=dev(pad(gq)), conv=(dev(conv), state), meta=meta,
+            xo, h = hip_ops.seq_norm(xs, width, eps, y=yk, g_post=dev(pad(gp)), g_pre=dev(pad(gq)), conv=(dev(conv, torch.bfloat16), state), meta=meta,
                                      act_dtype=torch.float32)
             assert torch.all(h[:, width:] == 0)
             r = 0
