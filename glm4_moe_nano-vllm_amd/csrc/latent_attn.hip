@@ -10,10 +10,8 @@
 //   latent_attn      split-KV flash loop over the pages; rows are (token, head) pairs; fp32 scores and softmax
 //   latent_up        merge of the KV splits (with the sink's mass) and out = W_uv ctx
 //
-// Roofline of latent_attn at decode: HBM — window * rank * 2 bytes per sequence, read once.  4 waves share every 32-key tile
-// through a ring of LDS-DMA stages (two tiles in flight): S^T = C . Q^T with the K dimension split over wave pairs and the keys
-// over the pairs' members, partial scores exchanged through LDS, the softmax evaluated redundantly by every wave, and
-// O^T += C^T . P^T with the latent dimension split over the waves.  One LDS image serves both products: chunk ^ swz(key) with
+// Roofline of latent_attn at decode: HBM — window * rank * 2 bytes per sequence, read once.  Four waves per 16 query rows share
+// every 64-key tile, double-buffered by LDS-DMA.  One LDS image serves both products: chunk ^ swz(key) with
 // swz(key) = (key & 3) << 1 | (key >> 2) & 1 is conflict-free for the ds_read_b128 row reads and for the transposed
 // ds_read_b64_tr_b16 reads.  Keys outside the sequence's range and padding columns are fetched from a page of zeros, never
 // from unused cache memory (whatever lies there would turn a zero weight into a NaN).
@@ -177,26 +175,29 @@ struct AttnArgs {
     float* part_ml;           // [Ta * H, nsplit, 2] running maximum (log2 units), mass
 };
 
-// Two workgroups per CU where registers and LDS allow (one computes while the other waits), else one with a deeper ring.
+// One wave per (16-row query tile, 16-key quarter of a 64-key tile): it computes those scores over the whole latent, their
+// weights, and hands them over through LDS; then the waves divide the latent's columns among themselves for O^T += C^T . P^T.
 template <int NCT, int MT>
 struct LaCfg {
-    static constexpr int TILEB = 32 * NCT * 128, SLAB = 2 * MT * 2 * 1024;
-    static constexpr bool TWO = NCT <= 8 && MT * NCT <= 16;
-    static constexpr int NST = TWO ? (3 * TILEB + SLAB + LA_BT * 4 <= 80 * 1024 ? 3 : 2) : (3 * TILEB <= 112 * 1024 ? 3 : 2);
-    static constexpr int LDS = NST * TILEB + SLAB + LA_BT * 4;
-    static_assert(LDS <= (TWO ? 80 : 160) * 1024, "LDS of a CU");
+    static constexpr int NW = 4 * MT, NT = 64 * NW;           // waves, threads
+    static constexpr int TILEB = 64 * NCT * 128;
+    static constexpr int NST = 2 * TILEB <= 144 * 1024 ? 2 : 1;
+    static constexpr int DPW = (4 * NCT + NW - 1) / NW;       // 16-column tiles of the latent per wave
+    static constexpr int PB = MT * 2048, MB = MT * 256;       // weights (bf16), row maxima
+    static constexpr int LDS = NST * TILEB + PB + MB + 16 + LA_BT * 4;
+    static_assert(LDS <= 160 * 1024, "LDS of a CU");
 };
 
 template <int NCT, int MT>
-__global__ __launch_bounds__(256, (LaCfg<NCT, MT>::TWO ? 2 : 1)) void latent_attn_kernel(const AttnArgs a) {
-    constexpr int RPAD = NCT * 64, ROWB = RPAD * 2, TILEB = 32 * ROWB, CPR = RPAD / 8;
-    constexpr int NST = LaCfg<NCT, MT>::NST, SLAB = LaCfg<NCT, MT>::SLAB;
-    constexpr int FG = NCT < 8 ? NCT : 8;  // fragments per request group
+__global__ __launch_bounds__(64 * 4 * MT) void latent_attn_kernel(const AttnArgs a) {
+    using C = LaCfg<NCT, MT>;
+    constexpr int RPAD = NCT * 64, ROWB = RPAD * 2, TILEB = C::TILEB, CPR = RPAD / 8, NST = C::NST, NW = C::NW, DPW = C::DPW, NT = C::NT;
+    constexpr int KS = 2 * NCT, NDMA = 8 * NCT, DMAW = (NDMA + NW - 1) / NW;
     extern __shared__ __attribute__((aligned(16))) char smem[];
     const int tid = threadIdx.x, lane = tid & 63;
     const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int c = lane & 15, g = lane >> 4;
-    const int kt = w & 1, kh = w >> 1;  // key half and K half of this wave's scores
+    const int kt = w & 3, mw = w >> 2;  // key quarter and row tile of this wave's scores
     int id = blockIdx.x;
     const int split = id % a.nsplit;
     id /= a.nsplit;
@@ -207,236 +208,249 @@ __global__ __launch_bounds__(256, (LaCfg<NCT, MT>::TWO ? 2 : 1)) void latent_att
     if (tok0 < 0 || tok0 >= a.Ta || ntok <= 0) return;
     const int p0 = a.pos[tok0], p1 = p0 + ntok - 1, seq = a.seq_of[tok0];
     const int nrows = ntok * hb;
-    // tiles start at multiples of 32, so that a tile lies in one cache block; the keys in front of the window's first are old
-    // latents of the same sequence (masked), keys behind the last row's are fetched from the zero page
-    const int lo = max(0, p0 - a.window + 1) & ~31;
-    const int ntile = p0 < 0 ? 0 : (p1 - lo + 32) >> 5;  // 32-key tiles of the whole range
+    // tiles start at multiples of 64: a tile lies in one cache block (its halves in one each, with blocks of 32); what is in front
+    // of the first visible key or behind the last row's comes from the zero page
+    const int first = max(0, p0 - a.window + 1), lo = first & ~63;
+    const int ntile = p0 < 0 ? 0 : (p1 - lo + 64) >> 6;  // 64-key tiles of the whole range
     const int per = (ntile + a.nsplit - 1) / a.nsplit;
     const int t0 = split * per, t1 = min(t0 + per, ntile), n = t1 - t0;
     if (n <= 0) {  // an empty split (or an unused row): no mass
-        for (int r = tid; r < nrows; r += 256) {
-            const int64_t grow = (int64_t)(tok0 + r / hb) * a.H + h0 + r % hb;
+        for (int r = tid; r < nrows; r += NT) {
+            const int64_t gr = (int64_t)(tok0 + r / hb) * a.H + h0 + r % hb;
             if (a.nsplit > 1) {
-                a.part_ml[(grow * a.nsplit + split) * 2] = -INFINITY;
-                a.part_ml[(grow * a.nsplit + split) * 2 + 1] = 0.f;
+                a.part_ml[(gr * a.nsplit + split) * 2] = -INFINITY;
+                a.part_ml[(gr * a.nsplit + split) * 2 + 1] = 0.f;
             } else {
-                for (int d = 0; d < a.rp; ++d) a.ctx[grow * a.rp + d] = 0;
+                for (int d = 0; d < a.rp; ++d) a.ctx[gr * a.rp + d] = 0;
             }
         }
         return;
     }
-    const int bs = 1 << a.bs_shift, bmask = bs - 1;
-    const int klo = lo + t0 * 32;                 // first key of this split
-    const int khi = min(p1, lo + t1 * 32 - 1);    // last key of this split
+    const int bmask = (1 << a.bs_shift) - 1;
+    const int klo = lo + t0 * 64;                 // first key of this split
+    const int khi = min(p1, lo + t1 * 64 - 1);    // last key of this split
     const int blk0 = klo >> a.bs_shift, nblk = (khi >> a.bs_shift) - blk0 + 1;
-    int* bt_lds = reinterpret_cast<int*>(smem + NST * TILEB + SLAB);
-    for (int i = tid; i < min(nblk, LA_BT); i += 256) {
+    char* aux = smem + NST * TILEB;
+    int* flags = reinterpret_cast<int*>(aux + C::PB + C::MB);
+    int* bt_lds = flags + 4;
+    // (entries of blocks in front of the window may have been given back, -1: no key of theirs is fetched)
+    for (int i = tid; i < min(nblk, LA_BT); i += NT) {
         const int64_t b = a.bt[(int64_t)seq * a.bt_stride + blk0 + i];
         bt_lds[i] = (int)min(max(b, (int64_t)0), a.n_blocks - 1);
     }
-    // query rows of this lane (one per row tile) and their fragments: K step 2 i + kh of wave pair kh
-    int rpos[MT];
-    int64_t grow[MT];
-    u32x4_t qf[MT][NCT];
+    if (tid < 4) flags[tid] = 0;
+    // this wave's query rows: row 16 mw + c
+    const int r_own = 16 * mw + c;
+    const bool own = r_own < nrows;
+    const int rpos = own ? p0 + r_own / hb : -1;
+    u32x4_t qf[KS];
+    {
+        const bf16_t* q = reinterpret_cast<const bf16_t*>(a.qa) + ((int64_t)(tok0 + (own ? r_own / hb : 0)) * a.H + h0 + (own ? r_own % hb : 0)) * a.rp;
 #pragma unroll
-    for (int m = 0; m < MT; ++m) {
-        const int r = 16 * m + c;
-        const bool ok = r < nrows;
-        const int to = ok ? r / hb : 0, hd = ok ? r % hb : 0;
-        rpos[m] = ok ? p0 + to : -1;
-        grow[m] = (int64_t)(tok0 + to) * a.H + h0 + hd;
-        const bf16_t* q = reinterpret_cast<const bf16_t*>(a.qa) + grow[m] * a.rp;
-#pragma unroll
-        for (int i = 0; i < NCT; ++i) {
-            const int k = 32 * (2 * i + kh) + 8 * g;
-            qf[m][i] = u32x4_t{0, 0, 0, 0};
-            if (ok && k < a.rp) qf[m][i] = *reinterpret_cast<const u32x4_t*>(q + k);
+        for (int i = 0; i < KS; ++i) {
+            const int k = 32 * i + 8 * g;
+            qf[i] = u32x4_t{0, 0, 0, 0};
+            if (own && k < a.rp) qf[i] = *reinterpret_cast<const u32x4_t*>(q + k);
         }
     }
     __syncthreads();
-    const unsigned base = lds_addr(smem), slab = base + NST * TILEB, bt_addr = slab + SLAB;
+    const unsigned base = lds_addr(smem), p_addr = base + NST * TILEB, m_addr = p_addr + C::PB, f_addr = m_addr + C::MB, bt_addr = f_addr + 16;
     const bf16_t* cache = reinterpret_cast<const bf16_t*>(a.cache);
     // per-lane source offsets (elements) of the DMA pieces inside a tile: constant over the tiles
-    unsigned off[NCT];
-    int orow[NCT];
+    unsigned off[DMAW];
+    int orow[DMAW];
     const bool padded = RPAD != a.rp;
 #pragma unroll
-    for (int i = 0; i < NCT; ++i) {
-        const int q = (w * NCT + i) * 64 + lane, row = q / CPR, ch = (q % CPR) ^ attn_swz(row);
+    for (int i = 0; i < DMAW; ++i) {
+        const int q = (i * NW + w) * 64 + lane, row = q / CPR, ch = (q % CPR) ^ attn_swz(row);
         orow[i] = (padded && ch * 8 >= a.rp) ? 1 << 30 : row;
-        off[i] = (unsigned)(row * a.rp + ch * 8);
+        off[i] = (unsigned)((row & 31) * a.rp + ch * 8);
     }
     auto issue = [&](int it) {
-        const int k0 = klo + it * 32;
-        int blk;
-        asm volatile("ds_read_b32 %0, %1\n\ts_waitcnt lgkmcnt(0)" : "=v"(blk) : "v"(bt_addr + ((k0 >> a.bs_shift) - blk0) * 4) : "memory");
-        blk = __builtin_amdgcn_readfirstlane(blk);
-        const bf16_t* src = cache + (((int64_t)blk << a.bs_shift) + (k0 & bmask)) * a.rp;
-        char* st = smem + (it % NST) * TILEB + w * NCT * 1024;
-        const int left = khi - k0;
-        if (left >= 31 && !padded) {
+        const int k0 = klo + it * 64;
+        int b0, b1;
+        const int i0 = (k0 >> a.bs_shift) - blk0, i1 = min(((k0 + 32) >> a.bs_shift) - blk0, nblk - 1);
+        asm volatile("ds_read_b32 %0, %2\n\tds_read_b32 %1, %3\n\ts_waitcnt lgkmcnt(0)" : "=&v"(b0), "=&v"(b1) : "v"(bt_addr + i0 * 4), "v"(bt_addr + i1 * 4) : "memory");
+        const bf16_t* s0 = cache + (((int64_t)__builtin_amdgcn_readfirstlane(b0) << a.bs_shift) + (k0 & bmask)) * a.rp;
+        const bf16_t* s1 = cache + (((int64_t)__builtin_amdgcn_readfirstlane(b1) << a.bs_shift) + ((k0 + 32) & bmask)) * a.rp;
+        char* st = smem + (NST == 2 ? (it & 1) * TILEB : 0);
+        const int left = khi - k0, skip = first - k0;
+        const bool plain = left >= 63 && skip <= 0 && !padded;
 #pragma unroll
-            for (int i = 0; i < NCT; ++i) lds_dma16(src + off[i], st + i * 1024);
-        } else {
-#pragma unroll
-            for (int i = 0; i < NCT; ++i) lds_dma16(orow[i] <= left ? (const void*)(src + off[i]) : (const void*)la_zero_page, st + i * 1024);
+        for (int i = 0; i < DMAW; ++i) {
+            const int piece = i * NW + w;
+            if (NDMA % NW != 0 && piece >= NDMA) continue;
+            const int row = orow[i];
+            const bf16_t* src = (((piece * 64 + lane) / CPR) & 32 ? s1 : s0) + off[i];
+            lds_dma16(plain || (row <= left && row >= skip) ? (const void*)src : (const void*)la_zero_page, st + piece * 1024);
         }
     };
-    f32x4_t acc[MT][NCT];
-    float m_run[MT], l_run[MT];
+    f32x4_t acc[MT][DPW];
+    float m_run[MT];
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
         m_run[m] = -INFINITY;
-        l_run[m] = 0.f;
 #pragma unroll
-        for (int d = 0; d < NCT; ++d) acc[m][d] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        for (int d = 0; d < DPW; ++d) acc[m][d] = f32x4_t{0.f, 0.f, 0.f, 0.f};
     }
+    float m_own = -INFINITY, l_own = 0.f;
     // loop-invariant LDS offsets of this lane's fragment reads
-    const unsigned k_rel = (16 * kt + c) * ROWB + (((4 * kh + g) ^ attn_swz(c)) << 4);
+    unsigned k_rel[2];
+#pragma unroll
+    for (int e = 0; e < 2; ++e) k_rel[e] = (16 * kt + c) * ROWB + (((4 * e + g) ^ attn_swz(c)) << 4);
     const int qq = (lane >> 2) & 3, pp = lane & 3, vrow = 4 * g + qq;
-    const unsigned v_rel = vrow * ROWB + (((2 * w + (pp >> 1)) ^ attn_swz(vrow)) << 4) + ((pp & 1) << 3);
+    // latent tile d of this wave: d NW + w = 4 (d MT + (w >> 2)) + (w & 3)
+    const unsigned v_rel = vrow * ROWB + (((2 * (w & 3) + (pp >> 1)) ^ attn_swz(vrow)) << 4) + ((pp & 1) << 3) + (w >> 2) * 128;
     const float sc = a.scale * LOG2E;
 #pragma unroll
-    for (int m = 0; m < MT; ++m)
-#pragma unroll
-        for (int i = 0; i < NCT; ++i) asm volatile("" : "+v"(qf[m][i]));  // landed before the ring starts counting vmcnt
-#pragma unroll
-    for (int i = 0; i < NST - 1; ++i)
-        if (i < n) issue(i);
+    for (int i = 0; i < KS; ++i) asm volatile("" : "+v"(qf[i]));  // landed before the DMAs are counted
+    issue(0);
     for (int it = 0; it < n; ++it) {
-        if (NST == 3 && it + 1 < n) wait_vm<NCT>();
-        else wait_vm<0>();
+        wait_vm<0>();
         __builtin_amdgcn_s_barrier();
-        if (it + NST - 1 < n) issue(it + NST - 1);
-        const unsigned st = base + (it % NST) * TILEB;
-        // ---- partial scores: keys 16 kt .. of the tile, K steps of parity kh ----
-        f32x4_t s[MT];
-#pragma unroll
-        for (int m = 0; m < MT; ++m) s[m] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-        static_for<(NCT + FG - 1) / FG>([&](auto G) {
-            constexpr int i0 = decltype(G)::value * FG, ni = NCT - i0 < FG ? NCT - i0 : FG;
+        if (NST == 2 && it + 1 < n) issue(it + 1);
+        if (tid == 0) asm volatile("ds_write_b32 %0, %1" ::"v"(f_addr + ((it + 1) & 1) * 4), "v"(0) : "memory");
+        const unsigned st = base + (NST == 2 ? (it & 1) * TILEB : 0);
+        // ---- scores of 16 keys x 16 rows over the whole latent, two accumulation chains ----
+        f32x4_t s2[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+        constexpr int FG = MT == 4 ? 4 : 8;  // fragments per request group
+        static_for<(KS + FG - 1) / FG>([&](auto G) {
+            constexpr int i0 = decltype(G)::value * FG, ni = KS - i0 < FG ? KS - i0 : FG;
             u32x4_t kf[FG];
-            static_for<ni>([&](auto I) { constexpr int i = decltype(I)::value; lds_read_b128<(i0 + i) * 128>(kf[i], st + k_rel); });
+            static_for<ni>([&](auto I) { constexpr int i = i0 + decltype(I)::value; lds_read_b128<(i >> 1) * 128>(kf[i - i0], st + k_rel[i & 1]); });
             wait_lds();
 #pragma unroll
             for (int i = 0; i < ni; ++i) asm volatile("" : "+v"(kf[i]));
 #pragma unroll
             for (int i = 0; i < ni; ++i)
-#pragma unroll
-                for (int m = 0; m < MT; ++m)
-                    s[m] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, kf[i]), __builtin_bit_cast(bf16x8_t, qf[m][i0 + i]), s[m], 0, 0, 0);
+                s2[i & 1] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, kf[i]), __builtin_bit_cast(bf16x8_t, qf[i0 + i]), s2[i & 1], 0, 0, 0);
         });
+        // ---- softmax of row c: this lane holds keys 16 kt + 4 g + r ----
+        const int key0 = klo + it * 64;
+        float x[4], mx = -INFINITY;
+        if (key0 > p1 - a.window && key0 + 63 <= p0) {  // every row sees every key
 #pragma unroll
-        for (int m = 0; m < MT; ++m) {
-            f32x4_t v;  // (an ordinary vector instruction between the matrix pipe's result and the store below)
+            for (int r = 0; r < 4; ++r) x[r] = (s2[0][r] + s2[1][r]) * sc;
+        } else {
+            const int d0 = rpos - (key0 + 16 * kt + 4 * g);
 #pragma unroll
-            for (int r = 0; r < 4; ++r) v[r] = s[m][r] * sc;
-            asm volatile("ds_write_b128 %0, %1" ::"v"(slab + ((kh * MT + m) * 2 + kt) * 1024 + lane * 16), "v"(v) : "memory");
+            for (int r = 0; r < 4; ++r) x[r] = (rpos >= 0 && d0 - r >= 0 && d0 - r < a.window) ? (s2[0][r] + s2[1][r]) * sc : -INFINITY;
         }
+#pragma unroll
+        for (int r = 0; r < 4; ++r) mx = fmaxf(mx, x[r]);
+        // The reference point of a row is raised only when a score exceeds it by more than 2^8 (it cancels in the end).  The
+        // weights are formed against the reference as it is; if any row of the workgroup needs a higher one, all waves see the
+        // flag behind the barrier, agree on new references and form the weights again.
+        auto weights = [&]() {
+            const float m_use = m_own == -INFINITY ? 0.f : m_own;
+            float p[4];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) p[r] = __builtin_amdgcn_exp2f(x[r] - m_use);
+            const u32x2_t v = {pack2bf(p[0], p[1]), pack2bf(p[2], p[3])};
+            asm volatile("ds_write_b64 %0, %1" ::"v"(p_addr + ((mw * 2 + (kt >> 1)) * 64 + lane) * 16 + (kt & 1) * 8), "v"(v) : "memory");
+            return (p[0] + p[1]) + (p[2] + p[3]);
+        };
+        float lp = weights();
+        if (__any(mx > m_own + 8.0f || (m_own == -INFINITY && mx > -INFINITY))) asm volatile("ds_write_b32 %0, %1" ::"v"(f_addr + (it & 1) * 4), "v"(1) : "memory");
         wait_lds();
         __builtin_amdgcn_s_barrier();
-        // ---- online softmax of row c of every row tile: this lane holds keys 16 t + 4 g + r ----
-        const int kbase = klo + it * 32 + 4 * g;
-        const bool inner = klo + it * 32 > p1 - a.window && klo + it * 32 + 31 <= p0;  // every row sees every key
-        bf16x8_t pf[MT];
-#pragma unroll
-        for (int m = 0; m < MT; ++m) {
-            f32x4_t sv[2][2];
-#pragma unroll
-            for (int t = 0; t < 2; ++t)
-#pragma unroll
-                for (int k2 = 0; k2 < 2; ++k2)
-                    asm volatile("ds_read_b128 %0, %1" : "=v"(sv[t][k2]) : "v"(slab + ((k2 * MT + m) * 2 + t) * 1024 + lane * 16));
+        int raise;
+        asm volatile("ds_read_b32 %0, %1\n\ts_waitcnt lgkmcnt(0)" : "=v"(raise) : "v"(f_addr + (it & 1) * 4) : "memory");
+        if (__builtin_amdgcn_readfirstlane(raise)) {
+            mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+            mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+            if (g == 0) asm volatile("ds_write_b32 %0, %1" ::"v"(m_addr + (mw * 16 + c) * 16 + kt * 4), "v"(mx) : "memory");
             wait_lds();
-            asm volatile("" : "+v"(sv[0][0]), "+v"(sv[0][1]), "+v"(sv[1][0]), "+v"(sv[1][1]));
-            float mx = -INFINITY, x[2][4];
-            if (inner) {
+            __builtin_amdgcn_s_barrier();
 #pragma unroll
-                for (int t = 0; t < 2; ++t)
-#pragma unroll
-                    for (int r = 0; r < 4; ++r) {
-                        x[t][r] = sv[t][0][r] + sv[t][1][r];
-                        mx = fmaxf(mx, x[t][r]);
-                    }
-            } else {
-                const int d0 = rpos[m] - kbase;
-#pragma unroll
-                for (int t = 0; t < 2; ++t)
-#pragma unroll
-                    for (int r = 0; r < 4; ++r) {
-                        const int d = d0 - 16 * t - r;
-                        x[t][r] = (rpos[m] >= 0 && d >= 0 && d < a.window) ? sv[t][0][r] + sv[t][1][r] : -INFINITY;
-                        mx = fmaxf(mx, x[t][r]);
-                    }
-            }
-            // the reference point is raised only when a score exceeds it by more than 2^8 (it cancels in the end); it is the
-            // same in the four lanes that share a row
-            if (__any(mx > m_run[m] + 8.0f || (m_run[m] == -INFINITY && mx > -INFINITY))) {
-                mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-                mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-                const float m_new = fmaxf(m_run[m], mx);
+            for (int m = 0; m < MT; ++m) {
+                f32x4_t q4;
+                asm volatile("ds_read_b128 %0, %1\n\ts_waitcnt lgkmcnt(0)" : "=v"(q4) : "v"(m_addr + (m * 16 + c) * 16) : "memory");
+                const float m_new = fmaxf(m_run[m], fmaxf(fmaxf(q4[0], q4[1]), fmaxf(q4[2], q4[3])));
                 const float alpha = m_new == -INFINITY ? 1.0f : __builtin_amdgcn_exp2f(m_run[m] - m_new);
-                l_run[m] *= alpha;
 #pragma unroll
-                for (int d = 0; d < NCT; ++d) acc[m][d] *= alpha;
+                for (int d = 0; d < DPW; ++d) acc[m][d] *= alpha;
                 m_run[m] = m_new;
-            }
-            const float m_use = m_run[m] == -INFINITY ? 0.f : m_run[m];
-#pragma unroll
-            for (int t = 0; t < 2; ++t)
-#pragma unroll
-                for (int r = 0; r < 4; ++r) {
-                    const float p = __builtin_amdgcn_exp2f(x[t][r] - m_use);
-                    l_run[m] += p;
-                    pf[m][4 * t + r] = (__bf16)p;
+                if (m == mw) {
+                    l_own *= alpha;
+                    m_own = m_new;
                 }
-        }
-        // ---- O^T += C^T . P^T on this wave's latent columns ----
-        static_for<(NCT + FG - 1) / FG>([&](auto G) {
-            constexpr int d0 = decltype(G)::value * FG, nd = NCT - d0 < FG ? NCT - d0 : FG;
-            u32x2_t vf[FG][2];
-            static_for<nd>([&](auto I) {
-                constexpr int d = decltype(I)::value;
-                lds_read_tr16_b64<(d0 + d) * 128>(vf[d][0], st + v_rel);
-                lds_read_tr16_b64<(d0 + d) * 128>(vf[d][1], st + v_rel + 16 * ROWB);
-            });
-            wait_lds();
-#pragma unroll
-            for (int d = 0; d < nd; ++d) asm volatile("" : "+v"(vf[d][0]), "+v"(vf[d][1]));
-#pragma unroll
-            for (int d = 0; d < nd; ++d) {
-                const u32x4_t vv = {vf[d][0][0], vf[d][0][1], vf[d][1][0], vf[d][1][1]};
-#pragma unroll
-                for (int m = 0; m < MT; ++m)
-                    acc[m][d0 + d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, vv), pf[m], acc[m][d0 + d], 0, 0, 0);
             }
-        });
+            lp = weights();
+            wait_lds();
+            __builtin_amdgcn_s_barrier();
+        }
+        l_own += lp;
+        // ---- O^T += C^T . P^T on this wave's latent columns, 32 keys at a time ----
+#pragma unroll
+        for (int k2 = 0; k2 < 2; ++k2) {
+            u32x4_t pf[MT];
+#pragma unroll
+            for (int m = 0; m < MT; ++m) asm volatile("ds_read_b128 %0, %1" : "=v"(pf[m]) : "v"(p_addr + ((m * 2 + k2) * 64 + lane) * 16));
+            const unsigned va = st + v_rel + k2 * 32 * ROWB;
+            static_for<(DPW + FG - 1) / FG>([&](auto G) {
+                constexpr int d0 = decltype(G)::value * FG, nd = DPW - d0 < FG ? DPW - d0 : FG;
+                u32x2_t vf[FG][2];
+                static_for<nd>([&](auto I) {
+                    constexpr int d = d0 + decltype(I)::value;
+                    if (4 * NCT % NW == 0 || d * NW + w < 4 * NCT) {
+                        lds_read_tr16_b64<d * MT * 128>(vf[d - d0][0], va);
+                        lds_read_tr16_b64<d * MT * 128>(vf[d - d0][1], va + 16 * ROWB);
+                    }
+                });
+                wait_lds();
+#pragma unroll
+                for (int m = 0; m < MT; ++m) asm volatile("" : "+v"(pf[m]));
+#pragma unroll
+                for (int d = 0; d < nd; ++d) asm volatile("" : "+v"(vf[d][0]), "+v"(vf[d][1]));
+#pragma unroll
+                for (int d = 0; d < nd; ++d) {
+                    const u32x4_t vv = {vf[d][0][0], vf[d][0][1], vf[d][1][0], vf[d][1][1]};
+                    if (4 * NCT % NW == 0 || (d0 + d) * NW + w < 4 * NCT) {
+#pragma unroll
+                        for (int m = 0; m < MT; ++m)
+                            acc[m][d0 + d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, vv), __builtin_bit_cast(bf16x8_t, pf[m]), acc[m][d0 + d], 0, 0, 0);
+                    }
+                }
+            });
+        }
+        if (NST == 1 && it + 1 < n) {
+            __builtin_amdgcn_s_barrier();
+            issue(it + 1);
+        }
     }
-    // ---- rows out: lane holds dims 64 d + 16 w + 4 g .. of row c ----
+    // ---- masses of the four key quarters meet in LDS ----
+    l_own += __shfl_xor(l_own, 16, 64);
+    l_own += __shfl_xor(l_own, 32, 64);
+    if (g == 0) asm volatile("ds_write_b32 %0, %1" ::"v"(m_addr + (mw * 16 + c) * 16 + kt * 4), "v"(l_own) : "memory");
+    wait_lds();
+    __builtin_amdgcn_s_barrier();
+    // ---- rows out: lane holds latent columns 16 (d NW + w) + 4 g .. of row c of every row tile ----
 #pragma unroll
     for (int m = 0; m < MT; ++m) {
-        float l = l_run[m];
-        l += __shfl_xor(l, 16, 64);
-        l += __shfl_xor(l, 32, 64);
-        const bool ok = 16 * m + c < nrows;
-        if (!ok) continue;
+        f32x4_t q4;
+        asm volatile("ds_read_b128 %0, %1\n\ts_waitcnt lgkmcnt(0)" : "=v"(q4) : "v"(m_addr + (m * 16 + c) * 16) : "memory");
+        const float l = (q4[0] + q4[1]) + (q4[2] + q4[3]);
+        const int r = 16 * m + c;
+        if (r >= nrows) continue;
+        const int hd = h0 + r % hb;
+        const int64_t gr = (int64_t)(tok0 + r / hb) * a.H + hd;
         if (a.nsplit == 1) {
-            const float sk = a.sink[grow[m] % a.H] * LOG2E;
+            const float sk = a.sink[hd] * LOG2E;
             const float M = fmaxf(m_run[m], sk);
             const float f = __builtin_amdgcn_exp2f(m_run[m] - M);
             const float inv = f / (l * f + __builtin_amdgcn_exp2f(sk - M));
 #pragma unroll
-            for (int d = 0; d < NCT; ++d) {
-                const int dim = 64 * d + 16 * w + 4 * g;
+            for (int d = 0; d < DPW; ++d) {
+                const int dim = 16 * (d * NW + w) + 4 * g;
                 if (dim < a.rp)
-                    *reinterpret_cast<u32x2_t*>(a.ctx + grow[m] * a.rp + dim) =
-                        u32x2_t{pack2bf(acc[m][d][0] * inv, acc[m][d][1] * inv), pack2bf(acc[m][d][2] * inv, acc[m][d][3] * inv)};
+                    *reinterpret_cast<u32x2_t*>(a.ctx + gr * a.rp + dim) = u32x2_t{pack2bf(acc[m][d][0] * inv, acc[m][d][1] * inv), pack2bf(acc[m][d][2] * inv, acc[m][d][3] * inv)};
             }
         } else {
-            const int64_t pr = grow[m] * a.nsplit + split;
+            const int64_t pr = gr * a.nsplit + split;
 #pragma unroll
-            for (int d = 0; d < NCT; ++d) {
-                const int dim = 64 * d + 16 * w + 4 * g;
+            for (int d = 0; d < DPW; ++d) {
+                const int dim = 16 * (d * NW + w) + 4 * g;
                 if (dim < a.rp) *reinterpret_cast<f32x4_t*>(a.part_o + pr * a.rp + dim) = acc[m][d];
             }
             if (w == 0 && g == 0) {
@@ -449,21 +463,28 @@ __global__ __launch_bounds__(256, (LaCfg<NCT, MT>::TWO ? 2 : 1)) void latent_att
 
 template <int NCT, int MT>
 int launch_latent_attn(const AttnArgs& a, hipStream_t st) {
-    constexpr int LDS = LaCfg<NCT, MT>::LDS;
+    using C = LaCfg<NCT, MT>;
     auto kern = latent_attn_kernel<NCT, MT>;
-    GLM_SET_MAX_LDS(kern, LDS, "glm_latent_attn");
+    GLM_SET_MAX_LDS(kern, C::LDS, "glm_latent_attn");
     const int64_t grid = (int64_t)a.n_tiles * a.n_hg * a.nsplit;
     GLM_CHECK_ARG(grid < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_latent_attn: grid too large");
-    hipLaunchKernelGGL(kern, dim3((unsigned)grid), dim3(256), LDS, st, a);
+    hipLaunchKernelGGL(kern, dim3((unsigned)grid), dim3(C::NT), C::LDS, st, a);
     GLM_CHECK_LAUNCH("glm_latent_attn");
     return GLM_OK;
 }
 
+// most query rows per workgroup (16 MT) whose fragments and sums the registers hold
+constexpr int la_max_rows(int nct) { return nct > 9 ? 16 : nct > 4 ? 32 : 64; }
+
 template <int NCT>
 int launch_latent_attn_mt(const AttnArgs& a, int mt, hipStream_t st) {
-    if (mt == 1) return launch_latent_attn<NCT, 1>(a, st);
-    if constexpr (NCT > 6) return launch_latent_attn<NCT, 2>(a, st);  // (four row tiles would not fit the registers)
-    else return mt == 2 ? launch_latent_attn<NCT, 2>(a, st) : launch_latent_attn<NCT, 4>(a, st);
+    if constexpr (la_max_rows(NCT) >= 64) {
+        if (mt > 2) return launch_latent_attn<NCT, 4>(a, st);
+    }
+    if constexpr (la_max_rows(NCT) >= 32) {
+        if (mt > 1) return launch_latent_attn<NCT, 2>(a, st);
+    }
+    return launch_latent_attn<NCT, 1>(a, st);
 }
 
 // ---------------------------------------------------------------------------------------------------------------------------
@@ -648,10 +669,10 @@ extern "C" int glm_latent_gather(const void* cache, int64_t n_slots, const int32
     return GLM_OK;
 }
 
-// rows per tile the absorbed kernel takes (16, 32 or 64) for a latent of rp columns
+// query rows (tokens x heads) per tile the absorbed kernel takes for a latent of rp columns: 16, 32 or 64
 extern "C" int glm_latent_attn_max_rows(int rp) {
     const int n = pick_nct(rp);
-    return n < 0 ? 0 : (n > 6 ? 32 : 64);
+    return n < 0 ? 0 : la_max_rows(n);
 }
 
 extern "C" int glm_latent_attn(const void* qa, const void* cache, int64_t n_blocks, int block_size, const int32_t* tile_tok, const int32_t* tile_n,
@@ -685,7 +706,7 @@ extern "C" int glm_latent_attn(const void* qa, const void* cache, int64_t n_bloc
     a.hb = (H + a.n_hg - 1) / a.n_hg;
     GLM_CHECK_ARG(tokens_per_tile * a.hb <= maxrows, GLM_ERR_INVALID, "glm_latent_attn: %d tokens x %d heads exceed %d rows", tokens_per_tile, a.hb, maxrows);
     const int64_t range = ((int64_t)bt_stride * block_size < (int64_t)window + tokens_per_tile ? (int64_t)bt_stride * block_size : (int64_t)window + tokens_per_tile);
-    GLM_CHECK_ARG((range / nsplit + 64) / block_size + 2 <= LA_BT, GLM_ERR_UNSUPPORTED, "glm_latent_attn: %ld keys per split exceed the block-table slice", (long)(range / nsplit));
+    GLM_CHECK_ARG((range / nsplit + 128) / block_size + 2 <= LA_BT, GLM_ERR_UNSUPPORTED, "glm_latent_attn: %ld keys per split exceed the block-table slice", (long)(range / nsplit));
     const int rows = tokens_per_tile * a.hb, mt = rows <= 16 ? 1 : rows <= 32 ? 2 : 4;
     switch (nct) {
         case 1: return launch_latent_attn_mt<1>(a, mt, st);

@@ -1377,11 +1377,11 @@ def latent_attn(qa: torch.Tensor, cache: torch.Tensor, tile_tok: torch.Tensor, t
     part_o = part_ml = None
     ns = 1
     if not f32:
-        # enough (tile, head group, KV split) workgroups to cover the chip, at least four 32-key tiles per split
+        # as many (tile, head group, KV split) workgroups as the chip has CUs, at least two 64-key tiles per split
         rows = latent_attn_max_rows(rp)
         wgs = tile_tok.numel() * -(-H // rows)
         keys = min(window + tokens_per_tile, block_tables.shape[1] * bs)
-        ns = num_splits or max(1, min(64, 512 // max(1, wgs), -(-keys // 128)))
+        ns = num_splits or max(1, min(64, 256 // max(1, wgs), -(-keys // 128)))
     ctx = torch.empty((Ta, H, rp), dtype=qa.dtype, device=qa.device)
     if ns > 1:
         part_o = torch.empty((Ta * H, ns, rp), dtype=torch.float32, device=qa.device)

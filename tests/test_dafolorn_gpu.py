@@ -125,7 +125,7 @@ def _standout(q, c, t, h, j, gain=40.0):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("H,rank,vdim,window,bs", [(6, 40, 24, 50, 64), (1, 264, 72, 1, 32), (32, 512, 128, 300, 64), (70, 24, 8, 33, 256),
+@pytest.mark.parametrize("H,rank,vdim,window,bs", [(6, 40, 24, 50, 64), (1, 264, 72, 1, 32), (2, 64, 16, 100, 32), (32, 512, 128, 300, 64), (70, 24, 8, 33, 256),
                                                    (16, 1000, 40, 64, 64), (40, 576, 16, 129, 64)])
 @pytest.mark.parametrize("n_q,splits", [(1, 0), (1, 1), (1, 5), (2, 0), (37, 3)])
 def test_latent_attn(dtype, H, rank, vdim, window, bs, n_q, splits):
