@@ -12,9 +12,10 @@ typedef __attribute__((address_space(3))) void attn_lds_void;
 typedef __attribute__((address_space(1))) const void attn_glb_void;
 
 __device__ __forceinline__ unsigned lds_addr(const void* p) { return (unsigned)(uintptr_t)(const attn_lds_void*)p; }
-// 64 lanes x 16 bytes from per-lane global addresses to 1 KiB of LDS at a wave-uniform address
+// 64 lanes x 16 bytes from per-lane global addresses to 1 KiB of LDS at a wave-uniform address; AUX 2: read once (nt)
+template <int AUX = 0>
 __device__ __forceinline__ void lds_dma16(const void* gsrc, void* lds_wave_base) {
-    __builtin_amdgcn_global_load_lds((attn_glb_void*)gsrc, (attn_lds_void*)lds_wave_base, 16, 0, 0);
+    __builtin_amdgcn_global_load_lds((attn_glb_void*)gsrc, (attn_lds_void*)lds_wave_base, 16, 0, AUX);
 }
 template <int OFF>
 __device__ __forceinline__ void lds_read_b128(u32x4_t& dst, unsigned addr) {
