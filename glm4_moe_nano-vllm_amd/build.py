@@ -20,8 +20,11 @@ LIBDIR = os.path.join(HERE, "lib")
 LIB = os.path.join(LIBDIR, "libglm4moe_hip.so")
 ARCH = "gfx950"
 SOURCES = ["api", "elementwise", "moe_misc", "paged_attn", "prefill_attn", "gemm_smallm", "gemm_tinym", "gemm_largem",
-           "decode_engine", "oneshot_allreduce", "seq_norm", "gemm_f32", "latent_attn",
-           "window_attn"]
+           "decode_engine", "oneshot_allreduce", "seq_norm", "gemm_f32", "latent_attn", "window_attn"]
+# kernel sets: what one model needs and nothing else (models/registry.py names the set), for a first run in a fresh checkout;
+# the library of everything is used where it is there
+KERNEL_SETS = {"dafolorn": (["api", "gemm_smallm", "gemm_tinym", "gemm_largem", "seq_norm", "gemm_f32", "latent_attn", "window_attn"],
+                            ["GLM_DENSE_ONLY=1"])}
 # kernels that were measured against the shipped ones and lost: only in the study library (`--study`), with their tests
 STUDY_SOURCES = ["prefill_attn64", "prefill_attn_persist"]
 STUDY_TAG = "_study"
@@ -91,6 +94,12 @@ def build_lib(force: bool = False, verbose: bool = True) -> str:
     return LIB
 
 
+def build_kernel_set(name: str) -> str:
+    """lib/libglm4moe_hip_<name>.so: the kernels of one model (KERNEL_SETS)."""
+    sources, defines = KERNEL_SETS[name]
+    return build_variant("_" + name, defines, sources)
+
+
 def build_study() -> str:
     """lib/libglm4moe_hip_study.so: the product sources + the measured-and-lost kernels (options fa_mfma32, fa_rows64)."""
     return build_variant(STUDY_TAG, ["GLM_STUDY_KERNELS=1"])
@@ -99,6 +108,8 @@ def build_study() -> str:
 if __name__ == "__main__":
     if "--study" in sys.argv:
         print(build_study())
+    elif "--kernel-set" in sys.argv:
+        print(build_kernel_set(sys.argv[sys.argv.index("--kernel-set") + 1]))
     elif "--variant" in sys.argv:  # python build.py --variant _abl1 GLM_ABLATE=1
         i = sys.argv.index("--variant")
         print(build_variant(sys.argv[i + 1], sys.argv[i + 2:]))

@@ -80,6 +80,7 @@ namespace {
 // rows per group above which the MFMA-bound tiled kernel is used instead of weight streaming
 constexpr int64_t LARGEM_MIN_AVG_ROWS = 96;
 
+#if !GLM_DENSE_ONLY
 // Many rows per group with fp8 weights (prefill): the GEMM is MFMA-bound.  First choice: the tiled kernel takes the fp8
 // bytes as they are (DMA-staged as fp8, converted exactly to bf16 between the fragment read and the MFMA; per-row
 // dequantisation scale on the fp32 accumulators) — no expansion pass, no scratch.  What that kernel does not cover (a K
@@ -108,6 +109,7 @@ int fp8w_large(int mode, GemmParams p, int rows, int cols, void* scratch, size_t
     p.w_gstride = (int64_t)rows * pitch;
     return glm_launch_gemm_largem(mode, p, st);  // p.wscale stays set
 }
+#endif  // !GLM_DENSE_ONLY
 
 // option tinym = 0 keeps the small-M kernels at one token row (A/B runs and the bit-identity tests of the fused launches)
 bool tinym_enabled() { return glm_option(GLM_OPT_TINYM) != 0; }
@@ -165,6 +167,7 @@ extern "C" int glm_gemm_bf16_act(const void* x, int64_t ldx, const void* w, int6
     return glm_launch_gemm_smallm(GEMM_PLAIN, p, glm_s(stream));
 }
 
+#if !GLM_DENSE_ONLY
 extern "C" int glm_gemm_qkv_rope_store(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* bias, int64_t T,
                                        int nh, int nkv, int hd, int K, const int64_t* positions, const float* cos_sin_cache,
                                        int rotary_dim, void* q_out, void* k_out, void* v_out, void* k_cache, void* v_cache,
@@ -236,6 +239,7 @@ extern "C" int glm_gemm_bf16_router_tail(const void* x, const void* w, int64_t l
                                              e_score_correction_bias, E, k, routed_scaling_factor, topk_idx, topk_w,
                                              expert_offsets, sorted_token, sorted_scale, pair_pos, with_shared, glm_s(stream));
 }
+#endif  // !GLM_DENSE_ONLY
 
 extern "C" int glm_gemm_bf16_partial_slices(int K, int want) { return glm_smallm_partial_slices(K, want); }
 
@@ -254,6 +258,7 @@ extern "C" int glm_gemm_bf16_partial(const void* x, int64_t ldx, const void* w, 
     return glm_launch_gemm_smallm_partial(p, glm_s(stream));
 }
 
+#if !GLM_DENSE_ONLY
 extern "C" int glm_grouped_gemm_gateup_silu(const void* x, int64_t ldx, const void* w13,
                                             int64_t w13_group_stride, int64_t w13_row_stride,
                                             const int32_t* expert_offsets, const int32_t* sorted_token,
@@ -493,3 +498,4 @@ extern "C" size_t glm_fp8w_expand_scratch_bytes(int G, int rows, int cols) {
     if (fp8w_native_enabled() && cols % 64 == 0) return 0;
     return (size_t)G * rows * glm_expand_pitch(cols) * sizeof(bf16_t);
 }
+#endif  // !GLM_DENSE_ONLY

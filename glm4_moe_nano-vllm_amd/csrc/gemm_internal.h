@@ -2,6 +2,12 @@
 #pragma once
 #include "common.h"
 
+// A library for models without experts, fp8 weights and fused QKV / router epilogues (build.py, kernel sets) compiles the GEMM
+// sources without those parts.
+#ifndef GLM_DENSE_ONLY
+#define GLM_DENSE_ONLY 0
+#endif
+
 enum GemmMode : int {
     GEMM_PLAIN = 0,   // y[r,n] = bf16(acc + bias[n])                              (a5, a10)
     GEMM_GATEUP = 1,  // act[r,i] = bf16(bf16(silu(bf16(g))) * bf16(u)), W rows gate|up  (a13)

@@ -1670,7 +1670,10 @@ int launch_largem_cfg(const GemmParams& p, hipStream_t st) {
     GLM_CHECK_ARG(total < (1ll << 31), GLM_ERR_UNSUPPORTED, "gemm_largem: grid too large");
     // the per-row scale of fp8-expanded weights is its own instantiation: as a run-time test it sat inside the epilogue's
     // element loop (a branch per accumulator register)
-    auto kern = (C::W8 || C::A8 || p.wscale) ? gemm_largem_kernel<MODE, C, VAR, true> : gemm_largem_kernel<MODE, C, VAR, !(C::W8 || C::A8) ? false : true>;
+    // (dense projections have no weight scales)
+    constexpr bool SCALES = MODE == GEMM_GATEUP || MODE == GEMM_DOWN;
+    auto kern = (C::W8 || C::A8 || (SCALES && p.wscale)) ? gemm_largem_kernel<MODE, C, VAR, SCALES || C::W8 || C::A8>
+                                                         : gemm_largem_kernel<MODE, C, VAR, !(C::W8 || C::A8) ? false : true>;
     constexpr int LDS_BYTES = (C::PH8 && (VAR & LM_PARK) != 0) ? 160 * 1024 : C::LDS + ((C::A8 && MODE == GEMM_DOWN) ? 16 * 1024 : 0);
     GLM_SET_MAX_LDS(kern, LDS_BYTES, "gemm_largem");
     // one workgroup per CU (the ring takes most of the LDS), a multiple of 8 so that every XCD gets the same count
@@ -1794,6 +1797,7 @@ int launch_largem(const GemmParams& p, hipStream_t st) {
 
 }  // namespace
 
+#if !GLM_DENSE_ONLY
 // fp8 x fp8 grouped expert projections on the block-scaled MFMA (r05): the product quadrant loop on
 // 256-row blocks.  Strides of x / w in BYTES.
 int glm_launch_gemm_largem_a8(int mode, const GemmParams& p, hipStream_t st) {
@@ -1829,6 +1833,7 @@ int glm_launch_gemm_largem_qkv(const GemmParams& p, hipStream_t st) {
     q.ldy = p.N;
     return launch_largem<GEMM_PLAIN>(q, st);
 }
+#endif  // !GLM_DENSE_ONLY
 
 int glm_launch_gemm_largem(int mode, const GemmParams& p, hipStream_t st) {
     GLM_CHECK_ARG(p.K % 8 == 0 && p.N % 4 == 0 && p.ldx % 8 == 0 && p.ldy % 4 == 0 && p.ldw % 8 == 0 &&
@@ -1836,8 +1841,10 @@ int glm_launch_gemm_largem(int mode, const GemmParams& p, hipStream_t st) {
                   GLM_ERR_UNSUPPORTED,
                   "gemm_largem: needs K%%8==0, N%%4==0, ldx%%8==0, ldy%%4==0, 16B-aligned x/W (K=%d N=%d)",
                   p.K, p.N);
+#if !GLM_DENSE_ONLY
     if (mode == GEMM_GATEUP) return launch_largem<GEMM_GATEUP>(p, st);
     if (mode == GEMM_DOWN) return launch_largem<GEMM_DOWN>(p, st);
+#endif  // !GLM_DENSE_ONLY
     if (mode == GEMM_ACT && p.yf == nullptr && p.act.kind == GLM_ACT_XIELU) return launch_largem<GEMM_XIELU>(p, st);
     if (mode == GEMM_ACT) return launch_largem<GEMM_ACT>(p, st);
     return launch_largem<GEMM_PLAIN>(p, st);

@@ -982,6 +982,7 @@ int glm_launch_gemm_smallm(int mode, const GemmParams& p, hipStream_t st) {
     // (tools/sweep_grouped.sh, two rounds): gate|up 4,1,2,2: 272 us; 8,4,2,2: 256; 4,2,2,2: 251; 4,4,2,2: 245-249.
     // down 4,1,2,2: 130 us; 8,1,1,2: 122; 2,1,1,2: 120; 4,2,1,2: 118-120.  Splitting K over the waves of a small
     // workgroup (16 act columns of gate|up, 32 columns of down) beats one long stream per wave.
+#if !GLM_DENSE_ONLY
 #ifndef GLM_SM_CFG_GATEUP
 #define GLM_SM_CFG_GATEUP 4, 4, 2, 2
 #endif
@@ -995,9 +996,6 @@ int glm_launch_gemm_smallm(int mode, const GemmParams& p, hipStream_t st) {
     // -DGLM_SM_NO_DMA builds the all-VGPR dispatch for A/B runs.
 #if !defined(GLM_SM_NO_DMA) && !defined(GLM_SM_DMA_GATEUP)
 #define GLM_SM_DMA_GATEUP 2, 2, 2, 2
-#endif
-#if !defined(GLM_SM_NO_DMA) && !defined(GLM_SM_DMA_MID)
-#define GLM_SM_DMA_MID 2, 1, 2, 2  // 23.7 us (4,2,2,2: 25.6; 1,1,2,2: 24.4; 4,1,2,2: 39.8)
 #endif
 #ifndef GLM_SM_DMA_MIN_ROWS
 #define GLM_SM_DMA_MIN_ROWS 17  // total rows from which the grouped projections take the LDS-DMA body
@@ -1038,6 +1036,10 @@ int glm_launch_gemm_smallm(int mode, const GemmParams& p, hipStream_t st) {
     if (mode == GEMM_DOWN && Rs <= 16) return launch_cfg<GEMM_DOWN, GLM_SM_CFG_DOWN_R16>(p, st);
     if (mode == GEMM_GATEUP) return launch_cfg<GEMM_GATEUP, GLM_SM_CFG_GATEUP>(p, st);
     if (mode == GEMM_DOWN) return launch_cfg<GEMM_DOWN, GLM_SM_CFG_DOWN>(p, st);
+#endif  // !GLM_DENSE_ONLY
+#if !defined(GLM_SM_NO_DMA) && !defined(GLM_SM_DMA_MID)
+#define GLM_SM_DMA_MID 2, 1, 2, 2  // 23.7 us (4,2,2,2: 25.6; 1,1,2,2: 24.4; 4,1,2,2: 39.8)
+#endif
     // dense projection: choose the K-split so that the grid covers the chip
     const int64_t rows = p.offs ? 64 : p.R;
     const int tiles32 = (p.N + 31) / 32;
@@ -1089,6 +1091,7 @@ int glm_launch_gemm_smallm_partial(const GemmParams& p, hipStream_t st) {
     return launch_cfg<GEMM_PLAIN, GLM_SM_CFG_PARTIAL>(p, st);
 }
 
+#if !GLM_DENSE_ONLY
 int glm_launch_gemm_smallm_fp8w(int mode, const GemmParams& p, hipStream_t st) {
     GLM_CHECK_ARG(p.K % 16 == 0 && p.N % 4 == 0 && p.ldx % 8 == 0 && p.ldy % 4 == 0 && p.ldw % 16 == 0 &&
                       p.w_gstride % 16 == 0 && glm_aligned16(p.x) && glm_aligned16(p.w) &&
@@ -1128,3 +1131,4 @@ int glm_launch_gemm_smallm_fp8w(int mode, const GemmParams& p, hipStream_t st) {
     glm_set_error("gemm_smallm(fp8 weights): only the grouped expert projections are quantised");
     return GLM_ERR_UNSUPPORTED;
 }
+#endif  // !GLM_DENSE_ONLY

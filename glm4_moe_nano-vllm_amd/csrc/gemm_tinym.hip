@@ -650,6 +650,7 @@ int glm_launch_gemm_tinym(int mode, const GemmParams& p, int n_tokens, hipStream
     GLM_CHECK_ARG(M == 1, GLM_ERR_UNSUPPORTED, "gemm_tinym: %d rows per block", M);
     // units: 4 rows x 4 KiB for long rows; a short K (expert down projection, 1408) as ONE unit of 3-KiB rows
     if (mode == GEMM_PLAIN) return launch_tiny<GEMM_PLAIN, 1, GLM_TM_SEGS_PLAIN, false, false, GLM_TM_RPW_PLAIN>(tp, 1, st);
+#if !GLM_DENSE_ONLY
     // grouped launches: rows per tile chosen for the TAIL of the launch — a workgroup's waves pull tiles from a counter, and
     // the launch ends when the slowest wave has finished its last tile; at Air dims one token gives 24.75 tiles of 4 rows per
     // workgroup for gate|up (7 waves take 3, one takes 4: +29 % on the critical wave), 49.5 tiles of 2 rows even that out
@@ -662,8 +663,12 @@ int glm_launch_gemm_tinym(int mode, const GemmParams& p, int n_tokens, hipStream
     if (mode == GEMM_GATEUP) return launch_tiny<GEMM_GATEUP, 1, (GLM_TM_RPW_GATEUP == 2 ? 8 : 4), false, false, GLM_TM_RPW_GATEUP>(tp, n_tokens, st);
     if (p.K <= 1536) return launch_tiny<GEMM_DOWN, 1, 3, false, false, GLM_TM_RPW_DOWN>(tp, (int)p.R, st);
     return launch_tiny<GEMM_DOWN, 1, 4, false, false, GLM_TM_RPW_DOWN>(tp, (int)p.R, st);
+#else
+    return GLM_ERR_UNSUPPORTED;
+#endif
 }
 
+#if !GLM_DENSE_ONLY
 // QKV projection (+bias) of ONE token row whose input is computed in the kernel: moe_combine of the previous layer's expert
 // rows + add-RMSNorm with `residual_in` (see the file header).  p.x is ignored; p.K = H.
 int glm_launch_gemm_tinym_combine_norm(const GemmParams& p, const void* y_prev, int64_t ld_yprev, const int32_t* pair_pos,
@@ -712,6 +717,7 @@ int glm_launch_gemm_tinym_router_tail(const GemmParams& p, unsigned* ticket, flo
     tp.tr_offs = offs; tp.tr_tok = tok; tp.tr_scale = (bf16_t*)scale; tp.tr_pos = pos; tp.tr_shared = with_shared;
     return launch_tiny<GEMM_PLAIN, 1, GLM_TM_SEGS_PLAIN, false, true, GLM_TM_RPW_PLAIN>(tp, 1, st);
 }
+#endif  // !GLM_DENSE_ONLY
 
 #if GLM_TM_STAMP
 extern "C" int glm_debug_tinym_stamps(unsigned long long* out, int n) {

@@ -71,36 +71,53 @@ __device__ __forceinline__ void la_st8(void* p, int64_t i, const float (&v)[8]) 
         for (int j = 0; j < 8; ++j) f[j] = v[j];
     }
 }
-template <typename E>
-__device__ void latent_norm_row(const PrepArgs& a, int64_t t, int lane) {
-    const int64_t base = t * a.ldq + a.c_off;
-    const int64_t slot = a.slots[t];
-    const bool st = slot >= 0 && slot < a.n_slots;
-    int64_t row = a.crow ? a.crow[t] : -1;
-    if (row >= a.n_crows) row = -1;
-    float v[8], s = 0.f;
-    for (int i = lane * 8; i < a.rp; i += 512) {
-        la_ld8<E>(a.qc, base + i, v);
+// R tokens t0 .. by one wave, their loads together
+template <typename E, int R>
+__device__ void latent_norm_rows(const PrepArgs& a, int64_t t0, int lane) {
+    int64_t slot[R], row[R];
+    float v[R][8], s[R];
 #pragma unroll
-        for (int j = 0; j < 8; ++j) s += v[j] * v[j];
+    for (int i = 0; i < R; ++i) {
+        const int64_t t = min(t0 + i, a.T - 1);
+        slot[i] = a.slots[t];
+        row[i] = a.crow ? a.crow[t] : -1;
+        s[i] = 0.f;
     }
-    const float r = 1.0f / sqrtf(wave_sum(s) / (float)a.rank + a.eps);
-    for (int i = lane * 8; i < a.rp; i += 512) {
-        if (a.rp > 512) la_ld8<E>(a.qc, base + i, v);  // (one step: the values are still in registers)
+    for (int k = lane * 8; k < a.rp; k += 512) {
 #pragma unroll
-        for (int j = 0; j < 8; ++j) v[j] = v[j] * r * a.norm_w[i + j];
-        if (st) la_st8<E>(a.cache, slot * a.rp + i, v);
-        if (row >= 0) la_st8<E>(a.c_out, row * a.rp + i, v);
+        for (int i = 0; i < R; ++i) la_ld8<E>(a.qc, min(t0 + i, a.T - 1) * a.ldq + a.c_off + k, v[i]);
+#pragma unroll
+        for (int i = 0; i < R; ++i)
+#pragma unroll
+            for (int j = 0; j < 8; ++j) s[i] += v[i][j] * v[i][j];
+    }
+#pragma unroll
+    for (int i = 0; i < R; ++i) s[i] = 1.0f / sqrtf(wave_sum(s[i]) / (float)a.rank + a.eps);
+    for (int k = lane * 8; k < a.rp; k += 512) {
+        float w[8];
+#pragma unroll
+        for (int j = 0; j < 8; ++j) w[j] = a.norm_w[k + j];
+#pragma unroll
+        for (int i = 0; i < R; ++i) {
+            if (t0 + i >= a.T) continue;
+            if (a.rp > 512) la_ld8<E>(a.qc, (t0 + i) * a.ldq + a.c_off + k, v[i]);  // (one step: the values are still in registers)
+#pragma unroll
+            for (int j = 0; j < 8; ++j) v[i][j] = v[i][j] * s[i] * w[j];
+            if (slot[i] >= 0 && slot[i] < a.n_slots) la_st8<E>(a.cache, slot[i] * a.rp + k, v[i]);
+            if (row[i] >= 0 && row[i] < a.n_crows) la_st8<E>(a.c_out, row[i] * a.rp + k, v[i]);
+        }
     }
 }
 
 constexpr int PREP_TT = 4;  // 16-token tiles per absorb workgroup
 
+// NR: tokens per wave of the norm's workgroups
+template <int NR>
 __global__ __launch_bounds__(256) void latent_prepare_kernel(const PrepArgs a, int n_absorb) {
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
     if ((int)blockIdx.x >= n_absorb) {
-        const int64_t t = (int64_t)((int)blockIdx.x - n_absorb) * 4 + wid;
-        if (t < a.T) latent_norm_row<bf16_t>(a, t, lane);
+        const int64_t t = ((int64_t)((int)blockIdx.x - n_absorb) * 4 + wid) * NR;
+        if (t < a.T) latent_norm_rows<bf16_t, NR>(a, t, lane);
         return;
     }
     // q'[t, h, r] = sum_d W_uk[h, d, r] q[t, h, d]: 64 latent rows x 64 tokens per workgroup, 16 x 64 per wave
@@ -141,7 +158,7 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(const PrepArgs a, i
 
 __global__ __launch_bounds__(256) void latent_norm_f32_kernel(const PrepArgs a) {
     const int64_t t = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (t < a.T) latent_norm_row<float>(a, t, threadIdx.x & 63);
+    if (t < a.T) latent_norm_rows<float, 1>(a, t, threadIdx.x & 63);
 }
 
 // cache rows -> contiguous rows (the history in front of a long portion): one wave per row, 16-byte chunks
@@ -651,13 +668,15 @@ extern "C" int glm_latent_prepare(const void* qc, int64_t ldq, int c_off, int64_
     GLM_CHECK_ARG(act_f32 || Ta == 0 || (wukt && qa && glm_aligned16(wukt) && glm_aligned16(qc)), GLM_ERR_INVALID, "glm_latent_prepare: absorbed rows need W_uk^T and q'");
     if (T == 0) return GLM_OK;
     PrepArgs a = {qc, ldq, c_off, T, Ta, H, dimp, rank, rp, norm_w, eps, slots, cache, n_slots, crow, c_out, n_crows, (const bf16_t*)wukt, (bf16_t*)qa};
-    const int64_t nnorm = (T + 3) / 4;
+    const bool many = !act_f32 && T >= 2048;
+    const int64_t nnorm = many ? (T + 15) / 16 : (T + 3) / 4;
     if (act_f32) {
         hipLaunchKernelGGL(latent_norm_f32_kernel, dim3((unsigned)nnorm), dim3(256), 0, glm_s(stream), a);
     } else {
         const int64_t nabs = Ta > 0 ? (int64_t)((rp + 63) / 64) * H * ((Ta + 16 * PREP_TT - 1) / (16 * PREP_TT)) : 0;
         GLM_CHECK_ARG(nabs + nnorm < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_latent_prepare: grid too large");
-        hipLaunchKernelGGL(latent_prepare_kernel, dim3((unsigned)(nabs + nnorm)), dim3(256), 0, glm_s(stream), a, (int)nabs);
+        if (many) hipLaunchKernelGGL(latent_prepare_kernel<4>, dim3((unsigned)(nabs + nnorm)), dim3(256), 0, glm_s(stream), a, (int)nabs);
+        else hipLaunchKernelGGL(latent_prepare_kernel<1>, dim3((unsigned)(nabs + nnorm)), dim3(256), 0, glm_s(stream), a, (int)nabs);
     }
     GLM_CHECK_LAUNCH("glm_latent_prepare");
     return GLM_OK;

@@ -14,6 +14,7 @@ class ModelEntry:
     default_block_size: int   # tokens per cache block
     block_multiple: int       # block sizes must be multiples of this
     dtypes: tuple             # activation dtypes the model runs in
+    kernel_set: str | None    # build.py kernel set that is enough for this model (None: the whole library)
     step_batches: bool        # True: the model runs StepBatch inputs (portions of prompts beside decoded tokens, recurrent state)
 
     @staticmethod
@@ -29,9 +30,9 @@ class ModelEntry:
 
 
 GLM4_MOE = ModelEntry("glm4_moe", "nanovllm.config:normalise_hf_config", "nanovllm.models.glm4_moe.model:Glm4MoeForCausalLM",
-                      256, 256, ("bfloat16",), False)
+                      256, 256, ("bfloat16",), None, False)
 DAFOLORN = ModelEntry("dafolorn", "nanovllm.models.dafolorn.config:read_config", "nanovllm.models.dafolorn.model:DafolornForCausalLM",
-                      64, 32, ("bfloat16", "float32"), True)
+                      64, 32, ("bfloat16", "float32"), "dafolorn", True)
 
 _ENTRIES = {e.name: e for e in (GLM4_MOE, DAFOLORN)}
 
