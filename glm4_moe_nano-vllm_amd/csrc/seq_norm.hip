@@ -426,18 +426,26 @@ int launch_seq_norm(const SeqNormArgs& a, hipStream_t st) {
 
 // one workgroup per token row: fp32 residual row and (optionally) the row in the activation dtype
 __global__ __launch_bounds__(SN_NT) void embed_rows_kernel(const int64_t* ids, const void* table, int64_t ldw, int64_t vocab, float* x,
-                                                           int64_t ldx, void* cast, int64_t ldc, int act_f32, int width, int wp) {
+                                                           int64_t ldx, void* cast, int64_t ldc, int act_f32, int width, int wp, int vec) {
     const int64_t t = blockIdx.x;
     const int64_t id = ids[t];
-    const bool ok = id >= 0 && id < vocab;
-    for (int c = threadIdx.x; c < wp; c += SN_NT) {
-        float v = 0.f;
-        if (ok && c < width) v = act_f32 ? reinterpret_cast<const float*>(table)[id * ldw + c] : bf2f(reinterpret_cast<const bf16_t*>(table)[id * ldw + c]);
-        x[t * ldx + c] = v;
-        if (cast) {
-            if (act_f32) reinterpret_cast<float*>(cast)[t * ldc + c] = v;
-            else reinterpret_cast<bf16_t*>(cast)[t * ldc + c] = f2bf(v);
+    const bool ok = id >= 0 && id < vocab;  // (an id outside the table gives a row of zeros)
+    for (int c = threadIdx.x * 4; c < wp; c += SN_NT * 4) {
+        f32x4_t v = {0.f, 0.f, 0.f, 0.f};
+        if (ok) {
+            if (vec) {  // whole rows of the table, padding included
+                if (act_f32) v = *reinterpret_cast<const f32x4_t*>(reinterpret_cast<const float*>(table) + id * ldw + c);
+                else {
+                    const u32x2_t u = *reinterpret_cast<const u32x2_t*>(reinterpret_cast<const bf16_t*>(table) + id * ldw + c);
+                    v = f32x4_t{bflo(u[0]), bfhi(u[0]), bflo(u[1]), bfhi(u[1])};
+                }
+            } else {
+                for (int i = 0; i < 4; ++i)
+                    if (c + i < width) v[i] = act_f32 ? reinterpret_cast<const float*>(table)[id * ldw + c + i] : bf2f(reinterpret_cast<const bf16_t*>(table)[id * ldw + c + i]);
+            }
         }
+        *reinterpret_cast<f32x4_t*>(x + t * ldx + c) = v;
+        if (cast) sn_store(cast, t * ldc + c, act_f32, v);
     }
 }
 
@@ -482,10 +490,11 @@ extern "C" int glm_seq_norm(const float* x_in, const int32_t* row_index, int64_t
 
 extern "C" int glm_embed_rows(const int64_t* ids, const void* table, int64_t ldw, int64_t vocab, float* x, int64_t ldx, void* cast,
                               int64_t ldc, int act_f32, int64_t T, int width, int wp, glm_stream_t stream) {
-    GLM_CHECK_ARG(ids && table && x && T >= 0 && width > 0 && wp >= width && ldw >= width && ldx >= wp && (!cast || ldc >= wp), GLM_ERR_INVALID,
-                  "glm_embed_rows: bad shape T=%ld width=%d wp=%d", (long)T, width, wp);
+    GLM_CHECK_ARG(ids && table && x && T >= 0 && width > 0 && wp >= width && wp % 8 == 0 && ldw >= width && ldx >= wp && ldx % 4 == 0 &&
+                      (!cast || (ldc >= wp && ldc % 4 == 0)), GLM_ERR_INVALID, "glm_embed_rows: bad shape T=%ld width=%d wp=%d", (long)T, width, wp);
     if (T == 0) return GLM_OK;
-    hipLaunchKernelGGL(embed_rows_kernel, dim3((unsigned)T), dim3(SN_NT), 0, glm_s(stream), ids, table, ldw, vocab, x, ldx, cast, ldc, act_f32, width, wp);
+    const int vec = width == wp && ldw % 8 == 0 && glm_aligned16(table);
+    hipLaunchKernelGGL(embed_rows_kernel, dim3((unsigned)T), dim3(SN_NT), 0, glm_s(stream), ids, table, ldw, vocab, x, ldx, cast, ldc, act_f32, width, wp, vec);
     GLM_CHECK_LAUNCH("glm_embed_rows");
     return GLM_OK;
 }

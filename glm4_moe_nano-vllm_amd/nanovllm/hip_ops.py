@@ -1384,7 +1384,8 @@ def latent_attn(qa: torch.Tensor, cache: torch.Tensor, tile_tok: torch.Tensor, t
         rows = latent_attn_max_rows(rp)
         wgs = tile_tok.numel() * -(-H // rows)
         keys = min(window + tokens_per_tile, block_tables.shape[1] * bs)
-        ns = num_splits or max(1, min(64, 256 // max(1, wgs), -(-keys // 128)))
+        # (and no more keys per split than a workgroup's slice of the block table covers)
+        ns = num_splits or max(1, min(64, 256 // max(1, wgs), -(-keys // 128)), -(-keys // (900 * bs)))
     ctx = torch.empty((Ta, H, rp), dtype=qa.dtype, device=qa.device)
     if ns > 1:
         part_o = torch.empty((Ta * H, ns, rp), dtype=torch.float32, device=qa.device)
@@ -1398,6 +1399,9 @@ def latent_attn(qa: torch.Tensor, cache: torch.Tensor, tile_tok: torch.Tensor, t
     if ns > 1:
         _check(lib.glm_latent_merge(_p(part_o), _p(part_ml), _p(sink), ns, _p(ctx), Ta, H, rp, _stream()), "glm_latent_merge")
     _check(lib.glm_latent_up(_p(ctx), _p(wuv), _p(out), out.stride(0), Ta, H, vdimp, rp, _stream()), "glm_latent_up")
+
+
+WINDOW_ATTN_MAX_DIM = 256  # head sizes of glm_window_attn_prefill
 
 
 def window_attn_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, out: torch.Tensor, q_start: torch.Tensor,

@@ -36,7 +36,9 @@ class LatentAttention(nn.Module):
         self.dimp, self.vdimp, self.rp = hip_ops.round8(dim), hip_ops.round8(vdim), hip_ops.round8(rank)
         H = self.heads
         self.qc_proj = PaddedLinear(width, [self.dimp] * H + [self.rp], dtype)     # query heads, raw latent
-        self.expand = PaddedLinear(rank, [self.dimp] * H + [self.vdimp] * H, dtype) if dtype == torch.bfloat16 else None
+        # (fp32, and heads beyond the expanded kernel's sizes: every portion attends in the absorbed form)
+        self.can_expand = dtype == torch.bfloat16 and max(self.dimp, self.vdimp) <= hip_ops.WINDOW_ATTN_MAX_DIM
+        self.expand = PaddedLinear(rank, [self.dimp] * H + [self.vdimp] * H, dtype) if self.can_expand else None
         self.o_proj = PaddedLinear([vdim] * H, [hip_ops.round8(width)], dtype)
         self.tokens_per_tile = hip_ops.latent_tokens_per_tile(self.rp, H) if dtype == torch.bfloat16 else 1
         self.break_even = absorb_break_even(self.rp, self.dimp, self.vdimp)

@@ -106,8 +106,10 @@ class DafolornForCausalLM(nn.Module):
 
     @property
     def max_short_portion(self) -> int:
-        """Longest portion of a sequence that attends in the absorbed form (fp32: every portion)."""
-        return 1 << 30 if self.dtype == torch.float32 else max(layer.mixer.break_even for layer in self.layers)
+        """Longest portion of a sequence that attends in the absorbed form."""
+        if all(layer.mixer.can_expand for layer in self.layers):
+            return max(layer.mixer.break_even for layer in self.layers)
+        return 1 << 30
 
     def cache_bytes_per_token(self) -> int:
         return sum(layer.mixer.cache_bytes_per_token() for layer in self.layers)

@@ -34,6 +34,8 @@ class TraceSession:
         from nanovllm.engine.sequence import Sequence
         batch = []
         for e in entries:
+            if not e["tokens"]:
+                continue
             seq = self.live.get(e["id"])
             if seq is None:
                 seq = self.live[e["id"]] = Sequence(e["tokens"])

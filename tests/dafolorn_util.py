@@ -26,6 +26,8 @@ CONFIGS = {
                    (1, 2, 1), 5.0, 1e-3),
     # many heads (several groups per tile), a latent of 536 columns, no loop
     "tall": config(64, 128, 2, [layer(40, 8, 8, 536, 48, 128), layer(70, 16, 8, 24, 300, 40)], None, 20.0),
+    # value heads beyond the expanded kernel: prompts attend in the absorbed form
+    "huge": config(72, 64, 3, [layer(2, 264, 24, 64, 40, 48, 0.05), layer(1, 16, 328, 48, 77, 48)], (0, 1, 2), 8.0),
     # loop up to the last layer, twice two layers
     "tail": config(200, 96, 4, [layer(6, 40, 24, 88, 64, 136), layer(4, 48, 32, 104, 64, 136), layer(6, 40, 24, 88, 31, 136)], (1, 3, 2), 12.0),
 }

@@ -72,6 +72,7 @@ def test_layer_runs():
     runs = {n: layer_runs(read_config(c)) for n, c in CONFIGS.items()}
     assert runs["odd"] == [(0, 0), (1, None), (0, 1), (1, None), (0, 2), (1, None), (2, None)]
     assert runs["wide"] == [(0, None), (1, 0), (2, None)] and runs["tall"] == [(0, None), (1, None)]
+    assert runs["huge"] == [(0, 0), (0, 1), (1, None)]
     assert runs["tail"] == [(0, None), (1, 0), (2, None), (1, 1), (2, None)]
 
 

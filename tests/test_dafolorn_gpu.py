@@ -41,6 +41,19 @@ def test_linear_act(dtype, M, N, K):
             assert torch.allclose(y.cpu().double(), ref, rtol=tol, atol=tol), (act[0], f32)
 
 
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("width", [72, 76, 1040])
+def test_embed_rows(dtype, width):
+    from nanovllm import hip_ops
+    wp = hip_ops.round8(width)
+    table = torch.randn(50, width, generator=g(1)).to(DT[dtype])
+    ids = torch.tensor([3, 49, 0, 3, 17])
+    cat = torch.full((5, 2 * wp), 7.0, dtype=DT[dtype], device="cuda")
+    x = hip_ops.embed_rows(dev(ids), dev(table), wp, cat[:, wp:]).cpu()
+    assert torch.equal(x[:, :width], table[ids].float()) and torch.all(x[:, width:] == 0)
+    assert torch.equal(cat[:, wp:].cpu().float(), x) and torch.all(cat[:, :wp] == 7)
+
+
 def _portions(lens_per_step):
     """Steps of (sequence, start, length) -> metadata of glm_seq_norm."""
     at, par, steps = {}, {}, []
