@@ -13,7 +13,7 @@ void glm_set_error(const char* fmt, ...) {
     va_end(ap);
 }
 
-extern "C" int glm_abi_version(void) { return 11; }
+extern "C" int glm_abi_version(void) { return 12; }
 extern "C" const char* glm_last_error(void) { return g_err; }
 
 // ---- launch-path options: name, environment variable read once, default ------------------------------------------------
@@ -165,6 +165,25 @@ extern "C" int glm_gemm_bf16_act(const void* x, int64_t ldx, const void* w, int6
     }
     if (M >= LARGEM_MIN_AVG_ROWS) return glm_launch_gemm_largem(GEMM_ACT, p, glm_s(stream));
     return glm_launch_gemm_smallm(GEMM_PLAIN, p, glm_s(stream));
+}
+
+extern "C" int glm_gemm_bf16_glu(const void* x, int64_t ldx, const void* w, int64_t ldw, void* y, int64_t ldy, int64_t M, int N, int K,
+                                 float limit, float slope, glm_stream_t stream) {
+    GLM_CHECK_ARG(x && w && y, GLM_ERR_INVALID, "glm_gemm_bf16_glu: null pointer");
+    GLM_CHECK_ARG(M >= 0 && N > 0 && K > 0 && ldx >= K && ldy >= N && ldw >= K, GLM_ERR_INVALID,
+                  "glm_gemm_bf16_glu: bad shape M=%ld N=%d K=%d ldx=%ld ldy=%ld", (long)M, N, K, (long)ldx, (long)ldy);
+    GemmParams p;
+    memset(&p, 0, sizeof(p));
+    p.x = (const bf16_t*)x; p.ldx = ldx;
+    p.w = (const bf16_t*)w; p.ldw = ldw;
+    p.y = (bf16_t*)y; p.ldy = ldy;
+    p.R = M; p.N = N; p.K = K; p.G = 1;
+    p.act = GlmAct{GLM_ACT_GLU_CLAMP, limit, slope};
+    if (M == 1 && tinym_enabled()) {
+        const int rc = glm_launch_gemm_tinym(GEMM_GLU, p, 1, glm_s(stream));
+        if (rc != GLM_ERR_UNSUPPORTED) return rc;
+    }
+    return dispatch(GEMM_GLU, p, glm_s(stream));
 }
 
 #if !GLM_DENSE_ONLY

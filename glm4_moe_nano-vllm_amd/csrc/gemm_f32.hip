@@ -67,7 +67,22 @@ __global__ __launch_bounds__(256) void gemm_f32_kernel(const GemmF32Args a) {
     }
 }
 
+// y = clamped gated unit of fp32 rows gate | up (bf16: the epilogue of glm_gemm_bf16_glu)
+__global__ __launch_bounds__(256) void glu_f32_kernel(const float* x, int64_t ldx, float* y, int64_t ldy, int64_t M, int N, GlmAct act) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x, r = i / N;
+    const int c = (int)(i - r * N);
+    if (r < M) y[r * ldy + c] = glm_glu_precise(act, x[r * ldx + c], x[r * ldx + N + c]);
+}
+
 }  // namespace
+
+extern "C" int glm_glu_f32(const float* x, int64_t ldx, float* y, int64_t ldy, int64_t M, int N, float limit, float slope, glm_stream_t stream) {
+    GLM_CHECK_ARG(x && y && M >= 0 && N > 0 && ldx >= 2 * (int64_t)N && ldy >= N && (M * N + 255) / 256 < (1ll << 31), GLM_ERR_INVALID, "glm_glu_f32: bad shape M=%ld N=%d", (long)M, N);
+    if (M == 0) return GLM_OK;
+    hipLaunchKernelGGL(glu_f32_kernel, dim3((unsigned)((M * N + 255) / 256)), dim3(256), 0, glm_s(stream), x, ldx, y, ldy, M, N, GlmAct{GLM_ACT_GLU_CLAMP, limit, slope});
+    GLM_CHECK_LAUNCH("glm_glu_f32");
+    return GLM_OK;
+}
 
 extern "C" int glm_gemm_f32(const float* x, int64_t ldx, int64_t xb, const float* w, int64_t ldw, int64_t wb, const float* bias, float* y,
                             int64_t ldy, int64_t yb, int64_t M, int N, int K, int batch, int act, float act_a, float act_b, glm_stream_t stream) {

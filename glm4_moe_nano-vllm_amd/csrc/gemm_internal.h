@@ -17,10 +17,12 @@ enum GemmMode : int {
     // bodies take p.act / p.yf in GEMM_PLAIN.)
     GEMM_ACT = 3,
     GEMM_XIELU = 4,  // xIELU, bf16 rows
+    GEMM_GLU = 5,    // GEMM_GATEUP's layout (W rows gate|up) with the clamped gated unit of p.act instead of SiLU; fp32 up to the store
 };
+__host__ __device__ constexpr bool gemm_paired(int mode) { return mode == GEMM_GATEUP || mode == GEMM_GLU; }
 
 // activation on the fp32 accumulator of a projection (after the bias)
-enum : int { GLM_ACT_NONE = GLM_EPI_NONE, GLM_ACT_XIELU = GLM_EPI_XIELU, GLM_ACT_SOFTCAP = GLM_EPI_SOFTCAP };
+enum : int { GLM_ACT_NONE = GLM_EPI_NONE, GLM_ACT_XIELU = GLM_EPI_XIELU, GLM_ACT_SOFTCAP = GLM_EPI_SOFTCAP, GLM_ACT_GLU_CLAMP = GLM_EPI_GLU_CLAMP };
 struct GlmAct {
     int kind;
     float a, b;
@@ -39,6 +41,19 @@ __device__ __forceinline__ float glm_xielu_fast(float a, float b, float z) {
 }
 __device__ __forceinline__ float glm_act_fast(const GlmAct& t, float z) {
     return t.kind == GLM_ACT_XIELU ? glm_xielu_fast(t.a, t.b, z) : glm_act_precise(t, z);
+}
+
+// clamped gated unit: limit t.a, slope t.b:  g sigmoid(b g) (u + 1) with g <= a, -a <= u <= a.  The fp32 form, and the one for outputs
+// that are rounded to bf16 right away (exp2 and reciprocal on the hardware units).
+__device__ __forceinline__ float glm_glu_precise(const GlmAct& t, float g, float u) {
+    g = fminf(g, t.a);
+    u = fminf(fmaxf(u, -t.a), t.a);
+    return g / (1.0f + expf(-t.b * g)) * (u + 1.0f);
+}
+__device__ __forceinline__ float glm_glu_fast(const GlmAct& t, float g, float u) {
+    g = fminf(g, t.a);
+    u = fminf(fmaxf(u, -t.a), t.a);
+    return g * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * t.b * g)) * (u + 1.0f);
 }
 
 struct GemmParams {

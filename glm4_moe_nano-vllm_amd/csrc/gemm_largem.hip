@@ -306,7 +306,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
     constexpr bool PARK = C::PH8 && (VAR & LM_PARK) != 0 && (VAR & LM_WIDEST) != 0 && (VAR & LM_NOSTORE) == 0;
     constexpr int PARK_N = 4;
     constexpr bool CONT = (VAR & LM_CONT) != 0 && C::PH8 && (VAR & LM_QW) != 0 && (VAR & LM_RFIRST) != 0 && (VAR & LM_P3X) == 0 &&
-                          !PARK && !C::A8 && !C::W8 && !WSCALE && (MODE == GEMM_GATEUP || MODE == GEMM_DOWN) && (VAR & LM_EPIORD) != 0;
+                          !PARK && !C::A8 && !C::W8 && !WSCALE && (gemm_paired(MODE) || MODE == GEMM_DOWN) && (VAR & LM_EPIORD) != 0;
     int* sh = reinterpret_cast<int*>(smem + C::NSTAGE * C::STAGE - ((C::ALIAS_SH || PARK) ? 16 : 0));
     const int tid = threadIdx.x, lane = tid & 63;
     const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
@@ -410,7 +410,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
                 const int row = (wid * C::W_DMA + i) * C::WRPI + lane / C::WCPR;
                 const int ch = (lane % C::WCPR) ^ C::wswz(row);
                 int wr;
-                if (MODE == GEMM_GATEUP) wr = (row >> 7) * p.N + min(ntile * 128 + (row & 127), p.N - 1);
+                if (gemm_paired(MODE)) wr = (row >> 7) * p.N + min(ntile * 128 + (row & 127), p.N - 1);
                 else wr = min(ntile * LM_BN + row, p.N - 1);
                 if constexpr (C::W8 || C::A8) wvo[i] = (unsigned)(wr * (int)p.ldw + ch * 16);
                 else wvo[i] = (unsigned)(wr * (int)p.ldw + ch * 8) * 2u;
@@ -433,7 +433,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
             const int ch = (lane % C::CPR) ^ C::swz(row);
             wch[i] = ch;
             int wr;
-            if (MODE == GEMM_GATEUP) {
+            if (gemm_paired(MODE)) {
                 const int half = row >> 7;  // 0: gate rows, 1: up rows
                 wr = half * p.N + min(ntile * 128 + (row & 127), p.N - 1);
             } else {
@@ -524,7 +524,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
 #pragma unroll
         for (int t = 0; t < 4; ++t) {
             int wrow;
-            if (MODE == GEMM_GATEUP) wrow = (t < 2 ? wn * 32 + 16 * t : 128 + wn * 32 + 16 * (t - 2)) + c;
+            if (gemm_paired(MODE)) wrow = (t < 2 ? wn * 32 + 16 * t : 128 + wn * 32 + 16 * (t - 2)) + c;
             else wrow = wn * 64 + 16 * t + c;
             if constexpr (C::W8)  // 8 bytes: k = 32 ks + 8 g4 .. +8 = chunk 2 ks + (g4 >> 1), half g4 & 1
                 rel[ks * (4 + C::MT) + t] = wrow * C::WRB + (((2 * ks + (g4 >> 1)) ^ C::wswz(wrow)) << 4) + ((g4 & 1) << 3);
@@ -568,7 +568,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
             static_for<4>([&](auto tc) {
                 constexpr int t = decltype(tc)::value;
                 constexpr int idx = ks * (4 + C::MT) + t;
-                constexpr int off = MODE == GEMM_GATEUP ? (t < 2 ? 16 * t : 128 + 16 * (t - 2)) * C::WRB : 16 * t * C::WRB;
+                constexpr int off = gemm_paired(MODE) ? (t < 2 ? 16 * t : 128 + 16 * (t - 2)) * C::WRB : 16 * t * C::WRB;
                 if (HALF == 0 || (HALF == 1) == (idx < C::NF / 2)) {
                     if constexpr (C::W8) lds_read_b64_o<off>(fr[ks * 4 + t], aw);  // fp8 as read; frags_cvt() fills f[idx]
                     else lds_read_b128_o<off>(f[idx], aw);
@@ -583,7 +583,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
     };
 
     // store instructions per wave of a full tile (16-byte stores: one per pair of output tiles)
-    constexpr int LM_NOUT = MODE == GEMM_GATEUP ? 2 : 4;
+    constexpr int LM_NOUT = gemm_paired(MODE) ? 2 : 4;
     constexpr int LM_STORES_FULL = C::MT * ((VAR & LM_WIDEST) ? LM_NOUT / 2 : LM_NOUT);
     int pending_stores = 0;
     bool park_pending = false;
@@ -762,7 +762,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
                 const unsigned aw = fbw[ks] + so;
                 static_for<NT>([&](auto tc) {
                     constexpr int t = t0 + decltype(tc)::value;
-                    constexpr int off = MODE == GEMM_GATEUP ? (t < 2 ? 16 * t : 128 + 16 * (t - 2)) * C::WRB : 16 * t * C::WRB;
+                    constexpr int off = gemm_paired(MODE) ? (t < 2 ? 16 * t : 128 + 16 * (t - 2)) * C::WRB : 16 * t * C::WRB;
                     if constexpr (C::W8) lds_read_b64_o<off>(fwr[ks * 4 + t], aw);
                     else lds_read_b128_o<off>(fw[ks * 4 + t], aw);
                 });
@@ -1381,8 +1381,8 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
 
         // ---- epilogue of the finished tile ----
         constexpr bool WIDE = (VAR & LM_WIDEST) != 0, NOSTORE = (VAR & LM_NOSTORE) != 0;
-        constexpr int NOUT = MODE == GEMM_GATEUP ? 2 : 4;  // 16-column output tiles per wave
-        const int ncol_w = MODE == GEMM_GATEUP ? ntile_c * 128 + wn * 32 : ntile_c * LM_BN + wn * 64;
+        constexpr int NOUT = gemm_paired(MODE) ? 2 : 4;  // 16-column output tiles per wave
+        const int ncol_w = gemm_paired(MODE) ? ntile_c * 128 + wn * 32 : ntile_c * LM_BN + wn * 64;
         const bool scaled = MODE == GEMM_DOWN && grp_c < p.n_scaled;
         bool qkv_epi = false;
         if constexpr (MODE == GEMM_PLAIN && WIDE && !WSCALE) qkv_epi = p.qkv_q != nullptr;
@@ -1451,7 +1451,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
                     }
                 }
             }
-        } else if constexpr (C::A8 && MODE == GEMM_GATEUP) {
+        } else if constexpr (C::A8 && gemm_paired(MODE)) {
             // ---- fp8 x fp8 gate|up (r05): the accumulator x weight-row scale x token scale is the bf16 GEMM's value up to the
             // fp8 roundings of its inputs; same rounding points behind it (mlp.py:49-53: bf16 gate_up, bf16 silu, bf16
             // product).  The product is then quantised for the down projection's fp8 operand in MX form, decided locally:
@@ -1542,7 +1542,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
                 float o[4];
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
-                    if (MODE == GEMM_GATEUP) {
+                    if (gemm_paired(MODE)) {
                         float ga = acc[t][mt][r], ua = acc[t + 2][mt][r];
                         if constexpr (WSCALE) {  // weights expanded from fp8: per-row scale on the fp32 accumulators (uniform branch)
                             const float* ws = p.wscale + (int64_t)grp_c * p.wscale_gstride;
@@ -1550,7 +1550,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
                             ga *= ws[n1];
                             ua *= ws[p.N + n1];
                         }
-                        o[r] = rbf(glm_silu(rbf(ga))) * rbf(ua);
+                        o[r] = MODE == GEMM_GLU ? glm_glu_fast(p.act, ga, ua) : rbf(glm_silu(rbf(ga))) * rbf(ua);
                     } else {
                         float a = acc[t][mt][r];
                         if constexpr (WSCALE) a *= wsv[t][r];
@@ -1630,7 +1630,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
         }
         if constexpr ((VAR & LM_EPIORD) != 0) {
             // exact only when every store instruction of the wave ran: all rows and columns of the tile exist
-            const bool full = !LATE_FILL && mcnt_c == C::BM && ncol_w + (MODE == GEMM_GATEUP ? 32 : 64) <= p.N && !NOSTORE &&
+            const bool full = !LATE_FILL && mcnt_c == C::BM && ncol_w + (gemm_paired(MODE) ? 32 : 64) <= p.N && !NOSTORE &&
                               !((VAR & LM_LDSEPI) != 0 && NOUT == 4) && !(MODE == GEMM_PLAIN && p.qkv_q != nullptr) && !(MODE == GEMM_ACT && p.yf != nullptr);
             pending_stores = full ? LM_STORES_FULL - (do_park ? PARK_N : 0) : 0;
         }
@@ -1661,7 +1661,7 @@ int env_variant() { return glm_option(GLM_OPT_LARGEM_VARIANT); }
 
 template <int MODE, class C, int VAR>
 int launch_largem_cfg(const GemmParams& p, hipStream_t st) {
-    const int cols_per_wg = MODE == GEMM_GATEUP ? 128 : LM_BN;
+    const int cols_per_wg = gemm_paired(MODE) ? 128 : LM_BN;
     const int n_tiles = (p.N + cols_per_wg - 1) / cols_per_wg;
     const int64_t combos = p.offs ? (p.R / C::BM + p.G) : (p.R + C::BM - 1) / C::BM;
     const int LM_BAND = g_largem_band;
@@ -1714,7 +1714,7 @@ int launch_largem(const GemmParams& p, hipStream_t st) {
     int var = g_largem_variant >= 0 ? g_largem_variant : env_variant() >= 0 ? env_variant() : GLM_LM_DEFAULT_VAR;
     if (var < 0) var = LM_LEAN | LM_WIDEST | LM_PH8 | LM_QW | LM_RFIRST | LM_NOPRIO | LM_EPIORD;
     const int bk = use_b ? ((var & LM_PH8) ? LmCfgC::BK : LmCfgB::BK) : LmCfgA::BK;
-    const int64_t wrows = MODE == GEMM_GATEUP ? 2 * (int64_t)p.N : (int64_t)p.N;
+    const int64_t wrows = gemm_paired(MODE) ? 2 * (int64_t)p.N : (int64_t)p.N;
     const bool lean_ok = p.K % bk == 0 && p.R * p.ldx * 2 < (1ll << 31) && wrows * p.ldw * 2 < (1ll << 31) &&
                          p.N % 8 == 0 && p.ldy % 8 == 0 && glm_aligned16(p.y);
     if (p.w_fp8) {
@@ -1725,7 +1725,7 @@ int launch_largem(const GemmParams& p, hipStream_t st) {
             glm_set_error("gemm_largem(fp8 weights): shape not covered (K=%d N=%d ldw=%ld)", p.K, p.N, (long)p.ldw);
             return GLM_ERR_UNSUPPORTED;
         }
-        if constexpr (MODE == GEMM_PLAIN || MODE == GEMM_ACT || MODE == GEMM_XIELU) {
+        if constexpr (MODE != GEMM_GATEUP && MODE != GEMM_DOWN) {
             glm_set_error("gemm_largem(fp8 weights): only the grouped expert projections are quantised");
             return GLM_ERR_UNSUPPORTED;
         } else {
@@ -1847,6 +1847,7 @@ int glm_launch_gemm_largem(int mode, const GemmParams& p, hipStream_t st) {
 #endif  // !GLM_DENSE_ONLY
     if (mode == GEMM_ACT && p.yf == nullptr && p.act.kind == GLM_ACT_XIELU) return launch_largem<GEMM_XIELU>(p, st);
     if (mode == GEMM_ACT) return launch_largem<GEMM_ACT>(p, st);
+    if (mode == GEMM_GLU) return launch_largem<GEMM_GLU>(p, st);
     return launch_largem<GEMM_PLAIN>(p, st);
 }
 

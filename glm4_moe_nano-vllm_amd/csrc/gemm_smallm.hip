@@ -105,7 +105,7 @@ __device__ __forceinline__ void smallm_epilogue(const GemmParams& p, f32x4_t (&a
         const int row = 16 * mt + c;
         if (row >= mcnt) continue;
         bf16_t* yrow = p.y + (int64_t)(m0 + row) * p.ldy;
-        if (MODE == GEMM_GATEUP) {
+        if (gemm_paired(MODE)) {
             // row tiles [0, RT/2) are gate columns, [RT/2, RT) the matching up columns
 #pragma unroll
             for (int j = 0; j < RT / 2; ++j) {
@@ -114,7 +114,8 @@ __device__ __forceinline__ void smallm_epilogue(const GemmParams& p, f32x4_t (&a
                     float o[4];
 #pragma unroll
                     for (int r = 0; r < 4; ++r)
-                        o[r] = rbf(glm_silu(rbf(acc[j][mt][r]))) * rbf(acc[RT / 2 + j][mt][r]);
+                        o[r] = MODE == GEMM_GLU ? glm_glu_fast(p.act, acc[j][mt][r], acc[RT / 2 + j][mt][r])
+                                                : rbf(glm_silu(rbf(acc[j][mt][r]))) * rbf(acc[RT / 2 + j][mt][r]);
                     u32x2_t v = {pack2bf(o[0], o[1]), pack2bf(o[2], o[3])};
                     *reinterpret_cast<u32x2_t*>(yrow + n) = v;
                 }
@@ -185,7 +186,7 @@ __device__ __forceinline__ void smallm_body(const GemmParams& p, char* smem, int
     const char* wrow[RT];
     int wrowi[RT];  // weight row index (for the fp8 per-row scale)
     int ncol0;  // first output column of this wave
-    if (MODE == GEMM_GATEUP) {
+    if (gemm_paired(MODE)) {
         ncol0 = (blockIdx.x * WR + wr) * 16;
         const int r = min(ncol0 + c, p.N - 1);
         wrowi[0] = r;
@@ -350,8 +351,8 @@ __device__ __forceinline__ void smallm_body(const GemmParams& p, char* smem, int
         const float* ws = p.wscale + (int64_t)grp * p.wscale_gstride;
 #pragma unroll
         for (int rt = 0; rt < RT; ++rt) {
-            const int rbase = (MODE == GEMM_GATEUP ? (rt == 0 ? ncol0 : p.N + ncol0) : ncol0 + 16 * rt) + 4 * g4;
-            const int rmax = MODE == GEMM_GATEUP ? 2 * p.N - 1 : p.N - 1;
+            const int rbase = (gemm_paired(MODE) ? (rt == 0 ? ncol0 : p.N + ncol0) : ncol0 + 16 * rt) + 4 * g4;
+            const int rmax = gemm_paired(MODE) ? 2 * p.N - 1 : p.N - 1;
             float sc[4];
 #pragma unroll
             for (int r = 0; r < 4; ++r) sc[r] = ws[min(rbase + r, rmax)];
@@ -379,7 +380,7 @@ __global__ __launch_bounds__(NWAVES * 64) void gemm_smallm_kernel(const GemmPara
     }
     constexpr int MB = 16 * MTMAX;
     constexpr int XBUF = WS * MB * SM_XROWB;  // bytes per x buffer (sized for MTMAX)
-    static_assert(MODE != GEMM_GATEUP || RT == 2, "gate|up needs two row tiles");
+    static_assert(!gemm_paired(MODE) || RT == 2, "gate|up needs two row tiles");
     extern __shared__ __attribute__((aligned(16))) char smem[];
     int* sh = reinterpret_cast<int*>(smem + 2 * XBUF);
     glm_locate_block(p.offs, p.G, p.R, MB, blockIdx.y, sh);
@@ -475,7 +476,7 @@ __device__ __forceinline__ void smallm_body_dma(const GemmParams& p, char* smem,
     constexpr int WROWS = 16 * RT, XROWS = 16 * MT;
     constexpr int WT = WROWS * 256, STAGE = (WROWS + XROWS) * 256;
     constexpr int NW_DMA = WROWS / 4, NX_DMA = XROWS / 4, NDMA = NW_DMA + NX_DMA;
-    constexpr int CPW = MODE == GEMM_GATEUP ? 8 * RT : 16 * RT;  // output columns per wave per tile
+    constexpr int CPW = gemm_paired(MODE) ? 8 * RT : 16 * RT;  // output columns per wave per tile
     const int tid = threadIdx.x, lane = tid & 63;
     const int wid = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int ws = wid % WS, wr = wid / WS;
@@ -499,7 +500,7 @@ __device__ __forceinline__ void smallm_body_dma(const GemmParams& p, char* smem,
     for (int i = 0; i < NW_DMA; ++i) {
         const int row = 4 * i + r4;  // 0 .. WROWS-1
         int wi;
-        if (MODE == GEMM_GATEUP)  // first half of the stage rows = gate columns, second half = the same up columns
+        if (gemm_paired(MODE))  // first half of the stage rows = gate columns, second half = the same up columns
             wi = (row < WROWS / 2 ? 0 : p.N) + min(ncol_first + row % (WROWS / 2), p.N - 1);
         else wi = min(ncol_first + row, p.N - 1);
         wsrc[i] = wg + (int64_t)wi * p.ldw;
@@ -607,14 +608,15 @@ __device__ __forceinline__ void smallm_body_dma(const GemmParams& p, char* smem,
                 const int row = 16 * mt + c;
                 if (row >= mcnt) continue;
                 bf16_t* yrow = p.y + (int64_t)(m0 + row) * p.ldy;
-                if (MODE == GEMM_GATEUP) {
+                if (gemm_paired(MODE)) {
 #pragma unroll
                     for (int j = 0; j < RT / 2; ++j) {
                         const int n = ncol0 + 16 * j + 4 * g4;
                         float o[4];
 #pragma unroll
                         for (int r = 0; r < 4; ++r)
-                            o[r] = rbf(glm_silu(rbf(acc[j][mt][r]))) * rbf(acc[RT / 2 + j][mt][r]);
+                            o[r] = MODE == GEMM_GLU ? glm_glu_fast(p.act, acc[j][mt][r], acc[RT / 2 + j][mt][r])
+                                                    : rbf(glm_silu(rbf(acc[j][mt][r]))) * rbf(acc[RT / 2 + j][mt][r]);
                         const u32x2_t v = {pack2bf(o[0], o[1]), pack2bf(o[2], o[3])};
                         *reinterpret_cast<u32x2_t*>(yrow + n) = v;
                     }
@@ -684,7 +686,7 @@ __global__ __launch_bounds__(NWAVES * 64) void gemm_smallm_dma_kernel(const Gemm
     }
     constexpr int MB = 16 * MTMAX;
     constexpr int RING = NWAVES * 2 * (16 * RT + 16 * MTMAX) * 256;
-    static_assert(MODE != GEMM_GATEUP || RT == 2 || RT == 4, "gate|up: gate and up tiles come in pairs");
+    static_assert(!gemm_paired(MODE) || RT == 2 || RT == 4, "gate|up: gate and up tiles come in pairs");
     extern __shared__ __attribute__((aligned(16))) char smem[];
     int* sh = reinterpret_cast<int*>(smem + RING);
     glm_locate_block(p.offs, p.G, p.R, MB, blockIdx.y, sh);
@@ -727,7 +729,7 @@ __device__ __forceinline__ void smallm_body_sx(const GemmParams& p, char* smem, 
     constexpr int NDMA = NW_DMA + NX_DMA;
     constexpr int XRPI = 1024 / XROWB;            // activation rows per DMA instruction (4 or 2)
     constexpr int XCPR = XROWB / 16;              // 16-B chunks per activation row (16 or 32)
-    constexpr int CPW = MODE == GEMM_GATEUP ? 8 * RT : 16 * RT;  // output columns per wave
+    constexpr int CPW = gemm_paired(MODE) ? 8 * RT : 16 * RT;  // output columns per wave
     constexpr int WB = W8 ? 1 : 2;
 
     const int tid = threadIdx.x, lane = tid & 63;
@@ -746,7 +748,7 @@ __device__ __forceinline__ void smallm_body_sx(const GemmParams& p, char* smem, 
     for (int i = 0; i < NW_DMA; ++i) {
         const int row = 4 * i + r4;
         int wi;
-        if (MODE == GEMM_GATEUP) wi = (row < WROWS / 2 ? 0 : p.N) + min(ncol0 + row % (WROWS / 2), p.N - 1);
+        if (gemm_paired(MODE)) wi = (row < WROWS / 2 ? 0 : p.N) + min(ncol0 + row % (WROWS / 2), p.N - 1);
         else wi = min(ncol0 + row, p.N - 1);
         wsrc[i] = wg + (int64_t)wi * p.ldw * WB;
         wk[i] = (pch ^ (row & 15)) << 4;
@@ -867,8 +869,8 @@ __device__ __forceinline__ void smallm_body_sx(const GemmParams& p, char* smem, 
         const float* ws = p.wscale + (int64_t)grp * p.wscale_gstride;
 #pragma unroll
         for (int rt = 0; rt < RT; ++rt) {
-            const int rb = (MODE == GEMM_GATEUP ? (rt < RT / 2 ? ncol0 + 16 * rt : p.N + ncol0 + 16 * (rt - RT / 2)) : ncol0 + 16 * rt) + 4 * g4;
-            const int rmax = MODE == GEMM_GATEUP ? 2 * p.N - 1 : p.N - 1;
+            const int rb = (gemm_paired(MODE) ? (rt < RT / 2 ? ncol0 + 16 * rt : p.N + ncol0 + 16 * (rt - RT / 2)) : ncol0 + 16 * rt) + 4 * g4;
+            const int rmax = gemm_paired(MODE) ? 2 * p.N - 1 : p.N - 1;
             float sc[4];
 #pragma unroll
             for (int r = 0; r < 4; ++r) sc[r] = ws[min(rb + r, rmax)];
@@ -907,7 +909,7 @@ int launch_cfg_sx(const GemmParams& p, hipStream_t st) {
     constexpr int RING = GLM_SM_SX_STAGES * (NW * 16 * RT * 256 + 16 * MTMAX * (W8 ? 512 : 256));
     static_assert(RING <= 160 * 1024, "the ring must fit the CU's 160 KiB of LDS");
     constexpr int LDS = RING;
-    const int cols_per_wg = MODE == GEMM_GATEUP ? NW * 8 * RT : NW * RT * 16;
+    const int cols_per_wg = gemm_paired(MODE) ? NW * 8 * RT : NW * RT * 16;
     const unsigned gx = (unsigned)((p.N + cols_per_wg - 1) / cols_per_wg);
     const int64_t combos = p.offs ? (p.R / MB + p.G) : (p.R + MB - 1) / MB;
     if (combos <= 0 || gx == 0) return GLM_OK;
@@ -923,7 +925,7 @@ template <int MODE, int NWAVES, int WS, int RT, int MTMAX, int TPW = 1>
 int launch_cfg_dma(const GemmParams& p, hipStream_t st) {
     static_assert(MTMAX <= 2, "the DMA variant stages at most 32 token rows");
     if (TPW > 1) {  // column-tile streams need whole tiles everywhere, else the plain one-tile kernel
-        const int step = (MODE == GEMM_GATEUP ? (NWAVES / WS) * 8 * RT : (NWAVES / WS) * RT * 16) * TPW;
+        const int step = (gemm_paired(MODE) ? (NWAVES / WS) * 8 * RT : (NWAVES / WS) * RT * 16) * TPW;
         if (p.N % step != 0) return launch_cfg_dma<MODE, NWAVES, WS, RT, MTMAX, 1>(p, st);
     }
     constexpr int WR = NWAVES / WS;
@@ -933,7 +935,7 @@ int launch_cfg_dma(const GemmParams& p, hipStream_t st) {
     static_assert(REDB <= RING, "reduction scratch must fit in the rings");
     static_assert(RING + 16 <= 160 * 1024, "the rings of all waves must fit the CU's 160 KiB of LDS");
     constexpr int LDS = RING + 16;
-    const int cols_per_wg = (MODE == GEMM_GATEUP ? WR * 8 * RT : WR * RT * 16) * TPW;
+    const int cols_per_wg = (gemm_paired(MODE) ? WR * 8 * RT : WR * RT * 16) * TPW;
     const unsigned gx = (unsigned)((p.N + cols_per_wg - 1) / cols_per_wg);
     const int64_t combos = p.offs ? (p.R / MB + p.G) : (p.R + MB - 1) / MB;
     if (combos <= 0 || gx == 0) return GLM_OK;
@@ -954,7 +956,7 @@ int launch_cfg(const GemmParams& p, hipStream_t st) {
     constexpr int REDB = WS > 1 ? WR * (WS - 1) * RT * MTMAX * 64 * 16 : 0;
     constexpr int LDS = (2 * XBUF > REDB ? 2 * XBUF : REDB) + 16;
     static_assert(REDB <= 2 * XBUF, "reduction scratch must fit in the x buffers");
-    const int cols_per_wg = MODE == GEMM_GATEUP ? WR * 16 : WR * RT * 16;
+    const int cols_per_wg = gemm_paired(MODE) ? WR * 16 : WR * RT * 16;
     const unsigned gx = (unsigned)((p.N + cols_per_wg - 1) / cols_per_wg);
     const int64_t combos = p.offs ? (p.R / MB + p.G) : (p.R + MB - 1) / MB;
     if (combos <= 0 || gx == 0) return GLM_OK;
@@ -982,10 +984,17 @@ int glm_launch_gemm_smallm(int mode, const GemmParams& p, hipStream_t st) {
     // (tools/sweep_grouped.sh, two rounds): gate|up 4,1,2,2: 272 us; 8,4,2,2: 256; 4,2,2,2: 251; 4,4,2,2: 245-249.
     // down 4,1,2,2: 130 us; 8,1,1,2: 122; 2,1,1,2: 120; 4,2,1,2: 118-120.  Splitting K over the waves of a small
     // workgroup (16 act columns of gate|up, 32 columns of down) beats one long stream per wave.
-#if !GLM_DENSE_ONLY
 #ifndef GLM_SM_CFG_GATEUP
 #define GLM_SM_CFG_GATEUP 4, 4, 2, 2
 #endif
+    // the dense gated projection: the grouped gate|up configurations (measured below)
+    if (mode == GEMM_GLU) {
+#ifndef GLM_SM_NO_DMA
+        if (Rs >= 17) return launch_cfg_dma<GEMM_GLU, 2, 2, 2, 2>(p, st);
+#endif
+        return launch_cfg<GEMM_GLU, GLM_SM_CFG_GATEUP>(p, st);
+    }
+#if !GLM_DENSE_ONLY
 #ifndef GLM_SM_CFG_DOWN
 #define GLM_SM_CFG_DOWN 4, 2, 1, 2
 #endif

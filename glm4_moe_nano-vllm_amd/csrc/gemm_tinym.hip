@@ -294,7 +294,7 @@ __device__ __forceinline__ void tinym_router_tail(const TinyParams& tp, char* sm
 template <int MODE, int M, int SEGS, bool PRO, bool TAIL = false, int RPW = TM_RPW>
 __global__ __launch_bounds__(TM_NT) void gemm_tinym_kernel(const TinyParams tp) {
     static_assert(RPW == 1 || RPW == 2 || RPW == 4, "1, 2 or 4 weight rows per tile");
-    static_assert(MODE != GEMM_GATEUP || RPW >= 2, "gate|up: a tile is gate rows + the matching up rows");
+    static_assert(!gemm_paired(MODE) || RPW >= 2, "gate|up: a tile is gate rows + the matching up rows");
     constexpr int HALF = RPW >= 2 ? RPW / 2 : 1;  // gate|up: HALF gate rows + the matching HALF up rows
     const GemmParams& p = tp.g;
     extern __shared__ __attribute__((aligned(16))) char smem[];
@@ -309,7 +309,7 @@ __global__ __launch_bounds__(TM_NT) void gemm_tinym_kernel(const TinyParams tp) 
     constexpr int KU = SEGS * 512;                 // k elements per unit
     const int nunits = (K + KU - 1) / KU;
     const int Kp = nunits * KU;                    // padded row length in LDS (pad = zeros)
-    const int tpg = MODE == GEMM_GATEUP ? p.N / HALF : p.N / RPW;  // tiles per group
+    const int tpg = gemm_paired(MODE) ? p.N / HALF : p.N / RPW;  // tiles per group
 
     // ---- non-empty groups (grouped modes) ----
     int nact = 1;
@@ -351,7 +351,7 @@ __global__ __launch_bounds__(TM_NT) void gemm_tinym_kernel(const TinyParams tp) 
         t.m0 = p.offs ? p.offs[grp] : 0;
         t.mcnt = p.offs ? min(p.offs[grp + 1] - t.m0, M) : (int)min((int64_t)M, p.R);
         const char* wg = reinterpret_cast<const char*>(p.w + (int64_t)grp * p.w_gstride);
-        if (MODE == GEMM_GATEUP) {  // rows: gate n .. n+HALF-1, then up n .. n+HALF-1
+        if (gemm_paired(MODE)) {  // rows: gate n .. n+HALF-1, then up n .. n+HALF-1
             t.ncol = HALF * ti;
 #pragma unroll
             for (int r = 0; r < RPW; ++r) t.wrow[r] = wg + ((int64_t)((r / HALF) * p.N + t.ncol + (r % HALF)) * p.ldw) * 2;
@@ -401,7 +401,7 @@ __global__ __launch_bounds__(TM_NT) void gemm_tinym_kernel(const TinyParams tp) 
 
     // ---- activation rows into LDS: [rows][Kp] bf16, pad zeroed ----
     //   PLAIN: rows 0..M-1 = x rows;  GATEUP: row t = token t (T = p.R / ... tokens, all of x);  DOWN: row r = act row r
-    const int xrows = MODE == GEMM_PLAIN ? M : (MODE == GEMM_GATEUP ? tp.n_tokens : (int)p.R);
+    const int xrows = MODE == GEMM_PLAIN ? M : (gemm_paired(MODE) ? tp.n_tokens : (int)p.R);
     bf16_t* xs = reinterpret_cast<bf16_t*>(smem);
     if (PRO) {
         // combine of the previous MoE block + input add-RMSNorm, token by token, exactly the stand-alone launch's code;
@@ -442,7 +442,7 @@ __global__ __launch_bounds__(TM_NT) void gemm_tinym_kernel(const TinyParams tp) 
         const int j = m < t.mcnt ? m : 0;  // a group with fewer rows than M: the extra column is computed and dropped
         int row;
         if (MODE == GEMM_PLAIN) row = j;
-        else if (MODE == GEMM_GATEUP) row = p.src ? p.src[t.m0 + j] : t.m0 + j;
+        else if (gemm_paired(MODE)) row = p.src ? p.src[t.m0 + j] : t.m0 + j;
         else row = t.m0 + j;
         return xs + (int64_t)row * Kp;
     };
@@ -474,10 +474,10 @@ __global__ __launch_bounds__(TM_NT) void gemm_tinym_kernel(const TinyParams tp) 
         for (int m = 0; m < M; ++m) {
             if (m >= t.mcnt) continue;
             const int64_t row = t.m0 + m;
-            if (MODE == GEMM_GATEUP) {
+            if (gemm_paired(MODE)) {
                 float a[HALF];
 #pragma unroll
-                for (int j = 0; j < HALF; ++j) a[j] = rbf(glm_silu(rbf(o[j][m]))) * rbf(o[HALF + j][m]);
+                for (int j = 0; j < HALF; ++j) a[j] = MODE == GEMM_GLU ? glm_glu_fast(p.act, o[j][m], o[HALF + j][m]) : rbf(glm_silu(rbf(o[j][m]))) * rbf(o[HALF + j][m]);
                 if constexpr (HALF == 2) *reinterpret_cast<unsigned*>(p.y + row * p.ldy + t.ncol) = pack2bf(a[0], a[1]);
                 else p.y[row * p.ldy + t.ncol] = f2bf(a[0]);
             } else {
@@ -607,7 +607,7 @@ int launch_tiny(const TinyParams& tp, int xrows, hipStream_t st) {
     GLM_CHECK_ARG(lds <= 156 * 1024, GLM_ERR_UNSUPPORTED, "gemm_tinym: %d activation rows of %d do not fit the LDS", xrows, Kp);
     auto kern = gemm_tinym_kernel<MODE, M, SEGS, PRO, TAIL, RPW>;
     GLM_SET_MAX_LDS(kern, 156 * 1024, "gemm_tinym");
-    const int64_t tiles = (int64_t)(p.offs ? p.G : 1) * (MODE == GEMM_GATEUP ? p.N / (RPW / 2) : p.N / RPW);
+    const int64_t tiles = (int64_t)(p.offs ? p.G : 1) * (gemm_paired(MODE) ? p.N / (RPW / 2) : p.N / RPW);
     int nwg = n_cus();
     if (tiles < nwg) nwg = (int)tiles;
     if (TAIL) {  // the tail's scratch lives in the (dead) activation area; behind it TR_ROWS gate rows
@@ -626,7 +626,7 @@ int launch_tiny(const TinyParams& tp, int xrows, hipStream_t st) {
 
 bool tiny_shape_ok(int mode, const GemmParams& p) {
     if (p.K % 8 != 0 || p.ldx % 8 != 0 || p.ldw % 8 != 0 || !glm_aligned16(p.x) || !glm_aligned16(p.w)) return false;
-    if (mode == GEMM_GATEUP) return p.N % 2 == 0 && p.ldy % 2 == 0 && (((uintptr_t)p.y) & 3) == 0;
+    if (gemm_paired(mode)) return p.N % 2 == 0 && p.ldy % 2 == 0 && (((uintptr_t)p.y) & 3) == 0;
     return p.N % TM_RPW == 0 && p.ldy % 4 == 0 && (((uintptr_t)p.y) & 7) == 0;
 }
 
@@ -650,6 +650,7 @@ int glm_launch_gemm_tinym(int mode, const GemmParams& p, int n_tokens, hipStream
     GLM_CHECK_ARG(M == 1, GLM_ERR_UNSUPPORTED, "gemm_tinym: %d rows per block", M);
     // units: 4 rows x 4 KiB for long rows; a short K (expert down projection, 1408) as ONE unit of 3-KiB rows
     if (mode == GEMM_PLAIN) return launch_tiny<GEMM_PLAIN, 1, GLM_TM_SEGS_PLAIN, false, false, GLM_TM_RPW_PLAIN>(tp, 1, st);
+    if (mode == GEMM_GLU) return launch_tiny<GEMM_GLU, 1, 8, false, false, 2>(tp, 1, st);
 #if !GLM_DENSE_ONLY
     // grouped launches: rows per tile chosen for the TAIL of the launch — a workgroup's waves pull tiles from a counter, and
     // the launch ends when the slowest wave has finished its last tile; at Air dims one token gives 24.75 tiles of 4 rows per

@@ -1,0 +1,719 @@
+// group_attn.hip — causal attention with grouped heads (H query heads over G key / value heads) read from paged caches, with
+// what a design may add to it, each a parameter: a sliding window or chunks (a token sees its own chunk only, chunks counted from
+// position 0 of the sequence), a distance bias per head (slope_h * (i - j) is taken off the scaled score), a learned sink per
+// head (mass exp(sink) in the denominator, without key or value).  Head sizes of keys and values are independent.  gfx950 only.
+//
+//   group_kv_store       rows of a projection -> the pages of both caches, [block][G][tokens of a block][head size]
+//   group_attn_prefill   long portions: 128 query rows of one head per workgroup
+//   group_attn_decode    decoded tokens and short portions: 16 (token, head) rows of one key / value head per workgroup, the keys
+//                        split over the waves and over workgroups (glm_attn_merge adds the splits up)
+//   group_attn_plain     any head size, bf16 or fp32: one (token, head) per workgroup, vector FMAs, every step in fp32
+//
+// All of them read keys and values of the step's own tokens from the cache, where group_kv_store has put them, so a portion of a
+// prompt, a decoded token and a layer that borrows another layer's cache are the same thing.
+//
+// Roofline: MFMA for prefill, HBM for decode (the visible keys and values, read once).  S^T = K . Q^T, fp32 online softmax per lane
+// column in log2 units, O^T += V^T . P^T straight from registers.  Tiles come in by LDS-DMA, double-buffered; keys behind
+// the last visible one are fetched from a page of zeros (unused cache memory may hold NaNs).  The running maximum is raised only when
+// a score exceeds it by more than 2^8 (the sums stay exact: the reference point cancels).
+#include "common.h"
+#include "attn_lds.h"
+
+namespace {
+
+constexpr float GA_LOG2E = 1.4426950408889634f;
+__device__ const u32x4_t ga_zero_page[4] = {};
+
+struct GroupArgs {
+    const void* q;        // [rows, ldq], head h at h*dk
+    int64_t ldq;
+    const void *kc, *vc;  // caches
+    int64_t n_blocks;
+    int bs, log2_bs;      // tokens per block (log2_bs < 0: not a power of two)
+    const int32_t* bt;    // [sequences, bt_stride]
+    int64_t bt_stride;
+    const int32_t *pos, *seq_of;  // of the rows of q
+    const int32_t *q_start, *tile_a, *tile_b;
+    int seq0, n_tiles, H, G, dk, dv, window, chunk, nsplit;
+    float scale;
+    const float *slope, *sink;  // [H] or nullptr
+    void* out;            // [rows, ldo], head h at h*dv
+    int64_t ldo;
+    float *part_o, *part_ml;    // nsplit > 1: [rows*H][nsplit][dv], [rows*H][nsplit][2]
+    int64_t rows;
+};
+
+// first position that position p sees
+__device__ __forceinline__ int ga_first(const GroupArgs& a, int p) {
+    int lo = 0;
+    if (a.window > 0) lo = max(lo, p - a.window + 1);
+    if (a.chunk > 0) lo = max(lo, p - p % a.chunk);
+    return lo;
+}
+__device__ __forceinline__ int ga_block(const GroupArgs& a, int j) { return a.log2_bs >= 0 ? j >> a.log2_bs : j / a.bs; }
+// row of a cache (in units of the head size) of key position j with block id blk, head g
+__device__ __forceinline__ int64_t ga_row(const GroupArgs& a, int blk, int j, int g) { return ((int64_t)blk * a.G + g) * a.bs + (j - ga_block(a, j) * a.bs); }
+__device__ __forceinline__ bool ga_ok(const GroupArgs& a, int blk) { return blk >= 0 && blk < a.n_blocks; }
+
+// ---------------------------------------------------------------------------------------------------------------------------
+struct StoreArgs {
+    const char* src;      // row r at r*ld bytes; keys at k_off, values at v_off (bytes)
+    int64_t ld, k_off, v_off;
+    const int32_t* slots; // [T] block * bs + place, < 0: no cache row
+    char *kc, *vc;
+    int64_t T, n_slots;
+    int G, bs, ku, vu;    // 16-byte units of a key / value head
+};
+__global__ __launch_bounds__(256) void group_kv_store_kernel(const StoreArgs a) {
+    const int per = a.G * (a.ku + a.vu);
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x;
+    const int64_t r = i / per;
+    if (r >= a.T) return;
+    int u = (int)(i - r * per);
+    const int64_t slot = a.slots[r];
+    if (slot < 0 || slot >= a.n_slots) return;
+    const bool val = u >= a.G * a.ku;
+    if (val) u -= a.G * a.ku;
+    const int w = val ? a.vu : a.ku, g = u / w, c = u - g * w;
+    const u32x4_t x = *reinterpret_cast<const u32x4_t*>(a.src + r * a.ld + (val ? a.v_off : a.k_off) + (int64_t)u * 16);
+    char* dst = val ? a.vc : a.kc;
+    *reinterpret_cast<u32x4_t*>(dst + (((slot / a.bs * a.G + g) * a.bs + slot % a.bs) * w + c) * 16) = x;
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------
+// the two products of a 32-key slab and the softmax between them, for NT tiles of 16 query rows (lane c holds row c of each)
+template <int DK, int DV, int NT>
+struct Slab {
+    static constexpr int KS = DK / 32, VT = DV / 16, KB = DK * 2, VB = DV * 2;
+    static constexpr bool VEARLY = DK + DV <= 256;                    // V fragments requested in front of the score products
+    static constexpr int KG = KS < 4 ? KS : 4, VG = VEARLY ? VT : 4;  // fragments per request group
+    u32x4_t qf[NT][KS];
+    f32x4_t acc[NT][VT];
+    float m_run[NT], l_run[NT], slope2[NT];
+    int rp[NT], rlo[NT];                                  // position of the lane's row and the first one it sees; rp < 0: no row
+    int any_lo[NT], any_hi[NT], full_lo[NT], full_hi[NT]; // keys that some row / every row of the tile sees
+    unsigned k_rel[2], v_rel[4];
+
+    __device__ __forceinline__ void init(int lane) {
+        const int c = lane & 15, g = lane >> 4;
+        // K row c, chunk 4 i + g (its low three bits depend on the parity of i only); V row 4 g + qq
+#pragma unroll
+        for (int e = 0; e < 2; ++e) k_rel[e] = c * KB + (((4 * e + g) ^ attn_swz(c)) << 4);
+        const int qq = (lane >> 2) & 3, pp = lane & 3, vr = 4 * g + qq;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v_rel[e] = vr * VB + (((2 * e + (pp >> 1)) ^ attn_swz(vr)) << 4) + ((pp & 1) << 3);
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+            m_run[t] = -INFINITY;
+            l_run[t] = 0.f;
+#pragma unroll
+            for (int d = 0; d < VT; ++d) acc[t][d] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        }
+    }
+    // kst, vst: LDS addresses of the slab's first key row and value row; j0: position of its first key
+    __device__ __forceinline__ void run(unsigned kst, unsigned vst, int j0, int g, float sc) {
+        bool live[NT], some = false;
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+            live[t] = j0 <= any_hi[t] && j0 + 31 >= any_lo[t];
+            some = some || live[t];
+        }
+        if (!some) return;
+        u32x2_t vf[VG][2];
+        auto read_v = [&](auto D0) {
+            static_for<VG>([&](auto I) {
+                constexpr int i = decltype(I)::value, d = decltype(D0)::value + i;
+                lds_read_tr16_b64<(d >> 2) * 128>(vf[i][0], vst + v_rel[d & 3]);
+                lds_read_tr16_b64<(d >> 2) * 128 + 16 * VB>(vf[i][1], vst + v_rel[d & 3]);
+            });
+        };
+        f32x4_t s[NT][2];
+#pragma unroll
+        for (int t = 0; t < NT; ++t)
+#pragma unroll
+            for (int kt = 0; kt < 2; ++kt) s[t][kt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        static_for<(KS + KG - 1) / KG>([&](auto GI) {
+            constexpr int k0 = decltype(GI)::value * KG, kn = KS - k0 < KG ? KS - k0 : KG;
+            constexpr bool last = k0 + KG >= KS;
+            u32x4_t kf[2][KG];
+            static_for<kn>([&](auto I) {
+                constexpr int i = k0 + decltype(I)::value;
+                lds_read_b128<(i >> 1) * 128>(kf[0][i - k0], kst + k_rel[i & 1]);
+                lds_read_b128<(i >> 1) * 128 + 16 * KB>(kf[1][i - k0], kst + k_rel[i & 1]);
+            });
+            if constexpr (last && VEARLY) {
+                read_v(std::integral_constant<int, 0>{});
+                // the K fragments are in; the V fragments (issued last) may still be on their way
+                asm volatile("s_waitcnt lgkmcnt(%0)" ::"i"(2 * VG <= 15 ? 2 * VG : 15) : "memory");
+            } else {
+                wait_lds();
+            }
+#pragma unroll
+            for (int i = 0; i < kn; ++i) asm volatile("" : "+v"(kf[0][i]), "+v"(kf[1][i]));
+#pragma unroll
+            for (int i = 0; i < kn; ++i)
+#pragma unroll
+                for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+                    for (int t = 0; t < NT; ++t)
+                        s[t][kt] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, kf[kt][i]), __builtin_bit_cast(bf16x8_t, qf[t][k0 + i]), s[t][kt], 0, 0, 0);
+        });
+        bf16x8_t pf[NT];
+#pragma unroll
+        for (int t = 0; t < NT; ++t) {
+            if (!live[t]) {
+#pragma unroll
+                for (int i = 0; i < 8; ++i) pf[t][i] = (__bf16)0.f;
+                continue;
+            }
+            const int jl = j0 + 4 * g;
+            const float b0 = slope2[t] * (float)(jl - rp[t]);
+            float mx = -INFINITY;
+            if (j0 >= full_lo[t] && j0 + 31 <= full_hi[t]) {
+#pragma unroll
+                for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) {
+                        s[t][kt][r] = fmaf(s[t][kt][r], sc, fmaf(slope2[t], (float)(16 * kt + r), b0));
+                        mx = fmaxf(mx, s[t][kt][r]);
+                    }
+            } else {
+#pragma unroll
+                for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) {
+                        const int j = jl + 16 * kt + r;
+                        const float v = fmaf(s[t][kt][r], sc, fmaf(slope2[t], (float)(16 * kt + r), b0));
+                        s[t][kt][r] = (j <= rp[t] && j >= rlo[t]) ? v : -INFINITY;
+                        mx = fmaxf(mx, s[t][kt][r]);
+                    }
+            }
+            if (__any(mx > m_run[t] + 8.0f || (m_run[t] == -INFINITY && mx > -INFINITY))) {
+                mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+                mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+                const float m_new = fmaxf(m_run[t], mx);
+                const float alpha = m_new == -INFINITY ? 1.0f : __builtin_amdgcn_exp2f(m_run[t] - m_new);
+                l_run[t] *= alpha;
+#pragma unroll
+                for (int d = 0; d < VT; ++d) acc[t][d] *= alpha;
+                m_run[t] = m_new;
+            }
+            const float m_use = m_run[t] == -INFINITY ? 0.f : m_run[t];
+#pragma unroll
+            for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const float p = __builtin_amdgcn_exp2f(s[t][kt][r] - m_use);
+                    l_run[t] += p;
+                    pf[t][4 * kt + r] = (__bf16)p;
+                }
+        }
+        static_for<VT / VG>([&](auto GI) {
+            constexpr int d0 = decltype(GI)::value * VG;
+            if constexpr (!VEARLY) read_v(std::integral_constant<int, d0>{});
+            wait_lds();
+#pragma unroll
+            for (int i = 0; i < VG; ++i) asm volatile("" : "+v"(vf[i][0]), "+v"(vf[i][1]));
+#pragma unroll
+            for (int i = 0; i < VG; ++i) {
+                const u32x4_t vv = {vf[i][0][0], vf[i][0][1], vf[i][1][0], vf[i][1][1]};
+#pragma unroll
+                for (int t = 0; t < NT; ++t)
+                    acc[t][d0 + i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, vv), pf[t], acc[t][d0 + i], 0, 0, 0);
+            }
+        });
+    }
+    __device__ __forceinline__ float mass(int t) const {
+        float l = l_run[t];
+        l += __shfl_xor(l, 16, 64);
+        l += __shfl_xor(l, 32, 64);
+        return l;
+    }
+};
+
+// ---------------------------------------------------------------------------------------------------------------------------
+// DK, DV: multiples of 64
+template <int DK, int DV>
+__global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void group_attn_prefill_kernel(const GroupArgs a) {
+    using SL = Slab<DK, DV, 2>;
+    constexpr int KS = SL::KS, VT = SL::VT, KB = SL::KB, VB = SL::VB, KTILE = 64 * KB, VTILE = 64 * VB, STAGE = KTILE + VTILE;
+    constexpr int KCPR = DK / 8, VCPR = DV / 8, KDMA = DK / 32, VDMA = DV / 32;
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int c = lane & 15, g = lane >> 4;
+    // XCD-aware order: workgroups with equal id % 8 share an XCD and take one contiguous run of (head, tile) items
+    const int total = a.n_tiles * a.H, per = (total + 7) >> 3;
+    const int item = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
+    if ((int)(blockIdx.x >> 3) >= per || item >= total) return;
+    const int h = item / a.n_tiles, tile = item % a.n_tiles, kvh = h / (a.H / a.G);
+    const int seq = a.tile_a[tile], qo = a.tile_b[tile];
+    const int qs = a.q_start[seq], nq = a.q_start[seq + 1] - qs;
+    if (qo >= nq) return;
+    const int p0 = a.pos[qs] + qo, plast = p0 + min(127, nq - 1 - qo);  // positions of the tile's first and last row
+    const int jlo = ga_first(a, p0) & ~63;
+    const int n = ((plast - jlo) >> 6) + 1;
+    const int32_t* bt = a.bt + (int64_t)(a.seq0 + seq) * a.bt_stride;
+    SL S;
+    S.init(lane);
+    const float sl = a.slope ? a.slope[h] * GA_LOG2E : 0.f;
+    // this wave's rows: tile t holds rows qo + 64 t + 16 w + c (the two half-dead tiles of the causal edge cost all waves the same)
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+        const int r0 = qo + 64 * t + 16 * w, r = r0 + c;
+        const bool some = r0 < nq;
+        S.rp[t] = r < nq ? p0 - qo + r : -1;
+        S.rlo[t] = r < nq ? ga_first(a, S.rp[t]) : 0;
+        S.slope2[t] = sl;
+        const int a0 = p0 - qo + r0, a1 = p0 - qo + min(r0 + 15, nq - 1);
+        S.any_lo[t] = some ? ga_first(a, a0) : 1 << 30;
+        S.any_hi[t] = some ? a1 : -1;
+        S.full_lo[t] = some ? ga_first(a, a1) : 1 << 30;
+        S.full_hi[t] = some ? a0 : -1;
+        const bf16_t* qp = reinterpret_cast<const bf16_t*>(a.q) + (int64_t)(qs + min(r, nq - 1)) * a.ldq + (int64_t)h * a.dk;
+#pragma unroll
+        for (int i = 0; i < KS; ++i) {
+            const int k = 32 * i + 8 * g;
+            S.qf[t][i] = u32x4_t{0, 0, 0, 0};
+            if (k < a.dk) S.qf[t][i] = *reinterpret_cast<const u32x4_t*>(qp + k);
+        }
+    }
+#pragma unroll
+    for (int t = 0; t < 2; ++t)
+#pragma unroll
+        for (int i = 0; i < KS; ++i) asm volatile("" : "+v"(S.qf[t][i]));
+    const unsigned base = lds_addr(smem);
+    // per-lane source offsets of the DMA pieces: constant over the tiles
+    unsigned koff[KDMA], voff[VDMA];
+    int krow[KDMA], vrow[VDMA];
+    bool kpad[KDMA], vpad[VDMA];
+#pragma unroll
+    for (int i = 0; i < KDMA; ++i) {
+        const int q = (w * KDMA + i) * 64 + lane, row = q / KCPR, ch = (q % KCPR) ^ attn_swz(row);
+        krow[i] = row;
+        kpad[i] = ch * 8 >= a.dk;
+        koff[i] = (unsigned)(row * a.dk + ch * 8);
+    }
+#pragma unroll
+    for (int i = 0; i < VDMA; ++i) {
+        const int q = (w * VDMA + i) * 64 + lane, row = q / VCPR, ch = (q % VCPR) ^ attn_swz(row);
+        vrow[i] = row;
+        vpad[i] = ch * 8 >= a.dv;
+        voff[i] = (unsigned)(row * a.dv + ch * 8);
+    }
+    auto issue = [&](int it, int blk) {
+        const int j0 = jlo + it * 64, left = ga_ok(a, blk) ? plast - j0 + 1 : 0;
+        const int64_t row = ga_row(a, blk, j0, kvh);
+        const bf16_t* kb = reinterpret_cast<const bf16_t*>(a.kc) + row * a.dk;
+        const bf16_t* vb = reinterpret_cast<const bf16_t*>(a.vc) + row * a.dv;
+        char* st = smem + (it & 1) * STAGE;
+#pragma unroll
+        for (int i = 0; i < KDMA; ++i) {
+            const void* s = (kpad[i] || krow[i] >= left) ? (const void*)ga_zero_page : (const void*)(kb + koff[i]);
+            lds_dma16(s, st + (w * KDMA + i) * 1024);
+        }
+#pragma unroll
+        for (int i = 0; i < VDMA; ++i) {
+            const void* s = (vpad[i] || vrow[i] >= left) ? (const void*)ga_zero_page : (const void*)(vb + voff[i]);
+            lds_dma16(s, st + KTILE + (w * VDMA + i) * 1024);
+        }
+    };
+    const float sc = a.scale * GA_LOG2E;
+    auto block_of = [&](int it) { return bt[ga_block(a, jlo + min(it, n - 1) * 64)]; };  // 64-key tiles lie in one block
+    int blk = block_of(1);
+    issue(0, block_of(0));
+    for (int it = 0; it < n; ++it) {
+        wait_vm<0>();
+        __builtin_amdgcn_s_barrier();
+        if (it + 1 < n) {
+            issue(it + 1, blk);
+            blk = block_of(it + 2);
+        }
+        const unsigned kst = base + (it & 1) * STAGE, vst = kst + KTILE;
+#pragma unroll
+        for (int s = 0; s < 2; ++s) S.run(kst + s * 32 * KB, vst + s * 32 * VB, jlo + it * 64 + s * 32, g, sc);
+    }
+    const float sk = a.sink ? a.sink[h] * GA_LOG2E : -INFINITY;
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+        const float l = S.mass(t);
+        const int r = qo + 64 * t + 16 * w + c;
+        if (r >= nq) continue;
+        const float M = fmaxf(S.m_run[t], sk), f = __builtin_amdgcn_exp2f(S.m_run[t] - M);
+        const float inv = f / (l * f + __builtin_amdgcn_exp2f(sk - M));
+        bf16_t* o = reinterpret_cast<bf16_t*>(a.out) + (int64_t)(qs + r) * a.ldo + (int64_t)h * a.dv;
+#pragma unroll
+        for (int d = 0; d < VT; ++d) {
+            const int dim = 16 * d + 4 * g;
+            const f32x4_t& v = S.acc[t][d];
+            if (dim < a.dv) *reinterpret_cast<u32x2_t*>(o + dim) = u32x2_t{pack2bf(v[0] * inv, v[1] * inv), pack2bf(v[2] * inv, v[3] * inv)};
+        }
+    }
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------
+// Workgroup = (token tile, key / value head, group of 16 rows, KV split).  Row rho of a tile is token rho / R, head rho % R of the
+// R = H / G heads that share the key / value head.  Every one of the NW waves takes each NW-th 32-key slab of the split with its own two LDS
+// stages and softmax state: no barrier in the loop.
+template <int DK, int DV, int NW>
+__global__ __launch_bounds__(NW * 64, 1) void group_attn_decode_kernel(const GroupArgs a, int row_groups) {
+    using SL = Slab<DK, DV, 1>;
+    constexpr int KS = SL::KS, VT = SL::VT, KB = SL::KB, VB = SL::VB, KSLAB = 32 * KB, STAGE = KSLAB + 32 * VB;
+    constexpr int KCPR = DK / 8, VCPR = DV / 8, KDMA = DK / 16, VDMA = DV / 16;
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int c = lane & 15, g = lane >> 4;
+    int item = blockIdx.x;
+    const int split = item % a.nsplit;
+    item /= a.nsplit;
+    const int rg = item % row_groups;
+    item /= row_groups;
+    const int kvh = item % a.G, tile = item / a.G;
+    const int tok0 = a.tile_a[tile], ntok = a.tile_b[tile], R = a.H / a.G;
+    const int pA = a.pos[tok0], pB = pA + ntok - 1;
+    const int rho = rg * 16 + c, tok = rho / R, hh = rho - tok * R, h = kvh * R + hh;
+    const bool row_ok = tok < ntok;
+    if (rg * 16 >= ntok * R) return;
+    const int jlo = pA >= 0 ? ga_first(a, pA) & ~31 : 0;
+    const int slabs = pA >= 0 ? ((pB - jlo) >> 5) + 1 : 0, per = (slabs + a.nsplit - 1) / a.nsplit;
+    const int s_lo = split * per, s_hi = min(s_lo + per, slabs);
+    const int n = s_hi > s_lo + w ? (s_hi - s_lo - w + NW - 1) / NW : 0;  // slabs of this wave: s_lo + w + NW k
+    SL S;
+    S.init(lane);
+    S.rp[0] = row_ok && pA >= 0 ? pA + tok : -1;
+    S.rlo[0] = S.rp[0] >= 0 ? ga_first(a, S.rp[0]) : 0;
+    S.slope2[0] = a.slope && row_ok ? a.slope[h] * GA_LOG2E : 0.f;
+    {
+        const int t0 = rg * 16 / R, t1 = min((rg * 16 + 15) / R, ntok - 1);
+        S.any_lo[0] = ga_first(a, max(pA, 0) + t0);
+        S.any_hi[0] = pA + t1;
+        S.full_lo[0] = ga_first(a, max(pA, 0) + t1);
+        S.full_hi[0] = rg * 16 + 16 <= ntok * R ? pA + t0 : -1;  // rows without a token: masked
+    }
+    const bf16_t* qp = reinterpret_cast<const bf16_t*>(a.q) + (int64_t)(tok0 + (row_ok ? tok : 0)) * a.ldq + (int64_t)(row_ok ? h : kvh * R) * a.dk;
+#pragma unroll
+    for (int i = 0; i < KS; ++i) {
+        const int k = 32 * i + 8 * g;
+        S.qf[0][i] = u32x4_t{0, 0, 0, 0};
+        if (k < a.dk && row_ok) S.qf[0][i] = *reinterpret_cast<const u32x4_t*>(qp + k);
+    }
+#pragma unroll
+    for (int i = 0; i < KS; ++i) asm volatile("" : "+v"(S.qf[0][i]));
+    const int32_t* bt = a.bt + (int64_t)(a.seq0 + a.seq_of[tok0]) * a.bt_stride;
+    char* mine = smem + w * 2 * STAGE;
+    const unsigned base = lds_addr(mine);
+    unsigned koff[KDMA], voff[VDMA];
+    int krow[KDMA], vrow[VDMA];
+    bool kpad[KDMA], vpad[VDMA];
+#pragma unroll
+    for (int i = 0; i < KDMA; ++i) {
+        const int q = i * 64 + lane, row = q / KCPR, ch = (q % KCPR) ^ attn_swz(row);
+        krow[i] = row;
+        kpad[i] = ch * 8 >= a.dk;
+        koff[i] = (unsigned)(row * a.dk + ch * 8);
+    }
+#pragma unroll
+    for (int i = 0; i < VDMA; ++i) {
+        const int q = i * 64 + lane, row = q / VCPR, ch = (q % VCPR) ^ attn_swz(row);
+        vrow[i] = row;
+        vpad[i] = ch * 8 >= a.dv;
+        voff[i] = (unsigned)(row * a.dv + ch * 8);
+    }
+    auto key0 = [&](int k) { return jlo + (s_lo + w + NW * k) * 32; };
+    // block ids of this wave's next 64 slabs, one per lane
+    auto blocks_from = [&](int k) { return k + lane < n ? bt[ga_block(a, key0(k + lane))] : -1; };
+    int ids = n > 0 ? blocks_from(0) : -1;
+    auto issue = [&](int k) {
+        const int j0 = key0(k), blk = __builtin_amdgcn_readlane(ids, k & 63);
+        const int left = ga_ok(a, blk) ? pB - j0 + 1 : 0;
+        const int64_t row = ga_row(a, blk, j0, kvh);
+        const bf16_t* kb = reinterpret_cast<const bf16_t*>(a.kc) + row * a.dk;
+        const bf16_t* vb = reinterpret_cast<const bf16_t*>(a.vc) + row * a.dv;
+        char* st = mine + (k & 1) * STAGE;
+#pragma unroll
+        for (int i = 0; i < KDMA; ++i) {
+            const void* s = (kpad[i] || krow[i] >= left) ? (const void*)ga_zero_page : (const void*)(kb + koff[i]);
+            lds_dma16<2>(s, st + i * 1024);
+        }
+#pragma unroll
+        for (int i = 0; i < VDMA; ++i) {
+            const void* s = (vpad[i] || vrow[i] >= left) ? (const void*)ga_zero_page : (const void*)(vb + voff[i]);
+            lds_dma16<2>(s, st + KSLAB + i * 1024);
+        }
+    };
+    const float sc = a.scale * GA_LOG2E;
+    if (n > 0) issue(0);
+    for (int k = 0; k < n; ++k) {
+        if (k + 1 < n) {
+            if (((k + 1) & 63) == 0) ids = blocks_from(k + 1);
+            issue(k + 1);
+            wait_vm<KDMA + VDMA>();  // slab k is in, slab k + 1 may be on its way
+        } else {
+            wait_vm<0>();
+        }
+        const unsigned kst = base + (k & 1) * STAGE;
+        S.run(kst, kst + KSLAB, key0(k), g, sc);
+    }
+    // ---- the waves' sums through LDS (over the stages: every wave is past its last read) ----
+    const float l = S.mass(0);
+    __syncthreads();
+    float* ml = reinterpret_cast<float*>(smem);                 // [NW][16][2]
+    float* po = reinterpret_cast<float*>(smem + NW * 16 * 2 * 4);  // [NW][16][DV + 4]
+    constexpr int PO = DV + 4;
+    if (g == 0) {
+        ml[(w * 16 + c) * 2] = S.m_run[0];
+        ml[(w * 16 + c) * 2 + 1] = l;
+    }
+#pragma unroll
+    for (int d = 0; d < VT; ++d) *reinterpret_cast<f32x4_t*>(po + (w * 16 + c) * PO + 16 * d + 4 * g) = S.acc[0][d];
+    __syncthreads();
+    constexpr int QPR = DV / 4;
+    for (int i = tid; i < 16 * QPR; i += NW * 64) {
+        const int rr = i / QPR, col = (i - rr * QPR) * 4;
+        const int rh = rg * 16 + rr, tk = rh / R, head = kvh * R + (rh - tk * R);
+        if (tk >= ntok || col >= a.dv) continue;
+        float M = -INFINITY;
+#pragma unroll
+        for (int x = 0; x < NW; ++x) M = fmaxf(M, ml[(x * 16 + rr) * 2]);
+        const float sk = (a.nsplit == 1 && a.sink) ? a.sink[head] * GA_LOG2E : -INFINITY;
+        const float Ms = fmaxf(M, sk);
+        float L = 0.f;
+        f32x4_t o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int x = 0; x < NW; ++x) {
+            const float mx = ml[(x * 16 + rr) * 2];
+            const float f = mx == -INFINITY ? 0.f : __builtin_amdgcn_exp2f(mx - Ms);
+            L += f * ml[(x * 16 + rr) * 2 + 1];
+            const f32x4_t v = *reinterpret_cast<const f32x4_t*>(po + (x * 16 + rr) * PO + col);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) o[e] += f * v[e];
+        }
+        const int64_t row = (int64_t)(tok0 + tk);
+        if (a.nsplit == 1) {
+            if (sk > -INFINITY) L += __builtin_amdgcn_exp2f(sk - Ms);
+            const float inv = L > 0.f ? 1.0f / L : 0.f;
+            *reinterpret_cast<u32x2_t*>(reinterpret_cast<bf16_t*>(a.out) + row * a.ldo + (int64_t)head * a.dv + col) =
+                u32x2_t{pack2bf(o[0] * inv, o[1] * inv), pack2bf(o[2] * inv, o[3] * inv)};
+        } else {
+            const int64_t pr = (row * a.H + head) * a.nsplit + split;
+            *reinterpret_cast<f32x4_t*>(a.part_o + pr * a.dv + col) = o;
+            if (col == 0) {
+                a.part_ml[pr * 2] = M;
+                a.part_ml[pr * 2 + 1] = L;
+            }
+        }
+    }
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------
+// any head size, fp32 arithmetic throughout: one (row, head) per workgroup, 256 keys at a time, one key per thread
+template <typename T>
+__device__ __forceinline__ float ga_f(T v);
+template <>
+__device__ __forceinline__ float ga_f<float>(float v) { return v; }
+template <>
+__device__ __forceinline__ float ga_f<bf16_t>(bf16_t v) { return bf2f(v); }
+
+template <typename T>
+__global__ __launch_bounds__(256) void group_attn_plain_kernel(const GroupArgs a) {
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    float* sq = reinterpret_cast<float*>(smem);  // [dk] query
+    float* so = sq + a.dk;                        // [dv] output
+    float* sp = so + a.dv;                        // [256] weights, then partial sums
+    __shared__ float s_red[4];
+    __shared__ int64_t s_row[256];
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+    const int h = blockIdx.x % a.H, kvh = h / (a.H / a.G);
+    const int64_t r = blockIdx.x / a.H;
+    const int p = a.pos[r];
+    T* out = reinterpret_cast<T*>(a.out) + r * a.ldo + (int64_t)h * a.dv;
+    auto put = [&](int d, float v) {
+        if constexpr (sizeof(T) == 4) out[d] = v;
+        else out[d] = f2bf(v);
+    };
+    if (p < 0) {
+        for (int d = tid; d < a.dv; d += 256) put(d, 0.f);
+        return;
+    }
+    const T* q = reinterpret_cast<const T*>(a.q) + r * a.ldq + (int64_t)h * a.dk;
+    for (int d = tid; d < a.dk; d += 256) sq[d] = ga_f<T>(q[d]);
+    for (int d = tid; d < a.dv; d += 256) so[d] = 0.f;
+    const int32_t* bt = a.bt + (int64_t)(a.seq0 + a.seq_of[r]) * a.bt_stride;
+    const int lo = ga_first(a, p);
+    const float slope = a.slope ? a.slope[h] : 0.f;
+    float m = a.sink ? a.sink[h] : -INFINITY, l = a.sink ? 1.0f : 0.f;  // the sink's mass from the start
+    const int ncol = min(a.dv, 256), parts = 256 / ncol;
+    for (int j0 = lo; j0 <= p; j0 += 256) {
+        const int j = j0 + tid;
+        float s = -INFINITY;
+        __syncthreads();
+        if (j <= p) {
+            const int blk = bt[ga_block(a, j)];
+            const int64_t row = ga_ok(a, blk) ? ga_row(a, blk, j, kvh) : 0;
+            s_row[tid] = row;
+            const T* k = reinterpret_cast<const T*>(a.kc) + row * a.dk;
+            float acc = 0.f;
+            for (int d = 0; d < a.dk; d += 4) {  // dk is a multiple of 8
+#pragma unroll
+                for (int e = 0; e < 4; ++e) acc = fmaf(sq[d + e], ga_f<T>(k[d + e]), acc);
+            }
+            s = acc * a.scale - slope * (float)(p - j);
+        }
+        const float bm = wave_max(s);
+        if (lane == 0) s_red[wid] = bm;
+        __syncthreads();
+        const float m_new = fmaxf(m, fmaxf(fmaxf(s_red[0], s_red[1]), fmaxf(s_red[2], s_red[3])));
+        const float e = j <= p ? expf(s - m_new) : 0.f;
+        sp[tid] = e;
+        const float bs = wave_sum(e);
+        __syncthreads();
+        if (lane == 0) s_red[wid] = bs;
+        __syncthreads();
+        const float alpha = m == -INFINITY ? 0.f : expf(m - m_new);
+        l = l * alpha + (s_red[0] + s_red[1] + s_red[2] + s_red[3]);
+        m = m_new;
+        const int nk = min(256, p - j0 + 1);
+        for (int c0 = 0; c0 < a.dv; c0 += ncol) {
+            const int col = c0 + tid % ncol, part = tid / ncol;
+            float acc = 0.f;
+            if (part < parts && col < a.dv)
+                for (int i = part; i < nk; i += parts) acc = fmaf(sp[i], ga_f<T>(reinterpret_cast<const T*>(a.vc)[s_row[i] * a.dv + col]), acc);
+            float* sums = sp + 256;
+            sums[tid] = acc;
+            __syncthreads();
+            if (part == 0 && col < a.dv) {
+                for (int i = 1; i < parts; ++i) acc += sums[i * ncol + tid];
+                so[col] = so[col] * alpha + acc;
+            }
+            __syncthreads();
+        }
+    }
+    __syncthreads();
+    for (int d = tid; d < a.dv; d += 256) put(d, so[d] / l);
+}
+
+template <int DK, int DV>
+int launch_prefill(const GroupArgs& a, hipStream_t st) {
+    constexpr int LDS = 2 * 64 * (DK + DV) * 2;
+    static_assert(LDS <= 160 * 1024, "LDS of a CU");
+    auto kern = group_attn_prefill_kernel<DK, DV>;
+    GLM_SET_MAX_LDS(kern, LDS, "glm_group_attn_prefill");
+    const int64_t per = ((int64_t)a.n_tiles * a.H + 7) / 8;
+    GLM_CHECK_ARG(per * 8 < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_group_attn_prefill: grid too large");
+    hipLaunchKernelGGL(kern, dim3((unsigned)(per * 8)), dim3(256), LDS, st, a);
+    GLM_CHECK_LAUNCH("glm_group_attn_prefill");
+    return GLM_OK;
+}
+
+template <int DK, int DV>
+int launch_decode(const GroupArgs& a, int row_groups, hipStream_t st) {
+    constexpr int NW = DK + DV <= 320 ? 4 : 2;  // as many waves as have room for two stages each
+    constexpr int STG = NW * 2 * 32 * (DK + DV) * 2, RED = NW * 16 * (2 + DV + 4) * 4, LDS = STG > RED ? STG : RED;
+    static_assert(LDS <= 160 * 1024, "LDS of a CU");
+    auto kern = group_attn_decode_kernel<DK, DV, NW>;
+    const int64_t grid = (int64_t)a.n_tiles * a.G * row_groups * a.nsplit;
+    GLM_CHECK_ARG(grid < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_group_attn_decode: grid too large");
+    GLM_SET_MAX_LDS(kern, LDS, "glm_group_attn_decode");
+    hipLaunchKernelGGL(kern, dim3((unsigned)grid), dim3(NW * 64), LDS, st, a, row_groups);
+    GLM_CHECK_LAUNCH("glm_group_attn_decode");
+    return GLM_OK;
+}
+
+#define GA_SIZES(F, ...)                                            \
+    do {                                                            \
+        const int kk = (a.dk + 63) / 64, vv = (a.dv + 63) / 64;     \
+        if (kk == 1 && vv == 1) return F<64, 64>(__VA_ARGS__);      \
+        if (kk == 1 && vv == 2) return F<64, 128>(__VA_ARGS__);     \
+        if (kk == 1) return F<64, 256>(__VA_ARGS__);                \
+        if (kk == 2 && vv == 1) return F<128, 64>(__VA_ARGS__);     \
+        if (kk == 2 && vv == 2) return F<128, 128>(__VA_ARGS__);    \
+        if (kk == 2) return F<128, 256>(__VA_ARGS__);               \
+        if (vv == 1) return F<256, 64>(__VA_ARGS__);                \
+        if (vv == 2) return F<256, 128>(__VA_ARGS__);               \
+        return F<256, 256>(__VA_ARGS__);                            \
+    } while (0)
+
+int run_prefill(const GroupArgs& a, hipStream_t st) { GA_SIZES(launch_prefill, a, st); }
+int run_decode(const GroupArgs& a, int row_groups, hipStream_t st) { GA_SIZES(launch_decode, a, row_groups, st); }
+
+int log2_of(int n) {
+    for (int i = 0; i < 30; ++i)
+        if (n == 1 << i) return i;
+    return -1;
+}
+
+// what the three attention entry points share
+int group_args(GroupArgs& a, const char* name, const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs, const int32_t* bt,
+               int64_t bt_stride, int seq0, int H, int G, int dk, int dv, int window, int chunk, float scale, const float* slope, const float* sink, void* out, int64_t ldo) {
+    GLM_CHECK_ARG(q && kc && vc && bt && out, GLM_ERR_INVALID, "%s: null pointer", name);
+    GLM_CHECK_ARG(H > 0 && G > 0 && H % G == 0 && dk > 0 && dv > 0 && dk % 8 == 0 && dv % 8 == 0 && ldq >= (int64_t)H * dk && ldo >= (int64_t)H * dv && ldq % 8 == 0 && ldo % 4 == 0 &&
+                      n_blocks > 0 && bs > 0 && bs % 64 == 0 && bt_stride > 0 && seq0 >= 0 && window >= 0 && chunk >= 0 && glm_aligned16(q) && glm_aligned16(kc) && glm_aligned16(vc) &&
+                      (((uintptr_t)out) & 7) == 0, GLM_ERR_INVALID, "%s: bad shape H=%d G=%d dk=%d dv=%d ldq=%ld ldo=%ld block=%d", name, H, G, dk, dv, (long)ldq, (long)ldo, bs);
+    a = GroupArgs{};
+    a.q = q; a.ldq = ldq; a.kc = kc; a.vc = vc; a.n_blocks = n_blocks; a.bs = bs; a.log2_bs = log2_of(bs); a.bt = bt; a.bt_stride = bt_stride; a.seq0 = seq0;
+    a.H = H; a.G = G; a.dk = dk; a.dv = dv; a.window = window; a.chunk = chunk; a.scale = scale; a.slope = slope; a.sink = sink; a.out = out; a.ldo = ldo; a.nsplit = 1;
+    return GLM_OK;
+}
+
+}  // namespace
+
+extern "C" int glm_group_kv_store(const void* src, int64_t ld, int64_t k_off, int64_t v_off, int f32, const int32_t* slots, int64_t T, void* kc, void* vc, int64_t n_slots, int bs,
+                                  int G, int dk, int dv, glm_stream_t stream) {
+    const int es = f32 ? 4 : 2;
+    GLM_CHECK_ARG(src && slots && kc && vc && T >= 0 && bs > 0 && n_slots > 0 && n_slots % bs == 0 && G > 0 && dk > 0 && dv > 0 && dk % 8 == 0 && dv % 8 == 0 && ld % 8 == 0 && k_off % 8 == 0 && v_off % 8 == 0 &&
+                      k_off >= 0 && v_off >= 0 && ld >= k_off + (int64_t)G * dk && ld >= v_off + (int64_t)G * dv && glm_aligned16(src) && glm_aligned16(kc) && glm_aligned16(vc), GLM_ERR_INVALID,
+                  "glm_group_kv_store: bad shape T=%ld G=%d dk=%d dv=%d ld=%ld", (long)T, G, dk, dv, (long)ld);
+    if (T == 0) return GLM_OK;
+    StoreArgs a = {(const char*)src, ld * es, k_off * es, v_off * es, slots, (char*)kc, (char*)vc, T, n_slots, G, bs, dk * es / 16, dv * es / 16};
+    const int64_t items = T * G * (a.ku + a.vu);
+    GLM_CHECK_ARG((items + 255) / 256 < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_group_kv_store: too many rows");
+    hipLaunchKernelGGL(group_kv_store_kernel, dim3((unsigned)((items + 255) / 256)), dim3(256), 0, glm_s(stream), a);
+    GLM_CHECK_LAUNCH("glm_group_kv_store");
+    return GLM_OK;
+}
+
+extern "C" int glm_group_attn_prefill(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs, const int32_t* block_tables, int64_t bt_stride, int seq0,
+                                      const int32_t* q_start, const int32_t* pos, const int32_t* tile_seq, const int32_t* tile_off, int n_tiles, int H, int G, int dk, int dv, int window,
+                                      int chunk, float scale, const float* slope, const float* sink, void* out, int64_t ldo, glm_stream_t stream) {
+    GroupArgs a;
+    const int rc = group_args(a, "glm_group_attn_prefill", q, ldq, kc, vc, n_blocks, bs, block_tables, bt_stride, seq0, H, G, dk, dv, window, chunk, scale, slope, sink, out, ldo);
+    if (rc != GLM_OK) return rc;
+    GLM_CHECK_ARG(q_start && pos && tile_seq && tile_off && n_tiles >= 0, GLM_ERR_INVALID, "glm_group_attn_prefill: no tiles");
+    GLM_CHECK_ARG(dk <= 256 && dv <= 256, GLM_ERR_UNSUPPORTED, "glm_group_attn_prefill: head sizes up to 256 (dk=%d dv=%d)", dk, dv);
+    if (n_tiles == 0) return GLM_OK;
+    a.q_start = q_start; a.pos = pos; a.tile_a = tile_seq; a.tile_b = tile_off; a.n_tiles = n_tiles;
+    return run_prefill(a, glm_s(stream));
+}
+
+extern "C" int glm_group_attn_decode(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs, const int32_t* block_tables, int64_t bt_stride,
+                                     const int32_t* pos, const int32_t* seq_of, const int32_t* tile_tok, const int32_t* tile_n, int n_tiles, int tokens_per_tile, int H, int G, int dk, int dv,
+                                     int window, int chunk, float scale, const float* slope, const float* sink, void* out, int64_t ldo, int nsplit, float* part_o, float* part_ml,
+                                     glm_stream_t stream) {
+    GroupArgs a;
+    const int rc = group_args(a, "glm_group_attn_decode", q, ldq, kc, vc, n_blocks, bs, block_tables, bt_stride, 0, H, G, dk, dv, window, chunk, scale, slope, sink, out, ldo);
+    if (rc != GLM_OK) return rc;
+    GLM_CHECK_ARG(pos && seq_of && tile_tok && tile_n && n_tiles >= 0 && tokens_per_tile >= 1 && nsplit >= 1 && nsplit <= 64 && (nsplit == 1 || (part_o && part_ml)), GLM_ERR_INVALID,
+                  "glm_group_attn_decode: bad tiles or splits (%d)", nsplit);
+    GLM_CHECK_ARG(dk <= 256 && dv <= 256, GLM_ERR_UNSUPPORTED, "glm_group_attn_decode: head sizes up to 256 (dk=%d dv=%d)", dk, dv);
+    if (n_tiles == 0) return GLM_OK;
+    a.pos = pos; a.seq_of = seq_of; a.tile_a = tile_tok; a.tile_b = tile_n; a.n_tiles = n_tiles; a.nsplit = nsplit; a.part_o = part_o; a.part_ml = part_ml;
+    return run_decode(a, (tokens_per_tile * (H / G) + 15) / 16, glm_s(stream));
+}
+
+extern "C" int glm_group_attn_plain(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs, const int32_t* block_tables, int64_t bt_stride, const int32_t* pos,
+                                    const int32_t* seq_of, int64_t rows, int H, int G, int dk, int dv, int window, int chunk, float scale, const float* slope, const float* sink, void* out,
+                                    int64_t ldo, int f32, glm_stream_t stream) {
+    GroupArgs a;
+    const int rc = group_args(a, "glm_group_attn_plain", q, ldq, kc, vc, n_blocks, bs, block_tables, bt_stride, 0, H, G, dk, dv, window, chunk, scale, slope, sink, out, ldo);
+    if (rc != GLM_OK) return rc;
+    GLM_CHECK_ARG(pos && seq_of && rows >= 0 && rows * H < (1ll << 31), GLM_ERR_INVALID, "glm_group_attn_plain: bad rows (%ld)", (long)rows);
+    const size_t lds = (size_t)(dk + dv + 512) * 4;
+    GLM_CHECK_ARG(lds <= 60 * 1024, GLM_ERR_UNSUPPORTED, "glm_group_attn_plain: head sizes %d + %d", dk, dv);
+    if (rows == 0) return GLM_OK;
+    a.pos = pos; a.seq_of = seq_of; a.rows = rows;
+    if (f32) hipLaunchKernelGGL(group_attn_plain_kernel<float>, dim3((unsigned)(rows * H)), dim3(256), lds, glm_s(stream), a);
+    else hipLaunchKernelGGL(group_attn_plain_kernel<bf16_t>, dim3((unsigned)(rows * H)), dim3(256), lds, glm_s(stream), a);
+    GLM_CHECK_LAUNCH("glm_group_attn_plain");
+    return GLM_OK;
+}

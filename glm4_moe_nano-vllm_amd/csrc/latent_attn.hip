@@ -570,47 +570,6 @@ __global__ __launch_bounds__(256) void latent_attn_f32_kernel(const AttnArgs a, 
         if (lane + 64 * i < a.rp) ctx[grow * a.rp + lane + 64 * i] = p < 0 ? 0.f : acc[i] * inv;
 }
 
-// ---------------------------------------------------------------------------------------------------------------------------
-// ctx = (sum over the KV splits, each brought to the common maximum) / (mass of the splits + the sink's): one wave per (token,
-// head) and 256 latent columns, sixteen splits in flight
-__global__ __launch_bounds__(256) void latent_merge_kernel(const float* __restrict__ part_o, const float* __restrict__ part_ml, const float* __restrict__ sink,
-                                                           int nsplit, bf16_t* __restrict__ ctx, int64_t rows, int H, int rp, int nchunk) {
-    const int lane = threadIdx.x & 63;
-    const int64_t item = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-    const int64_t grow = item / nchunk;
-    if (grow >= rows) return;
-    const int k = (int)(item % nchunk) * 256 + lane * 4;
-    const bool on = k < rp;
-    const float* p = part_o + grow * nsplit * rp + (on ? k : 0);
-    float m = -INFINITY, l = 0.f;
-    if (lane < nsplit) {
-        m = part_ml[(grow * nsplit + lane) * 2];
-        l = part_ml[(grow * nsplit + lane) * 2 + 1];
-    }
-    f32x4_t o = {0.f, 0.f, 0.f, 0.f};
-    float f = 0.f;
-    for (int s0 = 0; s0 < nsplit; s0 += 16) {
-        f32x4_t x[16];
-#pragma unroll
-        for (int j = 0; j < 16; ++j) x[j] = *reinterpret_cast<const f32x4_t*>(p + (int64_t)min(s0 + j, nsplit - 1) * rp);
-        if (s0 == 0) {
-            const float sk = sink[grow % H] * LOG2E;
-            const float M = fmaxf(wave_max(m), sk);
-            const float e = l > 0.f ? __builtin_amdgcn_exp2f(m - M) : 0.f;
-            f = e / (wave_sum(l * e) + __builtin_amdgcn_exp2f(sk - M));  // 0: an empty split, its sums were never written
-        }
-#pragma unroll
-        for (int j = 0; j < 16; ++j) {
-            const float fs = s0 + j < nsplit ? __shfl(f, s0 + j, 64) : 0.f;
-            if (fs != 0.f) {
-#pragma unroll
-                for (int i = 0; i < 4; ++i) o[i] += fs * x[j][i];
-            }
-        }
-    }
-    if (on) *reinterpret_cast<u32x2_t*>(ctx + grow * rp + k) = u32x2_t{pack2bf(o[0], o[1]), pack2bf(o[2], o[3])};
-}
-
 struct UpArgs {
     const bf16_t* ctx;   // [Ta, H, rp]
     const bf16_t* wuv;   // [H, vdimp, rp]
@@ -742,19 +701,6 @@ extern "C" int glm_latent_attn(const void* qa, const void* cache, int64_t n_bloc
         case 9: return launch_latent_attn_mt<9>(a, mt, st);
         default: return launch_latent_attn_mt<16>(a, mt, st);
     }
-}
-
-extern "C" int glm_latent_merge(const float* part_o, const float* part_ml, const float* sink, int nsplit, void* ctx, int64_t Ta, int H, int rp,
-                                glm_stream_t stream) {
-    GLM_CHECK_ARG(part_o && part_ml && sink && ctx && nsplit >= 1 && nsplit <= 64 && Ta >= 0 && H > 0 && rp > 0 && rp % 8 == 0, GLM_ERR_INVALID,
-                  "glm_latent_merge: bad shape Ta=%ld H=%d rp=%d splits=%d", (long)Ta, H, rp, nsplit);
-    GLM_CHECK_ARG(Ta * H < (1ll << 26), GLM_ERR_UNSUPPORTED, "glm_latent_merge: too many rows");
-    if (Ta == 0) return GLM_OK;
-    const int nchunk = (rp + 255) / 256;
-    hipLaunchKernelGGL(latent_merge_kernel, dim3((unsigned)((Ta * H * nchunk + 3) / 4)), dim3(256), 0, glm_s(stream), part_o, part_ml, sink, nsplit, (bf16_t*)ctx,
-                       Ta * H, H, rp, nchunk);
-    GLM_CHECK_LAUNCH("glm_latent_merge");
-    return GLM_OK;
 }
 
 extern "C" int glm_latent_up(const void* ctx, const void* wuv, void* out, int64_t ldo, int64_t Ta, int H, int vdimp, int rp, glm_stream_t stream) {

@@ -1,0 +1,768 @@
+// matrix_memory.hip — the gated matrix memory of a recurrent mixer (mLSTM of xLSTM).  Per head, with S [dim, vdim], n [dim] and a running
+// maximum m that all start at zero, log gates i and f,
+//
+//     i_t = cap tanh(a_t / cap)             f_t = log sigmoid(cap tanh(b_t / cap))         a, b: projections with their biases
+//     m_t = max(f_t + m_(t-1), i_t)
+//     S_t = e^(f_t + m_(t-1) - m_t) S_(t-1) + e^(i_t - m_t) k_t v_t^T                      n_t likewise with k_t alone
+//     o_t = S_t^T q_t dim^-1/2 / (max(|n_t . q_t| dim^-1/2, e^(-m_t)) + 1e-6)
+//     y_t = o_t / rms(o_t) . norm . sigmoid(g_t)
+//
+// State, gates and everything between the projections and y in fp32.  gfx950 only.
+//
+//   memory_recurrent   token by token, state in registers (decoded tokens, short portions, fp32): one (sequence, head) per workgroup, gate
+//                      projections and the output norm included; memory_recurrent_any for head sizes beyond its registers
+//   memory_chunkwise   long portions: 64 tokens at a time on the matrix cores, one (sequence, head, 64 value columns) per workgroup
+//   memory_output      norm and output gate of memory_chunkwise's rows
+//
+// Rooflines: the recurrent form is HBM-bound (the state is read once and written once per step), the chunkwise form is bound by the chain
+// of its chunks (the state of one is the input of the next).
+//
+// The chunkwise form, with b_t the running sum of f inside the chunk: m_t = b_t + max(m_in, max_(s<=t) (i_s - b_s)) is a scan over 64
+// lanes; with D_ts = e^(b_t - m_t + i_s - b_s) for s <= t and c_t = e^(b_t + m_in - m_t),
+//
+//     S_t^T q_t = c_t S_in^T q_t + sum_s D_ts (k_s . q_t) v_s            S_out = c_L S_in + sum_s e^(b_L - m_L + i_s - b_s) k_s v_s^T
+//
+// q, k and v are bf16 as the projection left them; the weights D (k . q), the decayed values and the state enter the matrix cores as a
+// bf16 pair hi + lo each, so the products keep about 16 bits of their fp32 operand.
+#include "common.h"
+#include "attn_lds.h"
+
+namespace {
+
+constexpr float MM_LOG2E = 1.4426950408889634f;
+__device__ const u32x4_t mm_zero_page[4] = {};
+
+__device__ __forceinline__ float mm_log_sigmoid(float z) { return fminf(z, 0.f) - log1pf(expf(-fabsf(z))); }
+__device__ __forceinline__ float mm_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
+__device__ __forceinline__ float mm_cap(float z, float cap) { return cap * tanhf(z / cap); }
+
+struct RecArgs {
+    const void* x;        // projection rows: q at h*dimp, k at k_off + h*dimp, v at v_off + h*vdimp, g at g_off + h*vdimp
+    int64_t ldx, k_off, v_off, g_off;
+    const void* hrow;     // [T, ldh] what the gates are projected from
+    int64_t ldh;
+    const void* wif;      // [2 H, ldw] rows i then f
+    int64_t ldw;
+    int wk;               // columns of hrow / wif
+    const float* bif;     // [2 H]
+    const float* norm;    // [H * vdimp]
+    void* y;              // [T, ldy] head h at h*vdimp
+    int64_t ldy;
+    float *S, *n, *m;     // [rows][H][dimp][vdimp], [rows][H][dimp], [rows][H]
+    int64_t n_state;
+    const int32_t *pos, *q_start, *state_in, *state_out;
+    int seqs, H, dim, dimp, vdim, vdimp;
+    float cap, eps;
+};
+
+template <typename T>
+__device__ __forceinline__ float mm_ld(const void* p, int64_t i) {
+    if constexpr (sizeof(T) == 4) return reinterpret_cast<const float*>(p)[i];
+    else return bf2f(reinterpret_cast<const bf16_t*>(p)[i]);
+}
+template <typename T>
+__device__ __forceinline__ void mm_st(void* p, int64_t i, float v) {
+    if constexpr (sizeof(T) == 4) reinterpret_cast<float*>(p)[i] = v;
+    else reinterpret_cast<bf16_t*>(p)[i] = f2bf(v);
+}
+template <typename T>
+__device__ __forceinline__ f32x4_t mm_ld4(const void* p, int64_t i) {
+    if constexpr (sizeof(T) == 4) return *reinterpret_cast<const f32x4_t*>(reinterpret_cast<const float*>(p) + i);
+    else {
+        const u32x2_t u = *reinterpret_cast<const u32x2_t*>(reinterpret_cast<const bf16_t*>(p) + i);
+        return f32x4_t{bflo(u[0]), bfhi(u[0]), bflo(u[1]), bfhi(u[1])};
+    }
+}
+// this thread's share of the two gate projections of row r, head h
+template <typename T>
+__device__ __forceinline__ void mm_gate_parts(const RecArgs& a, int64_t r, int h, int tid, int nt, float& gi, float& gf) {
+    gi = gf = 0.f;
+    for (int c = tid * 4; c < a.wk; c += nt * 4) {
+        const f32x4_t x = mm_ld4<T>(a.hrow, r * a.ldh + c), wi = mm_ld4<T>(a.wif, (int64_t)h * a.ldw + c), wf = mm_ld4<T>(a.wif, (int64_t)(a.H + h) * a.ldw + c);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            gi = fmaf(x[e], wi[e], gi);
+            gf = fmaf(x[e], wf[e], gf);
+        }
+    }
+}
+
+// dimp <= 16 KD, vdimp <= 64 NW.  256 NW threads: column block tid / 256 (64 columns), thread (rg, cq) of a block holds rows rg + 16 k of the
+// four columns cq.
+template <typename T, int KD, int NW>
+__global__ __launch_bounds__(256 * NW) void memory_recurrent_kernel(const RecArgs a) {
+    constexpr int NT = 256 * NW, NWV = 4 * NW;
+    __shared__ float s_q[16 * KD], s_k[16 * KD], s_g[2][NWV], s_nq[NWV], s_ss[NWV];
+    __shared__ __attribute__((aligned(16))) float s_o[NW][4][64];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const int cb = tid >> 8, cq = tid & 15, rg = (tid >> 4) & 15, wv = (tid >> 6) & 3;
+    const int seq = blockIdx.x / a.H, h = blockIdx.x % a.H;
+    const int r0 = a.q_start[seq], r1 = a.q_start[seq + 1];
+    const int col = cb * 64 + cq * 4;
+    const bool con = col < a.vdimp;
+    if (r1 <= r0) return;
+    if (a.pos[r0] < 0) {  // unused rows of a padded batch
+        for (int r = r0; r < r1; ++r)
+            for (int c = tid; c < a.vdimp; c += NT) mm_st<T>(a.y, (int64_t)r * a.ldy + (int64_t)h * a.vdimp + c, 0.f);
+        return;
+    }
+    f32x4_t S[KD];
+    float n = 0.f, m = 0.f;
+    const bool fresh = a.pos[r0] == 0;
+    const int64_t sin = min(max((int64_t)a.state_in[seq], (int64_t)0), a.n_state - 1) * a.H + h;
+#pragma unroll
+    for (int k = 0; k < KD; ++k) {
+        const int d = rg + 16 * k;
+        S[k] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        if (!fresh && con && d < a.dimp) S[k] = *reinterpret_cast<const f32x4_t*>(a.S + (sin * a.dimp + d) * a.vdimp + col);
+    }
+    if (!fresh) {
+        if (tid < a.dimp) n = a.n[sin * a.dimp + tid];
+        m = a.m[sin];
+    }
+    const float scale = 1.0f / sqrtf((float)a.dim), bi = a.bif[h], bf = a.bif[a.H + h], inv_v = 1.0f / (float)a.vdim;
+    for (int r = r0; r < r1; ++r) {
+        float gi, gf;
+        mm_gate_parts<T>(a, r, h, tid, NT, gi, gf);
+        gi = wave_sum(gi);
+        gf = wave_sum(gf);
+        if (lane == 0) {
+            s_g[0][wave] = gi;
+            s_g[1][wave] = gf;
+        }
+        const int64_t base = (int64_t)r * a.ldx;
+        float kd = 0.f, qd = 0.f;
+        if (tid < 16 * KD) {
+            if (tid < a.dimp) {
+                qd = mm_ld<T>(a.x, base + (int64_t)h * a.dimp + tid) * scale;
+                kd = mm_ld<T>(a.x, base + a.k_off + (int64_t)h * a.dimp + tid);
+            }
+            s_q[tid] = qd;
+            s_k[tid] = kd;
+        }
+        f32x4_t v = {0.f, 0.f, 0.f, 0.f};
+        if (con) v = mm_ld4<T>(a.x, base + a.v_off + (int64_t)h * a.vdimp + col);
+        __syncthreads();
+        float zi = 0.f, zf = 0.f;
+#pragma unroll
+        for (int w = 0; w < NWV; ++w) {
+            zi += s_g[0][w];
+            zf += s_g[1][w];
+        }
+        const float li = mm_cap(zi + bi, a.cap), lf = mm_log_sigmoid(mm_cap(zf + bf, a.cap));
+        const float mn = fmaxf(lf + m, li), keep = expf(lf + m - mn), add = expf(li - mn);
+        m = mn;
+        n = keep * n + add * kd;
+        f32x4_t o = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int k = 0; k < KD; ++k) {
+            const float ak = add * s_k[rg + 16 * k], q = s_q[rg + 16 * k];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) {
+                S[k][e] = fmaf(ak, v[e], keep * S[k][e]);
+                o[e] = fmaf(S[k][e], q, o[e]);
+            }
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            o[e] += __shfl_xor(o[e], 16, 64);
+            o[e] += __shfl_xor(o[e], 32, 64);
+        }
+        if (lane < 16) *reinterpret_cast<f32x4_t*>(&s_o[cb][wv][cq * 4]) = o;
+        const float nq = wave_sum(n * qd);
+        if (lane == 0) s_nq[wave] = nq;
+        __syncthreads();
+        float den = 0.f;
+#pragma unroll
+        for (int w = 0; w < NWV; ++w) den += s_nq[w];
+        den = fmaxf(fabsf(den), expf(-m)) + 1e-6f;
+        float ov = 0.f;  // thread tid owns column tid
+        if (tid < a.vdimp) ov = (s_o[tid >> 6][0][tid & 63] + s_o[tid >> 6][1][tid & 63] + s_o[tid >> 6][2][tid & 63] + s_o[tid >> 6][3][tid & 63]) / den;
+        const float ss = wave_sum(ov * ov);
+        if (lane == 0) s_ss[wave] = ss;
+        __syncthreads();
+        float sq = 0.f;
+#pragma unroll
+        for (int w = 0; w < NWV; ++w) sq += s_ss[w];
+        if (tid < a.vdimp) {
+            const float rms = sqrtf(sq * inv_v + a.eps), g = mm_ld<T>(a.x, base + a.g_off + (int64_t)h * a.vdimp + tid);
+            mm_st<T>(a.y, (int64_t)r * a.ldy + (int64_t)h * a.vdimp + tid, ov / rms * a.norm[(int64_t)h * a.vdimp + tid] * mm_sigmoid(g));
+        }
+    }
+    const int64_t so = a.state_out[seq];
+    if (so < 0 || so >= a.n_state) return;
+    const int64_t sout = so * a.H + h;
+#pragma unroll
+    for (int k = 0; k < KD; ++k) {
+        const int d = rg + 16 * k;
+        if (con && d < a.dimp) *reinterpret_cast<f32x4_t*>(a.S + (sout * a.dimp + d) * a.vdimp + col) = S[k];
+    }
+    if (tid < a.dimp) a.n[sout * a.dimp + tid] = n;
+    if (tid == 0) a.m[sout] = m;
+}
+
+// any head size: the state lives in its rows in memory (the row set that the step writes; scratch rows are not needed because a row set that
+// nobody keeps is only ever asked for by unused rows)
+template <typename T>
+__global__ __launch_bounds__(256) void memory_recurrent_any_kernel(const RecArgs a) {
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    float* s_q = reinterpret_cast<float*>(smem);  // [dimp]
+    float* s_k = s_q + a.dimp;                     // [dimp]
+    float* s_o = s_k + a.dimp;                     // [vdimp]
+    __shared__ __attribute__((aligned(16))) float s_part[16][64];
+    __shared__ float s_red[3][4];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, cq = tid & 15, rg = tid >> 4;
+    const int seq = blockIdx.x / a.H, h = blockIdx.x % a.H;
+    const int r0 = a.q_start[seq], r1 = a.q_start[seq + 1];
+    if (r1 <= r0) return;
+    const int64_t so = a.state_out[seq];
+    if (a.pos[r0] < 0 || so < 0 || so >= a.n_state) {
+        for (int r = r0; r < r1; ++r)
+            for (int c = tid; c < a.vdimp; c += 256) mm_st<T>(a.y, (int64_t)r * a.ldy + (int64_t)h * a.vdimp + c, 0.f);
+        return;
+    }
+    const int64_t sin = min(max((int64_t)a.state_in[seq], (int64_t)0), a.n_state - 1) * a.H + h, sout = so * a.H + h;
+    const bool fresh = a.pos[r0] == 0;
+    const float scale = 1.0f / sqrtf((float)a.dim), bi = a.bif[h], bf = a.bif[a.H + h], inv_v = 1.0f / (float)a.vdim;
+    float m = fresh ? 0.f : a.m[sin];
+    for (int r = r0; r < r1; ++r) {
+        const bool first = r == r0;
+        float gi, gf;
+        mm_gate_parts<T>(a, r, h, tid, 256, gi, gf);
+        gi = wave_sum(gi);
+        gf = wave_sum(gf);
+        __syncthreads();
+        if (lane == 0) {
+            s_red[0][wave] = gi;
+            s_red[1][wave] = gf;
+        }
+        const int64_t base = (int64_t)r * a.ldx;
+        for (int d = tid; d < a.dimp; d += 256) {
+            s_q[d] = mm_ld<T>(a.x, base + (int64_t)h * a.dimp + d) * scale;
+            s_k[d] = mm_ld<T>(a.x, base + a.k_off + (int64_t)h * a.dimp + d);
+        }
+        __syncthreads();
+        const float zi = s_red[0][0] + s_red[0][1] + s_red[0][2] + s_red[0][3], zf = s_red[1][0] + s_red[1][1] + s_red[1][2] + s_red[1][3];
+        const float li = mm_cap(zi + bi, a.cap), lf = mm_log_sigmoid(mm_cap(zf + bf, a.cap));
+        const float mn = fmaxf(lf + m, li), keep = expf(lf + m - mn), add = expf(li - mn);
+        m = mn;
+        float nq = 0.f;
+        for (int d = tid; d < a.dimp; d += 256) {
+            const float old = !first ? a.n[sout * a.dimp + d] : fresh ? 0.f : a.n[sin * a.dimp + d];
+            const float nn = keep * old + add * s_k[d];
+            a.n[sout * a.dimp + d] = nn;
+            nq += nn * s_q[d];
+        }
+        nq = wave_sum(nq);
+        if (lane == 0) s_red[2][wave] = nq;
+        __syncthreads();
+        const float den = fmaxf(fabsf(s_red[2][0] + s_red[2][1] + s_red[2][2] + s_red[2][3]), expf(-m)) + 1e-6f;
+        float ss = 0.f;
+        for (int c0 = 0; c0 < a.vdimp; c0 += 64) {
+            const int col = c0 + cq * 4;
+            f32x4_t o = {0.f, 0.f, 0.f, 0.f};
+            if (col < a.vdimp) {
+                const f32x4_t v = mm_ld4<T>(a.x, base + a.v_off + (int64_t)h * a.vdimp + col);
+                for (int d = rg; d < a.dimp; d += 16) {
+                    f32x4_t s = {0.f, 0.f, 0.f, 0.f};
+                    if (!first) s = *reinterpret_cast<const f32x4_t*>(a.S + (sout * a.dimp + d) * a.vdimp + col);
+                    else if (!fresh) s = *reinterpret_cast<const f32x4_t*>(a.S + (sin * a.dimp + d) * a.vdimp + col);
+                    const float ak = add * s_k[d], q = s_q[d];
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) {
+                        s[e] = fmaf(ak, v[e], keep * s[e]);
+                        o[e] = fmaf(s[e], q, o[e]);
+                    }
+                    *reinterpret_cast<f32x4_t*>(a.S + (sout * a.dimp + d) * a.vdimp + col) = s;
+                }
+            }
+            *reinterpret_cast<f32x4_t*>(&s_part[rg][cq * 4]) = o;
+            __syncthreads();
+            if (tid < 64 && c0 + tid < a.vdimp) {
+                float ov = 0.f;
+                for (int i = 0; i < 16; ++i) ov += s_part[i][tid];
+                ov /= den;
+                s_o[c0 + tid] = ov;
+                ss += ov * ov;
+            }
+            __syncthreads();
+        }
+        if (wave == 0) {
+            ss = wave_sum(ss);
+            if (lane == 0) s_red[0][0] = ss;
+        }
+        __syncthreads();
+        const float rms = sqrtf(s_red[0][0] * inv_v + a.eps);
+        for (int c = tid; c < a.vdimp; c += 256)
+            mm_st<T>(a.y, (int64_t)r * a.ldy + (int64_t)h * a.vdimp + c,
+                     s_o[c] / rms * a.norm[(int64_t)h * a.vdimp + c] * mm_sigmoid(mm_ld<T>(a.x, base + a.g_off + (int64_t)h * a.vdimp + c)));
+    }
+    if (tid == 0) a.m[sout] = m;
+}
+
+// ---------------------------------------------------------------------------------------------------------------------------
+struct ChunkArgs {
+    const bf16_t* x;      // projection rows (see RecArgs)
+    int64_t ldx, k_off, v_off;
+    const float* gates;   // [rows, ldg] a at h, b at H + h, biases included
+    int64_t ldg;
+    bf16_t* o;            // [rows, ldo] head h at h*vdimp, before the norm
+    int64_t ldo;
+    float *S, *n, *m;
+    int64_t n_state;
+    const int32_t *pos, *q_start, *state_in, *state_out;  // of the long portions; q_start and pos relative to x's first row
+    int H, dim, dimp, vdimp, vtiles;
+    float cap;
+};
+
+template <int OFF>
+__device__ __forceinline__ void lds_read_b64(u32x2_t& dst, unsigned addr) {
+    asm volatile("ds_read_b64 %0, %1 offset:%2" : "=v"(dst) : "v"(addr), "i"(OFF));
+}
+// v = hi + lo, two bf16 each
+__device__ __forceinline__ void mm_split(const float (&v)[8], bf16x8_t& hi, bf16x8_t& lo) {
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+        const __bf16 b = (__bf16)v[e];
+        hi[e] = b;
+        lo[e] = (__bf16)(v[e] - (float)b);
+    }
+}
+__device__ __forceinline__ f32x4_t mm_mfma(const bf16x8_t& x, const bf16x8_t& y, const f32x4_t& z) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(x, y, z, 0, 0, 0); }
+
+// D: multiple of 64, dimp <= D <= 256.  Four waves; wave w computes the scores of query rows 16 w .. + 15 and owns value columns
+// 16 w .. + 15 of the tile's 64: their state S[d][column], in the matrix cores' output layout (lane (c, g): column c, rows d = 16 i + 4 g + r),
+// is the left operand of the next chunk's readout without leaving the registers.
+template <int D>
+__global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(const ChunkArgs a) {
+    constexpr int KS = D / 32, DT = D / 16, RB = D * 2, CPR = D / 8, QT = 64 * RB, VTB = 64 * 128, STAGE = 2 * QT + VTB;
+    constexpr int QDMA = D / 32, VDMA = 2;          // 1 KiB pieces per wave
+    constexpr bool PALIAS = QT >= 16384;            // the weights (hi, lo: 16 KiB) go over the chunk's query rows, which are done by then
+    constexpr int POFF = PALIAS ? 0 : 2 * STAGE, SMALL = 2 * STAGE + (PALIAS ? 0 : 16384);
+    extern __shared__ __attribute__((aligned(16))) char smem[];
+    float* s_a = reinterpret_cast<float*>(smem + SMALL);  // i_s - b_s                   (log2 units)
+    float* s_row = s_a + 64;                               // b_t - m_t                   (log2 units)
+    float* s_in = s_row + 64;                              // c_t dim^-1/2
+    float* s_floor = s_in + 64;                            // e^(-m_t)
+    float* s_w = s_floor + 64;                             // e^(b_L - m_L + i_s - b_s)
+    float* s_den = s_w + 64;                               // n_t . q_t
+    float* s_n = s_den + 64;                               // [D]
+    const int tid = threadIdx.x, lane = tid & 63;
+    const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int c = lane & 15, g = lane >> 4;
+    const int vt = blockIdx.x % a.vtiles, h = (blockIdx.x / a.vtiles) % a.H, seq = blockIdx.x / (a.vtiles * a.H);
+    const int r0 = a.q_start[seq], T = a.q_start[seq + 1] - r0;
+    if (T <= 0) return;
+    const int n_chunks = (T + 63) >> 6;
+    const bool fresh = a.pos[r0] <= 0;
+    const int64_t sin = min(max((int64_t)a.state_in[seq], (int64_t)0), a.n_state - 1) * a.H + h;
+    const int col = vt * 64 + 16 * w + c;  // this lane's value column
+    const bool con = col < a.vdimp;
+    f32x4_t S[DT];
+#pragma unroll
+    for (int i = 0; i < DT; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int d = 16 * i + 4 * g + r;
+            S[i][r] = (!fresh && con && d < a.dimp) ? a.S[(sin * a.dimp + d) * a.vdimp + col] : 0.f;
+        }
+    // wave w keeps n of the rows d = 16 i + c with i = w mod 4 (the same in all four lane groups)
+    float nreg[DT / 4];
+#pragma unroll
+    for (int i = 0; i < DT / 4; ++i) {
+        const int d = 16 * (4 * i + w) + c;
+        nreg[i] = (!fresh && d < a.dimp) ? a.n[sin * a.dimp + d] : 0.f;
+        if (g == 0) s_n[d] = nreg[i];
+    }
+    float m_in = fresh ? 0.f : a.m[sin];
+    const float scale = 1.0f / sqrtf((float)a.dim);
+    const bf16_t* xq = a.x + (int64_t)r0 * a.ldx + (int64_t)h * a.dimp;
+    const bf16_t* xv = a.x + (int64_t)r0 * a.ldx + a.v_off + (int64_t)h * a.vdimp + vt * 64;
+    const float* gp = a.gates + (int64_t)r0 * a.ldg + h;
+    const unsigned base = lds_addr(smem);
+    auto issue = [&](int ch) {
+        char* st = smem + (ch & 1) * STAGE;
+        const int left = T - ch * 64;
+#pragma unroll
+        for (int i = 0; i < QDMA; ++i) {
+            const int p = (w * QDMA + i) * 64 + lane, row = p / CPR, cc = (p % CPR) ^ attn_swz(row);
+            const bool ok = row < left && cc * 8 < a.dimp;
+            const bf16_t* s = xq + (int64_t)(ch * 64 + row) * a.ldx + cc * 8;
+            lds_dma16(ok ? (const void*)s : (const void*)mm_zero_page, st + (w * QDMA + i) * 1024);
+            lds_dma16(ok ? (const void*)(s + a.k_off) : (const void*)mm_zero_page, st + QT + (w * QDMA + i) * 1024);
+        }
+#pragma unroll
+        for (int i = 0; i < VDMA; ++i) {
+            const int p = (w * VDMA + i) * 64 + lane, row = p >> 3, cc = (p & 7) ^ attn_swz(row);
+            const bool ok = row < left && vt * 64 + cc * 8 < a.vdimp;
+            lds_dma16(ok ? (const void*)(xv + (int64_t)(ch * 64 + row) * a.ldx + cc * 8) : (const void*)mm_zero_page, st + 2 * QT + (w * VDMA + i) * 1024);
+        }
+    };
+    // fragment offsets.  Rows by 16 (lane c), eight columns 32 i + 8 g: the scores.  Rows by 16, columns 32 i + 4 g and + 16: the readout,
+    // in the order of the state's registers.  Transposed reads, rows 4 g + qq: k and v over tokens.
+    unsigned row_rel[2], half_rel[2][2], tr_rel[4], vt_rel;
+#pragma unroll
+    for (int e = 0; e < 2; ++e) {
+        row_rel[e] = c * RB + (((4 * e + g) ^ attn_swz(c)) << 4);
+#pragma unroll
+        for (int u = 0; u < 2; ++u) half_rel[e][u] = c * RB + (((4 * e + 2 * u + (g >> 1)) ^ attn_swz(c)) << 4) + ((g & 1) << 3);
+    }
+    const int qq = (lane >> 2) & 3, pp = lane & 3, tr = 4 * g + qq;
+#pragma unroll
+    for (int e = 0; e < 4; ++e) tr_rel[e] = tr * RB + (((2 * e + (pp >> 1)) ^ attn_swz(tr)) << 4) + ((pp & 1) << 3);
+    vt_rel = tr * 128 + (((2 * w + (pp >> 1)) ^ attn_swz(tr)) << 4) + ((pp & 1) << 3);
+    float za = lane < T ? gp[(int64_t)lane * a.ldg] : 0.f, zb = lane < T ? gp[(int64_t)lane * a.ldg + a.H] : 0.f;
+    issue(0);
+    for (int ch = 0; ch < n_chunks; ++ch) {
+        const int left = T - ch * 64;
+        // ---- gates of the chunk, one token per lane, the same in every wave ----
+        const bool tok = lane < left;
+        const float li = tok ? mm_cap(za, a.cap) : -INFINITY, lf = tok ? mm_log_sigmoid(mm_cap(zb, a.cap)) : 0.f;
+        float b = lf;
+#pragma unroll
+        for (int o = 1; o < 64; o <<= 1) {
+            const float v = __shfl_up(b, o, 64);
+            if (lane >= o) b += v;
+        }
+        const float as = li - b;
+        float mx = as;
+#pragma unroll
+        for (int o = 1; o < 64; o <<= 1) {
+            const float v = __shfl_up(mx, o, 64);
+            if (lane >= o) mx = fmaxf(mx, v);
+        }
+        const float mt = b + fmaxf(m_in, mx);
+        const float bL = __shfl(b, 63, 64), mL = __shfl(mt, 63, 64);
+        const float carry = __builtin_amdgcn_exp2f((bL + m_in - mL) * MM_LOG2E);
+        wait_vm<0>();
+        __syncthreads();  // the chunk's rows are in; every wave is past its reads of the chunk before
+        if (ch + 1 < n_chunks) {
+            issue(ch + 1);
+            const int64_t t = (int64_t)(ch + 1) * 64 + lane;
+            za = t < T ? gp[t * a.ldg] : 0.f;
+            zb = t < T ? gp[t * a.ldg + a.H] : 0.f;
+        }
+        if (w == 0) {
+            s_a[lane] = as * MM_LOG2E;
+            s_row[lane] = (b - mt) * MM_LOG2E;
+            s_in[lane] = __builtin_amdgcn_exp2f((b + m_in - mt) * MM_LOG2E) * scale;
+            s_floor[lane] = __builtin_amdgcn_exp2f(-mt * MM_LOG2E);
+            s_w[lane] = __builtin_amdgcn_exp2f((bL - mL + as) * MM_LOG2E);
+        }
+        const unsigned qst = base + (ch & 1) * STAGE, kst = qst + QT, vst = kst + QT, pst = PALIAS ? qst : base + POFF;
+        char* pw = smem + (PALIAS ? (ch & 1) * STAGE : POFF);
+        // ---- scores of this wave's 16 query rows, and n . q of them ----
+        f32x4_t s[4];
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt) s[kt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        float nq = 0.f;
+        static_for<KS>([&](auto I) {
+            constexpr int i = decltype(I)::value;
+            u32x4_t qf, kf[4];
+            lds_read_b128<(i >> 1) * 128>(qf, qst + w * 16 * RB + row_rel[i & 1]);
+            static_for<4>([&](auto KT) { lds_read_b128<(i >> 1) * 128 + decltype(KT)::value * 16 * RB>(kf[decltype(KT)::value], kst + row_rel[i & 1]); });
+            wait_lds();
+            asm volatile("" : "+v"(qf), "+v"(kf[0]), "+v"(kf[1]), "+v"(kf[2]), "+v"(kf[3]));
+#pragma unroll
+            for (int kt = 0; kt < 4; ++kt) s[kt] = mm_mfma(__builtin_bit_cast(bf16x8_t, kf[kt]), __builtin_bit_cast(bf16x8_t, qf), s[kt]);
+            const f32x4_t n0 = *reinterpret_cast<const f32x4_t*>(s_n + 32 * i + 8 * g), n1 = *reinterpret_cast<const f32x4_t*>(s_n + 32 * i + 8 * g + 4);
+#pragma unroll
+            for (int e = 0; e < 2; ++e) {
+                nq = fmaf(bflo(qf[e]), n0[2 * e], nq);
+                nq = fmaf(bfhi(qf[e]), n0[2 * e + 1], nq);
+                nq = fmaf(bflo(qf[2 + e]), n1[2 * e], nq);
+                nq = fmaf(bfhi(qf[2 + e]), n1[2 * e + 1], nq);
+            }
+        });
+        // ---- what the state gives all 64 rows, in this wave's columns ----
+        f32x4_t acc[4];
+#pragma unroll
+        for (int rt = 0; rt < 4; ++rt) acc[rt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        static_for<KS>([&](auto I) {
+            constexpr int i = decltype(I)::value;
+            u32x2_t qh[4][2];
+            static_for<4>([&](auto RT) {
+                constexpr int rt = decltype(RT)::value;
+                lds_read_b64<(i >> 1) * 128 + rt * 16 * RB>(qh[rt][0], qst + half_rel[i & 1][0]);
+                lds_read_b64<(i >> 1) * 128 + rt * 16 * RB>(qh[rt][1], qst + half_rel[i & 1][1]);
+            });
+            const float sv[8] = {S[2 * i][0], S[2 * i][1], S[2 * i][2], S[2 * i][3], S[2 * i + 1][0], S[2 * i + 1][1], S[2 * i + 1][2], S[2 * i + 1][3]};
+            bf16x8_t hi, lo;
+            mm_split(sv, hi, lo);
+            wait_lds();
+#pragma unroll
+            for (int rt = 0; rt < 4; ++rt) asm volatile("" : "+v"(qh[rt][0]), "+v"(qh[rt][1]));
+#pragma unroll
+            for (int rt = 0; rt < 4; ++rt) {
+                const bf16x8_t q = __builtin_bit_cast(bf16x8_t, u32x4_t{qh[rt][0][0], qh[rt][0][1], qh[rt][1][0], qh[rt][1][1]});
+                acc[rt] = mm_mfma(hi, q, acc[rt]);
+                acc[rt] = mm_mfma(lo, q, acc[rt]);
+            }
+        });
+        __syncthreads();  // query rows read, gate arrays written
+        // ---- weights of this wave's rows: hi and lo, in the order the second product reads them ----
+        const int row = 16 * w + c;
+        const float rowc = s_row[row];
+        float dsum = 0.f;
+#pragma unroll
+        for (int sl = 0; sl < 2; ++sl) {
+            float p[8];
+#pragma unroll
+            for (int u = 0; u < 2; ++u) {
+                const int k0 = 32 * sl + 16 * u + 4 * g;
+                const f32x4_t av = *reinterpret_cast<const f32x4_t*>(s_a + k0);
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const float dw = k0 + r <= row ? __builtin_amdgcn_exp2f(rowc + av[r]) : 0.f;
+                    p[4 * u + r] = s[2 * sl + u][r] * scale * dw;
+                    dsum += p[4 * u + r];
+                }
+            }
+            bf16x8_t hi, lo;
+            mm_split(p, hi, lo);
+            const int chunk = ((4 * sl + g) ^ (c & 7)) << 4;
+            *reinterpret_cast<bf16x8_t*>(pw + row * 128 + chunk) = hi;
+            *reinterpret_cast<bf16x8_t*>(pw + 8192 + row * 128 + chunk) = lo;
+        }
+        nq = fmaf(nq, s_in[row], dsum);
+        nq += __shfl_xor(nq, 16, 64);
+        nq += __shfl_xor(nq, 32, 64);
+        if (g == 0) s_den[row] = nq;
+        __syncthreads();
+        // ---- output rows ----
+        u32x2_t vf[2][2];
+        lds_read_tr16_b64<0>(vf[0][0], vst + vt_rel);
+        lds_read_tr16_b64<16 * 128>(vf[0][1], vst + vt_rel);
+        lds_read_tr16_b64<32 * 128>(vf[1][0], vst + vt_rel);
+        lds_read_tr16_b64<48 * 128>(vf[1][1], vst + vt_rel);
+        wait_lds();
+#pragma unroll
+        for (int sl = 0; sl < 2; ++sl) asm volatile("" : "+v"(vf[sl][0]), "+v"(vf[sl][1]));
+        bf16x8_t vv[2];
+#pragma unroll
+        for (int sl = 0; sl < 2; ++sl) vv[sl] = __builtin_bit_cast(bf16x8_t, u32x4_t{vf[sl][0][0], vf[sl][0][1], vf[sl][1][0], vf[sl][1][1]});
+        static_for<4>([&](auto RT) {
+            constexpr int rt = decltype(RT)::value;
+            const int t = 16 * rt + c;
+            u32x4_t pf[2][2];
+            const unsigned pa0 = pst + c * 128 + ((g ^ (c & 7)) << 4), pa1 = pst + c * 128 + (((4 + g) ^ (c & 7)) << 4);
+            lds_read_b128<rt * 2048>(pf[0][0], pa0);
+            lds_read_b128<rt * 2048 + 8192>(pf[0][1], pa0);
+            lds_read_b128<rt * 2048>(pf[1][0], pa1);
+            lds_read_b128<rt * 2048 + 8192>(pf[1][1], pa1);
+            const float in = s_in[t], den = fmaxf(fabsf(s_den[t]), s_floor[t]) + 1e-6f;
+            f32x4_t o = acc[rt];
+#pragma unroll
+            for (int r = 0; r < 4; ++r) o[r] *= in;
+            wait_lds();
+#pragma unroll
+            for (int sl = 0; sl < 2; ++sl) asm volatile("" : "+v"(pf[sl][0]), "+v"(pf[sl][1]));
+#pragma unroll
+            for (int sl = 0; sl < 2; ++sl) {
+                if (sl == 1 && rt < 2) continue;  // keys 32 .. 63 of rows 0 .. 31: all in the future
+                o = mm_mfma(vv[sl], __builtin_bit_cast(bf16x8_t, pf[sl][0]), o);
+                o = mm_mfma(vv[sl], __builtin_bit_cast(bf16x8_t, pf[sl][1]), o);
+            }
+            const int vc = vt * 64 + 16 * w + 4 * g;
+            const float inv = 1.0f / den;
+            if (t < left && vc < a.vdimp)
+                *reinterpret_cast<u32x2_t*>(a.o + (int64_t)(r0 + ch * 64 + t) * a.ldo + (int64_t)h * a.vdimp + vc) =
+                    u32x2_t{pack2bf(o[0] * inv, o[1] * inv), pack2bf(o[2] * inv, o[3] * inv)};
+        });
+        // ---- state of the next chunk ----
+        bf16x8_t vhi[2], vlo[2];
+        float wt[2][8];
+#pragma unroll
+        for (int sl = 0; sl < 2; ++sl) {
+            const f32x4_t w0 = *reinterpret_cast<const f32x4_t*>(s_w + 32 * sl + 4 * g), w1 = *reinterpret_cast<const f32x4_t*>(s_w + 32 * sl + 16 + 4 * g);
+            float p[8];
+#pragma unroll
+            for (int e = 0; e < 8; ++e) {
+                wt[sl][e] = e < 4 ? w0[e] : w1[e - 4];
+                p[e] = wt[sl][e] * (float)vv[sl][e];
+            }
+            mm_split(p, vhi[sl], vlo[sl]);
+        }
+#pragma unroll
+        for (int i = 0; i < DT; ++i) S[i] *= carry;
+        static_for<DT>([&](auto I) {
+            constexpr int i = decltype(I)::value;
+            u32x2_t kf[2][2];
+            lds_read_tr16_b64<(i >> 2) * 128>(kf[0][0], kst + tr_rel[i & 3]);
+            lds_read_tr16_b64<(i >> 2) * 128 + 16 * RB>(kf[0][1], kst + tr_rel[i & 3]);
+            lds_read_tr16_b64<(i >> 2) * 128 + 32 * RB>(kf[1][0], kst + tr_rel[i & 3]);
+            lds_read_tr16_b64<(i >> 2) * 128 + 48 * RB>(kf[1][1], kst + tr_rel[i & 3]);
+            wait_lds();
+#pragma unroll
+            for (int sl = 0; sl < 2; ++sl) asm volatile("" : "+v"(kf[sl][0]), "+v"(kf[sl][1]));
+            float nn = 0.f;
+#pragma unroll
+            for (int sl = 0; sl < 2; ++sl) {
+                const bf16x8_t k = __builtin_bit_cast(bf16x8_t, u32x4_t{kf[sl][0][0], kf[sl][0][1], kf[sl][1][0], kf[sl][1][1]});
+                S[i] = mm_mfma(k, vhi[sl], S[i]);
+                S[i] = mm_mfma(k, vlo[sl], S[i]);
+                if ((i & 3) == w) {
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) nn = fmaf(wt[sl][e], (float)k[e], nn);
+                }
+            }
+            if ((i & 3) == w) {
+                nn += __shfl_xor(nn, 16, 64);
+                nn += __shfl_xor(nn, 32, 64);
+                nreg[i >> 2] = fmaf(carry, nreg[i >> 2], nn);
+                if (g == 0) s_n[16 * i + c] = nreg[i >> 2];  // read again behind the next barrier
+            }
+        });
+        m_in = mL;
+    }
+    const int64_t so = a.state_out[seq];
+    if (so < 0 || so >= a.n_state) return;
+    const int64_t sout = so * a.H + h;
+#pragma unroll
+    for (int i = 0; i < DT; ++i)
+#pragma unroll
+        for (int r = 0; r < 4; ++r) {
+            const int d = 16 * i + 4 * g + r;
+            if (con && d < a.dimp) a.S[(sout * a.dimp + d) * a.vdimp + col] = S[i][r];
+        }
+    if (vt == 0) {
+#pragma unroll
+        for (int i = 0; i < DT / 4; ++i) {
+            const int d = 16 * (4 * i + w) + c;
+            if (g == 0 && d < a.dimp) a.n[sout * a.dimp + d] = nreg[i];
+        }
+        if (tid == 0) a.m[sout] = m_in;
+    }
+}
+
+// y = o / rms(o) . norm . sigmoid(g) per (row, head); lph lanes (a power of two) per head, eight columns per lane and round
+struct OutArgs {
+    const bf16_t* o;
+    int64_t ldo;
+    const bf16_t* g;
+    int64_t ldg;
+    const float* norm;
+    bf16_t* y;
+    int64_t ldy, T;
+    int H, vdim, vdimp, lph;
+    float eps;
+};
+__global__ __launch_bounds__(256) void memory_output_kernel(const OutArgs a) {
+    const int64_t item = ((int64_t)blockIdx.x * 256 + threadIdx.x) / a.lph;
+    const int l = threadIdx.x & (a.lph - 1);
+    const bool on = item < a.T * a.H;
+    const int64_t r = on ? item / a.H : 0;
+    const int h = on ? (int)(item - r * a.H) : 0;
+    const bf16_t* o = a.o + r * a.ldo + (int64_t)h * a.vdimp;
+    float sq = 0.f;
+    for (int c = l * 8; c < a.vdimp; c += a.lph * 8) {
+        const u32x4_t u = *reinterpret_cast<const u32x4_t*>(o + c);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) sq += bflo(u[e]) * bflo(u[e]) + bfhi(u[e]) * bfhi(u[e]);
+    }
+    for (int x = 1; x < a.lph; x <<= 1) sq += __shfl_xor(sq, x, 64);
+    if (!on) return;
+    const float inv = 1.0f / sqrtf(sq / (float)a.vdim + a.eps);
+    const bf16_t* g = a.g + r * a.ldg + (int64_t)h * a.vdimp;
+    const float* nm = a.norm + (int64_t)h * a.vdimp;
+    bf16_t* y = a.y + r * a.ldy + (int64_t)h * a.vdimp;
+    for (int c = l * 8; c < a.vdimp; c += a.lph * 8) {
+        const u32x4_t u = *reinterpret_cast<const u32x4_t*>(o + c), gv = *reinterpret_cast<const u32x4_t*>(g + c);
+        u32x4_t out;
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+            const float g0 = bflo(gv[e]), g1 = bfhi(gv[e]);
+            out[e] = pack2bf(bflo(u[e]) * inv * nm[c + 2 * e] * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-MM_LOG2E * g0)),
+                             bfhi(u[e]) * inv * nm[c + 2 * e + 1] * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-MM_LOG2E * g1)));
+        }
+        *reinterpret_cast<u32x4_t*>(y + c) = out;
+    }
+}
+
+template <typename T, int KD, int NW>
+int launch_rec(const RecArgs& a, hipStream_t st) {
+    hipLaunchKernelGGL((memory_recurrent_kernel<T, KD, NW>), dim3((unsigned)(a.seqs * a.H)), dim3(256 * NW), 0, st, a);
+    GLM_CHECK_LAUNCH("glm_memory_recurrent");
+    return GLM_OK;
+}
+template <typename T, int KD>
+int launch_rec_v(const RecArgs& a, hipStream_t st) {
+    if (a.vdimp <= 64) return launch_rec<T, KD, 1>(a, st);
+    if (a.vdimp <= 128) return launch_rec<T, KD, 2>(a, st);
+    return launch_rec<T, KD, 4>(a, st);
+}
+template <typename T>
+int run_rec(const RecArgs& a, hipStream_t st) {
+    if (a.dimp <= 256 && a.vdimp <= 256) {
+        if (a.dimp <= 64) return launch_rec_v<T, 4>(a, st);
+        if (a.dimp <= 128) return launch_rec_v<T, 8>(a, st);
+        return launch_rec_v<T, 16>(a, st);
+    }
+    const size_t lds = (size_t)(2 * a.dimp + a.vdimp) * 4;
+    GLM_CHECK_ARG(lds <= 48 * 1024, GLM_ERR_UNSUPPORTED, "glm_memory_recurrent: head sizes %d + %d", a.dimp, a.vdimp);
+    hipLaunchKernelGGL(memory_recurrent_any_kernel<T>, dim3((unsigned)(a.seqs * a.H)), dim3(256), lds, st, a);
+    GLM_CHECK_LAUNCH("glm_memory_recurrent");
+    return GLM_OK;
+}
+
+template <int D>
+int launch_chunk(const ChunkArgs& a, int seqs, hipStream_t st) {
+    constexpr int STAGE = 2 * 64 * D * 2 + 8192, LDS = 2 * STAGE + (64 * D * 2 >= 16384 ? 0 : 16384) + 6 * 256 + D * 4;
+    static_assert(LDS <= 160 * 1024, "LDS of a CU");
+    auto kern = memory_chunkwise_kernel<D>;
+    GLM_SET_MAX_LDS(kern, LDS, "glm_memory_chunkwise");
+    hipLaunchKernelGGL(kern, dim3((unsigned)(seqs * a.H * a.vtiles)), dim3(256), LDS, st, a);
+    GLM_CHECK_LAUNCH("glm_memory_chunkwise");
+    return GLM_OK;
+}
+
+}  // namespace
+
+extern "C" int glm_memory_recurrent(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, int64_t g_off, const void* hrow, int64_t ldh, const void* wif, int64_t ldw, int wk,
+                                    const float* bif, const float* norm, void* y, int64_t ldy, float* S, float* n, float* m, int64_t n_state, const int32_t* pos,
+                                    const int32_t* q_start, const int32_t* state_in, const int32_t* state_out, int seqs, int H, int dim, int dimp, int vdim, int vdimp, float cap, float eps,
+                                    int f32, glm_stream_t stream) {
+    GLM_CHECK_ARG(x && hrow && wif && bif && norm && y && S && n && m && pos && q_start && state_in && state_out, GLM_ERR_INVALID, "glm_memory_recurrent: null pointer");
+    GLM_CHECK_ARG(seqs >= 0 && H > 0 && dim > 0 && dimp >= dim && dimp % 8 == 0 && vdim > 0 && vdimp >= vdim && vdimp % 8 == 0 && wk > 0 && wk % 8 == 0 && ldh >= wk && ldw >= wk && n_state > 0 &&
+                      k_off >= (int64_t)H * dimp && ldx >= k_off + (int64_t)H * dimp && ldx >= v_off + (int64_t)H * vdimp && ldx >= g_off + (int64_t)H * vdimp && ldy >= (int64_t)H * vdimp &&
+                      ldx % 8 == 0 && k_off % 8 == 0 && v_off % 8 == 0 && g_off % 8 == 0 && ldh % 8 == 0 && ldw % 8 == 0 && cap > 0.f && (int64_t)seqs * H < (1ll << 31) &&
+                      glm_aligned16(x) && glm_aligned16(hrow) && glm_aligned16(wif) && glm_aligned16(S), GLM_ERR_INVALID,
+                  "glm_memory_recurrent: bad shape H=%d dim=%d vdim=%d ldx=%ld", H, dim, vdim, (long)ldx);
+    if (seqs == 0) return GLM_OK;
+    RecArgs a = {x, ldx, k_off, v_off, g_off, hrow, ldh, wif, ldw, wk, bif, norm, y, ldy, S, n, m, n_state, pos, q_start, state_in, state_out, seqs, H, dim, dimp, vdim, vdimp, cap, eps};
+    return f32 ? run_rec<float>(a, glm_s(stream)) : run_rec<bf16_t>(a, glm_s(stream));
+}
+
+extern "C" int glm_memory_chunkwise(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* gates, int64_t ldg, void* o, int64_t ldo, float* S, float* n, float* m,
+                                    int64_t n_state, const int32_t* pos, const int32_t* q_start, const int32_t* state_in, const int32_t* state_out, int seqs, int H, int dim, int dimp,
+                                    int vdimp, float cap, glm_stream_t stream) {
+    GLM_CHECK_ARG(x && gates && o && S && n && m && pos && q_start && state_in && state_out, GLM_ERR_INVALID, "glm_memory_chunkwise: null pointer");
+    GLM_CHECK_ARG(seqs >= 0 && H > 0 && dim > 0 && dimp >= dim && dimp % 8 == 0 && vdimp > 0 && vdimp % 8 == 0 && n_state > 0 && k_off >= (int64_t)H * dimp && ldx >= k_off + (int64_t)H * dimp &&
+                      ldx >= v_off + (int64_t)H * vdimp && ldg >= 2 * H && ldo >= (int64_t)H * vdimp && ldx % 8 == 0 && k_off % 8 == 0 && v_off % 8 == 0 && ldo % 4 == 0 && cap > 0.f &&
+                      glm_aligned16(x) && (((uintptr_t)o) & 7) == 0, GLM_ERR_INVALID, "glm_memory_chunkwise: bad shape H=%d dim=%d vdimp=%d ldx=%ld", H, dim, vdimp, (long)ldx);
+    GLM_CHECK_ARG(dimp <= 256, GLM_ERR_UNSUPPORTED, "glm_memory_chunkwise: key size %d", dimp);
+    if (seqs == 0) return GLM_OK;
+    ChunkArgs a = {(const bf16_t*)x, ldx, k_off, v_off, gates, ldg, (bf16_t*)o, ldo, S, n, m, n_state, pos, q_start, state_in, state_out, H, dim, dimp, vdimp, (vdimp + 63) / 64, cap};
+    GLM_CHECK_ARG((int64_t)seqs * H * a.vtiles < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_memory_chunkwise: grid too large");
+    hipStream_t st = glm_s(stream);
+    if (dimp <= 64) return launch_chunk<64>(a, seqs, st);
+    if (dimp <= 128) return launch_chunk<128>(a, seqs, st);
+    return launch_chunk<256>(a, seqs, st);
+}
+
+extern "C" int glm_memory_output(const void* o, int64_t ldo, const void* g, int64_t ldg, const float* norm, void* y, int64_t ldy, int64_t T, int H, int vdim, int vdimp, float eps,
+                                 glm_stream_t stream) {
+    GLM_CHECK_ARG(o && g && norm && y && T >= 0 && H > 0 && vdim > 0 && vdimp >= vdim && vdimp % 8 == 0 && ldo >= (int64_t)H * vdimp && ldg >= (int64_t)H * vdimp && ldy >= (int64_t)H * vdimp &&
+                      ldo % 8 == 0 && ldg % 8 == 0 && ldy % 8 == 0 && glm_aligned16(o) && glm_aligned16(g) && glm_aligned16(y), GLM_ERR_INVALID,
+                  "glm_memory_output: bad shape T=%ld H=%d vdim=%d", (long)T, H, vdim);
+    if (T == 0) return GLM_OK;
+    int lph = 1;
+    while (lph < 64 && lph * 8 < vdimp) lph *= 2;
+    OutArgs a = {(const bf16_t*)o, ldo, (const bf16_t*)g, ldg, norm, (bf16_t*)y, ldy, T, H, vdim, vdimp, lph, eps};
+    const int64_t blocks = (T * H * lph + 255) / 256;
+    GLM_CHECK_ARG(blocks < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_memory_output: too many rows");
+    hipLaunchKernelGGL(memory_output_kernel, dim3((unsigned)blocks), dim3(256), 0, glm_s(stream), a);
+    GLM_CHECK_LAUNCH("glm_memory_output");
+    return GLM_OK;
+}
+

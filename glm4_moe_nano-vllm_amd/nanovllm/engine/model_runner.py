@@ -288,7 +288,9 @@ class ModelRunner:
             torch.cuda.empty_cache()
             free, total = torch.cuda.mem_get_info()
             budget = int(total * cfg.gpu_memory_utilization) - (total - free) - working - slots * m.state_bytes_per_slot()
-            cfg.num_kvcache_blocks = budget // (m.cache_bytes_per_token() * bs)
+            per_block = m.cache_bytes_per_token() * bs
+            # (a model without attention caches nothing per token: blocks then only count tokens)
+            cfg.num_kvcache_blocks = budget // per_block if per_block else slots * -(-cfg.max_model_len // bs)
             if self.world_size > 1:   # the ranks must agree on the pool
                 t = torch.tensor([cfg.num_kvcache_blocks], dtype=torch.int64, device="cpu")
                 dist.all_reduce(t, op=dist.ReduceOp.MIN, group=self.ctrl_group)

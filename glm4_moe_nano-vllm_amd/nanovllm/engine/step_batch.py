@@ -3,7 +3,7 @@ cache row), which rows belong to which sequence, where the recurrent state of a 
 lists of the attention kernels.  Everything the kernels read is packed into ONE int32 buffer: one copy to the device per step,
 and a captured step replays over a fixed buffer of the same layout.
 
-Rows are ordered short portions first (they attend in the absorbed form), then long ones; results go back in chunk order."""
+Rows are ordered short portions first (they take the kernels for few rows per sequence), then long ones; results go back in chunk order."""
 from __future__ import annotations
 
 from dataclasses import dataclass, field
@@ -49,12 +49,12 @@ class _Packer:
         return buf[self.offsets[i]: self.offsets[i] + a.size].view(a.shape)
 
 
-LONG_TILE = 128  # query rows of a long portion per workgroup (csrc/window_attn.hip)
+LONG_TILE = 128  # query rows of a long portion per workgroup (csrc/window_attn.hip, csrc/group_attn.hip)
 
 
 class StepBatch(SimpleNamespace):
     """Device views: ids int64 [T]; pos, seq_of, slots [T]; q_start [S+1]; state_in, state_out [S]; block_tables [S, width];
-    want [n]; tiles {tokens per tile: (first row, rows)}; Ta, max_short; and, if Ta < T: long_q_start, long_tile_seq,
+    want [n]; tiles {tokens per tile: (first row, rows)}; Ta rows of n_short short portions in front, max_short; and, if Ta < T: long_q_start, long_tile_seq,
     long_tile_off, windows {size: (rows, k_start, crow, hist_slots, hist_rows)}."""
 
 
@@ -133,7 +133,7 @@ def build_step(chunks: list[Chunk], spec, block_size: int, pad_rows: int = 0, ta
 
     def on_device(buf: torch.Tensor) -> StepBatch:
         v = lambda i: pk.view(buf, i)  # noqa: E731
-        b = StepBatch(**{name: v(i) for name, i in f.items()}, Ta=Ta, max_short=max_short,
+        b = StepBatch(**{name: v(i) for name, i in f.items()}, Ta=Ta, n_short=n_short, max_short=max_short,
                       tiles={s: (v(a), v(c)) for s, (a, c) in tiles.items()}, windows={})
         b.ids = b.ids.view(torch.int64)
         if longs is not None:

@@ -145,8 +145,8 @@ _SIGNATURES = {
     "glm_seq_norm": (c_int, [c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_int, c_int,
         c_int64, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p,
         c_void_p, c_void_p, c_int64, c_int, c_int64, c_int, c_int, c_float, c_void_p]),
-    "glm_embed_rows": (c_int, [c_void_p, c_void_p, c_int64, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_int,
-        c_int64, c_int, c_int, c_void_p]),
+    "glm_embed_rows": (c_int, [c_void_p, c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_int64,
+        c_int, c_int64, c_int, c_int, c_void_p]),
     "glm_latent_prepare": (c_int, [c_void_p, c_int64, c_int, c_int64, c_int64, c_int, c_int, c_int, c_int, c_void_p,
         c_float, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int, c_void_p]),
     "glm_latent_gather": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_int, c_void_p]),
@@ -154,11 +154,36 @@ _SIGNATURES = {
     "glm_latent_attn": (c_int, [c_void_p, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p,
         c_void_p, c_void_p, c_int64, c_int64, c_int, c_int, c_int, c_int, c_float, c_void_p, c_int, c_void_p, c_void_p,
         c_void_p, c_int, c_void_p]),
-    "glm_latent_merge": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int64, c_int, c_int, c_void_p]),
+    "glm_attn_merge": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int64, c_int, c_int, c_void_p]),
     "glm_latent_up": (c_int, [c_void_p, c_void_p, c_void_p, c_int64, c_int64, c_int, c_int, c_int, c_void_p]),
     "glm_window_attn_prefill": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_void_p,
         c_void_p, c_void_p, c_void_p, c_int, c_int, c_int64, c_int64, c_int, c_int, c_int, c_int, c_float, c_void_p,
         c_void_p]),
+    "glm_gemm_bf16_glu": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int, c_int, c_float, c_float,
+        c_void_p]),
+    "glm_glu_f32": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int, c_float, c_float, c_void_p]),
+    "glm_stream_norm": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_void_p, c_void_p,
+        c_void_p, c_float, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p,
+        c_void_p, c_int64, c_int, c_int64, c_int, c_int, c_int, c_float, c_void_p]),
+    "glm_group_kv_store": (c_int, [c_void_p, c_int64, c_int64, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int,
+        c_int, c_int, c_int, c_void_p]),
+    "glm_group_attn_prefill": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p, c_int64, c_int, c_void_p, c_void_p,
+        c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p, c_void_p,
+        c_void_p, c_int64, c_void_p]),
+    "glm_group_attn_decode": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p,
+        c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p,
+        c_void_p, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_void_p]),
+    "glm_group_attn_plain": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p,
+        c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_void_p, c_int64,
+        c_int, c_void_p]),
+    "glm_memory_recurrent": (c_int, [c_void_p, c_int64, c_int64, c_int64, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_int, c_void_p,
+        c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p,
+        c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_int, c_void_p]),
+    "glm_memory_chunkwise": (c_int, [c_void_p, c_int64, c_int64, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p,
+        c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
+        c_float, c_void_p]),
+    "glm_memory_output": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int, c_int, c_int,
+        c_float, c_void_p]),
 }
 
 EXPORTED_SYMBOLS = tuple(_SIGNATURES)
@@ -1258,13 +1283,16 @@ def batched_gemm_f32(x: torch.Tensor, w: torch.Tensor, y: torch.Tensor) -> None:
                                        y.stride(0), M, N, K, B, *NO_ACT, _stream()), "glm_gemm_f32")
 
 
-def embed_rows(ids: torch.Tensor, table: torch.Tensor, wp: int, cast: torch.Tensor | None = None) -> torch.Tensor:
-    """fp32 residual rows [T, wp] of the token ids; `cast` ([T, >= wp], the table's dtype) receives a copy."""
+def embed_rows(ids: torch.Tensor, table: torch.Tensor, wp: int, cast: torch.Tensor | None = None, pos: torch.Tensor | None = None,
+               freq: torch.Tensor | None = None) -> torch.Tensor:
+    """fp32 residual rows [T, wp] of the token ids; `cast` ([T, >= wp], the table's dtype) receives a copy.  freq (fp64, one per
+    pair of columns): the sinusoidal vector of the positions `pos` is added."""
     T = ids.numel()
     assert ids.dtype == torch.int64 and table.stride(1) == 1
     x = torch.empty((T, wp), dtype=torch.float32, device=table.device)
     assert cast is None or (cast.shape[0] == T and cast.stride(1) == 1 and cast.dtype == table.dtype)
-    _check(load_library().glm_embed_rows(_p(ids), _p(table), table.stride(0), table.shape[0], _p(x), wp, _p(cast),
+    assert freq is None or (freq.dtype == torch.float64 and freq.numel() >= (table.shape[1] + 1) // 2 and pos.dtype == torch.int32 and pos.numel() == T)
+    _check(load_library().glm_embed_rows(_p(ids), _p(table), table.stride(0), table.shape[0], _p(pos) if freq is not None else None, _p(freq), _p(x), wp, _p(cast),
                                          cast.stride(0) if cast is not None else wp, _is_f32(table.dtype), T, table.shape[1], wp,
                                          _stream()), "glm_embed_rows")
     return x
@@ -1397,7 +1425,7 @@ def latent_attn(qa: torch.Tensor, cache: torch.Tensor, tile_tok: torch.Tensor, t
         batched_gemm_f32(ctx.transpose(0, 1), wuv, out[:Ta].view(Ta, H, vdimp).transpose(0, 1))
         return
     if ns > 1:
-        _check(lib.glm_latent_merge(_p(part_o), _p(part_ml), _p(sink), ns, _p(ctx), Ta, H, rp, _stream()), "glm_latent_merge")
+        _check(lib.glm_attn_merge(_p(part_o), _p(part_ml), _p(sink), ns, _p(ctx), Ta, H, rp, _stream()), "glm_attn_merge")
     _check(lib.glm_latent_up(_p(ctx), _p(wuv), _p(out), out.stride(0), Ta, H, vdimp, rp, _stream()), "glm_latent_up")
 
 
@@ -1418,3 +1446,184 @@ def window_attn_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, out: 
     _check(load_library().glm_window_attn_prefill(
         _p(q), q.stride(0), _p(k), _p(v), k.stride(0), _p(out), out.stride(0), _p(q_start), _p(k_start), _p(tile_seq), _p(tile_off),
         tile_seq.numel(), S, q.shape[0], k.shape[0], heads, dk, dv, window, scale, _p(sink), _stream()), "glm_window_attn_prefill")
+
+
+# ------------------------------------------------------------------------------------------
+# decoders whose residual is several streams, with grouped-head attention over chunks and a gated matrix memory
+GLU_SLOPE = 1.702
+
+
+def gated_glu(x: torch.Tensor, w: torch.Tensor, limit: float, slope: float = GLU_SLOPE) -> torch.Tensor:
+    """Clamped gated unit of x @ w.T, w [2 N, K] rows gate | up -> [M, N]."""
+    M, K = x.shape
+    N = w.shape[0] // 2
+    assert w.shape == (2 * N, K) and w.dtype == x.dtype and x.stride(1) == 1 and w.stride(1) == 1
+    y = torch.empty((M, N), dtype=x.dtype, device=x.device)
+    if _is_f32(x.dtype):
+        z = linear_act(x, w)
+        _check(load_library().glm_glu_f32(_p(z), z.stride(0), _p(y), N, M, N, limit, slope, _stream()), "glm_glu_f32")
+    else:
+        _check(load_library().glm_gemm_bf16_glu(_p(x), x.stride(0), _p(w), w.stride(0), _p(y), N, M, N, K, limit, slope, _stream()),
+               "glm_gemm_bf16_glu")
+    return y
+
+
+def stream_norm(x: torch.Tensor, streams: int, width: int, eps: float, y: torch.Tensor | None = None, y_scale: torch.Tensor | None = None,
+                mix_out: torch.Tensor | None = None, w_in: torch.Tensor | None = None, gain: float = 1.0, shift: torch.Tensor | None = None,
+                state: torch.Tensor | None = None, meta=None, rows: torch.Tensor | None = None, act_dtype=torch.bfloat16, keep_x: bool = True):
+    """Between two sublayers (glm_stream_norm): returns (streams, h).  x: [T, wp] (all streams are that row) or [T, streams, wp], fp32;
+    y: the finished sublayer's output [T, wp]; w_in: weights of the next sublayer's input (None: no h); shift + state: token shift with
+    the step's `meta`; rows: gather of rows (streams are not kept)."""
+    wp = x.shape[-1]
+    assert x.dtype == torch.float32 and x.is_contiguous() and wp % 8 == 0 and width <= wp and (x.dim() == 2 or x.shape[1] == streams)
+    T = rows.numel() if rows is not None else x.shape[0]
+    for t, n in ((y_scale, wp), (mix_out, streams * (streams + 1)), (w_in, streams), (shift, wp)):
+        assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.numel() == n)
+    assert y is None or (y.stride(1) == 1 and y.shape == (x.shape[0], wp) and y_scale is not None and mix_out is not None)
+    x_out = torch.empty((T, streams, wp), dtype=torch.float32, device=x.device) if (y is not None and keep_x and rows is None) else None
+    h = torch.empty((T, wp), dtype=act_dtype, device=x.device) if w_in is not None else None
+    pos = seq_of = q_start = s_in = s_out = None
+    if shift is not None:
+        pos, seq_of, q_start, s_in, s_out = meta.pos, meta.seq_of, meta.q_start, meta.state_in, meta.state_out
+        assert pos.numel() == seq_of.numel() == T and q_start.numel() == s_in.numel() + 1 == s_out.numel() + 1
+        assert state.dtype == torch.float32 and state.is_contiguous() and state.shape[1] == wp
+    if x_out is not None or h is not None:
+        _check(load_library().glm_stream_norm(
+            _p(x), x.stride(0), x.stride(1) if x.dim() == 3 else 0, _p(rows), _p(x_out), _p(y), y.stride(0) if y is not None else wp,
+            _is_f32(y.dtype) if y is not None else 0, _p(y_scale), _p(mix_out), _p(w_in), gain, _p(shift), _p(state) if shift is not None else None,
+            state.shape[0] if shift is not None else 0, _p(pos), _p(seq_of), _p(q_start), _p(s_in), _p(s_out), _p(h), wp, _is_f32(act_dtype), T,
+            streams, width, wp, eps, _stream()), "glm_stream_norm")
+    return (x if x_out is None else x_out), h
+
+
+GROUP_ATTN_MAX_DIM = 256   # head sizes of glm_group_attn_prefill / _decode
+GROUP_ATTN_ROWS = 16       # (token, head) rows a decode workgroup takes
+
+
+def group_kv_store(src: torch.Tensor, k_off: int, v_off: int, slots: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor) -> None:
+    """Key and value columns of projection rows -> their cache rows.  Caches [blocks, G, block size, head size]."""
+    n, G, bs, dk = k_cache.shape
+    assert v_cache.shape[:3] == (n, G, bs) and k_cache.dtype == v_cache.dtype == src.dtype and k_cache.is_contiguous() and v_cache.is_contiguous()
+    assert slots.dtype == torch.int32 and slots.numel() == src.shape[0] and src.stride(1) == 1
+    _check(load_library().glm_group_kv_store(_p(src), src.stride(0), k_off, v_off, _is_f32(src.dtype), _p(slots), src.shape[0], _p(k_cache), _p(v_cache),
+                                             n * bs, bs, G, dk, v_cache.shape[3], _stream()), "glm_group_kv_store")
+
+
+def _group_shape(q, k_cache, v_cache, out, heads, slope, sink):
+    n, G, bs, dk = k_cache.shape
+    dv = v_cache.shape[3]
+    assert v_cache.shape[:3] == (n, G, bs) and k_cache.dtype == v_cache.dtype == q.dtype == out.dtype and k_cache.is_contiguous() and v_cache.is_contiguous()
+    assert q.shape[1] == heads * dk and out.shape[1] == heads * dv and q.stride(1) == out.stride(1) == 1 and out.shape[0] >= q.shape[0]
+    for t in (slope, sink):
+        assert t is None or (t.dtype == torch.float32 and t.numel() == heads)
+    return n, G, bs, dk, dv
+
+
+def group_attn_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor, seq0: int, q_start: torch.Tensor,
+                       pos: torch.Tensor, tile_seq: torch.Tensor, tile_off: torch.Tensor, heads: int, window: int, chunk: int, scale: float, slope, sink,
+                       out: torch.Tensor) -> None:
+    """Long portions (rows of q, q_start relative to them) over the paged caches; block table of portion s in row seq0 + s."""
+    n, G, bs, dk, dv = _group_shape(q, k_cache, v_cache, out, heads, slope, sink)
+    for t in (block_tables, q_start, pos, tile_seq, tile_off):
+        assert t.dtype == torch.int32
+    assert pos.numel() == q.shape[0] and tile_seq.numel() == tile_off.numel() and block_tables.shape[0] >= seq0 + q_start.numel() - 1
+    _check(load_library().glm_group_attn_prefill(
+        _p(q), q.stride(0), _p(k_cache), _p(v_cache), n, bs, _p(block_tables), block_tables.stride(0), seq0, _p(q_start), _p(pos), _p(tile_seq), _p(tile_off),
+        tile_seq.numel(), heads, G, dk, dv, window, chunk, scale, _p(slope), _p(sink), _p(out), out.stride(0), _stream()), "glm_group_attn_prefill")
+
+
+def group_attn_splits(tiles: int, tokens_per_tile: int, heads: int, kv_heads: int, keys: int) -> int:
+    """KV splits of a decode launch: about one workgroup per CU, at least 128 keys each."""
+    wgs = tiles * kv_heads * -(-tokens_per_tile * (heads // kv_heads) // GROUP_ATTN_ROWS)
+    return max(1, min(64, 256 // max(1, wgs), -(-keys // 128)))
+
+
+def group_attn_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor, pos: torch.Tensor, seq_of: torch.Tensor,
+                      tile_tok: torch.Tensor, tile_n: torch.Tensor, tokens_per_tile: int, heads: int, window: int, chunk: int, scale: float, slope, sink,
+                      out: torch.Tensor, num_splits: int = 0) -> None:
+    """Decoded tokens and short portions (the rows of q) over the paged caches; out is written row by row from its first."""
+    n, G, bs, dk, dv = _group_shape(q, k_cache, v_cache, out, heads, slope, sink)
+    T = q.shape[0]
+    if T == 0:
+        return
+    for t in (block_tables, pos, seq_of, tile_tok, tile_n):
+        assert t.dtype == torch.int32
+    assert pos.numel() >= T and seq_of.numel() >= T and tile_tok.numel() == tile_n.numel()
+    keys = block_tables.shape[1] * bs
+    for w in (window, chunk):
+        keys = min(keys, w + tokens_per_tile) if w else keys
+    ns = num_splits or (group_attn_splits(tile_tok.numel(), tokens_per_tile, heads, G, keys) if sink is not None and out.stride(0) == heads * dv else 1)
+    part_o = part_ml = None
+    if ns > 1:
+        part_o = torch.empty((T * heads, ns, dv), dtype=torch.float32, device=q.device)
+        part_ml = torch.empty((T * heads, ns, 2), dtype=torch.float32, device=q.device)
+    lib = load_library()
+    _check(lib.glm_group_attn_decode(
+        _p(q), q.stride(0), _p(k_cache), _p(v_cache), n, bs, _p(block_tables), block_tables.stride(0), _p(pos), _p(seq_of), _p(tile_tok), _p(tile_n),
+        tile_tok.numel(), tokens_per_tile, heads, G, dk, dv, window, chunk, scale, _p(slope), _p(sink), _p(out), out.stride(0), ns, _p(part_o), _p(part_ml),
+        _stream()), "glm_group_attn_decode")
+    if ns > 1:
+        assert sink is not None and out.stride(0) == heads * dv
+        _check(lib.glm_attn_merge(_p(part_o), _p(part_ml), _p(sink), ns, _p(out), T, heads, dv, _stream()), "glm_attn_merge")
+
+
+def group_attn_plain(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor, pos: torch.Tensor, seq_of: torch.Tensor,
+                     heads: int, window: int, chunk: int, scale: float, slope, sink, out: torch.Tensor) -> None:
+    """The same for any head size, in fp32 arithmetic whatever the dtype of the rows and caches."""
+    n, G, bs, dk, dv = _group_shape(q, k_cache, v_cache, out, heads, slope, sink)
+    for t in (block_tables, pos, seq_of):
+        assert t.dtype == torch.int32
+    assert pos.numel() >= q.shape[0] and seq_of.numel() >= q.shape[0]
+    _check(load_library().glm_group_attn_plain(
+        _p(q), q.stride(0), _p(k_cache), _p(v_cache), n, bs, _p(block_tables), block_tables.stride(0), _p(pos), _p(seq_of), q.shape[0], heads, G, dk, dv, window,
+        chunk, scale, _p(slope), _p(sink), _p(out), out.stride(0), _is_f32(q.dtype), _stream()), "glm_group_attn_plain")
+
+
+MEMORY_CHUNK_MAX_DIM = 256   # key size of glm_memory_chunkwise
+
+
+def _memory_state(state, heads, dimp, vdimp):
+    S, n, m = state
+    assert S.shape[1:] == (heads, dimp, vdimp) and n.shape == (S.shape[0], heads, dimp) and m.shape == (S.shape[0], heads)
+    for t in state:
+        assert t.dtype == torch.float32 and t.is_contiguous()
+    return S, n, m
+
+
+def memory_recurrent(x: torch.Tensor, hrow: torch.Tensor, wif: torch.Tensor, bif: torch.Tensor, norm: torch.Tensor, y: torch.Tensor, state, pos, q_start, state_in,
+                     state_out, heads: int, dim: int, vdim: int, cap: float, eps: float) -> None:
+    """Gated matrix memory token by token, gates and output norm included: rows x = q | k | v | g (heads padded to multiples of 8) -> y."""
+    dimp, vdimp = round8(dim), round8(vdim)
+    S, n, m = _memory_state(state, heads, dimp, vdimp)
+    kd, vd = heads * dimp, heads * vdimp
+    assert x.shape[1] >= 2 * kd + 2 * vd and x.stride(1) == hrow.stride(1) == wif.stride(1) == y.stride(1) == 1 and x.dtype == hrow.dtype == wif.dtype == y.dtype
+    assert wif.shape == (2 * heads, hrow.shape[1]) and bif.numel() == 2 * heads and norm.numel() == vd and bif.dtype == norm.dtype == torch.float32
+    for t in (pos, q_start, state_in, state_out):
+        assert t.dtype == torch.int32
+    seqs = q_start.numel() - 1
+    assert state_in.numel() >= seqs and state_out.numel() >= seqs
+    _check(load_library().glm_memory_recurrent(
+        _p(x), x.stride(0), kd, 2 * kd, 2 * kd + vd, _p(hrow), hrow.stride(0), _p(wif), wif.stride(0), hrow.shape[1], _p(bif), _p(norm), _p(y), y.stride(0), _p(S), _p(n),
+        _p(m), S.shape[0], _p(pos), _p(q_start), _p(state_in), _p(state_out), seqs, heads, dim, dimp, vdim, vdimp, cap, eps, _is_f32(x.dtype), _stream()),
+        "glm_memory_recurrent")
+
+
+def memory_chunkwise(x: torch.Tensor, gates: torch.Tensor, norm: torch.Tensor, y: torch.Tensor, state, pos, q_start, state_in, state_out, heads: int, dim: int,
+                     vdim: int, cap: float, eps: float) -> None:
+    """The same for long portions (bf16), 64 tokens at a time; gates: fp32 [rows, >= 2 heads] gate projections with their biases.  q_start
+    and pos relative to the rows of x."""
+    _bf16(x, "x"); _bf16(y, "y")
+    dimp, vdimp = round8(dim), round8(vdim)
+    S, n, m = _memory_state(state, heads, dimp, vdimp)
+    kd, vd, T = heads * dimp, heads * vdimp, x.shape[0]
+    assert x.shape[1] >= 2 * kd + 2 * vd and gates.dtype == torch.float32 and gates.shape[0] == T and gates.shape[1] >= 2 * heads and x.stride(1) == y.stride(1) == gates.stride(1) == 1
+    for t in (pos, q_start, state_in, state_out):
+        assert t.dtype == torch.int32
+    seqs = q_start.numel() - 1
+    assert state_in.numel() >= seqs and state_out.numel() >= seqs and pos.numel() == T
+    o = torch.empty((T, vd), dtype=x.dtype, device=x.device)
+    lib = load_library()
+    _check(lib.glm_memory_chunkwise(_p(x), x.stride(0), kd, 2 * kd, _p(gates), gates.stride(0), _p(o), vd, _p(S), _p(n), _p(m), S.shape[0], _p(pos), _p(q_start),
+                                    _p(state_in), _p(state_out), seqs, heads, dim, dimp, vdimp, cap, _stream()), "glm_memory_chunkwise")
+    _check(lib.glm_memory_output(_p(o), vd, _p(x[:, 2 * kd + vd:]), x.stride(0), _p(norm), _p(y), y.stride(0), T, heads, vdim, vdimp, eps, _stream()),
+           "glm_memory_output")

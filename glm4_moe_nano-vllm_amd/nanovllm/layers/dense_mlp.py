@@ -1,4 +1,4 @@
-"""Ungated feed-forward W_down act(W_up h) with the activation in the epilogue of the up projection."""
+"""Feed-forwards W_down act(W_up h) and W_down unit(W_gate h, W_up h), the activation in the epilogue of the first projection."""
 from __future__ import annotations
 
 import torch
@@ -38,6 +38,31 @@ class DenseMLP(nn.Module):
 
     def forward(self, h: torch.Tensor) -> torch.Tensor:
         y = self.down(self.up(h, act=self.act))
+        if self.tp_size > 1:
+            get_tp_group().all_reduce(y)
+        return y
+
+
+class GatedMLP(nn.Module):
+    """Clamped gated unit: g sigmoid(slope g) (u + 1) with g = min(gate, limit), u = up within +-limit."""
+
+    def __init__(self, width: int, ff: int, limit: float, dtype):
+        super().__init__()
+        tp = get_tp_group()
+        if ff % tp.world_size:
+            raise ValueError(f"a feed-forward of {ff} does not split over {tp.world_size} ranks")
+        self.tp_size, self.tp_rank, self.ff, self.limit = tp.world_size, tp.rank, ff // tp.world_size, limit
+        self.gate_up = PaddedLinear(width, [hip_ops.round8(self.ff)] * 2, dtype)
+        self.down = PaddedLinear(self.ff, [hip_ops.round8(width)], dtype)
+
+    def load(self, w: dict, device) -> None:
+        """w: gate, up, down."""
+        lo = self.tp_rank * self.ff
+        self.gate_up.load([w["gate"][lo: lo + self.ff], w["up"][lo: lo + self.ff]], device)
+        self.down.load([w["down"][:, lo: lo + self.ff]], device)
+
+    def forward(self, h: torch.Tensor) -> torch.Tensor:
+        y = self.down(hip_ops.gated_glu(h, self.gate_up.weight, self.limit))
         if self.tp_size > 1:
             get_tp_group().all_reduce(y)
         return y

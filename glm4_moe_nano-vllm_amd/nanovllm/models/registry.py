@@ -33,8 +33,10 @@ GLM4_MOE = ModelEntry("glm4_moe", "nanovllm.config:normalise_hf_config", "nanovl
                       256, 256, ("bfloat16",), None, False)
 DAFOLORN = ModelEntry("dafolorn", "nanovllm.models.dafolorn.config:read_config", "nanovllm.models.dafolorn.model:DafolornForCausalLM",
                       64, 32, ("bfloat16", "float32"), "dafolorn", True)
+NAPADRA = ModelEntry("napadra", "nanovllm.models.napadra.config:read_config", "nanovllm.models.napadra.model:NapadraForCausalLM",
+                     64, 64, ("bfloat16", "float32"), "napadra", True)
 
-_ENTRIES = {e.name: e for e in (GLM4_MOE, DAFOLORN)}
+_ENTRIES = {e.name: e for e in (GLM4_MOE, DAFOLORN, NAPADRA)}
 
 
 def find_model(cfg) -> ModelEntry:

@@ -492,9 +492,10 @@ int glm_allreduce_oneshot(const void* in, void* out, void* const* peer_bufs, voi
  * zero weights by the caller; kernels never read uninitialised memory into a product.                                       */
 
 /* activations of a projection's fp32 result: xIELU (z > 0: a z^2 + z/2; z <= 0: b (exp(z) - 1 - z) + z/2), soft cap a tanh(z/a) */
-#define GLM_EPI_NONE    0
-#define GLM_EPI_XIELU   1
-#define GLM_EPI_SOFTCAP 2
+#define GLM_EPI_NONE      0
+#define GLM_EPI_XIELU     1
+#define GLM_EPI_SOFTCAP   2
+#define GLM_EPI_GLU_CLAMP 3 /* glm_gemm_bf16_glu only */
 /* y = act(x . W^T + bias): glm_gemm_bf16 with an activation in the epilogue and, with out_f32, fp32 output rows (unrounded).  */
 int glm_gemm_bf16_act(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* bias, void* y, int64_t ldy, int64_t M,
                       int N, int K, int out_f32, int act, float act_a, float act_b, glm_stream_t stream);
@@ -502,6 +503,13 @@ int glm_gemm_bf16_act(const void* x, int64_t ldx, const void* w, int64_t ldw, co
 int glm_gemm_f32(const float* x, int64_t ldx, int64_t xb, const float* w, int64_t ldw, int64_t wb, const float* bias, float* y,
                  int64_t ldy, int64_t yb, int64_t M, int N, int K, int batch, int act, float act_a, float act_b,
                  glm_stream_t stream);
+
+/* Gated projection, W rows gate | up (2 N rows): y = g sigmoid(slope g) (u + 1), g = min(gate, limit), u = up clamped to [-limit, limit],
+ * on the fp32 accumulators.  glm_glu_f32: the unit alone, on fp32 rows gate | up (2 N columns).                              */
+int glm_gemm_bf16_glu(const void* x, int64_t ldx, const void* w, int64_t ldw, void* y, int64_t ldy, int64_t M, int N, int K,
+                      float limit, float slope, glm_stream_t stream);
+int glm_glu_f32(const float* x, int64_t ldx, float* y, int64_t ldy, int64_t M, int N, float limit, float slope,
+                glm_stream_t stream);
 
 /* Between two sublayers: x_out = x_in + rms(y) g_post (y bf16, or the sum of n_slabs fp32 slabs); h = rms(x_out) g_pre, then
  * h += depthwise causal convolution over time.  Gains fp32, conv_w [taps][wp] bf16, x fp32.  Rows of a step: row t belongs to
@@ -515,9 +523,62 @@ int glm_seq_norm(const float* x_in, const int32_t* row_index, int64_t ldx, float
                  const void* conv_w, int taps, float* state, int64_t n_state, const int32_t* pos, const int32_t* seq_of,
                  const int32_t* q_start, const int32_t* state_in, const int32_t* state_out, void* h, int64_t ldh, int act_f32,
                  int64_t T, int width, int wp, float eps, glm_stream_t stream);
-/* embedding rows as the fp32 residual and, optionally, in the activation dtype; columns [width, wp) are zeros                 */
-int glm_embed_rows(const int64_t* ids, const void* table, int64_t ldw, int64_t vocab, float* x, int64_t ldx, void* cast,
-                   int64_t ldc, int act_f32, int64_t T, int width, int wp, glm_stream_t stream);
+/* embedding rows as the fp32 residual and, optionally, in the activation dtype; columns [width, wp) are zeros.  freq [width / 2 rounded
+ * up] (double, or NULL) with pos [T]: sin(pos freq[i]) is added at column 2i, cos(pos freq[i]) at column 2i + 1             */
+int glm_embed_rows(const int64_t* ids, const void* table, int64_t ldw, int64_t vocab, const int32_t* pos, const double* freq,
+                   float* x, int64_t ldx, void* cast, int64_t ldc, int act_f32, int64_t T, int width, int wp, glm_stream_t stream);
+
+/* Between two sublayers of a decoder whose residual is S parallel streams: x'_t = sum_s mix[s, t] x_s + out[t] (y_scale . y), then
+ * u = sum_s w_in[s] x'_s, h = u / rms(u) gain, and with `shift` h += (h of the previous token - h) . shift.  x_in: row r, stream s at
+ * r*ldx + s*sx (sx = 0: one row stands for all streams); x_out [T][S][wp]; mix_out: S*S mix (from, to), then S out; y, x_out, h and
+ * shift are optional.  Rows of a step and state rows [n_state][wp] as for glm_seq_norm; row_index gathers rows (no shift, no x_out).  */
+int glm_stream_norm(const float* x_in, int64_t ldx, int64_t sx, const int32_t* row_index, float* x_out, const void* y, int64_t ldy,
+                    int y_f32, const float* y_scale, const float* mix_out, const float* w_in, float gain, const float* shift,
+                    float* state, int64_t n_state, const int32_t* pos, const int32_t* seq_of, const int32_t* q_start,
+                    const int32_t* state_in, const int32_t* state_out, void* h, int64_t ldh, int h_f32, int64_t T, int S,
+                    int width, int wp, float eps, glm_stream_t stream);
+
+/* Causal attention of H query heads over G key / value heads in paged caches [n_blocks][G][block_size][dk | dv] (block_size % 64 == 0;
+ * dk, dv multiples of 8).  A row at position p sees j <= p with p - j < window (window > 0) and in its own chunk of `chunk` positions
+ * (chunk > 0); score = scale q.k - slope[h] (p - j) (slope may be NULL); softmax with the extra mass exp(sink[h]) (sink may be NULL).
+ * store: key / value columns of projection rows -> cache rows slots[t] (< 0: none).
+ * prefill: 128-row tiles (sequence, first row inside the portion) of portions [q_start[s], q_start[s+1]), block table row seq0 + s.
+ * decode: tiles of tile_n[i] <= tokens_per_tile rows of one sequence from tile_tok[i]; nsplit > 1: unnormalised sums part_o
+ * [rows*H, nsplit, dv] and part_ml [rows*H, nsplit, 2] for glm_attn_merge.  Both bf16, dk, dv <= 256.  plain: any size, bf16 or fp32.  */
+int glm_group_kv_store(const void* src, int64_t ld, int64_t k_off, int64_t v_off, int f32, const int32_t* slots, int64_t T,
+                       void* kc, void* vc, int64_t n_slots, int bs, int G, int dk, int dv, glm_stream_t stream);
+int glm_group_attn_prefill(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs,
+                           const int32_t* block_tables, int64_t bt_stride, int seq0, const int32_t* q_start, const int32_t* pos,
+                           const int32_t* tile_seq, const int32_t* tile_off, int n_tiles, int H, int G, int dk, int dv, int window,
+                           int chunk, float scale, const float* slope, const float* sink, void* out, int64_t ldo,
+                           glm_stream_t stream);
+int glm_group_attn_decode(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs,
+                          const int32_t* block_tables, int64_t bt_stride, const int32_t* pos, const int32_t* seq_of,
+                          const int32_t* tile_tok, const int32_t* tile_n, int n_tiles, int tokens_per_tile, int H, int G, int dk,
+                          int dv, int window, int chunk, float scale, const float* slope, const float* sink, void* out,
+                          int64_t ldo, int nsplit, float* part_o, float* part_ml, glm_stream_t stream);
+int glm_group_attn_plain(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs,
+                         const int32_t* block_tables, int64_t bt_stride, const int32_t* pos, const int32_t* seq_of, int64_t rows,
+                         int H, int G, int dk, int dv, int window, int chunk, float scale, const float* slope, const float* sink,
+                         void* out, int64_t ldo, int f32, glm_stream_t stream);
+
+/* Gated matrix memory (mLSTM; the recurrence is written out in csrc/matrix_memory.hip).  Projection rows x hold q at h*dimp, k at
+ * k_off + h*dimp, v at v_off + h*vdimp and the output gate at g_off + h*vdimp.  State rows S [n_state][H][dimp][vdimp], n
+ * [n_state][H][dimp], m [n_state][H], fp32; sequence s reads row state_in[s] (not at position 0) and writes row state_out[s].
+ * recurrent: portions [q_start[s], q_start[s+1]) token by token; gate projections wif [2 H rows i | f, wk] of rows hrow, biases bif.
+ * chunkwise: bf16, dimp <= 256; gates [rows, >= 2 H] = the gate projections with their biases; o: rows in front of the norm.
+ * output: y = o / rms(o) norm sigmoid(g) per head.                                                                          */
+int glm_memory_recurrent(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, int64_t g_off, const void* hrow, int64_t ldh,
+                         const void* wif, int64_t ldw, int wk, const float* bif, const float* norm, void* y, int64_t ldy, float* S,
+                         float* n, float* m, int64_t n_state, const int32_t* pos, const int32_t* q_start, const int32_t* state_in,
+                         const int32_t* state_out, int seqs, int H, int dim, int dimp, int vdim, int vdimp, float cap, float eps,
+                         int f32, glm_stream_t stream);
+int glm_memory_chunkwise(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* gates, int64_t ldg, void* o,
+                         int64_t ldo, float* S, float* n, float* m, int64_t n_state, const int32_t* pos, const int32_t* q_start,
+                         const int32_t* state_in, const int32_t* state_out, int seqs, int H, int dim, int dimp, int vdimp, float cap,
+                         glm_stream_t stream);
+int glm_memory_output(const void* o, int64_t ldo, const void* g, int64_t ldg, const float* norm, void* y, int64_t ldy, int64_t T,
+                      int H, int vdim, int vdimp, float eps, glm_stream_t stream);
 
 /* Latent attention over a paged cache [n_blocks, block_size, rp] of latent rows (rp = rank rounded up to 8).
  * prepare: row t of qc holds the query heads at h*dimp and the raw latent at c_off; c = rms(raw) norm_w goes to cache row
@@ -530,15 +591,15 @@ int glm_latent_gather(const void* cache, int64_t n_slots, const int32_t* slots, 
 /* attn: query row (t, h) sees the latents of positions (pos[t] - window, pos[t]] of its sequence; softmax with the extra mass
  * exp(sink[h]).  Tiles: tile i covers tile_n[i] <= tokens_per_tile consecutive rows of one sequence from tile_tok[i]; tokens x
  * heads of a tile <= glm_latent_attn_max_rows(rp).  nsplit == 1: ctx [Ta, H, rp] normalised (bf16 / fp32); else part_o
- * [Ta*H, nsplit, rp], part_ml [Ta*H, nsplit, 2] for glm_latent_merge, which forms ctx.  fp32: tiles unused, nsplit 1.
+ * [Ta*H, nsplit, rp], part_ml [Ta*H, nsplit, 2] for glm_attn_merge, which forms ctx.  fp32: tiles unused, nsplit 1.
  * up: out[t, h*vdimp ..] = W_uv[h] ctx[t, h, :] (wuv [H, vdimp, rp]).                                                         */
 int glm_latent_attn_max_rows(int rp);
 int glm_latent_attn(const void* qa, const void* cache, int64_t n_blocks, int block_size, const int32_t* tile_tok,
                     const int32_t* tile_n, int n_tiles, int tokens_per_tile, const int32_t* pos, const int32_t* seq_of,
                     const int32_t* block_tables, int64_t bt_stride, int64_t Ta, int H, int rank, int rp, int window, float scale,
                     const float* sink, int nsplit, void* ctx, float* part_o, float* part_ml, int act_f32, glm_stream_t stream);
-int glm_latent_merge(const float* part_o, const float* part_ml, const float* sink, int nsplit, void* ctx, int64_t Ta, int H, int rp,
-                     glm_stream_t stream);
+int glm_attn_merge(const float* part_o, const float* part_ml, const float* sink, int nsplit, void* ctx, int64_t Ta, int H, int cols,
+                   glm_stream_t stream);
 int glm_latent_up(const void* ctx, const void* wuv, void* out, int64_t ldo, int64_t Ta, int H, int vdimp, int rp,
                   glm_stream_t stream);
 /* Prompts and long portions, bf16: q rows [q_start[s], q_start[s+1]) against expanded k / v rows [k_start[s], k_start[s+1]) — the
