@@ -131,7 +131,7 @@ class NapadraForCausalLM(nn.Module):
         """fp32 logits [meta.want_rows, vocab] of the wanted rows of a step.  residual_tap (a list) receives the sum of the
         streams [T, width] after every layer."""
         cfg, dt = self.config, self.dtype
-        x = hip_ops.embed_rows(meta.ids, self.embed, cfg.padded_width, pos=meta.pos, freq=self.freq)   # stands for all streams
+        x = hip_ops.embed_rows(meta.ids, self.embed[:, : cfg.hidden_size], cfg.padded_width, pos=meta.pos, freq=self.freq)   # stands for all streams
         finished = y = None          # the sublayer whose output y is not yet in x
         for layer in self.layers:
             x, h = layer.sub1.enter(x, finished, y, meta, dt)

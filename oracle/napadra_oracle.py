@@ -13,11 +13,18 @@ import torch
 
 
 class Weights:
-    def __init__(self, tensors: dict, dtype=torch.float64):
+    """noise: seed of a relative disturbance of every projection's result by up to 2^-8, about what 16-bit activations do (None: none)."""
+
+    def __init__(self, tensors: dict, dtype=torch.float64, noise: int | None = None):
         self.t, self.dtype = tensors, dtype
+        self.gen = None if noise is None else torch.Generator().manual_seed(noise)
 
     def __getitem__(self, name: str) -> torch.Tensor:
         return self.t[name].to(self.dtype)
+
+    def linear(self, h: torch.Tensor, name: str) -> torch.Tensor:
+        z = h @ self[name].T
+        return z if self.gen is None else z * (1 + 2.0 ** -8 * (2 * torch.rand(z.shape, generator=self.gen, dtype=z.dtype) - 1))
 
 
 # ---- embedding --------------------------------------------------------------------------------------------------------------
@@ -86,12 +93,12 @@ def slope(h: int, heads: int) -> float:
 
 def keys_values(h, W, pre, spec):
     T, G = h.shape[0], spec["kv_heads"]
-    return (h @ W[pre + "k"].T).view(T, G, spec["dim"]), (h @ W[pre + "v"].T).view(T, G, spec["vdim"])
+    return (W.linear(h, pre + "k")).view(T, G, spec["dim"]), (W.linear(h, pre + "v")).view(T, G, spec["vdim"])
 
 
 def attention(h, W, pre, spec, kv):
     H, G, T = spec["heads"], spec["kv_heads"], h.shape[0]
-    q = (h @ W[pre + "q"].T).view(T, H, spec["dim"])
+    q = (W.linear(h, pre + "q")).view(T, H, spec["dim"])
     k, v = kv
     dist = (torch.arange(T)[:, None] - torch.arange(T)[None, :]).to(h.dtype)
     visible, sink = chunk_mask(T, spec["mask"]["size"]), W[pre + "sink"]
@@ -100,7 +107,7 @@ def attention(h, W, pre, spec, kv):
         g = i // (H // G)
         a = sink_softmax((q[:, i] @ k[:, g].T) * spec["scale"] - slope(i, H) * dist, visible, sink[i])
         out[:, i] = a @ v[:, g]
-    return out.reshape(T, -1) @ W[pre + "o"].T
+    return W.linear(out.reshape(T, -1), pre + "o")
 
 
 # ---- matrix memory ------------------------------------------------------------------------------------------------------------------
@@ -121,18 +128,18 @@ def mlstm_cell(q, k, v, i, f):
 
 def mlstm(h, W, pre, spec, eps):
     H, d, dv, cap, T = spec["heads"], spec["dim"], spec["vdim"], spec["gate_cap"], h.shape[0]
-    q = (h @ W[pre + "q"].T).view(T, H, d) * d ** -0.5
-    k, v = (h @ W[pre + "k"].T).view(T, H, d), (h @ W[pre + "v"].T).view(T, H, dv)
-    i = soft_cap(h @ W[pre + "i"].T + W[pre + "i.b"], cap)
-    f = log_sigmoid(soft_cap(h @ W[pre + "f"].T + W[pre + "f.b"], cap))
+    q = (W.linear(h, pre + "q")).view(T, H, d) * d ** -0.5
+    k, v = (W.linear(h, pre + "k")).view(T, H, d), (W.linear(h, pre + "v")).view(T, H, dv)
+    i = soft_cap(W.linear(h, pre + "i") + W[pre + "i.b"], cap)
+    f = log_sigmoid(soft_cap(W.linear(h, pre + "f") + W[pre + "f.b"], cap))
     o = torch.stack([unit_rms(mlstm_cell(q[:, a], k[:, a], v[:, a], i[:, a], f[:, a]), eps) for a in range(H)], 1)
-    y = o.reshape(T, -1) * W[pre + "norm"] * torch.sigmoid(h @ W[pre + "g"].T)
-    return y @ W[pre + "o"].T
+    y = o.reshape(T, -1) * W[pre + "norm"] * torch.sigmoid(W.linear(h, pre + "g"))
+    return W.linear(y, pre + "o")
 
 
 # ---- feed-forward -------------------------------------------------------------------------------------------------------------------
 def dense_mlp(h, W, pre, limit):
-    return clamped_glu(h @ W[pre + "gate"].T, h @ W[pre + "up"].T, limit) @ W[pre + "down"].T
+    return W.linear(clamped_glu(W.linear(h, pre + "gate"), W.linear(h, pre + "up"), limit), pre + "down")
 
 
 # ---- layers and model ---------------------------------------------------------------------------------------------------------------
@@ -144,9 +151,9 @@ def sublayer(x, W, p, q, m, eps, shift, f):
     return spread(x, W[p + f"hc{q}.mix"], m * W[p + f"hc{q}.out"], W[p + f"ls{q}"] * f(h))
 
 
-def forward(cfg: dict, tensors: dict, tokens, dtype=torch.float64, layers_out: list | None = None):
+def forward(cfg: dict, tensors: dict, tokens, dtype=torch.float64, layers_out: list | None = None, noise: int | None = None):
     """Logits [T, vocab] of one sequence; layers_out (a list) receives the sum of the streams after every layer."""
-    W = Weights(tensors, dtype)
+    W = Weights(tensors, dtype, noise)
     eps, m = cfg["norm"]["eps"], cfg["residual_mult"]
     T = len(tokens)
     e = W["embed"][torch.as_tensor(tokens, dtype=torch.int64)] + sinusoid(T, cfg["width"]).to(dtype)
@@ -175,7 +182,7 @@ def random_tensors(cfg: dict, seed: int) -> dict:
     g = torch.Generator().manual_seed(seed)
 
     def n(*shape, std=1.0, mean=0.0):
-        return (torch.randn(*shape, generator=g) * std + mean).to(torch.bfloat16)
+        return (torch.randn(shape, generator=g) * std + mean).to(torch.bfloat16)
 
     w, V, S = cfg["width"], cfg["vocab"], cfg["streams"]
     t = {"embed": n(V, w, std=0.7), "head": n(V, w, std=w ** -0.5), "final.norm": n(std=0.1, mean=1.0)}
