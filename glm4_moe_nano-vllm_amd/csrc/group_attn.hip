@@ -9,11 +9,13 @@
 //                        split over the waves and over workgroups (glm_attn_merge adds the splits up)
 //   group_attn_plain     any head size, bf16 or fp32: one (token, head) per workgroup, vector FMAs, every step in fp32
 //
-// All of them read keys and values of the step's own tokens from the cache, where group_kv_store has put them, so a portion of a
-// prompt, a decoded token and a layer that borrows another layer's cache are the same thing.
+// Keys and values of the step's own tokens are in the cache like all others (group_kv_store), so a portion of a prompt, a decoded
+// token and a layer that borrows another layer's cache are the same thing.  The decode form may also take them from the
+// projection's rows and store them itself, which saves a decode step the launch in front.
 //
 // Roofline: MFMA for prefill, HBM for decode (the visible keys and values, read once).  S^T = K . Q^T, fp32 online softmax per lane
-// column in log2 units, O^T += V^T . P^T straight from registers.  Tiles come in by LDS-DMA, double-buffered; keys behind
+// column in log2 units (the distance bias, divided by the scale, is what the score products are added to), O^T += V^T . P^T straight from
+// registers.  Tiles come in by LDS-DMA, double-buffered; keys behind
 // the last visible one are fetched from a page of zeros (unused cache memory may hold NaNs).  The running maximum is raised only when
 // a score exceeds it by more than 2^8 (the sums stay exact: the reference point cancels).
 #include "common.h"
@@ -37,6 +39,9 @@ struct GroupArgs {
     int seq0, n_tiles, H, G, dk, dv, window, chunk, nsplit;
     float scale;
     const float *slope, *sink;  // [H] or nullptr
+    const void *knew, *vnew;    // decode: keys / values of the step's own rows, row r at r*ldkv, head g at g*dk / g*dv, or nullptr
+    int64_t ldkv;
+    const int32_t* slots;       // decode with knew: cache rows they are stored to
     void* out;            // [rows, ldo], head h at h*dv
     int64_t ldo;
     float *part_o, *part_ml;    // nsplit > 1: [rows*H][nsplit][dv], [rows*H][nsplit][2]
@@ -89,7 +94,7 @@ struct Slab {
     static constexpr int KG = KS < 4 ? KS : 4, VG = VEARLY ? VT : 4;  // fragments per request group
     u32x4_t qf[NT][KS];
     f32x4_t acc[NT][VT];
-    float m_run[NT], l_run[NT], slope2[NT];
+    float m_run[NT], l_run[NT], slope[NT];                // slope: per key, in units of the unscaled score
     int rp[NT], rlo[NT];                                  // position of the lane's row and the first one it sees; rp < 0: no row
     int any_lo[NT], any_hi[NT], full_lo[NT], full_hi[NT]; // keys that some row / every row of the tile sees
     unsigned k_rel[2], v_rel[4];
@@ -127,11 +132,15 @@ struct Slab {
                 lds_read_tr16_b64<(d >> 2) * 128 + 16 * VB>(vf[i][1], vst + v_rel[d & 3]);
             });
         };
-        f32x4_t s[NT][2];
+        f32x4_t s[NT][2];  // starts from the distance bias: the products are added to it
 #pragma unroll
-        for (int t = 0; t < NT; ++t)
+        for (int t = 0; t < NT; ++t) {
+            const float b0 = slope[t] * (float)(j0 + 4 * g - rp[t]);
 #pragma unroll
-            for (int kt = 0; kt < 2; ++kt) s[t][kt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+            for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) s[t][kt][r] = fmaf(slope[t], (float)(16 * kt + r), b0);
+        }
         static_for<(KS + KG - 1) / KG>([&](auto GI) {
             constexpr int k0 = decltype(GI)::value * KG, kn = KS - k0 < KG ? KS - k0 : KG;
             constexpr bool last = k0 + KG >= KS;
@@ -166,28 +175,22 @@ struct Slab {
                 for (int i = 0; i < 8; ++i) pf[t][i] = (__bf16)0.f;
                 continue;
             }
-            const int jl = j0 + 4 * g;
-            const float b0 = slope2[t] * (float)(jl - rp[t]);
-            float mx = -INFINITY;
-            if (j0 >= full_lo[t] && j0 + 31 <= full_hi[t]) {
-#pragma unroll
-                for (int kt = 0; kt < 2; ++kt)
-#pragma unroll
-                    for (int r = 0; r < 4; ++r) {
-                        s[t][kt][r] = fmaf(s[t][kt][r], sc, fmaf(slope2[t], (float)(16 * kt + r), b0));
-                        mx = fmaxf(mx, s[t][kt][r]);
-                    }
-            } else {
+            if (j0 < full_lo[t] || j0 + 31 > full_hi[t]) {
+                const int jl = j0 + 4 * g;
 #pragma unroll
                 for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
                     for (int r = 0; r < 4; ++r) {
                         const int j = jl + 16 * kt + r;
-                        const float v = fmaf(s[t][kt][r], sc, fmaf(slope2[t], (float)(16 * kt + r), b0));
-                        s[t][kt][r] = (j <= rp[t] && j >= rlo[t]) ? v : -INFINITY;
-                        mx = fmaxf(mx, s[t][kt][r]);
+                        if (j > rp[t] || j < rlo[t]) s[t][kt][r] = -INFINITY;
                     }
             }
+            float mx = -INFINITY;
+#pragma unroll
+            for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s[t][kt][r]);
+            mx *= sc;
             if (__any(mx > m_run[t] + 8.0f || (m_run[t] == -INFINITY && mx > -INFINITY))) {
                 mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
                 mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
@@ -203,7 +206,7 @@ struct Slab {
             for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
-                    const float p = __builtin_amdgcn_exp2f(s[t][kt][r] - m_use);
+                    const float p = __builtin_amdgcn_exp2f(fmaf(s[t][kt][r], sc, -m_use));
                     l_run[t] += p;
                     pf[t][4 * kt + r] = (__bf16)p;
                 }
@@ -256,7 +259,7 @@ __global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void group_attn_pref
     const int32_t* bt = a.bt + (int64_t)(a.seq0 + seq) * a.bt_stride;
     SL S;
     S.init(lane);
-    const float sl = a.slope ? a.slope[h] * GA_LOG2E : 0.f;
+    const float sl = a.slope ? a.slope[h] / a.scale : 0.f;
     // this wave's rows: tile t holds rows qo + 64 t + 16 w + c (the two half-dead tiles of the causal edge cost all waves the same)
 #pragma unroll
     for (int t = 0; t < 2; ++t) {
@@ -264,7 +267,7 @@ __global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void group_attn_pref
         const bool some = r0 < nq;
         S.rp[t] = r < nq ? p0 - qo + r : -1;
         S.rlo[t] = r < nq ? ga_first(a, S.rp[t]) : 0;
-        S.slope2[t] = sl;
+        S.slope[t] = sl;
         const int a0 = p0 - qo + r0, a1 = p0 - qo + min(r0 + 15, nq - 1);
         S.any_lo[t] = some ? ga_first(a, a0) : 1 << 30;
         S.any_hi[t] = some ? a1 : -1;
@@ -383,7 +386,7 @@ __global__ __launch_bounds__(NW * 64, 1) void group_attn_decode_kernel(const Gro
     S.init(lane);
     S.rp[0] = row_ok && pA >= 0 ? pA + tok : -1;
     S.rlo[0] = S.rp[0] >= 0 ? ga_first(a, S.rp[0]) : 0;
-    S.slope2[0] = a.slope && row_ok ? a.slope[h] * GA_LOG2E : 0.f;
+    S.slope[0] = a.slope && row_ok ? a.slope[h] / a.scale : 0.f;
     {
         const int t0 = rg * 16 / R, t1 = min((rg * 16 + 15) / R, ntok - 1);
         S.any_lo[0] = ga_first(a, max(pA, 0) + t0);
@@ -401,6 +404,20 @@ __global__ __launch_bounds__(NW * 64, 1) void group_attn_decode_kernel(const Gro
 #pragma unroll
     for (int i = 0; i < KS; ++i) asm volatile("" : "+v"(S.qf[0][i]));
     const int32_t* bt = a.bt + (int64_t)(a.seq0 + a.seq_of[tok0]) * a.bt_stride;
+    // keys of this step come straight from the projection's rows: positions from `own` on (the portion's first).  The tile's own tokens
+    // are put into the cache here, by the first of the workgroups that share them
+    const int own = a.knew ? pA - (tok0 - a.q_start[a.seq_of[tok0]]) : 1 << 30;
+    if (a.knew && split == 0 && rg == 0 && pA >= 0) {
+        const int ku = a.dk / 8, per_tok = ku + a.dv / 8;
+        for (int i = tid; i < ntok * per_tok; i += NW * 64) {
+            const int t = i / per_tok, u = i - t * per_tok;
+            const int64_t r = tok0 + t, slot = a.slots[r];
+            if (slot < 0 || slot >= a.n_blocks * a.bs) continue;
+            const int64_t dst = (slot / a.bs * a.G + kvh) * a.bs + slot % a.bs;
+            if (u < ku) reinterpret_cast<u32x4_t*>(const_cast<void*>(a.kc))[dst * ku + u] = *reinterpret_cast<const u32x4_t*>(reinterpret_cast<const bf16_t*>(a.knew) + r * a.ldkv + kvh * a.dk + u * 8);
+            else reinterpret_cast<u32x4_t*>(const_cast<void*>(a.vc))[dst * (per_tok - ku) + u - ku] = *reinterpret_cast<const u32x4_t*>(reinterpret_cast<const bf16_t*>(a.vnew) + r * a.ldkv + kvh * a.dv + (u - ku) * 8);
+        }
+    }
     char* mine = smem + w * 2 * STAGE;
     const unsigned base = lds_addr(mine);
     unsigned koff[KDMA], voff[VDMA];
@@ -431,15 +448,24 @@ __global__ __launch_bounds__(NW * 64, 1) void group_attn_decode_kernel(const Gro
         const bf16_t* kb = reinterpret_cast<const bf16_t*>(a.kc) + row * a.dk;
         const bf16_t* vb = reinterpret_cast<const bf16_t*>(a.vc) + row * a.dv;
         char* st = mine + (k & 1) * STAGE;
+        if (j0 + 31 < own) {
+#pragma unroll
+            for (int i = 0; i < KDMA; ++i) lds_dma16<2>((kpad[i] || krow[i] >= left) ? (const void*)ga_zero_page : (const void*)(kb + koff[i]), st + i * 1024);
+#pragma unroll
+            for (int i = 0; i < VDMA; ++i) lds_dma16<2>((vpad[i] || vrow[i] >= left) ? (const void*)ga_zero_page : (const void*)(vb + voff[i]), st + KSLAB + i * 1024);
+            return;
+        }
+        const bf16_t* kn = reinterpret_cast<const bf16_t*>(a.knew) + (int64_t)(tok0 + j0 - pA) * a.ldkv + kvh * a.dk;
+        const bf16_t* vn = reinterpret_cast<const bf16_t*>(a.vnew) + (int64_t)(tok0 + j0 - pA) * a.ldkv + kvh * a.dv;
 #pragma unroll
         for (int i = 0; i < KDMA; ++i) {
-            const void* s = (kpad[i] || krow[i] >= left) ? (const void*)ga_zero_page : (const void*)(kb + koff[i]);
-            lds_dma16<2>(s, st + i * 1024);
+            const bf16_t* s = j0 + krow[i] >= own ? kn + krow[i] * a.ldkv + ((int)koff[i] - krow[i] * a.dk) : kb + koff[i];
+            lds_dma16((kpad[i] || krow[i] >= left) ? (const void*)ga_zero_page : (const void*)s, st + i * 1024);
         }
 #pragma unroll
         for (int i = 0; i < VDMA; ++i) {
-            const void* s = (vpad[i] || vrow[i] >= left) ? (const void*)ga_zero_page : (const void*)(vb + voff[i]);
-            lds_dma16<2>(s, st + KSLAB + i * 1024);
+            const bf16_t* s = j0 + vrow[i] >= own ? vn + vrow[i] * a.ldkv + ((int)voff[i] - vrow[i] * a.dv) : vb + voff[i];
+            lds_dma16((vpad[i] || vrow[i] >= left) ? (const void*)ga_zero_page : (const void*)s, st + KSLAB + i * 1024);
         }
     };
     const float sc = a.scale * GA_LOG2E;
@@ -680,7 +706,7 @@ extern "C" int glm_group_attn_prefill(const void* q, int64_t ldq, const void* kc
     const int rc = group_args(a, "glm_group_attn_prefill", q, ldq, kc, vc, n_blocks, bs, block_tables, bt_stride, seq0, H, G, dk, dv, window, chunk, scale, slope, sink, out, ldo);
     if (rc != GLM_OK) return rc;
     GLM_CHECK_ARG(q_start && pos && tile_seq && tile_off && n_tiles >= 0, GLM_ERR_INVALID, "glm_group_attn_prefill: no tiles");
-    GLM_CHECK_ARG(dk <= 256 && dv <= 256, GLM_ERR_UNSUPPORTED, "glm_group_attn_prefill: head sizes up to 256 (dk=%d dv=%d)", dk, dv);
+    GLM_CHECK_ARG(dk <= 256 && dv <= 256 && scale > 0.f, GLM_ERR_UNSUPPORTED, "glm_group_attn_prefill: head sizes up to 256, a positive scale (dk=%d dv=%d)", dk, dv);
     if (n_tiles == 0) return GLM_OK;
     a.q_start = q_start; a.pos = pos; a.tile_a = tile_seq; a.tile_b = tile_off; a.n_tiles = n_tiles;
     return run_prefill(a, glm_s(stream));
@@ -688,15 +714,18 @@ extern "C" int glm_group_attn_prefill(const void* q, int64_t ldq, const void* kc
 
 extern "C" int glm_group_attn_decode(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs, const int32_t* block_tables, int64_t bt_stride,
                                      const int32_t* pos, const int32_t* seq_of, const int32_t* tile_tok, const int32_t* tile_n, int n_tiles, int tokens_per_tile, int H, int G, int dk, int dv,
-                                     int window, int chunk, float scale, const float* slope, const float* sink, void* out, int64_t ldo, int nsplit, float* part_o, float* part_ml,
-                                     glm_stream_t stream) {
+                                     int window, int chunk, float scale, const float* slope, const float* sink, const void* knew, const void* vnew, int64_t ldkv, const int32_t* q_start,
+                                     const int32_t* slots, void* out, int64_t ldo, int nsplit, float* part_o, float* part_ml, glm_stream_t stream) {
     GroupArgs a;
     const int rc = group_args(a, "glm_group_attn_decode", q, ldq, kc, vc, n_blocks, bs, block_tables, bt_stride, 0, H, G, dk, dv, window, chunk, scale, slope, sink, out, ldo);
     if (rc != GLM_OK) return rc;
     GLM_CHECK_ARG(pos && seq_of && tile_tok && tile_n && n_tiles >= 0 && tokens_per_tile >= 1 && nsplit >= 1 && nsplit <= 64 && (nsplit == 1 || (part_o && part_ml)), GLM_ERR_INVALID,
                   "glm_group_attn_decode: bad tiles or splits (%d)", nsplit);
-    GLM_CHECK_ARG(dk <= 256 && dv <= 256, GLM_ERR_UNSUPPORTED, "glm_group_attn_decode: head sizes up to 256 (dk=%d dv=%d)", dk, dv);
+    GLM_CHECK_ARG(dk <= 256 && dv <= 256 && scale > 0.f, GLM_ERR_UNSUPPORTED, "glm_group_attn_decode: head sizes up to 256, a positive scale (dk=%d dv=%d)", dk, dv);
+    GLM_CHECK_ARG(!knew || (vnew && q_start && slots && ldkv >= (int64_t)G * (dk > dv ? dk : dv) && ldkv % 8 == 0 && glm_aligned16(knew) && glm_aligned16(vnew)), GLM_ERR_INVALID,
+                  "glm_group_attn_decode: bad rows of new keys and values (ldkv=%ld)", (long)ldkv);
     if (n_tiles == 0) return GLM_OK;
+    a.knew = knew; a.vnew = vnew; a.ldkv = ldkv; a.q_start = q_start; a.slots = slots;
     a.pos = pos; a.seq_of = seq_of; a.tile_a = tile_tok; a.tile_b = tile_n; a.n_tiles = n_tiles; a.nsplit = nsplit; a.part_o = part_o; a.part_ml = part_ml;
     return run_decode(a, (tokens_per_tile * (H / G) + 15) / 16, glm_s(stream));
 }

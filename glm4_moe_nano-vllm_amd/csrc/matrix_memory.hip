@@ -11,6 +11,7 @@
 //
 //   memory_recurrent   token by token, state in registers (decoded tokens, short portions, fp32): one (sequence, head) per workgroup, gate
 //                      projections and the output norm included; memory_recurrent_any for head sizes beyond its registers
+//   memory_gates       gate projections of long portions and the part of the gates' scan that stays inside a chunk of 64 tokens
 //   memory_chunkwise   long portions: 64 tokens at a time on the matrix cores, one (sequence, head, 64 value columns) per workgroup
 //   memory_output      norm and output gate of memory_chunkwise's rows
 //
@@ -301,23 +302,125 @@ __global__ __launch_bounds__(256) void memory_recurrent_any_kernel(const RecArgs
 }
 
 // ---------------------------------------------------------------------------------------------------------------------------
+// Gates of long portions, 64 tokens of a portion and up to 16 heads per workgroup: the two projections on the matrix cores (the four
+// waves share K), then everything of a chunk that does not depend on the chunks before it.
+struct GateArgs {
+    const bf16_t* hrow;   // [rows, ldh]
+    int64_t ldh;
+    const bf16_t* wif;    // [2 H, ldw] rows i then f
+    int64_t ldw;
+    int wk;
+    const float* bif;     // [2 H]
+    float* gates;         // [3][H][rows], log2 units: i_s - b_s; b_s, the sum of f from the chunk's first token; running maximum of the first
+    int64_t rows;
+    const int32_t *q_start, *tile_seq, *tile_off;  // 128-row tiles
+    int H;
+    float cap;
+};
+__global__ __launch_bounds__(256) void memory_gates_kernel(const GateArgs a) {
+    __shared__ float s_z[4][32][64];
+    const int tid = threadIdx.x, lane = tid & 63, w = tid >> 6, c = lane & 15, g = lane >> 4;
+    const int tile = blockIdx.x >> 1, seq = a.tile_seq[tile], h0 = blockIdx.y * 16;
+    const int qs = a.q_start[seq], T = a.q_start[seq + 1] - qs, off = a.tile_off[tile] + (blockIdx.x & 1) * 64;
+    if (off >= T) return;
+    const int n = min(64, T - off);
+    f32x4_t acc[2][4];
+#pragma unroll
+    for (int m = 0; m < 2; ++m)
+#pragma unroll
+        for (int t = 0; t < 4; ++t) acc[m][t] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+    const int wrow = min(h0 + c, a.H - 1);  // (heads behind the last one: computed again, not used)
+    const bf16_t* wp[2] = {a.wif + (int64_t)wrow * a.ldw, a.wif + (int64_t)(a.H + wrow) * a.ldw};
+    const bf16_t* hp[4];
+#pragma unroll
+    for (int t = 0; t < 4; ++t) hp[t] = a.hrow + (int64_t)(qs + off + min(16 * t + c, n - 1)) * a.ldh;
+    const u32x4_t zero = {0, 0, 0, 0};
+#pragma unroll 4
+    for (int k = w * 32 + 8 * g; k - 8 * g < a.wk; k += 128) {
+        const bool on = k < a.wk;
+        u32x4_t x[4], y[2];
+#pragma unroll
+        for (int m = 0; m < 2; ++m) y[m] = on ? *reinterpret_cast<const u32x4_t*>(wp[m] + k) : zero;
+#pragma unroll
+        for (int t = 0; t < 4; ++t) x[t] = on ? *reinterpret_cast<const u32x4_t*>(hp[t] + k) : zero;
+#pragma unroll
+        for (int m = 0; m < 2; ++m)
+#pragma unroll
+            for (int t = 0; t < 4; ++t)
+                acc[m][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, y[m]), __builtin_bit_cast(bf16x8_t, x[t]), acc[m][t], 0, 0, 0);
+    }
+#pragma unroll
+    for (int m = 0; m < 2; ++m)
+#pragma unroll
+        for (int t = 0; t < 4; ++t)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) s_z[w][16 * m + 4 * g + r][16 * t + c] = acc[m][t][r];
+    __syncthreads();
+    for (int hh = w; hh < 16 && h0 + hh < a.H; hh += 4) {
+        const int h = h0 + hh;
+        float zi = a.bif[h], zf = a.bif[a.H + h];
+#pragma unroll
+        for (int x = 0; x < 4; ++x) {
+            zi += s_z[x][hh][lane];
+            zf += s_z[x][16 + hh][lane];
+        }
+        float b = mm_log_sigmoid(mm_cap(zf, a.cap));
+#pragma unroll
+        for (int o = 1; o < 64; o <<= 1) {
+            const float v = __shfl_up(b, o, 64);
+            if (lane >= o) b += v;
+        }
+        const float as = mm_cap(zi, a.cap) - b;
+        float mx = as;
+#pragma unroll
+        for (int o = 1; o < 64; o <<= 1) {
+            const float v = __shfl_up(mx, o, 64);
+            if (lane >= o) mx = fmaxf(mx, v);
+        }
+        if (lane < n) {
+            float* o = a.gates + (int64_t)h * a.rows + qs + off + lane;
+            const int64_t part = (int64_t)a.H * a.rows;
+            o[0] = as * MM_LOG2E;
+            o[part] = b * MM_LOG2E;
+            o[2 * part] = mx * MM_LOG2E;
+        }
+    }
+}
+
 struct ChunkArgs {
     const bf16_t* x;      // projection rows (see RecArgs)
     int64_t ldx, k_off, v_off;
-    const float* gates;   // [rows, ldg] a at h, b at H + h, biases included
-    int64_t ldg;
+    const float* gates;   // [3][H][rows] of memory_gates
+    int64_t rows;
     bf16_t* o;            // [rows, ldo] head h at h*vdimp, before the norm
     int64_t ldo;
     float *S, *n, *m;
     int64_t n_state;
     const int32_t *pos, *q_start, *state_in, *state_out;  // of the long portions; q_start and pos relative to x's first row
     int H, dim, dimp, vdimp, vtiles;
-    float cap;
 };
 
-template <int OFF>
-__device__ __forceinline__ void lds_read_b64(u32x2_t& dst, unsigned addr) {
-    asm volatile("ds_read_b64 %0, %1 offset:%2" : "=v"(dst) : "v"(addr), "i"(OFF));
+template <typename T>
+__device__ __forceinline__ T mm_lds(const char* p) { return *reinterpret_cast<const T*>(p); }
+// four transposed reads, complete when they return: the compiler would drain the LDS-DMA that is in flight in front of its own
+template <int O0, int O1, int O2, int O3>
+__device__ __forceinline__ void mm_lds_tr4(u32x2_t (&d)[2][2], const char* p) {
+    asm volatile("ds_read_b64_tr_b16 %0, %4 offset:%5\n\tds_read_b64_tr_b16 %1, %4 offset:%6\n\tds_read_b64_tr_b16 %2, %4 offset:%7\n\t"
+                 "ds_read_b64_tr_b16 %3, %4 offset:%8\n\ts_waitcnt lgkmcnt(0)"
+                 : "=&v"(d[0][0]), "=&v"(d[0][1]), "=&v"(d[1][0]), "=&v"(d[1][1]) : "v"(lds_addr(p)), "i"(O0), "i"(O1), "i"(O2), "i"(O3) : "memory");
+}
+// sixteen of them: rows 0, 16, 32, 48 (pitch RB) at four addresses
+template <int RB>
+__device__ __forceinline__ void mm_lds_tr16(u32x2_t (&d)[4][2][2], unsigned p0, unsigned p1, unsigned p2, unsigned p3) {
+#define MM_TR(D, P, O) "ds_read_b64_tr_b16 " D ", " P " offset:" O "\n\t"
+    asm volatile(MM_TR("%0", "%16", "%20") MM_TR("%1", "%16", "%21") MM_TR("%2", "%16", "%22") MM_TR("%3", "%16", "%23")
+                 MM_TR("%4", "%17", "%20") MM_TR("%5", "%17", "%21") MM_TR("%6", "%17", "%22") MM_TR("%7", "%17", "%23")
+                 MM_TR("%8", "%18", "%20") MM_TR("%9", "%18", "%21") MM_TR("%10", "%18", "%22") MM_TR("%11", "%18", "%23")
+                 MM_TR("%12", "%19", "%20") MM_TR("%13", "%19", "%21") MM_TR("%14", "%19", "%22") MM_TR("%15", "%19", "%23") "s_waitcnt lgkmcnt(0)"
+                 : "=&v"(d[0][0][0]), "=&v"(d[0][0][1]), "=&v"(d[0][1][0]), "=&v"(d[0][1][1]), "=&v"(d[1][0][0]), "=&v"(d[1][0][1]), "=&v"(d[1][1][0]), "=&v"(d[1][1][1]),
+                   "=&v"(d[2][0][0]), "=&v"(d[2][0][1]), "=&v"(d[2][1][0]), "=&v"(d[2][1][1]), "=&v"(d[3][0][0]), "=&v"(d[3][0][1]), "=&v"(d[3][1][0]), "=&v"(d[3][1][1])
+                 : "v"(p0), "v"(p1), "v"(p2), "v"(p3), "i"(0), "i"(16 * RB), "i"(32 * RB), "i"(48 * RB) : "memory");
+#undef MM_TR
 }
 // v = hi + lo, two bf16 each
 __device__ __forceinline__ void mm_split(const float (&v)[8], bf16x8_t& hi, bf16x8_t& lo) {
@@ -328,6 +431,14 @@ __device__ __forceinline__ void mm_split(const float (&v)[8], bf16x8_t& hi, bf16
         lo[e] = (__bf16)(v[e] - (float)b);
     }
 }
+// barrier that leaves LDS-DMA in flight
+__device__ __forceinline__ void mm_barrier() {
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");
+    __builtin_amdgcn_s_barrier();
+    asm volatile("" ::: "memory");
+}
+__device__ __forceinline__ bf16x8_t mm_frag(const u32x2_t& x, const u32x2_t& y) { return __builtin_bit_cast(bf16x8_t, u32x4_t{x[0], x[1], y[0], y[1]}); }
+__device__ __forceinline__ f32x4_t mm_f4(const u32x4_t& v) { return __builtin_bit_cast(f32x4_t, v); }
 __device__ __forceinline__ f32x4_t mm_mfma(const bf16x8_t& x, const bf16x8_t& y, const f32x4_t& z) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(x, y, z, 0, 0, 0); }
 
 // D: multiple of 64, dimp <= D <= 256.  Four waves; wave w computes the scores of query rows 16 w .. + 15 and owns value columns
@@ -378,8 +489,8 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
     const float scale = 1.0f / sqrtf((float)a.dim);
     const bf16_t* xq = a.x + (int64_t)r0 * a.ldx + (int64_t)h * a.dimp;
     const bf16_t* xv = a.x + (int64_t)r0 * a.ldx + a.v_off + (int64_t)h * a.vdimp + vt * 64;
-    const float* gp = a.gates + (int64_t)r0 * a.ldg + h;
-    const unsigned base = lds_addr(smem);
+    const float* gp = a.gates + (int64_t)h * a.rows + r0;
+    const int64_t gpart = (int64_t)a.H * a.rows;
     auto issue = [&](int ch) {
         char* st = smem + (ch & 1) * STAGE;
         const int left = T - ch * 64;
@@ -411,98 +522,110 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
 #pragma unroll
     for (int e = 0; e < 4; ++e) tr_rel[e] = tr * RB + (((2 * e + (pp >> 1)) ^ attn_swz(tr)) << 4) + ((pp & 1) << 3);
     vt_rel = tr * 128 + (((2 * w + (pp >> 1)) ^ attn_swz(tr)) << 4) + ((pp & 1) << 3);
-    float za = lane < T ? gp[(int64_t)lane * a.ldg] : 0.f, zb = lane < T ? gp[(int64_t)lane * a.ldg + a.H] : 0.f;
+    // gates of the chunk, one token per lane, the same in every wave
+    float ga, gb, gm;
+    auto load_gates = [&](int ch) {
+        const int64_t t = (int64_t)ch * 64 + lane;
+        const bool on = t < T;
+        ga = on ? gp[t] : -INFINITY;
+        gb = on ? gp[gpart + t] : 0.f;
+        gm = on ? gp[2 * gpart + t] : 0.f;
+    };
+    m_in *= MM_LOG2E;
+    load_gates(0);
     issue(0);
+    const char* sa = smem + SMALL;
     for (int ch = 0; ch < n_chunks; ++ch) {
         const int left = T - ch * 64;
-        // ---- gates of the chunk, one token per lane, the same in every wave ----
-        const bool tok = lane < left;
-        const float li = tok ? mm_cap(za, a.cap) : -INFINITY, lf = tok ? mm_log_sigmoid(mm_cap(zb, a.cap)) : 0.f;
-        float b = lf;
-#pragma unroll
-        for (int o = 1; o < 64; o <<= 1) {
-            const float v = __shfl_up(b, o, 64);
-            if (lane >= o) b += v;
-        }
-        const float as = li - b;
-        float mx = as;
-#pragma unroll
-        for (int o = 1; o < 64; o <<= 1) {
-            const float v = __shfl_up(mx, o, 64);
-            if (lane >= o) mx = fmaxf(mx, v);
-        }
-        const float mt = b + fmaxf(m_in, mx);
-        const float bL = __shfl(b, 63, 64), mL = __shfl(mt, 63, 64);
-        const float carry = __builtin_amdgcn_exp2f((bL + m_in - mL) * MM_LOG2E);
         wait_vm<0>();
-        __syncthreads();  // the chunk's rows are in; every wave is past its reads of the chunk before
-        if (ch + 1 < n_chunks) {
-            issue(ch + 1);
-            const int64_t t = (int64_t)(ch + 1) * 64 + lane;
-            za = t < T ? gp[t * a.ldg] : 0.f;
-            zb = t < T ? gp[t * a.ldg + a.H] : 0.f;
-        }
+        const float mt = gb + fmaxf(m_in, gm);
+        const int last = min(left, 64) - 1;
+        const float bL = __shfl(gb, last, 64), mL = __shfl(mt, last, 64);
+        const float carry = __builtin_amdgcn_exp2f(bL + m_in - mL);
+        mm_barrier();  // the chunk's rows are in; every wave is past its reads of the chunk before
         if (w == 0) {
-            s_a[lane] = as * MM_LOG2E;
-            s_row[lane] = (b - mt) * MM_LOG2E;
-            s_in[lane] = __builtin_amdgcn_exp2f((b + m_in - mt) * MM_LOG2E) * scale;
-            s_floor[lane] = __builtin_amdgcn_exp2f(-mt * MM_LOG2E);
-            s_w[lane] = __builtin_amdgcn_exp2f((bL - mL + as) * MM_LOG2E);
+            s_a[lane] = ga;
+            s_row[lane] = gb - mt;
+            s_in[lane] = __builtin_amdgcn_exp2f(gb + m_in - mt) * scale;
+            s_floor[lane] = __builtin_amdgcn_exp2f(-mt);
+            s_w[lane] = __builtin_amdgcn_exp2f(bL - mL + ga);
         }
-        const unsigned qst = base + (ch & 1) * STAGE, kst = qst + QT, vst = kst + QT, pst = PALIAS ? qst : base + POFF;
-        char* pw = smem + (PALIAS ? (ch & 1) * STAGE : POFF);
-        // ---- scores of this wave's 16 query rows, and n . q of them ----
+        if (ch + 1 < n_chunks) {
+            load_gates(ch + 1);
+            issue(ch + 1);
+        }
+        const char *qst = smem + (ch & 1) * STAGE, *kst = qst + QT, *vst = kst + QT;
+        char* pst = smem + (PALIAS ? (ch & 1) * STAGE : POFF);
+        // ---- scores of this wave's 16 query rows, and n . q of them; the readout's query fragments are on their way meanwhile ----
         f32x4_t s[4];
 #pragma unroll
         for (int kt = 0; kt < 4; ++kt) s[kt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
         float nq = 0.f;
-        static_for<KS>([&](auto I) {
-            constexpr int i = decltype(I)::value;
-            u32x4_t qf, kf[4];
-            lds_read_b128<(i >> 1) * 128>(qf, qst + w * 16 * RB + row_rel[i & 1]);
-            static_for<4>([&](auto KT) { lds_read_b128<(i >> 1) * 128 + decltype(KT)::value * 16 * RB>(kf[decltype(KT)::value], kst + row_rel[i & 1]); });
-            wait_lds();
-            asm volatile("" : "+v"(qf), "+v"(kf[0]), "+v"(kf[1]), "+v"(kf[2]), "+v"(kf[3]));
-#pragma unroll
-            for (int kt = 0; kt < 4; ++kt) s[kt] = mm_mfma(__builtin_bit_cast(bf16x8_t, kf[kt]), __builtin_bit_cast(bf16x8_t, qf), s[kt]);
-            const f32x4_t n0 = *reinterpret_cast<const f32x4_t*>(s_n + 32 * i + 8 * g), n1 = *reinterpret_cast<const f32x4_t*>(s_n + 32 * i + 8 * g + 4);
-#pragma unroll
-            for (int e = 0; e < 2; ++e) {
-                nq = fmaf(bflo(qf[e]), n0[2 * e], nq);
-                nq = fmaf(bfhi(qf[e]), n0[2 * e + 1], nq);
-                nq = fmaf(bflo(qf[2 + e]), n1[2 * e], nq);
-                nq = fmaf(bfhi(qf[2 + e]), n1[2 * e + 1], nq);
-            }
-        });
-        // ---- what the state gives all 64 rows, in this wave's columns ----
         f32x4_t acc[4];
 #pragma unroll
         for (int rt = 0; rt < 4; ++rt) acc[rt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-        static_for<KS>([&](auto I) {
-            constexpr int i = decltype(I)::value;
-            u32x2_t qh[4][2];
-            static_for<4>([&](auto RT) {
-                constexpr int rt = decltype(RT)::value;
-                lds_read_b64<(i >> 1) * 128 + rt * 16 * RB>(qh[rt][0], qst + half_rel[i & 1][0]);
-                lds_read_b64<(i >> 1) * 128 + rt * 16 * RB>(qh[rt][1], qst + half_rel[i & 1][1]);
+        static_for<KS / 2>([&](auto I2) {
+            constexpr int i0 = 2 * decltype(I2)::value;
+            u32x4_t qf[2], kf[2][4], nf[2][2];
+            u32x2_t qh[2][4][2];
+            static_for<2>([&](auto J) {
+                constexpr int jj = decltype(J)::value, i = i0 + jj;
+                qf[jj] = mm_lds<u32x4_t>(qst + w * 16 * RB + row_rel[i & 1] + ((i >> 1) * 128));
+                static_for<4>([&](auto KT) { kf[jj][decltype(KT)::value] = mm_lds<u32x4_t>(kst + row_rel[i & 1] + ((i >> 1) * 128 + decltype(KT)::value * 16 * RB)); });
+                nf[jj][0] = mm_lds<u32x4_t>(sa + 32 * g + (1536 + 128 * i));
+                nf[jj][1] = mm_lds<u32x4_t>(sa + 32 * g + (1536 + 128 * i + 16));
             });
-            const float sv[8] = {S[2 * i][0], S[2 * i][1], S[2 * i][2], S[2 * i][3], S[2 * i + 1][0], S[2 * i + 1][1], S[2 * i + 1][2], S[2 * i + 1][3]};
-            bf16x8_t hi, lo;
-            mm_split(sv, hi, lo);
-            wait_lds();
+            static_for<2>([&](auto J) {
+                constexpr int jj = decltype(J)::value, i = i0 + jj;
+                static_for<4>([&](auto RT) {
+                    constexpr int rt = decltype(RT)::value;
+                    qh[jj][rt][0] = mm_lds<u32x2_t>(qst + half_rel[i & 1][0] + ((i >> 1) * 128 + rt * 16 * RB));
+                    qh[jj][rt][1] = mm_lds<u32x2_t>(qst + half_rel[i & 1][1] + ((i >> 1) * 128 + rt * 16 * RB));
+                });
+            });
+            bf16x8_t hi[2], lo[2];
 #pragma unroll
-            for (int rt = 0; rt < 4; ++rt) asm volatile("" : "+v"(qh[rt][0]), "+v"(qh[rt][1]));
-#pragma unroll
-            for (int rt = 0; rt < 4; ++rt) {
-                const bf16x8_t q = __builtin_bit_cast(bf16x8_t, u32x4_t{qh[rt][0][0], qh[rt][0][1], qh[rt][1][0], qh[rt][1][1]});
-                acc[rt] = mm_mfma(hi, q, acc[rt]);
-                acc[rt] = mm_mfma(lo, q, acc[rt]);
+            for (int jj = 0; jj < 2; ++jj) {
+                const f32x4_t &u = S[2 * (i0 + jj)], &v = S[2 * (i0 + jj) + 1];
+                const float sv[8] = {u[0], u[1], u[2], u[3], v[0], v[1], v[2], v[3]};
+                mm_split(sv, hi[jj], lo[jj]);
             }
+#pragma unroll
+            for (int jj = 0; jj < 2; ++jj)
+#pragma unroll
+                for (int kt = 0; kt < 4; ++kt) s[kt] = mm_mfma(__builtin_bit_cast(bf16x8_t, kf[jj][kt]), __builtin_bit_cast(bf16x8_t, qf[jj]), s[kt]);
+#pragma unroll
+            for (int jj = 0; jj < 2; ++jj) {
+                const f32x4_t n0 = mm_f4(nf[jj][0]), n1 = mm_f4(nf[jj][1]);
+#pragma unroll
+                for (int e = 0; e < 2; ++e) {
+                    nq = fmaf(bflo(qf[jj][e]), n0[2 * e], nq);
+                    nq = fmaf(bfhi(qf[jj][e]), n0[2 * e + 1], nq);
+                    nq = fmaf(bflo(qf[jj][2 + e]), n1[2 * e], nq);
+                    nq = fmaf(bfhi(qf[jj][2 + e]), n1[2 * e + 1], nq);
+                }
+            }
+            // ---- what the state gives all 64 rows, in this wave's columns ----
+#pragma unroll
+            for (int jj = 0; jj < 2; ++jj)
+#pragma unroll
+                for (int x = 0; x < 2; ++x)
+#pragma unroll
+                    for (int rt = 0; rt < 4; ++rt) acc[rt] = mm_mfma(x ? lo[jj] : hi[jj], mm_frag(qh[jj][rt][0], qh[jj][rt][1]), acc[rt]);
         });
-        __syncthreads();  // query rows read, gate arrays written
+        // ---- operands of the state's update: values and keys over tokens ----
+        u32x2_t vf[2][2];
+        mm_lds_tr4<0, 16 * 128, 32 * 128, 48 * 128>(vf, vst + vt_rel);
+        mm_barrier();  // query rows read, gate arrays written
+        const bf16x8_t vv[2] = {mm_frag(vf[0][0], vf[0][1]), mm_frag(vf[1][0], vf[1][1])};
         // ---- weights of this wave's rows: hi and lo, in the order the second product reads them ----
         const int row = 16 * w + c;
-        const float rowc = s_row[row];
+        u32x4_t av[4], wq[4];
+        static_for<4>([&](auto X) { av[decltype(X)::value] = mm_lds<u32x4_t>(sa + 16 * g + (decltype(X)::value * 64)); });
+        static_for<4>([&](auto X) { wq[decltype(X)::value] = mm_lds<u32x4_t>(sa + 16 * g + (1024 + decltype(X)::value * 64)); });
+        float rowc, inc;
+        rowc = mm_lds<float>(sa + 4 * row + (256));
+        inc = mm_lds<float>(sa + 4 * row + (512));
         float dsum = 0.f;
 #pragma unroll
         for (int sl = 0; sl < 2; ++sl) {
@@ -510,109 +633,105 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
 #pragma unroll
             for (int u = 0; u < 2; ++u) {
                 const int k0 = 32 * sl + 16 * u + 4 * g;
-                const f32x4_t av = *reinterpret_cast<const f32x4_t*>(s_a + k0);
+                const f32x4_t ax = mm_f4(av[2 * sl + u]);
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
-                    const float dw = k0 + r <= row ? __builtin_amdgcn_exp2f(rowc + av[r]) : 0.f;
-                    p[4 * u + r] = s[2 * sl + u][r] * scale * dw;
+                    const float dw = k0 + r <= row ? __builtin_amdgcn_exp2f(rowc + ax[r]) * scale : 0.f;
+                    p[4 * u + r] = s[2 * sl + u][r] * dw;
                     dsum += p[4 * u + r];
                 }
             }
             bf16x8_t hi, lo;
             mm_split(p, hi, lo);
             const int chunk = ((4 * sl + g) ^ (c & 7)) << 4;
-            *reinterpret_cast<bf16x8_t*>(pw + row * 128 + chunk) = hi;
-            *reinterpret_cast<bf16x8_t*>(pw + 8192 + row * 128 + chunk) = lo;
+            *reinterpret_cast<bf16x8_t*>(pst + row * 128 + chunk) = hi;
+            *reinterpret_cast<bf16x8_t*>(pst + 8192 + row * 128 + chunk) = lo;
         }
-        nq = fmaf(nq, s_in[row], dsum);
+        nq = fmaf(nq, inc, dsum);
         nq += __shfl_xor(nq, 16, 64);
         nq += __shfl_xor(nq, 32, 64);
         if (g == 0) s_den[row] = nq;
-        __syncthreads();
-        // ---- output rows ----
-        u32x2_t vf[2][2];
-        lds_read_tr16_b64<0>(vf[0][0], vst + vt_rel);
-        lds_read_tr16_b64<16 * 128>(vf[0][1], vst + vt_rel);
-        lds_read_tr16_b64<32 * 128>(vf[1][0], vst + vt_rel);
-        lds_read_tr16_b64<48 * 128>(vf[1][1], vst + vt_rel);
-        wait_lds();
-#pragma unroll
-        for (int sl = 0; sl < 2; ++sl) asm volatile("" : "+v"(vf[sl][0]), "+v"(vf[sl][1]));
-        bf16x8_t vv[2];
-#pragma unroll
-        for (int sl = 0; sl < 2; ++sl) vv[sl] = __builtin_bit_cast(bf16x8_t, u32x4_t{vf[sl][0][0], vf[sl][0][1], vf[sl][1][0], vf[sl][1][1]});
-        static_for<4>([&](auto RT) {
-            constexpr int rt = decltype(RT)::value;
-            const int t = 16 * rt + c;
-            u32x4_t pf[2][2];
-            const unsigned pa0 = pst + c * 128 + ((g ^ (c & 7)) << 4), pa1 = pst + c * 128 + (((4 + g) ^ (c & 7)) << 4);
-            lds_read_b128<rt * 2048>(pf[0][0], pa0);
-            lds_read_b128<rt * 2048 + 8192>(pf[0][1], pa0);
-            lds_read_b128<rt * 2048>(pf[1][0], pa1);
-            lds_read_b128<rt * 2048 + 8192>(pf[1][1], pa1);
-            const float in = s_in[t], den = fmaxf(fabsf(s_den[t]), s_floor[t]) + 1e-6f;
-            f32x4_t o = acc[rt];
-#pragma unroll
-            for (int r = 0; r < 4; ++r) o[r] *= in;
-            wait_lds();
-#pragma unroll
-            for (int sl = 0; sl < 2; ++sl) asm volatile("" : "+v"(pf[sl][0]), "+v"(pf[sl][1]));
-#pragma unroll
-            for (int sl = 0; sl < 2; ++sl) {
-                if (sl == 1 && rt < 2) continue;  // keys 32 .. 63 of rows 0 .. 31: all in the future
-                o = mm_mfma(vv[sl], __builtin_bit_cast(bf16x8_t, pf[sl][0]), o);
-                o = mm_mfma(vv[sl], __builtin_bit_cast(bf16x8_t, pf[sl][1]), o);
-            }
-            const int vc = vt * 64 + 16 * w + 4 * g;
-            const float inv = 1.0f / den;
-            if (t < left && vc < a.vdimp)
-                *reinterpret_cast<u32x2_t*>(a.o + (int64_t)(r0 + ch * 64 + t) * a.ldo + (int64_t)h * a.vdimp + vc) =
-                    u32x2_t{pack2bf(o[0] * inv, o[1] * inv), pack2bf(o[2] * inv, o[3] * inv)};
-        });
         // ---- state of the next chunk ----
         bf16x8_t vhi[2], vlo[2];
         float wt[2][8];
 #pragma unroll
         for (int sl = 0; sl < 2; ++sl) {
-            const f32x4_t w0 = *reinterpret_cast<const f32x4_t*>(s_w + 32 * sl + 4 * g), w1 = *reinterpret_cast<const f32x4_t*>(s_w + 32 * sl + 16 + 4 * g);
             float p[8];
 #pragma unroll
             for (int e = 0; e < 8; ++e) {
-                wt[sl][e] = e < 4 ? w0[e] : w1[e - 4];
+                wt[sl][e] = mm_f4(wq[2 * sl + (e >> 2)])[e & 3];
                 p[e] = wt[sl][e] * (float)vv[sl][e];
             }
             mm_split(p, vhi[sl], vlo[sl]);
         }
+        static_for<DT / 4>([&](auto I4) {
+            constexpr int i0 = 4 * decltype(I4)::value;
+            u32x2_t kf[4][2][2];
+            const unsigned kb = lds_addr(kst) + (i0 >> 2) * 128;
+            mm_lds_tr16<RB>(kf, kb + tr_rel[0], kb + tr_rel[1], kb + tr_rel[2], kb + tr_rel[3]);
 #pragma unroll
-        for (int i = 0; i < DT; ++i) S[i] *= carry;
-        static_for<DT>([&](auto I) {
-            constexpr int i = decltype(I)::value;
-            u32x2_t kf[2][2];
-            lds_read_tr16_b64<(i >> 2) * 128>(kf[0][0], kst + tr_rel[i & 3]);
-            lds_read_tr16_b64<(i >> 2) * 128 + 16 * RB>(kf[0][1], kst + tr_rel[i & 3]);
-            lds_read_tr16_b64<(i >> 2) * 128 + 32 * RB>(kf[1][0], kst + tr_rel[i & 3]);
-            lds_read_tr16_b64<(i >> 2) * 128 + 48 * RB>(kf[1][1], kst + tr_rel[i & 3]);
-            wait_lds();
+            for (int jj = 0; jj < 4; ++jj) S[i0 + jj] *= carry;
 #pragma unroll
-            for (int sl = 0; sl < 2; ++sl) asm volatile("" : "+v"(kf[sl][0]), "+v"(kf[sl][1]));
-            float nn = 0.f;
+            for (int sl = 0; sl < 2; ++sl)
 #pragma unroll
-            for (int sl = 0; sl < 2; ++sl) {
-                const bf16x8_t k = __builtin_bit_cast(bf16x8_t, u32x4_t{kf[sl][0][0], kf[sl][0][1], kf[sl][1][0], kf[sl][1][1]});
-                S[i] = mm_mfma(k, vhi[sl], S[i]);
-                S[i] = mm_mfma(k, vlo[sl], S[i]);
-                if ((i & 3) == w) {
+                for (int x = 0; x < 2; ++x)
+#pragma unroll
+                    for (int jj = 0; jj < 4; ++jj) S[i0 + jj] = mm_mfma(mm_frag(kf[jj][sl][0], kf[jj][sl][1]), x ? vlo[sl] : vhi[sl], S[i0 + jj]);
+            float nn = 0.f;   // n of the rows 16 (i0 + w) + c
+#pragma unroll
+            for (int jj = 0; jj < 4; ++jj) {
+                if (jj != w) continue;
+#pragma unroll
+                for (int sl = 0; sl < 2; ++sl) {
+                    const bf16x8_t k = mm_frag(kf[jj][sl][0], kf[jj][sl][1]);
 #pragma unroll
                     for (int e = 0; e < 8; ++e) nn = fmaf(wt[sl][e], (float)k[e], nn);
                 }
             }
-            if ((i & 3) == w) {
-                nn += __shfl_xor(nn, 16, 64);
-                nn += __shfl_xor(nn, 32, 64);
-                nreg[i >> 2] = fmaf(carry, nreg[i >> 2], nn);
-                if (g == 0) s_n[16 * i + c] = nreg[i >> 2];  // read again behind the next barrier
-            }
+            nn += __shfl_xor(nn, 16, 64);
+            nn += __shfl_xor(nn, 32, 64);
+            nreg[i0 >> 2] = fmaf(carry, nreg[i0 >> 2], nn);
         });
+        mm_barrier();
+        // ---- output rows ----
+        u32x4_t pf[4][2][2];
+        const char *pa0 = pst + c * 128 + ((g ^ (c & 7)) << 4), *pa1 = pst + c * 128 + (((4 + g) ^ (c & 7)) << 4);
+        float in[4], dn[4], fl[4];
+        static_for<4>([&](auto RT) {
+            constexpr int rt = decltype(RT)::value;
+            pf[rt][0][0] = mm_lds<u32x4_t>(pa0 + (rt * 2048));
+            pf[rt][0][1] = mm_lds<u32x4_t>(pa0 + (rt * 2048 + 8192));
+            if constexpr (rt >= 2) {  // keys 32 .. 63 of rows 0 .. 31 are all in the future
+                pf[rt][1][0] = mm_lds<u32x4_t>(pa1 + (rt * 2048));
+                pf[rt][1][1] = mm_lds<u32x4_t>(pa1 + (rt * 2048 + 8192));
+            }
+            in[rt] = mm_lds<float>(sa + 4 * c + (512 + 64 * rt));
+            fl[rt] = mm_lds<float>(sa + 4 * c + (768 + 64 * rt));
+            dn[rt] = mm_lds<float>(sa + 4 * c + (1280 + 64 * rt));
+        });
+        if (g == 0) {
+#pragma unroll
+            for (int i = 0; i < DT / 4; ++i) s_n[16 * (4 * i + w) + c] = nreg[i];  // read again behind the next barrier
+        }
+#pragma unroll
+        for (int rt = 2; rt < 4; ++rt) asm volatile("" : "+v"(pf[rt][1][0]), "+v"(pf[rt][1][1]));
+#pragma unroll
+        for (int rt = 0; rt < 4; ++rt) acc[rt] *= in[rt];
+#pragma unroll
+        for (int sl = 0; sl < 2; ++sl)
+#pragma unroll
+            for (int x = 0; x < 2; ++x)
+#pragma unroll
+                for (int rt = 2 * sl; rt < 4; ++rt) acc[rt] = mm_mfma(vv[sl], __builtin_bit_cast(bf16x8_t, pf[rt][sl][x]), acc[rt]);
+        const int vc = vt * 64 + 16 * w + 4 * g;
+#pragma unroll
+        for (int rt = 0; rt < 4; ++rt) {
+            const int t = 16 * rt + c;
+            const float inv = 1.0f / (fmaxf(fabsf(dn[rt]), fl[rt]) + 1e-6f);
+            if (t < left && vc < a.vdimp)
+                *reinterpret_cast<u32x2_t*>(a.o + (int64_t)(r0 + ch * 64 + t) * a.ldo + (int64_t)h * a.vdimp + vc) =
+                    u32x2_t{pack2bf(acc[rt][0] * inv, acc[rt][1] * inv), pack2bf(acc[rt][2] * inv, acc[rt][3] * inv)};
+        }
         m_in = mL;
     }
     const int64_t so = a.state_out[seq];
@@ -631,7 +750,7 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
             const int d = 16 * (4 * i + w) + c;
             if (g == 0 && d < a.dimp) a.n[sout * a.dimp + d] = nreg[i];
         }
-        if (tid == 0) a.m[sout] = m_in;
+        if (tid == 0) a.m[sout] = m_in * (1.0f / MM_LOG2E);
     }
 }
 
@@ -733,16 +852,28 @@ extern "C" int glm_memory_recurrent(const void* x, int64_t ldx, int64_t k_off, i
     return f32 ? run_rec<float>(a, glm_s(stream)) : run_rec<bf16_t>(a, glm_s(stream));
 }
 
-extern "C" int glm_memory_chunkwise(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* gates, int64_t ldg, void* o, int64_t ldo, float* S, float* n, float* m,
+extern "C" int glm_memory_gates(const void* hrow, int64_t ldh, const void* wif, int64_t ldw, int wk, const float* bif, float* gates, int64_t rows, const int32_t* q_start,
+                                const int32_t* tile_seq, const int32_t* tile_off, int n_tiles, int H, float cap, glm_stream_t stream) {
+    GLM_CHECK_ARG(hrow && wif && bif && gates && q_start && tile_seq && tile_off, GLM_ERR_INVALID, "glm_memory_gates: null pointer");
+    GLM_CHECK_ARG(rows >= 0 && H > 0 && H <= 65535 * 16 && n_tiles >= 0 && n_tiles < (1 << 30) && wk > 0 && wk % 8 == 0 && ldh >= wk && ldw >= wk && ldh % 8 == 0 && ldw % 8 == 0 && cap > 0.f &&
+                      glm_aligned16(hrow) && glm_aligned16(wif), GLM_ERR_INVALID, "glm_memory_gates: bad shape rows=%ld H=%d wk=%d", (long)rows, H, wk);
+    if (n_tiles == 0) return GLM_OK;
+    GateArgs a = {(const bf16_t*)hrow, ldh, (const bf16_t*)wif, ldw, wk, bif, gates, rows, q_start, tile_seq, tile_off, H, cap};
+    hipLaunchKernelGGL(memory_gates_kernel, dim3((unsigned)(2 * n_tiles), (unsigned)((H + 15) / 16)), dim3(256), 0, glm_s(stream), a);
+    GLM_CHECK_LAUNCH("glm_memory_gates");
+    return GLM_OK;
+}
+
+extern "C" int glm_memory_chunkwise(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* gates, int64_t rows, void* o, int64_t ldo, float* S, float* n, float* m,
                                     int64_t n_state, const int32_t* pos, const int32_t* q_start, const int32_t* state_in, const int32_t* state_out, int seqs, int H, int dim, int dimp,
-                                    int vdimp, float cap, glm_stream_t stream) {
+                                    int vdimp, glm_stream_t stream) {
     GLM_CHECK_ARG(x && gates && o && S && n && m && pos && q_start && state_in && state_out, GLM_ERR_INVALID, "glm_memory_chunkwise: null pointer");
-    GLM_CHECK_ARG(seqs >= 0 && H > 0 && dim > 0 && dimp >= dim && dimp % 8 == 0 && vdimp > 0 && vdimp % 8 == 0 && n_state > 0 && k_off >= (int64_t)H * dimp && ldx >= k_off + (int64_t)H * dimp &&
-                      ldx >= v_off + (int64_t)H * vdimp && ldg >= 2 * H && ldo >= (int64_t)H * vdimp && ldx % 8 == 0 && k_off % 8 == 0 && v_off % 8 == 0 && ldo % 4 == 0 && cap > 0.f &&
+    GLM_CHECK_ARG(seqs >= 0 && rows >= 0 && H > 0 && dim > 0 && dimp >= dim && dimp % 8 == 0 && vdimp > 0 && vdimp % 8 == 0 && n_state > 0 && k_off >= (int64_t)H * dimp &&
+                      ldx >= k_off + (int64_t)H * dimp && ldx >= v_off + (int64_t)H * vdimp && ldo >= (int64_t)H * vdimp && ldx % 8 == 0 && k_off % 8 == 0 && v_off % 8 == 0 && ldo % 4 == 0 &&
                       glm_aligned16(x) && (((uintptr_t)o) & 7) == 0, GLM_ERR_INVALID, "glm_memory_chunkwise: bad shape H=%d dim=%d vdimp=%d ldx=%ld", H, dim, vdimp, (long)ldx);
     GLM_CHECK_ARG(dimp <= 256, GLM_ERR_UNSUPPORTED, "glm_memory_chunkwise: key size %d", dimp);
     if (seqs == 0) return GLM_OK;
-    ChunkArgs a = {(const bf16_t*)x, ldx, k_off, v_off, gates, ldg, (bf16_t*)o, ldo, S, n, m, n_state, pos, q_start, state_in, state_out, H, dim, dimp, vdimp, (vdimp + 63) / 64, cap};
+    ChunkArgs a = {(const bf16_t*)x, ldx, k_off, v_off, gates, rows, (bf16_t*)o, ldo, S, n, m, n_state, pos, q_start, state_in, state_out, H, dim, dimp, vdimp, (vdimp + 63) / 64};
     GLM_CHECK_ARG((int64_t)seqs * H * a.vtiles < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_memory_chunkwise: grid too large");
     hipStream_t st = glm_s(stream);
     if (dimp <= 64) return launch_chunk<64>(a, seqs, st);

@@ -262,7 +262,8 @@ __global__ __launch_bounds__(SW_NT) void stream_norm_any_kernel(const StreamNorm
 template <int S, int NV, int NT>
 int launch_stream(const StreamNormArgs& a, hipStream_t st) {
     // decode: one row per workgroup; else runs of rows long enough to spread the halo, short enough to fill the chip
-    int tr = a.T <= 512 ? 1 : (int)((a.T + 511) / 512);
+    constexpr int WGS = NT >= 512 ? 512 : 4096 / (NT / 64) > 2048 ? 2048 : 4096 / (NT / 64);   // four waves on every SIMD
+    int tr = a.T <= 512 ? 1 : (int)((a.T + WGS - 1) / WGS);
     if (tr > 1) tr = tr < 8 ? 8 : tr > 32 ? 32 : tr;
     hipLaunchKernelGGL((stream_norm_kernel<S, NV, NT>), dim3((unsigned)((a.T + tr - 1) / tr)), dim3(NT), 0, st, a, tr);
     GLM_CHECK_LAUNCH("glm_stream_norm");

@@ -172,16 +172,19 @@ _SIGNATURES = {
         c_void_p, c_int64, c_void_p]),
     "glm_group_attn_decode": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p,
         c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p,
-        c_void_p, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_void_p]),
+        c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_void_p,
+        c_void_p, c_void_p]),
     "glm_group_attn_plain": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p,
         c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_void_p, c_int64,
         c_int, c_void_p]),
     "glm_memory_recurrent": (c_int, [c_void_p, c_int64, c_int64, c_int64, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_int, c_void_p,
         c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p,
         c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_int, c_void_p]),
+    "glm_memory_gates": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_int64, c_void_p, c_void_p,
+        c_void_p, c_int, c_int, c_float, c_void_p]),
     "glm_memory_chunkwise": (c_int, [c_void_p, c_int64, c_int64, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p,
         c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int,
-        c_float, c_void_p]),
+        c_void_p]),
     "glm_memory_output": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int, c_int, c_int,
         c_float, c_void_p]),
 }
@@ -1540,8 +1543,9 @@ def group_attn_splits(tiles: int, tokens_per_tile: int, heads: int, kv_heads: in
 
 def group_attn_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor, pos: torch.Tensor, seq_of: torch.Tensor,
                       tile_tok: torch.Tensor, tile_n: torch.Tensor, tokens_per_tile: int, heads: int, window: int, chunk: int, scale: float, slope, sink,
-                      out: torch.Tensor, num_splits: int = 0) -> None:
-    """Decoded tokens and short portions (the rows of q) over the paged caches; out is written row by row from its first."""
+                      out: torch.Tensor, num_splits: int = 0, new=None) -> None:
+    """Decoded tokens and short portions (the rows of q) over the paged caches; out is written row by row from its first.  new =
+    (keys, values, q_start, slots): the rows' own keys and values are taken from there and stored to their cache rows."""
     n, G, bs, dk, dv = _group_shape(q, k_cache, v_cache, out, heads, slope, sink)
     T = q.shape[0]
     if T == 0:
@@ -1557,10 +1561,16 @@ def group_attn_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
     if ns > 1:
         part_o = torch.empty((T * heads, ns, dv), dtype=torch.float32, device=q.device)
         part_ml = torch.empty((T * heads, ns, 2), dtype=torch.float32, device=q.device)
+    kn = vn = q_start = slots = None
+    if new is not None:
+        kn, vn, q_start, slots = new
+        assert kn.shape == (T, G * dk) and vn.shape == (T, G * dv) and kn.stride() == vn.stride() and kn.stride(1) == 1 and kn.dtype == vn.dtype == q.dtype
+        assert q_start.dtype == slots.dtype == torch.int32 and slots.numel() >= T
     lib = load_library()
     _check(lib.glm_group_attn_decode(
         _p(q), q.stride(0), _p(k_cache), _p(v_cache), n, bs, _p(block_tables), block_tables.stride(0), _p(pos), _p(seq_of), _p(tile_tok), _p(tile_n),
-        tile_tok.numel(), tokens_per_tile, heads, G, dk, dv, window, chunk, scale, _p(slope), _p(sink), _p(out), out.stride(0), ns, _p(part_o), _p(part_ml),
+        tile_tok.numel(), tokens_per_tile, heads, G, dk, dv, window, chunk, scale, _p(slope), _p(sink), _p(kn), _p(vn),
+        kn.stride(0) if kn is not None else 0, _p(q_start), _p(slots), _p(out), out.stride(0), ns, _p(part_o), _p(part_ml),
         _stream()), "glm_group_attn_decode")
     if ns > 1:
         assert sink is not None and out.stride(0) == heads * dv
@@ -1608,22 +1618,25 @@ def memory_recurrent(x: torch.Tensor, hrow: torch.Tensor, wif: torch.Tensor, bif
         "glm_memory_recurrent")
 
 
-def memory_chunkwise(x: torch.Tensor, gates: torch.Tensor, norm: torch.Tensor, y: torch.Tensor, state, pos, q_start, state_in, state_out, heads: int, dim: int,
-                     vdim: int, cap: float, eps: float) -> None:
-    """The same for long portions (bf16), 64 tokens at a time; gates: fp32 [rows, >= 2 heads] gate projections with their biases.  q_start
-    and pos relative to the rows of x."""
-    _bf16(x, "x"); _bf16(y, "y")
+def memory_chunkwise(x: torch.Tensor, hrow: torch.Tensor, wif: torch.Tensor, bif: torch.Tensor, norm: torch.Tensor, y: torch.Tensor, state, pos, q_start, state_in,
+                     state_out, tile_seq, tile_off, heads: int, dim: int, vdim: int, cap: float, eps: float) -> None:
+    """The same for long portions (bf16), 64 tokens at a time; q_start, pos and the 128-row tiles relative to the rows of x."""
+    _bf16(x, "x"); _bf16(y, "y"); _bf16(hrow, "hrow"); _bf16(wif, "wif")
     dimp, vdimp = round8(dim), round8(vdim)
     S, n, m = _memory_state(state, heads, dimp, vdimp)
     kd, vd, T = heads * dimp, heads * vdimp, x.shape[0]
-    assert x.shape[1] >= 2 * kd + 2 * vd and gates.dtype == torch.float32 and gates.shape[0] == T and gates.shape[1] >= 2 * heads and x.stride(1) == y.stride(1) == gates.stride(1) == 1
-    for t in (pos, q_start, state_in, state_out):
+    assert x.shape[1] >= 2 * kd + 2 * vd and hrow.shape[0] == T and x.stride(1) == y.stride(1) == hrow.stride(1) == wif.stride(1) == 1
+    assert wif.shape == (2 * heads, hrow.shape[1]) and bif.numel() == 2 * heads and norm.numel() == vd and bif.dtype == norm.dtype == torch.float32
+    for t in (pos, q_start, state_in, state_out, tile_seq, tile_off):
         assert t.dtype == torch.int32
     seqs = q_start.numel() - 1
-    assert state_in.numel() >= seqs and state_out.numel() >= seqs and pos.numel() == T
+    assert state_in.numel() >= seqs and state_out.numel() >= seqs and pos.numel() == T and tile_seq.numel() == tile_off.numel()
     o = torch.empty((T, vd), dtype=x.dtype, device=x.device)
+    gates = torch.empty((3, heads, T), dtype=torch.float32, device=x.device)
     lib = load_library()
-    _check(lib.glm_memory_chunkwise(_p(x), x.stride(0), kd, 2 * kd, _p(gates), gates.stride(0), _p(o), vd, _p(S), _p(n), _p(m), S.shape[0], _p(pos), _p(q_start),
-                                    _p(state_in), _p(state_out), seqs, heads, dim, dimp, vdimp, cap, _stream()), "glm_memory_chunkwise")
+    _check(lib.glm_memory_gates(_p(hrow), hrow.stride(0), _p(wif), wif.stride(0), hrow.shape[1], _p(bif), _p(gates), T, _p(q_start), _p(tile_seq), _p(tile_off),
+                                tile_seq.numel(), heads, cap, _stream()), "glm_memory_gates")
+    _check(lib.glm_memory_chunkwise(_p(x), x.stride(0), kd, 2 * kd, _p(gates), T, _p(o), vd, _p(S), _p(n), _p(m), S.shape[0], _p(pos), _p(q_start),
+                                    _p(state_in), _p(state_out), seqs, heads, dim, dimp, vdimp, _stream()), "glm_memory_chunkwise")
     _check(lib.glm_memory_output(_p(o), vd, _p(x[:, 2 * kd + vd:]), x.stride(0), _p(norm), _p(y), y.stride(0), T, heads, vdim, vdimp, eps, _stream()),
            "glm_memory_output")

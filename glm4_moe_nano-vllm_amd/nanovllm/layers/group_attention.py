@@ -32,8 +32,8 @@ class GroupAttention(nn.Module):
         H, G = self.heads, self.kv_heads
         self.qkv_proj = PaddedLinear(width, [self.dimp] * H + ([self.dimp] * G + [self.vdimp] * G if own_kv else []), dtype)
         self.o_proj = PaddedLinear([vdim] * H, [hip_ops.round8(width)], dtype)
-        # (fp32, and heads beyond the tiled kernels' sizes: one evaluation for all portions)
-        self.tiled = dtype == torch.bfloat16 and max(self.dimp, self.vdimp) <= hip_ops.GROUP_ATTN_MAX_DIM
+        # (fp32, and what the tiled kernels do not take: one evaluation for all portions)
+        self.tiled = dtype == torch.bfloat16 and scale > 0 and max(self.dimp, self.vdimp) <= hip_ops.GROUP_ATTN_MAX_DIM
         self.tokens_per_tile = max(1, hip_ops.GROUP_ATTN_ROWS // (H // G)) if self.tiled else 1
         self.slope = self.sink = self.k_cache = self.v_cache = None
 
@@ -65,8 +65,10 @@ class GroupAttention(nn.Module):
         x = self.qkv_proj(h)
         nq = H * self.dimp
         kc, vc = cache or (self.k_cache, self.v_cache)
-        if self.own_kv:
-            hip_ops.group_kv_store(x, nq, nq + self.kv_heads * self.dimp, meta.slots, kc, vc)
+        nk = nq + self.kv_heads * self.dimp
+        Ts = Ta if self.tiled else 0    # the decode kernel stores its rows' keys and values itself
+        if self.own_kv and Ts < T:
+            hip_ops.group_kv_store(x[Ts:], nq, nk, meta.slots[Ts:], kc, vc)
         q = x[:, :nq]
         out = torch.empty((T, H * self.vdimp), dtype=h.dtype, device=h.device)
         form = (H, self.window, self.chunk, self.scale, self.slope, self.sink)
@@ -76,7 +78,8 @@ class GroupAttention(nn.Module):
             if Ta:
                 per = min(self.tokens_per_tile, meta.max_short)
                 tok, n = meta.tiles[per]
-                hip_ops.group_attn_decode(q[:Ta], kc, vc, meta.block_tables, meta.pos, meta.seq_of, tok, n, per, *form, out)
+                new = (x[:Ta, nq: nk], x[:Ta, nk:], meta.q_start, meta.slots) if self.own_kv else None
+                hip_ops.group_attn_decode(q[:Ta], kc, vc, meta.block_tables, meta.pos, meta.seq_of, tok, n, per, *form, out, new=new)
             if Ta < T:
                 hip_ops.group_attn_prefill(q[Ta:], kc, vc, meta.block_tables, meta.n_short, meta.long_q_start, meta.pos[Ta:], meta.long_tile_seq,
                                            meta.long_tile_off, *form, out[Ta:])

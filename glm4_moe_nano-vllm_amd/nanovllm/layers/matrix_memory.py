@@ -25,10 +25,10 @@ class MatrixMemory(nn.Module):
         self.dimp, self.vdimp, self.wp = hip_ops.round8(dim), hip_ops.round8(vdim), hip_ops.round8(width)
         H = self.heads
         self.in_proj = PaddedLinear(width, [self.dimp] * (2 * H) + [self.vdimp] * (2 * H), dtype)
-        self.gate_proj = PaddedLinear(width, [hip_ops.round8(2 * H)], dtype)
+        self.gates = PaddedLinear(width, [hip_ops.round8(2 * H)], dtype)   # rows i | f; projected where the recurrence needs them
         self.o_proj = PaddedLinear([vdim] * H, [hip_ops.round8(width)], dtype)
         self.chunkwise = dtype == torch.bfloat16 and self.dimp <= hip_ops.MEMORY_CHUNK_MAX_DIM
-        self.gate_bias = self.gate_bias_rows = self.norm = self.state = None
+        self.gate_bias = self.norm = self.state = None
 
     def load(self, w: dict, device) -> None:
         """w: q, k, v, g, o, norm, i, i.b, f, f.b."""
@@ -39,10 +39,8 @@ class MatrixMemory(nn.Module):
 
         d, v = self.dim, self.vdim
         self.in_proj.load(list(heads_of(w["q"], d)) + list(heads_of(w["k"], d)) + list(heads_of(w["v"], v)) + list(heads_of(w["g"], v)), device)
-        self.gate_proj.load([torch.cat([w["i"][h0: h0 + H], w["f"][h0: h0 + H]])], device)
+        self.gates.load([torch.cat([w["i"][h0: h0 + H], w["f"][h0: h0 + H]])], device)
         self.gate_bias = torch.cat([w["i.b"][h0: h0 + H], w["f.b"][h0: h0 + H]]).to(device=device, dtype=torch.float32)
-        self.gate_bias_rows = torch.zeros(self.gate_proj.N, dtype=self.dtype, device=device)
-        self.gate_bias_rows[: 2 * H] = self.gate_bias.to(self.dtype)
         norm = torch.zeros(H, self.vdimp, dtype=torch.float32, device=device)
         norm[:, :v] = heads_of(w["norm"], v)[..., 0].to(torch.float32)
         self.norm = norm.reshape(-1)
@@ -60,15 +58,15 @@ class MatrixMemory(nn.Module):
         H, T, Ta, ns = self.heads, h.shape[0], meta.Ta, meta.n_short
         x = self.in_proj(h)
         y = torch.empty((T, H * self.vdimp), dtype=h.dtype, device=h.device)
+        gates = (self.gates.weight[: 2 * H], self.gate_bias, self.norm)
         form = (H, self.dim, self.vdim, self.cap, self.eps)
         if not self.chunkwise:
             Ta, ns = T, meta.q_start.numel() - 1
         if Ta:
-            hip_ops.memory_recurrent(x[:Ta], h[:Ta], self.gate_proj.weight[: 2 * H], self.gate_bias, self.norm, y[:Ta], self.state, meta.pos, meta.q_start[: ns + 1],
-                                     meta.state_in, meta.state_out, *form)
+            hip_ops.memory_recurrent(x[:Ta], h[:Ta], *gates, y[:Ta], self.state, meta.pos, meta.q_start[: ns + 1], meta.state_in, meta.state_out, *form)
         if Ta < T:
-            gates = self.gate_proj(h[Ta:], bias=self.gate_bias_rows, out_f32=True)
-            hip_ops.memory_chunkwise(x[Ta:], gates, self.norm, y[Ta:], self.state, meta.pos[Ta:], meta.long_q_start, meta.state_in[ns:], meta.state_out[ns:], *form)
+            hip_ops.memory_chunkwise(x[Ta:], h[Ta:], *gates, y[Ta:], self.state, meta.pos[Ta:], meta.long_q_start, meta.state_in[ns:], meta.state_out[ns:],
+                                     meta.long_tile_seq, meta.long_tile_off, *form)
         y = self.o_proj(y)
         if self.tp_size > 1:
             get_tp_group().all_reduce(y)

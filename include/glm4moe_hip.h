@@ -544,7 +544,8 @@ int glm_stream_norm(const float* x_in, int64_t ldx, int64_t sx, const int32_t* r
  * store: key / value columns of projection rows -> cache rows slots[t] (< 0: none).
  * prefill: 128-row tiles (sequence, first row inside the portion) of portions [q_start[s], q_start[s+1]), block table row seq0 + s.
  * decode: tiles of tile_n[i] <= tokens_per_tile rows of one sequence from tile_tok[i]; nsplit > 1: unnormalised sums part_o
- * [rows*H, nsplit, dv] and part_ml [rows*H, nsplit, 2] for glm_attn_merge.  Both bf16, dk, dv <= 256.  plain: any size, bf16 or fp32.  */
+ * [rows*H, nsplit, dv] and part_ml [rows*H, nsplit, 2] for glm_attn_merge; knew / vnew (may be NULL): keys and values of the rows of q,
+ * head g at g*dk / g*dv, read instead of the cache's and stored to cache rows `slots`.  Both bf16, dk, dv <= 256, scale > 0.  plain: any size, bf16 or fp32.  */
 int glm_group_kv_store(const void* src, int64_t ld, int64_t k_off, int64_t v_off, int f32, const int32_t* slots, int64_t T,
                        void* kc, void* vc, int64_t n_slots, int bs, int G, int dk, int dv, glm_stream_t stream);
 int glm_group_attn_prefill(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs,
@@ -555,8 +556,9 @@ int glm_group_attn_prefill(const void* q, int64_t ldq, const void* kc, const voi
 int glm_group_attn_decode(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs,
                           const int32_t* block_tables, int64_t bt_stride, const int32_t* pos, const int32_t* seq_of,
                           const int32_t* tile_tok, const int32_t* tile_n, int n_tiles, int tokens_per_tile, int H, int G, int dk,
-                          int dv, int window, int chunk, float scale, const float* slope, const float* sink, void* out,
-                          int64_t ldo, int nsplit, float* part_o, float* part_ml, glm_stream_t stream);
+                          int dv, int window, int chunk, float scale, const float* slope, const float* sink, const void* knew,
+                          const void* vnew, int64_t ldkv, const int32_t* q_start, const int32_t* slots, void* out, int64_t ldo,
+                          int nsplit, float* part_o, float* part_ml, glm_stream_t stream);
 int glm_group_attn_plain(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs,
                          const int32_t* block_tables, int64_t bt_stride, const int32_t* pos, const int32_t* seq_of, int64_t rows,
                          int H, int G, int dk, int dv, int window, int chunk, float scale, const float* slope, const float* sink,
@@ -566,16 +568,20 @@ int glm_group_attn_plain(const void* q, int64_t ldq, const void* kc, const void*
  * k_off + h*dimp, v at v_off + h*vdimp and the output gate at g_off + h*vdimp.  State rows S [n_state][H][dimp][vdimp], n
  * [n_state][H][dimp], m [n_state][H], fp32; sequence s reads row state_in[s] (not at position 0) and writes row state_out[s].
  * recurrent: portions [q_start[s], q_start[s+1]) token by token; gate projections wif [2 H rows i | f, wk] of rows hrow, biases bif.
- * chunkwise: bf16, dimp <= 256; gates [rows, >= 2 H] = the gate projections with their biases; o: rows in front of the norm.
+ * gates: bf16, [3][H][rows] of long portions for chunkwise, by 128-row tiles (sequence, first row inside the portion).
+ * chunkwise: bf16, dimp <= 256; o: rows in front of the norm.
  * output: y = o / rms(o) norm sigmoid(g) per head.                                                                          */
 int glm_memory_recurrent(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, int64_t g_off, const void* hrow, int64_t ldh,
                          const void* wif, int64_t ldw, int wk, const float* bif, const float* norm, void* y, int64_t ldy, float* S,
                          float* n, float* m, int64_t n_state, const int32_t* pos, const int32_t* q_start, const int32_t* state_in,
                          const int32_t* state_out, int seqs, int H, int dim, int dimp, int vdim, int vdimp, float cap, float eps,
                          int f32, glm_stream_t stream);
-int glm_memory_chunkwise(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* gates, int64_t ldg, void* o,
+int glm_memory_gates(const void* hrow, int64_t ldh, const void* wif, int64_t ldw, int wk, const float* bif, float* gates,
+                     int64_t rows, const int32_t* q_start, const int32_t* tile_seq, const int32_t* tile_off, int n_tiles, int H,
+                     float cap, glm_stream_t stream);
+int glm_memory_chunkwise(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* gates, int64_t rows, void* o,
                          int64_t ldo, float* S, float* n, float* m, int64_t n_state, const int32_t* pos, const int32_t* q_start,
-                         const int32_t* state_in, const int32_t* state_out, int seqs, int H, int dim, int dimp, int vdimp, float cap,
+                         const int32_t* state_in, const int32_t* state_out, int seqs, int H, int dim, int dimp, int vdimp,
                          glm_stream_t stream);
 int glm_memory_output(const void* o, int64_t ldo, const void* g, int64_t ldg, const float* norm, void* y, int64_t ldy, int64_t T,
                       int H, int vdim, int vdimp, float eps, glm_stream_t stream);

@@ -194,7 +194,7 @@ FORMS = [(6, 2, 24, 40, 0, 50, 64), (4, 4, 128, 128, 0, 200, 64), (3, 1, 136, 20
 
 
 @pytest.mark.parametrize("H,G,dk,dv,window,chunk,bs", FORMS)
-@pytest.mark.parametrize("kind", ["decode1", "decode1_split", "decode5", "prefill", "plain", "plain_f32"])
+@pytest.mark.parametrize("kind", ["decode1", "decode1_split", "decode5", "decode1_new", "decode5_new", "prefill", "plain", "plain_f32"])
 def test_group_attention(H, G, dk, dv, window, chunk, bs, kind):
     """Every form over pages in disorder, with NaNs wherever nothing was stored; with bias and sink, and without."""
     from nanovllm import hip_ops
@@ -202,7 +202,7 @@ def test_group_attention(H, G, dk, dv, window, chunk, bs, kind):
     dt, span = DT[dtype], max(window, chunk, 90)
     if kind.startswith("decode1"):
         lens, n_q = [1, span + 1, 2 * span, span + 37, 321], [1] * 5
-    elif kind == "decode5":
+    elif kind.startswith("decode5"):
         lens, n_q = [5, span + 2, 2 * span + 1, 2, 130], [5, 5, 3, 2, 4]
     else:
         lens, n_q = [300, span + 60, 2 * span + 129, 2, 64], [300, 60, 129, 2, 64]
@@ -221,6 +221,14 @@ def test_group_attention(H, G, dk, dv, window, chunk, bs, kind):
         out = torch.full((T, H * dv), float("nan"), dtype=dt, device="cuda")
         form = (H, window, chunk, 0.9, dev(slope) if slope is not None else None, dev(sink) if sink is not None else None)
         args = (dev(qr, dt), dev(kc, dt), dev(vc, dt), i32(bt))
+        new = None
+        if kind.endswith("_new"):   # the step's own keys and values are not in the cache yet: it must hold them afterwards
+            rows = torch.cat([torch.cat([t[s][lens[s] - n_q[s]:].reshape(n_q[s], -1) for s in range(len(lens))]) for t in (k, v)], 1)
+            slots = torch.cat([bt[s, torch.arange(n - m, n) // bs] * bs + torch.arange(n - m, n) % bs for s, (n, m) in enumerate(zip(lens, n_q))])
+            for c in args[1:3]:
+                c[dev(slots) // bs, :, dev(slots) % bs] = float("nan")
+            rows = dev(rows, dt)
+            new = (rows[:, : G * dk], rows[:, G * dk:], i32(qs), i32(slots))
         if kind == "prefill":
             tiles = [(s, o) for s, n in enumerate(n_q) for o in range(0, n, 128)]
             wide = torch.full((3 + bt.shape[0], bt.shape[1]), -1, dtype=torch.int32)
@@ -231,10 +239,12 @@ def test_group_attention(H, G, dk, dv, window, chunk, bs, kind):
         else:
             if kind == "decode1_split" and sink is None:
                 continue
-            per = max(1, min(max(n_q), hip_ops.GROUP_ATTN_ROWS // (H // G)))
+            per = max(1, min(max(n_q), hip_ops.GROUP_ATTN_ROWS // (H // G)))   # (five rows of a portion may be several tiles)
             tok = [qs[s] + o for s, n in enumerate(n_q) for o in range(0, n, per)]
             cnt = [min(per, n - o) for n in n_q for o in range(0, n, per)]
-            hip_ops.group_attn_decode(*args, pos, seq_of, i32(tok), i32(cnt), per, *form, out, num_splits=7 if kind == "decode1_split" else 1)
+            hip_ops.group_attn_decode(*args, pos, seq_of, i32(tok), i32(cnt), per, *form, out, num_splits=7 if kind == "decode1_split" else 1, new=new)
+            if new is not None:
+                assert torch.equal(args[1].nan_to_num(), dev(kc, dt).nan_to_num()) and torch.equal(args[2].nan_to_num(), dev(vc, dt).nan_to_num())
         got = out.cpu().double().view(T, H, dv)
         for s in range(len(lens)):
             ref = _attn_reference(q[s], k[s], v[s], window, chunk, 0.9, slope, sink)
@@ -277,10 +287,9 @@ def test_matrix_memory(H, dim, vdim, cap, form):
     wif, bif, norm = r16(rnd(500, 2 * H, width) * 0.4), torch.cat([rnd(501, H), 6 * rnd(502, H)]), 1 + 0.2 * rnd(503, H * vdim)
     if H == 1:
         bif[1] = 30.0        # hardly forgets
-    ref, gates = {}, {}
+    ref = {}
     for s in L:
         z = h[s].double() @ wif.double().T + bif.double()
-        gates[s] = z.float()
         i, f = O.soft_cap(z[:, :H], cap), O.log_sigmoid(O.soft_cap(z[:, H:], cap))
         o = torch.stack([O.unit_rms(O.mlstm_cell(q[s][:, a].double() * dim ** -0.5, k[s][:, a].double(), v[s][:, a].double(), i[:, a], f[:, a]), eps) for a in range(H)], 1)
         ref[s] = o.reshape(len(o), -1) * norm.double() * torch.sigmoid(gt[s].reshape(len(o), -1).double())
@@ -294,11 +303,13 @@ def test_matrix_memory(H, dim, vdim, cap, form):
             cut = lambda t: torch.cat([t[s][at[s]: at[s] + n] for s, n in step])  # noqa: E731
             xs, T = dev(cut(x), dt), sum(n for _, n in step)
             y = torch.full((T, H * vdimp), float("nan"), dtype=dt, device="cuda")
+            rows = (xs, dev(cut(h), dt), dev(wif, dt), dev(bif), dev(normp), y)
             rest = (state, meta.pos, meta.q_start, meta.state_in, meta.state_out, H, dim, vdim, cap, eps)
             if form == "chunkwise":
-                hip_ops.memory_chunkwise(xs, dev(cut(gates)), dev(normp), y, *rest)
+                tiles = [(s, o) for s, (_, n) in enumerate(step) for o in range(0, n, 128)]
+                hip_ops.memory_chunkwise(*rows, *rest[:5], i32([t[0] for t in tiles]), i32([t[1] for t in tiles]), *rest[5:])
             else:
-                hip_ops.memory_recurrent(xs, dev(cut(h), dt), dev(wif, dt), dev(bif), dev(normp), y, *rest)
+                hip_ops.memory_recurrent(*rows, *rest)
             y, r = y.cpu().double().view(T, H, vdimp), 0
             assert torch.all(y[..., vdim:] == 0)
             for s, n in step:
