@@ -58,6 +58,7 @@ __device__ __forceinline__ int ga_first(const GroupArgs& a, int p) {
 __device__ __forceinline__ int ga_block(const GroupArgs& a, int j) { return a.log2_bs >= 0 ? j >> a.log2_bs : j / a.bs; }
 // row of a cache (in units of the head size) of key position j with block id blk, head g
 __device__ __forceinline__ int64_t ga_row(const GroupArgs& a, int blk, int j, int g) { return ((int64_t)blk * a.G + g) * a.bs + (j - ga_block(a, j) * a.bs); }
+__device__ __forceinline__ int ga_uniform(int v) { return __builtin_amdgcn_readfirstlane(v); }
 __device__ __forceinline__ bool ga_ok(const GroupArgs& a, int blk) { return blk >= 0 && blk < a.n_blocks; }
 
 // ---------------------------------------------------------------------------------------------------------------------------
@@ -250,10 +251,10 @@ __global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void group_attn_pref
     const int item = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
     if ((int)(blockIdx.x >> 3) >= per || item >= total) return;
     const int h = item / a.n_tiles, tile = item % a.n_tiles, kvh = h / (a.H / a.G);
-    const int seq = a.tile_a[tile], qo = a.tile_b[tile];
-    const int qs = a.q_start[seq], nq = a.q_start[seq + 1] - qs;
+    const int seq = ga_uniform(a.tile_a[tile]), qo = ga_uniform(a.tile_b[tile]);
+    const int qs = ga_uniform(a.q_start[seq]), nq = ga_uniform(a.q_start[seq + 1]) - qs;
     if (qo >= nq) return;
-    const int p0 = a.pos[qs] + qo, plast = p0 + min(127, nq - 1 - qo);  // positions of the tile's first and last row
+    const int p0 = ga_uniform(a.pos[qs]) + qo, plast = p0 + min(127, nq - 1 - qo);  // positions of the tile's first and last row
     const int jlo = ga_first(a, p0) & ~63;
     const int n = ((plast - jlo) >> 6) + 1;
     const int32_t* bt = a.bt + (int64_t)(a.seq0 + seq) * a.bt_stride;
@@ -304,8 +305,9 @@ __global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void group_attn_pref
         vpad[i] = ch * 8 >= a.dv;
         voff[i] = (unsigned)(row * a.dv + ch * 8);
     }
+    // tiles from the last keys to the first: under a distance bias the maximum is found early and stays
     auto issue = [&](int it, int blk) {
-        const int j0 = jlo + it * 64, left = ga_ok(a, blk) ? plast - j0 + 1 : 0;
+        const int j0 = jlo + (n - 1 - it) * 64, left = ga_ok(a, blk) ? plast - j0 + 1 : 0;
         const int64_t row = ga_row(a, blk, j0, kvh);
         const bf16_t* kb = reinterpret_cast<const bf16_t*>(a.kc) + row * a.dk;
         const bf16_t* vb = reinterpret_cast<const bf16_t*>(a.vc) + row * a.dv;
@@ -322,19 +324,19 @@ __global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void group_attn_pref
         }
     };
     const float sc = a.scale * GA_LOG2E;
-    auto block_of = [&](int it) { return bt[ga_block(a, jlo + min(it, n - 1) * 64)]; };  // 64-key tiles lie in one block
+    auto block_of = [&](int it) { return bt[ga_block(a, jlo + max(n - 1 - it, 0) * 64)]; };  // 64-key tiles lie in one block
     int blk = block_of(1);
-    issue(0, block_of(0));
+    issue(0, ga_uniform(block_of(0)));
     for (int it = 0; it < n; ++it) {
         wait_vm<0>();
         __builtin_amdgcn_s_barrier();
         if (it + 1 < n) {
-            issue(it + 1, blk);
+            issue(it + 1, ga_uniform(blk));
             blk = block_of(it + 2);
         }
         const unsigned kst = base + (it & 1) * STAGE, vst = kst + KTILE;
 #pragma unroll
-        for (int s = 0; s < 2; ++s) S.run(kst + s * 32 * KB, vst + s * 32 * VB, jlo + it * 64 + s * 32, g, sc);
+        for (int s = 1; s >= 0; --s) S.run(kst + s * 32 * KB, vst + s * 32 * VB, jlo + (n - 1 - it) * 64 + s * 32, g, sc);
     }
     const float sk = a.sink ? a.sink[h] * GA_LOG2E : -INFINITY;
 #pragma unroll
@@ -373,15 +375,15 @@ __global__ __launch_bounds__(NW * 64, 1) void group_attn_decode_kernel(const Gro
     const int rg = item % row_groups;
     item /= row_groups;
     const int kvh = item % a.G, tile = item / a.G;
-    const int tok0 = a.tile_a[tile], ntok = a.tile_b[tile], R = a.H / a.G;
-    const int pA = a.pos[tok0], pB = pA + ntok - 1;
+    const int tok0 = ga_uniform(a.tile_a[tile]), ntok = ga_uniform(a.tile_b[tile]), R = a.H / a.G;
+    const int pA = ga_uniform(a.pos[tok0]), pB = pA + ntok - 1;
     const int rho = rg * 16 + c, tok = rho / R, hh = rho - tok * R, h = kvh * R + hh;
     const bool row_ok = tok < ntok;
     if (rg * 16 >= ntok * R) return;
     const int jlo = pA >= 0 ? ga_first(a, pA) & ~31 : 0;
     const int slabs = pA >= 0 ? ((pB - jlo) >> 5) + 1 : 0, per = (slabs + a.nsplit - 1) / a.nsplit;
     const int s_lo = split * per, s_hi = min(s_lo + per, slabs);
-    const int n = s_hi > s_lo + w ? (s_hi - s_lo - w + NW - 1) / NW : 0;  // slabs of this wave: s_lo + w + NW k
+    const int n = s_hi > s_lo + w ? (s_hi - s_lo - w + NW - 1) / NW : 0;  // slabs of this wave: s_hi - 1 - w - NW k, last keys first
     SL S;
     S.init(lane);
     S.rp[0] = row_ok && pA >= 0 ? pA + tok : -1;
@@ -437,7 +439,7 @@ __global__ __launch_bounds__(NW * 64, 1) void group_attn_decode_kernel(const Gro
         vpad[i] = ch * 8 >= a.dv;
         voff[i] = (unsigned)(row * a.dv + ch * 8);
     }
-    auto key0 = [&](int k) { return jlo + (s_lo + w + NW * k) * 32; };
+    auto key0 = [&](int k) { return jlo + (s_hi - 1 - w - NW * k) * 32; };
     // block ids of this wave's next 64 slabs, one per lane
     auto blocks_from = [&](int k) { return k + lane < n ? bt[ga_block(a, key0(k + lane))] : -1; };
     int ids = n > 0 ? blocks_from(0) : -1;

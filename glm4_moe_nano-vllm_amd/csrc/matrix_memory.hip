@@ -424,12 +424,16 @@ __device__ __forceinline__ void mm_lds_tr16(u32x2_t (&d)[4][2][2], unsigned p0, 
 }
 // v = hi + lo, two bf16 each
 __device__ __forceinline__ void mm_split(const float (&v)[8], bf16x8_t& hi, bf16x8_t& lo) {
+    typedef __attribute__((ext_vector_type(2))) float f32x2;
+    typedef __attribute__((ext_vector_type(2))) __bf16 bf16x2;
+    u32x4_t h, l;
 #pragma unroll
-    for (int e = 0; e < 8; ++e) {
-        const __bf16 b = (__bf16)v[e];
-        hi[e] = b;
-        lo[e] = (__bf16)(v[e] - (float)b);
+    for (int e = 0; e < 4; ++e) {
+        h[e] = __builtin_bit_cast(unsigned, __builtin_convertvector((f32x2{v[2 * e], v[2 * e + 1]}), bf16x2));
+        l[e] = __builtin_bit_cast(unsigned, __builtin_convertvector((f32x2{v[2 * e] - bflo(h[e]), v[2 * e + 1] - bfhi(h[e])}), bf16x2));
     }
+    hi = __builtin_bit_cast(bf16x8_t, h);
+    lo = __builtin_bit_cast(bf16x8_t, l);
 }
 // barrier that leaves LDS-DMA in flight
 __device__ __forceinline__ void mm_barrier() {
@@ -491,22 +495,45 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
     const bf16_t* xv = a.x + (int64_t)r0 * a.ldx + a.v_off + (int64_t)h * a.vdimp + vt * 64;
     const float* gp = a.gates + (int64_t)h * a.rows + r0;
     const int64_t gpart = (int64_t)a.H * a.rows;
+    // per-lane source offsets of the DMA pieces: constant over the chunks
+    unsigned qoff[QDMA], voff[VDMA];
+#pragma unroll
+    for (int i = 0; i < QDMA; ++i) {
+        const int p = (w * QDMA + i) * 64 + lane, row = p / CPR;
+        qoff[i] = (unsigned)(row * (int)a.ldx + ((p % CPR) ^ attn_swz(row)) * 8);
+    }
+#pragma unroll
+    for (int i = 0; i < VDMA; ++i) {
+        const int p = (w * VDMA + i) * 64 + lane, row = p >> 3;
+        voff[i] = (unsigned)(row * (int)a.ldx + ((p & 7) ^ attn_swz(row)) * 8);
+    }
+    const bool whole = a.dimp == D && vt * 64 + 64 <= a.vdimp;  // no padding columns in this workgroup's tiles
     auto issue = [&](int ch) {
         char* st = smem + (ch & 1) * STAGE;
         const int left = T - ch * 64;
+        const bf16_t *q = xq + (int64_t)ch * 64 * a.ldx, *k = q + a.k_off, *v = xv + (int64_t)ch * 64 * a.ldx;
+        if (whole && left >= 64) {
+#pragma unroll
+            for (int i = 0; i < QDMA; ++i) {
+                lds_dma16(q + qoff[i], st + (w * QDMA + i) * 1024);
+                lds_dma16(k + qoff[i], st + QT + (w * QDMA + i) * 1024);
+            }
+#pragma unroll
+            for (int i = 0; i < VDMA; ++i) lds_dma16(v + voff[i], st + 2 * QT + (w * VDMA + i) * 1024);
+            return;
+        }
 #pragma unroll
         for (int i = 0; i < QDMA; ++i) {
             const int p = (w * QDMA + i) * 64 + lane, row = p / CPR, cc = (p % CPR) ^ attn_swz(row);
             const bool ok = row < left && cc * 8 < a.dimp;
-            const bf16_t* s = xq + (int64_t)(ch * 64 + row) * a.ldx + cc * 8;
-            lds_dma16(ok ? (const void*)s : (const void*)mm_zero_page, st + (w * QDMA + i) * 1024);
-            lds_dma16(ok ? (const void*)(s + a.k_off) : (const void*)mm_zero_page, st + QT + (w * QDMA + i) * 1024);
+            lds_dma16(ok ? (const void*)(q + qoff[i]) : (const void*)mm_zero_page, st + (w * QDMA + i) * 1024);
+            lds_dma16(ok ? (const void*)(k + qoff[i]) : (const void*)mm_zero_page, st + QT + (w * QDMA + i) * 1024);
         }
 #pragma unroll
         for (int i = 0; i < VDMA; ++i) {
             const int p = (w * VDMA + i) * 64 + lane, row = p >> 3, cc = (p & 7) ^ attn_swz(row);
             const bool ok = row < left && vt * 64 + cc * 8 < a.vdimp;
-            lds_dma16(ok ? (const void*)(xv + (int64_t)(ch * 64 + row) * a.ldx + cc * 8) : (const void*)mm_zero_page, st + 2 * QT + (w * VDMA + i) * 1024);
+            lds_dma16(ok ? (const void*)(v + voff[i]) : (const void*)mm_zero_page, st + 2 * QT + (w * VDMA + i) * 1024);
         }
     };
     // fragment offsets.  Rows by 16 (lane c), eight columns 32 i + 8 g: the scores.  Rows by 16, columns 32 i + 4 g and + 16: the readout,
@@ -612,6 +639,7 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
                 for (int x = 0; x < 2; ++x)
 #pragma unroll
                     for (int rt = 0; rt < 4; ++rt) acc[rt] = mm_mfma(x ? lo[jj] : hi[jj], mm_frag(qh[jj][rt][0], qh[jj][rt][1]), acc[rt]);
+            asm volatile("" ::: "memory");  // one group's fragments at a time
         });
         // ---- operands of the state's update: values and keys over tokens ----
         u32x2_t vf[2][2];
@@ -727,7 +755,7 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
 #pragma unroll
         for (int rt = 0; rt < 4; ++rt) {
             const int t = 16 * rt + c;
-            const float inv = 1.0f / (fmaxf(fabsf(dn[rt]), fl[rt]) + 1e-6f);
+            const float inv = __builtin_amdgcn_rcpf(fmaxf(fabsf(dn[rt]), fl[rt]) + 1e-6f);
             if (t < left && vc < a.vdimp)
                 *reinterpret_cast<u32x2_t*>(a.o + (int64_t)(r0 + ch * 64 + t) * a.ldo + (int64_t)h * a.vdimp + vc) =
                     u32x2_t{pack2bf(acc[rt][0] * inv, acc[rt][1] * inv), pack2bf(acc[rt][2] * inv, acc[rt][3] * inv)};
@@ -869,7 +897,7 @@ extern "C" int glm_memory_chunkwise(const void* x, int64_t ldx, int64_t k_off, i
                                     int vdimp, glm_stream_t stream) {
     GLM_CHECK_ARG(x && gates && o && S && n && m && pos && q_start && state_in && state_out, GLM_ERR_INVALID, "glm_memory_chunkwise: null pointer");
     GLM_CHECK_ARG(seqs >= 0 && rows >= 0 && H > 0 && dim > 0 && dimp >= dim && dimp % 8 == 0 && vdimp > 0 && vdimp % 8 == 0 && n_state > 0 && k_off >= (int64_t)H * dimp &&
-                      ldx >= k_off + (int64_t)H * dimp && ldx >= v_off + (int64_t)H * vdimp && ldo >= (int64_t)H * vdimp && ldx % 8 == 0 && k_off % 8 == 0 && v_off % 8 == 0 && ldo % 4 == 0 &&
+                      ldx >= k_off + (int64_t)H * dimp && ldx >= v_off + (int64_t)H * vdimp && ldo >= (int64_t)H * vdimp && ldx % 8 == 0 && k_off % 8 == 0 && v_off % 8 == 0 && ldo % 4 == 0 && ldx < (1 << 24) &&
                       glm_aligned16(x) && (((uintptr_t)o) & 7) == 0, GLM_ERR_INVALID, "glm_memory_chunkwise: bad shape H=%d dim=%d vdimp=%d ldx=%ld", H, dim, vdimp, (long)ldx);
     GLM_CHECK_ARG(dimp <= 256, GLM_ERR_UNSUPPORTED, "glm_memory_chunkwise: key size %d", dimp);
     if (seqs == 0) return GLM_OK;
