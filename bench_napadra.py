@@ -131,8 +131,8 @@ def napadra_kernels(m, meta, mode, B, n):
             2 * B * pairs * 2 * G * d, 4 * B * pairs * H * d)
     else:
         out["attention"] = (
-            [lambda l=l: ops.group_attn_prefill(qkv[:, :nq], l.mixer.k_cache, l.mixer.v_cache, meta.block_tables, meta.n_short, meta.long_q_start, meta.pos, meta.long_tile_seq,
-                                                meta.long_tile_off, *form(l)) for l in own],
+            [lambda l=l: ops.group_attn_prefill(qkv[:, :nq], l.mixer.k_cache, l.mixer.v_cache, meta.block_tables, meta.n_short, meta.long_q_start, meta.pos,
+                                                *meta.chunk_tiles[a.chunk, a.tile_rows], *form(l)) for l in own],
             2 * T * (2 * H + 2 * G) * d, 4 * B * pairs * H * d)
     gemm("gemm memory q|k|v|g", [l.mixer.in_proj for l in mem], h)
     gemm("gemm memory o", [l.mixer.o_proj for l in mem], rnd(T, e.heads * e.vdimp))

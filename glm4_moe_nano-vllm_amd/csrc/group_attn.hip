@@ -4,7 +4,7 @@
 // head (mass exp(sink) in the denominator, without key or value).  Head sizes of keys and values are independent.  gfx950 only.
 //
 //   group_kv_store       rows of a projection -> the pages of both caches, [block][G][tokens of a block][head size]
-//   group_attn_prefill   long portions: 128 query rows of one head per workgroup
+//   group_attn_prefill   long portions: 128 query rows of one head, or 64 of two heads of a group, per workgroup
 //   group_attn_decode    decoded tokens and short portions: 16 (token, head) rows of one key / value head per workgroup, the keys
 //                        split over the waves and over workgroups (glm_attn_merge adds the splits up)
 //   group_attn_plain     any head size, bf16 or fp32: one (token, head) per workgroup, vector FMAs, every step in fp32
@@ -36,7 +36,7 @@ struct GroupArgs {
     int64_t bt_stride;
     const int32_t *pos, *seq_of;  // of the rows of q
     const int32_t *q_start, *tile_a, *tile_b;
-    int seq0, n_tiles, H, G, dk, dv, window, chunk, nsplit;
+    int seq0, n_tiles, H, G, dk, dv, window, chunk, nsplit, pair;  // pair: prefill tiles of 64 rows of two heads
     float scale;
     const float *slope, *sink;  // [H] or nullptr
     const void *knew, *vnew;    // decode: keys / values of the step's own rows, row r at r*ldkv, head g at g*dk / g*dv, or nullptr
@@ -247,28 +247,29 @@ __global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void group_attn_pref
     const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
     const int c = lane & 15, g = lane >> 4;
     // XCD-aware order: workgroups with equal id % 8 share an XCD and take one contiguous run of (head, tile) items
-    const int total = a.n_tiles * a.H, per = (total + 7) >> 3;
+    const int total = a.n_tiles * (a.H >> a.pair), per = (total + 7) >> 3;
     const int item = (blockIdx.x & 7) * per + (blockIdx.x >> 3);
     if ((int)(blockIdx.x >> 3) >= per || item >= total) return;
-    const int h = item / a.n_tiles, tile = item % a.n_tiles, kvh = h / (a.H / a.G);
+    const int h0 = (item / a.n_tiles) << a.pair, tile = item % a.n_tiles, kvh = h0 / (a.H / a.G);
     const int seq = ga_uniform(a.tile_a[tile]), qo = ga_uniform(a.tile_b[tile]);
     const int qs = ga_uniform(a.q_start[seq]), nq = ga_uniform(a.q_start[seq + 1]) - qs;
     if (qo >= nq) return;
-    const int p0 = ga_uniform(a.pos[qs]) + qo, plast = p0 + min(127, nq - 1 - qo);  // positions of the tile's first and last row
+    const int p0 = ga_uniform(a.pos[qs]) + qo, plast = p0 + min((128 >> a.pair) - 1, nq - 1 - qo);  // positions of the tile's first and last row
     const int jlo = ga_first(a, p0) & ~63;
     const int n = ((plast - jlo) >> 6) + 1;
     const int32_t* bt = a.bt + (int64_t)(a.seq0 + seq) * a.bt_stride;
     SL S;
     S.init(lane);
-    const float sl = a.slope ? a.slope[h] / a.scale : 0.f;
-    // this wave's rows: tile t holds rows qo + 64 t + 16 w + c (the two half-dead tiles of the causal edge cost all waves the same)
+    // this wave's rows: tile t holds rows qo + 64 t + 16 w + c of the head (the two half-dead tiles of the causal edge cost all waves the
+    // same) or, of a pair, rows qo + 16 w + c of its head t
+    const int trow = a.pair ? 0 : 64;
 #pragma unroll
     for (int t = 0; t < 2; ++t) {
-        const int r0 = qo + 64 * t + 16 * w, r = r0 + c;
+        const int r0 = qo + trow * t + 16 * w, r = r0 + c, h = h0 + a.pair * t;
         const bool some = r0 < nq;
         S.rp[t] = r < nq ? p0 - qo + r : -1;
         S.rlo[t] = r < nq ? ga_first(a, S.rp[t]) : 0;
-        S.slope[t] = sl;
+        S.slope[t] = a.slope ? a.slope[h] / a.scale : 0.f;
         const int a0 = p0 - qo + r0, a1 = p0 - qo + min(r0 + 15, nq - 1);
         S.any_lo[t] = some ? ga_first(a, a0) : 1 << 30;
         S.any_hi[t] = some ? a1 : -1;
@@ -338,12 +339,12 @@ __global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void group_attn_pref
 #pragma unroll
         for (int s = 1; s >= 0; --s) S.run(kst + s * 32 * KB, vst + s * 32 * VB, jlo + (n - 1 - it) * 64 + s * 32, g, sc);
     }
-    const float sk = a.sink ? a.sink[h] * GA_LOG2E : -INFINITY;
 #pragma unroll
     for (int t = 0; t < 2; ++t) {
         const float l = S.mass(t);
-        const int r = qo + 64 * t + 16 * w + c;
+        const int r = qo + trow * t + 16 * w + c, h = h0 + a.pair * t;
         if (r >= nq) continue;
+        const float sk = a.sink ? a.sink[h] * GA_LOG2E : -INFINITY;
         const float M = fmaxf(S.m_run[t], sk), f = __builtin_amdgcn_exp2f(S.m_run[t] - M);
         const float inv = f / (l * f + __builtin_amdgcn_exp2f(sk - M));
         bf16_t* o = reinterpret_cast<bf16_t*>(a.out) + (int64_t)(qs + r) * a.ldo + (int64_t)h * a.dv;
@@ -627,7 +628,7 @@ int launch_prefill(const GroupArgs& a, hipStream_t st) {
     static_assert(LDS <= 160 * 1024, "LDS of a CU");
     auto kern = group_attn_prefill_kernel<DK, DV>;
     GLM_SET_MAX_LDS(kern, LDS, "glm_group_attn_prefill");
-    const int64_t per = ((int64_t)a.n_tiles * a.H + 7) / 8;
+    const int64_t per = ((int64_t)a.n_tiles * (a.H >> a.pair) + 7) / 8;
     GLM_CHECK_ARG(per * 8 < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_group_attn_prefill: grid too large");
     hipLaunchKernelGGL(kern, dim3((unsigned)(per * 8)), dim3(256), LDS, st, a);
     GLM_CHECK_LAUNCH("glm_group_attn_prefill");
@@ -702,14 +703,16 @@ extern "C" int glm_group_kv_store(const void* src, int64_t ld, int64_t k_off, in
 }
 
 extern "C" int glm_group_attn_prefill(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs, const int32_t* block_tables, int64_t bt_stride, int seq0,
-                                      const int32_t* q_start, const int32_t* pos, const int32_t* tile_seq, const int32_t* tile_off, int n_tiles, int H, int G, int dk, int dv, int window,
-                                      int chunk, float scale, const float* slope, const float* sink, void* out, int64_t ldo, glm_stream_t stream) {
+                                      const int32_t* q_start, const int32_t* pos, const int32_t* tile_seq, const int32_t* tile_off, int n_tiles, int tile_rows, int H, int G, int dk, int dv,
+                                      int window, int chunk, float scale, const float* slope, const float* sink, void* out, int64_t ldo, glm_stream_t stream) {
     GroupArgs a;
     const int rc = group_args(a, "glm_group_attn_prefill", q, ldq, kc, vc, n_blocks, bs, block_tables, bt_stride, seq0, H, G, dk, dv, window, chunk, scale, slope, sink, out, ldo);
     if (rc != GLM_OK) return rc;
     GLM_CHECK_ARG(q_start && pos && tile_seq && tile_off && n_tiles >= 0, GLM_ERR_INVALID, "glm_group_attn_prefill: no tiles");
     GLM_CHECK_ARG(dk <= 256 && dv <= 256 && scale > 0.f, GLM_ERR_UNSUPPORTED, "glm_group_attn_prefill: head sizes up to 256, a positive scale (dk=%d dv=%d)", dk, dv);
+    GLM_CHECK_ARG(tile_rows == 128 || (tile_rows == 64 && (H / G) % 2 == 0), GLM_ERR_UNSUPPORTED, "glm_group_attn_prefill: tiles of %d rows (128, or 64 where heads pair up)", tile_rows);
     if (n_tiles == 0) return GLM_OK;
+    a.pair = tile_rows == 64;
     a.q_start = q_start; a.pos = pos; a.tile_a = tile_seq; a.tile_b = tile_off; a.n_tiles = n_tiles;
     return run_prefill(a, glm_s(stream));
 }

@@ -450,10 +450,11 @@ __device__ __forceinline__ f32x4_t mm_mfma(const bf16x8_t& x, const bf16x8_t& y,
 // is the left operand of the next chunk's readout without leaving the registers.
 template <int D>
 __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(const ChunkArgs a) {
-    constexpr int KS = D / 32, DT = D / 16, RB = D * 2, CPR = D / 8, QT = 64 * RB, VTB = 64 * 128, STAGE = 2 * QT + VTB;
+    constexpr int KS = D / 32, DT = D / 16, RB = D * 2, CPR = D / 8, QT = 64 * RB, VTB = 64 * 128, GT = 1024, STAGE = 2 * QT + VTB + GT;
+    constexpr int NST = D <= 128 ? 3 : 2;           // LDS stages: chunks on their way are NST - 1
     constexpr int QDMA = D / 32, VDMA = 2;          // 1 KiB pieces per wave
     constexpr bool PALIAS = QT >= 16384;            // the weights (hi, lo: 16 KiB) go over the chunk's query rows, which are done by then
-    constexpr int POFF = PALIAS ? 0 : 2 * STAGE, SMALL = 2 * STAGE + (PALIAS ? 0 : 16384);
+    constexpr int POFF = PALIAS ? 0 : NST * STAGE, SMALL = NST * STAGE + (PALIAS ? 0 : 16384);
     extern __shared__ __attribute__((aligned(16))) char smem[];
     float* s_a = reinterpret_cast<float*>(smem + SMALL);  // i_s - b_s                   (log2 units)
     float* s_row = s_a + 64;                               // b_t - m_t                   (log2 units)
@@ -509,8 +510,10 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
     }
     const bool whole = a.dimp == D && vt * 64 + 64 <= a.vdimp;  // no padding columns in this workgroup's tiles
     auto issue = [&](int ch) {
-        char* st = smem + (ch & 1) * STAGE;
+        char* st = smem + (ch % NST) * STAGE;
         const int left = T - ch * 64;
+        // gates: i - b, b and the running maximum, 256 bytes each (the fourth wave's piece is not used)
+        __builtin_amdgcn_global_load_lds((attn_glb_void*)(gp + min(w, 2) * gpart + ch * 64 + min(lane, left - 1)), (attn_lds_void*)(st + 2 * QT + VTB + w * 256), 4, 0, 0);
         const bf16_t *q = xq + (int64_t)ch * 64 * a.ldx, *k = q + a.k_off, *v = xv + (int64_t)ch * 64 * a.ldx;
         if (whole && left >= 64) {
 #pragma unroll
@@ -549,27 +552,39 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
 #pragma unroll
     for (int e = 0; e < 4; ++e) tr_rel[e] = tr * RB + (((2 * e + (pp >> 1)) ^ attn_swz(tr)) << 4) + ((pp & 1) << 3);
     vt_rel = tr * 128 + (((2 * w + (pp >> 1)) ^ attn_swz(tr)) << 4) + ((pp & 1) << 3);
-    // gates of the chunk, one token per lane, the same in every wave
-    float ga, gb, gm;
-    auto load_gates = [&](int ch) {
-        const int64_t t = (int64_t)ch * 64 + lane;
-        const bool on = t < T;
-        ga = on ? gp[t] : -INFINITY;
-        gb = on ? gp[gpart + t] : 0.f;
-        gm = on ? gp[2 * gpart + t] : 0.f;
-    };
     m_in *= MM_LOG2E;
-    load_gates(0);
-    issue(0);
+#pragma unroll
+    for (int i = 0; i < NST - 1; ++i)
+        if (i < n_chunks) issue(i);
     const char* sa = smem + SMALL;
+    // a chunk's output rows are stored behind the next chunk's first barrier: their way to memory is then not waited for
+    u32x2_t rows_out[4];
+    const int vc = vt * 64 + 16 * w + 4 * g;
+    auto store_rows = [&](int ch) {
+        const int left = T - ch * 64;
+        bf16_t* o = a.o + (int64_t)(r0 + ch * 64 + c) * a.ldo + (int64_t)h * a.vdimp + vc;
+#pragma unroll
+        for (int rt = 0; rt < 4; ++rt)
+            if (16 * rt + c < left && vc < a.vdimp) *reinterpret_cast<u32x2_t*>(o + (int64_t)(16 * rt) * a.ldo) = rows_out[rt];
+    };
     for (int ch = 0; ch < n_chunks; ++ch) {
         const int left = T - ch * 64;
-        wait_vm<0>();
+        // the chunk is in (what was issued behind it may be on its way): loads return in order
+        if (ch + NST - 2 < n_chunks) wait_vm<(NST - 2) * (2 * QDMA + VDMA + 1)>();
+        else wait_vm<0>();
+        mm_barrier();  // ... for every wave, and every wave is past its reads of the chunk before
+        if (ch > 0) store_rows(ch - 1);
+        if (ch + NST - 1 < n_chunks) issue(ch + NST - 1);
+        const char *qst = smem + (ch % NST) * STAGE, *kst = qst + QT, *vst = kst + QT, *gst = vst + VTB;
+        char* pst = smem + (PALIAS ? (ch % NST) * STAGE : POFF);
+        // gates of the chunk, one token per lane, the same in every wave
+        const bool tok = lane < left;
+        const float ga = tok ? mm_lds<float>(gst + 4 * lane) : -INFINITY, gb = tok ? mm_lds<float>(gst + 256 + 4 * lane) : 0.f,
+                    gm = tok ? mm_lds<float>(gst + 512 + 4 * lane) : 0.f;
         const float mt = gb + fmaxf(m_in, gm);
         const int last = min(left, 64) - 1;
         const float bL = __shfl(gb, last, 64), mL = __shfl(mt, last, 64);
         const float carry = __builtin_amdgcn_exp2f(bL + m_in - mL);
-        mm_barrier();  // the chunk's rows are in; every wave is past its reads of the chunk before
         if (w == 0) {
             s_a[lane] = ga;
             s_row[lane] = gb - mt;
@@ -577,12 +592,6 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
             s_floor[lane] = __builtin_amdgcn_exp2f(-mt);
             s_w[lane] = __builtin_amdgcn_exp2f(bL - mL + ga);
         }
-        if (ch + 1 < n_chunks) {
-            load_gates(ch + 1);
-            issue(ch + 1);
-        }
-        const char *qst = smem + (ch & 1) * STAGE, *kst = qst + QT, *vst = kst + QT;
-        char* pst = smem + (PALIAS ? (ch & 1) * STAGE : POFF);
         // ---- scores of this wave's 16 query rows, and n . q of them; the readout's query fragments are on their way meanwhile ----
         f32x4_t s[4];
 #pragma unroll
@@ -751,17 +760,14 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
             for (int x = 0; x < 2; ++x)
 #pragma unroll
                 for (int rt = 2 * sl; rt < 4; ++rt) acc[rt] = mm_mfma(vv[sl], __builtin_bit_cast(bf16x8_t, pf[rt][sl][x]), acc[rt]);
-        const int vc = vt * 64 + 16 * w + 4 * g;
 #pragma unroll
         for (int rt = 0; rt < 4; ++rt) {
-            const int t = 16 * rt + c;
             const float inv = __builtin_amdgcn_rcpf(fmaxf(fabsf(dn[rt]), fl[rt]) + 1e-6f);
-            if (t < left && vc < a.vdimp)
-                *reinterpret_cast<u32x2_t*>(a.o + (int64_t)(r0 + ch * 64 + t) * a.ldo + (int64_t)h * a.vdimp + vc) =
-                    u32x2_t{pack2bf(acc[rt][0] * inv, acc[rt][1] * inv), pack2bf(acc[rt][2] * inv, acc[rt][3] * inv)};
+            rows_out[rt] = u32x2_t{pack2bf(acc[rt][0] * inv, acc[rt][1] * inv), pack2bf(acc[rt][2] * inv, acc[rt][3] * inv)};
         }
         m_in = mL;
     }
+    store_rows(n_chunks - 1);
     const int64_t so = a.state_out[seq];
     if (so < 0 || so >= a.n_state) return;
     const int64_t sout = so * a.H + h;
@@ -854,7 +860,7 @@ int run_rec(const RecArgs& a, hipStream_t st) {
 
 template <int D>
 int launch_chunk(const ChunkArgs& a, int seqs, hipStream_t st) {
-    constexpr int STAGE = 2 * 64 * D * 2 + 8192, LDS = 2 * STAGE + (64 * D * 2 >= 16384 ? 0 : 16384) + 6 * 256 + D * 4;
+    constexpr int STAGE = 2 * 64 * D * 2 + 8192 + 1024, LDS = (D <= 128 ? 3 : 2) * STAGE + (64 * D * 2 >= 16384 ? 0 : 16384) + 6 * 256 + D * 4;
     static_assert(LDS <= 160 * 1024, "LDS of a CU");
     auto kern = memory_chunkwise_kernel<D>;
     GLM_SET_MAX_LDS(kern, LDS, "glm_memory_chunkwise");

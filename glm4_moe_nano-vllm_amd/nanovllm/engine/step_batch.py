@@ -55,11 +55,11 @@ LONG_TILE = 128  # query rows of a long portion per workgroup (csrc/window_attn.
 class StepBatch(SimpleNamespace):
     """Device views: ids int64 [T]; pos, seq_of, slots [T]; q_start [S+1]; state_in, state_out [S]; block_tables [S, width];
     want [n]; tiles {tokens per tile: (first row, rows)}; Ta rows of n_short short portions in front, max_short; and, if Ta < T: long_q_start, long_tile_seq,
-    long_tile_off, windows {size: (rows, k_start, crow, hist_slots, hist_rows)}."""
+    long_tile_off, chunk_tiles {(chunk, rows): tiles of that many rows}, windows {size: (rows, k_start, crow, hist_slots, hist_rows)}."""
 
 
 def build_step(chunks: list[Chunk], spec, block_size: int, pad_rows: int = 0, table_width: int = 0):
-    """spec: the model (windows, tile_sizes, max_short_portion).  pad_rows > 0: a decode step of exactly that many rows, the
+    """spec: the model (windows, tile_sizes, max_short_portion; chunk_tiles if it wants some).  pad_rows > 0: a decode step of exactly that many rows, the
     missing ones unused (position -1), with block tables of table_width columns.
     Returns (host int32 buffer, function device buffer -> StepBatch, order of the wanted rows in chunk order)."""
     limit = spec.max_short_portion
@@ -111,7 +111,7 @@ def build_step(chunks: list[Chunk], spec, block_size: int, pad_rows: int = 0, ta
             cnt = np.minimum(size, all_lens[tseq] - k * size)
         tiles[size] = (pk.add(tok), pk.add(cnt))
 
-    longs, windows = None, {}
+    longs, windows, chunk_tiles = None, {}, {}
     if Ta < T:
         L = np.arange(n_short, S)
         n_tiles = -(-all_lens[L] // LONG_TILE)
@@ -119,6 +119,13 @@ def build_step(chunks: list[Chunk], spec, block_size: int, pad_rows: int = 0, ta
         k = np.arange(len(tseq)) - np.repeat(np.cumsum(n_tiles) - n_tiles, n_tiles)
         tseq, k = tseq[::-1], k[::-1]   # a portion's last rows see the most keys: they start first
         longs = (pk.add(q_start[n_short:] - Ta), pk.add(tseq), pk.add(k * LONG_TILE))
+        for c, rows in getattr(spec, "chunk_tiles", ()):            # tiles for attention over chunks, the ones with the most keys first
+            m = -(-all_lens[L] // rows)
+            tseq = np.repeat(np.arange(len(L)), m)
+            off = (np.arange(len(tseq)) - np.repeat(np.cumsum(m) - m, m)) * rows
+            last = starts[n_short:][tseq] + np.minimum(off + rows, all_lens[L][tseq]) - 1   # position of a tile's last row
+            o = np.argsort(-(last % c), kind="stable")
+            chunk_tiles[c, rows] = (pk.add(tseq[o]), pk.add(off[o]))
         for w in spec.windows:
             hist = np.minimum(starts[n_short:], w - 1)           # tokens in front of the portion that its first row still sees
             k_start = np.concatenate([[0], np.cumsum(hist + all_lens[L])])
@@ -138,6 +145,7 @@ def build_step(chunks: list[Chunk], spec, block_size: int, pad_rows: int = 0, ta
         b.ids = b.ids.view(torch.int64)
         if longs is not None:
             b.long_q_start, b.long_tile_seq, b.long_tile_off = (v(i) for i in longs)
+            b.chunk_tiles = {k: (v(q), v(o)) for k, (q, o) in chunk_tiles.items()}
             b.windows = {w: SimpleNamespace(rows=n, k_start=v(a), crow=v(c), hist_slots=v(h), hist_rows=v(r))
                          for w, (n, a, c, h, r) in windows.items()}
         return b

@@ -168,8 +168,8 @@ _SIGNATURES = {
     "glm_group_kv_store": (c_int, [c_void_p, c_int64, c_int64, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int,
         c_int, c_int, c_int, c_void_p]),
     "glm_group_attn_prefill": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p, c_int64, c_int, c_void_p, c_void_p,
-        c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p, c_void_p,
-        c_void_p, c_int64, c_void_p]),
+        c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p,
+        c_void_p, c_void_p, c_int64, c_void_p]),
     "glm_group_attn_decode": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p,
         c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p,
         c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_void_p,
@@ -1522,17 +1522,24 @@ def _group_shape(q, k_cache, v_cache, out, heads, slope, sink):
     return n, G, bs, dk, dv
 
 
+def group_attn_tile_rows(heads: int, kv_heads: int) -> int:
+    """Query rows per workgroup of glm_group_attn_prefill: two heads of a group share a tile where they pair up."""
+    return 64 if (heads // kv_heads) % 2 == 0 else 128
+
+
 def group_attn_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor, seq0: int, q_start: torch.Tensor,
                        pos: torch.Tensor, tile_seq: torch.Tensor, tile_off: torch.Tensor, heads: int, window: int, chunk: int, scale: float, slope, sink,
                        out: torch.Tensor) -> None:
-    """Long portions (rows of q, q_start relative to them) over the paged caches; block table of portion s in row seq0 + s."""
+    """Long portions (rows of q, q_start relative to them) over the paged caches; block table of portion s in row seq0 + s; tiles of
+    group_attn_tile_rows rows."""
     n, G, bs, dk, dv = _group_shape(q, k_cache, v_cache, out, heads, slope, sink)
     for t in (block_tables, q_start, pos, tile_seq, tile_off):
         assert t.dtype == torch.int32
     assert pos.numel() == q.shape[0] and tile_seq.numel() == tile_off.numel() and block_tables.shape[0] >= seq0 + q_start.numel() - 1
     _check(load_library().glm_group_attn_prefill(
         _p(q), q.stride(0), _p(k_cache), _p(v_cache), n, bs, _p(block_tables), block_tables.stride(0), seq0, _p(q_start), _p(pos), _p(tile_seq), _p(tile_off),
-        tile_seq.numel(), heads, G, dk, dv, window, chunk, scale, _p(slope), _p(sink), _p(out), out.stride(0), _stream()), "glm_group_attn_prefill")
+        tile_seq.numel(), group_attn_tile_rows(heads, G), heads, G, dk, dv, window, chunk, scale, _p(slope), _p(sink), _p(out), out.stride(0), _stream()),
+        "glm_group_attn_prefill")
 
 
 def group_attn_splits(tiles: int, tokens_per_tile: int, heads: int, kv_heads: int, keys: int) -> int:

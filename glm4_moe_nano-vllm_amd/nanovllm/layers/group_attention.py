@@ -35,6 +35,7 @@ class GroupAttention(nn.Module):
         # (fp32, and what the tiled kernels do not take: one evaluation for all portions)
         self.tiled = dtype == torch.bfloat16 and scale > 0 and max(self.dimp, self.vdimp) <= hip_ops.GROUP_ATTN_MAX_DIM
         self.tokens_per_tile = max(1, hip_ops.GROUP_ATTN_ROWS // (H // G)) if self.tiled else 1
+        self.tile_rows = hip_ops.group_attn_tile_rows(H, G)
         self.slope = self.sink = self.k_cache = self.v_cache = None
 
     def load(self, w: dict, device) -> None:
@@ -81,8 +82,8 @@ class GroupAttention(nn.Module):
                 new = (x[:Ta, nq: nk], x[:Ta, nk:], meta.q_start, meta.slots) if self.own_kv else None
                 hip_ops.group_attn_decode(q[:Ta], kc, vc, meta.block_tables, meta.pos, meta.seq_of, tok, n, per, *form, out, new=new)
             if Ta < T:
-                hip_ops.group_attn_prefill(q[Ta:], kc, vc, meta.block_tables, meta.n_short, meta.long_q_start, meta.pos[Ta:], meta.long_tile_seq,
-                                           meta.long_tile_off, *form, out[Ta:])
+                hip_ops.group_attn_prefill(q[Ta:], kc, vc, meta.block_tables, meta.n_short, meta.long_q_start, meta.pos[Ta:],
+                                           *meta.chunk_tiles[self.chunk, self.tile_rows], *form, out[Ta:])
         y = self.o_proj(out)
         if self.tp_size > 1:
             get_tp_group().all_reduce(y)

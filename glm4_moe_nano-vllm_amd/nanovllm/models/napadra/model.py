@@ -98,6 +98,10 @@ class NapadraForCausalLM(nn.Module):
         return [layer.mixer for layer in self.layers if isinstance(layer.mixer, GroupAttention)]
 
     @property
+    def chunk_tiles(self) -> list[tuple]:
+        return sorted({(m.chunk, m.tile_rows) for m in self._attention})
+
+    @property
     def tile_sizes(self) -> list[int]:
         return sorted({m.tokens_per_tile for m in self._attention})
 

@@ -542,7 +542,7 @@ int glm_stream_norm(const float* x_in, int64_t ldx, int64_t sx, const int32_t* r
  * dk, dv multiples of 8).  A row at position p sees j <= p with p - j < window (window > 0) and in its own chunk of `chunk` positions
  * (chunk > 0); score = scale q.k - slope[h] (p - j) (slope may be NULL); softmax with the extra mass exp(sink[h]) (sink may be NULL).
  * store: key / value columns of projection rows -> cache rows slots[t] (< 0: none).
- * prefill: 128-row tiles (sequence, first row inside the portion) of portions [q_start[s], q_start[s+1]), block table row seq0 + s.
+ * prefill: tiles (sequence, first row inside the portion) of tile_rows rows (128; 64 if H/G is even) of portions [q_start[s], q_start[s+1]), block table row seq0 + s.
  * decode: tiles of tile_n[i] <= tokens_per_tile rows of one sequence from tile_tok[i]; nsplit > 1: unnormalised sums part_o
  * [rows*H, nsplit, dv] and part_ml [rows*H, nsplit, 2] for glm_attn_merge; knew / vnew (may be NULL): keys and values of the rows of q,
  * head g at g*dk / g*dv, read instead of the cache's and stored to cache rows `slots`.  Both bf16, dk, dv <= 256, scale > 0.  plain: any size, bf16 or fp32.  */
@@ -550,8 +550,8 @@ int glm_group_kv_store(const void* src, int64_t ld, int64_t k_off, int64_t v_off
                        void* kc, void* vc, int64_t n_slots, int bs, int G, int dk, int dv, glm_stream_t stream);
 int glm_group_attn_prefill(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs,
                            const int32_t* block_tables, int64_t bt_stride, int seq0, const int32_t* q_start, const int32_t* pos,
-                           const int32_t* tile_seq, const int32_t* tile_off, int n_tiles, int H, int G, int dk, int dv, int window,
-                           int chunk, float scale, const float* slope, const float* sink, void* out, int64_t ldo,
+                           const int32_t* tile_seq, const int32_t* tile_off, int n_tiles, int tile_rows, int H, int G, int dk,
+                           int dv, int window, int chunk, float scale, const float* slope, const float* sink, void* out, int64_t ldo,
                            glm_stream_t stream);
 int glm_group_attn_decode(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs,
                           const int32_t* block_tables, int64_t bt_stride, const int32_t* pos, const int32_t* seq_of,

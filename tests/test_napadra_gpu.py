@@ -230,7 +230,7 @@ def test_group_attention(H, G, dk, dv, window, chunk, bs, kind):
             rows = dev(rows, dt)
             new = (rows[:, : G * dk], rows[:, G * dk:], i32(qs), i32(slots))
         if kind == "prefill":
-            tiles = [(s, o) for s, n in enumerate(n_q) for o in range(0, n, 128)]
+            tiles = [(s, o) for s, n in enumerate(n_q) for o in range(0, n, hip_ops.group_attn_tile_rows(H, G))]
             wide = torch.full((3 + bt.shape[0], bt.shape[1]), -1, dtype=torch.int32)
             wide[3:] = bt       # portions whose block tables are not the first rows
             hip_ops.group_attn_prefill(*args[:3], i32(wide), 3, i32(qs), pos, i32([t[0] for t in tiles]), i32([t[1] for t in tiles]), *form, out)
