@@ -124,7 +124,7 @@ def build_step(chunks: list[Chunk], spec, block_size: int, pad_rows: int = 0, ta
             tseq = np.repeat(np.arange(len(L)), m)
             off = (np.arange(len(tseq)) - np.repeat(np.cumsum(m) - m, m)) * rows
             last = starts[n_short:][tseq] + np.minimum(off + rows, all_lens[L][tseq]) - 1   # position of a tile's last row
-            o = np.argsort(-(last % c), kind="stable")
+            o = np.argsort(-(last % c if c else last), kind="stable")
             chunk_tiles[c, rows] = (pk.add(tseq[o]), pk.add(off[o]))
         for w in spec.windows:
             hist = np.minimum(starts[n_short:], w - 1)           # tokens in front of the portion that its first row still sees

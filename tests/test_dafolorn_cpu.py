@@ -182,7 +182,7 @@ def _drive(sch, seqs, check=lambda batch: None, window=50):
         for seq, c in batch:
             assert c.start == seq.num_computed_tokens and c.tokens == seq.token_ids[c.start: c.start + len(c.tokens)]
             assert len(c.block_table) * 32 >= c.start + len(c.tokens)
-            first = max(0, c.start - window + 1)
+            first = max(0, c.start - window + 1)   # (window 0: the caller checks the blocks)
             assert all(b >= 0 for b in c.block_table[first // 32: -(-(c.start + len(c.tokens)) // 32)])
             assert {c.state_in, c.state_out} == {2 * seq.state_slot, 2 * seq.state_slot + 1}
             if c.want:
