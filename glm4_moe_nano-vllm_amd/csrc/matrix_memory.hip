@@ -445,26 +445,30 @@ __device__ __forceinline__ bf16x8_t mm_frag(const u32x2_t& x, const u32x2_t& y) 
 __device__ __forceinline__ f32x4_t mm_f4(const u32x4_t& v) { return __builtin_bit_cast(f32x4_t, v); }
 __device__ __forceinline__ f32x4_t mm_mfma(const bf16x8_t& x, const bf16x8_t& y, const f32x4_t& z) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(x, y, z, 0, 0, 0); }
 
-// D: multiple of 64, dimp <= D <= 256.  Four waves; wave w computes the scores of query rows 16 w .. + 15 and owns value columns
-// 16 w .. + 15 of the tile's 64: their state S[d][column], in the matrix cores' output layout (lane (c, g): column c, rows d = 16 i + 4 g + r),
-// is the left operand of the next chunk's readout without leaving the registers.
+// D: multiple of 64, dimp <= D <= 256.  Eight waves; wave (v, dh) = (w & 3, w >> 2) computes the scores of query rows 16 v .. + 15 with half dh
+// of the keys, and owns the part d in half dh, value columns 16 v .. + 15 of the state.  That part, in the matrix cores' output layout
+// (lane (c, g): column c, rows d = 16 i + 4 g + r), is the left operand of the next chunk's readout without leaving the registers.  Of
+// the 64 output rows, half 0 finishes row tiles 0 and 3, half 1 tiles 1 and 2 (equal work under the causal mask); the readouts of the
+// other half come through LDS.
 template <int D>
-__global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(const ChunkArgs a) {
-    constexpr int KS = D / 32, DT = D / 16, RB = D * 2, CPR = D / 8, QT = 64 * RB, VTB = 64 * 128, GT = 1024, STAGE = 2 * QT + VTB + GT;
+__global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArgs a) {
+    constexpr int KS = D / 32, DT = D / 16, HT = DT / 2, RB = D * 2, CPR = D / 8, QT = 64 * RB, VTB = 64 * 128, GT = 1024, STAGE = 2 * QT + VTB + GT;
     constexpr int NST = D <= 128 ? 3 : 2;           // LDS stages: chunks on their way are NST - 1
-    constexpr int QDMA = D / 32, VDMA = 2;          // 1 KiB pieces per wave
-    constexpr bool PALIAS = QT >= 16384;            // the weights (hi, lo: 16 KiB) go over the chunk's query rows, which are done by then
-    constexpr int POFF = PALIAS ? 0 : NST * STAGE, SMALL = NST * STAGE + (PALIAS ? 0 : 16384);
+    constexpr int QDMA = D / 64;                    // 1 KiB pieces per wave (of q, of k; one of v, one of the gates)
+    // the weights (hi, lo: 16 KiB) and the readouts that change hands (16 KiB) go over the chunk's query rows, which are done by then, as far as
+    // these reach
+    constexpr bool PALIAS = QT >= 16384, XALIAS = QT >= 32768;
+    constexpr int POFF = PALIAS ? 0 : NST * STAGE, XOFF = XALIAS ? 16384 : NST * STAGE + (PALIAS ? 0 : 16384), SMALL = NST * STAGE + (PALIAS ? 0 : 16384) + (XALIAS ? 0 : 16384);
     extern __shared__ __attribute__((aligned(16))) char smem[];
     float* s_a = reinterpret_cast<float*>(smem + SMALL);  // i_s - b_s                   (log2 units)
     float* s_row = s_a + 64;                               // b_t - m_t                   (log2 units)
     float* s_in = s_row + 64;                              // c_t dim^-1/2
     float* s_floor = s_in + 64;                            // e^(-m_t)
     float* s_w = s_floor + 64;                             // e^(b_L - m_L + i_s - b_s)
-    float* s_den = s_w + 64;                               // n_t . q_t
-    float* s_n = s_den + 64;                               // [D]
+    float* s_den = s_w + 64;                               // n_t . q_t, two parts [2][64]
+    float* s_n = s_den + 128;                              // [D]
     const int tid = threadIdx.x, lane = tid & 63;
-    const int w = __builtin_amdgcn_readfirstlane(tid >> 6);
+    const int w = __builtin_amdgcn_readfirstlane(tid >> 6), v = w & 3, dh = w >> 2;
     const int c = lane & 15, g = lane >> 4;
     const int vt = blockIdx.x % a.vtiles, h = (blockIdx.x / a.vtiles) % a.H, seq = blockIdx.x / (a.vtiles * a.H);
     const int r0 = a.q_start[seq], T = a.q_start[seq + 1] - r0;
@@ -472,23 +476,24 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
     const int n_chunks = (T + 63) >> 6;
     const bool fresh = a.pos[r0] <= 0;
     const int64_t sin = min(max((int64_t)a.state_in[seq], (int64_t)0), a.n_state - 1) * a.H + h;
-    const int col = vt * 64 + 16 * w + c;  // this lane's value column
+    const int col = vt * 64 + 16 * v + c;  // this lane's value column
     const bool con = col < a.vdimp;
-    f32x4_t S[DT];
+    f32x4_t S[HT];
 #pragma unroll
-    for (int i = 0; i < DT; ++i)
+    for (int i = 0; i < HT; ++i)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            const int d = 16 * i + 4 * g + r;
+            const int d = 16 * (dh * HT + i) + 4 * g + r;
             S[i][r] = (!fresh && con && d < a.dimp) ? a.S[(sin * a.dimp + d) * a.vdimp + col] : 0.f;
         }
-    // wave w keeps n of the rows d = 16 i + c with i = w mod 4 (the same in all four lane groups)
-    float nreg[DT / 4];
+    // n of the rows d = 16 (dh HT + i) + c with i = v mod 4 (the same in all four lane groups)
+    constexpr int NR = HT > 4 ? HT / 4 : 1;
+    float nreg[NR];
 #pragma unroll
-    for (int i = 0; i < DT / 4; ++i) {
-        const int d = 16 * (4 * i + w) + c;
-        nreg[i] = (!fresh && d < a.dimp) ? a.n[sin * a.dimp + d] : 0.f;
-        if (g == 0) s_n[d] = nreg[i];
+    for (int i = 0; i < NR; ++i) {
+        const int d = 16 * (dh * HT + 4 * i + v) + c;
+        nreg[i] = (!fresh && v < HT && d < a.dimp) ? a.n[sin * a.dimp + d] : 0.f;
+        if (g == 0 && v < HT) s_n[d] = nreg[i];
     }
     float m_in = fresh ? 0.f : a.m[sin];
     const float scale = 1.0f / sqrtf((float)a.dim);
@@ -497,32 +502,28 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
     const float* gp = a.gates + (int64_t)h * a.rows + r0;
     const int64_t gpart = (int64_t)a.H * a.rows;
     // per-lane source offsets of the DMA pieces: constant over the chunks
-    unsigned qoff[QDMA], voff[VDMA];
+    unsigned qoff[QDMA];
 #pragma unroll
     for (int i = 0; i < QDMA; ++i) {
         const int p = (w * QDMA + i) * 64 + lane, row = p / CPR;
         qoff[i] = (unsigned)(row * (int)a.ldx + ((p % CPR) ^ attn_swz(row)) * 8);
     }
-#pragma unroll
-    for (int i = 0; i < VDMA; ++i) {
-        const int p = (w * VDMA + i) * 64 + lane, row = p >> 3;
-        voff[i] = (unsigned)(row * (int)a.ldx + ((p & 7) ^ attn_swz(row)) * 8);
-    }
+    const int vrow = w * 8 + (lane >> 3), vcc = (lane & 7) ^ attn_swz(vrow);
+    const unsigned voff = (unsigned)(vrow * (int)a.ldx + vcc * 8);
     const bool whole = a.dimp == D && vt * 64 + 64 <= a.vdimp;  // no padding columns in this workgroup's tiles
     auto issue = [&](int ch) {
         char* st = smem + (ch % NST) * STAGE;
         const int left = T - ch * 64;
-        // gates: i - b, b and the running maximum, 256 bytes each (the fourth wave's piece is not used)
-        __builtin_amdgcn_global_load_lds((attn_glb_void*)(gp + min(w, 2) * gpart + ch * 64 + min(lane, left - 1)), (attn_lds_void*)(st + 2 * QT + VTB + w * 256), 4, 0, 0);
-        const bf16_t *q = xq + (int64_t)ch * 64 * a.ldx, *k = q + a.k_off, *v = xv + (int64_t)ch * 64 * a.ldx;
+        // gates: i - b, b and the running maximum, 256 bytes each (the other waves' piece is not used)
+        __builtin_amdgcn_global_load_lds((attn_glb_void*)(gp + min(w, 2) * gpart + ch * 64 + min(lane, left - 1)), (attn_lds_void*)(st + 2 * QT + VTB + min(w, 3) * 256), 4, 0, 0);
+        const bf16_t *q = xq + (int64_t)ch * 64 * a.ldx, *k = q + a.k_off, *vv = xv + (int64_t)ch * 64 * a.ldx;
         if (whole && left >= 64) {
 #pragma unroll
             for (int i = 0; i < QDMA; ++i) {
                 lds_dma16(q + qoff[i], st + (w * QDMA + i) * 1024);
                 lds_dma16(k + qoff[i], st + QT + (w * QDMA + i) * 1024);
             }
-#pragma unroll
-            for (int i = 0; i < VDMA; ++i) lds_dma16(v + voff[i], st + 2 * QT + (w * VDMA + i) * 1024);
+            lds_dma16(vv + voff, st + 2 * QT + w * 1024);
             return;
         }
 #pragma unroll
@@ -532,12 +533,8 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
             lds_dma16(ok ? (const void*)(q + qoff[i]) : (const void*)mm_zero_page, st + (w * QDMA + i) * 1024);
             lds_dma16(ok ? (const void*)(k + qoff[i]) : (const void*)mm_zero_page, st + QT + (w * QDMA + i) * 1024);
         }
-#pragma unroll
-        for (int i = 0; i < VDMA; ++i) {
-            const int p = (w * VDMA + i) * 64 + lane, row = p >> 3, cc = (p & 7) ^ attn_swz(row);
-            const bool ok = row < left && vt * 64 + cc * 8 < a.vdimp;
-            lds_dma16(ok ? (const void*)(v + voff[i]) : (const void*)mm_zero_page, st + 2 * QT + (w * VDMA + i) * 1024);
-        }
+        const bool ok = vrow < left && vt * 64 + vcc * 8 < a.vdimp;
+        lds_dma16(ok ? (const void*)(vv + voff) : (const void*)mm_zero_page, st + 2 * QT + w * 1024);
     };
     // fragment offsets.  Rows by 16 (lane c), eight columns 32 i + 8 g: the scores.  Rows by 16, columns 32 i + 4 g and + 16: the readout,
     // in the order of the state's registers.  Transposed reads, rows 4 g + qq: k and v over tokens.
@@ -551,32 +548,32 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
     const int qq = (lane >> 2) & 3, pp = lane & 3, tr = 4 * g + qq;
 #pragma unroll
     for (int e = 0; e < 4; ++e) tr_rel[e] = tr * RB + (((2 * e + (pp >> 1)) ^ attn_swz(tr)) << 4) + ((pp & 1) << 3);
-    vt_rel = tr * 128 + (((2 * w + (pp >> 1)) ^ attn_swz(tr)) << 4) + ((pp & 1) << 3);
+    vt_rel = tr * 128 + (((2 * v + (pp >> 1)) ^ attn_swz(tr)) << 4) + ((pp & 1) << 3);
+    const int rt_a = dh ? 1 : 0, rt_b = dh ? 2 : 3;   // the output row tiles this wave finishes
     m_in *= MM_LOG2E;
 #pragma unroll
     for (int i = 0; i < NST - 1; ++i)
         if (i < n_chunks) issue(i);
     const char* sa = smem + SMALL;
     // a chunk's output rows are stored behind the next chunk's first barrier: their way to memory is then not waited for
-    u32x2_t rows_out[4];
-    const int vc = vt * 64 + 16 * w + 4 * g;
+    u32x2_t rows_out[2];
+    const int vc = vt * 64 + 16 * v + 4 * g;
     auto store_rows = [&](int ch) {
         const int left = T - ch * 64;
         bf16_t* o = a.o + (int64_t)(r0 + ch * 64 + c) * a.ldo + (int64_t)h * a.vdimp + vc;
-#pragma unroll
-        for (int rt = 0; rt < 4; ++rt)
-            if (16 * rt + c < left && vc < a.vdimp) *reinterpret_cast<u32x2_t*>(o + (int64_t)(16 * rt) * a.ldo) = rows_out[rt];
+        if (16 * rt_a + c < left && vc < a.vdimp) *reinterpret_cast<u32x2_t*>(o + (int64_t)(16 * rt_a) * a.ldo) = rows_out[0];
+        if (16 * rt_b + c < left && vc < a.vdimp) *reinterpret_cast<u32x2_t*>(o + (int64_t)(16 * rt_b) * a.ldo) = rows_out[1];
     };
     for (int ch = 0; ch < n_chunks; ++ch) {
         const int left = T - ch * 64;
         // the chunk is in (what was issued behind it may be on its way): loads return in order
-        if (ch + NST - 2 < n_chunks) wait_vm<(NST - 2) * (2 * QDMA + VDMA + 1)>();
+        if (ch + NST - 2 < n_chunks) wait_vm<(NST - 2) * (2 * QDMA + 2)>();
         else wait_vm<0>();
         mm_barrier();  // ... for every wave, and every wave is past its reads of the chunk before
         if (ch > 0) store_rows(ch - 1);
         if (ch + NST - 1 < n_chunks) issue(ch + NST - 1);
         const char *qst = smem + (ch % NST) * STAGE, *kst = qst + QT, *vst = kst + QT, *gst = vst + VTB;
-        char* pst = smem + (PALIAS ? (ch % NST) * STAGE : POFF);
+        char *pst = smem + (PALIAS ? (ch % NST) * STAGE : POFF), *xst = smem + (XALIAS ? (ch % NST) * STAGE : 0) + XOFF;
         // gates of the chunk, one token per lane, the same in every wave
         const bool tok = lane < left;
         const float ga = tok ? mm_lds<float>(gst + 4 * lane) : -INFINITY, gb = tok ? mm_lds<float>(gst + 256 + 4 * lane) : 0.f,
@@ -592,132 +589,117 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
             s_floor[lane] = __builtin_amdgcn_exp2f(-mt);
             s_w[lane] = __builtin_amdgcn_exp2f(bL - mL + ga);
         }
-        // ---- scores of this wave's 16 query rows, and n . q of them; the readout's query fragments are on their way meanwhile ----
-        f32x4_t s[4];
-#pragma unroll
-        for (int kt = 0; kt < 4; ++kt) s[kt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+        // ---- scores of 16 query rows with 32 keys; n . q of these rows, over this half's d ----
+        f32x4_t s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
         float nq = 0.f;
+        static_for<KS>([&](auto I) {
+            constexpr int i = decltype(I)::value;
+            const u32x4_t qf = mm_lds<u32x4_t>(qst + v * 16 * RB + row_rel[i & 1] + (i >> 1) * 128);
+            const u32x4_t k0 = mm_lds<u32x4_t>(kst + dh * 32 * RB + row_rel[i & 1] + (i >> 1) * 128), k1 = mm_lds<u32x4_t>(kst + dh * 32 * RB + row_rel[i & 1] + (i >> 1) * 128 + 16 * RB);
+            s[0] = mm_mfma(__builtin_bit_cast(bf16x8_t, k0), __builtin_bit_cast(bf16x8_t, qf), s[0]);
+            s[1] = mm_mfma(__builtin_bit_cast(bf16x8_t, k1), __builtin_bit_cast(bf16x8_t, qf), s[1]);
+            if (i / (KS / 2) == dh) {
+                const f32x4_t n0 = mm_lds<f32x4_t>(sa + 1792 + 128 * i + 32 * g), n1 = mm_lds<f32x4_t>(sa + 1792 + 128 * i + 32 * g + 16);
+#pragma unroll
+                for (int e = 0; e < 2; ++e) {
+                    nq = fmaf(bflo(qf[e]), n0[2 * e], nq);
+                    nq = fmaf(bfhi(qf[e]), n0[2 * e + 1], nq);
+                    nq = fmaf(bflo(qf[2 + e]), n1[2 * e], nq);
+                    nq = fmaf(bfhi(qf[2 + e]), n1[2 * e + 1], nq);
+                }
+            }
+        });
+        // ---- what this part of the state gives all 64 rows, in this wave's columns ----
         f32x4_t acc[4];
 #pragma unroll
         for (int rt = 0; rt < 4; ++rt) acc[rt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
-        static_for<KS / 2>([&](auto I2) {
-            constexpr int i0 = 2 * decltype(I2)::value;
-            u32x4_t qf[2], kf[2][4], nf[2][2];
-            u32x2_t qh[2][4][2];
-            static_for<2>([&](auto J) {
-                constexpr int jj = decltype(J)::value, i = i0 + jj;
-                qf[jj] = mm_lds<u32x4_t>(qst + w * 16 * RB + row_rel[i & 1] + ((i >> 1) * 128));
-                static_for<4>([&](auto KT) { kf[jj][decltype(KT)::value] = mm_lds<u32x4_t>(kst + row_rel[i & 1] + ((i >> 1) * 128 + decltype(KT)::value * 16 * RB)); });
-                nf[jj][0] = mm_lds<u32x4_t>(sa + 32 * g + (1536 + 128 * i));
-                nf[jj][1] = mm_lds<u32x4_t>(sa + 32 * g + (1536 + 128 * i + 16));
-            });
-            static_for<2>([&](auto J) {
-                constexpr int jj = decltype(J)::value, i = i0 + jj;
-                static_for<4>([&](auto RT) {
-                    constexpr int rt = decltype(RT)::value;
-                    qh[jj][rt][0] = mm_lds<u32x2_t>(qst + half_rel[i & 1][0] + ((i >> 1) * 128 + rt * 16 * RB));
-                    qh[jj][rt][1] = mm_lds<u32x2_t>(qst + half_rel[i & 1][1] + ((i >> 1) * 128 + rt * 16 * RB));
-                });
-            });
-            bf16x8_t hi[2], lo[2];
+        const char* qh_st = qst + (KS / 2 >= 2 ? dh * (KS / 4) * 128 : 0);   // columns of this half: 128 bytes hold 64 of them
+        static_for<KS / 2>([&](auto I) {
+            constexpr int i = decltype(I)::value;
+            const unsigned ra = KS / 2 >= 2 ? half_rel[i & 1][0] : (dh ? half_rel[1][0] : half_rel[0][0]), rb = KS / 2 >= 2 ? half_rel[i & 1][1] : (dh ? half_rel[1][1] : half_rel[0][1]);
+            const f32x4_t &u = S[2 * i], &x = S[2 * i + 1];
+            const float sv[8] = {u[0], u[1], u[2], u[3], x[0], x[1], x[2], x[3]};
+            bf16x8_t hi, lo, q[4];
+            mm_split(sv, hi, lo);
 #pragma unroll
-            for (int jj = 0; jj < 2; ++jj) {
-                const f32x4_t &u = S[2 * (i0 + jj)], &v = S[2 * (i0 + jj) + 1];
-                const float sv[8] = {u[0], u[1], u[2], u[3], v[0], v[1], v[2], v[3]};
-                mm_split(sv, hi[jj], lo[jj]);
-            }
+            for (int rt = 0; rt < 4; ++rt) q[rt] = mm_frag(mm_lds<u32x2_t>(qh_st + ra + (i >> 1) * 128 + rt * 16 * RB), mm_lds<u32x2_t>(qh_st + rb + (i >> 1) * 128 + rt * 16 * RB));
 #pragma unroll
-            for (int jj = 0; jj < 2; ++jj)
+            for (int rt = 0; rt < 4; ++rt) acc[rt] = mm_mfma(hi, q[rt], acc[rt]);
 #pragma unroll
-                for (int kt = 0; kt < 4; ++kt) s[kt] = mm_mfma(__builtin_bit_cast(bf16x8_t, kf[jj][kt]), __builtin_bit_cast(bf16x8_t, qf[jj]), s[kt]);
-#pragma unroll
-            for (int jj = 0; jj < 2; ++jj) {
-                const f32x4_t n0 = mm_f4(nf[jj][0]), n1 = mm_f4(nf[jj][1]);
-#pragma unroll
-                for (int e = 0; e < 2; ++e) {
-                    nq = fmaf(bflo(qf[jj][e]), n0[2 * e], nq);
-                    nq = fmaf(bfhi(qf[jj][e]), n0[2 * e + 1], nq);
-                    nq = fmaf(bflo(qf[jj][2 + e]), n1[2 * e], nq);
-                    nq = fmaf(bfhi(qf[jj][2 + e]), n1[2 * e + 1], nq);
-                }
-            }
-            // ---- what the state gives all 64 rows, in this wave's columns ----
-#pragma unroll
-            for (int jj = 0; jj < 2; ++jj)
-#pragma unroll
-                for (int x = 0; x < 2; ++x)
-#pragma unroll
-                    for (int rt = 0; rt < 4; ++rt) acc[rt] = mm_mfma(x ? lo[jj] : hi[jj], mm_frag(qh[jj][rt][0], qh[jj][rt][1]), acc[rt]);
-            asm volatile("" ::: "memory");  // one group's fragments at a time
+            for (int rt = 0; rt < 4; ++rt) acc[rt] = mm_mfma(lo, q[rt], acc[rt]);
         });
-        // ---- operands of the state's update: values and keys over tokens ----
+        f32x4_t o_a = dh ? acc[1] : acc[0], o_b = dh ? acc[2] : acc[3];
+        const f32x4_t x_a = dh ? acc[0] : acc[1], x_b = dh ? acc[3] : acc[2];   // for the other half
+        // ---- operands of the state's update: values over tokens ----
         u32x2_t vf[2][2];
         mm_lds_tr4<0, 16 * 128, 32 * 128, 48 * 128>(vf, vst + vt_rel);
         mm_barrier();  // query rows read, gate arrays written
         const bf16x8_t vv[2] = {mm_frag(vf[0][0], vf[0][1]), mm_frag(vf[1][0], vf[1][1])};
-        // ---- weights of this wave's rows: hi and lo, in the order the second product reads them ----
-        const int row = 16 * w + c;
-        u32x4_t av[4], wq[4];
-        static_for<4>([&](auto X) { av[decltype(X)::value] = mm_lds<u32x4_t>(sa + 16 * g + (decltype(X)::value * 64)); });
-        static_for<4>([&](auto X) { wq[decltype(X)::value] = mm_lds<u32x4_t>(sa + 16 * g + (1024 + decltype(X)::value * 64)); });
-        float rowc, inc;
-        rowc = mm_lds<float>(sa + 4 * row + (256));
-        inc = mm_lds<float>(sa + 4 * row + (512));
-        float dsum = 0.f;
-#pragma unroll
-        for (int sl = 0; sl < 2; ++sl) {
-            float p[8];
+        // ---- weights of this wave's rows and keys: hi and lo, in the order the second product reads them ----
+        const int row = 16 * v + c;
+        const float rowc = mm_lds<float>(sa + 256 + 4 * row), inc = mm_lds<float>(sa + 512 + 4 * row);
+        {
+            *reinterpret_cast<f32x4_t*>(xst + (w * 2 * 64 + lane) * 16) = x_a;
+            *reinterpret_cast<f32x4_t*>(xst + ((w * 2 + 1) * 64 + lane) * 16) = x_b;
+            float p[8], dsum = 0.f;
 #pragma unroll
             for (int u = 0; u < 2; ++u) {
-                const int k0 = 32 * sl + 16 * u + 4 * g;
-                const f32x4_t ax = mm_f4(av[2 * sl + u]);
+                const int k0 = 32 * dh + 16 * u + 4 * g;
+                const f32x4_t ax = mm_lds<f32x4_t>(sa + 4 * k0);
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
                     const float dw = k0 + r <= row ? __builtin_amdgcn_exp2f(rowc + ax[r]) * scale : 0.f;
-                    p[4 * u + r] = s[2 * sl + u][r] * dw;
+                    p[4 * u + r] = s[u][r] * dw;
                     dsum += p[4 * u + r];
                 }
             }
             bf16x8_t hi, lo;
             mm_split(p, hi, lo);
-            const int chunk = ((4 * sl + g) ^ (c & 7)) << 4;
+            const int chunk = ((4 * dh + g) ^ (c & 7)) << 4;
             *reinterpret_cast<bf16x8_t*>(pst + row * 128 + chunk) = hi;
             *reinterpret_cast<bf16x8_t*>(pst + 8192 + row * 128 + chunk) = lo;
+            nq = fmaf(nq, inc, dsum);
+            nq += __shfl_xor(nq, 16, 64);
+            nq += __shfl_xor(nq, 32, 64);
+            if (g == 0) s_den[64 * dh + row] = nq;
         }
-        nq = fmaf(nq, inc, dsum);
-        nq += __shfl_xor(nq, 16, 64);
-        nq += __shfl_xor(nq, 32, 64);
-        if (g == 0) s_den[row] = nq;
         // ---- state of the next chunk ----
         bf16x8_t vhi[2], vlo[2];
         float wt[2][8];
 #pragma unroll
         for (int sl = 0; sl < 2; ++sl) {
+            const f32x4_t w0 = mm_lds<f32x4_t>(sa + 1024 + 128 * sl + 16 * g), w1 = mm_lds<f32x4_t>(sa + 1024 + 128 * sl + 64 + 16 * g);
             float p[8];
 #pragma unroll
             for (int e = 0; e < 8; ++e) {
-                wt[sl][e] = mm_f4(wq[2 * sl + (e >> 2)])[e & 3];
+                wt[sl][e] = e < 4 ? w0[e & 3] : w1[e & 3];
                 p[e] = wt[sl][e] * (float)vv[sl][e];
             }
             mm_split(p, vhi[sl], vlo[sl]);
         }
-        static_for<DT / 4>([&](auto I4) {
-            constexpr int i0 = 4 * decltype(I4)::value;
-            u32x2_t kf[4][2][2];
-            const unsigned kb = lds_addr(kst) + (i0 >> 2) * 128;
-            mm_lds_tr16<RB>(kf, kb + tr_rel[0], kb + tr_rel[1], kb + tr_rel[2], kb + tr_rel[3]);
+        constexpr int GI = HT >= 4 ? 4 : HT;   // row tiles of the state per group of reads
+        static_for<HT / GI>([&](auto I4) {
+            constexpr int i0 = GI * decltype(I4)::value;
+            u32x2_t kf[GI][2][2];
+            if constexpr (GI == 4) {
+                const unsigned kb = lds_addr(kst) + (dh * HT / 4 + (i0 >> 2)) * 128;
+                mm_lds_tr16<RB>(kf, kb + tr_rel[0], kb + tr_rel[1], kb + tr_rel[2], kb + tr_rel[3]);
+            } else {
 #pragma unroll
-            for (int jj = 0; jj < 4; ++jj) S[i0 + jj] *= carry;
+                for (int jj = 0; jj < GI; ++jj) mm_lds_tr4<0, 16 * RB, 32 * RB, 48 * RB>(kf[jj], kst + (dh ? tr_rel[2 + jj] : tr_rel[jj]));
+            }
+#pragma unroll
+            for (int jj = 0; jj < GI; ++jj) S[i0 + jj] *= carry;
 #pragma unroll
             for (int sl = 0; sl < 2; ++sl)
 #pragma unroll
                 for (int x = 0; x < 2; ++x)
 #pragma unroll
-                    for (int jj = 0; jj < 4; ++jj) S[i0 + jj] = mm_mfma(mm_frag(kf[jj][sl][0], kf[jj][sl][1]), x ? vlo[sl] : vhi[sl], S[i0 + jj]);
-            float nn = 0.f;   // n of the rows 16 (i0 + w) + c
+                    for (int jj = 0; jj < GI; ++jj) S[i0 + jj] = mm_mfma(mm_frag(kf[jj][sl][0], kf[jj][sl][1]), x ? vlo[sl] : vhi[sl], S[i0 + jj]);
+            float nn = 0.f;   // n of the rows 16 (dh HT + i0 + v) + c
 #pragma unroll
-            for (int jj = 0; jj < 4; ++jj) {
-                if (jj != w) continue;
+            for (int jj = 0; jj < GI; ++jj) {
+                if (jj != v) continue;
 #pragma unroll
                 for (int sl = 0; sl < 2; ++sl) {
                     const bf16x8_t k = mm_frag(kf[jj][sl][0], kf[jj][sl][1]);
@@ -731,40 +713,30 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
         });
         mm_barrier();
         // ---- output rows ----
-        u32x4_t pf[4][2][2];
-        const char *pa0 = pst + c * 128 + ((g ^ (c & 7)) << 4), *pa1 = pst + c * 128 + (((4 + g) ^ (c & 7)) << 4);
-        float in[4], dn[4], fl[4];
-        static_for<4>([&](auto RT) {
-            constexpr int rt = decltype(RT)::value;
-            pf[rt][0][0] = mm_lds<u32x4_t>(pa0 + (rt * 2048));
-            pf[rt][0][1] = mm_lds<u32x4_t>(pa0 + (rt * 2048 + 8192));
-            if constexpr (rt >= 2) {  // keys 32 .. 63 of rows 0 .. 31 are all in the future
-                pf[rt][1][0] = mm_lds<u32x4_t>(pa1 + (rt * 2048));
-                pf[rt][1][1] = mm_lds<u32x4_t>(pa1 + (rt * 2048 + 8192));
-            }
-            in[rt] = mm_lds<float>(sa + 4 * c + (512 + 64 * rt));
-            fl[rt] = mm_lds<float>(sa + 4 * c + (768 + 64 * rt));
-            dn[rt] = mm_lds<float>(sa + 4 * c + (1280 + 64 * rt));
-        });
-        if (g == 0) {
+        if (g == 0 && v < HT) {
 #pragma unroll
-            for (int i = 0; i < DT / 4; ++i) s_n[16 * (4 * i + w) + c] = nreg[i];  // read again behind the next barrier
+            for (int i = 0; i < NR; ++i) s_n[16 * (dh * HT + 4 * i + v) + c] = nreg[i];  // read again behind the next barrier
         }
-#pragma unroll
-        for (int rt = 2; rt < 4; ++rt) asm volatile("" : "+v"(pf[rt][1][0]), "+v"(pf[rt][1][1]));
-#pragma unroll
-        for (int rt = 0; rt < 4; ++rt) acc[rt] *= in[rt];
-#pragma unroll
-        for (int sl = 0; sl < 2; ++sl)
-#pragma unroll
-            for (int x = 0; x < 2; ++x)
-#pragma unroll
-                for (int rt = 2 * sl; rt < 4; ++rt) acc[rt] = mm_mfma(vv[sl], __builtin_bit_cast(bf16x8_t, pf[rt][sl][x]), acc[rt]);
-#pragma unroll
-        for (int rt = 0; rt < 4; ++rt) {
-            const float inv = __builtin_amdgcn_rcpf(fmaxf(fabsf(dn[rt]), fl[rt]) + 1e-6f);
-            rows_out[rt] = u32x2_t{pack2bf(acc[rt][0] * inv, acc[rt][1] * inv), pack2bf(acc[rt][2] * inv, acc[rt][3] * inv)};
-        }
+        const int ow = v + 4 * (1 - dh);       // the wave whose readout of these rows this one finishes
+        o_a += mm_lds<f32x4_t>(xst + (ow * 2 * 64 + lane) * 16);
+        o_b += mm_lds<f32x4_t>(xst + ((ow * 2 + 1) * 64 + lane) * 16);
+        const int ta = 16 * rt_a + c, tb = 16 * rt_b + c;
+        o_a *= mm_lds<float>(sa + 512 + 4 * ta);
+        o_b *= mm_lds<float>(sa + 512 + 4 * tb);
+        const unsigned ca = (g ^ (c & 7)) << 4, cb = ((4 + g) ^ (c & 7)) << 4;
+        const bf16x8_t pa0 = mm_lds<bf16x8_t>(pst + ta * 128 + ca), pa1 = mm_lds<bf16x8_t>(pst + 8192 + ta * 128 + ca);   // tiles 0 and 1: keys 32 .. 63 are all in the future
+        const bf16x8_t pb0 = mm_lds<bf16x8_t>(pst + tb * 128 + ca), pb1 = mm_lds<bf16x8_t>(pst + 8192 + tb * 128 + ca);
+        const bf16x8_t pb2 = mm_lds<bf16x8_t>(pst + tb * 128 + cb), pb3 = mm_lds<bf16x8_t>(pst + 8192 + tb * 128 + cb);
+        o_b = mm_mfma(vv[0], pb0, o_b);
+        o_a = mm_mfma(vv[0], pa0, o_a);
+        o_b = mm_mfma(vv[0], pb1, o_b);
+        o_a = mm_mfma(vv[0], pa1, o_a);
+        o_b = mm_mfma(vv[1], pb2, o_b);
+        o_b = mm_mfma(vv[1], pb3, o_b);
+        const float ia = __builtin_amdgcn_rcpf(fmaxf(fabsf(mm_lds<float>(sa + 1280 + 4 * ta) + mm_lds<float>(sa + 1536 + 4 * ta)), mm_lds<float>(sa + 768 + 4 * ta)) + 1e-6f);
+        const float ib = __builtin_amdgcn_rcpf(fmaxf(fabsf(mm_lds<float>(sa + 1280 + 4 * tb) + mm_lds<float>(sa + 1536 + 4 * tb)), mm_lds<float>(sa + 768 + 4 * tb)) + 1e-6f);
+        rows_out[0] = u32x2_t{pack2bf(o_a[0] * ia, o_a[1] * ia), pack2bf(o_a[2] * ia, o_a[3] * ia)};
+        rows_out[1] = u32x2_t{pack2bf(o_b[0] * ib, o_b[1] * ib), pack2bf(o_b[2] * ib, o_b[3] * ib)};
         m_in = mL;
     }
     store_rows(n_chunks - 1);
@@ -772,17 +744,17 @@ __global__ __launch_bounds__(256, D <= 64 ? 2 : 1) void memory_chunkwise_kernel(
     if (so < 0 || so >= a.n_state) return;
     const int64_t sout = so * a.H + h;
 #pragma unroll
-    for (int i = 0; i < DT; ++i)
+    for (int i = 0; i < HT; ++i)
 #pragma unroll
         for (int r = 0; r < 4; ++r) {
-            const int d = 16 * i + 4 * g + r;
+            const int d = 16 * (dh * HT + i) + 4 * g + r;
             if (con && d < a.dimp) a.S[(sout * a.dimp + d) * a.vdimp + col] = S[i][r];
         }
     if (vt == 0) {
 #pragma unroll
-        for (int i = 0; i < DT / 4; ++i) {
-            const int d = 16 * (4 * i + w) + c;
-            if (g == 0 && d < a.dimp) a.n[sout * a.dimp + d] = nreg[i];
+        for (int i = 0; i < NR; ++i) {
+            const int d = 16 * (dh * HT + 4 * i + v) + c;
+            if (g == 0 && v < HT && d < a.dimp) a.n[sout * a.dimp + d] = nreg[i];
         }
         if (tid == 0) a.m[sout] = m_in * (1.0f / MM_LOG2E);
     }
@@ -860,11 +832,12 @@ int run_rec(const RecArgs& a, hipStream_t st) {
 
 template <int D>
 int launch_chunk(const ChunkArgs& a, int seqs, hipStream_t st) {
-    constexpr int STAGE = 2 * 64 * D * 2 + 8192 + 1024, LDS = (D <= 128 ? 3 : 2) * STAGE + (64 * D * 2 >= 16384 ? 0 : 16384) + 6 * 256 + D * 4;
+    constexpr int QT = 64 * D * 2, STAGE = 2 * QT + 8192 + 1024;
+    constexpr int LDS = (D <= 128 ? 3 : 2) * STAGE + (QT >= 16384 ? 0 : 16384) + (QT >= 32768 ? 0 : 16384) + 7 * 256 + D * 4;
     static_assert(LDS <= 160 * 1024, "LDS of a CU");
     auto kern = memory_chunkwise_kernel<D>;
     GLM_SET_MAX_LDS(kern, LDS, "glm_memory_chunkwise");
-    hipLaunchKernelGGL(kern, dim3((unsigned)(seqs * a.H * a.vtiles)), dim3(256), LDS, st, a);
+    hipLaunchKernelGGL(kern, dim3((unsigned)(seqs * a.H * a.vtiles)), dim3(512), LDS, st, a);
     GLM_CHECK_LAUNCH("glm_memory_chunkwise");
     return GLM_OK;
 }
