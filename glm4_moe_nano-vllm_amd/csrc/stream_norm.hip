@@ -100,7 +100,7 @@ __global__ __launch_bounds__(NT) void stream_norm_kernel(const StreamNormArgs a,
         for (int j = 0; j < NV; ++j) {
             if (!on[j]) continue;
 #pragma unroll
-            for (int t = 0; t < S; ++t) x[t][j] = *reinterpret_cast<const f32x4_t*>(a.x_in + row * a.ldx + t * a.sx + col[j]);
+            for (int t = 0; t < S; ++t) x[t][j] = __builtin_nontemporal_load(reinterpret_cast<const f32x4_t*>(a.x_in + row * a.ldx + t * a.sx + col[j]));
             if (a.y) y[j] = st_load4(a.y, row * a.ldy + col[j], a.y_f32);
         }
     };
@@ -136,7 +136,7 @@ __global__ __launch_bounds__(NT) void stream_norm_kernel(const StreamNormArgs a,
             }
             if (a.x_out && r >= r0 && on[j]) {
 #pragma unroll
-                for (int t = 0; t < S; ++t) *reinterpret_cast<f32x4_t*>(a.x_out + (r * S + t) * a.wp + col[j]) = x[t][j];
+                for (int t = 0; t < S; ++t) __builtin_nontemporal_store(x[t][j], reinterpret_cast<f32x4_t*>(a.x_out + (r * S + t) * a.wp + col[j]));
             }
             u[j] = zero;
 #pragma unroll
