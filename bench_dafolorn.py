@@ -161,7 +161,7 @@ def dafolorn_kernels(m, meta, mode, B, n):
             [lambda mx=layer.mixer: ops.latent_prepare(qc, H * d, H, d, r, mx.c_gain, mx.eps, meta.slots, mx.caches[0], T, mx.wukt) for layer in L],
             2 * (H * d * r + T * (H * d + 2 * r + H * r)), 2 * T * H * d * r)
         out["latent attention + merge, W_uv"] = (
-            [lambda mx=layer.mixer: ops.latent_attn(qa, mx.caches[0], tok, cnt, 1, meta.pos, meta.seq_of, meta.block_tables, r, W, mx.scale, mx.sink,
+            [lambda mx=layer.mixer: ops.latent_attn(qa, mx.caches[0], tok, cnt, 1, meta.pos, meta.seq_of, meta.block_tables, W, mx.scale, mx.sink,
                                                     mx.wuv, o2) for layer in L],
             2 * (B * keys * r + H * v * r + T * H * (r + v)), 2 * T * H * (2 * keys * r + r * v))
     else:

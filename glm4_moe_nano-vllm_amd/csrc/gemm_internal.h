@@ -3,9 +3,12 @@
 #include "common.h"
 
 // A library for models without experts, fp8 weights and fused QKV / router epilogues (build.py, kernel sets) compiles the GEMM
-// sources without those parts.
+// sources without those parts; with GLM_EXPERTS the grouped bf16 projections of experts stay in.
 #ifndef GLM_DENSE_ONLY
 #define GLM_DENSE_ONLY 0
+#endif
+#ifndef GLM_EXPERTS
+#define GLM_EXPERTS !GLM_DENSE_ONLY
 #endif
 
 enum GemmMode : int {
@@ -17,18 +20,24 @@ enum GemmMode : int {
     // bodies take p.act / p.yf in GEMM_PLAIN.)
     GEMM_ACT = 3,
     GEMM_XIELU = 4,  // xIELU, bf16 rows
+    GEMM_COLS = 6,   // per-column activation (glm_act_cols), bf16 rows
     GEMM_GLU = 5,    // GEMM_GATEUP's layout (W rows gate|up) with the clamped gated unit of p.act instead of SiLU; fp32 up to the store
 };
 __host__ __device__ constexpr bool gemm_paired(int mode) { return mode == GEMM_GATEUP || mode == GEMM_GLU; }
 
 // activation on the fp32 accumulator of a projection (after the bias)
-enum : int { GLM_ACT_NONE = GLM_EPI_NONE, GLM_ACT_XIELU = GLM_EPI_XIELU, GLM_ACT_SOFTCAP = GLM_EPI_SOFTCAP, GLM_ACT_GLU_CLAMP = GLM_EPI_GLU_CLAMP };
+enum : int { GLM_ACT_NONE = GLM_EPI_NONE, GLM_ACT_XIELU = GLM_EPI_XIELU, GLM_ACT_SOFTCAP = GLM_EPI_SOFTCAP, GLM_ACT_GLU_CLAMP = GLM_EPI_GLU_CLAMP,
+              GLM_ACT_GATE = GLM_EPI_GATE, GLM_ACT_SILU_GATE = GLM_EPI_SILU_GATE };
 struct GlmAct {
     int kind;
     float a, b;
 };
 // z > 0: a z^2 + z / 2;  z <= 0: b (exp(z) - 1 - z) + z / 2.   The fp32 form, for fp32 outputs.
-__device__ __forceinline__ float glm_act_precise(const GlmAct& t, float z) {
+__device__ __forceinline__ float glm_act_precise(const GlmAct& t, float z, int n) {
+    if (t.kind >= GLM_ACT_GATE) {
+        const float s = 1.0f / (1.0f + expf(-z));
+        return n >= (int)t.a ? s : t.kind == GLM_ACT_SILU_GATE ? z * s : z;
+    }
     if (t.kind == GLM_ACT_XIELU) return z > 0.f ? t.a * z * z + 0.5f * z : t.b * (expm1f(z) - z) + 0.5f * z;
     if (t.kind == GLM_ACT_SOFTCAP) return t.a * tanhf(z / t.a);
     return z;
@@ -39,8 +48,14 @@ __device__ __forceinline__ float glm_xielu_fast(float a, float b, float z) {
     const float neg = b * (__builtin_amdgcn_exp2f(1.4426950408889634f * fminf(z, 0.f)) - 1.0f - z);
     return (z > 0.f ? a * z * z : neg) + 0.5f * z;
 }
-__device__ __forceinline__ float glm_act_fast(const GlmAct& t, float z) {
-    return t.kind == GLM_ACT_XIELU ? glm_xielu_fast(t.a, t.b, z) : glm_act_precise(t, z);
+// per-column activations: the first t.a columns pass (or go through SiLU), the others through the sigmoid (a gate)
+__device__ __forceinline__ float glm_act_cols(const GlmAct& t, float z, int n) {
+    const float s = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+    return n >= (int)t.a ? s : t.kind == GLM_ACT_SILU_GATE ? z * s : z;
+}
+__device__ __forceinline__ float glm_act_fast(const GlmAct& t, float z, int n) {
+    if (t.kind >= GLM_ACT_GATE) return glm_act_cols(t, z, n);
+    return t.kind == GLM_ACT_XIELU ? glm_xielu_fast(t.a, t.b, z) : glm_act_precise(t, z, n);
 }
 
 // clamped gated unit: limit t.a, slope t.b:  g sigmoid(b g) (u + 1) with g <= a, -a <= u <= a.  The fp32 form, and the one for outputs

@@ -1554,10 +1554,11 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
                     } else {
                         float a = acc[t][mt][r];
                         if constexpr (WSCALE) a *= wsv[t][r];
-                        if ((MODE == GEMM_PLAIN || MODE == GEMM_ACT || MODE == GEMM_XIELU) && p.bias) a += bf2f(p.bias[min(ncol_w + 16 * t + 4 * g4 + r, p.N - 1)]);
+                        if ((MODE == GEMM_PLAIN || MODE == GEMM_ACT || MODE == GEMM_XIELU || MODE == GEMM_COLS) && p.bias) a += bf2f(p.bias[min(ncol_w + 16 * t + 4 * g4 + r, p.N - 1)]);
                         if (scaled) a = rbf(a) * sc;
                         if (MODE == GEMM_XIELU) a = glm_xielu_fast(p.act.a, p.act.b, a);
-                        if (MODE == GEMM_ACT) a = p.yf != nullptr ? glm_act_precise(p.act, a) : glm_act_fast(p.act, a);
+                        if (MODE == GEMM_COLS) a = glm_act_cols(p.act, a, ncol_w + 16 * t + 4 * g4 + r);
+                        if (MODE == GEMM_ACT) a = p.yf != nullptr ? glm_act_precise(p.act, a, ncol_w + 16 * t + 4 * g4 + r) : glm_act_fast(p.act, a, ncol_w + 16 * t + 4 * g4 + r);
                         o[r] = a;
                     }
                 }
@@ -1706,7 +1707,7 @@ int launch_largem(const GemmParams& p, hipStream_t st) {
     const int64_t avg_rows = (p.R_hint > 0 ? p.R_hint : p.R) / (p.G > 0 ? p.G : 1);
     // ... and a projection onto <= 128 columns (the router logits at prefill: N = E = 64) is one column tile however the rows
     // are cut, so its parallelism is its row-block count: 128-row blocks (75.8 -> 55.1 us at T = 16384)
-    const bool use_b = ch == 2 || (ch == 0 && avg_rows >= 192 && !((MODE == GEMM_PLAIN || MODE == GEMM_ACT || MODE == GEMM_XIELU) && p.offs == nullptr && p.N <= 128));
+    const bool use_b = ch == 2 || (ch == 0 && avg_rows >= 192 && !((MODE == GEMM_PLAIN || MODE == GEMM_ACT || MODE == GEMM_XIELU || MODE == GEMM_COLS) && p.offs == nullptr && p.N <= 128));
     // the lean load phase addresses x and the group's weights through 32-bit buffer offsets and has no K tail path
     // default (tools/largem_ab.py, one process, T = 16384): the quadrant-phase loop with 4 x 2-tile quadrants and the
     // fragment reads of a load interval issued before its DMA, no priority flips (86531: +1 % over 86019), epilogue
@@ -1841,10 +1842,11 @@ int glm_launch_gemm_largem(int mode, const GemmParams& p, hipStream_t st) {
                   GLM_ERR_UNSUPPORTED,
                   "gemm_largem: needs K%%8==0, N%%4==0, ldx%%8==0, ldy%%4==0, 16B-aligned x/W (K=%d N=%d)",
                   p.K, p.N);
-#if !GLM_DENSE_ONLY
+#if GLM_EXPERTS
     if (mode == GEMM_GATEUP) return launch_largem<GEMM_GATEUP>(p, st);
     if (mode == GEMM_DOWN) return launch_largem<GEMM_DOWN>(p, st);
-#endif  // !GLM_DENSE_ONLY
+#endif  // GLM_EXPERTS
+    if (mode == GEMM_ACT && p.yf == nullptr && p.act.kind >= GLM_ACT_GATE) return launch_largem<GEMM_COLS>(p, st);
     if (mode == GEMM_ACT && p.yf == nullptr && p.act.kind == GLM_ACT_XIELU) return launch_largem<GEMM_XIELU>(p, st);
     if (mode == GEMM_ACT) return launch_largem<GEMM_ACT>(p, st);
     if (mode == GEMM_GLU) return launch_largem<GEMM_GLU>(p, st);

@@ -143,13 +143,13 @@ __device__ __forceinline__ void smallm_epilogue(const GemmParams& p, f32x4_t (&a
                     if (p.yf != nullptr) {
                         f32x4_t v;
 #pragma unroll
-                        for (int r = 0; r < 4; ++r) v[r] = glm_act_precise(p.act, o[r]);
+                        for (int r = 0; r < 4; ++r) v[r] = glm_act_precise(p.act, o[r], n + r);
                         *reinterpret_cast<f32x4_t*>(p.yf + (int64_t)(m0 + row) * p.ldy + n) = v;
                         continue;
                     }
                     if (p.act.kind != GLM_ACT_NONE) {
 #pragma unroll
-                        for (int r = 0; r < 4; ++r) o[r] = glm_act_fast(p.act, o[r]);
+                        for (int r = 0; r < 4; ++r) o[r] = glm_act_fast(p.act, o[r], n + r);
                     }
                 }
                 u32x2_t v = {pack2bf(o[0], o[1]), pack2bf(o[2], o[3])};
@@ -994,7 +994,7 @@ int glm_launch_gemm_smallm(int mode, const GemmParams& p, hipStream_t st) {
 #endif
         return launch_cfg<GEMM_GLU, GLM_SM_CFG_GATEUP>(p, st);
     }
-#if !GLM_DENSE_ONLY
+#if GLM_EXPERTS
 #ifndef GLM_SM_CFG_DOWN
 #define GLM_SM_CFG_DOWN 4, 2, 1, 2
 #endif
@@ -1045,7 +1045,7 @@ int glm_launch_gemm_smallm(int mode, const GemmParams& p, hipStream_t st) {
     if (mode == GEMM_DOWN && Rs <= 16) return launch_cfg<GEMM_DOWN, GLM_SM_CFG_DOWN_R16>(p, st);
     if (mode == GEMM_GATEUP) return launch_cfg<GEMM_GATEUP, GLM_SM_CFG_GATEUP>(p, st);
     if (mode == GEMM_DOWN) return launch_cfg<GEMM_DOWN, GLM_SM_CFG_DOWN>(p, st);
-#endif  // !GLM_DENSE_ONLY
+#endif  // GLM_EXPERTS
 #if !defined(GLM_SM_NO_DMA) && !defined(GLM_SM_DMA_MID)
 #define GLM_SM_DMA_MID 2, 1, 2, 2  // 23.7 us (4,2,2,2: 25.6; 1,1,2,2: 24.4; 4,1,2,2: 39.8)
 #endif

@@ -495,12 +495,12 @@ __global__ __launch_bounds__(TM_NT) void gemm_tinym_kernel(const TinyParams tp) 
                 if (MODE == GEMM_PLAIN && !TAIL) {
                     if (p.yf != nullptr) {
 #pragma unroll
-                        for (int r = 0; r < RPW; ++r) p.yf[row * p.ldy + t.ncol + r] = glm_act_precise(p.act, v[r]);
+                        for (int r = 0; r < RPW; ++r) p.yf[row * p.ldy + t.ncol + r] = glm_act_precise(p.act, v[r], t.ncol + r);
                         continue;
                     }
                     if (p.act.kind != GLM_ACT_NONE) {
 #pragma unroll
-                        for (int r = 0; r < RPW; ++r) v[r] = glm_act_fast(p.act, v[r]);
+                        for (int r = 0; r < RPW; ++r) v[r] = glm_act_fast(p.act, v[r], t.ncol + r);
                     }
                 }
                 if constexpr (RPW == 4) {
@@ -651,7 +651,7 @@ int glm_launch_gemm_tinym(int mode, const GemmParams& p, int n_tokens, hipStream
     // units: 4 rows x 4 KiB for long rows; a short K (expert down projection, 1408) as ONE unit of 3-KiB rows
     if (mode == GEMM_PLAIN) return launch_tiny<GEMM_PLAIN, 1, GLM_TM_SEGS_PLAIN, false, false, GLM_TM_RPW_PLAIN>(tp, 1, st);
     if (mode == GEMM_GLU) return launch_tiny<GEMM_GLU, 1, 8, false, false, 2>(tp, 1, st);
-#if !GLM_DENSE_ONLY
+#if GLM_EXPERTS
     // grouped launches: rows per tile chosen for the TAIL of the launch — a workgroup's waves pull tiles from a counter, and
     // the launch ends when the slowest wave has finished its last tile; at Air dims one token gives 24.75 tiles of 4 rows per
     // workgroup for gate|up (7 waves take 3, one takes 4: +29 % on the critical wave), 49.5 tiles of 2 rows even that out

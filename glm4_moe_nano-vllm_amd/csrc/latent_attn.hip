@@ -8,7 +8,12 @@
 //
 //   latent_prepare   one launch: latent norm + cache store of the step's tokens, and q' = W_uk^T q of the absorbed rows
 //   latent_attn      split-KV flash loop over the pages; rows are (token, head) pairs; fp32 scores and softmax
-//   latent_up        merge of the KV splits (with the sink's mass) and out = W_uv ctx
+//   latent_up        out = W_uv ctx, times an output gate if there is one
+//
+// With a rotated key part that all heads share (rotp columns behind the latent's rp in a cache row), queries that go through a latent of
+// their own and positions, latent_prepare is two launches: latent_rows (both latents' norms, the rotated key, cache store) in front of
+// the query projection and latent_absorb (q' and the rotated query part behind it) after it; the scores then run over rp + rotp
+// columns, the values over the first rp.
 //
 // Roofline of latent_attn at decode: HBM — window * rank * 2 bytes per sequence, read once.  Four waves per 16 query rows share
 // every 64-key tile, double-buffered by LDS-DMA.  One LDS image serves both products: chunk ^ swz(key) with
@@ -27,21 +32,30 @@ __device__ const u32x4_t la_zero_page[4] = {};
 
 // ---------------------------------------------------------------------------------------------------------------------------
 struct PrepArgs {
-    const void* qc;        // [T, ldq] projection rows: q heads at h*dimp, raw latent at c_off
+    const void* q;         // [T, ldqq] queries, head h at h*hd: dimp unrotated columns, then rotp rotated ones
+    int64_t ldqq;
+    int hd;
+    const void* qc;        // [T, ldq] projection rows: raw latent at c_off, raw rotated key part at c_off + rp
     int64_t ldq;
     int c_off;
     int64_t T, Ta;         // rows; rows [0, Ta) are absorbed
     int H, dimp, rank, rp; // rp = rank rounded up to 8
+    int rotp, rc;          // rotated columns; rc = rp + rotp, the pitch of cache, c_out and qa rows
+    const float* cs;       // [T, rotp / 2, 2] cos, sin of the pairs of columns (2i, 2i+1)
+    int cq_off, cq_rank, cq_rp;  // latent of the queries in qc, or cq_out = nullptr
+    const float* cq_norm;  // [cq_rp]
+    void* cq_out;          // [T, ld_cq]
+    int64_t ld_cq;
     const float* norm_w;   // [rp]
     float eps;
     const int32_t* slots;  // [T] cache row of the token, < 0: none
-    void* cache;           // [n_slots, rp]
+    void* cache;           // [n_slots, rc]
     int64_t n_slots;
     const int32_t* crow;   // [T] row of c_out, < 0: none (nullptr: no c_out)
-    void* c_out;           // [n_crows, rp]
+    void* c_out;           // [n_crows, rc]
     int64_t n_crows;
     const bf16_t* wukt;    // [H, rp, dimp]
-    bf16_t* qa;            // [Ta, H, rp]
+    bf16_t* qa;            // [Ta, H, rc]
 };
 
 // latent norm of one token by one wave, eight columns per lane and step (the padding columns of the projection are zeros)
@@ -71,42 +85,73 @@ __device__ __forceinline__ void la_st8(void* p, int64_t i, const float (&v)[8]) 
         for (int j = 0; j < 8; ++j) f[j] = v[j];
     }
 }
-// R tokens t0 .. by one wave, their loads together
-template <typename E, int R>
-__device__ void latent_norm_rows(const PrepArgs& a, int64_t t0, int lane) {
-    int64_t slot[R], row[R];
+// RMS norm of columns [off, off + rp) of R rows t0 .. by one wave, their loads together; put(row, column, eight values)
+template <typename E, int R, class Put>
+__device__ __forceinline__ void norm_rows(const void* x, int64_t ld, int off, int64_t T, int64_t t0, int lane, int rank, int rp, const float* gain, float eps, Put put) {
     float v[R][8], s[R];
 #pragma unroll
-    for (int i = 0; i < R; ++i) {
-        const int64_t t = min(t0 + i, a.T - 1);
-        slot[i] = a.slots[t];
-        row[i] = a.crow ? a.crow[t] : -1;
-        s[i] = 0.f;
-    }
-    for (int k = lane * 8; k < a.rp; k += 512) {
+    for (int i = 0; i < R; ++i) s[i] = 0.f;
+    for (int k = lane * 8; k < rp; k += 512) {
 #pragma unroll
-        for (int i = 0; i < R; ++i) la_ld8<E>(a.qc, min(t0 + i, a.T - 1) * a.ldq + a.c_off + k, v[i]);
+        for (int i = 0; i < R; ++i) la_ld8<E>(x, min(t0 + i, T - 1) * ld + off + k, v[i]);
 #pragma unroll
         for (int i = 0; i < R; ++i)
 #pragma unroll
             for (int j = 0; j < 8; ++j) s[i] += v[i][j] * v[i][j];
     }
 #pragma unroll
-    for (int i = 0; i < R; ++i) s[i] = 1.0f / sqrtf(wave_sum(s[i]) / (float)a.rank + a.eps);
-    for (int k = lane * 8; k < a.rp; k += 512) {
+    for (int i = 0; i < R; ++i) s[i] = 1.0f / sqrtf(wave_sum(s[i]) / (float)rank + eps);
+    for (int k = lane * 8; k < rp; k += 512) {
         float w[8];
 #pragma unroll
-        for (int j = 0; j < 8; ++j) w[j] = a.norm_w[k + j];
+        for (int j = 0; j < 8; ++j) w[j] = gain[k + j];
+#pragma unroll
+        for (int i = 0; i < R; ++i) {
+            if (t0 + i >= T) continue;
+            if (rp > 512) la_ld8<E>(x, (t0 + i) * ld + off + k, v[i]);  // (one step: the values are still in registers)
+#pragma unroll
+            for (int j = 0; j < 8; ++j) v[i][j] = v[i][j] * s[i] * w[j];
+            put(i, k, v[i]);
+        }
+    }
+}
+// pairs (u, v) of eight columns -> (u cos - v sin, v cos + u sin)
+__device__ __forceinline__ void la_rotate8(float (&x)[8], const float* cs) {
+#pragma unroll
+    for (int j = 0; j < 4; ++j) {
+        const float c = cs[2 * j], s = cs[2 * j + 1], u = x[2 * j], v = x[2 * j + 1];
+        x[2 * j] = u * c - v * s;
+        x[2 * j + 1] = v * c + u * s;
+    }
+}
+template <typename E, int R>
+__device__ void latent_norm_rows(const PrepArgs& a, int64_t t0, int lane) {
+    int64_t slot[R], row[R];
+#pragma unroll
+    for (int i = 0; i < R; ++i) {
+        const int64_t t = min(t0 + i, a.T - 1);
+        slot[i] = a.slots[t];
+        row[i] = a.crow ? a.crow[t] : -1;
+    }
+    auto put = [&](int i, int k, const float (&v)[8]) {
+        if (slot[i] >= 0 && slot[i] < a.n_slots) la_st8<E>(a.cache, slot[i] * a.rc + k, v);
+        if (row[i] >= 0 && row[i] < a.n_crows) la_st8<E>(a.c_out, row[i] * a.rc + k, v);
+    };
+    norm_rows<E, R>(a.qc, a.ldq, a.c_off, a.T, t0, lane, a.rank, a.rp, a.norm_w, a.eps, put);
+    for (int k = lane * 8; k < a.rotp; k += 512)
 #pragma unroll
         for (int i = 0; i < R; ++i) {
             if (t0 + i >= a.T) continue;
-            if (a.rp > 512) la_ld8<E>(a.qc, (t0 + i) * a.ldq + a.c_off + k, v[i]);  // (one step: the values are still in registers)
-#pragma unroll
-            for (int j = 0; j < 8; ++j) v[i][j] = v[i][j] * s[i] * w[j];
-            if (slot[i] >= 0 && slot[i] < a.n_slots) la_st8<E>(a.cache, slot[i] * a.rp + k, v[i]);
-            if (row[i] >= 0 && row[i] < a.n_crows) la_st8<E>(a.c_out, row[i] * a.rp + k, v[i]);
+            float v[8];
+            la_ld8<E>(a.qc, (t0 + i) * a.ldq + a.c_off + a.rp + k, v);
+            la_rotate8(v, a.cs + (t0 + i) * a.rotp + k);
+            put(i, a.rp + k, v);
         }
-    }
+}
+template <typename E, int R>
+__device__ void latent_query_rows(const PrepArgs& a, int64_t t0, int lane) {
+    norm_rows<E, R>(a.qc, a.ldq, a.cq_off, a.T, t0, lane, a.cq_rank, a.cq_rp, a.cq_norm, a.eps,
+                    [&](int i, int k, const float (&v)[8]) { la_st8<E>(a.cq_out, (t0 + i) * a.ld_cq + k, v); });
 }
 
 constexpr int PREP_TT = 4;  // 16-token tiles per absorb workgroup
@@ -121,16 +166,28 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(const PrepArgs a, i
         return;
     }
     // q'[t, h, r] = sum_d W_uk[h, d, r] q[t, h, d]: 64 latent rows x 64 tokens per workgroup, 16 x 64 per wave
-    const int nr = (a.rp + 63) / 64;
+    const int nb = (a.rp + 63) / 64, nr = nb + (a.rotp > 0);
     int b = blockIdx.x;
     const int rb = b % nr;
     b /= nr;
     const int h = b % a.H;
     const int64_t t0 = (int64_t)(b / a.H) * (16 * PREP_TT);
+    if (rb == nb) {  // the rotated part
+        for (int i = tid; i < 16 * PREP_TT * (a.rotp / 8); i += 256) {
+            const int64_t t = t0 + i / (a.rotp / 8);
+            const int k = i % (a.rotp / 8) * 8;
+            if (t >= a.Ta) continue;
+            float v[8];
+            la_ld8<bf16_t>(a.q, t * a.ldqq + (int64_t)h * a.hd + a.dimp + k, v);
+            la_rotate8(v, a.cs + t * a.rotp + k);
+            la_st8<bf16_t>(a.qa, (t * a.H + h) * a.rc + a.rp + k, v);
+        }
+        return;
+    }
     const int c = lane & 15, g = lane >> 4;
     const int r0 = rb * 64 + wid * 16;
     const int ar = r0 + c;  // A row of this lane
-    const bf16_t* q = reinterpret_cast<const bf16_t*>(a.qc);
+    const bf16_t* q = reinterpret_cast<const bf16_t*>(a.q);
     f32x4_t acc[PREP_TT];
 #pragma unroll
     for (int i = 0; i < PREP_TT; ++i) acc[i] = f32x4_t{0.f, 0.f, 0.f, 0.f};
@@ -141,7 +198,7 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(const PrepArgs a, i
         for (int i = 0; i < PREP_TT; ++i) {
             const int64_t t = t0 + 16 * i + c;
             u32x4_t bv = {0, 0, 0, 0};
-            if (k < a.dimp && t < a.Ta) bv = *reinterpret_cast<const u32x4_t*>(q + t * a.ldq + (int64_t)h * a.dimp + k);
+            if (k < a.dimp && t < a.Ta) bv = *reinterpret_cast<const u32x4_t*>(q + t * a.ldqq + (int64_t)h * a.hd + k);
             acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, av), __builtin_bit_cast(bf16x8_t, bv), acc[i], 0, 0, 0);
         }
     }
@@ -151,9 +208,47 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(const PrepArgs a, i
         for (int i = 0; i < PREP_TT; ++i) {
             const int64_t t = t0 + 16 * i + c;
             if (t < a.Ta)
-                *reinterpret_cast<u32x2_t*>(a.qa + (t * a.H + h) * a.rp + r) = u32x2_t{pack2bf(acc[i][0], acc[i][1]), pack2bf(acc[i][2], acc[i][3])};
+                *reinterpret_cast<u32x2_t*>(a.qa + (t * a.H + h) * a.rc + r) = u32x2_t{pack2bf(acc[i][0], acc[i][1]), pack2bf(acc[i][2], acc[i][3])};
         }
     }
+}
+
+// both latents' norms, the rotated key part and the cache store; blockIdx.y: key side, query side
+template <typename E, int NR>
+__global__ __launch_bounds__(256) void latent_rows_kernel(const PrepArgs a) {
+    const int64_t t = ((int64_t)blockIdx.x * 4 + (threadIdx.x >> 6)) * NR;
+    if (t >= a.T) return;
+    if (blockIdx.y == 0) latent_norm_rows<E, NR>(a, t, threadIdx.x & 63);
+    else latent_query_rows<E, NR>(a, t, threadIdx.x & 63);
+}
+
+// fp32: the rotated query part alone
+__global__ __launch_bounds__(256) void latent_rotate_f32_kernel(const PrepArgs a) {
+    const int n = a.rotp / 8;
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x, th = i / n, t = th / a.H;
+    const int k = (int)(i % n) * 8, h = (int)(th % a.H);
+    if (t >= a.Ta) return;
+    float v[8];
+    la_ld8<float>(a.q, t * a.ldqq + (int64_t)h * a.hd + a.dimp + k, v);
+    la_rotate8(v, a.cs + t * a.rotp + k);
+    la_st8<float>(a.qa, th * a.rc + a.rp + k, v);
+}
+
+// cos and sin of every pair of rotated columns at the positions of a step, times mscale; the angle is taken in double and brought into
+// one turn before it is rounded, so far positions are as exact as near ones.  Pairs behind the last frequency do not turn.
+__global__ __launch_bounds__(256) void rope_pairs_kernel(const int32_t* pos, const double* freq, int n_freq, float mscale, float* cs, int64_t T, int pairs) {
+    const int64_t i = (int64_t)blockIdx.x * 256 + threadIdx.x, t = i / pairs;
+    const int j = (int)(i % pairs);
+    if (t >= T) return;
+    float c = 1.f, s = 0.f;
+    if (j < n_freq) {
+        const double turns = (double)max(pos[t], 0) * freq[j] * 0.15915494309189533577;
+        const float ang = (float)((turns - rint(turns)) * 6.28318530717958647693);
+        c = cosf(ang) * mscale;
+        s = sinf(ang) * mscale;
+    }
+    cs[i * 2] = c;
+    cs[i * 2 + 1] = s;
 }
 
 __global__ __launch_bounds__(256) void latent_norm_f32_kernel(const PrepArgs a) {
@@ -183,12 +278,12 @@ struct AttnArgs {
     int64_t n_blocks;
     int bs_shift;             // log2(block size)
     int64_t Ta;
-    int H, rank, rp, window;
+    int H, rp, vp, window;      // rp: columns of a cache row (scores), the first vp of them are the values
     float scale;
     const float* sink;        // [H]
     int n_tiles, hb, n_hg, tq, nsplit;  // heads per workgroup, head groups, tokens per tile (at most)
-    bf16_t* ctx;              // nsplit == 1: [Ta, H, rp] normalised context
-    float* part_o;            // nsplit > 1: [Ta * H, nsplit, rp] unnormalised
+    bf16_t* ctx;              // nsplit == 1: [Ta, H, vp] normalised context
+    float* part_o;            // nsplit > 1: [Ta * H, nsplit, vp] unnormalised
     float* part_ml;           // [Ta * H, nsplit, 2] running maximum (log2 units), mass
 };
 
@@ -238,7 +333,7 @@ __global__ __launch_bounds__(64 * 4 * MT) void latent_attn_kernel(const AttnArgs
                 a.part_ml[(gr * a.nsplit + split) * 2] = -INFINITY;
                 a.part_ml[(gr * a.nsplit + split) * 2 + 1] = 0.f;
             } else {
-                for (int d = 0; d < a.rp; ++d) a.ctx[gr * a.rp + d] = 0;
+                for (int d = 0; d < a.vp; ++d) a.ctx[gr * a.vp + d] = 0;
             }
         }
         return;
@@ -318,6 +413,7 @@ __global__ __launch_bounds__(64 * 4 * MT) void latent_attn_kernel(const AttnArgs
     const int qq = (lane >> 2) & 3, pp = lane & 3, vrow = 4 * g + qq;
     // latent tile d of this wave: d NW + w = 4 (d MT + (w >> 2)) + (w & 3)
     const unsigned v_rel = vrow * ROWB + (((2 * (w & 3) + (pp >> 1)) ^ attn_swz(vrow)) << 4) + ((pp & 1) << 3) + (w >> 2) * 128;
+    const bool last_v = (DPW - 1) * NW * 16 < a.vp;  // this wave's last column tile may hold values
     const float sc = a.scale * LOG2E;
 #pragma unroll
     for (int i = 0; i < KS; ++i) asm volatile("" : "+v"(qf[i]));  // landed before the DMAs are counted
@@ -410,7 +506,7 @@ __global__ __launch_bounds__(64 * 4 * MT) void latent_attn_kernel(const AttnArgs
                 u32x2_t vf[FG][2];
                 static_for<nd>([&](auto I) {
                     constexpr int d = d0 + decltype(I)::value;
-                    if (4 * NCT % NW == 0 || d * NW + w < 4 * NCT) {
+                    if ((4 * NCT % NW == 0 || d * NW + w < 4 * NCT) && (d + 1 < DPW || last_v)) {
                         lds_read_tr16_b64<d * MT * 128>(vf[d - d0][0], va);
                         lds_read_tr16_b64<d * MT * 128>(vf[d - d0][1], va + 16 * ROWB);
                     }
@@ -423,7 +519,7 @@ __global__ __launch_bounds__(64 * 4 * MT) void latent_attn_kernel(const AttnArgs
 #pragma unroll
                 for (int d = 0; d < nd; ++d) {
                     const u32x4_t vv = {vf[d][0][0], vf[d][0][1], vf[d][1][0], vf[d][1][1]};
-                    if (4 * NCT % NW == 0 || (d0 + d) * NW + w < 4 * NCT) {
+                    if ((4 * NCT % NW == 0 || (d0 + d) * NW + w < 4 * NCT) && (d0 + d + 1 < DPW || last_v)) {
 #pragma unroll
                         for (int m = 0; m < MT; ++m)
                             acc[m][d0 + d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, vv), __builtin_bit_cast(bf16x8_t, pf[m]), acc[m][d0 + d], 0, 0, 0);
@@ -460,15 +556,15 @@ __global__ __launch_bounds__(64 * 4 * MT) void latent_attn_kernel(const AttnArgs
 #pragma unroll
             for (int d = 0; d < DPW; ++d) {
                 const int dim = 16 * (d * NW + w) + 4 * g;
-                if (dim < a.rp)
-                    *reinterpret_cast<u32x2_t*>(a.ctx + gr * a.rp + dim) = u32x2_t{pack2bf(acc[m][d][0] * inv, acc[m][d][1] * inv), pack2bf(acc[m][d][2] * inv, acc[m][d][3] * inv)};
+                if (dim < a.vp)
+                    *reinterpret_cast<u32x2_t*>(a.ctx + gr * a.vp + dim) = u32x2_t{pack2bf(acc[m][d][0] * inv, acc[m][d][1] * inv), pack2bf(acc[m][d][2] * inv, acc[m][d][3] * inv)};
             }
         } else {
             const int64_t pr = gr * a.nsplit + split;
 #pragma unroll
             for (int d = 0; d < DPW; ++d) {
                 const int dim = 16 * (d * NW + w) + 4 * g;
-                if (dim < a.rp) *reinterpret_cast<f32x4_t*>(a.part_o + pr * a.rp + dim) = acc[m][d];
+                if (dim < a.vp) *reinterpret_cast<f32x4_t*>(a.part_o + pr * a.vp + dim) = acc[m][d];
             }
             if (w == 0 && g == 0) {
                 a.part_ml[pr * 2] = m_run[m];
@@ -561,19 +657,21 @@ __global__ __launch_bounds__(256) void latent_attn_f32_kernel(const AttnArgs a, 
             const int64_t rk = __shfl((long long)row, k, 64);
 #pragma unroll
             for (int i = 0; i < NV; ++i)
-                if (lane + 64 * i < a.rp) acc[i] = fmaf(pk, cache[rk * a.rp + lane + 64 * i], acc[i]);
+                if (lane + 64 * i < a.vp) acc[i] = fmaf(pk, cache[rk * a.rp + lane + 64 * i], acc[i]);
         }
     }
     const float inv = 1.0f / l;
 #pragma unroll
     for (int i = 0; i < NV; ++i)
-        if (lane + 64 * i < a.rp) ctx[grow * a.rp + lane + 64 * i] = p < 0 ? 0.f : acc[i] * inv;
+        if (lane + 64 * i < a.vp) ctx[grow * a.vp + lane + 64 * i] = p < 0 ? 0.f : acc[i] * inv;
 }
 
 struct UpArgs {
     const bf16_t* ctx;   // [Ta, H, rp]
     const bf16_t* wuv;   // [H, vdimp, rp]
     bf16_t* out;         // [T, ldo], head h at h*vdimp
+    const bf16_t* gate;  // [T, ldg] laid out like out: factors of the rows, or nullptr
+    int64_t ldg;
     int64_t ldo, Ta;
     int H, vdimp, rp;
 };
@@ -606,6 +704,10 @@ __global__ __launch_bounds__(256) void latent_up_kernel(const UpArgs a) {
             acc = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(bf16x8_t, av[i]), __builtin_bit_cast(bf16x8_t, bv[i]), acc, 0, 0, 0);
     }
     const int v = v0 + 4 * g;
+    if (a.gate && t < a.Ta && v < a.vdimp) {
+        const u32x2_t gt = *reinterpret_cast<const u32x2_t*>(a.gate + t * a.ldg + (int64_t)h * a.vdimp + v);
+        acc *= f32x4_t{bflo(gt[0]), bfhi(gt[0]), bflo(gt[1]), bfhi(gt[1])};
+    }
     if (t < a.Ta && v < a.vdimp)
         *reinterpret_cast<u32x2_t*>(a.out + t * a.ldo + (int64_t)h * a.vdimp + v) = u32x2_t{pack2bf(acc[0], acc[1]), pack2bf(acc[2], acc[3])};
 }
@@ -626,7 +728,11 @@ extern "C" int glm_latent_prepare(const void* qc, int64_t ldq, int c_off, int64_
                   GLM_ERR_INVALID, "glm_latent_prepare: bad shape T=%ld Ta=%ld H=%d dimp=%d rank=%d", (long)T, (long)Ta, H, dimp, rank);
     GLM_CHECK_ARG(act_f32 || Ta == 0 || (wukt && qa && glm_aligned16(wukt) && glm_aligned16(qc)), GLM_ERR_INVALID, "glm_latent_prepare: absorbed rows need W_uk^T and q'");
     if (T == 0) return GLM_OK;
-    PrepArgs a = {qc, ldq, c_off, T, Ta, H, dimp, rank, rp, norm_w, eps, slots, cache, n_slots, crow, c_out, n_crows, (const bf16_t*)wukt, (bf16_t*)qa};
+    PrepArgs a = {};
+    a.q = a.qc = qc; a.ldqq = a.ldq = ldq; a.hd = dimp; a.c_off = c_off;
+    a.T = T; a.Ta = Ta; a.H = H; a.dimp = dimp; a.rank = rank; a.rp = a.rc = rp;
+    a.norm_w = norm_w; a.eps = eps; a.slots = slots; a.cache = cache; a.n_slots = n_slots; a.crow = crow; a.c_out = c_out; a.n_crows = n_crows;
+    a.wukt = (const bf16_t*)wukt; a.qa = (bf16_t*)qa;
     const bool many = !act_f32 && T >= 2048;
     const int64_t nnorm = many ? (T + 15) / 16 : (T + 3) / 4;
     if (act_f32) {
@@ -638,6 +744,54 @@ extern "C" int glm_latent_prepare(const void* qc, int64_t ldq, int c_off, int64_
         else hipLaunchKernelGGL(latent_prepare_kernel<1>, dim3((unsigned)(nabs + nnorm)), dim3(256), 0, glm_s(stream), a, (int)nabs);
     }
     GLM_CHECK_LAUNCH("glm_latent_prepare");
+    return GLM_OK;
+}
+
+extern "C" int glm_rope_pairs(const int32_t* pos, const double* freq, int n_freq, float mscale, float* cs, int64_t T, int pairs, glm_stream_t stream) {
+    GLM_CHECK_ARG(pos && cs && (freq || n_freq == 0) && T >= 0 && pairs > 0 && n_freq >= 0 && n_freq <= pairs && (T * pairs + 255) / 256 < (1ll << 31), GLM_ERR_INVALID,
+                  "glm_rope_pairs: bad shape T=%ld pairs=%d freq=%d", (long)T, pairs, n_freq);
+    if (T == 0) return GLM_OK;
+    hipLaunchKernelGGL(rope_pairs_kernel, dim3((unsigned)((T * pairs + 255) / 256)), dim3(256), 0, glm_s(stream), pos, freq, n_freq, mscale, cs, T, pairs);
+    GLM_CHECK_LAUNCH("glm_rope_pairs");
+    return GLM_OK;
+}
+
+extern "C" int glm_latent_rows(const void* qc, int64_t ldq, int c_off, int rank, int rp, int rotp, const float* norm_w, const float* cs, float eps, const int32_t* slots, void* cache,
+                               int64_t n_slots, const int32_t* crow, void* c_out, int64_t n_crows, int cq_off, int cq_rank, int cq_rp, const float* cq_norm, void* cq_out,
+                               int64_t ld_cq, int64_t T, int act_f32, glm_stream_t stream) {
+    GLM_CHECK_ARG(qc && norm_w && slots && cache && T >= 0 && rank > 0 && rp >= rank && rp % 8 == 0 && rotp >= 0 && rotp % 8 == 0 && (rotp == 0 || cs) && c_off >= 0 && c_off % 8 == 0 &&
+                      ldq % 8 == 0 && ldq >= (int64_t)c_off + rp + rotp && n_slots > 0 && (!crow || (c_out && n_crows > 0)) && glm_aligned16(qc) && glm_aligned16(cache), GLM_ERR_INVALID,
+                  "glm_latent_rows: bad shape T=%ld rank=%d rot=%d", (long)T, rank, rotp);
+    GLM_CHECK_ARG(!cq_out || (cq_norm && cq_off >= 0 && cq_off % 8 == 0 && cq_rank > 0 && cq_rp >= cq_rank && cq_rp % 8 == 0 && ldq >= (int64_t)cq_off + cq_rp && ld_cq >= cq_rp &&
+                              ld_cq % 8 == 0 && glm_aligned16(cq_out)), GLM_ERR_INVALID, "glm_latent_rows: bad query latent of %d columns", cq_rank);
+    if (T == 0) return GLM_OK;
+    PrepArgs a = {};
+    a.qc = qc; a.ldq = ldq; a.c_off = c_off; a.T = T; a.rank = rank; a.rp = rp; a.rotp = rotp; a.rc = rp + rotp; a.cs = cs;
+    a.norm_w = norm_w; a.eps = eps; a.slots = slots; a.cache = cache; a.n_slots = n_slots; a.crow = crow; a.c_out = c_out; a.n_crows = n_crows;
+    a.cq_off = cq_off; a.cq_rank = cq_rank; a.cq_rp = cq_rp; a.cq_norm = cq_norm; a.cq_out = cq_out; a.ld_cq = ld_cq;
+    const int nr = !act_f32 && T >= 2048 ? 4 : 1;
+    const dim3 grid((unsigned)((T + 4 * nr - 1) / (4 * nr)), cq_out ? 2 : 1);
+    if (act_f32) hipLaunchKernelGGL((latent_rows_kernel<float, 1>), grid, dim3(256), 0, glm_s(stream), a);
+    else if (nr == 4) hipLaunchKernelGGL((latent_rows_kernel<bf16_t, 4>), grid, dim3(256), 0, glm_s(stream), a);
+    else hipLaunchKernelGGL((latent_rows_kernel<bf16_t, 1>), grid, dim3(256), 0, glm_s(stream), a);
+    GLM_CHECK_LAUNCH("glm_latent_rows");
+    return GLM_OK;
+}
+
+extern "C" int glm_latent_absorb(const void* q, int64_t ldq, int64_t Ta, int H, int dimp, int rp, int rotp, const float* cs, const void* wukt, void* qa, int act_f32,
+                                 glm_stream_t stream) {
+    GLM_CHECK_ARG(q && qa && Ta >= 0 && H > 0 && dimp > 0 && dimp % 8 == 0 && rp > 0 && rp % 8 == 0 && rotp >= 0 && rotp % 8 == 0 && (rotp == 0 || cs) && ldq % 8 == 0 &&
+                      ldq >= (int64_t)H * (dimp + rotp) && (act_f32 || (wukt && glm_aligned16(wukt))) && glm_aligned16(q) && glm_aligned16(qa), GLM_ERR_INVALID,
+                  "glm_latent_absorb: bad shape Ta=%ld H=%d dimp=%d", (long)Ta, H, dimp);
+    if (Ta == 0 || (act_f32 && rotp == 0)) return GLM_OK;
+    PrepArgs a = {};
+    a.q = q; a.ldqq = ldq; a.hd = dimp + rotp; a.T = Ta; a.Ta = Ta; a.H = H; a.dimp = dimp; a.rank = a.rp = rp; a.rotp = rotp; a.rc = rp + rotp; a.cs = cs;
+    a.wukt = (const bf16_t*)wukt; a.qa = (bf16_t*)qa;
+    const int64_t nb = act_f32 ? (Ta * H * (rotp / 8) + 255) / 256 : (int64_t)((rp + 63) / 64 + (rotp > 0)) * H * ((Ta + 16 * PREP_TT - 1) / (16 * PREP_TT));
+    GLM_CHECK_ARG(nb < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_latent_absorb: grid too large");
+    if (act_f32) hipLaunchKernelGGL(latent_rotate_f32_kernel, dim3((unsigned)nb), dim3(256), 0, glm_s(stream), a);
+    else hipLaunchKernelGGL(latent_prepare_kernel<1>, dim3((unsigned)nb), dim3(256), 0, glm_s(stream), a, (int)nb);
+    GLM_CHECK_LAUNCH("glm_latent_absorb");
     return GLM_OK;
 }
 
@@ -660,15 +814,15 @@ extern "C" int glm_latent_attn_max_rows(int rp) {
 
 extern "C" int glm_latent_attn(const void* qa, const void* cache, int64_t n_blocks, int block_size, const int32_t* tile_tok, const int32_t* tile_n,
                                int n_tiles, int tokens_per_tile, const int32_t* pos, const int32_t* seq_of, const int32_t* block_tables, int64_t bt_stride,
-                               int64_t Ta, int H, int rank, int rp, int window, float scale, const float* sink, int nsplit, void* ctx, float* part_o,
+                               int64_t Ta, int H, int rp, int vp, int window, float scale, const float* sink, int nsplit, void* ctx, float* part_o,
                                float* part_ml, int act_f32, glm_stream_t stream) {
-    GLM_CHECK_ARG(qa && cache && pos && seq_of && block_tables && sink && n_blocks > 0 && Ta >= 0 && H > 0 && rank > 0 && rp >= rank && rp % 8 == 0 && window > 0 &&
+    GLM_CHECK_ARG(qa && cache && pos && seq_of && block_tables && sink && n_blocks > 0 && Ta >= 0 && H > 0 && vp > 0 && rp >= vp && rp % 8 == 0 && vp % 8 == 0 && window > 0 &&
                       bt_stride > 0, GLM_ERR_INVALID, "glm_latent_attn: bad shape Ta=%ld H=%d rp=%d window=%d", (long)Ta, H, rp, window);
     int sh = 0;
     while ((1 << sh) < block_size) ++sh;
     GLM_CHECK_ARG((1 << sh) == block_size && block_size >= 32, GLM_ERR_UNSUPPORTED, "glm_latent_attn: block size %d is not a power of two >= 32", block_size);
     if (Ta == 0) return GLM_OK;
-    AttnArgs a = {qa, cache, tile_tok, tile_n, pos, seq_of, block_tables, bt_stride, n_blocks, sh, Ta, H, rank, rp, window, scale, sink,
+    AttnArgs a = {qa, cache, tile_tok, tile_n, pos, seq_of, block_tables, bt_stride, n_blocks, sh, Ta, H, rp, vp, window, scale, sink,
                   n_tiles, 0, 0, tokens_per_tile, nsplit, (bf16_t*)ctx, part_o, part_ml};
     hipStream_t st = glm_s(stream);
     if (act_f32) {
@@ -703,12 +857,13 @@ extern "C" int glm_latent_attn(const void* qa, const void* cache, int64_t n_bloc
     }
 }
 
-extern "C" int glm_latent_up(const void* ctx, const void* wuv, void* out, int64_t ldo, int64_t Ta, int H, int vdimp, int rp, glm_stream_t stream) {
+extern "C" int glm_latent_up(const void* ctx, const void* wuv, void* out, const void* gate, int64_t ldg, int64_t ldo, int64_t Ta, int H, int vdimp, int rp, glm_stream_t stream) {
+    GLM_CHECK_ARG((!gate || (ldg >= (int64_t)H * vdimp && ldg % 4 == 0)), GLM_ERR_INVALID, "glm_latent_up: bad gate (ldg=%ld)", (long)ldg);
     GLM_CHECK_ARG(ctx && wuv && out && Ta >= 0 && H > 0 && vdimp > 0 && vdimp % 8 == 0 && rp > 0 && rp % 8 == 0 && ldo >= (int64_t)H * vdimp && ldo % 4 == 0 &&
                       glm_aligned16(ctx) && glm_aligned16(wuv), GLM_ERR_INVALID, "glm_latent_up: bad shape Ta=%ld H=%d vdimp=%d", (long)Ta, H, vdimp);
     GLM_CHECK_ARG((Ta + 15) / 16 <= 65535, GLM_ERR_UNSUPPORTED, "glm_latent_up: too many rows");
     if (Ta == 0) return GLM_OK;
-    UpArgs a = {(const bf16_t*)ctx, (const bf16_t*)wuv, (bf16_t*)out, ldo, Ta, H, vdimp, rp};
+    UpArgs a = {(const bf16_t*)ctx, (const bf16_t*)wuv, (bf16_t*)out, (const bf16_t*)gate, ldg, ldo, Ta, H, vdimp, rp};
     const int items = H * ((vdimp + 15) / 16);
     hipLaunchKernelGGL(latent_up_kernel, dim3((unsigned)((items + 3) / 4), (unsigned)((Ta + 15) / 16)), dim3(256), 0, glm_s(stream), a);
     GLM_CHECK_LAUNCH("glm_latent_up");

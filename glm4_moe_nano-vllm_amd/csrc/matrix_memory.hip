@@ -9,11 +9,16 @@
 //
 // State, gates and everything between the projections and y in fp32.  gfx950 only.
 //
+// And its plain relative, the linear memory of attention with a constant decay per head (GATED = false):
+//
+//     S_t = decay S_(t-1) + k_t v_t^T        o_t = S_t^T q_t        y_t = o_t / rms(o_t) . norm . gate_t      the norm over all heads together
+//
 //   memory_recurrent   token by token, state in registers (decoded tokens, short portions, fp32): one (sequence, head) per workgroup, gate
 //                      projections and the output norm included; memory_recurrent_any for head sizes beyond its registers
 //   memory_gates       gate projections of long portions and the part of the gates' scan that stays inside a chunk of 64 tokens
 //   memory_chunkwise   long portions: 64 tokens at a time on the matrix cores, one (sequence, head, 64 value columns) per workgroup
 //   memory_output      norm and output gate of memory_chunkwise's rows
+//   row_norm_gate      the linear memory's norm and gate, for rows of either form
 //
 // Rooflines: the recurrent form is HBM-bound (the state is read once and written once per step), the chunkwise form is bound by the chain
 // of its chunks (the state of one is the input of the next).
@@ -22,6 +27,8 @@
 // lanes; with D_ts = e^(b_t - m_t + i_s - b_s) for s <= t and c_t = e^(b_t + m_in - m_t),
 //
 //     S_t^T q_t = c_t S_in^T q_t + sum_s D_ts (k_s . q_t) v_s            S_out = c_L S_in + sum_s e^(b_L - m_L + i_s - b_s) k_s v_s^T
+//
+// (the linear memory: D_ts = decay^(t-s), c_t = decay^(t+1), from a table of powers; they are the same in every chunk and stay in registers)
 //
 // q, k and v are bf16 as the projection left them; the weights D (k . q), the decayed values and the state enter the matrix cores as a
 // bf16 pair hi + lo each, so the products keep about 16 bits of their fp32 operand.
@@ -54,6 +61,7 @@ struct RecArgs {
     const int32_t *pos, *q_start, *state_in, *state_out;
     int seqs, H, dim, dimp, vdim, vdimp;
     float cap, eps;
+    const float* decay;   // [H]: the linear memory; y is then fp32 and holds o as it is
 };
 
 template <typename T>
@@ -88,9 +96,11 @@ __device__ __forceinline__ void mm_gate_parts(const RecArgs& a, int64_t r, int h
     }
 }
 
+__device__ __forceinline__ void mm_st_o(const RecArgs& a, int64_t r, int h, int c, float v) { reinterpret_cast<float*>(a.y)[r * a.ldy + (int64_t)h * a.vdimp + c] = v; }
+
 // dimp <= 16 KD, vdimp <= 64 NW.  256 NW threads: column block tid / 256 (64 columns), thread (rg, cq) of a block holds rows rg + 16 k of the
 // four columns cq.
-template <typename T, int KD, int NW>
+template <typename T, int KD, int NW, bool GATED>
 __global__ __launch_bounds__(256 * NW) void memory_recurrent_kernel(const RecArgs a) {
     constexpr int NT = 256 * NW, NWV = 4 * NW;
     __shared__ float s_q[16 * KD], s_k[16 * KD], s_g[2][NWV], s_nq[NWV], s_ss[NWV];
@@ -104,7 +114,10 @@ __global__ __launch_bounds__(256 * NW) void memory_recurrent_kernel(const RecArg
     if (r1 <= r0) return;
     if (a.pos[r0] < 0) {  // unused rows of a padded batch
         for (int r = r0; r < r1; ++r)
-            for (int c = tid; c < a.vdimp; c += NT) mm_st<T>(a.y, (int64_t)r * a.ldy + (int64_t)h * a.vdimp + c, 0.f);
+            for (int c = tid; c < a.vdimp; c += NT) {
+                if constexpr (GATED) mm_st<T>(a.y, (int64_t)r * a.ldy + (int64_t)h * a.vdimp + c, 0.f);
+                else mm_st_o(a, r, h, c, 0.f);
+            }
         return;
     }
     f32x4_t S[KD];
@@ -117,19 +130,22 @@ __global__ __launch_bounds__(256 * NW) void memory_recurrent_kernel(const RecArg
         S[k] = f32x4_t{0.f, 0.f, 0.f, 0.f};
         if (!fresh && con && d < a.dimp) S[k] = *reinterpret_cast<const f32x4_t*>(a.S + (sin * a.dimp + d) * a.vdimp + col);
     }
-    if (!fresh) {
+    if (GATED && !fresh) {
         if (tid < a.dimp) n = a.n[sin * a.dimp + tid];
         m = a.m[sin];
     }
-    const float scale = 1.0f / sqrtf((float)a.dim), bi = a.bif[h], bf = a.bif[a.H + h], inv_v = 1.0f / (float)a.vdim;
+    const float scale = GATED ? 1.0f / sqrtf((float)a.dim) : 1.0f, bi = GATED ? a.bif[h] : 0.f, bf = GATED ? a.bif[a.H + h] : 0.f, inv_v = 1.0f / (float)a.vdim;
+    float keep = GATED ? 0.f : a.decay[h], add = 1.0f;
     for (int r = r0; r < r1; ++r) {
-        float gi, gf;
-        mm_gate_parts<T>(a, r, h, tid, NT, gi, gf);
-        gi = wave_sum(gi);
-        gf = wave_sum(gf);
-        if (lane == 0) {
-            s_g[0][wave] = gi;
-            s_g[1][wave] = gf;
+        if constexpr (GATED) {
+            float gi, gf;
+            mm_gate_parts<T>(a, r, h, tid, NT, gi, gf);
+            gi = wave_sum(gi);
+            gf = wave_sum(gf);
+            if (lane == 0) {
+                s_g[0][wave] = gi;
+                s_g[1][wave] = gf;
+            }
         }
         const int64_t base = (int64_t)r * a.ldx;
         float kd = 0.f, qd = 0.f;
@@ -144,16 +160,20 @@ __global__ __launch_bounds__(256 * NW) void memory_recurrent_kernel(const RecArg
         f32x4_t v = {0.f, 0.f, 0.f, 0.f};
         if (con) v = mm_ld4<T>(a.x, base + a.v_off + (int64_t)h * a.vdimp + col);
         __syncthreads();
-        float zi = 0.f, zf = 0.f;
+        if constexpr (GATED) {
+            float zi = 0.f, zf = 0.f;
 #pragma unroll
-        for (int w = 0; w < NWV; ++w) {
-            zi += s_g[0][w];
-            zf += s_g[1][w];
+            for (int w = 0; w < NWV; ++w) {
+                zi += s_g[0][w];
+                zf += s_g[1][w];
+            }
+            const float li = mm_cap(zi + bi, a.cap), lf = mm_log_sigmoid(mm_cap(zf + bf, a.cap));
+            const float mn = fmaxf(lf + m, li);
+            keep = expf(lf + m - mn);
+            add = expf(li - mn);
+            m = mn;
+            n = keep * n + add * kd;
         }
-        const float li = mm_cap(zi + bi, a.cap), lf = mm_log_sigmoid(mm_cap(zf + bf, a.cap));
-        const float mn = fmaxf(lf + m, li), keep = expf(lf + m - mn), add = expf(li - mn);
-        m = mn;
-        n = keep * n + add * kd;
         f32x4_t o = {0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int k = 0; k < KD; ++k) {
@@ -170,10 +190,16 @@ __global__ __launch_bounds__(256 * NW) void memory_recurrent_kernel(const RecArg
             o[e] += __shfl_xor(o[e], 32, 64);
         }
         if (lane < 16) *reinterpret_cast<f32x4_t*>(&s_o[cb][wv][cq * 4]) = o;
-        const float nq = wave_sum(n * qd);
-        if (lane == 0) s_nq[wave] = nq;
-        __syncthreads();
         float den = 0.f;
+        if constexpr (GATED) {
+            const float nq = wave_sum(n * qd);
+            if (lane == 0) s_nq[wave] = nq;
+        }
+        __syncthreads();
+        if constexpr (!GATED) {  // (s_o is written again behind the next token's first barrier)
+            if (tid < a.vdimp) mm_st_o(a, r, h, tid, (s_o[tid >> 6][0][tid & 63] + s_o[tid >> 6][1][tid & 63]) + (s_o[tid >> 6][2][tid & 63] + s_o[tid >> 6][3][tid & 63]));
+            continue;
+        }
 #pragma unroll
         for (int w = 0; w < NWV; ++w) den += s_nq[w];
         den = fmaxf(fabsf(den), expf(-m)) + 1e-6f;
@@ -198,13 +224,15 @@ __global__ __launch_bounds__(256 * NW) void memory_recurrent_kernel(const RecArg
         const int d = rg + 16 * k;
         if (con && d < a.dimp) *reinterpret_cast<f32x4_t*>(a.S + (sout * a.dimp + d) * a.vdimp + col) = S[k];
     }
-    if (tid < a.dimp) a.n[sout * a.dimp + tid] = n;
-    if (tid == 0) a.m[sout] = m;
+    if constexpr (GATED) {
+        if (tid < a.dimp) a.n[sout * a.dimp + tid] = n;
+        if (tid == 0) a.m[sout] = m;
+    }
 }
 
 // any head size: the state lives in its rows in memory (the row set that the step writes; scratch rows are not needed because a row set that
 // nobody keeps is only ever asked for by unused rows)
-template <typename T>
+template <typename T, bool GATED>
 __global__ __launch_bounds__(256) void memory_recurrent_any_kernel(const RecArgs a) {
     extern __shared__ __attribute__((aligned(16))) char smem[];
     float* s_q = reinterpret_cast<float*>(smem);  // [dimp]
@@ -219,19 +247,25 @@ __global__ __launch_bounds__(256) void memory_recurrent_any_kernel(const RecArgs
     const int64_t so = a.state_out[seq];
     if (a.pos[r0] < 0 || so < 0 || so >= a.n_state) {
         for (int r = r0; r < r1; ++r)
-            for (int c = tid; c < a.vdimp; c += 256) mm_st<T>(a.y, (int64_t)r * a.ldy + (int64_t)h * a.vdimp + c, 0.f);
+            for (int c = tid; c < a.vdimp; c += 256) {
+                if constexpr (GATED) mm_st<T>(a.y, (int64_t)r * a.ldy + (int64_t)h * a.vdimp + c, 0.f);
+                else mm_st_o(a, r, h, c, 0.f);
+            }
         return;
     }
     const int64_t sin = min(max((int64_t)a.state_in[seq], (int64_t)0), a.n_state - 1) * a.H + h, sout = so * a.H + h;
     const bool fresh = a.pos[r0] == 0;
-    const float scale = 1.0f / sqrtf((float)a.dim), bi = a.bif[h], bf = a.bif[a.H + h], inv_v = 1.0f / (float)a.vdim;
-    float m = fresh ? 0.f : a.m[sin];
+    const float scale = GATED ? 1.0f / sqrtf((float)a.dim) : 1.0f, bi = GATED ? a.bif[h] : 0.f, bf = GATED ? a.bif[a.H + h] : 0.f, inv_v = 1.0f / (float)a.vdim;
+    float m = !GATED || fresh ? 0.f : a.m[sin];
+    float keep = GATED ? 0.f : a.decay[h], add = 1.0f;
     for (int r = r0; r < r1; ++r) {
         const bool first = r == r0;
-        float gi, gf;
-        mm_gate_parts<T>(a, r, h, tid, 256, gi, gf);
-        gi = wave_sum(gi);
-        gf = wave_sum(gf);
+        float gi = 0.f, gf = 0.f;
+        if constexpr (GATED) {
+            mm_gate_parts<T>(a, r, h, tid, 256, gi, gf);
+            gi = wave_sum(gi);
+            gf = wave_sum(gf);
+        }
         __syncthreads();
         if (lane == 0) {
             s_red[0][wave] = gi;
@@ -244,20 +278,25 @@ __global__ __launch_bounds__(256) void memory_recurrent_any_kernel(const RecArgs
         }
         __syncthreads();
         const float zi = s_red[0][0] + s_red[0][1] + s_red[0][2] + s_red[0][3], zf = s_red[1][0] + s_red[1][1] + s_red[1][2] + s_red[1][3];
-        const float li = mm_cap(zi + bi, a.cap), lf = mm_log_sigmoid(mm_cap(zf + bf, a.cap));
-        const float mn = fmaxf(lf + m, li), keep = expf(lf + m - mn), add = expf(li - mn);
-        m = mn;
-        float nq = 0.f;
-        for (int d = tid; d < a.dimp; d += 256) {
-            const float old = !first ? a.n[sout * a.dimp + d] : fresh ? 0.f : a.n[sin * a.dimp + d];
-            const float nn = keep * old + add * s_k[d];
-            a.n[sout * a.dimp + d] = nn;
-            nq += nn * s_q[d];
+        float den = 1.0f;
+        if constexpr (GATED) {
+            const float li = mm_cap(zi + bi, a.cap), lf = mm_log_sigmoid(mm_cap(zf + bf, a.cap));
+            const float mn = fmaxf(lf + m, li);
+            keep = expf(lf + m - mn);
+            add = expf(li - mn);
+            m = mn;
+            float nq = 0.f;
+            for (int d = tid; d < a.dimp; d += 256) {
+                const float old = !first ? a.n[sout * a.dimp + d] : fresh ? 0.f : a.n[sin * a.dimp + d];
+                const float nn = keep * old + add * s_k[d];
+                a.n[sout * a.dimp + d] = nn;
+                nq += nn * s_q[d];
+            }
+            nq = wave_sum(nq);
+            if (lane == 0) s_red[2][wave] = nq;
+            __syncthreads();
+            den = fmaxf(fabsf(s_red[2][0] + s_red[2][1] + s_red[2][2] + s_red[2][3]), expf(-m)) + 1e-6f;
         }
-        nq = wave_sum(nq);
-        if (lane == 0) s_red[2][wave] = nq;
-        __syncthreads();
-        const float den = fmaxf(fabsf(s_red[2][0] + s_red[2][1] + s_red[2][2] + s_red[2][3]), expf(-m)) + 1e-6f;
         float ss = 0.f;
         for (int c0 = 0; c0 < a.vdimp; c0 += 64) {
             const int col = c0 + cq * 4;
@@ -282,12 +321,14 @@ __global__ __launch_bounds__(256) void memory_recurrent_any_kernel(const RecArgs
             if (tid < 64 && c0 + tid < a.vdimp) {
                 float ov = 0.f;
                 for (int i = 0; i < 16; ++i) ov += s_part[i][tid];
-                ov /= den;
+                if constexpr (GATED) ov /= den;
+                else mm_st_o(a, r, h, c0 + tid, ov);
                 s_o[c0 + tid] = ov;
                 ss += ov * ov;
             }
             __syncthreads();
         }
+        if constexpr (!GATED) continue;
         if (wave == 0) {
             ss = wave_sum(ss);
             if (lane == 0) s_red[0][0] = ss;
@@ -298,7 +339,7 @@ __global__ __launch_bounds__(256) void memory_recurrent_any_kernel(const RecArgs
             mm_st<T>(a.y, (int64_t)r * a.ldy + (int64_t)h * a.vdimp + c,
                      s_o[c] / rms * a.norm[(int64_t)h * a.vdimp + c] * mm_sigmoid(mm_ld<T>(a.x, base + a.g_off + (int64_t)h * a.vdimp + c)));
     }
-    if (tid == 0) a.m[sout] = m;
+    if (GATED && tid == 0) a.m[sout] = m;
 }
 
 // ---------------------------------------------------------------------------------------------------------------------------
@@ -398,6 +439,7 @@ struct ChunkArgs {
     int64_t n_state;
     const int32_t *pos, *q_start, *state_in, *state_out;  // of the long portions; q_start and pos relative to x's first row
     int H, dim, dimp, vdimp, vtiles;
+    const float* powers;  // [H][65] decay^j: the linear memory
 };
 
 template <typename T>
@@ -450,7 +492,7 @@ __device__ __forceinline__ f32x4_t mm_mfma(const bf16x8_t& x, const bf16x8_t& y,
 // (lane (c, g): column c, rows d = 16 i + 4 g + r), is the left operand of the next chunk's readout without leaving the registers.  Of
 // the 64 output rows, half 0 finishes row tiles 0 and 3, half 1 tiles 1 and 2 (equal work under the causal mask); the readouts of the
 // other half come through LDS.
-template <int D>
+template <int D, bool GATED>
 __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArgs a) {
     constexpr int KS = D / 32, DT = D / 16, HT = DT / 2, RB = D * 2, CPR = D / 8, QT = 64 * RB, VTB = 64 * 128, GT = 1024, STAGE = 2 * QT + VTB + GT;
     constexpr int NST = D <= 128 ? 3 : 2;           // LDS stages: chunks on their way are NST - 1
@@ -492,14 +534,33 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
 #pragma unroll
     for (int i = 0; i < NR; ++i) {
         const int d = 16 * (dh * HT + 4 * i + v) + c;
-        nreg[i] = (!fresh && v < HT && d < a.dimp) ? a.n[sin * a.dimp + d] : 0.f;
-        if (g == 0 && v < HT) s_n[d] = nreg[i];
+        nreg[i] = (GATED && !fresh && v < HT && d < a.dimp) ? a.n[sin * a.dimp + d] : 0.f;
+        if (GATED && g == 0 && v < HT) s_n[d] = nreg[i];
     }
-    float m_in = fresh ? 0.f : a.m[sin];
-    const float scale = 1.0f / sqrtf((float)a.dim);
+    float m_in = !GATED || fresh ? 0.f : a.m[sin];
+    const float scale = GATED ? 1.0f / sqrtf((float)a.dim) : 1.0f;
+    // the linear memory's weights: of this wave's rows and keys, of its output rows, of a token in the state behind a whole chunk
+    float dw_c[2][4], wt_c[2][8], inc_a = 0.f, inc_b = 0.f, carry_c = 0.f;
+    const float* pw = GATED ? nullptr : a.powers + h * 65;
+    if constexpr (!GATED) {
+#pragma unroll
+        for (int u = 0; u < 2; ++u)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) {
+                const int d = 16 * v + c - (32 * dh + 16 * u + 4 * g + r);
+                dw_c[u][r] = d >= 0 ? pw[d] : 0.f;
+            }
+#pragma unroll
+        for (int sl = 0; sl < 2; ++sl)
+#pragma unroll
+            for (int e = 0; e < 8; ++e) wt_c[sl][e] = pw[63 - (32 * sl + 4 * g + (e & 3) + (e & 4) * 4)];
+        inc_a = pw[16 * (dh ? 1 : 0) + c + 1];
+        inc_b = pw[16 * (dh ? 2 : 3) + c + 1];
+        carry_c = pw[64];
+    }
     const bf16_t* xq = a.x + (int64_t)r0 * a.ldx + (int64_t)h * a.dimp;
     const bf16_t* xv = a.x + (int64_t)r0 * a.ldx + a.v_off + (int64_t)h * a.vdimp + vt * 64;
-    const float* gp = a.gates + (int64_t)h * a.rows + r0;
+    const float* gp = GATED ? a.gates + (int64_t)h * a.rows + r0 : nullptr;
     const int64_t gpart = (int64_t)a.H * a.rows;
     // per-lane source offsets of the DMA pieces: constant over the chunks
     unsigned qoff[QDMA];
@@ -515,7 +576,7 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
         char* st = smem + (ch % NST) * STAGE;
         const int left = T - ch * 64;
         // gates: i - b, b and the running maximum, 256 bytes each (the other waves' piece is not used)
-        __builtin_amdgcn_global_load_lds((attn_glb_void*)(gp + min(w, 2) * gpart + ch * 64 + min(lane, left - 1)), (attn_lds_void*)(st + 2 * QT + VTB + min(w, 3) * 256), 4, 0, 0);
+        if constexpr (GATED) __builtin_amdgcn_global_load_lds((attn_glb_void*)(gp + min(w, 2) * gpart + ch * 64 + min(lane, left - 1)), (attn_lds_void*)(st + 2 * QT + VTB + min(w, 3) * 256), 4, 0, 0);
         const bf16_t *q = xq + (int64_t)ch * 64 * a.ldx, *k = q + a.k_off, *vv = xv + (int64_t)ch * 64 * a.ldx;
         if (whole && left >= 64) {
 #pragma unroll
@@ -567,7 +628,7 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
     for (int ch = 0; ch < n_chunks; ++ch) {
         const int left = T - ch * 64;
         // the chunk is in (what was issued behind it may be on its way): loads return in order
-        if (ch + NST - 2 < n_chunks) wait_vm<(NST - 2) * (2 * QDMA + 2)>();
+        if (ch + NST - 2 < n_chunks) wait_vm<(NST - 2) * (2 * QDMA + (GATED ? 2 : 1))>();
         else wait_vm<0>();
         mm_barrier();  // ... for every wave, and every wave is past its reads of the chunk before
         if (ch > 0) store_rows(ch - 1);
@@ -575,14 +636,20 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
         const char *qst = smem + (ch % NST) * STAGE, *kst = qst + QT, *vst = kst + QT, *gst = vst + VTB;
         char *pst = smem + (PALIAS ? (ch % NST) * STAGE : POFF), *xst = smem + (XALIAS ? (ch % NST) * STAGE : 0) + XOFF;
         // gates of the chunk, one token per lane, the same in every wave
-        const bool tok = lane < left;
+        const bool tok = GATED && lane < left;
         const float ga = tok ? mm_lds<float>(gst + 4 * lane) : -INFINITY, gb = tok ? mm_lds<float>(gst + 256 + 4 * lane) : 0.f,
                     gm = tok ? mm_lds<float>(gst + 512 + 4 * lane) : 0.f;
         const float mt = gb + fmaxf(m_in, gm);
         const int last = min(left, 64) - 1;
-        const float bL = __shfl(gb, last, 64), mL = __shfl(mt, last, 64);
-        const float carry = __builtin_amdgcn_exp2f(bL + m_in - mL);
-        if (w == 0) {
+        float bL = 0.f, mL = 0.f, carry;
+        if constexpr (GATED) {
+            bL = __shfl(gb, last, 64);
+            mL = __shfl(mt, last, 64);
+            carry = __builtin_amdgcn_exp2f(bL + m_in - mL);
+        } else {
+            carry = last == 63 ? carry_c : pw[last + 1];
+        }
+        if (GATED && w == 0) {
             s_a[lane] = ga;
             s_row[lane] = gb - mt;
             s_in[lane] = __builtin_amdgcn_exp2f(gb + m_in - mt) * scale;
@@ -598,7 +665,7 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
             const u32x4_t k0 = mm_lds<u32x4_t>(kst + dh * 32 * RB + row_rel[i & 1] + (i >> 1) * 128), k1 = mm_lds<u32x4_t>(kst + dh * 32 * RB + row_rel[i & 1] + (i >> 1) * 128 + 16 * RB);
             s[0] = mm_mfma(__builtin_bit_cast(bf16x8_t, k0), __builtin_bit_cast(bf16x8_t, qf), s[0]);
             s[1] = mm_mfma(__builtin_bit_cast(bf16x8_t, k1), __builtin_bit_cast(bf16x8_t, qf), s[1]);
-            if (i / (KS / 2) == dh) {
+            if (GATED && i / (KS / 2) == dh) {
                 const f32x4_t n0 = mm_lds<f32x4_t>(sa + 1792 + 128 * i + 32 * g), n1 = mm_lds<f32x4_t>(sa + 1792 + 128 * i + 32 * g + 16);
 #pragma unroll
                 for (int e = 0; e < 2; ++e) {
@@ -637,7 +704,7 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
         const bf16x8_t vv[2] = {mm_frag(vf[0][0], vf[0][1]), mm_frag(vf[1][0], vf[1][1])};
         // ---- weights of this wave's rows and keys: hi and lo, in the order the second product reads them ----
         const int row = 16 * v + c;
-        const float rowc = mm_lds<float>(sa + 256 + 4 * row), inc = mm_lds<float>(sa + 512 + 4 * row);
+        const float rowc = GATED ? mm_lds<float>(sa + 256 + 4 * row) : 0.f, inc = GATED ? mm_lds<float>(sa + 512 + 4 * row) : 0.f;
         {
             *reinterpret_cast<f32x4_t*>(xst + (w * 2 * 64 + lane) * 16) = x_a;
             *reinterpret_cast<f32x4_t*>(xst + ((w * 2 + 1) * 64 + lane) * 16) = x_b;
@@ -645,10 +712,11 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
 #pragma unroll
             for (int u = 0; u < 2; ++u) {
                 const int k0 = 32 * dh + 16 * u + 4 * g;
-                const f32x4_t ax = mm_lds<f32x4_t>(sa + 4 * k0);
+                f32x4_t ax = {0.f, 0.f, 0.f, 0.f};
+                if constexpr (GATED) ax = mm_lds<f32x4_t>(sa + 4 * k0);
 #pragma unroll
                 for (int r = 0; r < 4; ++r) {
-                    const float dw = k0 + r <= row ? __builtin_amdgcn_exp2f(rowc + ax[r]) * scale : 0.f;
+                    const float dw = !GATED ? dw_c[u][r] : k0 + r <= row ? __builtin_amdgcn_exp2f(rowc + ax[r]) * scale : 0.f;
                     p[4 * u + r] = s[u][r] * dw;
                     dsum += p[4 * u + r];
                 }
@@ -658,21 +726,35 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
             const int chunk = ((4 * dh + g) ^ (c & 7)) << 4;
             *reinterpret_cast<bf16x8_t*>(pst + row * 128 + chunk) = hi;
             *reinterpret_cast<bf16x8_t*>(pst + 8192 + row * 128 + chunk) = lo;
-            nq = fmaf(nq, inc, dsum);
-            nq += __shfl_xor(nq, 16, 64);
-            nq += __shfl_xor(nq, 32, 64);
-            if (g == 0) s_den[64 * dh + row] = nq;
+            if constexpr (GATED) {
+                nq = fmaf(nq, inc, dsum);
+                nq += __shfl_xor(nq, 16, 64);
+                nq += __shfl_xor(nq, 32, 64);
+                if (g == 0) s_den[64 * dh + row] = nq;
+            }
         }
         // ---- state of the next chunk ----
         bf16x8_t vhi[2], vlo[2];
         float wt[2][8];
 #pragma unroll
         for (int sl = 0; sl < 2; ++sl) {
-            const f32x4_t w0 = mm_lds<f32x4_t>(sa + 1024 + 128 * sl + 16 * g), w1 = mm_lds<f32x4_t>(sa + 1024 + 128 * sl + 64 + 16 * g);
+            f32x4_t w0 = {0.f, 0.f, 0.f, 0.f}, w1 = w0;
+            if constexpr (GATED) {
+                w0 = mm_lds<f32x4_t>(sa + 1024 + 128 * sl + 16 * g);
+                w1 = mm_lds<f32x4_t>(sa + 1024 + 128 * sl + 64 + 16 * g);
+            }
             float p[8];
 #pragma unroll
             for (int e = 0; e < 8; ++e) {
-                wt[sl][e] = e < 4 ? w0[e & 3] : w1[e & 3];
+                if constexpr (GATED) {
+                    wt[sl][e] = e < 4 ? w0[e & 3] : w1[e & 3];
+                } else {
+                    wt[sl][e] = wt_c[sl][e];
+                    if (last < 63) {  // the portion's last chunk
+                        const int d = last - (32 * sl + 4 * g + (e & 3) + (e & 4) * 4);
+                        wt[sl][e] = d >= 0 ? pw[d] : 0.f;
+                    }
+                }
                 p[e] = wt[sl][e] * (float)vv[sl][e];
             }
             mm_split(p, vhi[sl], vlo[sl]);
@@ -696,6 +778,7 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
                 for (int x = 0; x < 2; ++x)
 #pragma unroll
                     for (int jj = 0; jj < GI; ++jj) S[i0 + jj] = mm_mfma(mm_frag(kf[jj][sl][0], kf[jj][sl][1]), x ? vlo[sl] : vhi[sl], S[i0 + jj]);
+            if constexpr (!GATED) return;
             float nn = 0.f;   // n of the rows 16 (dh HT + i0 + v) + c
 #pragma unroll
             for (int jj = 0; jj < GI; ++jj) {
@@ -713,7 +796,7 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
         });
         mm_barrier();
         // ---- output rows ----
-        if (g == 0 && v < HT) {
+        if (GATED && g == 0 && v < HT) {
 #pragma unroll
             for (int i = 0; i < NR; ++i) s_n[16 * (dh * HT + 4 * i + v) + c] = nreg[i];  // read again behind the next barrier
         }
@@ -721,8 +804,8 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
         o_a += mm_lds<f32x4_t>(xst + (ow * 2 * 64 + lane) * 16);
         o_b += mm_lds<f32x4_t>(xst + ((ow * 2 + 1) * 64 + lane) * 16);
         const int ta = 16 * rt_a + c, tb = 16 * rt_b + c;
-        o_a *= mm_lds<float>(sa + 512 + 4 * ta);
-        o_b *= mm_lds<float>(sa + 512 + 4 * tb);
+        o_a *= GATED ? mm_lds<float>(sa + 512 + 4 * ta) : inc_a;
+        o_b *= GATED ? mm_lds<float>(sa + 512 + 4 * tb) : inc_b;
         const unsigned ca = (g ^ (c & 7)) << 4, cb = ((4 + g) ^ (c & 7)) << 4;
         const bf16x8_t pa0 = mm_lds<bf16x8_t>(pst + ta * 128 + ca), pa1 = mm_lds<bf16x8_t>(pst + 8192 + ta * 128 + ca);   // tiles 0 and 1: keys 32 .. 63 are all in the future
         const bf16x8_t pb0 = mm_lds<bf16x8_t>(pst + tb * 128 + ca), pb1 = mm_lds<bf16x8_t>(pst + 8192 + tb * 128 + ca);
@@ -733,8 +816,11 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
         o_a = mm_mfma(vv[0], pa1, o_a);
         o_b = mm_mfma(vv[1], pb2, o_b);
         o_b = mm_mfma(vv[1], pb3, o_b);
-        const float ia = __builtin_amdgcn_rcpf(fmaxf(fabsf(mm_lds<float>(sa + 1280 + 4 * ta) + mm_lds<float>(sa + 1536 + 4 * ta)), mm_lds<float>(sa + 768 + 4 * ta)) + 1e-6f);
-        const float ib = __builtin_amdgcn_rcpf(fmaxf(fabsf(mm_lds<float>(sa + 1280 + 4 * tb) + mm_lds<float>(sa + 1536 + 4 * tb)), mm_lds<float>(sa + 768 + 4 * tb)) + 1e-6f);
+        float ia = 1.0f, ib = 1.0f;
+        if constexpr (GATED) {
+            ia = __builtin_amdgcn_rcpf(fmaxf(fabsf(mm_lds<float>(sa + 1280 + 4 * ta) + mm_lds<float>(sa + 1536 + 4 * ta)), mm_lds<float>(sa + 768 + 4 * ta)) + 1e-6f);
+            ib = __builtin_amdgcn_rcpf(fmaxf(fabsf(mm_lds<float>(sa + 1280 + 4 * tb) + mm_lds<float>(sa + 1536 + 4 * tb)), mm_lds<float>(sa + 768 + 4 * tb)) + 1e-6f);
+        }
         rows_out[0] = u32x2_t{pack2bf(o_a[0] * ia, o_a[1] * ia), pack2bf(o_a[2] * ia, o_a[3] * ia)};
         rows_out[1] = u32x2_t{pack2bf(o_b[0] * ib, o_b[1] * ib), pack2bf(o_b[2] * ib, o_b[3] * ib)};
         m_in = mL;
@@ -750,7 +836,7 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
             const int d = 16 * (dh * HT + i) + 4 * g + r;
             if (con && d < a.dimp) a.S[(sout * a.dimp + d) * a.vdimp + col] = S[i][r];
         }
-    if (vt == 0) {
+    if (GATED && vt == 0) {
 #pragma unroll
         for (int i = 0; i < NR; ++i) {
             const int d = 16 * (dh * HT + 4 * i + v) + c;
@@ -804,9 +890,41 @@ __global__ __launch_bounds__(256) void memory_output_kernel(const OutArgs a) {
     }
 }
 
+// y = o / rms(o) . norm . gate over whole rows, one wave per row; n: true number of columns (padding columns of o are zeros)
+template <typename O, typename Y>
+__global__ __launch_bounds__(256) void row_norm_gate_kernel(const O* __restrict__ o, int64_t ldo, const Y* __restrict__ gate, int64_t ldg, const float* __restrict__ norm,
+                                                            Y* __restrict__ y, int64_t ldy, int64_t T, int n, int np, float eps) {
+    const int lane = threadIdx.x & 63;
+    const int64_t r = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (r >= T) return;
+    float sq = 0.f;
+    f32x4_t u[2][2];  // up to 1024 columns stay in registers
+    for (int c = lane * 8, i = 0; c < np; c += 512, ++i) {
+        const f32x4_t a = mm_ld4<O>(o, r * ldo + c), b = mm_ld4<O>(o, r * ldo + c + 4);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) sq += a[e] * a[e] + b[e] * b[e];
+        if (i < 2) {
+            if (i == 0) { u[0][0] = a; u[0][1] = b; } else { u[1][0] = a; u[1][1] = b; }
+        }
+    }
+    const float inv = 1.0f / sqrtf(wave_sum(sq) / (float)n + eps);
+    for (int c = lane * 8, i = 0; c < np; c += 512, ++i) {
+#pragma unroll
+        for (int hlf = 0; hlf < 2; ++hlf) {
+            f32x4_t v = i == 0 ? u[0][hlf] : i == 1 ? u[1][hlf] : mm_ld4<O>(o, r * ldo + c + 4 * hlf);
+            const f32x4_t g = mm_ld4<Y>(gate, r * ldg + c + 4 * hlf), w = *reinterpret_cast<const f32x4_t*>(norm + c + 4 * hlf);
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = v[e] * inv * w[e] * g[e];
+            if constexpr (sizeof(Y) == 4) *reinterpret_cast<f32x4_t*>(y + r * ldy + c + 4 * hlf) = v;
+            else *reinterpret_cast<u32x2_t*>(y + r * ldy + c + 4 * hlf) = u32x2_t{pack2bf(v[0], v[1]), pack2bf(v[2], v[3])};
+        }
+    }
+}
+
 template <typename T, int KD, int NW>
 int launch_rec(const RecArgs& a, hipStream_t st) {
-    hipLaunchKernelGGL((memory_recurrent_kernel<T, KD, NW>), dim3((unsigned)(a.seqs * a.H)), dim3(256 * NW), 0, st, a);
+    if (a.decay) hipLaunchKernelGGL((memory_recurrent_kernel<T, KD, NW, false>), dim3((unsigned)(a.seqs * a.H)), dim3(256 * NW), 0, st, a);
+    else hipLaunchKernelGGL((memory_recurrent_kernel<T, KD, NW, true>), dim3((unsigned)(a.seqs * a.H)), dim3(256 * NW), 0, st, a);
     GLM_CHECK_LAUNCH("glm_memory_recurrent");
     return GLM_OK;
 }
@@ -825,17 +943,18 @@ int run_rec(const RecArgs& a, hipStream_t st) {
     }
     const size_t lds = (size_t)(2 * a.dimp + a.vdimp) * 4;
     GLM_CHECK_ARG(lds <= 48 * 1024, GLM_ERR_UNSUPPORTED, "glm_memory_recurrent: head sizes %d + %d", a.dimp, a.vdimp);
-    hipLaunchKernelGGL(memory_recurrent_any_kernel<T>, dim3((unsigned)(a.seqs * a.H)), dim3(256), lds, st, a);
+    if (a.decay) hipLaunchKernelGGL((memory_recurrent_any_kernel<T, false>), dim3((unsigned)(a.seqs * a.H)), dim3(256), lds, st, a);
+    else hipLaunchKernelGGL((memory_recurrent_any_kernel<T, true>), dim3((unsigned)(a.seqs * a.H)), dim3(256), lds, st, a);
     GLM_CHECK_LAUNCH("glm_memory_recurrent");
     return GLM_OK;
 }
 
-template <int D>
+template <int D, bool GATED>
 int launch_chunk(const ChunkArgs& a, int seqs, hipStream_t st) {
     constexpr int QT = 64 * D * 2, STAGE = 2 * QT + 8192 + 1024;
     constexpr int LDS = (D <= 128 ? 3 : 2) * STAGE + (QT >= 16384 ? 0 : 16384) + (QT >= 32768 ? 0 : 16384) + 7 * 256 + D * 4;
     static_assert(LDS <= 160 * 1024, "LDS of a CU");
-    auto kern = memory_chunkwise_kernel<D>;
+    auto kern = memory_chunkwise_kernel<D, GATED>;
     GLM_SET_MAX_LDS(kern, LDS, "glm_memory_chunkwise");
     hipLaunchKernelGGL(kern, dim3((unsigned)(seqs * a.H * a.vtiles)), dim3(512), LDS, st, a);
     GLM_CHECK_LAUNCH("glm_memory_chunkwise");
@@ -855,7 +974,7 @@ extern "C" int glm_memory_recurrent(const void* x, int64_t ldx, int64_t k_off, i
                       glm_aligned16(x) && glm_aligned16(hrow) && glm_aligned16(wif) && glm_aligned16(S), GLM_ERR_INVALID,
                   "glm_memory_recurrent: bad shape H=%d dim=%d vdim=%d ldx=%ld", H, dim, vdim, (long)ldx);
     if (seqs == 0) return GLM_OK;
-    RecArgs a = {x, ldx, k_off, v_off, g_off, hrow, ldh, wif, ldw, wk, bif, norm, y, ldy, S, n, m, n_state, pos, q_start, state_in, state_out, seqs, H, dim, dimp, vdim, vdimp, cap, eps};
+    RecArgs a = {x, ldx, k_off, v_off, g_off, hrow, ldh, wif, ldw, wk, bif, norm, y, ldy, S, n, m, n_state, pos, q_start, state_in, state_out, seqs, H, dim, dimp, vdim, vdimp, cap, eps, nullptr};
     return f32 ? run_rec<float>(a, glm_s(stream)) : run_rec<bf16_t>(a, glm_s(stream));
 }
 
@@ -880,12 +999,12 @@ extern "C" int glm_memory_chunkwise(const void* x, int64_t ldx, int64_t k_off, i
                       glm_aligned16(x) && (((uintptr_t)o) & 7) == 0, GLM_ERR_INVALID, "glm_memory_chunkwise: bad shape H=%d dim=%d vdimp=%d ldx=%ld", H, dim, vdimp, (long)ldx);
     GLM_CHECK_ARG(dimp <= 256, GLM_ERR_UNSUPPORTED, "glm_memory_chunkwise: key size %d", dimp);
     if (seqs == 0) return GLM_OK;
-    ChunkArgs a = {(const bf16_t*)x, ldx, k_off, v_off, gates, rows, (bf16_t*)o, ldo, S, n, m, n_state, pos, q_start, state_in, state_out, H, dim, dimp, vdimp, (vdimp + 63) / 64};
+    ChunkArgs a = {(const bf16_t*)x, ldx, k_off, v_off, gates, rows, (bf16_t*)o, ldo, S, n, m, n_state, pos, q_start, state_in, state_out, H, dim, dimp, vdimp, (vdimp + 63) / 64, nullptr};
     GLM_CHECK_ARG((int64_t)seqs * H * a.vtiles < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_memory_chunkwise: grid too large");
     hipStream_t st = glm_s(stream);
-    if (dimp <= 64) return launch_chunk<64>(a, seqs, st);
-    if (dimp <= 128) return launch_chunk<128>(a, seqs, st);
-    return launch_chunk<256>(a, seqs, st);
+    if (dimp <= 64) return launch_chunk<64, true>(a, seqs, st);
+    if (dimp <= 128) return launch_chunk<128, true>(a, seqs, st);
+    return launch_chunk<256, true>(a, seqs, st);
 }
 
 extern "C" int glm_memory_output(const void* o, int64_t ldo, const void* g, int64_t ldg, const float* norm, void* y, int64_t ldy, int64_t T, int H, int vdim, int vdimp, float eps,
@@ -904,3 +1023,47 @@ extern "C" int glm_memory_output(const void* o, int64_t ldo, const void* g, int6
     return GLM_OK;
 }
 
+extern "C" int glm_linear_recurrent(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* decay, float* o, int64_t ldo, float* S, int64_t n_state, const int32_t* pos,
+                                    const int32_t* q_start, const int32_t* state_in, const int32_t* state_out, int seqs, int H, int dimp, int vdimp, int f32, glm_stream_t stream) {
+    GLM_CHECK_ARG(x && decay && o && S && pos && q_start && state_in && state_out, GLM_ERR_INVALID, "glm_linear_recurrent: null pointer");
+    GLM_CHECK_ARG(seqs >= 0 && H > 0 && dimp > 0 && dimp % 8 == 0 && vdimp > 0 && vdimp % 8 == 0 && n_state > 0 && k_off >= (int64_t)H * dimp && ldx >= k_off + (int64_t)H * dimp &&
+                      ldx >= v_off + (int64_t)H * vdimp && ldo >= (int64_t)H * vdimp && ldx % 8 == 0 && k_off % 8 == 0 && v_off % 8 == 0 && (int64_t)seqs * H < (1ll << 31) &&
+                      glm_aligned16(x) && glm_aligned16(S), GLM_ERR_INVALID, "glm_linear_recurrent: bad shape H=%d dimp=%d vdimp=%d ldx=%ld", H, dimp, vdimp, (long)ldx);
+    if (seqs == 0) return GLM_OK;
+    RecArgs a = {};
+    a.x = x; a.ldx = ldx; a.k_off = k_off; a.v_off = v_off; a.y = o; a.ldy = ldo; a.S = S; a.n_state = n_state; a.pos = pos; a.q_start = q_start; a.state_in = state_in;
+    a.state_out = state_out; a.seqs = seqs; a.H = H; a.dim = a.dimp = dimp; a.vdim = a.vdimp = vdimp; a.decay = decay;
+    return f32 ? run_rec<float>(a, glm_s(stream)) : run_rec<bf16_t>(a, glm_s(stream));
+}
+
+extern "C" int glm_linear_chunkwise(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* powers, void* o, int64_t ldo, float* S, int64_t n_state, const int32_t* pos,
+                                    const int32_t* q_start, const int32_t* state_in, const int32_t* state_out, int seqs, int H, int dimp, int vdimp, glm_stream_t stream) {
+    GLM_CHECK_ARG(x && powers && o && S && pos && q_start && state_in && state_out, GLM_ERR_INVALID, "glm_linear_chunkwise: null pointer");
+    GLM_CHECK_ARG(seqs >= 0 && H > 0 && dimp > 0 && dimp % 8 == 0 && vdimp > 0 && vdimp % 8 == 0 && n_state > 0 && k_off >= (int64_t)H * dimp && ldx >= k_off + (int64_t)H * dimp &&
+                      ldx >= v_off + (int64_t)H * vdimp && ldo >= (int64_t)H * vdimp && ldx % 8 == 0 && k_off % 8 == 0 && v_off % 8 == 0 && ldo % 4 == 0 && ldx < (1 << 24) &&
+                      glm_aligned16(x) && (((uintptr_t)o) & 7) == 0, GLM_ERR_INVALID, "glm_linear_chunkwise: bad shape H=%d dimp=%d vdimp=%d ldx=%ld", H, dimp, vdimp, (long)ldx);
+    GLM_CHECK_ARG(dimp <= 256, GLM_ERR_UNSUPPORTED, "glm_linear_chunkwise: key size %d", dimp);
+    if (seqs == 0) return GLM_OK;
+    ChunkArgs a = {(const bf16_t*)x, ldx, k_off, v_off, nullptr, 0, (bf16_t*)o, ldo, S, nullptr, nullptr, n_state, pos, q_start, state_in, state_out, H, dimp, dimp, vdimp, (vdimp + 63) / 64, powers};
+    GLM_CHECK_ARG((int64_t)seqs * H * a.vtiles < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_linear_chunkwise: grid too large");
+    hipStream_t st = glm_s(stream);
+    if (dimp <= 64) return launch_chunk<64, false>(a, seqs, st);
+    if (dimp <= 128) return launch_chunk<128, false>(a, seqs, st);
+    return launch_chunk<256, false>(a, seqs, st);
+}
+
+extern "C" int glm_row_norm_gate(const void* o, int64_t ldo, int o_f32, const void* gate, int64_t ldg, const float* norm, void* y, int64_t ldy, int64_t T, int n, int np, float eps,
+                                 int act_f32, glm_stream_t stream) {
+    GLM_CHECK_ARG(o && gate && norm && y && T >= 0 && n > 0 && np >= n && np % 8 == 0 && ldo >= np && ldg >= np && ldy >= np && ldo % 8 == 0 && ldg % 8 == 0 && ldy % 8 == 0 &&
+                      glm_aligned16(o) && glm_aligned16(gate) && glm_aligned16(norm) && glm_aligned16(y) && (o_f32 || !act_f32), GLM_ERR_INVALID,
+                  "glm_row_norm_gate: bad shape T=%ld n=%d np=%d", (long)T, n, np);
+    GLM_CHECK_ARG((T + 3) / 4 < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_row_norm_gate: too many rows");
+    if (T == 0) return GLM_OK;
+    const dim3 grid((unsigned)((T + 3) / 4));
+    hipStream_t st = glm_s(stream);
+    if (act_f32) hipLaunchKernelGGL((row_norm_gate_kernel<float, float>), grid, dim3(256), 0, st, (const float*)o, ldo, (const float*)gate, ldg, norm, (float*)y, ldy, T, n, np, eps);
+    else if (o_f32) hipLaunchKernelGGL((row_norm_gate_kernel<float, bf16_t>), grid, dim3(256), 0, st, (const float*)o, ldo, (const bf16_t*)gate, ldg, norm, (bf16_t*)y, ldy, T, n, np, eps);
+    else hipLaunchKernelGGL((row_norm_gate_kernel<bf16_t, bf16_t>), grid, dim3(256), 0, st, (const bf16_t*)o, ldo, (const bf16_t*)gate, ldg, norm, (bf16_t*)y, ldy, T, n, np, eps);
+    GLM_CHECK_LAUNCH("glm_row_norm_gate");
+    return GLM_OK;
+}

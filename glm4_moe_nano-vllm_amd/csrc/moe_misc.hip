@@ -46,7 +46,7 @@ __device__ __forceinline__ void moe_align_body(const int64_t* topk_idx, const bf
             if (SC1) {
                 const unsigned pr = ld_sc1_u32(topk_w + (p & ~(int64_t)1));
                 w_first = (bf16_t)((p & 1) ? (pr >> 16) : (pr & 0xffffu));
-            } else {
+            } else if (topk_w) {
                 w_first = topk_w[p];
             }
         }
@@ -85,9 +85,9 @@ __device__ __forceinline__ void moe_align_body(const int64_t* topk_idx, const bf
                 const unsigned pr = ld_sc1_u32(topk_w + (p & ~(int64_t)1));
                 wv = (bf16_t)((p & 1) ? (pr >> 16) : (pr & 0xffffu));
             } else {
-                wv = topk_w[p];
+                wv = topk_w ? topk_w[p] : (bf16_t)0;
             }
-            sorted_scale[pos] = wv;
+            if (sorted_scale) sorted_scale[pos] = wv;
             pair_pos[p] = pos;
         } else {
             pair_pos[p] = -1;
@@ -620,7 +620,7 @@ __global__ __launch_bounds__(1024) void moe_align_scatter_kernel(
             if (e >= 0 && e < E) {
                 const int pos = atomicAdd(&cur[(int)e], 1);
                 sorted_token[pos] = (int32_t)(p / k);
-                sorted_scale[pos] = topk_w[p];
+                if (sorted_scale) sorted_scale[pos] = topk_w[p];
                 pair_pos[p] = pos;
             } else {
                 pair_pos[p] = -1;
@@ -634,6 +634,87 @@ __global__ __launch_bounds__(1024) void moe_align_scatter_kernel(
             sorted_token[sbase + t] = (int32_t)t;
             sorted_scale[sbase + t] = 0x3F80;  // bf16 1.0
         }
+    }
+}
+
+// ------------------------------------------------------------------------------------------
+// Softmax router: from fp32 logits the k largest scores of softmax over all E experts, not renormalised, in fp32; one wave per token,
+// 64 EPL >= E.  Order: descending, ties to the lower index.
+template <int EPL>
+__device__ __forceinline__ void softmax_select_wave(const float* __restrict__ lg, int E, int k, int lane, int64_t* idx, float* w) {
+    float v[EPL], m = -INFINITY, z = 0.f;
+#pragma unroll
+    for (int i = 0; i < EPL; ++i) {
+        v[i] = lane + 64 * i < E ? lg[lane + 64 * i] : -INFINITY;
+        m = fmaxf(m, v[i]);
+    }
+    m = wave_max(m);
+#pragma unroll
+    for (int i = 0; i < EPL; ++i) z += lane + 64 * i < E ? expf(v[i] - m) : 0.f;
+    const float inv = 1.0f / wave_sum(z);
+    for (int j = 0; j < k; ++j) {
+        float b = -INFINITY;
+        int e = 1 << 30;
+#pragma unroll
+        for (int i = 0; i < EPL; ++i)
+            if (v[i] > b) {
+                b = v[i];
+                e = lane + 64 * i;
+            }
+#pragma unroll
+        for (int o = 32; o > 0; o >>= 1) {
+            const float ob = __shfl_xor(b, o, 64);
+            const int oe = __shfl_xor(e, o, 64);
+            if (ob > b || (ob == b && oe < e)) {
+                b = ob;
+                e = oe;
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < EPL; ++i)
+            if (lane + 64 * i == e) v[i] = -INFINITY;
+        if (lane == 0) {  // (no number among the logits: no expert, which the bucketing leaves out)
+            idx[j] = e < E ? e : -1;
+            w[j] = e < E ? expf(b - m) * inv : 0.f;
+        }
+    }
+}
+
+template <int EPL>
+__global__ __launch_bounds__(256) void router_softmax_kernel(const float* __restrict__ logits, int64_t ld, int64_t* __restrict__ topk_idx,
+                                                             float* __restrict__ topk_w, int64_t T, int E, int k) {
+    const int64_t t = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    if (t < T) softmax_select_wave<EPL>(logits + t * ld, E, k, threadIdx.x & 63, topk_idx + t * k, topk_w + t * k);
+}
+
+// ... and the bucketing, for the few tokens of a decode step, by one workgroup
+template <int EPL>
+__global__ __launch_bounds__(1024) void router_softmax_align_kernel(const float* logits, int64_t ld, int64_t* topk_idx, float* topk_w, int32_t* expert_offsets,
+                                                                    int32_t* sorted_token, int32_t* pair_pos, int64_t T, int E, int k) {
+    __shared__ int cnt[ALIGN_MAX_G + 1];
+    __shared__ int cur[ALIGN_MAX_G + 1];
+    for (int64_t t = threadIdx.x >> 6; t < T; t += 16) softmax_select_wave<EPL>(logits + t * ld, E, k, threadIdx.x & 63, topk_idx + t * k, topk_w + t * k);
+    __syncthreads();
+    moe_align_body<false>(topk_idx, nullptr, expert_offsets, sorted_token, nullptr, pair_pos, T, k, E, 0, cnt, cur);
+}
+
+// out[t] = sum_j w[t, j] y[pair_pos[t, j]], fp32 sum
+template <typename E>
+__global__ __launch_bounds__(256) void moe_combine_weighted_kernel(const E* __restrict__ y, int64_t ldy, int64_t R, const int32_t* __restrict__ pair_pos,
+                                                                   const float* __restrict__ w, E* __restrict__ out, int64_t ldo, int k, int H) {
+    const int64_t t = blockIdx.x;
+    for (int c = threadIdx.x; c < H; c += 256) {
+        float s = 0.f;
+        for (int j = 0; j < k; ++j) {
+            const int p = pair_pos[t * k + j];
+            if (p < 0 || p >= R) continue;
+            float v;
+            if constexpr (sizeof(E) == 4) v = y[(int64_t)p * ldy + c];
+            else v = bf2f(y[(int64_t)p * ldy + c]);
+            s = fmaf(w[t * k + j], v, s);
+        }
+        if constexpr (sizeof(E) == 4) out[t * ldo + c] = s;
+        else out[t * ldo + c] = f2bf(s);
     }
 }
 
@@ -910,7 +991,7 @@ static int add_rmsnorm_router_impl(const void* x, const float* part, int nslices
 extern "C" int glm_moe_align(const int64_t* topk_idx, const void* topk_w, int32_t* expert_offsets,
                              int32_t* sorted_token, void* sorted_scale, int32_t* pair_pos,
                              int64_t T, int k, int E, int with_shared, glm_stream_t stream) {
-    GLM_CHECK_ARG(topk_idx && topk_w && expert_offsets && sorted_token && sorted_scale && pair_pos,
+    GLM_CHECK_ARG(topk_idx && expert_offsets && sorted_token && pair_pos && (!topk_w) == (!sorted_scale) && (sorted_scale || !with_shared),
                   GLM_ERR_INVALID, "glm_moe_align: null pointer");
     GLM_CHECK_ARG(T >= 0 && k > 0 && E > 0, GLM_ERR_INVALID, "glm_moe_align: bad shape");
     GLM_CHECK_ARG(E < ALIGN_MAX_G && T * (int64_t)(k + 1) < (1ll << 31), GLM_ERR_UNSUPPORTED,
@@ -934,7 +1015,7 @@ extern "C" int glm_moe_align_parallel(const int64_t* topk_idx, const void* topk_
                                       int32_t* sorted_token, void* sorted_scale, int32_t* pair_pos, int64_t T, int k,
                                       int E, int with_shared, int32_t* workspace, size_t workspace_bytes,
                                       glm_stream_t stream) {
-    GLM_CHECK_ARG(topk_idx && topk_w && expert_offsets && sorted_token && sorted_scale && pair_pos && workspace,
+    GLM_CHECK_ARG(topk_idx && expert_offsets && sorted_token && pair_pos && workspace && (!topk_w) == (!sorted_scale) && (sorted_scale || !with_shared),
                   GLM_ERR_INVALID, "glm_moe_align_parallel: null pointer");
     GLM_CHECK_ARG(T >= 0 && k > 0 && E > 0, GLM_ERR_INVALID, "glm_moe_align_parallel: bad shape");
     GLM_CHECK_ARG(E < ALIGN_MAX_G && T * (int64_t)(k + 1) < (1ll << 31), GLM_ERR_UNSUPPORTED,
@@ -953,6 +1034,42 @@ extern "C" int glm_moe_align_parallel(const int64_t* topk_idx, const void* topk_
         hipLaunchKernelGGL(moe_align_scatter_kernel, dim3(chunks), dim3(1024), 0, st, topk_idx, (const bf16_t*)topk_w,
                            expert_offsets, base, sorted_token, (bf16_t*)sorted_scale, pair_pos, T, k, E, with_shared);
     GLM_CHECK_LAUNCH("glm_moe_align_parallel");
+    return GLM_OK;
+}
+
+extern "C" int glm_router_softmax(const float* logits, int64_t ld, int64_t* topk_idx, float* topk_w, int64_t T, int E, int k, glm_stream_t stream) {
+    GLM_CHECK_ARG(logits && topk_idx && topk_w && T >= 0 && E > 0 && k > 0 && k <= E && ld >= E, GLM_ERR_INVALID, "glm_router_softmax: bad shape T=%ld E=%d k=%d", (long)T, E, k);
+    GLM_CHECK_ARG(E < ALIGN_MAX_G && T < (1ll << 32), GLM_ERR_UNSUPPORTED, "glm_router_softmax: %d experts", E);
+    if (T == 0) return GLM_OK;
+    const dim3 grid((unsigned)((T + 3) / 4));
+    hipStream_t st = glm_s(stream);
+    if (E <= 64) hipLaunchKernelGGL(router_softmax_kernel<1>, grid, dim3(256), 0, st, logits, ld, topk_idx, topk_w, T, E, k);
+    else if (E <= 256) hipLaunchKernelGGL(router_softmax_kernel<4>, grid, dim3(256), 0, st, logits, ld, topk_idx, topk_w, T, E, k);
+    else hipLaunchKernelGGL(router_softmax_kernel<16>, grid, dim3(256), 0, st, logits, ld, topk_idx, topk_w, T, E, k);
+    GLM_CHECK_LAUNCH("glm_router_softmax");
+    return GLM_OK;
+}
+
+extern "C" int glm_router_softmax_align(const float* logits, int64_t ld, int64_t* topk_idx, float* topk_w, int32_t* expert_offsets, int32_t* sorted_token,
+                                        int32_t* pair_pos, int64_t T, int E, int k, glm_stream_t stream) {
+    GLM_CHECK_ARG(logits && topk_idx && topk_w && expert_offsets && sorted_token && pair_pos && T >= 0 && E > 0 && k > 0 && k <= E && ld >= E, GLM_ERR_INVALID,
+                  "glm_router_softmax_align: bad shape T=%ld E=%d k=%d", (long)T, E, k);
+    GLM_CHECK_ARG(E < ALIGN_MAX_G && T * (int64_t)k < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_router_softmax_align: %d experts", E);
+    hipStream_t st = glm_s(stream);
+    if (E <= 64) hipLaunchKernelGGL(router_softmax_align_kernel<1>, dim3(1), dim3(1024), 0, st, logits, ld, topk_idx, topk_w, expert_offsets, sorted_token, pair_pos, T, E, k);
+    else if (E <= 256) hipLaunchKernelGGL(router_softmax_align_kernel<4>, dim3(1), dim3(1024), 0, st, logits, ld, topk_idx, topk_w, expert_offsets, sorted_token, pair_pos, T, E, k);
+    else hipLaunchKernelGGL(router_softmax_align_kernel<16>, dim3(1), dim3(1024), 0, st, logits, ld, topk_idx, topk_w, expert_offsets, sorted_token, pair_pos, T, E, k);
+    GLM_CHECK_LAUNCH("glm_router_softmax_align");
+    return GLM_OK;
+}
+
+extern "C" int glm_moe_combine_weighted(const void* y, int64_t ldy, int64_t R, const int32_t* pair_pos, const float* w, void* out, int64_t ldo, int64_t T, int k, int H, int f32,
+                                        glm_stream_t stream) {
+    GLM_CHECK_ARG(y && pair_pos && w && out && T >= 0 && T < (1ll << 31) && k > 0 && H > 0 && ldy >= H && ldo >= H, GLM_ERR_INVALID, "glm_moe_combine_weighted: bad shape T=%ld H=%d", (long)T, H);
+    if (T == 0) return GLM_OK;
+    if (f32) hipLaunchKernelGGL(moe_combine_weighted_kernel<float>, dim3((unsigned)T), dim3(256), 0, glm_s(stream), (const float*)y, ldy, R, pair_pos, w, (float*)out, ldo, k, H);
+    else hipLaunchKernelGGL(moe_combine_weighted_kernel<bf16_t>, dim3((unsigned)T), dim3(256), 0, glm_s(stream), (const bf16_t*)y, ldy, R, pair_pos, w, (bf16_t*)out, ldo, k, H);
+    GLM_CHECK_LAUNCH("glm_moe_combine_weighted");
     return GLM_OK;
 }
 

@@ -424,11 +424,11 @@ int launch_seq_norm(const SeqNormArgs& a, hipStream_t st) {
     return GLM_OK;
 }
 
-// one workgroup per token row: fp32 residual row and (optionally) the row in the activation dtype.  freq: a sinusoidal position
+// one workgroup per token row: fp32 residual row (the table's row times `scale`) and (optionally) the row in the activation dtype.  freq: a sinusoidal position
 // vector is added, sin(p f_i) at the even columns 2i and cos(p f_i) at the odd ones; the angle is taken in double and brought into
 // one turn before it is rounded, so far positions are as exact as near ones.
 __global__ __launch_bounds__(SN_NT) void embed_rows_kernel(const int64_t* ids, const void* table, int64_t ldw, int64_t vocab, const int32_t* pos,
-                                                           const double* freq, float* x, int64_t ldx, void* cast, int64_t ldc, int act_f32, int width, int wp, int vec) {
+                                                           const double* freq, float* x, int64_t ldx, void* cast, int64_t ldc, int act_f32, int width, int wp, int vec, float scale) {
     const int64_t t = blockIdx.x;
     const int64_t id = ids[t];
     const bool ok = id >= 0 && id < vocab;  // (an id outside the table gives a row of zeros)
@@ -446,6 +446,8 @@ __global__ __launch_bounds__(SN_NT) void embed_rows_kernel(const int64_t* ids, c
                     if (c + i < width) v[i] = act_f32 ? reinterpret_cast<const float*>(table)[id * ldw + c + i] : bf2f(reinterpret_cast<const bf16_t*>(table)[id * ldw + c + i]);
             }
         }
+#pragma unroll
+        for (int i = 0; i < 4; ++i) v[i] *= scale;
         if (freq) {
             const double p = (double)max(pos[t], 0);
 #pragma unroll
@@ -502,12 +504,13 @@ extern "C" int glm_seq_norm(const float* x_in, const int32_t* row_index, int64_t
 }
 
 extern "C" int glm_embed_rows(const int64_t* ids, const void* table, int64_t ldw, int64_t vocab, const int32_t* pos, const double* freq,
-                              float* x, int64_t ldx, void* cast, int64_t ldc, int act_f32, int64_t T, int width, int wp, glm_stream_t stream) {
+                              float* x, int64_t ldx, void* cast, int64_t ldc, int act_f32, int64_t T, int width, int wp, float scale,
+                              glm_stream_t stream) {
     GLM_CHECK_ARG(ids && table && x && T >= 0 && width > 0 && wp >= width && wp % 8 == 0 && ldw >= width && ldx >= wp && ldx % 4 == 0 &&
                       (!cast || (ldc >= wp && ldc % 4 == 0)) && (!freq || pos), GLM_ERR_INVALID, "glm_embed_rows: bad shape T=%ld width=%d wp=%d", (long)T, width, wp);
     if (T == 0) return GLM_OK;
     const int vec = width == wp && ldw % 8 == 0 && glm_aligned16(table);
-    hipLaunchKernelGGL(embed_rows_kernel, dim3((unsigned)T), dim3(SN_NT), 0, glm_s(stream), ids, table, ldw, vocab, pos, freq, x, ldx, cast, ldc, act_f32, width, wp, vec);
+    hipLaunchKernelGGL(embed_rows_kernel, dim3((unsigned)T), dim3(SN_NT), 0, glm_s(stream), ids, table, ldw, vocab, pos, freq, x, ldx, cast, ldc, act_f32, width, wp, vec, scale);
     GLM_CHECK_LAUNCH("glm_embed_rows");
     return GLM_OK;
 }

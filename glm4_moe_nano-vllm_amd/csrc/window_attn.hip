@@ -19,15 +19,20 @@ __device__ const u32x4_t wa_zero_page[4] = {};
 struct WinArgs {
     const bf16_t* q;   // [rows, ldq], head h at h*dk
     int64_t ldq;
-    const bf16_t *k, *v;  // [Tk, ldkv], head h at h*dk / h*dv
+    const bf16_t *k, *v;  // [Tk, ldkv], head h at h*dkn / h*dv
     int64_t ldkv;
+    const bf16_t* kr;  // [Tk, ldr] the last dk - dkn key columns, shared by all heads
+    int64_t ldr;
+    const float* cs;   // [rows, (dk - dkn) / 2, 2] rotation of those query columns, pairs (2i, 2i+1)
+    const bf16_t* gate;  // [rows, ldg] factors of the output, laid out like out, or nullptr
+    int64_t ldg;
     bf16_t* out;       // [rows, ldo], head h at h*dv
     int64_t ldo;
     const int32_t *q_start;  // [S+1] first q / out row of every sequence's portion
     const int32_t *k_start;  // [S+1] first k / v row
     const int32_t *tile_seq, *tile_off;  // [n_tiles]
     const float* sink;
-    int S, n_tiles, H, dk, dv, window;
+    int S, n_tiles, H, dk, dkn, dv, window;
     int64_t Tq, Tk;
     float scale;
 };
@@ -70,6 +75,14 @@ __global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void window_attn_ker
             const int k = 32 * i + 8 * g;
             qf[t][i] = u32x4_t{0, 0, 0, 0};
             if (k < a.dk) qf[t][i] = *reinterpret_cast<const u32x4_t*>(qp + k);
+            if (k >= a.dkn && k < a.dk) {  // rotated here: a lane holds whole pairs
+                const float* cs = a.cs + (int64_t)(qs + min(r, nq - 1)) * (a.dk - a.dkn) + (k - a.dkn);
+#pragma unroll
+                for (int j = 0; j < 4; ++j) {
+                    const float u = bflo(qf[t][i][j]), v = bfhi(qf[t][i][j]), co = cs[2 * j], si = cs[2 * j + 1];
+                    qf[t][i][j] = pack2bf(u * co - v * si, v * co + u * si);
+                }
+            }
         }
     }
 #pragma unroll
@@ -77,19 +90,21 @@ __global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void window_attn_ker
 #pragma unroll
         for (int i = 0; i < KS; ++i) asm volatile("" : "+v"(qf[t][i]));
     const unsigned base = lds_addr(smem);
-    const bf16_t* kbase = a.k + (int64_t)(ks0 + jlo) * a.ldkv + (int64_t)h * a.dk;
+    const bf16_t* kbase = a.k + (int64_t)(ks0 + jlo) * a.ldkv + (int64_t)h * a.dkn;
+    const bf16_t* rbase = a.kr ? a.kr + (int64_t)(ks0 + jlo) * a.ldr : kbase;
     const bf16_t* vbase = a.v + (int64_t)(ks0 + jlo) * a.ldkv + (int64_t)h * a.dv;
     const int nkeys = jhi - jlo + 1;
     // per-lane source offsets of the DMA pieces: constant over the tiles
     unsigned koff[KDMA], voff[VDMA];
     int krow[KDMA], vrow_[VDMA];
-    bool kpad[KDMA], vpad[VDMA];
+    bool kpad[KDMA], krot[KDMA], vpad[VDMA];
 #pragma unroll
     for (int i = 0; i < KDMA; ++i) {
         const int q = (w * KDMA + i) * 64 + lane, row = q / KCPR, ch = (q % KCPR) ^ attn_swz(row);
         krow[i] = row;
         kpad[i] = ch * 8 >= a.dk;
-        koff[i] = (unsigned)(row * (int)a.ldkv + ch * 8);
+        krot[i] = ch * 8 >= a.dkn;
+        koff[i] = (unsigned)(krot[i] ? row * (int)a.ldr + ch * 8 - a.dkn : row * (int)a.ldkv + ch * 8);
     }
 #pragma unroll
     for (int i = 0; i < VDMA; ++i) {
@@ -99,12 +114,12 @@ __global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void window_attn_ker
         voff[i] = (unsigned)(row * (int)a.ldkv + ch * 8);
     }
     auto issue = [&](int it) {
-        const int64_t adv = (int64_t)it * 64 * a.ldkv;
+        const int64_t adv = (int64_t)it * 64 * a.ldkv, advr = (int64_t)it * 64 * a.ldr;
         const int left = nkeys - it * 64;
         char* st = smem + (it & 1) * STAGE;
 #pragma unroll
         for (int i = 0; i < KDMA; ++i) {
-            const void* s = (kpad[i] || krow[i] >= left) ? (const void*)wa_zero_page : (const void*)(kbase + adv + koff[i]);
+            const void* s = (kpad[i] || krow[i] >= left) ? (const void*)wa_zero_page : (const void*)((krot[i] ? rbase + advr : kbase + adv) + koff[i]);
             lds_dma16(s, st + (w * KDMA + i) * 1024);
         }
 #pragma unroll
@@ -267,6 +282,10 @@ __global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void window_attn_ker
 #pragma unroll
         for (int d = 0; d < VT; ++d) {
             const int dim = 16 * d + 4 * g;
+            if (a.gate && dim < a.dv) {
+                const u32x2_t gt = *reinterpret_cast<const u32x2_t*>(a.gate + (int64_t)(qs + r) * a.ldg + (int64_t)h * a.dv + dim);
+                acc[t][d] *= f32x4_t{bflo(gt[0]), bfhi(gt[0]), bflo(gt[1]), bfhi(gt[1])};
+            }
             if (dim < a.dv) *reinterpret_cast<u32x2_t*>(o + dim) = u32x2_t{pack2bf(acc[t][d][0] * inv, acc[t][d][1] * inv), pack2bf(acc[t][d][2] * inv, acc[t][d][3] * inv)};
         }
     }
@@ -295,18 +314,21 @@ int launch_window_dv(const WinArgs& a, hipStream_t st) {
 
 }  // namespace
 
-extern "C" int glm_window_attn_prefill(const void* q, int64_t ldq, const void* k, const void* v, int64_t ldkv, void* out, int64_t ldo,
+extern "C" int glm_window_attn_prefill(const void* q, int64_t ldq, const void* k, const void* v, int64_t ldkv, const void* kr, int64_t ldr, int rotp, const float* cs,
+                                       const void* gate, int64_t ldg, void* out, int64_t ldo,
                                        const int32_t* q_start, const int32_t* k_start, const int32_t* tile_seq, const int32_t* tile_off, int n_tiles, int S,
                                        int64_t Tq, int64_t Tk, int H, int dk, int dv, int window, float scale, const float* sink, glm_stream_t stream) {
     GLM_CHECK_ARG(q && k && v && out && q_start && k_start && tile_seq && tile_off && sink, GLM_ERR_INVALID, "glm_window_attn_prefill: null pointer");
-    GLM_CHECK_ARG(H > 0 && dk > 0 && dv > 0 && dk % 8 == 0 && dv % 8 == 0 && ldq >= (int64_t)H * dk && ldkv >= (int64_t)H * (dk > dv ? dk : dv) && ldo >= (int64_t)H * dv &&
+    GLM_CHECK_ARG(H > 0 && dk > 0 && dv > 0 && dk % 8 == 0 && dv % 8 == 0 && ldq >= (int64_t)H * dk && ldkv >= (int64_t)H * (dk - rotp > dv ? dk - rotp : dv) && ldo >= (int64_t)H * dv &&
                       ldq % 8 == 0 && ldkv % 8 == 0 && ldo % 4 == 0 && window > 0 && S > 0 && n_tiles >= 0 && Tq >= 0 && Tk >= Tq && ldkv < (1 << 24) &&
                       glm_aligned16(q) && glm_aligned16(k) && glm_aligned16(v), GLM_ERR_INVALID,
                   "glm_window_attn_prefill: bad shape H=%d dk=%d dv=%d ldq=%ld ldkv=%ld window=%d", H, dk, dv, (long)ldq, (long)ldkv, window);
     GLM_CHECK_ARG(dk <= 256 && dv <= 256, GLM_ERR_UNSUPPORTED, "glm_window_attn_prefill: head sizes up to 256 (dk=%d dv=%d)", dk, dv);
+    GLM_CHECK_ARG(rotp >= 0 && rotp < dk && rotp % 8 == 0 && (rotp == 0 || (kr && cs && ldr >= rotp && ldr % 8 == 0 && ldr < (1 << 24) && glm_aligned16(kr))) &&
+                      (!gate || (ldg >= (int64_t)H * dv && ldg % 4 == 0)), GLM_ERR_INVALID, "glm_window_attn_prefill: bad rotated part of %d columns or gate", rotp);
     if (n_tiles == 0) return GLM_OK;
-    WinArgs a = {(const bf16_t*)q, ldq, (const bf16_t*)k, (const bf16_t*)v, ldkv, (bf16_t*)out, ldo, q_start, k_start, tile_seq, tile_off, sink,
-                 S, n_tiles, H, dk, dv, window, Tq, Tk, scale};
+    WinArgs a = {(const bf16_t*)q, ldq, (const bf16_t*)k, (const bf16_t*)v, ldkv, rotp ? (const bf16_t*)kr : nullptr, ldr, cs, (const bf16_t*)gate, ldg, (bf16_t*)out, ldo,
+                 q_start, k_start, tile_seq, tile_off, sink, S, n_tiles, H, dk, dk - rotp, dv, window, Tq, Tk, scale};
     hipStream_t st = glm_s(stream);
     if (dk <= 64) return launch_window_dv<64>(a, st);
     if (dk <= 128) return launch_window_dv<128>(a, st);

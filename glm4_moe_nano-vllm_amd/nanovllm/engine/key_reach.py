@@ -3,6 +3,8 @@ from __future__ import annotations
 
 from dataclasses import dataclass
 
+EVERYTHING = 1 << 30   # window of a layer that sees every earlier token
+
 
 @dataclass(frozen=True)
 class KeyReach:

@@ -145,20 +145,19 @@ _SIGNATURES = {
     "glm_seq_norm": (c_int, [c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_int, c_int,
         c_int64, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p,
         c_void_p, c_void_p, c_int64, c_int, c_int64, c_int, c_int, c_float, c_void_p]),
-    "glm_embed_rows": (c_int, [c_void_p, c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_int64,
-        c_int, c_int64, c_int, c_int, c_void_p]),
+    "glm_embed_rows": (c_int, [c_void_p, c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_int,
+        c_int64, c_int, c_int, c_float, c_void_p]),
     "glm_latent_prepare": (c_int, [c_void_p, c_int64, c_int, c_int64, c_int64, c_int, c_int, c_int, c_int, c_void_p,
         c_float, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int, c_void_p]),
     "glm_latent_gather": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_int, c_void_p]),
     "glm_latent_attn_max_rows": (c_int, [c_int]),
-    "glm_latent_attn": (c_int, [c_void_p, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p,
-        c_void_p, c_void_p, c_int64, c_int64, c_int, c_int, c_int, c_int, c_float, c_void_p, c_int, c_void_p, c_void_p,
-        c_void_p, c_int, c_void_p]),
+    "glm_latent_attn": (c_int, [c_void_p, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p,
+        c_int64, c_int64, c_int, c_int, c_int, c_int, c_float, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p]),
     "glm_attn_merge": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int64, c_int, c_int, c_void_p]),
-    "glm_latent_up": (c_int, [c_void_p, c_void_p, c_void_p, c_int64, c_int64, c_int, c_int, c_int, c_void_p]),
-    "glm_window_attn_prefill": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_void_p,
-        c_void_p, c_void_p, c_void_p, c_int, c_int, c_int64, c_int64, c_int, c_int, c_int, c_int, c_float, c_void_p,
-        c_void_p]),
+    "glm_latent_up": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_int64, c_int64, c_int64, c_int, c_int, c_int, c_void_p]),
+    "glm_window_attn_prefill": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_int, c_void_p, c_void_p,
+        c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int64, c_int64, c_int, c_int, c_int, c_int,
+        c_float, c_void_p, c_void_p]),
     "glm_gemm_bf16_glu": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int, c_int, c_float, c_float,
         c_void_p]),
     "glm_glu_f32": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int, c_float, c_float, c_void_p]),
@@ -187,6 +186,29 @@ _SIGNATURES = {
         c_void_p]),
     "glm_memory_output": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int, c_int, c_int,
         c_float, c_void_p]),
+    "glm_linear_recurrent": (c_int, [c_void_p, c_int64, c_int64, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_void_p,
+        c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p]),
+    "glm_linear_chunkwise": (c_int, [c_void_p, c_int64, c_int64, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_void_p,
+        c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p]),
+    "glm_row_norm_gate": (c_int, [c_void_p, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int, c_int,
+        c_float, c_int, c_void_p]),
+    "glm_depth_norm_taps": (c_int, [c_int]),
+    "glm_depth_norm": (c_int, [c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_int, c_int64, c_void_p, c_void_p,
+        c_void_p, c_int64, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int64, c_void_p,
+        c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int64, c_int, c_int, c_int, c_float, c_void_p]),
+    "glm_router_softmax": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_int, c_void_p]),
+    "glm_router_softmax_align": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int,
+        c_void_p]),
+    "glm_moe_combine_weighted": (c_int, [c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_int64, c_int, c_int, c_int,
+        c_void_p]),
+    "glm_grouped_gemm_f32": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_int64,
+        c_int, c_int, c_int, c_void_p]),
+    "glm_swiglu_f32": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int, c_void_p]),
+    "glm_mul_f32": (c_int, [c_void_p, c_int64, c_void_p, c_int64, c_int64, c_int, c_void_p]),
+    "glm_rope_pairs": (c_int, [c_void_p, c_void_p, c_int, c_float, c_void_p, c_int64, c_int, c_void_p]),
+    "glm_latent_rows": (c_int, [c_void_p, c_int64, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_float, c_void_p, c_void_p, c_int64,
+        c_void_p, c_void_p, c_int64, c_int, c_int, c_int, c_void_p, c_void_p, c_int64, c_int64, c_int, c_void_p]),
+    "glm_latent_absorb": (c_int, [c_void_p, c_int64, c_int64, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p]),
 }
 
 EXPORTED_SYMBOLS = tuple(_SIGNATURES)
@@ -730,14 +752,15 @@ def add_rmsnorm_router_topk(x, residual: torch.Tensor, norm_weight: torch.Tensor
 ALIGN_PARALLEL_MIN_PAIRS = 16384  # from here on the one-workgroup bucketing kernel is the slower one (200 us at 131072 pairs)
 
 
-def moe_align(topk_idx: torch.Tensor, topk_w: torch.Tensor, E: int, with_shared: bool):
+def moe_align(topk_idx: torch.Tensor, topk_w: torch.Tensor | None, E: int, with_shared: bool):
+    """topk_w None: no scales (the rows are weighed where they are summed up)."""
     T, k = topk_idx.shape
     G = E + (1 if with_shared else 0)
     R = T * k + (T if with_shared else 0)
     dev = topk_idx.device
     offs = torch.empty(G + 1, dtype=torch.int32, device=dev)
     tok = torch.empty(R, dtype=torch.int32, device=dev)
-    scale = torch.empty(R, dtype=torch.bfloat16, device=dev)
+    scale = torch.empty(R, dtype=torch.bfloat16, device=dev) if topk_w is not None else None
     pos = torch.empty(T * k, dtype=torch.int32, device=dev)
     if T * k >= ALIGN_PARALLEL_MIN_PAIRS:  # prefill sizes: count / offsets / scatter over many workgroups
         lib = load_library()
@@ -1241,6 +1264,7 @@ def gemm_bf16(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None
 # decoders with a 32-bit residual stream, latent attention and short convolutions over time (no counterpart in the
 # reference).  Activations are bf16 or fp32 (`act dtype`): every op below takes either and picks the kernel by dtype.
 ACT_NONE, ACT_XIELU, ACT_SOFTCAP = 0, 1, 2
+ACT_GATE, ACT_SILU_GATE = 4, 5     # columns below the constant pass / go through SiLU, the others through the sigmoid
 NO_ACT = (ACT_NONE, 0.0, 0.0)
 
 
@@ -1287,17 +1311,18 @@ def batched_gemm_f32(x: torch.Tensor, w: torch.Tensor, y: torch.Tensor) -> None:
 
 
 def embed_rows(ids: torch.Tensor, table: torch.Tensor, wp: int, cast: torch.Tensor | None = None, pos: torch.Tensor | None = None,
-               freq: torch.Tensor | None = None) -> torch.Tensor:
-    """fp32 residual rows [T, wp] of the token ids; `cast` ([T, >= wp], the table's dtype) receives a copy.  freq (fp64, one per
+               freq: torch.Tensor | None = None, scale: float = 1.0, out: torch.Tensor | None = None) -> torch.Tensor:
+    """fp32 residual rows [T, wp] (`out` or new) of the token ids, times scale; `cast` ([T, >= wp], the table's dtype) receives a copy.  freq (fp64, one per
     pair of columns): the sinusoidal vector of the positions `pos` is added."""
     T = ids.numel()
     assert ids.dtype == torch.int64 and table.stride(1) == 1
-    x = torch.empty((T, wp), dtype=torch.float32, device=table.device)
+    x = torch.empty((T, wp), dtype=torch.float32, device=table.device) if out is None else out
+    assert x.shape == (T, wp) and x.dtype == torch.float32 and x.is_contiguous()
     assert cast is None or (cast.shape[0] == T and cast.stride(1) == 1 and cast.dtype == table.dtype)
     assert freq is None or (freq.dtype == torch.float64 and freq.numel() >= (table.shape[1] + 1) // 2 and pos.dtype == torch.int32 and pos.numel() == T)
     _check(load_library().glm_embed_rows(_p(ids), _p(table), table.stride(0), table.shape[0], _p(pos) if freq is not None else None, _p(freq), _p(x), wp, _p(cast),
                                          cast.stride(0) if cast is not None else wp, _is_f32(table.dtype), T, table.shape[1], wp,
-                                         _stream()), "glm_embed_rows")
+                                         scale, _stream()), "glm_embed_rows")
     return x
 
 
@@ -1370,6 +1395,52 @@ def latent_prepare(qc: torch.Tensor, c_off: int, heads: int, dimp: int, rank: in
     return qa, c_out
 
 
+def mul_f32(y: torch.Tensor, g: torch.Tensor) -> None:
+    """y *= g, fp32 rows."""
+    assert y.shape == g.shape and y.dtype == g.dtype == torch.float32 and y.stride(1) == g.stride(1) == 1
+    _check(load_library().glm_mul_f32(_p(y), y.stride(0), _p(g), g.stride(0), y.shape[0], y.shape[1], _stream()), "glm_mul_f32")
+
+
+def rope_pairs(pos: torch.Tensor, freq: torch.Tensor, mscale: float, pairs: int) -> torch.Tensor:
+    """cos and sin [T, pairs, 2] of pos x freq (fp64) times mscale; pairs behind the last frequency do not turn."""
+    assert pos.dtype == torch.int32 and freq.dtype == torch.float64 and freq.numel() <= pairs
+    cs = torch.empty((pos.numel(), pairs, 2), dtype=torch.float32, device=pos.device)
+    _check(load_library().glm_rope_pairs(_p(pos), _p(freq), freq.numel(), mscale, _p(cs), pos.numel(), pairs, _stream()), "glm_rope_pairs")
+    return cs
+
+
+def latent_rows(x: torch.Tensor, c_off: int, rank: int, norm_w: torch.Tensor, cs: torch.Tensor | None, eps: float, slots: torch.Tensor, cache: torch.Tensor,
+                query: tuple | None = None, crow: torch.Tensor | None = None, n_crows: int = 0):
+    """In front of the query projection: rows x hold the raw latent (and the rotated key part behind it) at c_off; norm, rotation and cache
+    store; query = (column, rank, gain) of the queries' latent.  Returns (query latent [T, round8(rank)], c_out [n_crows, cache columns])."""
+    T, rc, rp = x.shape[0], cache.shape[-1], round8(rank)
+    assert x.stride(1) == 1 and cache.is_contiguous() and cache.dtype == x.dtype and slots.numel() == T and slots.dtype == torch.int32
+    assert norm_w.dtype == torch.float32 and norm_w.numel() == rp and (crow is None or (crow.dtype == torch.int32 and crow.numel() == T))
+    assert rc == rp or (cs.dtype == torch.float32 and cs.is_contiguous() and cs.numel() == T * (rc - rp))
+    c_out = torch.empty((n_crows, rc), dtype=x.dtype, device=x.device) if crow is not None else None
+    q_off, q_rank, q_gain = query or (0, 0, None)
+    assert q_gain is None or (q_gain.dtype == torch.float32 and q_gain.numel() == round8(q_rank))
+    cq = torch.empty((T, round8(q_rank)), dtype=x.dtype, device=x.device) if query else None
+    _check(load_library().glm_latent_rows(
+        _p(x), x.stride(0), c_off, rank, rp, rc - rp, _p(norm_w), _p(cs), eps, _p(slots), _p(cache), cache.numel() // rc, _p(crow), _p(c_out), n_crows, q_off, q_rank,
+        round8(q_rank), _p(q_gain), _p(cq), round8(q_rank), T, _is_f32(x.dtype), _stream()), "glm_latent_rows")
+    return cq, c_out
+
+
+def latent_absorb(q: torch.Tensor, heads: int, dimp: int, cs: torch.Tensor | None, wukt: torch.Tensor, rotp: int) -> torch.Tensor:
+    """W_uk^T q | rotated rest for every row and head of q ([Ta, heads * (dimp + rotp)])."""
+    Ta, rp = q.shape[0], wukt.shape[1]
+    assert q.shape[1] == heads * (dimp + rotp) and q.stride(1) == 1 and wukt.shape == (heads, rp, dimp) and wukt.is_contiguous()
+    assert rotp == 0 or (cs.dtype == torch.float32 and cs.is_contiguous() and cs.numel() >= Ta * rotp)
+    qa = torch.empty((Ta, heads, rp + rotp), dtype=q.dtype, device=q.device)
+    f32 = _is_f32(q.dtype)
+    _check(load_library().glm_latent_absorb(_p(q), q.stride(0), Ta, heads, dimp, rp, rotp, _p(cs), _p(wukt), _p(qa), f32, _stream()), "glm_latent_absorb")
+    if f32 and Ta:
+        qh = q.as_strided((Ta, heads, dimp), (q.stride(0), dimp + rotp, 1), q.storage_offset())
+        batched_gemm_f32(qh.transpose(0, 1), wukt, qa[..., :rp].transpose(0, 1))
+    return qa
+
+
 def latent_gather(cache: torch.Tensor, slots: torch.Tensor, rows: torch.Tensor, out: torch.Tensor) -> None:
     """out[rows[i]] = cache row slots[i]."""
     rp = cache.shape[-1]
@@ -1394,19 +1465,21 @@ def latent_tokens_per_tile(rp: int, heads: int) -> int:
 
 
 def latent_attn(qa: torch.Tensor, cache: torch.Tensor, tile_tok: torch.Tensor, tile_n: torch.Tensor, tokens_per_tile: int,
-                pos: torch.Tensor, seq_of: torch.Tensor, block_tables: torch.Tensor, rank: int, window: int, scale: float,
-                sink: torch.Tensor, wuv: torch.Tensor, out: torch.Tensor, num_splits: int = 0) -> None:
-    """Absorbed attention of the rows qa [Ta, H, rp] over the paged latents, then W_uv: writes out[:Ta] ([T, H * vdimp])."""
+                pos: torch.Tensor, seq_of: torch.Tensor, block_tables: torch.Tensor, window: int, scale: float,
+                sink: torch.Tensor, wuv: torch.Tensor, out: torch.Tensor, num_splits: int = 0, gate: torch.Tensor | None = None) -> None:
+    """Absorbed attention of the rows qa [Ta, H, rp] over the paged rows (all rp columns make the scores, the first wuv.shape[2] of
+    them are the latent), then W_uv and the gate rows ([T, H * vdimp], factors): writes out[:Ta] ([T, H * vdimp])."""
     Ta, H, rp = qa.shape
     n_blocks, bs, _ = cache.shape
-    vdimp = wuv.shape[1]
+    vdimp, vp = wuv.shape[1:]
     if Ta == 0:
         return
     assert qa.is_contiguous() and cache.is_contiguous() and cache.dtype == qa.dtype and wuv.is_contiguous()
-    assert wuv.shape == (H, vdimp, rp) and sink.dtype == torch.float32 and sink.numel() == H and block_tables.stride(1) == 1
+    assert wuv.shape[0] == H and vp <= rp == cache.shape[2] and sink.dtype == torch.float32 and sink.numel() == H and block_tables.stride(1) == 1
     for t in (tile_tok, tile_n, pos, seq_of, block_tables):
         assert t.dtype == torch.int32
     assert pos.numel() >= Ta and seq_of.numel() >= Ta and out.stride(1) == 1 and out.shape[0] >= Ta and out.shape[1] == H * vdimp
+    assert gate is None or (gate.dtype == out.dtype and gate.stride(1) == 1 and gate.shape[0] >= Ta and gate.shape[1] == H * vdimp)
     lib, f32 = load_library(), _is_f32(qa.dtype)
     part_o = part_ml = None
     ns = 1
@@ -1417,19 +1490,22 @@ def latent_attn(qa: torch.Tensor, cache: torch.Tensor, tile_tok: torch.Tensor, t
         keys = min(window + tokens_per_tile, block_tables.shape[1] * bs)
         # (and no more keys per split than a workgroup's slice of the block table covers)
         ns = num_splits or max(1, min(64, 256 // max(1, wgs), -(-keys // 128)), -(-keys // (900 * bs)))
-    ctx = torch.empty((Ta, H, rp), dtype=qa.dtype, device=qa.device)
+    ctx = torch.empty((Ta, H, vp), dtype=qa.dtype, device=qa.device)
     if ns > 1:
-        part_o = torch.empty((Ta * H, ns, rp), dtype=torch.float32, device=qa.device)
+        part_o = torch.empty((Ta * H, ns, vp), dtype=torch.float32, device=qa.device)
         part_ml = torch.empty((Ta * H, ns, 2), dtype=torch.float32, device=qa.device)
     _check(lib.glm_latent_attn(_p(qa), _p(cache), n_blocks, bs, _p(tile_tok), _p(tile_n), tile_tok.numel(), tokens_per_tile, _p(pos),
-                               _p(seq_of), _p(block_tables), block_tables.stride(0), Ta, H, rank, rp, window, scale, _p(sink), ns,
+                               _p(seq_of), _p(block_tables), block_tables.stride(0), Ta, H, rp, vp, window, scale, _p(sink), ns,
                                _p(ctx), _p(part_o), _p(part_ml), f32, _stream()), "glm_latent_attn")
     if f32:
         batched_gemm_f32(ctx.transpose(0, 1), wuv, out[:Ta].view(Ta, H, vdimp).transpose(0, 1))
+        if gate is not None:
+            mul_f32(out[:Ta], gate[:Ta])
         return
     if ns > 1:
-        _check(lib.glm_attn_merge(_p(part_o), _p(part_ml), _p(sink), ns, _p(ctx), Ta, H, rp, _stream()), "glm_attn_merge")
-    _check(lib.glm_latent_up(_p(ctx), _p(wuv), _p(out), out.stride(0), Ta, H, vdimp, rp, _stream()), "glm_latent_up")
+        _check(lib.glm_attn_merge(_p(part_o), _p(part_ml), _p(sink), ns, _p(ctx), Ta, H, vp, _stream()), "glm_attn_merge")
+    _check(lib.glm_latent_up(_p(ctx), _p(wuv), _p(out), _p(gate), gate.stride(0) if gate is not None else 0, out.stride(0), Ta, H, vdimp, vp, _stream()),
+           "glm_latent_up")
 
 
 WINDOW_ATTN_MAX_DIM = 256  # head sizes of glm_window_attn_prefill
@@ -1437,17 +1513,27 @@ WINDOW_ATTN_MAX_DIM = 256  # head sizes of glm_window_attn_prefill
 
 def window_attn_prefill(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, out: torch.Tensor, q_start: torch.Tensor,
                         k_start: torch.Tensor, tile_seq: torch.Tensor, tile_off: torch.Tensor, heads: int, dk: int, dv: int,
-                        window: int, scale: float, sink: torch.Tensor) -> None:
-    """q, out: rows of the step's long portions (views with free row pitch); k, v: expanded rows, see the header."""
+                        window: int, scale: float, sink: torch.Tensor, kr: torch.Tensor | None = None, cs: torch.Tensor | None = None,
+                        gate: torch.Tensor | None = None) -> None:
+    """q, out: rows of the step's long portions (views with free row pitch); k, v: expanded rows, see the header.  kr [Tk, rotp]: the
+    rotated key part that all heads share, the last of dk columns (k holds the others), cs the rotation of these query columns."""
     _bf16(q, "q"); _bf16(k, "k"); _bf16(v, "v"); _bf16(out, "out")
-    assert q.shape[1] == k.shape[1] == heads * dk and v.shape[1] == out.shape[1] == heads * dv and k.stride(0) == v.stride(0)
+    rotp = kr.shape[1] if kr is not None else 0
+    assert q.shape[1] == heads * dk and k.shape[1] == heads * (dk - rotp) and v.shape[1] == out.shape[1] == heads * dv and k.stride(0) == v.stride(0)
     assert k.shape[0] == v.shape[0] and out.shape[0] == q.shape[0] and sink.dtype == torch.float32 and sink.numel() == heads
     for t in (q_start, k_start, tile_seq, tile_off):
         assert t.dtype == torch.int32
     S = q_start.numel() - 1
     assert k_start.numel() == S + 1 and tile_seq.numel() == tile_off.numel()
+    if rotp:
+        _bf16(kr, "kr")
+        assert kr.shape[0] == k.shape[0] and kr.stride(1) == 1 and cs.dtype == torch.float32 and cs.is_contiguous() and cs.numel() == q.shape[0] * rotp
+    if gate is not None:
+        _bf16(gate, "gate")
+        assert gate.shape == out.shape and gate.stride(1) == 1
     _check(load_library().glm_window_attn_prefill(
-        _p(q), q.stride(0), _p(k), _p(v), k.stride(0), _p(out), out.stride(0), _p(q_start), _p(k_start), _p(tile_seq), _p(tile_off),
+        _p(q), q.stride(0), _p(k), _p(v), k.stride(0), _p(kr), kr.stride(0) if rotp else 0, rotp, _p(cs), _p(gate), gate.stride(0) if gate is not None else 0,
+        _p(out), out.stride(0), _p(q_start), _p(k_start), _p(tile_seq), _p(tile_off),
         tile_seq.numel(), S, q.shape[0], k.shape[0], heads, dk, dv, window, scale, _p(sink), _stream()), "glm_window_attn_prefill")
 
 
@@ -1647,3 +1733,176 @@ def memory_chunkwise(x: torch.Tensor, hrow: torch.Tensor, wif: torch.Tensor, bif
                                     _p(state_in), _p(state_out), seqs, heads, dim, dimp, vdimp, _stream()), "glm_memory_chunkwise")
     _check(lib.glm_memory_output(_p(o), vd, _p(x[:, 2 * kd + vd:]), x.stride(0), _p(norm), _p(y), y.stride(0), T, heads, vdim, vdimp, eps, _stream()),
            "glm_memory_output")
+
+
+def linear_recurrent(x: torch.Tensor, decay: torch.Tensor, S: torch.Tensor, pos, q_start, state_in, state_out, heads: int, dimp: int, vdimp: int) -> torch.Tensor:
+    """Linear memory (constant decay) token by token: rows x = q | k | v | ... -> fp32 rows o [T, heads * vdimp] in front of their norm."""
+    kd, T = heads * dimp, x.shape[0]
+    assert S.shape[1:] == (heads, dimp, vdimp) and S.dtype == torch.float32 and S.is_contiguous() and decay.dtype == torch.float32 and decay.numel() == heads
+    assert x.shape[1] >= 2 * kd + heads * vdimp and x.stride(1) == 1
+    for t in (pos, q_start, state_in, state_out):
+        assert t.dtype == torch.int32
+    seqs = q_start.numel() - 1
+    assert state_in.numel() >= seqs and state_out.numel() >= seqs
+    o = torch.empty((T, heads * vdimp), dtype=torch.float32, device=x.device)
+    _check(load_library().glm_linear_recurrent(
+        _p(x), x.stride(0), kd, 2 * kd, _p(decay), _p(o), heads * vdimp, _p(S), S.shape[0], _p(pos), _p(q_start), _p(state_in), _p(state_out), seqs, heads, dimp, vdimp,
+        _is_f32(x.dtype), _stream()), "glm_linear_recurrent")
+    return o
+
+
+def linear_chunkwise(x: torch.Tensor, powers: torch.Tensor, S: torch.Tensor, pos, q_start, state_in, state_out, heads: int, dimp: int, vdimp: int) -> torch.Tensor:
+    """The same for long portions (bf16), 64 tokens at a time; powers [heads, 65] = decay^j; q_start and pos relative to the rows of x."""
+    _bf16(x, "x")
+    kd, T = heads * dimp, x.shape[0]
+    assert S.shape[1:] == (heads, dimp, vdimp) and S.dtype == torch.float32 and S.is_contiguous() and powers.dtype == torch.float32 and powers.shape == (heads, 65) and powers.is_contiguous()
+    assert x.shape[1] >= 2 * kd + heads * vdimp and x.stride(1) == 1 and pos.numel() == T
+    for t in (pos, q_start, state_in, state_out):
+        assert t.dtype == torch.int32
+    seqs = q_start.numel() - 1
+    assert state_in.numel() >= seqs and state_out.numel() >= seqs
+    o = torch.empty((T, heads * vdimp), dtype=x.dtype, device=x.device)
+    _check(load_library().glm_linear_chunkwise(
+        _p(x), x.stride(0), kd, 2 * kd, _p(powers), _p(o), heads * vdimp, _p(S), S.shape[0], _p(pos), _p(q_start), _p(state_in), _p(state_out), seqs, heads, dimp, vdimp,
+        _stream()), "glm_linear_chunkwise")
+    return o
+
+
+def row_norm_gate(o: torch.Tensor, gate: torch.Tensor, norm: torch.Tensor, n: int, eps: float, y: torch.Tensor) -> None:
+    """y = o / rms(o) . norm . gate per row; n of the columns are true, the others zeros."""
+    T, np_ = o.shape
+    assert gate.shape == y.shape == o.shape and gate.dtype == y.dtype and o.stride(1) == gate.stride(1) == y.stride(1) == 1 and norm.dtype == torch.float32 and norm.numel() == np_
+    _check(load_library().glm_row_norm_gate(_p(o), o.stride(0), _is_f32(o.dtype), _p(gate), gate.stride(0), _p(norm), _p(y), y.stride(0), T, n, np_, eps, _is_f32(y.dtype), _stream()),
+           "glm_row_norm_gate")
+
+
+# ------------------------------------------------------------------------------------------
+# decoders whose sublayers read the residual as it is, with norms in groups, an average over depth and softmax-routed experts
+def depth_norm_taps(taps: int) -> int:
+    t = load_library().glm_depth_norm_taps(taps)
+    if t < 0:
+        raise NotImplementedError(f"a convolution over {taps} tokens is not built")
+    return t
+
+
+class ExpertRows:
+    """Unscaled rows of the experts [R, N] with the row and the fp32 weight of each of a token's k experts: what a feed-forward of experts
+    hands to the launch that closes it."""
+
+    def __init__(self, rows: torch.Tensor, pair_pos: torch.Tensor, weights: torch.Tensor):
+        self.rows, self.pair_pos, self.weights = rows, pair_pos, weights
+
+
+def depth_norm(x: torch.Tensor, width: int, groups: int, eps: float, y=None, g_post: torch.Tensor | None = None, x_out: torch.Tensor | None = None,
+               cast: bool = False, depth: tuple | None = None, x_next: torch.Tensor | None = None, g_pre: torch.Tensor | None = None, conv: tuple | None = None,
+               meta=None, rows: torch.Tensor | None = None, act_dtype=torch.bfloat16):
+    """Between two sublayers (glm_depth_norm).  y: sublayer output [T, wp] or ExpertRows, g_post the gain of its norm; x_out receives the
+    residual behind it, cast: also in the activation dtype (returned); depth = (planes [n, T, wp], coefficients [n + 1]), their average
+    goes to x_next; h is the result of `conv` (bf16 weights, state) or of the norm with gain g_pre.  Returns (cast, h)."""
+    wp = x.shape[1]
+    T = rows.numel() if rows is not None else x.shape[0]
+    dev, f32 = x.device, _is_f32(act_dtype)
+    for t in (x, x_out, x_next):
+        assert t is None or (t.dtype == torch.float32 and t.is_contiguous() and t.shape[1] == wp)
+    assert x_out is None or x_out.shape[0] == T
+    assert x_next is None or x_next.shape[0] == T
+    yp = pos_p = w_p = None
+    ldy, k, n_rows = wp, 0, 0
+    if y is not None:
+        t = y.rows if isinstance(y, ExpertRows) else y
+        assert t.dtype == act_dtype and t.stride(1) == 1 and t.shape[1] == wp and g_post is not None
+        yp, ldy = _p(t), t.stride(0)
+        if isinstance(y, ExpertRows):
+            k, n_rows = y.weights.shape[1], t.shape[0]
+            assert y.weights.shape[0] == x.shape[0] and y.weights.dtype == torch.float32 and y.pair_pos.dtype == torch.int32 and y.pair_pos.numel() == y.weights.numel()
+            pos_p, w_p = _p(y.pair_pos), _p(y.weights)
+        else:
+            assert t.shape[0] == x.shape[0]
+    for g in (g_post, g_pre):
+        assert g is None or (g.dtype == torch.float32 and g.is_contiguous() and g.numel() == wp)
+    dp = cp = None
+    n_depth = stride = 0
+    if depth is not None:
+        planes, coef = depth
+        n_depth, stride = planes.shape[0], planes.stride(0)
+        assert planes.shape[1:] == x.shape and planes.dtype == torch.float32 and planes.stride(1) == wp and planes.stride(2) == 1
+        assert coef.dtype == torch.float32 and coef.numel() == n_depth + 1
+        dp, cp = _p(planes), _p(coef)
+    x_cast = torch.empty((T, wp), dtype=act_dtype, device=dev) if cast else None
+    h = torch.empty((T, wp), dtype=act_dtype, device=dev) if (conv is not None or g_pre is not None) else None
+    taps, n_state, cw, st = 1, 0, None, None
+    args = (None,) * 5
+    if conv is not None:
+        cw, st = conv
+        taps, n_state = cw.shape[0], st.shape[0]
+        assert cw.dtype == torch.bfloat16 and st.dtype == torch.float32 and cw.is_contiguous() and st.is_contiguous() and cw.shape[1] == wp
+        if taps == 1:
+            raise ValueError("a convolution of one tap keeps two (depth_norm_taps)")
+        assert st.shape[1:] == (taps - 1, wp) and rows is None
+        args = (meta.pos, meta.seq_of, meta.q_start, meta.state_in, meta.state_out)
+        assert meta.pos.numel() == meta.seq_of.numel() == T
+    _check(load_library().glm_depth_norm(
+        _p(x), _p(rows), wp, yp, ldy, pos_p, w_p, k, n_rows, _p(g_post) if y is not None else None, _p(x_out), _p(x_cast), wp, dp, stride, n_depth, cp, _p(x_next), _p(g_pre),
+        _p(cw), taps, _p(st), n_state, *(_p(a) for a in args), _p(h), wp, f32, T, width, wp, groups, eps, _stream()), "glm_depth_norm")
+    return x_cast, h
+
+
+def softmax_router(logits: torch.Tensor, E: int, k: int):
+    """The k largest scores of softmax(logits[:, :E]) per row: (experts int64 [T, k], weights fp32 [T, k]), not renormalised."""
+    T = logits.shape[0]
+    assert logits.dtype == torch.float32 and logits.stride(1) == 1 and logits.shape[1] >= E
+    idx = torch.empty((T, k), dtype=torch.int64, device=logits.device)
+    w = torch.empty((T, k), dtype=torch.float32, device=logits.device)
+    _check(load_library().glm_router_softmax(_p(logits), logits.stride(0), _p(idx), _p(w), T, E, k, _stream()), "glm_router_softmax")
+    return idx, w
+
+
+ROUTER_ALIGN_MAX_ROWS = 128   # rows up to which one workgroup routes and buckets them
+
+
+def softmax_router_align(logits: torch.Tensor, E: int, k: int):
+    """softmax_router and the bucketing of its pairs: (weights [T, k], offsets [E + 1], source rows [T k], pair positions [T k])."""
+    T, dev = logits.shape[0], logits.device
+    if T > ROUTER_ALIGN_MAX_ROWS:
+        idx, w = softmax_router(logits, E, k)
+        offs, tok, _, pos = moe_align(idx, None, E, False)
+        return w, offs, tok, pos
+    assert logits.dtype == torch.float32 and logits.stride(1) == 1 and logits.shape[1] >= E
+    idx = torch.empty((T, k), dtype=torch.int64, device=dev)
+    w = torch.empty((T, k), dtype=torch.float32, device=dev)
+    offs, tok, pos = (torch.empty(n, dtype=torch.int32, device=dev) for n in (E + 1, T * k, T * k))
+    _check(load_library().glm_router_softmax_align(_p(logits), logits.stride(0), _p(idx), _p(w), _p(offs), _p(tok), _p(pos), T, E, k, _stream()), "glm_router_softmax_align")
+    return w, offs, tok, pos
+
+
+def combine_weighted(y: ExpertRows) -> torch.Tensor:
+    """Sum of the experts' rows with their weights, one row per token."""
+    r, (T, k) = y.rows, y.weights.shape
+    out = torch.empty((T, r.shape[1]), dtype=r.dtype, device=r.device)
+    _check(load_library().glm_moe_combine_weighted(_p(r), r.stride(0), r.shape[0], _p(y.pair_pos), _p(y.weights), _p(out), out.stride(0), T, k, r.shape[1], _is_f32(r.dtype), _stream()),
+           "glm_moe_combine_weighted")
+    return out
+
+
+def grouped_swiglu(x: torch.Tensor, w13: torch.Tensor, offs: torch.Tensor, tok: torch.Tensor) -> torch.Tensor:
+    """silu(gate) up of the gathered rows, w13 [G, 2 I, K] rows gate | up, bf16 or fp32 -> [rows, I]."""
+    if x.dtype == torch.bfloat16:
+        return grouped_gemm_gateup_silu(x, w13, offs, tok, tok.numel(), max_rows_per_group=x.shape[0])
+    G, I2, K = w13.shape
+    R = tok.numel()
+    t = torch.empty((R, I2), dtype=x.dtype, device=x.device)
+    act = torch.empty((R, I2 // 2), dtype=x.dtype, device=x.device)
+    lib = load_library()
+    _check(lib.glm_grouped_gemm_f32(_p(x), x.stride(0), _p(w13), w13.stride(0), w13.stride(1), _p(offs), _p(tok), _p(t), I2, R, I2, K, G, _stream()), "glm_grouped_gemm_f32")
+    _check(lib.glm_swiglu_f32(_p(t), I2, _p(act), I2 // 2, R, I2 // 2, _stream()), "glm_swiglu_f32")
+    return act
+
+
+def grouped_down(act: torch.Tensor, w2: torch.Tensor, offs: torch.Tensor, max_rows_per_group: int) -> torch.Tensor:
+    """Unscaled down projection of the experts' rows, w2 [G, N, I]."""
+    if act.dtype == torch.bfloat16:
+        return grouped_gemm_down(act, w2, offs, None, 0, max_rows_per_group=max_rows_per_group)
+    G, N, I = w2.shape
+    y = torch.empty((act.shape[0], N), dtype=act.dtype, device=act.device)
+    _check(load_library().glm_grouped_gemm_f32(_p(act), I, _p(w2), w2.stride(0), w2.stride(1), _p(offs), None, _p(y), N, act.shape[0], N, I, G, _stream()), "glm_grouped_gemm_f32")
+    return y

@@ -1,5 +1,6 @@
-"""Latent attention over a paged cache of one latent row per token, with a sliding window and a sink per head, without
-positions (csrc/latent_attn.hip, csrc/window_attn.hip).
+"""Latent attention over a paged cache of one latent row per token, with a sink per head, with or without a sliding window, a rotated
+key part that all heads share (cached behind the latent), queries that go through a latent of their own, and an output gate
+(csrc/latent_attn.hip, csrc/window_attn.hip).
 
 Two evaluations of the same mechanism share a step: short portions (decoded tokens above all) attend in the absorbed form over
 the cached latents, long portions expand keys and values.  The step's batch says which rows are which (StepBatch.Ta)."""
@@ -11,6 +12,7 @@ from torch import nn
 from nanovllm import hip_ops
 from nanovllm.distributed.parallel_state import get_tp_group
 from nanovllm.layers.linear import PaddedLinear
+from nanovllm.layers.rotary_embedding import PairRotary
 from nanovllm.layers.seq_norm import norm_gain
 
 
@@ -25,7 +27,10 @@ def absorb_break_even(rank: int, dim: int, vdim: int) -> int:
 
 class LatentAttention(nn.Module):
 
-    def __init__(self, width: int, heads: int, dim: int, vdim: int, rank: int, window: int, scale: float, eps: float, dtype, runs: int = 1):
+    def __init__(self, width: int, heads: int, dim: int, vdim: int, rank: int, window: int, scale: float, eps: float, dtype, runs: int = 1,
+                 q_rank: int | None = None, rot_dim: int = 0, rot: PairRotary | None = None, gated: bool = False):
+        """q_rank: size of the queries' latent (None: queries straight from the input); rot_dim: rotated columns of a head behind the
+        `dim` unrotated ones, turned by `rot`; gated: sigmoid gate on the heads, projected from the input."""
         super().__init__()
         tp = get_tp_group()
         if heads % tp.world_size:
@@ -34,26 +39,43 @@ class LatentAttention(nn.Module):
         self.heads = heads // tp.world_size
         self.dim, self.vdim, self.rank, self.window, self.scale, self.eps, self.dtype = dim, vdim, rank, window, scale, eps, dtype
         self.dimp, self.vdimp, self.rp = hip_ops.round8(dim), hip_ops.round8(vdim), hip_ops.round8(rank)
+        self.q_rank, self.rot_dim, self.rotp, self.rot, self.gated = q_rank, rot_dim, hip_ops.round8(rot_dim), rot, gated
         H = self.heads
-        self.qc_proj = PaddedLinear(width, [self.dimp] * H + [self.rp], dtype)     # query heads, raw latent
+        self.rc = self.rp + self.rotp                   # columns of a cache row
+        head = [self.dimp] + ([self.rotp] if rot_dim else [])
+        # queries (heads, or their raw latent), raw latent, raw rotated key part, gate
+        queries = head * H if q_rank is None else [hip_ops.round8(q_rank)]
+        self.c_off = sum(queries)
+        self.qc_proj = PaddedLinear(width, queries + [self.rp] + ([self.rotp] if rot_dim else []) + ([self.vdimp] * H if gated else []), dtype)
+        self.g_off = self.c_off + self.rc
+        self.act = (hip_ops.ACT_GATE, float(self.g_off), 0.0) if gated else hip_ops.NO_ACT
+        self.uq_proj = PaddedLinear(q_rank, head * H, dtype) if q_rank is not None else None
         # (fp32, and heads beyond the expanded kernel's sizes: every portion attends in the absorbed form)
-        self.can_expand = dtype == torch.bfloat16 and max(self.dimp, self.vdimp) <= hip_ops.WINDOW_ATTN_MAX_DIM
+        self.can_expand = dtype == torch.bfloat16 and max(self.dimp + self.rotp, self.vdimp) <= hip_ops.WINDOW_ATTN_MAX_DIM
         self.expand = PaddedLinear(rank, [self.dimp] * H + [self.vdimp] * H, dtype) if self.can_expand else None
         self.o_proj = PaddedLinear([vdim] * H, [hip_ops.round8(width)], dtype)
-        self.tokens_per_tile = hip_ops.latent_tokens_per_tile(self.rp, H) if dtype == torch.bfloat16 else 1
+        self.tokens_per_tile = hip_ops.latent_tokens_per_tile(self.rc, H) if dtype == torch.bfloat16 else 1
         self.break_even = absorb_break_even(self.rp, self.dimp, self.vdimp)
         self.caches: list = [None] * runs
         self.runs = runs
 
     def load(self, w: dict, device) -> None:
-        """w: q, dkv, dkv.norm, uk, uv, sink, o."""
+        """w: q or dq, dq.norm, uq; dkv, dkv.norm, uk, uv, sink, o; g if there is a gate."""
         H, h0 = self.heads, self.tp_rank * self.heads
 
         def heads_of(t, size):  # this rank's heads of a head-by-head layout
             return t.view(H * self.tp_size, size, -1)[h0: h0 + H].to(device)
 
-        q, uk, uv = heads_of(w["q"], self.dim), heads_of(w["uk"], self.dim), heads_of(w["uv"], self.vdim)
-        self.qc_proj.load(list(q) + [w["dkv"]], device)
+        uk, uv = heads_of(w["uk"], self.dim), heads_of(w["uv"], self.vdim)
+        q = heads_of(w["q" if self.q_rank is None else "uq"], self.dim + self.rot_dim)
+        blocks = [b for t in q for b in ((t[: self.dim], t[self.dim:]) if self.rot_dim else (t,))]
+        if self.q_rank is not None:
+            self.uq_proj.load(blocks, device)
+            self.cq_gain = norm_gain(w["dq.norm"], hip_ops.round8(self.q_rank), device, zero_centred=False)
+            blocks = [w["dq"]]
+        assert w["dkv"].shape[0] == self.rank + self.rot_dim
+        blocks += [w["dkv"][: self.rank]] + ([w["dkv"][self.rank:]] if self.rot_dim else [])
+        self.qc_proj.load(blocks + (list(heads_of(w["g"], self.vdim)) if self.gated else []), device)
         if self.expand is not None:
             self.expand.load(list(uk) + list(uv), device)
         self.wukt = torch.zeros(H, self.rp, self.dimp, dtype=self.dtype, device=device)
@@ -65,30 +87,44 @@ class LatentAttention(nn.Module):
         self.o_proj.load([w["o"][:, h0 * self.vdim: (h0 + H) * self.vdim]], device)
 
     def cache_bytes_per_token(self) -> int:
-        return self.runs * self.rp * self.dtype.itemsize
+        return self.runs * self.rc * self.dtype.itemsize
 
     def allocate_cache(self, num_blocks: int, block_size: int, device) -> None:
-        self.caches = [torch.empty(num_blocks, block_size, self.rp, dtype=self.dtype, device=device) for _ in range(self.runs)]
+        self.caches = [torch.empty(num_blocks, block_size, self.rc, dtype=self.dtype, device=device) for _ in range(self.runs)]
 
-    def forward(self, h: torch.Tensor, meta, run: int) -> torch.Tensor:
+    def _queries(self, h: torch.Tensor, meta, cache, win, cs):
+        """Projections, norms, cache store.  Returns (query rows, absorbed queries of the first Ta rows, latent rows for the expanded
+        form, gate rows)."""
+        H, Ta, T = self.heads, meta.Ta, h.shape[0]
+        x = self.qc_proj(h, act=self.act)
+        gate = x[:, self.g_off:] if self.gated else None
+        crow, n_crows = (win.crow, win.rows) if win else (None, 0)
+        if self.q_rank is None and not self.rotp:
+            qa, c_all = hip_ops.latent_prepare(x, self.c_off, H, self.dimp, self.rank, self.c_gain, self.eps, meta.slots, cache, Ta, self.wukt, crow, n_crows)
+            return x[:, : self.c_off], qa, c_all, gate
+        query = (0, self.q_rank, self.cq_gain) if self.q_rank is not None else None
+        cq, c_all = hip_ops.latent_rows(x, self.c_off, self.rank, self.c_gain, cs, self.eps, meta.slots, cache, query, crow, n_crows)
+        q = self.uq_proj(cq) if query else x[:, : self.c_off]
+        return q, hip_ops.latent_absorb(q[:Ta], H, self.dimp, cs, self.wukt, self.rotp) if Ta else None, c_all, gate
+
+    def forward(self, h: torch.Tensor, meta, run: int = 0, cs: torch.Tensor | None = None) -> torch.Tensor:
+        """cs: the step's rotation table of self.rot (PairRotary.table)."""
         H, Ta, T = self.heads, meta.Ta, h.shape[0]
         cache = self.caches[run]
-        qc = self.qc_proj(h)
-        nq = H * self.dimp
         win = meta.windows[self.window] if Ta < T else None
-        qa, c_all = hip_ops.latent_prepare(qc, nq, H, self.dimp, self.rank, self.c_gain, self.eps, meta.slots, cache, Ta, self.wukt,
-                                           win.crow if win else None, win.rows if win else 0)
+        q, qa, c_all, gate = self._queries(h, meta, cache, win, cs)
         out = torch.empty((T, H * self.vdimp), dtype=h.dtype, device=h.device)
         if Ta:
             tok, n = meta.tiles[min(self.tokens_per_tile, meta.max_short)]
             hip_ops.latent_attn(qa, cache, tok, n, min(self.tokens_per_tile, meta.max_short), meta.pos, meta.seq_of, meta.block_tables,
-                                self.rank, self.window, self.scale, self.sink, self.wuv, out)
+                                self.window, self.scale, self.sink, self.wuv, out, gate=gate)
         if Ta < T:
             if win.hist_rows.numel():
                 hip_ops.latent_gather(cache, win.hist_slots, win.hist_rows, c_all)
-            kv = self.expand(c_all)
-            hip_ops.window_attn_prefill(qc[Ta:, :nq], kv[:, :nq], kv[:, nq:], out[Ta:], meta.long_q_start, win.k_start, meta.long_tile_seq,
-                                        meta.long_tile_off, H, self.dimp, self.vdimp, self.window, self.scale, self.sink)
+            kv, nk = self.expand(c_all[:, : self.rp]), H * self.dimp
+            rotated = dict(kr=c_all[:, self.rp:], cs=cs[Ta:]) if self.rotp else {}
+            hip_ops.window_attn_prefill(q[Ta:], kv[:, :nk], kv[:, nk:], out[Ta:], meta.long_q_start, win.k_start, meta.long_tile_seq, meta.long_tile_off, H,
+                                        self.dimp + self.rotp, self.vdimp, self.window, self.scale, self.sink, gate=gate[Ta:] if gate is not None else None, **rotated)
         y = self.o_proj(out)
         if self.tp_size > 1:
             get_tp_group().all_reduce(y)

@@ -1,8 +1,12 @@
 """NeoX rotary embedding on the first rotary_dim dims of each head — reference:
 layers/rotary_embedding.py:17-71.  The cos/sin table is built on the host with the same torch
-ops as the reference (so the table is bit-identical); the rotation is glm_rope_neox."""
+ops as the reference (so the table is bit-identical); the rotation is glm_rope_neox.
+
+PairRotary: rotation of neighbouring columns, with YaRN's scaling, for models that run step batches (no counterpart in the
+reference)."""
 from __future__ import annotations
 
+import math
 from functools import lru_cache
 
 import torch
@@ -36,3 +40,44 @@ def get_rope(head_size: int, rotary_dim: int, max_position: int, base: float,
     if partial_rotary_factor < 1.0:
         rotary_dim = int(head_size * partial_rotary_factor)
     return RotaryEmbedding(head_size, rotary_dim, max_position, base)
+
+
+def yarn_frequencies(base: float, dims: int, factor: float, original: float, fast: float, slow: float) -> list[float]:
+    """Frequencies of dims / 2 pairs with YaRN's interpolation: pairs that turn more than `fast` times over the original length keep
+    theirs, those that turn less than `slow` times are slowed down by `factor`, with a linear ramp over the pair index between."""
+    def pair_of(turns):
+        return dims * math.log(original / (2 * math.pi * turns)) / (2 * math.log(base))
+
+    lo, hi = max(math.floor(pair_of(fast)), 0), min(math.ceil(pair_of(slow)), dims - 1)
+    width = max(hi - lo, 0.001)
+    freq = []
+    for i in range(dims // 2):
+        f, ramp = base ** (-2.0 * i / dims), min(max((i - lo) / width, 0.0), 1.0)
+        freq.append(f / factor * ramp + f * (1.0 - ramp))
+    return freq
+
+
+class PairRotary:
+    """Rotation of the column pairs (2i, 2i+1), i < dims / 2, of a head's rotated part of rot_dim columns (the rest do not turn).  The
+    table of a step is made on the device from its positions, so no length is built in; layers with the same rotation share it."""
+
+    def __init__(self, rot_dim: int, dims: int, base: float, scaling: dict | None = None):
+        if dims % 2 or rot_dim % 2 or not 0 < dims <= rot_dim:
+            raise ValueError(f"a rotation of {dims} of {rot_dim} columns")
+        self.pairs = hip_ops.round8(rot_dim) // 2
+        if scaling is None:
+            self.freq, self.mscale = tuple(base ** (-2.0 * i / dims) for i in range(dims // 2)), 1.0
+        else:
+            self.freq = tuple(yarn_frequencies(base, dims, *(scaling[k] for k in ("factor", "original", "fast", "slow"))))
+            self.mscale = 0.1 * math.log(scaling["factor"]) + 1.0
+        self.key = (self.pairs, self.freq, self.mscale)
+        self._dev = {}
+
+    def prepare(self, device) -> None:
+        """The frequencies on the device (at load time: a captured step only reads them)."""
+        if device not in self._dev:
+            self._dev[device] = torch.tensor(self.freq, dtype=torch.float64, device="cpu").to(device)
+
+    def table(self, pos: torch.Tensor) -> torch.Tensor:
+        """cos, sin [T, pairs, 2] at the positions of a step."""
+        return hip_ops.rope_pairs(pos, self._dev[pos.device], self.mscale, self.pairs)

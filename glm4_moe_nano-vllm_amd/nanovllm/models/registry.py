@@ -35,8 +35,10 @@ DAFOLORN = ModelEntry("dafolorn", "nanovllm.models.dafolorn.config:read_config",
                       64, 32, ("bfloat16", "float32"), "dafolorn", True)
 NAPADRA = ModelEntry("napadra", "nanovllm.models.napadra.config:read_config", "nanovllm.models.napadra.model:NapadraForCausalLM",
                      64, 64, ("bfloat16", "float32"), "napadra", True)
+GULOZEN = ModelEntry("gulozen", "nanovllm.models.gulozen.config:read_config", "nanovllm.models.gulozen.model:GulozenForCausalLM",
+                     64, 32, ("bfloat16", "float32"), "gulozen", True)
 
-_ENTRIES = {e.name: e for e in (GLM4_MOE, DAFOLORN, NAPADRA)}
+_ENTRIES = {e.name: e for e in (GLM4_MOE, DAFOLORN, NAPADRA, GULOZEN)}
 
 
 def find_model(cfg) -> ModelEntry:

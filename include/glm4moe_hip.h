@@ -171,7 +171,8 @@ int glm_router_select(const void* logits, int64_t ld_logits, const float* e_scor
  *     group (id E) holding every token once is appended (the shared expert, moe.py:165).
  *     G = E + (with_shared?1:0), R = T*k + (with_shared?T:0).
  *     expert_offsets int32 [G+1]; sorted_token int32 [R]; sorted_scale bf16 [R] (routing
- *     weight of the row; 1.0 for shared rows); pair_pos int32 [T*k] (sorted row of pair).    */
+ *     weight of the row; 1.0 for shared rows); pair_pos int32 [T*k] (sorted row of pair).  Without a shared
+ *     group topk_w and sorted_scale may both be NULL (the caller weighs the rows itself).    */
 int glm_moe_align(const int64_t* topk_idx, const void* topk_w,
                   int32_t* expert_offsets, int32_t* sorted_token, void* sorted_scale,
                   int32_t* pair_pos, int64_t T, int k, int E, int with_shared,
@@ -496,6 +497,8 @@ int glm_allreduce_oneshot(const void* in, void* out, void* const* peer_bufs, voi
 #define GLM_EPI_XIELU     1
 #define GLM_EPI_SOFTCAP   2
 #define GLM_EPI_GLU_CLAMP 3 /* glm_gemm_bf16_glu only */
+#define GLM_EPI_GATE      4 /* columns below a: z; the others: sigmoid(z) */
+#define GLM_EPI_SILU_GATE 5 /* columns below a: z sigmoid(z); the others: sigmoid(z) */
 /* y = act(x . W^T + bias): glm_gemm_bf16 with an activation in the epilogue and, with out_f32, fp32 output rows (unrounded).  */
 int glm_gemm_bf16_act(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* bias, void* y, int64_t ldy, int64_t M,
                       int N, int K, int out_f32, int act, float act_a, float act_b, glm_stream_t stream);
@@ -524,9 +527,11 @@ int glm_seq_norm(const float* x_in, const int32_t* row_index, int64_t ldx, float
                  const int32_t* q_start, const int32_t* state_in, const int32_t* state_out, void* h, int64_t ldh, int act_f32,
                  int64_t T, int width, int wp, float eps, glm_stream_t stream);
 /* embedding rows as the fp32 residual and, optionally, in the activation dtype; columns [width, wp) are zeros.  freq [width / 2 rounded
- * up] (double, or NULL) with pos [T]: sin(pos freq[i]) is added at column 2i, cos(pos freq[i]) at column 2i + 1             */
+ * up] (double, or NULL) with pos [T]: sin(pos freq[i]) is added at column 2i, cos(pos freq[i]) at column 2i + 1; the table's rows are
+ * multiplied by scale                                                                                                       */
 int glm_embed_rows(const int64_t* ids, const void* table, int64_t ldw, int64_t vocab, const int32_t* pos, const double* freq,
-                   float* x, int64_t ldx, void* cast, int64_t ldc, int act_f32, int64_t T, int width, int wp, glm_stream_t stream);
+                   float* x, int64_t ldx, void* cast, int64_t ldc, int act_f32, int64_t T, int width, int wp, float scale,
+                   glm_stream_t stream);
 
 /* Between two sublayers of a decoder whose residual is S parallel streams: x'_t = sum_s mix[s, t] x_s + out[t] (y_scale . y), then
  * u = sum_s w_in[s] x'_s, h = u / rms(u) gain, and with `shift` h += (h of the previous token - h) . shift.  x_in: row r, stream s at
@@ -586,32 +591,85 @@ int glm_memory_chunkwise(const void* x, int64_t ldx, int64_t k_off, int64_t v_of
 int glm_memory_output(const void* o, int64_t ldo, const void* g, int64_t ldg, const float* norm, void* y, int64_t ldy, int64_t T,
                       int H, int vdim, int vdimp, float eps, glm_stream_t stream);
 
+/* The linear memory (attention with a constant decay per head): S_t = decay S_(t-1) + k v^T, o_t = S_t^T q.  x rows hold q at h*dimp, k at
+ * k_off + h*dimp, v at v_off + h*vdimp; state S [n_state][H][dimp][vdimp] fp32.  recurrent: o fp32 rows [T, ldo]; chunkwise (long
+ * portions, bf16, dimp <= 256): powers [H][65] = decay^j, o bf16 rows.  row_norm_gate: y = o / rms(o) norm gate over np columns of a row,
+ * n of them true (the others zeros).                                                                                          */
+int glm_linear_recurrent(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* decay, float* o, int64_t ldo, float* S,
+                         int64_t n_state, const int32_t* pos, const int32_t* q_start, const int32_t* state_in, const int32_t* state_out,
+                         int seqs, int H, int dimp, int vdimp, int f32, glm_stream_t stream);
+int glm_linear_chunkwise(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* powers, void* o, int64_t ldo, float* S,
+                         int64_t n_state, const int32_t* pos, const int32_t* q_start, const int32_t* state_in, const int32_t* state_out,
+                         int seqs, int H, int dimp, int vdimp, glm_stream_t stream);
+int glm_row_norm_gate(const void* o, int64_t ldo, int o_f32, const void* gate, int64_t ldg, const float* norm, void* y, int64_t ldy,
+                      int64_t T, int n, int np, float eps, int act_f32, glm_stream_t stream);
+
+/* Between two sublayers of a decoder whose sublayers read the fp32 residual as it is: x_out = x_in + norm(y) g_post (the norm divides each
+ * of `groups` equal parts by its own root mean square), x_next = sum_j coef[j] depth_j + coef[n_depth] x_out (depth_j at depth + j
+ * depth_stride), and h = x_next + conv(x_next) or, with g_pre, norm(x_next) g_pre.  y: rows of the sublayer, or with pair_pos [T, k] the
+ * experts' rows, weighed by pair_w in fp32.  All fp32 rows have pitch ld; every part is optional; taps as glm_depth_norm_taps; rows of a
+ * step and state rows [n_state][taps-1][wp] as for glm_seq_norm; row_index gathers rows of x_in, y and the depths (no convolution).   */
+int glm_depth_norm_taps(int taps);
+int glm_depth_norm(const float* x_in, const int32_t* row_index, int64_t ld, const void* y, int64_t ldy, const int32_t* pair_pos,
+                   const float* pair_w, int k, int64_t n_rows, const float* g_post, float* x_out, void* x_cast, int64_t ldc,
+                   const float* depth, int64_t depth_stride, int n_depth, const float* coef, float* x_next, const float* g_pre,
+                   const void* conv_w, int taps, float* state, int64_t n_state, const int32_t* pos, const int32_t* seq_of,
+                   const int32_t* q_start, const int32_t* state_in, const int32_t* state_out, void* h, int64_t ldh, int act_f32,
+                   int64_t T, int width, int wp, int groups, float eps, glm_stream_t stream);
+
+/* Softmax router: the k largest of softmax(logits) over E experts, fp32 weights, not renormalised; descending.  _align: and the bucketing
+ * of glm_moe_align (no shared group, no scales) in one launch, for few tokens.  combine_weighted: out[t] = sum_j w[t,j] y[pair_pos[t,j]]. */
+int glm_router_softmax(const float* logits, int64_t ld, int64_t* topk_idx, float* topk_w, int64_t T, int E, int k, glm_stream_t stream);
+int glm_router_softmax_align(const float* logits, int64_t ld, int64_t* topk_idx, float* topk_w, int32_t* expert_offsets,
+                             int32_t* sorted_token, int32_t* pair_pos, int64_t T, int E, int k, glm_stream_t stream);
+int glm_moe_combine_weighted(const void* y, int64_t ldy, int64_t R, const int32_t* pair_pos, const float* w, void* out, int64_t ldo,
+                             int64_t T, int k, int H, int f32, glm_stream_t stream);
+/* fp32 forms of the grouped projections: rows [offsets[g], offsets[g+1]) of y = x[src[r]] w_g^T; silu(gate) up of rows gate | up; y *= g */
+int glm_grouped_gemm_f32(const float* x, int64_t ldx, const float* w, int64_t w_group_stride, int64_t ldw, const int32_t* offsets,
+                         const int32_t* src, float* y, int64_t ldy, int64_t R, int N, int K, int G, glm_stream_t stream);
+int glm_swiglu_f32(const float* x, int64_t ldx, float* y, int64_t ldy, int64_t M, int N, glm_stream_t stream);
+int glm_mul_f32(float* y, int64_t ldy, const float* g, int64_t ldg, int64_t M, int N, glm_stream_t stream);
+
 /* Latent attention over a paged cache [n_blocks, block_size, rp] of latent rows (rp = rank rounded up to 8).
  * prepare: row t of qc holds the query heads at h*dimp and the raw latent at c_off; c = rms(raw) norm_w goes to cache row
  * slots[t] (< 0: none) and to row crow[t] of c_out; for rows [0, Ta): qa[t, h, :] = W_uk[h]^T q[t, h, :] (wukt [H, rp, dimp]; bf16 only). */
 int glm_latent_prepare(const void* qc, int64_t ldq, int c_off, int64_t T, int64_t Ta, int H, int dimp, int rank, int rp,
                        const float* norm_w, float eps, const int32_t* slots, void* cache, int64_t n_slots, const int32_t* crow,
                        void* c_out, int64_t n_crows, const void* wukt, void* qa, int act_f32, glm_stream_t stream);
+/* The same with a rotated key part of rotp columns that all heads share and queries of a latent of their own, in two launches: cache rows are
+ * [latent rp | rotated part rotp].  rope_pairs: cs [T, pairs, 2] = mscale (cos, sin)(pos freq), pairs behind n_freq are (1, 0).  rows (in
+ * front of the query projection): qc holds the raw latent at c_off, the raw key part behind it and the queries' raw latent at cq_off, whose
+ * norm goes to cq_out.  absorb: qa[t, h] = W_uk^T q[t, h] | rotated rest of q[t, h] (fp32: only the rotated part).            */
+int glm_rope_pairs(const int32_t* pos, const double* freq, int n_freq, float mscale, float* cs, int64_t T, int pairs, glm_stream_t stream);
+int glm_latent_rows(const void* qc, int64_t ldq, int c_off, int rank, int rp, int rotp, const float* norm_w, const float* cs, float eps,
+                    const int32_t* slots, void* cache, int64_t n_slots, const int32_t* crow, void* c_out, int64_t n_crows, int cq_off,
+                    int cq_rank, int cq_rp, const float* cq_norm, void* cq_out, int64_t ld_cq, int64_t T, int act_f32,
+                    glm_stream_t stream);
+int glm_latent_absorb(const void* q, int64_t ldq, int64_t Ta, int H, int dimp, int rp, int rotp, const float* cs, const void* wukt,
+                      void* qa, int act_f32, glm_stream_t stream);
 int glm_latent_gather(const void* cache, int64_t n_slots, const int32_t* slots, const int32_t* rows, int64_t n, void* out,
                       int64_t n_rows, int row_bytes, glm_stream_t stream);
 /* attn: query row (t, h) sees the latents of positions (pos[t] - window, pos[t]] of its sequence; softmax with the extra mass
  * exp(sink[h]).  Tiles: tile i covers tile_n[i] <= tokens_per_tile consecutive rows of one sequence from tile_tok[i]; tokens x
- * heads of a tile <= glm_latent_attn_max_rows(rp).  nsplit == 1: ctx [Ta, H, rp] normalised (bf16 / fp32); else part_o
- * [Ta*H, nsplit, rp], part_ml [Ta*H, nsplit, 2] for glm_attn_merge, which forms ctx.  fp32: tiles unused, nsplit 1.
- * up: out[t, h*vdimp ..] = W_uv[h] ctx[t, h, :] (wuv [H, vdimp, rp]).                                                         */
+ * heads of a tile <= glm_latent_attn_max_rows(rp).  rp columns of a cache row make the scores, the first vp of them are summed up.
+ * nsplit == 1: ctx [Ta, H, vp] normalised (bf16 / fp32); else part_o [Ta*H, nsplit, vp], part_ml [Ta*H, nsplit, 2] for glm_attn_merge, which forms ctx.  fp32: tiles unused, nsplit 1.
+ * up: out[t, h*vdimp ..] = W_uv[h] ctx[t, h, :] (wuv [H, vdimp, rp]), times the row of gate (or NULL).                                                         */
 int glm_latent_attn_max_rows(int rp);
 int glm_latent_attn(const void* qa, const void* cache, int64_t n_blocks, int block_size, const int32_t* tile_tok,
                     const int32_t* tile_n, int n_tiles, int tokens_per_tile, const int32_t* pos, const int32_t* seq_of,
-                    const int32_t* block_tables, int64_t bt_stride, int64_t Ta, int H, int rank, int rp, int window, float scale,
+                    const int32_t* block_tables, int64_t bt_stride, int64_t Ta, int H, int rp, int vp, int window, float scale,
                     const float* sink, int nsplit, void* ctx, float* part_o, float* part_ml, int act_f32, glm_stream_t stream);
 int glm_attn_merge(const float* part_o, const float* part_ml, const float* sink, int nsplit, void* ctx, int64_t Ta, int H, int cols,
                    glm_stream_t stream);
-int glm_latent_up(const void* ctx, const void* wuv, void* out, int64_t ldo, int64_t Ta, int H, int vdimp, int rp,
+int glm_latent_up(const void* ctx, const void* wuv, void* out, const void* gate, int64_t ldg, int64_t ldo, int64_t Ta, int H, int vdimp, int rp,
                   glm_stream_t stream);
 /* Prompts and long portions, bf16: q rows [q_start[s], q_start[s+1]) against expanded k / v rows [k_start[s], k_start[s+1]) — the
  * portion's own tokens last, in front of them the history the window still reaches.  Head h at h*dk (q, k) / h*dv (v, out).
- * Tiles of 128 query rows: (sequence, first row inside the portion).  dk, dv <= 256, multiples of 8.                          */
-int glm_window_attn_prefill(const void* q, int64_t ldq, const void* k, const void* v, int64_t ldkv, void* out, int64_t ldo,
+ * Tiles of 128 query rows: (sequence, first row inside the portion).  dk, dv <= 256, multiples of 8.  rotp > 0: the last rotp of
+ * a head's dk columns are rotated on the way in (queries, by cs rows of glm_rope_pairs) and come from kr rows shared by all heads (keys,
+ * rotated already; k rows then hold dk - rotp columns per head).  gate (or NULL): factors of the output rows.                  */
+int glm_window_attn_prefill(const void* q, int64_t ldq, const void* k, const void* v, int64_t ldkv, const void* kr, int64_t ldr, int rotp,
+                            const float* cs, const void* gate, int64_t ldg, void* out, int64_t ldo,
                             const int32_t* q_start, const int32_t* k_start, const int32_t* tile_seq, const int32_t* tile_off,
                             int n_tiles, int S, int64_t Tq, int64_t Tk, int H, int dk, int dv, int window, float scale,
                             const float* sink, glm_stream_t stream);

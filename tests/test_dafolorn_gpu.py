@@ -167,7 +167,7 @@ def test_latent_attn(dtype, H, rank, vdim, window, bs, n_q, splits):
     tok = [s * n_q + k for s in range(S) for k in range(0, n_q, tpt)]
     cnt = [min(tpt, n_q - k) for s in range(S) for k in range(0, n_q, tpt)]
     out = torch.full((S * n_q, H * vdim), float("nan"), dtype=dt, device="cuda")
-    hip_ops.latent_attn(dev(q.reshape(S * n_q, H, rp)), dev(cache, dt), i32(tok), i32(cnt), tpt, i32(pos), i32(seq_of), i32(bt), rank, window, 1.0,
+    hip_ops.latent_attn(dev(q.reshape(S * n_q, H, rp)), dev(cache, dt), i32(tok), i32(cnt), tpt, i32(pos), i32(seq_of), i32(bt), window, 1.0,
                         dev(sink), dev(wuv), out, num_splits=splits)
     got = out.cpu().double().view(S, n_q, H, vdim)
     for s, n in enumerate(lens):
