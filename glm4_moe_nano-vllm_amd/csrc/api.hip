@@ -163,7 +163,8 @@ extern "C" int glm_gemm_bf16_act(const void* x, int64_t ldx, const void* w, int6
         const int rc = glm_launch_gemm_tinym(GEMM_PLAIN, p, 1, glm_s(stream));
         if (rc != GLM_ERR_UNSUPPORTED) return rc;
     }
-    if (M >= LARGEM_MIN_AVG_ROWS) return glm_launch_gemm_largem(GEMM_ACT, p, glm_s(stream));
+    // (a few hundred rows on a few columns, a router's logits: the tiled kernel would be a handful of workgroups)
+    if (M >= LARGEM_MIN_AVG_ROWS && !(N <= 256 && M < 1024)) return glm_launch_gemm_largem(GEMM_ACT, p, glm_s(stream));
     return glm_launch_gemm_smallm(GEMM_PLAIN, p, glm_s(stream));
 }
 

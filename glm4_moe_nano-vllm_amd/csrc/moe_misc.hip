@@ -639,52 +639,48 @@ __global__ __launch_bounds__(1024) void moe_align_scatter_kernel(
 
 // ------------------------------------------------------------------------------------------
 // Softmax router: from fp32 logits the k largest scores of softmax over all E experts, not renormalised, in fp32; one wave per token,
-// 64 EPL >= E.  Order: descending, ties to the lower index.
+// 64 EPL >= E.  Order: descending, ties to the lower index.  A lane counts how many logits are ahead of each of its own (they pass by in
+// LDS, four at a time): the count is the place in the order, nothing is searched for k times.  row: 64 EPL floats of this wave.
 template <int EPL>
-__device__ __forceinline__ void softmax_select_wave(const float* __restrict__ lg, int E, int k, int lane, int64_t* idx, float* w) {
+__device__ __forceinline__ void softmax_select_wave(const float* lg, int E, int k, int lane, float* row, int64_t* idx, float* w) {
     float v[EPL], m = -INFINITY, z = 0.f;
+    int ahead[EPL];
 #pragma unroll
     for (int i = 0; i < EPL; ++i) {
-        v[i] = lane + 64 * i < E ? lg[lane + 64 * i] : -INFINITY;
+        const int e = lane + 64 * i;
+        v[i] = e < E ? lg[e] : -INFINITY;
+        v[i] = v[i] == v[i] ? v[i] : -INFINITY;   // (not a number: behind all others)
+        row[e] = v[i];
+        ahead[i] = 0;
         m = fmaxf(m, v[i]);
     }
     m = wave_max(m);
 #pragma unroll
     for (int i = 0; i < EPL; ++i) z += lane + 64 * i < E ? expf(v[i] - m) : 0.f;
     const float inv = 1.0f / wave_sum(z);
-    for (int j = 0; j < k; ++j) {
-        float b = -INFINITY;
-        int e = 1 << 30;
+    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");   // the row is this wave's own
+    for (int e0 = 0; e0 < E; e0 += 4) {
+        const f32x4_t u = *reinterpret_cast<const f32x4_t*>(row + e0);
 #pragma unroll
         for (int i = 0; i < EPL; ++i)
-            if (v[i] > b) {
-                b = v[i];
-                e = lane + 64 * i;
-            }
 #pragma unroll
-        for (int o = 32; o > 0; o >>= 1) {
-            const float ob = __shfl_xor(b, o, 64);
-            const int oe = __shfl_xor(e, o, 64);
-            if (ob > b || (ob == b && oe < e)) {
-                b = ob;
-                e = oe;
-            }
-        }
-#pragma unroll
-        for (int i = 0; i < EPL; ++i)
-            if (lane + 64 * i == e) v[i] = -INFINITY;
-        if (lane == 0) {  // (no number among the logits: no expert, which the bucketing leaves out)
-            idx[j] = e < E ? e : -1;
-            w[j] = e < E ? expf(b - m) * inv : 0.f;
-        }
+            for (int j = 0; j < 4; ++j) ahead[i] += (u[j] > v[i] || (u[j] == v[i] && e0 + j < lane + 64 * i)) ? 1 : 0;
     }
+#pragma unroll
+    for (int i = 0; i < EPL; ++i)
+        if (lane + 64 * i < E && ahead[i] < k) {
+            idx[ahead[i]] = lane + 64 * i;
+            w[ahead[i]] = expf(v[i] - m) * inv;
+        }
+    asm volatile("" ::: "memory");   // the row is written again for the next token
 }
 
 template <int EPL>
 __global__ __launch_bounds__(256) void router_softmax_kernel(const float* __restrict__ logits, int64_t ld, int64_t* __restrict__ topk_idx,
                                                              float* __restrict__ topk_w, int64_t T, int E, int k) {
+    __shared__ __attribute__((aligned(16))) float rows[4][64 * EPL];
     const int64_t t = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (t < T) softmax_select_wave<EPL>(logits + t * ld, E, k, threadIdx.x & 63, topk_idx + t * k, topk_w + t * k);
+    if (t < T) softmax_select_wave<EPL>(logits + t * ld, E, k, threadIdx.x & 63, rows[threadIdx.x >> 6], topk_idx + t * k, topk_w + t * k);
 }
 
 // ... and the bucketing, for the few tokens of a decode step, by one workgroup
@@ -693,7 +689,9 @@ __global__ __launch_bounds__(1024) void router_softmax_align_kernel(const float*
                                                                     int32_t* sorted_token, int32_t* pair_pos, int64_t T, int E, int k) {
     __shared__ int cnt[ALIGN_MAX_G + 1];
     __shared__ int cur[ALIGN_MAX_G + 1];
-    for (int64_t t = threadIdx.x >> 6; t < T; t += 16) softmax_select_wave<EPL>(logits + t * ld, E, k, threadIdx.x & 63, topk_idx + t * k, topk_w + t * k);
+    __shared__ __attribute__((aligned(16))) float rows[16][64 * EPL];
+    const int wid = threadIdx.x >> 6;
+    for (int64_t t = wid; t < T; t += 16) softmax_select_wave<EPL>(logits + t * ld, E, k, threadIdx.x & 63, rows[wid], topk_idx + t * k, topk_w + t * k);
     __syncthreads();
     moe_align_body<false>(topk_idx, nullptr, expert_offsets, sorted_token, nullptr, pair_pos, T, k, E, 0, cnt, cur);
 }
@@ -1054,11 +1052,10 @@ extern "C" int glm_router_softmax_align(const float* logits, int64_t ld, int64_t
                                         int32_t* pair_pos, int64_t T, int E, int k, glm_stream_t stream) {
     GLM_CHECK_ARG(logits && topk_idx && topk_w && expert_offsets && sorted_token && pair_pos && T >= 0 && E > 0 && k > 0 && k <= E && ld >= E, GLM_ERR_INVALID,
                   "glm_router_softmax_align: bad shape T=%ld E=%d k=%d", (long)T, E, k);
-    GLM_CHECK_ARG(E < ALIGN_MAX_G && T * (int64_t)k < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_router_softmax_align: %d experts", E);
+    GLM_CHECK_ARG(E <= 256 && T * (int64_t)k < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_router_softmax_align: %d experts (256 at most; glm_router_softmax + glm_moe_align take more)", E);
     hipStream_t st = glm_s(stream);
     if (E <= 64) hipLaunchKernelGGL(router_softmax_align_kernel<1>, dim3(1), dim3(1024), 0, st, logits, ld, topk_idx, topk_w, expert_offsets, sorted_token, pair_pos, T, E, k);
-    else if (E <= 256) hipLaunchKernelGGL(router_softmax_align_kernel<4>, dim3(1), dim3(1024), 0, st, logits, ld, topk_idx, topk_w, expert_offsets, sorted_token, pair_pos, T, E, k);
-    else hipLaunchKernelGGL(router_softmax_align_kernel<16>, dim3(1), dim3(1024), 0, st, logits, ld, topk_idx, topk_w, expert_offsets, sorted_token, pair_pos, T, E, k);
+    else hipLaunchKernelGGL(router_softmax_align_kernel<4>, dim3(1), dim3(1024), 0, st, logits, ld, topk_idx, topk_w, expert_offsets, sorted_token, pair_pos, T, E, k);
     GLM_CHECK_LAUNCH("glm_router_softmax_align");
     return GLM_OK;
 }

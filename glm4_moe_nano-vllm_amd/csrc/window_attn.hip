@@ -39,7 +39,7 @@ struct WinArgs {
 
 // DK, DV: multiples of 64
 template <int DK, int DV>
-__global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void window_attn_kernel(const WinArgs a) {
+__global__ __launch_bounds__(256, (DK + DV) <= 320 ? 2 : 1) void window_attn_kernel(const WinArgs a) {
     constexpr int KS = DK / 32, VT = DV / 16;
     constexpr bool VEARLY = DK + DV <= 256;                      // V fragments requested in front of the score products
     constexpr int KG = KS < 4 ? KS : 4, VG = VEARLY ? VT : 4;    // fragments per request group

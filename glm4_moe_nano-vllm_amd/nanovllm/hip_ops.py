@@ -1863,7 +1863,7 @@ ROUTER_ALIGN_MAX_ROWS = 128   # rows up to which one workgroup routes and bucket
 def softmax_router_align(logits: torch.Tensor, E: int, k: int):
     """softmax_router and the bucketing of its pairs: (weights [T, k], offsets [E + 1], source rows [T k], pair positions [T k])."""
     T, dev = logits.shape[0], logits.device
-    if T > ROUTER_ALIGN_MAX_ROWS:
+    if T > ROUTER_ALIGN_MAX_ROWS or E > 256:
         idx, w = softmax_router(logits, E, k)
         offs, tok, _, pos = moe_align(idx, None, E, False)
         return w, offs, tok, pos
