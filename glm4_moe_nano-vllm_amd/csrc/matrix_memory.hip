@@ -109,15 +109,18 @@ __global__ __launch_bounds__(256 * NW) void memory_recurrent_kernel(const RecArg
     const int cb = tid >> 8, cq = tid & 15, rg = (tid >> 4) & 15, wv = (tid >> 6) & 3;
     const int seq = blockIdx.x / a.H, h = blockIdx.x % a.H;
     const int r0 = a.q_start[seq], r1 = a.q_start[seq + 1];
-    const int col = cb * 64 + cq * 4;
+    const int c0 = GATED ? 0 : blockIdx.y * 64 * NW;   // (no sum over a head's value columns: they are shared out)
+    const int col = c0 + cb * 64 + cq * 4;
     const bool con = col < a.vdimp;
     if (r1 <= r0) return;
     if (a.pos[r0] < 0) {  // unused rows of a padded batch
-        for (int r = r0; r < r1; ++r)
-            for (int c = tid; c < a.vdimp; c += NT) {
-                if constexpr (GATED) mm_st<T>(a.y, (int64_t)r * a.ldy + (int64_t)h * a.vdimp + c, 0.f);
-                else mm_st_o(a, r, h, c, 0.f);
+        for (int r = r0; r < r1; ++r) {
+            if constexpr (GATED) {
+                for (int c = tid; c < a.vdimp; c += NT) mm_st<T>(a.y, (int64_t)r * a.ldy + (int64_t)h * a.vdimp + c, 0.f);
+            } else if (tid < 64 * NW && c0 + tid < a.vdimp) {
+                mm_st_o(a, r, h, c0 + tid, 0.f);
             }
+        }
         return;
     }
     f32x4_t S[KD];
@@ -197,7 +200,7 @@ __global__ __launch_bounds__(256 * NW) void memory_recurrent_kernel(const RecArg
         }
         __syncthreads();
         if constexpr (!GATED) {  // (s_o is written again behind the next token's first barrier)
-            if (tid < a.vdimp) mm_st_o(a, r, h, tid, (s_o[tid >> 6][0][tid & 63] + s_o[tid >> 6][1][tid & 63]) + (s_o[tid >> 6][2][tid & 63] + s_o[tid >> 6][3][tid & 63]));
+            if (tid < 64 * NW && c0 + tid < a.vdimp) mm_st_o(a, r, h, c0 + tid, (s_o[tid >> 6][0][tid & 63] + s_o[tid >> 6][1][tid & 63]) + (s_o[tid >> 6][2][tid & 63] + s_o[tid >> 6][3][tid & 63]));
             continue;
         }
 #pragma unroll
@@ -890,53 +893,84 @@ __global__ __launch_bounds__(256) void memory_output_kernel(const OutArgs a) {
     }
 }
 
-// y = o / rms(o) . norm . gate over whole rows, one wave per row; n: true number of columns (padding columns of o are zeros)
+// y = o / rms(o) . norm . gate over whole rows, one row per workgroup, eight columns per thread and round (two rounds stay in registers); n: true
+// number of columns (padding columns of o are zeros)
 template <typename O, typename Y>
-__global__ __launch_bounds__(256) void row_norm_gate_kernel(const O* __restrict__ o, int64_t ldo, const Y* __restrict__ gate, int64_t ldg, const float* __restrict__ norm,
-                                                            Y* __restrict__ y, int64_t ldy, int64_t T, int n, int np, float eps) {
-    const int lane = threadIdx.x & 63;
-    const int64_t r = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (r >= T) return;
+__global__ __launch_bounds__(1024) void row_norm_gate_kernel(const O* __restrict__ o, int64_t ldo, const Y* __restrict__ gate, int64_t ldg, const float* __restrict__ norm,
+                                                             Y* __restrict__ y, int64_t ldy, int n, int np, float eps) {
+    __shared__ float s_red[16];
+    const int tid = threadIdx.x, nt = blockDim.x;
+    const int64_t r = blockIdx.x;
+    f32x4_t u[2][2], g[2][2], w[2][2];
     float sq = 0.f;
-    f32x4_t u[2][2];  // up to 1024 columns stay in registers
-    for (int c = lane * 8, i = 0; c < np; c += 512, ++i) {
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+        const int c = (tid + i * nt) * 8;
+#pragma unroll
+        for (int hf = 0; hf < 2; ++hf) {
+            u[i][hf] = g[i][hf] = w[i][hf] = f32x4_t{0.f, 0.f, 0.f, 0.f};
+            if (c < np) {
+                u[i][hf] = mm_ld4<O>(o, r * ldo + c + 4 * hf);
+                g[i][hf] = mm_ld4<Y>(gate, r * ldg + c + 4 * hf);
+                w[i][hf] = *reinterpret_cast<const f32x4_t*>(norm + c + 4 * hf);
+            }
+        }
+#pragma unroll
+        for (int e = 0; e < 4; ++e) sq += u[i][0][e] * u[i][0][e] + u[i][1][e] * u[i][1][e];
+    }
+    for (int c = (tid + 2 * nt) * 8; c < np; c += nt * 8) {
         const f32x4_t a = mm_ld4<O>(o, r * ldo + c), b = mm_ld4<O>(o, r * ldo + c + 4);
 #pragma unroll
         for (int e = 0; e < 4; ++e) sq += a[e] * a[e] + b[e] * b[e];
-        if (i < 2) {
-            if (i == 0) { u[0][0] = a; u[0][1] = b; } else { u[1][0] = a; u[1][1] = b; }
+    }
+    sq = wave_sum(sq);
+    if ((tid & 63) == 0) s_red[tid >> 6] = sq;
+    __syncthreads();
+    sq = 0.f;
+    for (int i = 0; i < nt / 64; ++i) sq += s_red[i];
+    const float inv = 1.0f / sqrtf(sq / (float)n + eps);
+    auto put = [&](int c, f32x4_t v, const f32x4_t& gv, const f32x4_t& wv) {
+#pragma unroll
+        for (int e = 0; e < 4; ++e) v[e] = v[e] * inv * wv[e] * gv[e];
+        if constexpr (sizeof(Y) == 4) *reinterpret_cast<f32x4_t*>(y + r * ldy + c) = v;
+        else *reinterpret_cast<u32x2_t*>(y + r * ldy + c) = u32x2_t{pack2bf(v[0], v[1]), pack2bf(v[2], v[3])};
+    };
+#pragma unroll
+    for (int i = 0; i < 2; ++i) {
+        const int c = (tid + i * nt) * 8;
+        if (c < np) {
+            put(c, u[i][0], g[i][0], w[i][0]);
+            put(c + 4, u[i][1], g[i][1], w[i][1]);
         }
     }
-    const float inv = 1.0f / sqrtf(wave_sum(sq) / (float)n + eps);
-    for (int c = lane * 8, i = 0; c < np; c += 512, ++i) {
+    for (int c = (tid + 2 * nt) * 8; c < np; c += nt * 8)
 #pragma unroll
-        for (int hlf = 0; hlf < 2; ++hlf) {
-            f32x4_t v = i == 0 ? u[0][hlf] : i == 1 ? u[1][hlf] : mm_ld4<O>(o, r * ldo + c + 4 * hlf);
-            const f32x4_t g = mm_ld4<Y>(gate, r * ldg + c + 4 * hlf), w = *reinterpret_cast<const f32x4_t*>(norm + c + 4 * hlf);
-#pragma unroll
-            for (int e = 0; e < 4; ++e) v[e] = v[e] * inv * w[e] * g[e];
-            if constexpr (sizeof(Y) == 4) *reinterpret_cast<f32x4_t*>(y + r * ldy + c + 4 * hlf) = v;
-            else *reinterpret_cast<u32x2_t*>(y + r * ldy + c + 4 * hlf) = u32x2_t{pack2bf(v[0], v[1]), pack2bf(v[2], v[3])};
-        }
-    }
+        for (int hf = 0; hf < 2; ++hf)
+            put(c + 4 * hf, mm_ld4<O>(o, r * ldo + c + 4 * hf), mm_ld4<Y>(gate, r * ldg + c + 4 * hf), *reinterpret_cast<const f32x4_t*>(norm + c + 4 * hf));
 }
 
 template <typename T, int KD, int NW>
 int launch_rec(const RecArgs& a, hipStream_t st) {
-    if (a.decay) hipLaunchKernelGGL((memory_recurrent_kernel<T, KD, NW, false>), dim3((unsigned)(a.seqs * a.H)), dim3(256 * NW), 0, st, a);
-    else hipLaunchKernelGGL((memory_recurrent_kernel<T, KD, NW, true>), dim3((unsigned)(a.seqs * a.H)), dim3(256 * NW), 0, st, a);
+    if constexpr (NW == 1) {
+        if (a.decay) {
+            hipLaunchKernelGGL((memory_recurrent_kernel<T, KD, 1, false>), dim3((unsigned)(a.seqs * a.H), (unsigned)((a.vdimp + 63) / 64)), dim3(256), 0, st, a);
+            GLM_CHECK_LAUNCH("glm_linear_recurrent");
+            return GLM_OK;
+        }
+    }
+    hipLaunchKernelGGL((memory_recurrent_kernel<T, KD, NW, true>), dim3((unsigned)(a.seqs * a.H)), dim3(256 * NW), 0, st, a);
     GLM_CHECK_LAUNCH("glm_memory_recurrent");
     return GLM_OK;
 }
 template <typename T, int KD>
 int launch_rec_v(const RecArgs& a, hipStream_t st) {
-    if (a.vdimp <= 64) return launch_rec<T, KD, 1>(a, st);
+    if (a.vdimp <= 64 || a.decay) return launch_rec<T, KD, 1>(a, st);
     if (a.vdimp <= 128) return launch_rec<T, KD, 2>(a, st);
     return launch_rec<T, KD, 4>(a, st);
 }
 template <typename T>
 int run_rec(const RecArgs& a, hipStream_t st) {
-    if (a.dimp <= 256 && a.vdimp <= 256) {
+    if (a.dimp <= 256 && (a.vdimp <= 256 || (a.decay && a.vdimp <= 65535 * 64))) {
         if (a.dimp <= 64) return launch_rec_v<T, 4>(a, st);
         if (a.dimp <= 128) return launch_rec_v<T, 8>(a, st);
         return launch_rec_v<T, 16>(a, st);
@@ -1057,13 +1091,16 @@ extern "C" int glm_row_norm_gate(const void* o, int64_t ldo, int o_f32, const vo
     GLM_CHECK_ARG(o && gate && norm && y && T >= 0 && n > 0 && np >= n && np % 8 == 0 && ldo >= np && ldg >= np && ldy >= np && ldo % 8 == 0 && ldg % 8 == 0 && ldy % 8 == 0 &&
                       glm_aligned16(o) && glm_aligned16(gate) && glm_aligned16(norm) && glm_aligned16(y) && (o_f32 || !act_f32), GLM_ERR_INVALID,
                   "glm_row_norm_gate: bad shape T=%ld n=%d np=%d", (long)T, n, np);
-    GLM_CHECK_ARG((T + 3) / 4 < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_row_norm_gate: too many rows");
+    GLM_CHECK_ARG(T < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_row_norm_gate: too many rows");
     if (T == 0) return GLM_OK;
-    const dim3 grid((unsigned)((T + 3) / 4));
+    const dim3 grid((unsigned)T);
+    int nt = (np / 8 + 63) / 64 * 64;   // (many rows: half as many threads, two rounds each)
+    if (T > 1024 && nt > 64) nt = (nt / 2 + 63) / 64 * 64;
+    nt = nt > 1024 ? 1024 : nt;
     hipStream_t st = glm_s(stream);
-    if (act_f32) hipLaunchKernelGGL((row_norm_gate_kernel<float, float>), grid, dim3(256), 0, st, (const float*)o, ldo, (const float*)gate, ldg, norm, (float*)y, ldy, T, n, np, eps);
-    else if (o_f32) hipLaunchKernelGGL((row_norm_gate_kernel<float, bf16_t>), grid, dim3(256), 0, st, (const float*)o, ldo, (const bf16_t*)gate, ldg, norm, (bf16_t*)y, ldy, T, n, np, eps);
-    else hipLaunchKernelGGL((row_norm_gate_kernel<bf16_t, bf16_t>), grid, dim3(256), 0, st, (const bf16_t*)o, ldo, (const bf16_t*)gate, ldg, norm, (bf16_t*)y, ldy, T, n, np, eps);
+    if (act_f32) hipLaunchKernelGGL((row_norm_gate_kernel<float, float>), grid, dim3(nt), 0, st, (const float*)o, ldo, (const float*)gate, ldg, norm, (float*)y, ldy, n, np, eps);
+    else if (o_f32) hipLaunchKernelGGL((row_norm_gate_kernel<float, bf16_t>), grid, dim3(nt), 0, st, (const float*)o, ldo, (const bf16_t*)gate, ldg, norm, (bf16_t*)y, ldy, n, np, eps);
+    else hipLaunchKernelGGL((row_norm_gate_kernel<bf16_t, bf16_t>), grid, dim3(nt), 0, st, (const bf16_t*)o, ldo, (const bf16_t*)gate, ldg, norm, (bf16_t*)y, ldy, n, np, eps);
     GLM_CHECK_LAUNCH("glm_row_norm_gate");
     return GLM_OK;
 }

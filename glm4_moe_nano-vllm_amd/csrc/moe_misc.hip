@@ -639,61 +639,113 @@ __global__ __launch_bounds__(1024) void moe_align_scatter_kernel(
 
 // ------------------------------------------------------------------------------------------
 // Softmax router: from fp32 logits the k largest scores of softmax over all E experts, not renormalised, in fp32; one wave per token,
-// 64 EPL >= E.  Order: descending, ties to the lower index.  A lane counts how many logits are ahead of each of its own (they pass by in
-// LDS, four at a time): the count is the place in the order, nothing is searched for k times.  row: 64 EPL floats of this wave.
+// 64 EPL >= E.  Order: descending, ties to the lower index.  Maxima and sums over the wave run on DPP row shifts, the place of a maximum
+// is a ballot.  put(j, expert, weight) is called by all lanes.
+__device__ __forceinline__ float dpp_max(float v) {  // the maximum over the wave, in lane 63
+#define GLM_DPP_MAX(CTRL, ROWS) v = fmaxf(v, __int_as_float(__builtin_amdgcn_update_dpp(__float_as_int(v), __float_as_int(v), CTRL, ROWS, 0xf, false)));
+    GLM_DPP_MAX(0x111, 0xf) GLM_DPP_MAX(0x112, 0xf) GLM_DPP_MAX(0x114, 0xf) GLM_DPP_MAX(0x118, 0xf) GLM_DPP_MAX(0x142, 0xa) GLM_DPP_MAX(0x143, 0xc)
+#undef GLM_DPP_MAX
+    return __int_as_float(__builtin_amdgcn_readlane(__float_as_int(v), 63));
+}
 template <int EPL>
-__device__ __forceinline__ void softmax_select_wave(const float* lg, int E, int k, int lane, float* row, int64_t* idx, float* w) {
-    float v[EPL], m = -INFINITY, z = 0.f;
-    int ahead[EPL];
+__device__ __forceinline__ void load_logits(const float* lg, int E, int lane, float (&v)[EPL]) {
+#pragma unroll
+    for (int i = 0; i < EPL; ++i) v[i] = lane + 64 * i < E ? lg[lane + 64 * i] : -INFINITY;
+}
+template <int EPL, class Put>
+__device__ __forceinline__ void softmax_select_wave(float (&v)[EPL], int E, int k, int lane, Put put) {
+    float z = 0.f, m = -INFINITY;
+    bool there[EPL];
 #pragma unroll
     for (int i = 0; i < EPL; ++i) {
-        const int e = lane + 64 * i;
-        v[i] = e < E ? lg[e] : -INFINITY;
-        v[i] = v[i] == v[i] ? v[i] : -INFINITY;   // (not a number: behind all others)
-        row[e] = v[i];
-        ahead[i] = 0;
+        there[i] = lane + 64 * i < E;
         m = fmaxf(m, v[i]);
     }
-    m = wave_max(m);
+    m = dpp_max(m);
 #pragma unroll
-    for (int i = 0; i < EPL; ++i) z += lane + 64 * i < E ? expf(v[i] - m) : 0.f;
+    for (int i = 0; i < EPL; ++i) z += there[i] ? expf(v[i] - m) : 0.f;
     const float inv = 1.0f / wave_sum(z);
-    asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");   // the row is this wave's own
-    for (int e0 = 0; e0 < E; e0 += 4) {
-        const f32x4_t u = *reinterpret_cast<const f32x4_t*>(row + e0);
+    for (int j = 0; j < k; ++j) {
+        float b = -INFINITY;
+#pragma unroll
+        for (int i = 0; i < EPL; ++i) b = there[i] ? fmaxf(b, v[i]) : b;
+        b = dpp_max(b);
+        int e = -1;   // (only numbers are found: without one among the logits there is no expert, which the bucketing leaves out)
+#pragma unroll
+        for (int i = EPL - 1; i >= 0; --i) {
+            const unsigned long long at = __ballot(there[i] && v[i] == b);
+            if (at) e = 64 * i + __builtin_ctzll(at);
+        }
 #pragma unroll
         for (int i = 0; i < EPL; ++i)
-#pragma unroll
-            for (int j = 0; j < 4; ++j) ahead[i] += (u[j] > v[i] || (u[j] == v[i] && e0 + j < lane + 64 * i)) ? 1 : 0;
+            if (lane + 64 * i == e) there[i] = false;
+        put(j, e, e < 0 ? 0.f : expf(b - m) * inv);
     }
-#pragma unroll
-    for (int i = 0; i < EPL; ++i)
-        if (lane + 64 * i < E && ahead[i] < k) {
-            idx[ahead[i]] = lane + 64 * i;
-            w[ahead[i]] = expf(v[i] - m) * inv;
-        }
-    asm volatile("" ::: "memory");   // the row is written again for the next token
 }
 
 template <int EPL>
 __global__ __launch_bounds__(256) void router_softmax_kernel(const float* __restrict__ logits, int64_t ld, int64_t* __restrict__ topk_idx,
                                                              float* __restrict__ topk_w, int64_t T, int E, int k) {
-    __shared__ __attribute__((aligned(16))) float rows[4][64 * EPL];
     const int64_t t = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
-    if (t < T) softmax_select_wave<EPL>(logits + t * ld, E, k, threadIdx.x & 63, rows[threadIdx.x >> 6], topk_idx + t * k, topk_w + t * k);
+    if (t >= T) return;
+    const int lane = threadIdx.x & 63;
+    float v[EPL];
+    load_logits<EPL>(logits + t * ld, E, lane, v);
+    softmax_select_wave<EPL>(v, E, k, lane, [&](int j, int e, float w) {
+        if (lane == 0) {
+            topk_idx[t * k + j] = e;
+            topk_w[t * k + j] = w;
+        }
+    });
 }
 
-// ... and the bucketing, for the few tokens of a decode step, by one workgroup
+// ... and the bucketing, for the few tokens of a decode step, by one workgroup: a pair's place inside its expert's group is what its count
+// of the expert returned
+constexpr int ROUTER_ALIGN_PAIRS = 1024;
 template <int EPL>
 __global__ __launch_bounds__(1024) void router_softmax_align_kernel(const float* logits, int64_t ld, int64_t* topk_idx, float* topk_w, int32_t* expert_offsets,
-                                                                    int32_t* sorted_token, int32_t* pair_pos, int64_t T, int E, int k) {
-    __shared__ int cnt[ALIGN_MAX_G + 1];
-    __shared__ int cur[ALIGN_MAX_G + 1];
-    __shared__ __attribute__((aligned(16))) float rows[16][64 * EPL];
-    const int wid = threadIdx.x >> 6;
-    for (int64_t t = wid; t < T; t += 16) softmax_select_wave<EPL>(logits + t * ld, E, k, threadIdx.x & 63, rows[wid], topk_idx + t * k, topk_w + t * k);
+                                                                    int32_t* sorted_token, int32_t* pair_pos, int T, int E, int k) {
+    __shared__ int cnt[64 * EPL], off[64 * EPL], s_e[ROUTER_ALIGN_PAIRS], s_r[ROUTER_ALIGN_PAIRS];
+    const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
+    if (tid < 64 * EPL) cnt[tid] = 0;
     __syncthreads();
-    moe_align_body<false>(topk_idx, nullptr, expert_offsets, sorted_token, nullptr, pair_pos, T, k, E, 0, cnt, cur);
+    for (int t0 = wid; t0 < T; t0 += 64) {   // four tokens of this wave, their logits together
+        float v[4][EPL];
+#pragma unroll
+        for (int u = 0; u < 4; ++u) load_logits<EPL>(logits + (int64_t)min(t0 + 16 * u, T - 1) * ld, E, lane, v[u]);
+#pragma unroll
+        for (int u = 0; u < 4; ++u) {
+            const int t = t0 + 16 * u;
+            if (t >= T) break;
+            softmax_select_wave<EPL>(v[u], E, k, lane, [&](int j, int e, float w) {
+                if (lane == 0) {
+                    const int p = t * k + j;
+                    topk_idx[p] = e;
+                    topk_w[p] = w;
+                    s_e[p] = e;
+                    s_r[p] = e >= 0 ? atomicAdd(&cnt[e], 1) : 0;
+                }
+            });
+        }
+    }
+    __syncthreads();
+    if (wid == 0) {
+        int run = 0;
+#pragma unroll
+        for (int i = 0; i < EPL; ++i) {
+            const int e = lane + 64 * i, c = cnt[e], incl = wave_scan_incl(c);
+            off[e] = run + incl - c;
+            if (e < E) expert_offsets[e] = run + incl - c;
+            run += __builtin_amdgcn_readlane(incl, 63);
+        }
+        if (lane == 0) expert_offsets[E] = run;
+    }
+    __syncthreads();
+    for (int p = tid; p < T * k; p += 1024) {
+        const int e = s_e[p], pos = e >= 0 ? off[e] + s_r[p] : -1;
+        pair_pos[p] = pos;
+        if (pos >= 0) sorted_token[pos] = p / k;
+    }
 }
 
 // out[t] = sum_j w[t, j] y[pair_pos[t, j]], fp32 sum
@@ -1052,10 +1104,11 @@ extern "C" int glm_router_softmax_align(const float* logits, int64_t ld, int64_t
                                         int32_t* pair_pos, int64_t T, int E, int k, glm_stream_t stream) {
     GLM_CHECK_ARG(logits && topk_idx && topk_w && expert_offsets && sorted_token && pair_pos && T >= 0 && E > 0 && k > 0 && k <= E && ld >= E, GLM_ERR_INVALID,
                   "glm_router_softmax_align: bad shape T=%ld E=%d k=%d", (long)T, E, k);
-    GLM_CHECK_ARG(E <= 256 && T * (int64_t)k < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_router_softmax_align: %d experts (256 at most; glm_router_softmax + glm_moe_align take more)", E);
+    GLM_CHECK_ARG(E <= 256 && T * (int64_t)k <= ROUTER_ALIGN_PAIRS, GLM_ERR_UNSUPPORTED, "glm_router_softmax_align: %ld pairs, %d experts (%d and 256 at most; glm_router_softmax + glm_moe_align take more)", (long)(T * k), E, ROUTER_ALIGN_PAIRS);
+    if (T == 0) return GLM_OK;
     hipStream_t st = glm_s(stream);
-    if (E <= 64) hipLaunchKernelGGL(router_softmax_align_kernel<1>, dim3(1), dim3(1024), 0, st, logits, ld, topk_idx, topk_w, expert_offsets, sorted_token, pair_pos, T, E, k);
-    else hipLaunchKernelGGL(router_softmax_align_kernel<4>, dim3(1), dim3(1024), 0, st, logits, ld, topk_idx, topk_w, expert_offsets, sorted_token, pair_pos, T, E, k);
+    if (E <= 64) hipLaunchKernelGGL(router_softmax_align_kernel<1>, dim3(1), dim3(1024), 0, st, logits, ld, topk_idx, topk_w, expert_offsets, sorted_token, pair_pos, (int)T, E, k);
+    else hipLaunchKernelGGL(router_softmax_align_kernel<4>, dim3(1), dim3(1024), 0, st, logits, ld, topk_idx, topk_w, expert_offsets, sorted_token, pair_pos, (int)T, E, k);
     GLM_CHECK_LAUNCH("glm_router_softmax_align");
     return GLM_OK;
 }

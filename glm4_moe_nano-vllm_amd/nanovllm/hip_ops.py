@@ -1857,13 +1857,13 @@ def softmax_router(logits: torch.Tensor, E: int, k: int):
     return idx, w
 
 
-ROUTER_ALIGN_MAX_ROWS = 128   # rows up to which one workgroup routes and buckets them
+ROUTER_ALIGN_MAX_ROWS = 64    # rows up to which one workgroup routes and buckets them (1024 pairs at most)
 
 
 def softmax_router_align(logits: torch.Tensor, E: int, k: int):
     """softmax_router and the bucketing of its pairs: (weights [T, k], offsets [E + 1], source rows [T k], pair positions [T k])."""
     T, dev = logits.shape[0], logits.device
-    if T > ROUTER_ALIGN_MAX_ROWS or E > 256:
+    if T > ROUTER_ALIGN_MAX_ROWS or E > 256 or T * k > 1024:
         idx, w = softmax_router(logits, E, k)
         offs, tok, _, pos = moe_align(idx, None, E, False)
         return w, offs, tok, pos

@@ -618,7 +618,7 @@ int glm_depth_norm(const float* x_in, const int32_t* row_index, int64_t ld, cons
                    int64_t T, int width, int wp, int groups, float eps, glm_stream_t stream);
 
 /* Softmax router: the k largest of softmax(logits) over E experts, fp32 weights, not renormalised; descending.  _align: and the bucketing
- * of glm_moe_align (no shared group, no scales) in one launch, for few tokens and E <= 256.  combine_weighted: out[t] = sum_j w[t,j] y[pair_pos[t,j]]. */
+ * of glm_moe_align (no shared group, no scales) in one launch, for few tokens (T k <= 1024, E <= 256).  combine_weighted: out[t] = sum_j w[t,j] y[pair_pos[t,j]]. */
 int glm_router_softmax(const float* logits, int64_t ld, int64_t* topk_idx, float* topk_w, int64_t T, int E, int k, glm_stream_t stream);
 int glm_router_softmax_align(const float* logits, int64_t ld, int64_t* topk_idx, float* topk_w, int32_t* expert_offsets,
                              int32_t* sorted_token, int32_t* pair_pos, int64_t T, int E, int k, glm_stream_t stream);
