@@ -101,7 +101,7 @@ __device__ __forceinline__ void mm_st_o(const RecArgs& a, int64_t r, int h, int 
 // dimp <= 16 KD, vdimp <= 64 NW.  256 NW threads: column block tid / 256 (64 columns), thread (rg, cq) of a block holds rows rg + 16 k of the
 // four columns cq.
 template <typename T, int KD, int NW, bool GATED>
-__global__ __launch_bounds__(256 * NW) void memory_recurrent_kernel(const RecArgs a) {
+__global__ __launch_bounds__(256 * NW, GATED ? 1 : KD <= 8 ? 6 : 4) void memory_recurrent_kernel(const RecArgs a) {
     constexpr int NT = 256 * NW, NWV = 4 * NW;
     __shared__ float s_q[16 * KD], s_k[16 * KD], s_g[2][NWV], s_nq[NWV], s_ss[NWV];
     __shared__ __attribute__((aligned(16))) float s_o[NW][4][64];
