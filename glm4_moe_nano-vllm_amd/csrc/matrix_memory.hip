@@ -431,6 +431,7 @@ __global__ __launch_bounds__(256) void memory_gates_kernel(const GateArgs a) {
     }
 }
 
+constexpr int MM_MAX_SEG = 8;
 struct ChunkArgs {
     const bf16_t* x;      // projection rows (see RecArgs)
     int64_t ldx, k_off, v_off;
@@ -443,6 +444,7 @@ struct ChunkArgs {
     const int32_t *pos, *q_start, *state_in, *state_out;  // of the long portions; q_start and pos relative to x's first row
     int H, dim, dimp, vdimp, vtiles;
     const float* powers;  // [H][65] decay^j: the linear memory
+    float seg[MM_MAX_SEG + 1];  // where its segments begin, as parts of a sequence
 };
 
 template <typename T>
@@ -518,7 +520,15 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
     const int vt = blockIdx.x % a.vtiles, h = (blockIdx.x / a.vtiles) % a.H, seq = blockIdx.x / (a.vtiles * a.H);
     const int r0 = a.q_start[seq], T = a.q_start[seq + 1] - r0;
     if (T <= 0) return;
-    const int n_chunks = (T + 63) >> 6;
+    // chunks [ch0, n_chunks) are this workgroup's.  The linear memory's few (sequence, head) pairs are cut into segments: a workgroup brings the
+    // state up to its segment by itself, which costs a fraction of a chunk's work (no scores, no readout)
+    int n_chunks = (T + 63) >> 6, ch0 = 0;
+    const bool keeps = GATED || blockIdx.y + 1 == gridDim.y;
+    if constexpr (!GATED) {
+        ch0 = (int)((float)n_chunks * a.seg[blockIdx.y]);
+        if (!keeps) n_chunks = (int)((float)n_chunks * a.seg[blockIdx.y + 1]);
+        if (ch0 >= n_chunks) return;
+    }
     const bool fresh = a.pos[r0] <= 0;
     const int64_t sin = min(max((int64_t)a.state_in[seq], (int64_t)0), a.n_state - 1) * a.H + h;
     const int col = vt * 64 + 16 * v + c;  // this lane's value column
@@ -581,10 +591,11 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
         // gates: i - b, b and the running maximum, 256 bytes each (the other waves' piece is not used)
         if constexpr (GATED) __builtin_amdgcn_global_load_lds((attn_glb_void*)(gp + min(w, 2) * gpart + ch * 64 + min(lane, left - 1)), (attn_lds_void*)(st + 2 * QT + VTB + min(w, 3) * 256), 4, 0, 0);
         const bf16_t *q = xq + (int64_t)ch * 64 * a.ldx, *k = q + a.k_off, *vv = xv + (int64_t)ch * 64 * a.ldx;
+        const bool full = GATED || ch >= ch0;
         if (whole && left >= 64) {
 #pragma unroll
             for (int i = 0; i < QDMA; ++i) {
-                lds_dma16(q + qoff[i], st + (w * QDMA + i) * 1024);
+                if (full) lds_dma16(q + qoff[i], st + (w * QDMA + i) * 1024);
                 lds_dma16(k + qoff[i], st + QT + (w * QDMA + i) * 1024);
             }
             lds_dma16(vv + voff, st + 2 * QT + w * 1024);
@@ -594,7 +605,7 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
         for (int i = 0; i < QDMA; ++i) {
             const int p = (w * QDMA + i) * 64 + lane, row = p / CPR, cc = (p % CPR) ^ attn_swz(row);
             const bool ok = row < left && cc * 8 < a.dimp;
-            lds_dma16(ok ? (const void*)(q + qoff[i]) : (const void*)mm_zero_page, st + (w * QDMA + i) * 1024);
+            if (full) lds_dma16(ok ? (const void*)(q + qoff[i]) : (const void*)mm_zero_page, st + (w * QDMA + i) * 1024);
             lds_dma16(ok ? (const void*)(k + qoff[i]) : (const void*)mm_zero_page, st + QT + (w * QDMA + i) * 1024);
         }
         const bool ok = vrow < left && vt * 64 + vcc * 8 < a.vdimp;
@@ -631,10 +642,12 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
     for (int ch = 0; ch < n_chunks; ++ch) {
         const int left = T - ch * 64;
         // the chunk is in (what was issued behind it may be on its way): loads return in order
-        if (ch + NST - 2 < n_chunks) wait_vm<(NST - 2) * (2 * QDMA + (GATED ? 2 : 1))>();
-        else wait_vm<0>();
+        const bool full = GATED || ch >= ch0;
+        if (ch + NST - 2 >= n_chunks) wait_vm<0>();
+        else if (GATED || ch + NST - 2 >= ch0) wait_vm<(NST - 2) * (2 * QDMA + (GATED ? 2 : 1))>();
+        else wait_vm<(NST - 2) * (QDMA + 1)>();
         mm_barrier();  // ... for every wave, and every wave is past its reads of the chunk before
-        if (ch > 0) store_rows(ch - 1);
+        if (ch > ch0) store_rows(ch - 1);
         if (ch + NST - 1 < n_chunks) issue(ch + NST - 1);
         const char *qst = smem + (ch % NST) * STAGE, *kst = qst + QT, *vst = kst + QT, *gst = vst + VTB;
         char *pst = smem + (PALIAS ? (ch % NST) * STAGE : POFF), *xst = smem + (XALIAS ? (ch % NST) * STAGE : 0) + XOFF;
@@ -662,7 +675,7 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
         // ---- scores of 16 query rows with 32 keys; n . q of these rows, over this half's d ----
         f32x4_t s[2] = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
         float nq = 0.f;
-        static_for<KS>([&](auto I) {
+        if (full) static_for<KS>([&](auto I) {
             constexpr int i = decltype(I)::value;
             const u32x4_t qf = mm_lds<u32x4_t>(qst + v * 16 * RB + row_rel[i & 1] + (i >> 1) * 128);
             const u32x4_t k0 = mm_lds<u32x4_t>(kst + dh * 32 * RB + row_rel[i & 1] + (i >> 1) * 128), k1 = mm_lds<u32x4_t>(kst + dh * 32 * RB + row_rel[i & 1] + (i >> 1) * 128 + 16 * RB);
@@ -684,7 +697,7 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
 #pragma unroll
         for (int rt = 0; rt < 4; ++rt) acc[rt] = f32x4_t{0.f, 0.f, 0.f, 0.f};
         const char* qh_st = qst + (KS / 2 >= 2 ? dh * (KS / 4) * 128 : 0);   // columns of this half: 128 bytes hold 64 of them
-        static_for<KS / 2>([&](auto I) {
+        if (full) static_for<KS / 2>([&](auto I) {
             constexpr int i = decltype(I)::value;
             const unsigned ra = KS / 2 >= 2 ? half_rel[i & 1][0] : (dh ? half_rel[1][0] : half_rel[0][0]), rb = KS / 2 >= 2 ? half_rel[i & 1][1] : (dh ? half_rel[1][1] : half_rel[0][1]);
             const f32x4_t &u = S[2 * i], &x = S[2 * i + 1];
@@ -703,12 +716,12 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
         // ---- operands of the state's update: values over tokens ----
         u32x2_t vf[2][2];
         mm_lds_tr4<0, 16 * 128, 32 * 128, 48 * 128>(vf, vst + vt_rel);
-        mm_barrier();  // query rows read, gate arrays written
+        if (full) mm_barrier();  // query rows read, gate arrays written
         const bf16x8_t vv[2] = {mm_frag(vf[0][0], vf[0][1]), mm_frag(vf[1][0], vf[1][1])};
         // ---- weights of this wave's rows and keys: hi and lo, in the order the second product reads them ----
         const int row = 16 * v + c;
         const float rowc = GATED ? mm_lds<float>(sa + 256 + 4 * row) : 0.f, inc = GATED ? mm_lds<float>(sa + 512 + 4 * row) : 0.f;
-        {
+        if (full) {
             *reinterpret_cast<f32x4_t*>(xst + (w * 2 * 64 + lane) * 16) = x_a;
             *reinterpret_cast<f32x4_t*>(xst + ((w * 2 + 1) * 64 + lane) * 16) = x_b;
             float p[8], dsum = 0.f;
@@ -797,6 +810,7 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
             nn += __shfl_xor(nn, 32, 64);
             nreg[i0 >> 2] = fmaf(carry, nreg[i0 >> 2], nn);
         });
+        if (!full) continue;
         mm_barrier();
         // ---- output rows ----
         if (GATED && g == 0 && v < HT) {
@@ -830,7 +844,7 @@ __global__ __launch_bounds__(512, 2) void memory_chunkwise_kernel(const ChunkArg
     }
     store_rows(n_chunks - 1);
     const int64_t so = a.state_out[seq];
-    if (so < 0 || so >= a.n_state) return;
+    if (!keeps || so < 0 || so >= a.n_state) return;
     const int64_t sout = so * a.H + h;
 #pragma unroll
     for (int i = 0; i < HT; ++i)
@@ -984,13 +998,13 @@ int run_rec(const RecArgs& a, hipStream_t st) {
 }
 
 template <int D, bool GATED>
-int launch_chunk(const ChunkArgs& a, int seqs, hipStream_t st) {
+int launch_chunk(const ChunkArgs& a, int seqs, int nseg, hipStream_t st) {
     constexpr int QT = 64 * D * 2, STAGE = 2 * QT + 8192 + 1024;
     constexpr int LDS = (D <= 128 ? 3 : 2) * STAGE + (QT >= 16384 ? 0 : 16384) + (QT >= 32768 ? 0 : 16384) + 7 * 256 + D * 4;
     static_assert(LDS <= 160 * 1024, "LDS of a CU");
     auto kern = memory_chunkwise_kernel<D, GATED>;
     GLM_SET_MAX_LDS(kern, LDS, "glm_memory_chunkwise");
-    hipLaunchKernelGGL(kern, dim3((unsigned)(seqs * a.H * a.vtiles)), dim3(512), LDS, st, a);
+    hipLaunchKernelGGL(kern, dim3((unsigned)(seqs * a.H * a.vtiles), (unsigned)nseg), dim3(512), LDS, st, a);
     GLM_CHECK_LAUNCH("glm_memory_chunkwise");
     return GLM_OK;
 }
@@ -1033,12 +1047,12 @@ extern "C" int glm_memory_chunkwise(const void* x, int64_t ldx, int64_t k_off, i
                       glm_aligned16(x) && (((uintptr_t)o) & 7) == 0, GLM_ERR_INVALID, "glm_memory_chunkwise: bad shape H=%d dim=%d vdimp=%d ldx=%ld", H, dim, vdimp, (long)ldx);
     GLM_CHECK_ARG(dimp <= 256, GLM_ERR_UNSUPPORTED, "glm_memory_chunkwise: key size %d", dimp);
     if (seqs == 0) return GLM_OK;
-    ChunkArgs a = {(const bf16_t*)x, ldx, k_off, v_off, gates, rows, (bf16_t*)o, ldo, S, n, m, n_state, pos, q_start, state_in, state_out, H, dim, dimp, vdimp, (vdimp + 63) / 64, nullptr};
+    ChunkArgs a = {(const bf16_t*)x, ldx, k_off, v_off, gates, rows, (bf16_t*)o, ldo, S, n, m, n_state, pos, q_start, state_in, state_out, H, dim, dimp, vdimp, (vdimp + 63) / 64, nullptr, {}};
     GLM_CHECK_ARG((int64_t)seqs * H * a.vtiles < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_memory_chunkwise: grid too large");
     hipStream_t st = glm_s(stream);
-    if (dimp <= 64) return launch_chunk<64, true>(a, seqs, st);
-    if (dimp <= 128) return launch_chunk<128, true>(a, seqs, st);
-    return launch_chunk<256, true>(a, seqs, st);
+    if (dimp <= 64) return launch_chunk<64, true>(a, seqs, 1, st);
+    if (dimp <= 128) return launch_chunk<128, true>(a, seqs, 1, st);
+    return launch_chunk<256, true>(a, seqs, 1, st);
 }
 
 extern "C" int glm_memory_output(const void* o, int64_t ldo, const void* g, int64_t ldg, const float* norm, void* y, int64_t ldy, int64_t T, int H, int vdim, int vdimp, float eps,
@@ -1070,20 +1084,29 @@ extern "C" int glm_linear_recurrent(const void* x, int64_t ldx, int64_t k_off, i
     return f32 ? run_rec<float>(a, glm_s(stream)) : run_rec<bf16_t>(a, glm_s(stream));
 }
 
-extern "C" int glm_linear_chunkwise(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* powers, void* o, int64_t ldo, float* S, int64_t n_state, const int32_t* pos,
+extern "C" int glm_linear_chunkwise(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* powers, int64_t rows, void* o, int64_t ldo, float* S, int64_t n_state, const int32_t* pos,
                                     const int32_t* q_start, const int32_t* state_in, const int32_t* state_out, int seqs, int H, int dimp, int vdimp, glm_stream_t stream) {
     GLM_CHECK_ARG(x && powers && o && S && pos && q_start && state_in && state_out, GLM_ERR_INVALID, "glm_linear_chunkwise: null pointer");
-    GLM_CHECK_ARG(seqs >= 0 && H > 0 && dimp > 0 && dimp % 8 == 0 && vdimp > 0 && vdimp % 8 == 0 && n_state > 0 && k_off >= (int64_t)H * dimp && ldx >= k_off + (int64_t)H * dimp &&
+    GLM_CHECK_ARG(seqs >= 0 && rows >= 0 && H > 0 && dimp > 0 && dimp % 8 == 0 && vdimp > 0 && vdimp % 8 == 0 && n_state > 0 && k_off >= (int64_t)H * dimp && ldx >= k_off + (int64_t)H * dimp &&
                       ldx >= v_off + (int64_t)H * vdimp && ldo >= (int64_t)H * vdimp && ldx % 8 == 0 && k_off % 8 == 0 && v_off % 8 == 0 && ldo % 4 == 0 && ldx < (1 << 24) &&
                       glm_aligned16(x) && (((uintptr_t)o) & 7) == 0, GLM_ERR_INVALID, "glm_linear_chunkwise: bad shape H=%d dimp=%d vdimp=%d ldx=%ld", H, dimp, vdimp, (long)ldx);
     GLM_CHECK_ARG(dimp <= 256, GLM_ERR_UNSUPPORTED, "glm_linear_chunkwise: key size %d", dimp);
     if (seqs == 0) return GLM_OK;
-    ChunkArgs a = {(const bf16_t*)x, ldx, k_off, v_off, nullptr, 0, (bf16_t*)o, ldo, S, nullptr, nullptr, n_state, pos, q_start, state_in, state_out, H, dimp, dimp, vdimp, (vdimp + 63) / 64, powers};
+    // segments as long as the chip has room: a chunk that only moves the state costs about a third of a whole one, and all segments shall
+    // take the same time, c (t_(s+1) - t_s) + c / 3 t_s
+    const int64_t wgs = (int64_t)seqs * H * ((vdimp + 63) / 64);
+    int nseg = (int)(256 / (wgs > 0 ? wgs : 1)), most = (int)(rows / seqs / 256);
+    nseg = nseg > most ? most : nseg;
+    nseg = nseg > MM_MAX_SEG ? MM_MAX_SEG : nseg < 1 ? 1 : nseg;
+    ChunkArgs a = {(const bf16_t*)x, ldx, k_off, v_off, nullptr, 0, (bf16_t*)o, ldo, S, nullptr, nullptr, n_state, pos, q_start, state_in, state_out, H, dimp, dimp, vdimp, (vdimp + 63) / 64, powers, {}};
+    float left = 1.0f, all = 1.0f;
+    for (int i = 0; i < nseg; ++i) all *= 2.0f / 3;
+    for (int i = 0; i <= nseg; ++i, left *= 2.0f / 3) a.seg[i] = i == nseg ? 1.0f : (1.0f - left) / (1.0f - all);
     GLM_CHECK_ARG((int64_t)seqs * H * a.vtiles < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_linear_chunkwise: grid too large");
     hipStream_t st = glm_s(stream);
-    if (dimp <= 64) return launch_chunk<64, false>(a, seqs, st);
-    if (dimp <= 128) return launch_chunk<128, false>(a, seqs, st);
-    return launch_chunk<256, false>(a, seqs, st);
+    if (dimp <= 64) return launch_chunk<64, false>(a, seqs, nseg, st);
+    if (dimp <= 128) return launch_chunk<128, false>(a, seqs, nseg, st);
+    return launch_chunk<256, false>(a, seqs, nseg, st);
 }
 
 extern "C" int glm_row_norm_gate(const void* o, int64_t ldo, int o_f32, const void* gate, int64_t ldg, const float* norm, void* y, int64_t ldy, int64_t T, int n, int np, float eps,

@@ -188,7 +188,7 @@ _SIGNATURES = {
         c_float, c_void_p]),
     "glm_linear_recurrent": (c_int, [c_void_p, c_int64, c_int64, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_void_p,
         c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_void_p]),
-    "glm_linear_chunkwise": (c_int, [c_void_p, c_int64, c_int64, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_void_p,
+    "glm_linear_chunkwise": (c_int, [c_void_p, c_int64, c_int64, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_void_p,
         c_void_p, c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_void_p]),
     "glm_row_norm_gate": (c_int, [c_void_p, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int64, c_int, c_int,
         c_float, c_int, c_void_p]),
@@ -1763,7 +1763,7 @@ def linear_chunkwise(x: torch.Tensor, powers: torch.Tensor, S: torch.Tensor, pos
     assert state_in.numel() >= seqs and state_out.numel() >= seqs
     o = torch.empty((T, heads * vdimp), dtype=x.dtype, device=x.device)
     _check(load_library().glm_linear_chunkwise(
-        _p(x), x.stride(0), kd, 2 * kd, _p(powers), _p(o), heads * vdimp, _p(S), S.shape[0], _p(pos), _p(q_start), _p(state_in), _p(state_out), seqs, heads, dimp, vdimp,
+        _p(x), x.stride(0), kd, 2 * kd, _p(powers), T, _p(o), heads * vdimp, _p(S), S.shape[0], _p(pos), _p(q_start), _p(state_in), _p(state_out), seqs, heads, dimp, vdimp,
         _stream()), "glm_linear_chunkwise")
     return o
 

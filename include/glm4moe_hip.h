@@ -593,12 +593,12 @@ int glm_memory_output(const void* o, int64_t ldo, const void* g, int64_t ldg, co
 
 /* The linear memory (attention with a constant decay per head): S_t = decay S_(t-1) + k v^T, o_t = S_t^T q.  x rows hold q at h*dimp, k at
  * k_off + h*dimp, v at v_off + h*vdimp; state S [n_state][H][dimp][vdimp] fp32.  recurrent: o fp32 rows [T, ldo]; chunkwise (long
- * portions, bf16, dimp <= 256): powers [H][65] = decay^j, o bf16 rows.  row_norm_gate: y = o / rms(o) norm gate over np columns of a row,
+ * portions, bf16, dimp <= 256): powers [H][65] = decay^j, o bf16 rows, `rows` of them.  row_norm_gate: y = o / rms(o) norm gate over np columns of a row,
  * n of them true (the others zeros).                                                                                          */
 int glm_linear_recurrent(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* decay, float* o, int64_t ldo, float* S,
                          int64_t n_state, const int32_t* pos, const int32_t* q_start, const int32_t* state_in, const int32_t* state_out,
                          int seqs, int H, int dimp, int vdimp, int f32, glm_stream_t stream);
-int glm_linear_chunkwise(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* powers, void* o, int64_t ldo, float* S,
+int glm_linear_chunkwise(const void* x, int64_t ldx, int64_t k_off, int64_t v_off, const float* powers, int64_t rows, void* o, int64_t ldo, float* S,
                          int64_t n_state, const int32_t* pos, const int32_t* q_start, const int32_t* state_in, const int32_t* state_out,
                          int seqs, int H, int dimp, int vdimp, glm_stream_t stream);
 int glm_row_norm_gate(const void* o, int64_t ldo, int o_f32, const void* gate, int64_t ldg, const float* norm, void* y, int64_t ldy,

@@ -296,6 +296,22 @@ def test_linear_attention(form, H, dim, vd, decay):
             assert distance(a, b) < (1e-5 if dtype == "float32" else 3e-2), form
 
 
+@pytest.mark.parametrize("H,dim,vd,lens", [(1, 40, 24, (2100,)), (2, 64, 72, (1500, 70, 1130)), (1, 136, 64, (1200, 900))])
+def test_linear_attention_in_segments(H, dim, vd, lens):
+    """Long portions of few heads are cut into segments that bring the state up to their beginning by themselves."""
+    from nanovllm.layers.linear_attention import LinearAttention
+    width, e = 40, lightning(H, dim, vd, None, [1.0, 0.998][:H])
+    w = mixer_weights(config(width, 16, 2, 2, [e]), 5)
+    mod = LinearAttention(width, H, dim, vd, e["mixer"]["decay"], 1e-5, torch.bfloat16)
+    mod.load(w, "cuda")
+    hs = [torch.randn(n, width, generator=g(n)).to(torch.bfloat16).float() for n in lens]
+    W = O.Weights({"m." + k: v for k, v in w.items()})
+    ref = [O.lightning(h.double(), W, "m.", e["mixer"], 1e-5, O.Project()) for h in hs]
+    for plan in ([dict.fromkeys(range(len(lens)), 4000)], [dict.fromkeys(range(len(lens)), 601), dict.fromkeys(range(len(lens)), 4000)]):
+        for a, b in zip(run_mixer(mod, hs, plan, 1, torch.bfloat16), ref):
+            assert distance(a, b) < 3e-2
+
+
 # ---- the model through the engine -------------------------------------------------------------------------------------------
 @pytest.fixture(scope="module", params=list(CONFIGS))
 def model(request, tmp_path_factory):
