@@ -460,7 +460,9 @@ def test_memory_sized_pool_and_sampling(tmp_path, name):
     sample."""
     from nanovllm import LLM, SamplingParams
     cfg, t = make_model(tmp_path, name, 5)
-    llm = LLM(str(tmp_path), max_num_seqs=5, max_num_batched_tokens=256, max_model_len=256, gpu_memory_utilization=0.05)
+    torch.cuda.empty_cache()
+    free, total = torch.cuda.mem_get_info()    # (other tests of the process may hold memory)
+    llm = LLM(str(tmp_path), max_num_seqs=5, max_num_batched_tokens=256, max_model_len=256, gpu_memory_utilization=1.0 - free / total + 0.03)
     try:
         assert llm.config.num_kvcache_blocks >= (1000 if name == "odd" else 20)
         a, b = (llm.generate([tokens(cfg, t, 20, 1)], SamplingParams(temperature=x, max_tokens=24, ignore_eos=True), use_tqdm=False)[0]["token_ids"]
