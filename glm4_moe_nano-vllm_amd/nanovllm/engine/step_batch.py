@@ -117,7 +117,10 @@ def build_step(chunks: list[Chunk], spec, block_size: int, pad_rows: int = 0, ta
         n_tiles = -(-all_lens[L] // LONG_TILE)
         tseq = np.repeat(np.arange(len(L)), n_tiles)
         k = np.arange(len(tseq)) - np.repeat(np.cumsum(n_tiles) - n_tiles, n_tiles)
-        tseq, k = tseq[::-1], k[::-1]   # a portion's last rows see the most keys: they start first
+        tseq, k = tseq[::-1], k[::-1]   # a portion's last rows see the most keys: they start first, over all portions
+        keys = np.minimum(starts[n_short:][tseq] + (k + 1) * LONG_TILE, max(spec.windows, default=1 << 30))
+        o = np.argsort(-keys, kind="stable")
+        tseq, k = tseq[o], k[o]
         longs = (pk.add(q_start[n_short:] - Ta), pk.add(tseq), pk.add(k * LONG_TILE))
         for c, rows in getattr(spec, "chunk_tiles", ()):            # tiles for attention over chunks, the ones with the most keys first
             m = -(-all_lens[L] // rows)
