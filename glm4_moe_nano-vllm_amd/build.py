@@ -21,13 +21,14 @@ LIB = os.path.join(LIBDIR, "libglm4moe_hip.so")
 ARCH = "gfx950"
 SOURCES = ["api", "elementwise", "moe_misc", "paged_attn", "prefill_attn", "gemm_smallm", "gemm_tinym", "gemm_largem",
            "decode_engine", "oneshot_allreduce", "seq_norm", "gemm_f32", "latent_attn", "window_attn", "attn_merge", "stream_norm", "group_attn",
-           "matrix_memory", "depth_norm"]
+           "matrix_memory", "depth_norm", "rope_pairs", "residual_norm", "group_rows"]
 # kernel sets: what one model needs and nothing else (models/registry.py names the set), for a first run in a fresh checkout;
 # the library of everything is used where it is there
 _DENSE = ["api", "gemm_smallm", "gemm_tinym", "gemm_largem", "seq_norm", "gemm_f32", "attn_merge"]
 KERNEL_SETS = {"dafolorn": (_DENSE + ["latent_attn", "window_attn"], ["GLM_DENSE_ONLY=1"]),
                "napadra": (_DENSE + ["stream_norm", "group_attn", "matrix_memory"], ["GLM_DENSE_ONLY=1"]),
-               "gulozen": (_DENSE + ["moe_misc", "latent_attn", "window_attn", "matrix_memory", "depth_norm"], ["GLM_DENSE_ONLY=1", "GLM_EXPERTS=1"])}
+               "gulozen": (_DENSE + ["moe_misc", "latent_attn", "window_attn", "matrix_memory", "depth_norm", "rope_pairs"], ["GLM_DENSE_ONLY=1", "GLM_EXPERTS=1"]),
+               "loselix": ([s for s in _DENSE if s != "seq_norm"] + ["rope_pairs", "residual_norm", "group_rows", "group_attn"], ["GLM_DENSE_ONLY=1"])}
 # kernels that were measured against the shipped ones and lost: only in the study library (`--study`), with their tests
 STUDY_SOURCES = ["prefill_attn64", "prefill_attn_persist"]
 STUDY_TAG = "_study"

@@ -13,7 +13,7 @@ void glm_set_error(const char* fmt, ...) {
     va_end(ap);
 }
 
-extern "C" int glm_abi_version(void) { return 13; }
+extern "C" int glm_abi_version(void) { return 14; }
 extern "C" const char* glm_last_error(void) { return g_err; }
 
 // ---- launch-path options: name, environment variable read once, default ------------------------------------------------
@@ -147,7 +147,7 @@ extern "C" int glm_gemm_bf16_act(const void* x, int64_t ldx, const void* w, int6
     GLM_CHECK_ARG(x && w && y, GLM_ERR_INVALID, "glm_gemm_bf16_act: null pointer");
     GLM_CHECK_ARG(M >= 0 && N > 0 && K > 0 && ldx >= K && ldy >= N && ldw >= K, GLM_ERR_INVALID,
                   "glm_gemm_bf16_act: bad shape M=%ld N=%d K=%d ldx=%ld ldy=%ld", (long)M, N, K, (long)ldx, (long)ldy);
-    GLM_CHECK_ARG(act >= GLM_ACT_NONE && act <= GLM_ACT_SILU_GATE && act != GLM_ACT_GLU_CLAMP, GLM_ERR_INVALID, "glm_gemm_bf16_act: unknown activation %d", act);
+    GLM_CHECK_ARG(act >= GLM_ACT_NONE && act <= GLM_ACT_RELU2_GATE && act != GLM_ACT_GLU_CLAMP, GLM_ERR_INVALID, "glm_gemm_bf16_act: unknown activation %d", act);
     GLM_CHECK_ARG(!out_f32 || (glm_aligned16(y) && ldy % 4 == 0), GLM_ERR_UNSUPPORTED, "glm_gemm_bf16_act: fp32 rows need 16-byte alignment");
     GemmParams p;
     memset(&p, 0, sizeof(p));

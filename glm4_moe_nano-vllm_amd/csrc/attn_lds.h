@@ -17,6 +17,10 @@ template <int AUX = 0>
 __device__ __forceinline__ void lds_dma16(const void* gsrc, void* lds_wave_base) {
     __builtin_amdgcn_global_load_lds((attn_glb_void*)gsrc, (attn_lds_void*)lds_wave_base, 16, 0, AUX);
 }
+// 64 lanes x 4 bytes: 256 bytes of LDS
+__device__ __forceinline__ void lds_dma4(const void* gsrc, void* lds_wave_base) {
+    __builtin_amdgcn_global_load_lds((attn_glb_void*)gsrc, (attn_lds_void*)lds_wave_base, 4, 0, 0);
+}
 template <int OFF>
 __device__ __forceinline__ void lds_read_b128(u32x4_t& dst, unsigned addr) {
     asm volatile("ds_read_b128 %0, %1 offset:%2" : "=v"(dst) : "v"(addr), "i"(OFF));

@@ -153,7 +153,7 @@ extern "C" int glm_gemm_f32(const float* x, int64_t ldx, int64_t xb, const float
                   "glm_gemm_f32: bad shape M=%ld N=%d K=%d", (long)M, N, K);
     GLM_CHECK_ARG(K % 4 == 0 && ldx % 4 == 0 && ldw % 4 == 0 && xb % 4 == 0 && wb % 4 == 0 && glm_aligned16(x) && glm_aligned16(w), GLM_ERR_UNSUPPORTED,
                   "glm_gemm_f32: needs K, ldx, ldw, batch strides %% 4 == 0 and 16-byte aligned operands (K=%d)", K);
-    GLM_CHECK_ARG(act >= GLM_ACT_NONE && act <= GLM_ACT_SILU_GATE && act != GLM_ACT_GLU_CLAMP, GLM_ERR_INVALID, "glm_gemm_f32: unknown activation %d", act);
+    GLM_CHECK_ARG(act >= GLM_ACT_NONE && act <= GLM_ACT_RELU2_GATE && act != GLM_ACT_GLU_CLAMP, GLM_ERR_INVALID, "glm_gemm_f32: unknown activation %d", act);
     const int64_t gy = (M + GF_B - 1) / GF_B;
     GLM_CHECK_ARG(gy <= 65535 && batch <= 65535, GLM_ERR_UNSUPPORTED, "glm_gemm_f32: too many rows (%ld)", (long)M);
     if (M == 0) return GLM_OK;

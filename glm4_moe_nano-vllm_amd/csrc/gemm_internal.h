@@ -27,15 +27,17 @@ __host__ __device__ constexpr bool gemm_paired(int mode) { return mode == GEMM_G
 
 // activation on the fp32 accumulator of a projection (after the bias)
 enum : int { GLM_ACT_NONE = GLM_EPI_NONE, GLM_ACT_XIELU = GLM_EPI_XIELU, GLM_ACT_SOFTCAP = GLM_EPI_SOFTCAP, GLM_ACT_GLU_CLAMP = GLM_EPI_GLU_CLAMP,
-              GLM_ACT_GATE = GLM_EPI_GATE, GLM_ACT_SILU_GATE = GLM_EPI_SILU_GATE };
+              GLM_ACT_GATE = GLM_EPI_GATE, GLM_ACT_SILU_GATE = GLM_EPI_SILU_GATE, GLM_ACT_RELU2_GATE = GLM_EPI_RELU2_GATE };
 struct GlmAct {
     int kind;
     float a, b;
 };
 // z > 0: a z^2 + z / 2;  z <= 0: b (exp(z) - 1 - z) + z / 2.   The fp32 form, for fp32 outputs.
 __device__ __forceinline__ float glm_act_precise(const GlmAct& t, float z, int n) {
+    if (t.kind == GLM_ACT_RELU2_GATE && n < (int)t.b) return n < (int)t.a ? fmaxf(z, 0.f) * fmaxf(z, 0.f) : z;
     if (t.kind >= GLM_ACT_GATE) {
         const float s = 1.0f / (1.0f + expf(-z));
+        if (t.kind == GLM_ACT_RELU2_GATE) return s;
         return n >= (int)t.a ? s : t.kind == GLM_ACT_SILU_GATE ? z * s : z;
     }
     if (t.kind == GLM_ACT_XIELU) return z > 0.f ? t.a * z * z + 0.5f * z : t.b * (expm1f(z) - z) + 0.5f * z;
@@ -48,9 +50,12 @@ __device__ __forceinline__ float glm_xielu_fast(float a, float b, float z) {
     const float neg = b * (__builtin_amdgcn_exp2f(1.4426950408889634f * fminf(z, 0.f)) - 1.0f - z);
     return (z > 0.f ? a * z * z : neg) + 0.5f * z;
 }
-// per-column activations: the first t.a columns pass (or go through SiLU), the others through the sigmoid (a gate)
+// per-column activations: the first t.a columns pass (or go through SiLU), the others through the sigmoid (a gate); or the first t.a
+// columns are the square of relu, those up to t.b pass, the others go through the sigmoid
 __device__ __forceinline__ float glm_act_cols(const GlmAct& t, float z, int n) {
+    if (t.kind == GLM_ACT_RELU2_GATE && n < (int)t.b) return n < (int)t.a ? fmaxf(z, 0.f) * fmaxf(z, 0.f) : z;
     const float s = __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+    if (t.kind == GLM_ACT_RELU2_GATE) return s;
     return n >= (int)t.a ? s : t.kind == GLM_ACT_SILU_GATE ? z * s : z;
 }
 __device__ __forceinline__ float glm_act_fast(const GlmAct& t, float z, int n) {

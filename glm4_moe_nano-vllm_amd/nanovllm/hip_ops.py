@@ -8,6 +8,7 @@ from __future__ import annotations
 
 import ctypes
 import os
+from dataclasses import dataclass
 from ctypes import c_char_p, c_float, c_int, c_int64, c_size_t, c_void_p
 
 import torch
@@ -153,7 +154,7 @@ _SIGNATURES = {
     "glm_latent_attn_max_rows": (c_int, [c_int]),
     "glm_latent_attn": (c_int, [c_void_p, c_void_p, c_int64, c_int, c_void_p, c_void_p, c_int, c_int, c_void_p, c_void_p, c_void_p,
         c_int64, c_int64, c_int, c_int, c_int, c_int, c_float, c_void_p, c_int, c_void_p, c_void_p, c_void_p, c_int, c_void_p]),
-    "glm_attn_merge": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int64, c_int, c_int, c_void_p]),
+    "glm_attn_merge": (c_int, [c_void_p, c_void_p, c_void_p, c_int, c_void_p, c_int64, c_int64, c_int, c_int, c_void_p, c_void_p]),
     "glm_latent_up": (c_int, [c_void_p, c_void_p, c_void_p, c_void_p, c_int64, c_int64, c_int64, c_int, c_int, c_int, c_void_p]),
     "glm_window_attn_prefill": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_void_p, c_int64, c_int, c_void_p, c_void_p,
         c_int64, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_void_p, c_int, c_int, c_int64, c_int64, c_int, c_int, c_int, c_int,
@@ -167,15 +168,18 @@ _SIGNATURES = {
     "glm_group_kv_store": (c_int, [c_void_p, c_int64, c_int64, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int,
         c_int, c_int, c_int, c_void_p]),
     "glm_group_attn_prefill": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p, c_int64, c_int, c_void_p, c_void_p,
-        c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p,
-        c_void_p, c_void_p, c_int64, c_void_p]),
+        c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_int64, c_void_p]),
     "glm_group_attn_decode": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p,
-        c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p,
-        c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_int, c_void_p,
-        c_void_p, c_void_p]),
-    "glm_group_attn_plain": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p,
-        c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_void_p, c_void_p, c_void_p, c_int64,
-        c_int, c_void_p]),
+        c_void_p, c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p,
+        c_int64, c_int, c_void_p, c_void_p, c_void_p]),
+    "glm_group_attn_plain": (c_int, [c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p, c_int64, c_void_p, c_void_p, c_int64,
+        c_int, c_int, c_int, c_int, c_void_p, c_void_p, c_int64, c_int, c_void_p]),
+    "glm_group_rotate_store": (c_int, [c_void_p, c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int,
+        c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p]),
+    "glm_group_norm_store": (c_int, [c_void_p, c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int, c_int, c_int, c_float,
+        c_float, c_int, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p]),
+    "glm_residual_norm": (c_int, [c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int, c_int64, c_void_p, c_int64, c_int64, c_void_p, c_void_p,
+        c_void_p, c_void_p, c_int64, c_int, c_int64, c_int, c_int, c_float, c_void_p]),
     "glm_memory_recurrent": (c_int, [c_void_p, c_int64, c_int64, c_int64, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_int, c_void_p,
         c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_void_p,
         c_void_p, c_int, c_int, c_int, c_int, c_int, c_int, c_float, c_float, c_int, c_void_p]),
@@ -1265,6 +1269,7 @@ def gemm_bf16(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None
 # reference).  Activations are bf16 or fp32 (`act dtype`): every op below takes either and picks the kernel by dtype.
 ACT_NONE, ACT_XIELU, ACT_SOFTCAP = 0, 1, 2
 ACT_GATE, ACT_SILU_GATE = 4, 5     # columns below the constant pass / go through SiLU, the others through the sigmoid
+ACT_RELU2_GATE = 6                 # columns below the first constant: relu squared; below the second: pass; the others: sigmoid
 NO_ACT = (ACT_NONE, 0.0, 0.0)
 
 
@@ -1280,22 +1285,25 @@ def _is_f32(dtype) -> int:
     raise TypeError(f"activations are bfloat16 or float32, not {dtype}")
 
 
-def linear_act(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, act=NO_ACT, out_f32: bool = False) -> torch.Tensor:
-    """act(x @ w.T + bias), x [M, K], w [N, K] (row pitches free), in x's dtype or — out_f32 — unrounded fp32."""
+def linear_act(x: torch.Tensor, w: torch.Tensor, bias: torch.Tensor | None = None, act=NO_ACT, out_f32: bool = False, out: torch.Tensor | None = None) -> torch.Tensor:
+    """act(x @ w.T + bias), x [M, K], w [N, K] (row pitches free), in x's dtype or — out_f32 — unrounded fp32; out: where to (a view with
+    its own row pitch)."""
     M, K = x.shape
     N = w.shape[0]
     assert w.shape[1] == K and w.dtype == x.dtype and x.stride(1) == 1 and w.stride(1) == 1
     f32 = _is_f32(x.dtype)
     assert bias is None or (bias.dtype == x.dtype and bias.numel() == N and bias.is_contiguous())
-    y = torch.empty((M, N), dtype=torch.float32 if (f32 or out_f32) else x.dtype, device=x.device)
+    dt = torch.float32 if (f32 or out_f32) else x.dtype
+    y = torch.empty((M, N), dtype=dt, device=x.device) if out is None else out
+    assert y.shape == (M, N) and y.dtype == dt and y.stride(1) == 1
     if f32:
-        _check(load_library().glm_gemm_f32(_p(x), x.stride(0), 0, _p(w), w.stride(0), 0, _p(bias), _p(y), N, 0, M, N, K, 1, *act,
+        _check(load_library().glm_gemm_f32(_p(x), x.stride(0), 0, _p(w), w.stride(0), 0, _p(bias), _p(y), y.stride(0), 0, M, N, K, 1, *act,
                                            _stream()), "glm_gemm_f32")
     elif act[0] == ACT_NONE and not out_f32:
-        _check(load_library().glm_gemm_bf16(_p(x), x.stride(0), _p(w), w.stride(0), _p(bias), _p(y), N, M, N, K, _stream()),
+        _check(load_library().glm_gemm_bf16(_p(x), x.stride(0), _p(w), w.stride(0), _p(bias), _p(y), y.stride(0), M, N, K, _stream()),
                "glm_gemm_bf16")
     else:
-        _check(load_library().glm_gemm_bf16_act(_p(x), x.stride(0), _p(w), w.stride(0), _p(bias), _p(y), N, M, N, K,
+        _check(load_library().glm_gemm_bf16_act(_p(x), x.stride(0), _p(w), w.stride(0), _p(bias), _p(y), y.stride(0), M, N, K,
                                                 int(out_f32), *act, _stream()), "glm_gemm_bf16_act")
     return y
 
@@ -1503,7 +1511,7 @@ def latent_attn(qa: torch.Tensor, cache: torch.Tensor, tile_tok: torch.Tensor, t
             mul_f32(out[:Ta], gate[:Ta])
         return
     if ns > 1:
-        _check(lib.glm_attn_merge(_p(part_o), _p(part_ml), _p(sink), ns, _p(ctx), Ta, H, vp, _stream()), "glm_attn_merge")
+        _check(lib.glm_attn_merge(_p(part_o), _p(part_ml), _p(sink), ns, _p(ctx), H * vp, Ta, H, vp, None, _stream()), "glm_attn_merge")
     _check(lib.glm_latent_up(_p(ctx), _p(wuv), _p(out), _p(gate), gate.stride(0) if gate is not None else 0, out.stride(0), Ta, H, vdimp, vp, _stream()),
            "glm_latent_up")
 
@@ -1598,6 +1606,40 @@ def group_kv_store(src: torch.Tensor, k_off: int, v_off: int, slots: torch.Tenso
                                              n * bs, bs, G, dk, v_cache.shape[3], _stream()), "glm_group_kv_store")
 
 
+class _GroupForm(ctypes.Structure):
+    _fields_ = [("window", c_int), ("chunk", c_int), ("scale", c_float), ("slope", c_void_p), ("sink", c_void_p), ("cap", c_float), ("maps", c_int),
+                ("lam", c_float), ("post", c_float), ("eps", c_float), ("vn", c_int), ("sigmoid", c_int), ("bias", c_void_p), ("kscale", c_void_p),
+                ("gate", c_void_p), ("ldg", c_int64), ("gate_cols", c_int)]
+
+
+@dataclass
+class GroupParts:
+    """What an attention with grouped heads may have beside window, chunk, slope and sink (include/glm4moe_hip.h, glm_group_form)."""
+    cap: float = 0.0                       # soft cap on the scores
+    maps: int = 1                          # 2: two queries / keys per head side by side, output post d / rms(d), d = o_1 - lam o_2, over vn columns
+    lam: float = 0.0
+    post: float = 1.0
+    eps: float = 0.0
+    vn: int = 0
+    sigmoid: bool = False                  # weights sigmoid(score + bias), not normalised
+    bias: torch.Tensor | None = None       # fp32 [heads]
+    kscale: torch.Tensor | None = None     # fp32 [blocks, block size]: the keys are the values, their products times this
+    gate: torch.Tensor | None = None       # factors of the output, a row per row of q; [T, heads] or, gate_cols, [T, heads * value columns]
+    gate_cols: bool = False
+
+
+NO_PARTS = GroupParts()
+
+
+def _group_form(window, chunk, scale, slope, sink, p: GroupParts, q, k_cache, v_cache, heads: int) -> _GroupForm:
+    assert p.bias is None or (p.bias.dtype == torch.float32 and p.bias.numel() == heads)
+    assert p.kscale is None or (p.kscale.dtype == torch.float32 and p.kscale.is_contiguous() and p.kscale.numel() == k_cache.shape[0] * k_cache.shape[2])
+    assert p.gate is None or (p.gate.dtype == q.dtype and p.gate.stride(1) == 1 and p.gate.shape[0] >= q.shape[0]
+                              and p.gate.shape[1] >= (heads * v_cache.shape[3] if p.gate_cols else heads))
+    return _GroupForm(window, chunk, scale, _p(slope), _p(sink), p.cap, p.maps, p.lam, p.post, p.eps, p.vn, int(p.sigmoid), _p(p.bias), _p(p.kscale), _p(p.gate),
+                      p.gate.stride(0) if p.gate is not None else 0, int(p.gate_cols))
+
+
 def _group_shape(q, k_cache, v_cache, out, heads, slope, sink):
     n, G, bs, dk = k_cache.shape
     dv = v_cache.shape[3]
@@ -1608,35 +1650,41 @@ def _group_shape(q, k_cache, v_cache, out, heads, slope, sink):
     return n, G, bs, dk, dv
 
 
-def group_attn_tile_rows(heads: int, kv_heads: int) -> int:
-    """Query rows per workgroup of glm_group_attn_prefill: two heads of a group share a tile where they pair up."""
-    return 64 if (heads // kv_heads) % 2 == 0 else 128
+def group_attn_tile_rows(heads: int, kv_heads: int, maps: int = 1) -> int:
+    """Query rows per workgroup of glm_group_attn_prefill: two heads of a group share a tile where they pair up, and so do two maps."""
+    return 64 if maps == 2 or (heads // kv_heads) % 2 == 0 else 128
+
+
+def group_attn_rows(maps: int = 1) -> int:
+    """(token, head) rows a workgroup of glm_group_attn_decode takes."""
+    return GROUP_ATTN_ROWS // maps
 
 
 def group_attn_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor, seq0: int, q_start: torch.Tensor,
                        pos: torch.Tensor, tile_seq: torch.Tensor, tile_off: torch.Tensor, heads: int, window: int, chunk: int, scale: float, slope, sink,
-                       out: torch.Tensor) -> None:
+                       out: torch.Tensor, parts: GroupParts = NO_PARTS) -> None:
     """Long portions (rows of q, q_start relative to them) over the paged caches; block table of portion s in row seq0 + s; tiles of
     group_attn_tile_rows rows."""
     n, G, bs, dk, dv = _group_shape(q, k_cache, v_cache, out, heads, slope, sink)
     for t in (block_tables, q_start, pos, tile_seq, tile_off):
         assert t.dtype == torch.int32
     assert pos.numel() == q.shape[0] and tile_seq.numel() == tile_off.numel() and block_tables.shape[0] >= seq0 + q_start.numel() - 1
+    form = _group_form(window, chunk, scale, slope, sink, parts, q, k_cache, v_cache, heads)
     _check(load_library().glm_group_attn_prefill(
         _p(q), q.stride(0), _p(k_cache), _p(v_cache), n, bs, _p(block_tables), block_tables.stride(0), seq0, _p(q_start), _p(pos), _p(tile_seq), _p(tile_off),
-        tile_seq.numel(), group_attn_tile_rows(heads, G), heads, G, dk, dv, window, chunk, scale, _p(slope), _p(sink), _p(out), out.stride(0), _stream()),
+        tile_seq.numel(), group_attn_tile_rows(heads, G, parts.maps), heads, G, dk, dv, ctypes.byref(form), _p(out), out.stride(0), _stream()),
         "glm_group_attn_prefill")
 
 
-def group_attn_splits(tiles: int, tokens_per_tile: int, heads: int, kv_heads: int, keys: int) -> int:
+def group_attn_splits(tiles: int, tokens_per_tile: int, heads: int, kv_heads: int, keys: int, maps: int = 1) -> int:
     """KV splits of a decode launch: about one workgroup per CU, at least 128 keys each."""
-    wgs = tiles * kv_heads * -(-tokens_per_tile * (heads // kv_heads) // GROUP_ATTN_ROWS)
+    wgs = tiles * kv_heads * -(-tokens_per_tile * (heads // kv_heads) // group_attn_rows(maps))
     return max(1, min(64, 256 // max(1, wgs), -(-keys // 128)))
 
 
 def group_attn_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor, pos: torch.Tensor, seq_of: torch.Tensor,
                       tile_tok: torch.Tensor, tile_n: torch.Tensor, tokens_per_tile: int, heads: int, window: int, chunk: int, scale: float, slope, sink,
-                      out: torch.Tensor, num_splits: int = 0, new=None) -> None:
+                      out: torch.Tensor, num_splits: int = 0, new=None, parts: GroupParts = NO_PARTS) -> None:
     """Decoded tokens and short portions (the rows of q) over the paged caches; out is written row by row from its first.  new =
     (keys, values, q_start, slots): the rows' own keys and values are taken from there and stored to their cache rows."""
     n, G, bs, dk, dv = _group_shape(q, k_cache, v_cache, out, heads, slope, sink)
@@ -1649,37 +1697,92 @@ def group_attn_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Ten
     keys = block_tables.shape[1] * bs
     for w in (window, chunk):
         keys = min(keys, w + tokens_per_tile) if w else keys
-    ns = num_splits or (group_attn_splits(tile_tok.numel(), tokens_per_tile, heads, G, keys) if sink is not None and out.stride(0) == heads * dv else 1)
+    ns = num_splits or group_attn_splits(tile_tok.numel(), tokens_per_tile, heads, G, keys, parts.maps)
     part_o = part_ml = None
-    if ns > 1:
-        part_o = torch.empty((T * heads, ns, dv), dtype=torch.float32, device=q.device)
-        part_ml = torch.empty((T * heads, ns, 2), dtype=torch.float32, device=q.device)
+    if ns > 1 or parts.maps > 1:
+        part_o = torch.empty((T * heads * parts.maps, ns, dv), dtype=torch.float32, device=q.device)
+        part_ml = torch.empty((T * heads * parts.maps, ns, 2), dtype=torch.float32, device=q.device)
     kn = vn = q_start = slots = None
     if new is not None:
         kn, vn, q_start, slots = new
         assert kn.shape == (T, G * dk) and vn.shape == (T, G * dv) and kn.stride() == vn.stride() and kn.stride(1) == 1 and kn.dtype == vn.dtype == q.dtype
         assert q_start.dtype == slots.dtype == torch.int32 and slots.numel() >= T
-    lib = load_library()
+    lib, form = load_library(), _group_form(window, chunk, scale, slope, sink, parts, q, k_cache, v_cache, heads)
     _check(lib.glm_group_attn_decode(
         _p(q), q.stride(0), _p(k_cache), _p(v_cache), n, bs, _p(block_tables), block_tables.stride(0), _p(pos), _p(seq_of), _p(tile_tok), _p(tile_n),
-        tile_tok.numel(), tokens_per_tile, heads, G, dk, dv, window, chunk, scale, _p(slope), _p(sink), _p(kn), _p(vn),
+        tile_tok.numel(), tokens_per_tile, heads, G, dk, dv, ctypes.byref(form), _p(kn), _p(vn),
         kn.stride(0) if kn is not None else 0, _p(q_start), _p(slots), _p(out), out.stride(0), ns, _p(part_o), _p(part_ml),
         _stream()), "glm_group_attn_decode")
-    if ns > 1:
-        assert sink is not None and out.stride(0) == heads * dv
-        _check(lib.glm_attn_merge(_p(part_o), _p(part_ml), _p(sink), ns, _p(out), T, heads, dv, _stream()), "glm_attn_merge")
+    if part_o is not None:
+        _check(lib.glm_attn_merge(_p(part_o), _p(part_ml), _p(sink), ns, _p(out), out.stride(0), T, heads, dv, ctypes.byref(form), _stream()), "glm_attn_merge")
 
 
 def group_attn_plain(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tensor, block_tables: torch.Tensor, pos: torch.Tensor, seq_of: torch.Tensor,
-                     heads: int, window: int, chunk: int, scale: float, slope, sink, out: torch.Tensor) -> None:
+                     heads: int, window: int, chunk: int, scale: float, slope, sink, out: torch.Tensor, parts: GroupParts = NO_PARTS) -> None:
     """The same for any head size, in fp32 arithmetic whatever the dtype of the rows and caches."""
     n, G, bs, dk, dv = _group_shape(q, k_cache, v_cache, out, heads, slope, sink)
     for t in (block_tables, pos, seq_of):
         assert t.dtype == torch.int32
     assert pos.numel() >= q.shape[0] and seq_of.numel() >= q.shape[0]
+    form = _group_form(window, chunk, scale, slope, sink, parts, q, k_cache, v_cache, heads)
     _check(load_library().glm_group_attn_plain(
-        _p(q), q.stride(0), _p(k_cache), _p(v_cache), n, bs, _p(block_tables), block_tables.stride(0), _p(pos), _p(seq_of), q.shape[0], heads, G, dk, dv, window,
-        chunk, scale, _p(slope), _p(sink), _p(out), out.stride(0), _is_f32(q.dtype), _stream()), "glm_group_attn_plain")
+        _p(q), q.stride(0), _p(k_cache), _p(v_cache), n, bs, _p(block_tables), block_tables.stride(0), _p(pos), _p(seq_of), q.shape[0], heads, G, dk, dv,
+        ctypes.byref(form), _p(out), out.stride(0), _is_f32(q.dtype), _stream()), "glm_group_attn_plain")
+
+
+def group_rotate_store(x: torch.Tensor, q_off: int, k_off: int, v_off: int, heads: int, maps: int, dims: int, cs: torch.Tensor, slots: torch.Tensor,
+                       k_cache: torch.Tensor, v_cache: torch.Tensor) -> None:
+    """Rows of a projection: queries at q_off are rotated in place (column i < dims / 2 of a head's map with column i + dims / 2, table cs of
+    rope_pairs), rotated keys at k_off and the values at v_off go to their cache rows [blocks, G, block size, maps * columns | value columns]."""
+    n, G, bs, dk = k_cache.shape
+    dv, T = v_cache.shape[3], x.shape[0]
+    assert v_cache.shape[:3] == (n, G, bs) and k_cache.dtype == v_cache.dtype == x.dtype and k_cache.is_contiguous() and v_cache.is_contiguous() and x.stride(1) == 1
+    assert slots.dtype == torch.int32 and slots.numel() == T and cs.dtype == torch.float32 and cs.shape[0] == T and cs.is_contiguous() and dk % maps == 0
+    assert max(q_off + heads * dk, k_off + G * dk, v_off + G * dv) <= x.shape[1]
+    _check(load_library().glm_group_rotate_store(_p(x), x.stride(0), q_off, k_off, v_off, _is_f32(x.dtype), heads, G, maps, dk // maps, dv, dims, _p(cs), cs.shape[1],
+                                                 _p(slots), T, _p(k_cache), _p(v_cache), n * bs, bs, _stream()), "glm_group_rotate_store")
+
+
+def group_norm_store(x: torch.Tensor, q_off: int, k_off: int, gain: torch.Tensor, q_true: int, k_cols: int, k_true: int, first: int, eps: float, pos: torch.Tensor,
+                     slots: torch.Tensor, cache: torch.Tensor, kscale: torch.Tensor, temperature: tuple = (0.0, 0)) -> None:
+    """Rows of a projection whose keys are the values: queries at q_off (as many columns as gain, q_true of them true) <- q / rms(q) gain, times
+    1 + coef ln(floor((p + 1) / every) + 1) with temperature = (coef, every); key heads `first`.. of the k_cols columns at k_off go to the
+    cache as they are, 1 / rms of all of them (k_true true ones) to kscale."""
+    n, G, bs, dm = cache.shape
+    T = x.shape[0]
+    assert cache.dtype == x.dtype and cache.is_contiguous() and x.stride(1) == 1 and gain.dtype == torch.float32 and gain.is_contiguous()
+    assert kscale.dtype == torch.float32 and kscale.is_contiguous() and kscale.numel() == n * bs
+    assert pos.dtype == slots.dtype == torch.int32 and pos.numel() == slots.numel() == T and max(q_off + gain.numel(), k_off + k_cols) <= x.shape[1]
+    _check(load_library().glm_group_norm_store(_p(x), x.stride(0), q_off, gain.numel(), q_true, k_off, k_cols, k_true, _is_f32(x.dtype), _p(gain), dm, first, G, eps,
+                                               *temperature, _p(pos), _p(slots), T, _p(cache), _p(kscale), n * bs, bs, _stream()), "glm_group_norm_store")
+
+
+def residual_norm(x: torch.Tensor | None, width: int, wp: int, eps: float, y=None, embed: tuple | None = None, g: torch.Tensor | None = None, rows: torch.Tensor | None = None,
+                  act_dtype=torch.bfloat16, keep_x: bool = True):
+    """Between two layers (glm_residual_norm): returns (x_out, h) with x_out = x + y + rows of an embedding table and h its norm with gain g (None: no
+    h).  y: [T, wp] in bf16, fp32 or a PartialSum; embed: (ids, table); rows: gather of rows."""
+    T = rows.numel() if rows is not None else (x.shape[0] if x is not None else embed[0].numel())
+    dev = embed[1].device if x is None else x.device
+    assert x is None or (x.dtype == torch.float32 and x.is_contiguous() and x.shape[1] == wp)
+    yp, ldy, y_f32, ns, sstride = None, wp, 0, 1, 0
+    if y is not None:
+        t = y.part if isinstance(y, PartialSum) else y
+        assert t.shape[-1] == wp and t.is_contiguous() and (x is None or t.shape[-2] == x.shape[0])
+        yp, y_f32 = _p(t), _is_f32(t.dtype)
+        if isinstance(y, PartialSum):
+            ns, sstride = t.shape[0], t.shape[1] * t.shape[2]
+    ids, table = embed or (None, None)
+    if embed is not None:
+        assert ids.dtype == torch.int64 and ids.is_contiguous() and table.stride(1) == 1 and table.shape[1] >= wp and table.dtype == act_dtype
+        assert x is None or ids.numel() == x.shape[0]
+    assert rows is None or rows.dtype == torch.int32
+    assert g is None or (g.dtype == torch.float32 and g.numel() == wp)
+    x_out = torch.empty((T, wp), dtype=torch.float32, device=dev) if keep_x else None
+    h = torch.empty((T, wp), dtype=act_dtype, device=dev) if g is not None else None
+    _check(load_library().glm_residual_norm(_p(x), _p(rows), yp, ldy, y_f32, ns, sstride, _p(table), table.stride(0) if table is not None else wp,
+                                            table.shape[0] if table is not None else 0, _p(ids), _p(x_out), _p(g), _p(h), wp, _is_f32(act_dtype), T, width, wp, eps, _stream()),
+           "glm_residual_norm")
+    return x_out, h
 
 
 MEMORY_CHUNK_MAX_DIM = 256   # key size of glm_memory_chunkwise

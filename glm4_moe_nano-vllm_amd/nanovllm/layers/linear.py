@@ -189,5 +189,5 @@ class PaddedLinear(nn.Module):
         self.weight = hip_ops.padded_weight(self.N, self.K, dtype=self.dtype, device=device)
         self.weight.copy_(full)
 
-    def forward(self, x: torch.Tensor, bias: torch.Tensor | None = None, act=hip_ops.NO_ACT, out_f32: bool = False) -> torch.Tensor:
-        return hip_ops.linear_act(x, self.weight, bias, act, out_f32)
+    def forward(self, x: torch.Tensor, bias: torch.Tensor | None = None, act=hip_ops.NO_ACT, out_f32: bool = False, out: torch.Tensor | None = None) -> torch.Tensor:
+        return hip_ops.linear_act(x, self.weight, bias, act, out_f32, out)

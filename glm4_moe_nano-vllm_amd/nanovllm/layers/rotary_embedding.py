@@ -2,8 +2,8 @@
 layers/rotary_embedding.py:17-71.  The cos/sin table is built on the host with the same torch
 ops as the reference (so the table is bit-identical); the rotation is glm_rope_neox.
 
-PairRotary: rotation of neighbouring columns, with YaRN's scaling, for models that run step batches (no counterpart in the
-reference)."""
+StepRotation, PairRotary, HalfRotary: rotations of neighbouring columns (with YaRN's scaling) or of columns half the rotated part apart,
+for models that run step batches (no counterpart in the reference)."""
 from __future__ import annotations
 
 import math
@@ -57,20 +57,13 @@ def yarn_frequencies(base: float, dims: int, factor: float, original: float, fas
     return freq
 
 
-class PairRotary:
-    """Rotation of the column pairs (2i, 2i+1), i < dims / 2, of a head's rotated part of rot_dim columns (the rest do not turn).  The
-    table of a step is made on the device from its positions, so no length is built in; layers with the same rotation share it."""
+class StepRotation:
+    """A rotation whose table is made on the device from a step's positions, so no length is built in; layers with the same rotation share
+    it (`key`).  freq: frequency of every pair that turns; pairs: pairs of the table."""
 
-    def __init__(self, rot_dim: int, dims: int, base: float, scaling: dict | None = None):
-        if dims % 2 or rot_dim % 2 or not 0 < dims <= rot_dim:
-            raise ValueError(f"a rotation of {dims} of {rot_dim} columns")
-        self.pairs = hip_ops.round8(rot_dim) // 2
-        if scaling is None:
-            self.freq, self.mscale = tuple(base ** (-2.0 * i / dims) for i in range(dims // 2)), 1.0
-        else:
-            self.freq = tuple(yarn_frequencies(base, dims, *(scaling[k] for k in ("factor", "original", "fast", "slow"))))
-            self.mscale = 0.1 * math.log(scaling["factor"]) + 1.0
-        self.key = (self.pairs, self.freq, self.mscale)
+    def __init__(self, freq: tuple, mscale: float, pairs: int):
+        self.freq, self.mscale, self.pairs = freq, mscale, pairs
+        self.key = (pairs, freq, mscale)
         self._dev = {}
 
     def prepare(self, device) -> None:
@@ -81,3 +74,33 @@ class PairRotary:
     def table(self, pos: torch.Tensor) -> torch.Tensor:
         """cos, sin [T, pairs, 2] at the positions of a step."""
         return hip_ops.rope_pairs(pos, self._dev[pos.device], self.mscale, self.pairs)
+
+    def shared_table(self, pos: torch.Tensor, tables: dict) -> torch.Tensor:
+        """The table of a step, made once for all layers with this rotation (`tables`: of the step)."""
+        if self.key not in tables:
+            tables[self.key] = self.table(pos)
+        return tables[self.key]
+
+
+class PairRotary(StepRotation):
+    """Rotation of the column pairs (2i, 2i+1), i < dims / 2, of a head's rotated part of rot_dim columns (the rest do not turn)."""
+
+    def __init__(self, rot_dim: int, dims: int, base: float, scaling: dict | None = None):
+        if dims % 2 or rot_dim % 2 or not 0 < dims <= rot_dim:
+            raise ValueError(f"a rotation of {dims} of {rot_dim} columns")
+        if scaling is None:
+            freq, mscale = tuple(base ** (-2.0 * i / dims) for i in range(dims // 2)), 1.0
+        else:
+            freq = tuple(yarn_frequencies(base, dims, *(scaling[k] for k in ("factor", "original", "fast", "slow"))))
+            mscale = 0.1 * math.log(scaling["factor"]) + 1.0
+        super().__init__(freq, mscale, hip_ops.round8(rot_dim) // 2)
+
+
+class HalfRotary(StepRotation):
+    """Rotation of the column pairs (i, i + dims / 2), i < dims / 2, of a head of dim columns (those from dims on do not turn)."""
+
+    def __init__(self, dim: int, dims: int, base: float):
+        if dims % 2 or not 0 < dims <= dim:
+            raise ValueError(f"a rotation of {dims} of {dim} columns")
+        self.dims = dims
+        super().__init__(tuple(base ** (-2.0 * i / dims) for i in range(dims // 2)), 1.0, dims // 2)

@@ -7,6 +7,7 @@ import types
 import torch
 
 from nanovllm.hip_ops import round8
+from nanovllm.models.layer_loop import layer_runs, read_loop  # noqa: F401
 
 MAX_POSITIONS = 1 << 30  # attention has no positional term: nothing limits a sequence but memory
 
@@ -35,26 +36,10 @@ def _layer(i: int, e: dict) -> LayerSpec:
 def read_config(raw: dict) -> types.SimpleNamespace:
     d = raw if isinstance(raw, dict) else dict(vars(raw))
     layers = [_layer(i, e) for i, e in enumerate(d["layers"])]
-    loop = d.get("loop")
-    if loop is not None:
-        loop = types.SimpleNamespace(start=int(loop["start"]), stop=int(loop["stop"]), times=int(loop["times"]))
-        if not 0 <= loop.start < loop.stop <= len(layers) or loop.times < 1:
-            raise ValueError(f"loop {vars(loop)} does not fit {len(layers)} layers")
+    loop = read_loop(d.get("loop"), len(layers))
     cap = d.get("logit_softcap")
     return types.SimpleNamespace(
         raw=d, model_type="dafolorn", vocab_size=int(d["vocab"]), hidden_size=int(d["width"]), padded_width=round8(int(d["width"])),
         layers=layers, loop=loop, rms_norm_eps=float(d["norm"]["eps"]), conv_taps=int(d["canon"]["taps"]),
         logit_softcap=None if cap is None else float(cap), num_hidden_layers=len(layers), max_position_embeddings=MAX_POSITIONS,
         max_window=max(s.window for s in layers), torch_dtype=torch.bfloat16)
-
-
-def layer_runs(cfg) -> list:
-    """The layers in the order they run: (layer index, pass number if this is the first layer of a pass else None)."""
-    n = len(cfg.layers)
-    if cfg.loop is None:
-        return [(i, None) for i in range(n)]
-    lo, hi = cfg.loop.start, cfg.loop.stop
-    runs = [(i, None) for i in range(lo)]
-    for t in range(cfg.loop.times):
-        runs += [(i, t if i == lo else None) for i in range(lo, hi)]
-    return runs + [(i, None) for i in range(hi, n)]

@@ -14,8 +14,8 @@ from nanovllm.layers.dense_mlp import DenseMLP
 from nanovllm.layers.latent_attention import LatentAttention
 from nanovllm.layers.linear import PaddedLinear
 from nanovllm.layers.seq_norm import SublayerEntry, norm_gain
+from nanovllm.models.layer_loop import layer_runs, run_indices
 from nanovllm.utils.loader import load_prefixed
-from .config import layer_runs
 
 
 class DafolornLayer(nn.Module):
@@ -57,11 +57,7 @@ class DafolornForCausalLM(nn.Module):
         self.config = config
         self.dtype = config.torch_dtype
         self.runs = layer_runs(config)
-        count = [0] * len(config.layers)
-        self.run_index = []          # which run of its layer an entry of self.runs is
-        for i, _ in self.runs:
-            self.run_index.append(count[i])
-            count[i] += 1
+        self.run_index, count = run_indices(config)
         self.layers = nn.ModuleList([DafolornLayer(config, s, count[s.index]) for s in config.layers])
         w = config.hidden_size
         self.loop_in = PaddedLinear([w, w], [config.padded_width], self.dtype) if config.loop else None

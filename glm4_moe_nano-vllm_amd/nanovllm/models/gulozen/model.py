@@ -130,10 +130,7 @@ class GulozenForCausalLM(nn.Module):
     def _mix(self, layer, h, meta, tables):
         if isinstance(layer.mixer, LinearAttention):
             return layer.mixer(h, meta)
-        rot = layer.mixer.rot
-        if rot.key not in tables:    # one table for all layers with the same rotation
-            tables[rot.key] = rot.table(meta.pos)
-        return layer.mixer(h, meta, cs=tables[rot.key])
+        return layer.mixer(h, meta, cs=layer.mixer.rot.shared_table(meta.pos, tables))
 
     def forward(self, meta, residual_tap: list | None = None) -> torch.Tensor:
         """fp32 logits [meta.want_rows, vocab] of the wanted rows of a step.  residual_tap (a list) receives what every layer hands on

@@ -37,8 +37,10 @@ NAPADRA = ModelEntry("napadra", "nanovllm.models.napadra.config:read_config", "n
                      64, 64, ("bfloat16", "float32"), "napadra", True)
 GULOZEN = ModelEntry("gulozen", "nanovllm.models.gulozen.config:read_config", "nanovllm.models.gulozen.model:GulozenForCausalLM",
                      64, 32, ("bfloat16", "float32"), "gulozen", True)
+LOSELIX = ModelEntry("loselix", "nanovllm.models.loselix.config:read_config", "nanovllm.models.loselix.model:LoselixForCausalLM",
+                     64, 64, ("bfloat16", "float32"), "loselix", True)
 
-_ENTRIES = {e.name: e for e in (GLM4_MOE, DAFOLORN, NAPADRA, GULOZEN)}
+_ENTRIES = {e.name: e for e in (GLM4_MOE, DAFOLORN, NAPADRA, GULOZEN, LOSELIX)}
 
 
 def find_model(cfg) -> ModelEntry:

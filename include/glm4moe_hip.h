@@ -499,6 +499,7 @@ int glm_allreduce_oneshot(const void* in, void* out, void* const* peer_bufs, voi
 #define GLM_EPI_GLU_CLAMP 3 /* glm_gemm_bf16_glu only */
 #define GLM_EPI_GATE      4 /* columns below a: z; the others: sigmoid(z) */
 #define GLM_EPI_SILU_GATE 5 /* columns below a: z sigmoid(z); the others: sigmoid(z) */
+#define GLM_EPI_RELU2_GATE 6 /* columns below a: relu(z)^2; those below b: z; the others: sigmoid(z) */
 /* y = act(x . W^T + bias): glm_gemm_bf16 with an activation in the epilogue and, with out_f32, fp32 output rows (unrounded).  */
 int glm_gemm_bf16_act(const void* x, int64_t ldx, const void* w, int64_t ldw, const void* bias, void* y, int64_t ldy, int64_t M,
                       int N, int K, int out_f32, int act, float act_a, float act_b, glm_stream_t stream);
@@ -546,28 +547,60 @@ int glm_stream_norm(const float* x_in, int64_t ldx, int64_t sx, const int32_t* r
 /* Causal attention of H query heads over G key / value heads in paged caches [n_blocks][G][block_size][dk | dv] (block_size % 64 == 0;
  * dk, dv multiples of 8).  A row at position p sees j <= p with p - j < window (window > 0) and in its own chunk of `chunk` positions
  * (chunk > 0); score = scale q.k - slope[h] (p - j) (slope may be NULL); softmax with the extra mass exp(sink[h]) (sink may be NULL).
+ * Further parts: glm_group_form.
  * store: key / value columns of projection rows -> cache rows slots[t] (< 0: none).
- * prefill: tiles (sequence, first row inside the portion) of tile_rows rows (128; 64 if H/G is even) of portions [q_start[s], q_start[s+1]), block table row seq0 + s.
- * decode: tiles of tile_n[i] <= tokens_per_tile rows of one sequence from tile_tok[i]; nsplit > 1: unnormalised sums part_o
- * [rows*H, nsplit, dv] and part_ml [rows*H, nsplit, 2] for glm_attn_merge; knew / vnew (may be NULL): keys and values of the rows of q,
+ * prefill: tiles (sequence, first row inside the portion) of tile_rows rows (128; 64 if H/G is even or a head has two maps) of portions [q_start[s], q_start[s+1]), block table row seq0 + s.
+ * decode: tiles of tile_n[i] <= tokens_per_tile rows of one sequence from tile_tok[i]; nsplit > 1 or two maps: unnormalised sums part_o
+ * [rows*H*maps, nsplit, dv] and part_ml [rows*H*maps, nsplit, 2] for glm_attn_merge; knew / vnew (may be NULL): keys and values of the rows of q,
  * head g at g*dk / g*dv, read instead of the cache's and stored to cache rows `slots`.  Both bf16, dk, dv <= 256, scale > 0.  plain: any size, bf16 or fp32.  */
+typedef struct {
+    int window, chunk;
+    float scale;
+    const float *slope, *sink;
+    float cap;            /* score <- cap tanh(score / cap); 0: none */
+    int maps;             /* 1, or 2: a head's dk columns are two queries / keys side by side over the same values, and its output is
+                             post d / sqrt(mean(d^2) + eps) with d = o_1 - lam o_2, the mean over vn columns */
+    float lam, post, eps;
+    int vn;
+    int sigmoid;          /* weights sigmoid(score + bias[h]), not normalised */
+    const float* bias;    /* [H] or NULL */
+    const float* kscale;  /* sigmoid: the keys are the values (kc == vc) and a key's products are multiplied by kscale[cache row]; or NULL */
+    const void* gate;     /* output factors in the activation dtype, row t at t*ldg: head h at h, or with gate_cols at h*dv + column; or NULL */
+    int64_t ldg;
+    int gate_cols;
+} glm_group_form;
 int glm_group_kv_store(const void* src, int64_t ld, int64_t k_off, int64_t v_off, int f32, const int32_t* slots, int64_t T,
                        void* kc, void* vc, int64_t n_slots, int bs, int G, int dk, int dv, glm_stream_t stream);
 int glm_group_attn_prefill(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs,
                            const int32_t* block_tables, int64_t bt_stride, int seq0, const int32_t* q_start, const int32_t* pos,
                            const int32_t* tile_seq, const int32_t* tile_off, int n_tiles, int tile_rows, int H, int G, int dk,
-                           int dv, int window, int chunk, float scale, const float* slope, const float* sink, void* out, int64_t ldo,
-                           glm_stream_t stream);
+                           int dv, const glm_group_form* form, void* out, int64_t ldo, glm_stream_t stream);
 int glm_group_attn_decode(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs,
                           const int32_t* block_tables, int64_t bt_stride, const int32_t* pos, const int32_t* seq_of,
                           const int32_t* tile_tok, const int32_t* tile_n, int n_tiles, int tokens_per_tile, int H, int G, int dk,
-                          int dv, int window, int chunk, float scale, const float* slope, const float* sink, const void* knew,
+                          int dv, const glm_group_form* form, const void* knew,
                           const void* vnew, int64_t ldkv, const int32_t* q_start, const int32_t* slots, void* out, int64_t ldo,
                           int nsplit, float* part_o, float* part_ml, glm_stream_t stream);
 int glm_group_attn_plain(const void* q, int64_t ldq, const void* kc, const void* vc, int64_t n_blocks, int bs,
                          const int32_t* block_tables, int64_t bt_stride, const int32_t* pos, const int32_t* seq_of, int64_t rows,
-                         int H, int G, int dk, int dv, int window, int chunk, float scale, const float* slope, const float* sink,
-                         void* out, int64_t ldo, int f32, glm_stream_t stream);
+                         int H, int G, int dk, int dv, const glm_group_form* form, void* out, int64_t ldo, int f32,
+                         glm_stream_t stream);
+/* Rows of a projection on their way into that attention.  rotate_store: column i < dims / 2 of a head (of each map) turns with column i + dims / 2
+ * by the table cs [T, pairs, 2] of glm_rope_pairs; H*maps query heads of dm columns at q_off stay where they are, G*maps keys at k_off and G
+ * values at v_off go to cache rows slots[t].  norm_store (keys are values, one map): queries <- q / rms(q) gq (1 + coef ln(floor((p + 1) / every) + 1)),
+ * the mean over q_n of nq columns; kscale[slots[t]] = 1 / rms of the nk key columns (k_n true ones); key heads [g0, g0 + G) go to the cache as they are. */
+int glm_group_rotate_store(void* x, int64_t ld, int q_off, int k_off, int v_off, int f32, int H, int G, int maps, int dm, int dv,
+                           int dims, const float* cs, int pairs, const int32_t* slots, int64_t T, void* kc, void* vc,
+                           int64_t n_slots, int bs, glm_stream_t stream);
+int glm_group_norm_store(void* x, int64_t ld, int q_off, int nq, int q_n, int k_off, int nk, int k_n, int f32, const float* gq,
+                         int dm, int g0, int G, float eps, float coef, int every, const int32_t* pos, const int32_t* slots,
+                         int64_t T, void* kc, float* kscale, int64_t n_slots, int bs, glm_stream_t stream);
+
+/* Between two layers: x_out = x_in + y + table[ids] (each optional; y bf16, or the sum of n_slabs fp32 slabs; table in the activation
+ * dtype), h = x_out / rms(x_out) g (optional).  Rows of pitch wp; rows (or NULL) gathers x_in, y and ids.                        */
+int glm_residual_norm(const float* x_in, const int32_t* rows, const void* y, int64_t ldy, int y_f32, int n_slabs, int64_t slab_stride,
+                      const void* table, int64_t ldt, int64_t vocab, const int64_t* ids, float* x_out, const float* g, void* h,
+                      int64_t ldh, int act_f32, int64_t T, int width, int wp, float eps, glm_stream_t stream);
 
 /* Gated matrix memory (mLSTM; the recurrence is written out in csrc/matrix_memory.hip).  Projection rows x hold q at h*dimp, k at
  * k_off + h*dimp, v at v_off + h*vdimp and the output gate at g_off + h*vdimp.  State rows S [n_state][H][dimp][vdimp], n
@@ -659,8 +692,9 @@ int glm_latent_attn(const void* qa, const void* cache, int64_t n_blocks, int blo
                     const int32_t* tile_n, int n_tiles, int tokens_per_tile, const int32_t* pos, const int32_t* seq_of,
                     const int32_t* block_tables, int64_t bt_stride, int64_t Ta, int H, int rp, int vp, int window, float scale,
                     const float* sink, int nsplit, void* ctx, float* part_o, float* part_ml, int act_f32, glm_stream_t stream);
-int glm_attn_merge(const float* part_o, const float* part_ml, const float* sink, int nsplit, void* ctx, int64_t Ta, int H, int cols,
-                   glm_stream_t stream);
+/* sum of the splits, finished: row (t, h) to out[t*ldo + h*cols]; sink may be NULL; form (or NULL): what of it concerns the result */
+int glm_attn_merge(const float* part_o, const float* part_ml, const float* sink, int nsplit, void* out, int64_t ldo, int64_t Ta, int H,
+                   int cols, const glm_group_form* form, glm_stream_t stream);
 int glm_latent_up(const void* ctx, const void* wuv, void* out, const void* gate, int64_t ldg, int64_t ldo, int64_t Ta, int H, int vdimp, int rp,
                   glm_stream_t stream);
 /* Prompts and long portions, bf16: q rows [q_start[s], q_start[s+1]) against expanded k / v rows [k_start[s], k_start[s+1]) — the
