@@ -115,8 +115,8 @@ def main():
                     help="BASELINE config 4 flavour: the experts are partitioned over the ranks (E/N each, full intermediate "
                          "size) and token rows travel by an all-to-all of fixed-capacity slots planned on the device "
                          "(graph-capturable); attention stays tensor-parallel.  The headline run is the default (TP only)")
-    ap.add_argument("--design", choices=("glm4_moe", "dafolorn", "napadra", "gulozen"), default="glm4_moe",
-                    help="dafolorn, napadra, gulozen: prefill / decode and per-kernel numbers of that design beside GLM layers of equal size (bench_<design>.py)")
+    ap.add_argument("--design", choices=("glm4_moe", "dafolorn", "napadra", "gulozen", "loselix"), default="glm4_moe",
+                    help="dafolorn, napadra, gulozen, loselix: prefill / decode and per-kernel numbers of that design beside GLM layers of equal size (bench_<design>.py)")
     ap.add_argument("--design-sizes", default="", help="with another design: comma-separated sizes")
     ap.add_argument("--probe-capture", action="store_true", help=argparse.SUPPRESS)
     ap.add_argument("--graph-body-only", action="store_true",
@@ -137,6 +137,9 @@ def main():
     if args.design == "gulozen":
         import bench_gulozen
         return bench_gulozen.run(args)
+    if args.design == "loselix":
+        import bench_loselix
+        return bench_loselix.run(args)
 
     if args.gpus > 1 and "WORLD_SIZE" not in os.environ:
         # plain `python bench.py --gpus N`: this process becomes the launcher.  It has not touched a GPU (importing

@@ -237,8 +237,6 @@ def test_group_attention(H, G, dk, dv, window, chunk, bs, kind):
         elif kind.startswith("plain"):
             hip_ops.group_attn_plain(*args, pos, seq_of, *form, out)
         else:
-            if kind == "decode1_split" and sink is None:
-                continue
             per = max(1, min(max(n_q), hip_ops.GROUP_ATTN_ROWS // (H // G)))   # (five rows of a portion may be several tiles)
             tok = [qs[s] + o for s, n in enumerate(n_q) for o in range(0, n, per)]
             cnt = [min(per, n - o) for n in n_q for o in range(0, n, per)]
