@@ -263,6 +263,17 @@ extern "C" int glm_gemm_bf16_router_tail(const void* x, const void* w, int64_t l
 
 extern "C" int glm_gemm_bf16_partial_slices(int K, int want) { return glm_smallm_partial_slices(K, want); }
 
+// more rows than the weight-streaming kernel splits K for: equal slices of whole K tiles, as many as bring the launch to a workgroup per CU
+extern "C" int glm_gemm_bf16_slices(int64_t M, int N, int K) {
+    if (M < LARGEM_MIN_AVG_ROWS || K % 64 != 0) return 1;
+    const int rows = M >= 192 ? 256 : 128;
+    const int64_t tiles = (M + rows - 1) / rows * ((N + 255) / 256);
+    int best = 1;
+    for (int s = 2; s <= 16 && s * tiles <= 256 && K / s >= 512; ++s)
+        if (K % (64 * s) == 0) best = s;
+    return best;
+}
+
 extern "C" int glm_gemm_bf16_partial(const void* x, int64_t ldx, const void* w, int64_t ldw, float* ypart,
                                      int64_t M, int N, int K, int nslices, glm_stream_t stream) {
     GLM_CHECK_ARG(x && w && ypart, GLM_ERR_INVALID, "glm_gemm_bf16_partial: null pointer");
@@ -274,6 +285,12 @@ extern "C" int glm_gemm_bf16_partial(const void* x, int64_t ldx, const void* w, 
     p.x = (const bf16_t*)x; p.ldx = ldx;
     p.w = (const bf16_t*)w; p.w_gstride = 0; p.ldw = ldw;
     p.R = M; p.N = N; p.K = K; p.G = 1;
+    if (M >= LARGEM_MIN_AVG_ROWS) {
+        GLM_CHECK_ARG(K % (64 * nslices) == 0 && glm_aligned16(ypart) && N % 8 == 0, GLM_ERR_UNSUPPORTED, "glm_gemm_bf16_partial: K=%d in %d slices of whole tiles", K, nslices);
+        p.K = K / nslices; p.G = nslices; p.w_gstride = p.K;
+        p.yf = ypart; p.y = (bf16_t*)ypart; p.ldy = N;  // (y: alignment checks only)
+        return glm_launch_gemm_largem(GEMM_SLICES, p, glm_s(stream));
+    }
     p.ksplit = nslices; p.ypart = ypart;
     return glm_launch_gemm_smallm_partial(p, glm_s(stream));
 }

@@ -21,9 +21,11 @@ struct MergeArgs {
     int vn;
 };
 
-// sum over the KV splits of one row's columns k .. k + 4, each split brought to the common maximum, over the mass of all and the sink's:
-// sixteen splits in flight
-__device__ __forceinline__ f32x4_t merge_row(const MergeArgs& a, int64_t prow, int h, int k, int lane) {
+// The splits of one row, sixteen in flight: this wave adds up splits w, w + WPR, ... of the row's columns k .. k + 4, each weighed with its
+// share of the row's mass (brought to the common maximum, over the mass of all and the sink's)
+template <int WPR>
+__device__ __forceinline__ f32x4_t merge_row(const MergeArgs& a, int64_t prow, int h, int k, int lane, int w) {
+    constexpr int N = WPR == 1 ? 16 : 8;
     const float* p = a.part_o + prow * a.nsplit * a.cols + k;
     float m = -INFINITY, l = 0.f;
     if (lane < a.nsplit) {
@@ -32,10 +34,10 @@ __device__ __forceinline__ f32x4_t merge_row(const MergeArgs& a, int64_t prow, i
     }
     f32x4_t o = {0.f, 0.f, 0.f, 0.f};
     float f = 0.f;
-    for (int s0 = 0; s0 < a.nsplit; s0 += 16) {
-        f32x4_t x[16];
+    for (int s0 = 0; s0 < a.nsplit; s0 += N * WPR) {
+        f32x4_t x[N];
 #pragma unroll
-        for (int j = 0; j < 16; ++j) x[j] = *reinterpret_cast<const f32x4_t*>(p + (int64_t)min(s0 + j, a.nsplit - 1) * a.cols);
+        for (int j = 0; j < N; ++j) x[j] = *reinterpret_cast<const f32x4_t*>(p + (int64_t)min(s0 + j * WPR + w, a.nsplit - 1) * a.cols);
         if (s0 == 0) {
             const float sk = a.sink ? a.sink[h] * LOG2E : -INFINITY;
             const float M = fmaxf(wave_max(m), sk);
@@ -44,8 +46,9 @@ __device__ __forceinline__ f32x4_t merge_row(const MergeArgs& a, int64_t prow, i
             f = a.plain_sum ? (l > 0.f ? 1.0f : 0.f) : mass > 0.f ? e / mass : 0.f;  // 0: an empty split, its sums were never written
         }
 #pragma unroll
-        for (int j = 0; j < 16; ++j) {
-            const float fs = s0 + j < a.nsplit ? __shfl(f, s0 + j, 64) : 0.f;
+        for (int j = 0; j < N; ++j) {
+            const int s = s0 + j * WPR + w;
+            const float fs = s < a.nsplit ? __shfl(f, s, 64) : 0.f;
             if (fs != 0.f) {
 #pragma unroll
                 for (int i = 0; i < 4; ++i) o[i] += fs * x[j][i];
@@ -55,27 +58,44 @@ __device__ __forceinline__ f32x4_t merge_row(const MergeArgs& a, int64_t prow, i
     return o;
 }
 
-// one wave per (token, head) and 256 columns; two maps: all columns of a head in one wave
-template <bool TWO>
+// WPR waves (1 or 4) per (token, head) and 256 columns; two maps: all columns of a head together
+template <bool TWO, int WPR>
 __global__ __launch_bounds__(256) void attn_merge_kernel(const MergeArgs a) {
-    const int lane = threadIdx.x & 63;
-    const int64_t item = (int64_t)blockIdx.x * 4 + (threadIdx.x >> 6);
+    __shared__ f32x4_t sums[WPR == 1 ? 1 : (TWO ? 2 : 1) * (WPR - 1)][64];
+    const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
+    const int64_t item = WPR == 1 ? (int64_t)blockIdx.x * 4 + w : (int64_t)blockIdx.x;
     const int64_t grow = item / a.nchunk, t = grow / a.H;
     if (grow >= a.rows) return;
-    const int k = (int)(item % a.nchunk) * 256 + lane * 4, h = (int)(grow - t * a.H);
+    const int k = (int)(item % a.nchunk) * 256 + lane * 4, h = (int)(grow - t * a.H), kk = k < a.cols ? k : 0;
     const bool on = k < a.cols;
-    f32x4_t o;
+    f32x4_t o, y;
     if constexpr (TWO) {
-        const f32x4_t x = merge_row(a, grow * 2, h, on ? k : 0, lane), y = merge_row(a, grow * 2 + 1, h, on ? k : 0, lane);
+        o = merge_row<WPR>(a, grow * 2, h, kk, lane, WPR == 1 ? 0 : w);
+        y = merge_row<WPR>(a, grow * 2 + 1, h, kk, lane, WPR == 1 ? 0 : w);
+    } else {
+        o = merge_row<WPR>(a, grow, h, kk, lane, WPR == 1 ? 0 : w);
+    }
+    if constexpr (WPR > 1) {
+        if (w > 0) {
+            sums[w - 1][lane] = o;
+            if constexpr (TWO) sums[WPR - 1 + w - 1][lane] = y;
+        }
+        __syncthreads();
+        if (w > 0) return;
+#pragma unroll
+        for (int i = 0; i < WPR - 1; ++i) {
+            o += sums[i][lane];
+            if constexpr (TWO) y += sums[WPR - 1 + i][lane];
+        }
+    }
+    if constexpr (TWO) {
         float ss = 0.f;
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-            o[i] = x[i] - a.lam * y[i];
+            o[i] = o[i] - a.lam * y[i];
             ss += on ? o[i] * o[i] : 0.f;
         }
         o *= a.post / sqrtf(wave_sum(ss) / (float)a.vn + a.eps);
-    } else {
-        o = merge_row(a, grow, h, on ? k : 0, lane);
     }
     if (!on) return;
     if (a.gate) {
@@ -84,6 +104,14 @@ __global__ __launch_bounds__(256) void attn_merge_kernel(const MergeArgs a) {
         for (int i = 0; i < 4; ++i) o[i] *= bf2f(a.gate_cols ? g[i] : g[0]);
     }
     *reinterpret_cast<u32x2_t*>(a.out + t * a.ldo + (int64_t)h * a.cols + k) = u32x2_t{pack2bf(o[0], o[1]), pack2bf(o[2], o[3])};
+}
+
+template <int WPR>
+void launch(const MergeArgs& a, int maps, hipStream_t st) {
+    const int64_t items = a.rows * a.nchunk;
+    const dim3 grid((unsigned)(WPR == 1 ? (items + 3) / 4 : items));
+    if (maps == 2) hipLaunchKernelGGL((attn_merge_kernel<true, WPR>), grid, dim3(256), 0, st, a);
+    else hipLaunchKernelGGL((attn_merge_kernel<false, WPR>), grid, dim3(256), 0, st, a);
 }
 
 }  // namespace
@@ -102,9 +130,8 @@ extern "C" int glm_attn_merge(const float* part_o, const float* part_ml, const f
         a.gate = (const bf16_t*)form->gate; a.ldg = form->ldg; a.gate_cols = form->gate_cols;
         a.lam = form->lam; a.post = form->post; a.eps = form->eps; a.vn = form->vn;
     }
-    const dim3 grid((unsigned)((a.rows * a.nchunk + 3) / 4));
-    if (maps == 2) hipLaunchKernelGGL(attn_merge_kernel<true>, grid, dim3(256), 0, glm_s(stream), a);
-    else hipLaunchKernelGGL(attn_merge_kernel<false>, grid, dim3(256), 0, glm_s(stream), a);
+    if (a.rows * a.nchunk <= 2048 && nsplit > 4) launch<4>(a, maps, glm_s(stream));
+    else launch<1>(a, maps, glm_s(stream));
     GLM_CHECK_LAUNCH("glm_attn_merge");
     return GLM_OK;
 }

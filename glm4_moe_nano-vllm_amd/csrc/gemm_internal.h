@@ -21,6 +21,7 @@ enum GemmMode : int {
     GEMM_ACT = 3,
     GEMM_XIELU = 4,  // xIELU, bf16 rows
     GEMM_COLS = 6,   // per-column activation (glm_act_cols), bf16 rows
+    GEMM_SLICES = 7, // G slices of K side by side, K the length of one: fp32 partial sums, slab s of R rows at yf + s R ldy
     GEMM_GLU = 5,    // GEMM_GATEUP's layout (W rows gate|up) with the clamped gated unit of p.act instead of SiLU; fp32 up to the store
 };
 __host__ __device__ constexpr bool gemm_paired(int mode) { return mode == GEMM_GATEUP || mode == GEMM_GLU; }
@@ -177,9 +178,10 @@ __device__ __forceinline__ void glm_locate_block(const int32_t* __restrict__ off
     const int tid = threadIdx.x;
     if (offs == nullptr) {
         if (tid == 0) {
-            const int64_t m0 = (int64_t)target * MB;
-            if (m0 < R) {
-                sh[0] = 0;
+            const int nb = (int)((R + MB - 1) / MB);  // (all groups have the R rows)
+            const int64_t m0 = (int64_t)(target % nb) * MB;
+            if (target < nb * G) {
+                sh[0] = target / nb;
                 sh[1] = (int)m0;
                 sh[2] = (int)((R - m0) < MB ? (R - m0) : MB);
             } else {

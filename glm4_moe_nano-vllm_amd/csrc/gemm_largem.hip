@@ -251,10 +251,11 @@ __device__ __forceinline__ void lm_locate_wave(const int32_t* __restrict__ offs,
     g = -1;
     m0 = 0;
     cnt = 0;
-    if (offs == nullptr) {
-        const int64_t r0 = (int64_t)target * MB;
-        if (r0 < R) {
-            g = 0;
+    if (offs == nullptr) {  // all groups have the R rows (one group, or the K slices of GEMM_SLICES)
+        const int nb = (int)((R + MB - 1) / MB);
+        const int64_t r0 = (int64_t)(target % nb) * MB;
+        if (target < nb * G) {
+            g = target / nb;
             m0 = (int)r0;
             cnt = (int)((R - r0) < MB ? (R - r0) : MB);
         }
@@ -297,6 +298,7 @@ __device__ __forceinline__ void lm_locate_wave(const int32_t* __restrict__ offs,
 template <int MODE, class C, int VAR, bool WSCALE>
 __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, int n_tiles, int total_tiles, int LM_BAND) {
     constexpr bool LEAN = (VAR & LM_LEAN) != 0;
+    constexpr bool F32ROWS = MODE == GEMM_ACT || MODE == GEMM_SLICES;  // may store fp32 rows (p.yf)
     // DMA instructions of a K tile issued from the MFMA phase (the rest from the load phase)
     constexpr int S2 = !LEAN ? 0 : (VAR & LM_DMA4) ? C::DPW : (VAR & LM_DMA2) ? C::DPW / 2 : 0;
     extern __shared__ __attribute__((aligned(16))) char smem[];
@@ -422,7 +424,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
                 const int mr = row < mcnt ? row : 0;
                 const int srow = PRE ? nsrow[i] : (p.src ? p.src[m0 + mr] : m0 + mr);
                 if constexpr (C::A8) xvo[i] = (unsigned)(srow * (int)p.ldx + ch * 16);  // fp8 activations: ldx in bytes
-                else xvo[i] = (unsigned)(srow * (int)p.ldx + ch * 8) * 2u;
+                else xvo[i] = (unsigned)(srow * (int)p.ldx + (MODE == GEMM_SLICES ? grp * K : 0) + ch * 8) * 2u;
             }
             return;
         }
@@ -448,7 +450,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
             xch[i] = ch;
             const int mr = row < mcnt ? row : 0;
             const int64_t srow = p.src ? (int64_t)p.src[m0 + mr] : (int64_t)(m0 + mr);
-            xsrc[i] = p.x + srow * p.ldx + ch * 8;
+            xsrc[i] = p.x + srow * p.ldx + (MODE == GEMM_SLICES ? (int64_t)grp * K : 0) + ch * 8;
         }
     };
     const bf16_t* zero = reinterpret_cast<const bf16_t*>(g_zero_page_lm);
@@ -1562,14 +1564,15 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
                         o[r] = a;
                     }
                 }
-                if (MODE == GEMM_ACT && p.yf != nullptr) {  // fp32 rows: four columns per store
+                if (F32ROWS && p.yf != nullptr) {  // fp32 rows: four columns per store
                     const int n = ncol_w + 16 * t + 4 * g4;
-                    if (row_ok && n < p.N && !NOSTORE) *reinterpret_cast<f32x4_t*>(p.yf + (int64_t)(m0_c + row) * p.ldy + n) = f32x4_t{o[0], o[1], o[2], o[3]};
+                    const int64_t slab = MODE == GEMM_SLICES ? (int64_t)grp_c * p.R : 0;
+                    if (row_ok && n < p.N && !NOSTORE) *reinterpret_cast<f32x4_t*>(p.yf + (slab + m0_c + row) * p.ldy + n) = f32x4_t{o[0], o[1], o[2], o[3]};
                     continue;
                 }
                 v[t] = u32x2_t{pack2bf(o[0], o[1]), pack2bf(o[2], o[3])};
             }
-            if (MODE == GEMM_ACT && p.yf != nullptr) continue;
+            if (F32ROWS && p.yf != nullptr) continue;
             if (NOSTORE) {
 #pragma unroll
                 for (int t = 0; t < NOUT; ++t) asm volatile("" ::"v"(v[t][0]), "v"(v[t][1]));
@@ -1632,7 +1635,7 @@ __global__ __launch_bounds__(512) void gemm_largem_kernel(const GemmParams p, in
         if constexpr ((VAR & LM_EPIORD) != 0) {
             // exact only when every store instruction of the wave ran: all rows and columns of the tile exist
             const bool full = !LATE_FILL && mcnt_c == C::BM && ncol_w + (gemm_paired(MODE) ? 32 : 64) <= p.N && !NOSTORE &&
-                              !((VAR & LM_LDSEPI) != 0 && NOUT == 4) && !(MODE == GEMM_PLAIN && p.qkv_q != nullptr) && !(MODE == GEMM_ACT && p.yf != nullptr);
+                              !((VAR & LM_LDSEPI) != 0 && NOUT == 4) && !(MODE == GEMM_PLAIN && p.qkv_q != nullptr) && !(F32ROWS && p.yf != nullptr);
             pending_stores = full ? LM_STORES_FULL - (do_park ? PARK_N : 0) : 0;
         }
         if constexpr (PARK) {
@@ -1664,8 +1667,10 @@ template <int MODE, class C, int VAR>
 int launch_largem_cfg(const GemmParams& p, hipStream_t st) {
     const int cols_per_wg = gemm_paired(MODE) ? 128 : LM_BN;
     const int n_tiles = (p.N + cols_per_wg - 1) / cols_per_wg;
-    const int64_t combos = p.offs ? (p.R / C::BM + p.G) : (p.R + C::BM - 1) / C::BM;
-    const int LM_BAND = g_largem_band;
+    const int64_t combos = p.offs ? (p.R / C::BM + p.G) : (p.R + C::BM - 1) / C::BM * (MODE == GEMM_SLICES ? p.G : 1);
+    // (a band higher than the rows' blocks would be mostly positions without a tile: 74 tiles of one block took two rounds of 256
+    // workgroups)
+    const int LM_BAND = p.offs ? g_largem_band : (int)(combos < g_largem_band ? combos : (int64_t)g_largem_band);
     const int64_t total = (combos + LM_BAND - 1) / LM_BAND * LM_BAND * n_tiles;
     if (total <= 0) return GLM_OK;
     GLM_CHECK_ARG(total < (1ll << 31), GLM_ERR_UNSUPPORTED, "gemm_largem: grid too large");
@@ -1704,7 +1709,7 @@ template <int MODE>
 int launch_largem(const GemmParams& p, hipStream_t st) {
     // 256-row blocks pay off once a group fills most of one; smaller groups keep the 128-row tile
     const int ch = cfg_choice();
-    const int64_t avg_rows = (p.R_hint > 0 ? p.R_hint : p.R) / (p.G > 0 ? p.G : 1);
+    const int64_t avg_rows = (p.R_hint > 0 ? p.R_hint : p.R) / (p.G > 0 && MODE != GEMM_SLICES ? p.G : 1);
     // ... and a projection onto <= 128 columns (the router logits at prefill: N = E = 64) is one column tile however the rows
     // are cut, so its parallelism is its row-block count: 128-row blocks (75.8 -> 55.1 us at T = 16384)
     const bool use_b = ch == 2 || (ch == 0 && avg_rows >= 192 && !((MODE == GEMM_PLAIN || MODE == GEMM_ACT || MODE == GEMM_XIELU || MODE == GEMM_COLS) && p.offs == nullptr && p.N <= 128));
@@ -1848,6 +1853,7 @@ int glm_launch_gemm_largem(int mode, const GemmParams& p, hipStream_t st) {
 #endif  // GLM_EXPERTS
     if (mode == GEMM_ACT && p.yf == nullptr && p.act.kind >= GLM_ACT_GATE) return launch_largem<GEMM_COLS>(p, st);
     if (mode == GEMM_ACT && p.yf == nullptr && p.act.kind == GLM_ACT_XIELU) return launch_largem<GEMM_XIELU>(p, st);
+    if (mode == GEMM_SLICES) return launch_largem<GEMM_SLICES>(p, st);
     if (mode == GEMM_ACT) return launch_largem<GEMM_ACT>(p, st);
     if (mode == GEMM_GLU) return launch_largem<GEMM_GLU>(p, st);
     return launch_largem<GEMM_PLAIN>(p, st);

@@ -1060,6 +1060,14 @@ int glm_launch_gemm_smallm(int mode, const GemmParams& p, hipStream_t st) {
     if (p.G <= 1 && rows <= 32 && tiles32 >= 1024 && p.K >= 512) return launch_cfg_dma<GEMM_PLAIN, 2, 1, 2, 2>(p, st);
 #endif
     if (p.G > 1 || rows > 32 || tiles32 >= 1024) return launch_cfg<GEMM_PLAIN, 4, 1, 2, 4>(p, st);
+#ifndef GLM_SM_NO_DMA
+    // several projections in one (their activations in the epilogue): small workgroups.  Cold weights, 32 rows: 9728 x 2048 22.0 -> 14.9 us
+    // (1,1,2,2: 15.5), 18944 x 4096 47.9 -> 36.8 us (2,2,1,2: 48.0; 4,4,2,2: 45.2)
+    if (p.act.kind != GLM_ACT_NONE && p.yf == nullptr && p.K >= 512 && tiles32 >= 128) {
+        if (tiles32 < 384) return launch_cfg_dma<GEMM_PLAIN, 2, 2, 1, 2>(p, st);
+        return launch_cfg_dma<GEMM_PLAIN, 1, 1, 2, 2>(p, st);
+    }
+#endif
     // (waves, K-split waves, row tiles per wave, max 16-row activation tiles); overridable for A/B builds
 #ifndef GLM_SM_CFG_MID
 #define GLM_SM_CFG_MID 8, 2, 1, 2  // QKV at M=32: 26.9 us (4,4,2,2: 33.2; 4,2,2,2: 28.9; 8,4,2,2: 29.5)

