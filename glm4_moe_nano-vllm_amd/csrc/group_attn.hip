@@ -86,7 +86,10 @@ __device__ __forceinline__ f32x4_t ga_gate(const GroupArgs& a, int64_t row, int 
     return f32x4_t{bflo(u[0]), bfhi(u[0]), bflo(u[1]), bfhi(u[1])};
 }
 // forms of the tiled kernels
-enum : int { GA_SOFTMAX = 0, GA_TWO_MAPS = 1, GA_SIGMOID_KV = 2 };
+// (GA_TWO_MAPS: the scores have a soft cap that 2^score fits under as it is; GA_TWO_MAPS_ANY: any cap, or none)
+enum : int { GA_SOFTMAX = 0, GA_TWO_MAPS = 1, GA_SIGMOID_KV = 2, GA_TWO_MAPS_ANY = 3 };
+constexpr float GA_CAP_FITS = 55.f;  // cap log2(e) <= 80: the sums of 2^score stay far inside fp32 whatever their number
+__host__ __device__ constexpr bool ga_two(int form) { return form == GA_TWO_MAPS || form == GA_TWO_MAPS_ANY; }
 
 // ---------------------------------------------------------------------------------------------------------------------------
 struct StoreArgs {
@@ -119,7 +122,7 @@ __global__ __launch_bounds__(256) void group_kv_store_kernel(const StoreArgs a) 
 // zeros in the other map's half)
 template <int DK, int DV, int NT, int F>
 struct Slab {
-    static constexpr bool SPLIT = F == GA_TWO_MAPS && NT == 2;
+    static constexpr bool SPLIT = ga_two(F) && NT == 2;
     static constexpr int KS = DK / 32, KQ = SPLIT ? KS / 2 : KS, VT = DV / 16, KB = DK * 2, VB = DV * 2;
     static constexpr bool VEARLY = DK + DV <= 256;                    // V fragments requested in front of the score products
     static constexpr int KG = KS < 4 ? KS : 4, VG = VEARLY ? VT : 4;  // fragments per request group
@@ -127,6 +130,7 @@ struct Slab {
     f32x4_t acc[NT][VT];
     float m_run[NT], l_run[NT], slope[NT];                // slope: per key, in units of the unscaled score; sigmoid: the bias in log2 units
     float cap_in, cap_out;                                // soft cap: exponent per unit of score, cap in log2 units (0: none)
+    float cap_lim, ca0, ca1, ca2, ca3;                    // scores up to cap_lim: odd polynomial
     int rp[NT], rlo[NT];                                  // position of the lane's row and the first one it sees; rp < 0: no row
     int any_lo[NT], any_hi[NT], full_lo[NT], full_hi[NT]; // keys that some row / every row of the tile sees
     unsigned k_rel[2], v_rel[4];
@@ -146,6 +150,37 @@ struct Slab {
 #pragma unroll
             for (int d = 0; d < VT; ++d) acc[t][d] = f32x4_t{0.f, 0.f, 0.f, 0.f};
         }
+    }
+    // cap tanh(s / cap) in log2 units, by tanh y = 1 - 2 / (1 + e^(2 y))
+    __device__ __forceinline__ void cap_exact(f32x4_t (&s)[2]) const {
+#pragma unroll
+        for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+            for (int r = 0; r < 4; ++r) s[kt][r] = fmaf(-2.f * cap_out, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s[kt][r] * cap_in)), cap_out);
+    }
+    // all tiles: up to a fifth of the cap tanh is its odd polynomial of degree 7 (the next term is below 2e-8 of the cap)
+    __device__ __forceinline__ void cap_scores(f32x4_t (&s)[NT][2]) const {
+        float big = 0.f;
+#pragma unroll
+        for (int t = 0; t < NT; ++t)
+#pragma unroll
+            for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) big = fmaxf(big, fabsf(s[t][kt][r]));
+        if (__any(big > cap_lim)) {
+#pragma unroll
+            for (int t = 0; t < NT; ++t) cap_exact(s[t]);
+            return;
+        }
+#pragma unroll
+        for (int t = 0; t < NT; ++t)
+#pragma unroll
+            for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+                for (int r = 0; r < 4; ++r) {
+                    const float u = s[t][kt][r] * s[t][kt][r];
+                    s[t][kt][r] *= fmaf(fmaf(fmaf(ca3, u, ca2), u, ca1), u, ca0);
+                }
     }
     // kst, vst: LDS addresses of the slab's first key row and value row; j0: position of its first key
     // kst, vst, fst: ... and of the keys' factors (sigmoid form)
@@ -209,73 +244,93 @@ struct Slab {
         });
         if constexpr (F == GA_SIGMOID_KV) asm volatile("" : "+v"(ks[0]), "+v"(ks[1]));
         bf16x8_t pf[NT];
-#pragma unroll
-        for (int t = 0; t < NT; ++t) {
-            if (!live[t]) {
-#pragma unroll
-                for (int i = 0; i < 8; ++i) pf[t][i] = (__bf16)0.f;
-                continue;
-            }
-            if constexpr (F == GA_TWO_MAPS) {
-                // cap tanh(s / cap) in log2 units: tanh y = 1 - 2 / (1 + e^(2 y))
-                if (cap_out > 0.f) {
-#pragma unroll
-                    for (int kt = 0; kt < 2; ++kt)
-#pragma unroll
-                        for (int r = 0; r < 4; ++r)
-                            s[t][kt][r] = fmaf(-2.f * cap_out, __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(s[t][kt][r] * cap_in)), cap_out);
-                }
-            }
+        if constexpr (F == GA_TWO_MAPS || F == GA_SIGMOID_KV) {  // no maximum: all tiles go through every step together
+            if constexpr (F == GA_TWO_MAPS) cap_scores(s);
             if constexpr (F == GA_SIGMOID_KV) {
 #pragma unroll
-                for (int kt = 0; kt < 2; ++kt) {
-                    const f32x4_t f = __builtin_bit_cast(f32x4_t, ks[kt]);
+                for (int t = 0; t < NT; ++t)
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) s[t][kt][r] = fmaf(s[t][kt][r] * sc, f[r], slope[t]);
-                }
+                    for (int kt = 0; kt < 2; ++kt) {
+                        const f32x4_t f = __builtin_bit_cast(f32x4_t, ks[kt]);
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) s[t][kt][r] = fmaf(s[t][kt][r] * sc, f[r], slope[t]);
+                    }
             }
-            if (j0 < full_lo[t] || j0 + 31 > full_hi[t]) {
+            bool edge = false;
+#pragma unroll
+            for (int t = 0; t < NT; ++t) edge = edge || j0 < full_lo[t] || j0 + 31 > full_hi[t];
+            if (edge) {
                 const int jl = j0 + 4 * g;
 #pragma unroll
                 for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) {
-                        const int j = jl + 16 * kt + r;
-                        if (j > rp[t] || j < rlo[t]) s[t][kt][r] = -INFINITY;
-                    }
+                    for (int r = 0; r < 4; ++r)
+#pragma unroll
+                        for (int t = 0; t < NT; ++t) {
+                            const int j = jl + 16 * kt + r, row = F == GA_TWO_MAPS ? 0 : t;  // (two maps: the same tokens)
+                            if (j > rp[row] || j < rlo[row]) s[t][kt][r] = -INFINITY;
+                        }
             }
-            if constexpr (F == GA_SIGMOID_KV) {
+#pragma unroll
+            for (int t = 0; t < NT; ++t)
 #pragma unroll
                 for (int kt = 0; kt < 2; ++kt)
 #pragma unroll
-                    for (int r = 0; r < 4; ++r) pf[t][4 * kt + r] = (__bf16)__builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-s[t][kt][r]));
-                continue;
-            }
-            float mx = -INFINITY;
+                    for (int r = 0; r < 4; ++r) {
+                        float p;
+                        if constexpr (F == GA_SIGMOID_KV) {
+                            p = __builtin_amdgcn_rcpf(1.f + __builtin_amdgcn_exp2f(-s[t][kt][r]));
+                        } else {
+                            p = __builtin_amdgcn_exp2f(s[t][kt][r]);
+                            l_run[t] += p;
+                        }
+                        pf[t][4 * kt + r] = (__bf16)p;
+                    }
+        } else {
 #pragma unroll
-            for (int kt = 0; kt < 2; ++kt)
+            for (int t = 0; t < NT; ++t) {
+                if (!live[t]) {
 #pragma unroll
-                for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s[t][kt][r]);
-            mx *= sc;
-            if (__any(mx > m_run[t] + 8.0f || (m_run[t] == -INFINITY && mx > -INFINITY))) {
-                mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
-                mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
-                const float m_new = fmaxf(m_run[t], mx);
-                const float alpha = m_new == -INFINITY ? 1.0f : __builtin_amdgcn_exp2f(m_run[t] - m_new);
-                l_run[t] *= alpha;
-#pragma unroll
-                for (int d = 0; d < VT; ++d) acc[t][d] *= alpha;
-                m_run[t] = m_new;
-            }
-            const float m_use = m_run[t] == -INFINITY ? 0.f : m_run[t];
-#pragma unroll
-            for (int kt = 0; kt < 2; ++kt)
-#pragma unroll
-                for (int r = 0; r < 4; ++r) {
-                    const float p = __builtin_amdgcn_exp2f(fmaf(s[t][kt][r], sc, -m_use));
-                    l_run[t] += p;
-                    pf[t][4 * kt + r] = (__bf16)p;
+                    for (int i = 0; i < 8; ++i) pf[t][i] = (__bf16)0.f;
+                    continue;
                 }
+                if (F == GA_TWO_MAPS_ANY && cap_out > 0.f) cap_exact(s[t]);
+                if (j0 < full_lo[t] || j0 + 31 > full_hi[t]) {
+                    const int jl = j0 + 4 * g;
+#pragma unroll
+                    for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+                        for (int r = 0; r < 4; ++r) {
+                            const int j = jl + 16 * kt + r;
+                            if (j > rp[t] || j < rlo[t]) s[t][kt][r] = -INFINITY;
+                        }
+                }
+                float mx = -INFINITY;
+#pragma unroll
+                for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) mx = fmaxf(mx, s[t][kt][r]);
+                mx *= sc;
+                if (__any(mx > m_run[t] + 8.0f || (m_run[t] == -INFINITY && mx > -INFINITY))) {
+                    mx = fmaxf(mx, __shfl_xor(mx, 16, 64));
+                    mx = fmaxf(mx, __shfl_xor(mx, 32, 64));
+                    const float m_new = fmaxf(m_run[t], mx);
+                    const float alpha = m_new == -INFINITY ? 1.0f : __builtin_amdgcn_exp2f(m_run[t] - m_new);
+                    l_run[t] *= alpha;
+#pragma unroll
+                    for (int d = 0; d < VT; ++d) acc[t][d] *= alpha;
+                    m_run[t] = m_new;
+                }
+                const float m_use = m_run[t] == -INFINITY ? 0.f : m_run[t];
+#pragma unroll
+                for (int kt = 0; kt < 2; ++kt)
+#pragma unroll
+                    for (int r = 0; r < 4; ++r) {
+                        const float p = __builtin_amdgcn_exp2f(fmaf(s[t][kt][r], sc, -m_use));
+                        l_run[t] += p;
+                        pf[t][4 * kt + r] = (__bf16)p;
+                    }
+            }
         }
         static_for<VT / VG>([&](auto GI) {
             constexpr int d0 = decltype(GI)::value * VG;
@@ -293,8 +348,19 @@ struct Slab {
         });
     }
     __device__ __forceinline__ void set_cap(const GroupArgs& a) {
+        if constexpr (!ga_two(F)) return;
         cap_in = a.cap > 0.f ? 2.f * GA_LOG2E * a.scale / a.cap : 0.f;
         cap_out = a.cap * GA_LOG2E;
+        const float k = a.cap > 0.f ? a.scale / a.cap : 0.f, kk = k * k;
+        cap_lim = k > 0.f ? 0.2f / k : 0.f;
+        ca0 = cap_out * k;
+        ca1 = ca0 * kk * (-1.f / 3.f);
+        ca2 = ca0 * kk * kk * (2.f / 15.f);
+        ca3 = ca0 * kk * kk * kk * (-17.f / 315.f);
+        if constexpr (F == GA_TWO_MAPS) {
+#pragma unroll
+            for (int t = 0; t < NT; ++t) m_run[t] = 0.f;
+        }
     }
     __device__ __forceinline__ float mass(int t) const {
         float l = l_run[t];
@@ -309,7 +375,7 @@ struct Slab {
 template <int DK, int DV, int F>
 __global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void group_attn_prefill_kernel(const GroupArgs a) {
     using SL = Slab<DK, DV, 2, F>;
-    constexpr bool TWO = F == GA_TWO_MAPS, KV = F == GA_SIGMOID_KV;
+    constexpr bool TWO = ga_two(F), KV = F == GA_SIGMOID_KV;
     constexpr int KQ = SL::KQ, VT = SL::VT, KB = SL::KB, VB = SL::VB, KTILE = 64 * KB, VTILE = KV ? 256 : 64 * VB, STAGE = KTILE + VTILE;  // (behind the keys: values, or the keys' factors)
     constexpr int KCPR = DK / 8, VCPR = DV / 8, KDMA = DK / 32, VDMA = KV ? 0 : DV / 32;
     constexpr int MAPC = TWO ? KCPR / 2 : KCPR;  // chunks of one map in an LDS row
@@ -471,7 +537,7 @@ __global__ __launch_bounds__(256, (DK + DV) <= 256 ? 2 : 1) void group_attn_pref
 // stages and softmax state: no barrier in the loop.
 template <int DK, int DV, int NW, int F>
 __global__ __launch_bounds__(NW * 64, 1) void group_attn_decode_kernel(const GroupArgs a, int row_groups) {
-    constexpr bool TWO = F == GA_TWO_MAPS, KV = F == GA_SIGMOID_KV;
+    constexpr bool TWO = ga_two(F), KV = F == GA_SIGMOID_KV;
     constexpr int RPG = TWO ? 8 : 16;  // (token, head) rows of a group: 16, or 8 of either map
     using SL = Slab<DK, DV, 1, F>;
     constexpr int KS = SL::KS, VT = SL::VT, KB = SL::KB, VB = SL::VB, KSLAB = 32 * KB, STAGE = KSLAB + (KV ? 256 : 32 * VB);
@@ -775,7 +841,7 @@ int launch_prefill(const GroupArgs& a, hipStream_t st) {
     static_assert(LDS <= 160 * 1024, "LDS of a CU");
     auto kern = group_attn_prefill_kernel<DK, DV, F>;
     GLM_SET_MAX_LDS(kern, LDS, "glm_group_attn_prefill");
-    const int64_t per = ((int64_t)a.n_tiles * (a.H >> (F == GA_TWO_MAPS ? 0 : a.pair)) + 7) / 8;
+    const int64_t per = ((int64_t)a.n_tiles * (a.H >> (ga_two(F) ? 0 : a.pair)) + 7) / 8;
     GLM_CHECK_ARG(per * 8 < (1ll << 31), GLM_ERR_UNSUPPORTED, "glm_group_attn_prefill: grid too large");
     hipLaunchKernelGGL(kern, dim3((unsigned)(per * 8)), dim3(256), LDS, st, a);
     GLM_CHECK_LAUNCH("glm_group_attn_prefill");
@@ -818,7 +884,8 @@ int launch_decode(const GroupArgs& a, int row_groups, hipStream_t st) {
             if (kk == 2) return F<128, 128, GA_SIGMOID_KV>(__VA_ARGS__);                             \
             return F<256, 256, GA_SIGMOID_KV>(__VA_ARGS__);                                          \
         }                                                                                            \
-        if (a.maps == 2) GA_SIZES(F, kk, vv, GA_TWO_MAPS, __VA_ARGS__);                              \
+        if (a.maps == 2 && a.cap > 0.f && a.cap <= GA_CAP_FITS) GA_SIZES(F, kk, vv, GA_TWO_MAPS, __VA_ARGS__); \
+        if (a.maps == 2) GA_SIZES(F, kk, vv, GA_TWO_MAPS_ANY, __VA_ARGS__);                          \
         GA_SIZES(F, kk, vv, GA_SOFTMAX, __VA_ARGS__);                                                \
     } while (0)
 

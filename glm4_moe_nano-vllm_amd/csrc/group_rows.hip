@@ -71,13 +71,13 @@ __device__ __forceinline__ int64_t gr_base(int slot, int bs, int log2_bs, int G)
 }
 
 // UNIT 8: half of the rotated columns is a multiple of eight, pieces of eight; 1: column by column (the values still by eight).  An item is
-// eight pairs (or one), eight columns of a key that do not turn (or one), eight columns of a value; workgroup (row, 256 items of it)
+// eight pairs (or one), eight columns of a key that do not turn (or one), eight columns of a value; workgroup (row, part of its items)
 template <typename T, int UNIT>
-__global__ __launch_bounds__(256) void group_rotate_store_kernel(const RotArgs a) {
+__global__ __launch_bounds__(512) void group_rotate_store_kernel(const RotArgs a) {
     const int half = a.dims / 2, pi = half / UNIT, ri = (a.dm - a.dims) / UNIT, nk = a.G * a.maps;
     const int n_q = a.nq * pi, n_k = nk * pi, n_r = nk * ri;
     const int64_t r = blockIdx.x;
-    int i = blockIdx.y * 256 + threadIdx.x;
+    int i = blockIdx.y * blockDim.x + threadIdx.x;
     if (i >= a.per) return;
     const int slot = a.slots[r];
     T* row = reinterpret_cast<T*>(a.x) + r * a.ld;
@@ -241,9 +241,10 @@ template <typename T>
 void launch_rotate(RotArgs a, hipStream_t st) {
     const int unit = a.dims % 16 == 0 ? 8 : 1, half = a.dims / 2, nk = a.G * a.maps;
     a.per = (a.nq + nk) * (half / unit) + nk * ((a.dm - a.dims) / unit) + a.G * (a.dv / 8);
-    const dim3 grid((unsigned)a.T, (unsigned)((a.per + 255) / 256));
-    if (unit == 8) hipLaunchKernelGGL((group_rotate_store_kernel<T, 8>), grid, dim3(256), 0, st, a);
-    else hipLaunchKernelGGL((group_rotate_store_kernel<T, 1>), grid, dim3(256), 0, st, a);
+    const int parts = (a.per + 511) / 512, size = ((a.per + parts - 1) / parts + 63) / 64 * 64;  // equal parts of whole waves
+    const dim3 grid((unsigned)a.T, (unsigned)parts);
+    if (unit == 8) hipLaunchKernelGGL((group_rotate_store_kernel<T, 8>), grid, dim3(size), 0, st, a);
+    else hipLaunchKernelGGL((group_rotate_store_kernel<T, 1>), grid, dim3(size), 0, st, a);
 }
 template <typename T>
 void launch_norm(const NormArgs& a, int64_t rows, hipStream_t st) {

@@ -89,6 +89,21 @@ def test_residual_norm_many_rows():
             assert torch.allclose(a[k].float(), torch.cat([p[k] for p in b]).float(), rtol=1e-6 if k == 0 else 1e-2, atol=1e-6)
 
 
+@pytest.mark.parametrize("M,N,K", [(97, 264, 1024), (128, 2048, 4096), (200, 520, 2048), (300, 1032, 8192), (500, 64, 1536)])
+def test_slices_of_k(M, N, K):
+    """Partial sums of a projection of some hundred rows, out of a part of wider rows: as many slices as the chip has room for, and given numbers."""
+    from nanovllm import hip_ops
+    rows = torch.randn(M, K + 72, generator=g(1)).to(torch.bfloat16)
+    w = (torch.randn(N, K, generator=g(2)) * K ** -0.5).to(torch.bfloat16)
+    want = rows[:, 8: 8 + K].double() @ w.double().T
+    assert hip_ops.gemm_slices(M, N, K) > 1 and hip_ops.gemm_slices(40, N, K) == 1 and hip_ops.gemm_slices(M, N, K + 8) == 1 and hip_ops.gemm_slices(16384, 4096, K) == 1
+    for ns in {hip_ops.gemm_slices(M, N, K), 2, 4, 8}:
+        part = hip_ops.gemm_bf16_partial(dev(rows)[:, 8: 8 + K], dev(w), ns).part
+        assert part.shape == (ns, M, N) and close(part.sum(0), want, 1e-4), ns
+        k = K // ns
+        assert close(part[1], rows[:, 8 + k: 8 + 2 * k].double() @ w[:, k: 2 * k].double().T, 1e-4)
+
+
 def test_rotation_far_positions():
     from nanovllm.layers.rotary_embedding import HalfRotary
     rot = HalfRotary(40, 20, 500000.0)
