@@ -209,7 +209,7 @@ def _paged(rows, G, bs, n_blocks, perm, fill=float("nan")):
 
 
 FORMS = [("two_maps", 6, 2, 24, 40, 64), ("two_maps", 4, 4, 64, 128, 64), ("two_maps", 12, 1, 128, 256, 128), ("two_maps", 2, 2, 8, 8, 64), ("two_maps", 5, 1, 72, 64, 192),
-         ("two_maps", 3, 1, 32, 200, 64),
+         ("two_maps", 3, 1, 32, 200, 64), ("two_maps_70", 6, 2, 24, 40, 64), ("two_maps_70", 4, 1, 64, 128, 64), ("two_maps_0", 4, 2, 40, 72, 64),
          ("sigmoid", 6, 2, 24, 24, 64), ("sigmoid", 20, 1, 128, 128, 64), ("sigmoid", 3, 3, 200, 200, 128), ("sigmoid", 8, 2, 64, 64, 64),
          ("softmax", 6, 3, 40, 72, 64), ("softmax", 17, 1, 128, 64, 64)]
 
@@ -217,10 +217,11 @@ FORMS = [("two_maps", 6, 2, 24, 40, 64), ("two_maps", 4, 4, 64, 128, 64), ("two_
 @pytest.mark.parametrize("form,H,G,dim,dv,bs", FORMS)
 @pytest.mark.parametrize("kind", ["decode1", "decode1_split", "decode5", "prefill", "plain", "plain_f32"])
 def test_group_attention_forms(form, H, G, dim, dv, bs, kind):
-    """Two maps with a soft cap, sigmoid weights over keys that are the values, a softmax without sinks; gates per head, per column, none.  Pages in
+    """Two maps with a soft cap that scores come near, a high one, none; sigmoid weights over keys that are the values, a softmax without sinks; gates per head, per column, none.  Pages in
     disorder, NaNs wherever nothing was stored; single keys that stand out: the first one, those at page borders, the row's own."""
     from nanovllm import hip_ops
     dtype = "float32" if kind == "plain_f32" else "bfloat16"
+    form, cap = (form[:8], float(form[9:] or 20)) if form.startswith("two_maps") else (form, 0.0)
     dt, R, maps = DT[dtype], H // G, 2 if form == "two_maps" else 1
     r = lambda t: t.to(dt).float()  # noqa: E731
     if kind.startswith("decode1"):
@@ -232,7 +233,7 @@ def test_group_attention_forms(form, H, G, dim, dv, bs, kind):
     k = [torch.randn(n, G, maps, dim, generator=g(s)) * 0.7 for s, n in enumerate(lens)]
     v = [torch.randn(n, G, dv, generator=g(50 + s)) for s, n in enumerate(lens)]
     q = [torch.randn(m, H, maps, dim, generator=g(90 + s)) * 0.7 for s, m in enumerate(n_q)]
-    scale, cap, lam, post, eps = 0.9, 20.0, 0.4, 0.6, 1e-3
+    scale, lam, post, eps = 0.9, 0.4, 0.6, 1e-3
     for s, n in enumerate(lens):
         for h, j in ((0, 0), (H - 1, (n - 1) // 64 * 64), (H // 2, (n - 1) // 64 * 64 - 1), (H // 3, n - 1)):
             if 0 <= j < n:
@@ -288,7 +289,7 @@ def test_group_attention_forms(form, H, G, dim, dv, bs, kind):
                     if form == "sigmoid":
                         a = O.sigmoid(z * ks[s][:, 0, 0].double() + bias[h].double()) * visible
                     else:
-                        z = (O.soft_cap(z, cap) if form == "two_maps" else z).masked_fill(~visible, -math.inf)
+                        z = (O.soft_cap(z, cap) if cap else z).masked_fill(~visible, -math.inf)
                         a = torch.softmax(z, -1)
                     res.append(a @ v[s][:, h // R].double())
                 want = res[0] if maps == 1 else O.unit_rms(res[0] - lam * res[1], eps) * post
