@@ -21,11 +21,10 @@ struct MergeArgs {
     int vn;
 };
 
-// The splits of one row, sixteen in flight: this wave adds up splits w, w + WPR, ... of the row's columns k .. k + 4, each weighed with its
+// The splits of one row, N in flight: this wave adds up splits w, w + WPR, ... of the row's columns k .. k + 4, each weighed with its
 // share of the row's mass (brought to the common maximum, over the mass of all and the sink's)
-template <int WPR>
+template <int WPR, int N>
 __device__ __forceinline__ f32x4_t merge_row(const MergeArgs& a, int64_t prow, int h, int k, int lane, int w) {
-    constexpr int N = WPR == 1 ? 16 : 8;
     const float* p = a.part_o + prow * a.nsplit * a.cols + k;
     float m = -INFINITY, l = 0.f;
     if (lane < a.nsplit) {
@@ -59,7 +58,7 @@ __device__ __forceinline__ f32x4_t merge_row(const MergeArgs& a, int64_t prow, i
 }
 
 // WPR waves (1 or 4) per (token, head) and 256 columns; two maps: all columns of a head together
-template <bool TWO, int WPR>
+template <bool TWO, int WPR, int N>
 __global__ __launch_bounds__(256) void attn_merge_kernel(const MergeArgs a) {
     __shared__ f32x4_t sums[WPR == 1 ? 1 : (TWO ? 2 : 1) * (WPR - 1)][64];
     const int lane = threadIdx.x & 63, w = threadIdx.x >> 6;
@@ -70,10 +69,10 @@ __global__ __launch_bounds__(256) void attn_merge_kernel(const MergeArgs a) {
     const bool on = k < a.cols;
     f32x4_t o, y;
     if constexpr (TWO) {
-        o = merge_row<WPR>(a, grow * 2, h, kk, lane, WPR == 1 ? 0 : w);
-        y = merge_row<WPR>(a, grow * 2 + 1, h, kk, lane, WPR == 1 ? 0 : w);
+        o = merge_row<WPR, N>(a, grow * 2, h, kk, lane, WPR == 1 ? 0 : w);
+        y = merge_row<WPR, N>(a, grow * 2 + 1, h, kk, lane, WPR == 1 ? 0 : w);
     } else {
-        o = merge_row<WPR>(a, grow, h, kk, lane, WPR == 1 ? 0 : w);
+        o = merge_row<WPR, N>(a, grow, h, kk, lane, WPR == 1 ? 0 : w);
     }
     if constexpr (WPR > 1) {
         if (w > 0) {
@@ -106,12 +105,12 @@ __global__ __launch_bounds__(256) void attn_merge_kernel(const MergeArgs a) {
     *reinterpret_cast<u32x2_t*>(a.out + t * a.ldo + (int64_t)h * a.cols + k) = u32x2_t{pack2bf(o[0], o[1]), pack2bf(o[2], o[3])};
 }
 
-template <int WPR>
+template <int WPR, int N>
 void launch(const MergeArgs& a, int maps, hipStream_t st) {
     const int64_t items = a.rows * a.nchunk;
     const dim3 grid((unsigned)(WPR == 1 ? (items + 3) / 4 : items));
-    if (maps == 2) hipLaunchKernelGGL((attn_merge_kernel<true, WPR>), grid, dim3(256), 0, st, a);
-    else hipLaunchKernelGGL((attn_merge_kernel<false, WPR>), grid, dim3(256), 0, st, a);
+    if (maps == 2) hipLaunchKernelGGL((attn_merge_kernel<true, WPR, N>), grid, dim3(256), 0, st, a);
+    else hipLaunchKernelGGL((attn_merge_kernel<false, WPR, N>), grid, dim3(256), 0, st, a);
 }
 
 }  // namespace
@@ -130,8 +129,9 @@ extern "C" int glm_attn_merge(const float* part_o, const float* part_ml, const f
         a.gate = (const bf16_t*)form->gate; a.ldg = form->ldg; a.gate_cols = form->gate_cols;
         a.lam = form->lam; a.post = form->post; a.eps = form->eps; a.vn = form->vn;
     }
-    if (a.rows * a.nchunk <= 2048 && nsplit > 4) launch<4>(a, maps, glm_s(stream));
-    else launch<1>(a, maps, glm_s(stream));
+    if (nsplit <= 4) launch<1, 4>(a, maps, glm_s(stream));
+    else if (a.rows * a.nchunk <= 2048) launch<4, 8>(a, maps, glm_s(stream));
+    else launch<1, 16>(a, maps, glm_s(stream));
     GLM_CHECK_LAUNCH("glm_attn_merge");
     return GLM_OK;
 }
