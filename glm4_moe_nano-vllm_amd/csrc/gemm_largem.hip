@@ -1668,7 +1668,7 @@ int launch_largem_cfg(const GemmParams& p, hipStream_t st) {
     const int cols_per_wg = gemm_paired(MODE) ? 128 : LM_BN;
     const int n_tiles = (p.N + cols_per_wg - 1) / cols_per_wg;
     const int64_t combos = p.offs ? (p.R / C::BM + p.G) : (p.R + C::BM - 1) / C::BM * (MODE == GEMM_SLICES ? p.G : 1);
-    // (a band higher than the rows' blocks would be mostly positions without a tile: 74 tiles of one block took two rounds of 256
+    // (a band higher than the rows' blocks would be mostly positions without a tile: 74 tiles of one block took two passes of 256
     // workgroups)
     const int LM_BAND = p.offs ? g_largem_band : (int)(combos < g_largem_band ? combos : (int64_t)g_largem_band);
     const int64_t total = (combos + LM_BAND - 1) / LM_BAND * LM_BAND * n_tiles;
